@@ -551,6 +551,61 @@ int lvllm_rope_cache_paged_attention_q(
 int64_t lvllm_get_device_attribute(int64_t attribute, int64_t device_id);
 int64_t lvllm_get_max_shared_memory_per_block_device_attribute(int64_t device_id);
 
+/* ---- hybrid decoders: paged attention beside recurrent mixers (csrc/token_mix.hip, recurrent.hip, head_attention.hip) ----
+ * A step's rows are the new tokens of num_seqs sequences back to back: rows query_start_loc[s] .. query_start_loc[s+1]
+ * (int32 [num_seqs + 1]) end sequence s at position seq_lens[s] - 1.  Rows past the last sequence are padding.
+ * state_slots int32 [num_seqs]: the sequence's slot of a state tensor (< 0 or >= num_slots: none -- the state starts at
+ * zero and is not stored).  A sequence whose tokens are all in the step (seq_lens == its rows) starts at zero too.
+ * `y` / `partials`: a projection result to add, [rows, width] elements, or num_partials fp32 slabs of it (the split-K
+ * output of lvllm_skinny_gemm_ex); both null: nothing is added.  Residuals, norm weights and gates are fp32. */
+
+/* x_out = x_in + y; h = T(tanh(alpha * x_out) * weight + bias).  x_out may be x_in. */
+int lvllm_add_dyt(float* x_out, const float* x_in, const void* y, const float* partials, int num_partials, void* h,
+                  const float* alpha, const float* weight, const float* bias, int rows, int width, int dtype, void* stream);
+/* the same norm, then mix[m] = T(h + (h' - h) * mu[m]) with h' the row before (token shift): mix [num_mix, rows, width],
+ * mu float [num_mix, width]; carried float [num_slots, carried_stride]: the last normed row of each sequence.
+ * x_out != x_in. */
+int lvllm_add_dyt_shift_mix(float* x_out, const float* x_in, const void* y, const float* partials, int num_partials,
+                            void* mix, const float* mu, int num_mix, const float* alpha, const float* weight,
+                            const float* bias, float* carried, int64_t carried_stride, const int32_t* state_slots,
+                            int num_slots, const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows,
+                            int width, int dtype, void* stream);
+/* out = max(x, 0)^2 (out may be x) */
+int lvllm_relu_squared(void* out, const void* x, int64_t n, int dtype, void* stream);
+/* Per-head RMS norm of q and k (weights float [dim], shared by heads), normed keys and the values into a paged cache of
+ * unequal key and value sizes: key_cache [num_blocks, kv_heads, kpad/x, block_size, x], value_cache [num_blocks, kv_heads,
+ * vpad, block_size]; q_out [rows, heads, kpad].  Padding elements are written as zeros.  slot_mapping int64 [rows]
+ * (outside the cache: nothing cached). */
+int lvllm_qk_norm_cache(void* q_out, void* key_cache, void* value_cache, const void* q, const void* k, const void* v,
+                        int64_t row_stride, const float* q_weight, const float* k_weight, float eps, int rows, int heads,
+                        int kv_heads, int dim, int vdim, int kpad, int vpad, const int64_t* slot_mapping,
+                        int64_t num_blocks, int block_size, int64_t k_block_stride, int64_t v_block_stride, int dtype,
+                        void* stream);
+/* out[row, h * vdim + d] = T(attn[row, h, d] * sigmoid(gate[row, h]) * scale) */
+int lvllm_head_gate(void* out, int64_t out_stride, const void* attn, int64_t attn_head_stride, const void* gate,
+                    int64_t gate_stride, int rows, int heads, int vdim, float scale, int dtype, void* stream);
+/* out = T(o / rms(o over vdim) * weight * silu(gate) * scale) per head; o float [rows, heads, vdim]; weight float,
+ * weight_head_stride apart between heads (0: shared) */
+int lvllm_head_norm_gate(void* out, int64_t out_stride, const float* o, const void* gate, int64_t gate_stride,
+                         const float* weight, int weight_head_stride, float eps, float scale, int rows, int heads,
+                         int vdim, int dtype, void* stream);
+/* ln w [rows, channels] = logsigmoid(z) * inv_tau (kind 0) or -exp(z) (kind 1), z = A f(u) + bias with f = identity
+ * (kind 0) or tanh (kind 1); a_t float [rank, channels] = A transposed */
+int lvllm_log_decay(float* out, const void* u, int64_t u_stride, const float* a_t, const float* bias, int kind,
+                    float inv_tau, int rows, int rank, int channels, int dtype, void* stream);
+/* S_t = diag(w_t) S_{t-1} + k_t v_t^T; o_t = S_t^T q_t, or with bonus (float [heads, dk]) o_t = (S_{t-1} + diag(bonus)
+ * k_t v_t^T)^T q_t.  q is multiplied by q_scale.  state float [num_slots, heads, dk, dv], slots state_stride apart. */
+int lvllm_recurrent_scan(float* o, const void* q, const void* k, const void* v, int64_t q_stride, int64_t k_stride,
+                         int64_t v_stride, const float* log_decay, const float* bonus, float q_scale, float* state,
+                         int64_t state_stride, const int32_t* state_slots, int num_slots, const int32_t* query_start_loc,
+                         const int32_t* seq_lens, int num_seqs, int heads, int dk, int dv, int dtype, void* stream);
+/* Causal attention over the cache of lvllm_qk_norm_cache; q [rows, heads, kpad], out [rows, heads, vpad]. */
+int lvllm_head_attention(void* out, const void* q, const void* key_cache, const void* value_cache,
+                         const int32_t* block_tables, const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs,
+                         int rows, int heads, int kv_heads, int kpad, int vpad, int max_blocks, int block_size,
+                         int64_t num_blocks, float scale, int64_t k_block_stride, int64_t v_block_stride, int dtype,
+                         void* stream);
+
 #ifdef __cplusplus
 }
 #endif

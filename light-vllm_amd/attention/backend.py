@@ -106,6 +106,8 @@ class PagedAttnMetadata:
     # (not in the reference) paged_attention_v2 scratch (exp_sums, max_logits, tmp_out) owned by the caller: a
     # captured step brings its own, so that two graphs replaying on two streams never share one
     decode_scratch: Optional[tuple] = None
+    # (not in the reference) slot of each sequence's recurrent state, int32 [num_seqs]: models that have one
+    state_slots: Optional[torch.Tensor] = None
 
     @property
     def prefill_metadata(self) -> Optional["PagedAttnMetadata"]:
@@ -178,6 +180,7 @@ class PagedAttnMetadataBuilder:
         self.context_lens: List[int] = []
         self.block_tables: List[List[int]] = []
         self.curr_seq_lens: List[int] = []
+        self.state_slots: List[int] = []
         self.num_prefills = 0
         self.num_prefill_tokens = 0
         self.num_decode_tokens = 0
@@ -194,6 +197,8 @@ class PagedAttnMetadataBuilder:
             context_len = inter_data.context_lens[i]
             curr_sw_blocks = inter_data.curr_sliding_window_blocks[i]
             self.context_lens.append(context_len)
+            if getattr(inter_data, "state_slots", None) is not None:
+                self.state_slots.append(inter_data.state_slots[seq_id])
             if is_prompt:
                 self.num_prefills += 1
                 self.num_prefill_tokens += token_len
@@ -246,7 +251,8 @@ class PagedAttnMetadataBuilder:
             max_decode_seq_len=max(self.curr_seq_lens, default=0),
             query_start_loc=query_start_loc, seq_start_loc=seq_start_loc,
             context_lens_tensor=cpu(self.context_lens, torch.int32), block_tables=block_tables,
-            use_cuda_graph=False, query_lens=list(query_lens), context_lens=list(self.context_lens))
+            use_cuda_graph=False, query_lens=list(query_lens), context_lens=list(self.context_lens),
+            state_slots=cpu(self.state_slots, torch.int32) if self.state_slots else None)
 
     def __call__(self, *args, **kwargs):
         """AttentionMetadataBuilder's abstract call hook (backends/attention/abstract.py:90-92); the

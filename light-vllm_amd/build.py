@@ -1,12 +1,15 @@
 """Build the gfx950 native libraries in-tree (no cmake, no hipify).
 
-  liblvllm_hip.so   hand-written HIP kernels behind the C-ABI of include/lvllm_hip.h
+  liblvllm_base.so  what every model needs: error plumbing, cache block movement, the weight-streaming GEMMs of decode
+                    steps, step inputs, the sampler, and the kernels of the hybrid (attention + recurrent) decoders
+  liblvllm_hip.so   the rest of the C-ABI of include/lvllm_hip.h (paged and prefill attention of the rotary decoders,
+                    norms, fp8); it needs liblvllm_base.so, so a handle on it resolves every symbol of the header
                     (hipcc --offload-arch=gfx950, one object per .hip, linked -shared)
-  _C.so             torch op registrations (`torch.ops._C`, `_C_cache_ops`,
-                    `_C_cuda_utils`) forwarding to the C-ABI; host-only C++,
-                    built with g++ against the torch headers.
+  _C_base.so, _C.so torch op registrations (`torch.ops._C`, `_C_cache_ops`, `_C_cuda_utils`, `_C_amd`) forwarding to
+                    the C-ABI; host-only C++, built with g++ against the torch headers.
 
-Both land in light-vllm_amd/lib/.  Objects are cached under build/ keyed on the
+`build_all(("base",))` builds the first pair only: all that a model whose registry entry says so will load.
+All land in light-vllm_amd/lib/.  Objects are cached under build/ keyed on the
 source mtime, so a rebuild after touching one kernel takes seconds.
 """
 import os
@@ -21,24 +24,33 @@ LIBDIR = os.path.join(PKG, "lib")
 OBJDIR = os.path.join(ROOT, "build", "obj")
 ARCH = "gfx950"
 
-HIP_SOURCES = [
+BASE_SOURCES = [
     "capi.hip",
     "cache.hip",
+    "skinny_gemm.hip",
+    "prepare_inputs.hip",
+    "sampler.hip",
+    "activation.hip",
+    "token_mix.hip",
+    "recurrent.hip",
+    "head_attention.hip",
+]
+FULL_SOURCES = [
     "layernorm.hip",
     "pos_encoding.hip",
-    "activation.hip",
     "attention.hip",
     "attention_bf16.hip",
     "attention_f16.hip",
-    "skinny_gemm.hip",
     "prefill_attention.hip",
-    "prepare_inputs.hip",
     "fp8_quant.hip",
-    "sampler.hip",
 ]
+COMPONENTS = {"base": (BASE_SOURCES, "liblvllm_base.so", "torch_bindings_base.cpp", "_C_base.so"),
+              "full": (FULL_SOURCES, "liblvllm_hip.so", "torch_bindings.cpp", "_C.so")}
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # tuning experiments: e.g. LVLLM_EXTRA_HIPCC_FLAGS="-DLVLLM_ATTN_NBUF=2 -DLVLLM_ATTN_TUNE_ONLY"
+# No packed fp32 arithmetic (v_pk_add / mul / fma_f32): some of its forms have given wrong results on this hardware.
+BASE_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 EXTRA_FLAGS = os.environ.get("LVLLM_EXTRA_HIPCC_FLAGS", "").split()
 
 
@@ -69,65 +81,76 @@ def _run(cmd):
 PER_SOURCE_FLAGS = {"prefill_attention.hip": ["-fno-honor-nans"]}
 
 
-def build_kernels(verbose=False):
+def build_kernels(components=("base", "full"), verbose=False, force=False):
     os.makedirs(OBJDIR, exist_ok=True)
     os.makedirs(LIBDIR, exist_ok=True)
     hdrs = _headers()
     jobs = []
-    objs = []
-    for src in HIP_SOURCES:
-        s = os.path.join(CSRC, src)
-        o = os.path.join(OBJDIR, src.replace(".hip", ".o"))
-        objs.append(o)
-        if _newer(o, [s] + hdrs):
-            jobs.append([HIPCC, "--offload-arch=" + ARCH, "-O3", "-std=c++17", "-fPIC",
-                         "-ffp-contract=off", "-Wall", "-Wno-unused-function"] +
-                        PER_SOURCE_FLAGS.get(src, []) + EXTRA_FLAGS + ["-c", s, "-o", o])
+    objs = {c: [] for c in components}
+    for c in components:
+        for src in COMPONENTS[c][0]:
+            s = os.path.join(CSRC, src)
+            o = os.path.join(OBJDIR, src.replace(".hip", ".o"))
+            objs[c].append(o)
+            if force or _newer(o, [s] + hdrs):
+                jobs.append([HIPCC, "--offload-arch=" + ARCH, "-O3", "-std=c++17", "-fPIC",
+                             "-ffp-contract=off", "-Wall", "-Wno-unused-function"] + BASE_FLAGS +
+                            PER_SOURCE_FLAGS.get(src, []) + EXTRA_FLAGS + ["-c", s, "-o", o])
     if jobs:
         with ThreadPoolExecutor(max_workers=min(6, len(jobs))) as ex:
             for out in ex.map(_run, jobs):
                 if verbose and out.strip():
                     print(out)
-    lib = os.path.join(LIBDIR, "liblvllm_hip.so")
-    if jobs or _newer(lib, objs):
-        # no rpath to /opt/rocm on purpose: inside a torch process the HIP
-        # runtime torch already loaded (same SONAME) must be the one used.
-        _run([HIPCC, "--offload-arch=" + ARCH, "-shared", "-fPIC", "-o", lib] + objs)
-    return lib
+    libs = []
+    for c in components:
+        lib = os.path.join(LIBDIR, COMPONENTS[c][1])
+        libs.append(lib)
+        if force or _newer(lib, objs[c] + [os.path.abspath(__file__)]):
+            # no rpath to /opt/rocm on purpose: inside a torch process the HIP
+            # runtime torch already loaded (same SONAME) must be the one used.
+            link = [] if c == "base" else ["-L", LIBDIR, "-llvllm_base", "-Wl,-rpath,$ORIGIN"]
+            _run([HIPCC, "--offload-arch=" + ARCH, "-shared", "-fPIC", "-o", lib] + objs[c] + link)
+    return libs
 
 
-def build_torch_bindings(verbose=False):
+def build_torch_bindings(components=("base", "full"), verbose=False, force=False):
     import torch  # noqa: F401  (header + library locations)
     from torch.utils import cpp_extension as ce
-
-    os.makedirs(LIBDIR, exist_ok=True)
-    src = os.path.join(CSRC, "torch_bindings.cpp")
-    out = os.path.join(LIBDIR, "_C.so")
-    if not _newer(out, [src, os.path.join(ROOT, "include", "lvllm_hip.h")]):
-        return out
     import sysconfig
 
+    os.makedirs(LIBDIR, exist_ok=True)
     incs = ce.include_paths("cuda") + [sysconfig.get_paths()["include"], os.path.join(ROOT, "include")]
     torch_lib = os.path.join(os.path.dirname(torch.__file__), "lib")
-    cmd = ["g++", "-O2", "-std=c++17", "-fPIC", "-shared", "-D__HIP_PLATFORM_AMD__=1",
-           "-DUSE_ROCM=1", "-DTORCH_EXTENSION_NAME=_C",
-           "-D_GLIBCXX_USE_CXX11_ABI=%d" % int(torch._C._GLIBCXX_USE_CXX11_ABI),
-           "-Wno-deprecated-declarations"]
-    for i in incs:
-        cmd += ["-I", i]
-    cmd += [src, "-o", out, "-L", torch_lib, "-L", LIBDIR,
-            "-ltorch", "-ltorch_cpu", "-ltorch_hip", "-lc10", "-lc10_hip", "-llvllm_hip",
-            "-Wl,-rpath,$ORIGIN"]
-    o = _run(cmd)
-    if verbose and o.strip():
-        print(o)
-    return out
+    hdrs = [os.path.join(CSRC, "torch_bindings.h"), os.path.join(ROOT, "include", "lvllm_hip.h")]
+    jobs, outs = [], []
+    for c in components:
+        src = os.path.join(CSRC, COMPONENTS[c][2])
+        name = COMPONENTS[c][3]
+        out = os.path.join(LIBDIR, name)
+        outs.append(out)
+        if not force and not _newer(out, [src] + hdrs):
+            continue
+        cmd = ["g++", "-O2", "-std=c++17", "-fPIC", "-shared", "-D__HIP_PLATFORM_AMD__=1",
+               "-DUSE_ROCM=1", "-DTORCH_EXTENSION_NAME=" + name[:-3],
+               "-D_GLIBCXX_USE_CXX11_ABI=%d" % int(torch._C._GLIBCXX_USE_CXX11_ABI),
+               "-Wno-deprecated-declarations"]
+        for i in incs:
+            cmd += ["-I", i]
+        jobs.append(cmd + [src, "-o", out, "-L", torch_lib, "-L", LIBDIR,
+                           "-ltorch", "-ltorch_cpu", "-ltorch_hip", "-lc10", "-lc10_hip"] +
+                    (["-llvllm_hip"] if c == "full" else []) + ["-llvllm_base", "-Wl,-rpath,$ORIGIN"])
+    if jobs:
+        with ThreadPoolExecutor(max_workers=len(jobs)) as ex:
+            for o in ex.map(_run, jobs):
+                if verbose and o.strip():
+                    print(o)
+    return outs
 
 
-def build_all(verbose=False):
-    lib = build_kernels(verbose)
-    ext = build_torch_bindings(verbose)
-    return lib, ext
+def build_all(components=("base", "full"), verbose=False, force=False):
+    """(kernel libraries, torch extensions) of the components, built where they are missing or older than a source
+    (`force`: all of them)."""
+    return build_kernels(components, verbose, force), build_torch_bindings(components, verbose, force)
 
 
 if __name__ == "__main__":

@@ -150,6 +150,42 @@ struct Vec16 {
   typename T::store_t v[N];
 };
 
+// 4 consecutive elements <-> floats (the address is a multiple of 4 elements)
+template <typename T>
+__device__ __forceinline__ void load4(const typename T::store_t* p, float (&v)[4]) {
+  if constexpr (sizeof(typename T::store_t) == 4) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+  } else {
+    const uint2 a = *reinterpret_cast<const uint2*>(p);
+    v[0] = T::to_float((uint16_t)a.x); v[1] = T::to_float((uint16_t)(a.x >> 16));
+    v[2] = T::to_float((uint16_t)a.y); v[3] = T::to_float((uint16_t)(a.y >> 16));
+  }
+}
+template <typename T>
+__device__ __forceinline__ void store4(typename T::store_t* p, const float (&v)[4]) {
+  if constexpr (sizeof(typename T::store_t) == 4) {
+    *reinterpret_cast<float4*>(p) = float4{v[0], v[1], v[2], v[3]};
+  } else {
+    uint2 a;
+    a.x = (uint32_t)T::from_float(v[0]) | ((uint32_t)T::from_float(v[1]) << 16);
+    a.y = (uint32_t)T::from_float(v[2]) | ((uint32_t)T::from_float(v[3]) << 16);
+    *reinterpret_cast<uint2*>(p) = a;
+  }
+}
+
+// The sequence that owns `row` of a step's token batch: the s with query_start_loc[s] <= row < query_start_loc[s + 1],
+// num_seqs for rows past the last sequence (padding).  Sequences without tokens own nothing.
+__device__ __forceinline__ int find_seq(const int32_t* __restrict__ query_start_loc, int num_seqs, int row) {
+  int lo = 0, hi = num_seqs;  // first s with query_start_loc[s + 1] > row
+  while (lo < hi) {
+    const int mid = (lo + hi) >> 1;
+    if (query_start_loc[mid + 1] > row) hi = mid;
+    else lo = mid + 1;
+  }
+  return lo;
+}
+
 __device__ inline float wave_sum(float v) {
 #pragma unroll
   for (int m = 32; m >= 1; m >>= 1) v += __shfl_xor(v, m);

@@ -1,0 +1,82 @@
+// Helpers shared by the torch op registrations (torch_bindings_base.cpp, torch_bindings.cpp): dtype codes, argument
+// checks, the current stream, the C-ABI's error string as an exception.  Host-only C++.
+#pragma once
+#include <Python.h>
+#include <ATen/hip/impl/HIPGuardImplMasqueradingAsCUDA.h>
+#include <ATen/hip/impl/HIPStreamMasqueradingAsCUDA.h>
+#include <torch/all.h>
+#include <torch/library.h>
+
+#include <optional>
+#include <string>
+#include <vector>
+
+#include "lvllm_hip.h"
+
+namespace {
+
+[[maybe_unused]] int dtype_code(const torch::Tensor& t, const char* what) {
+  switch (t.scalar_type()) {
+    case at::ScalarType::Float: return LVLLM_F32;
+    case at::ScalarType::Half: return LVLLM_F16;
+    case at::ScalarType::BFloat16: return LVLLM_BF16;
+    default: TORCH_CHECK(false, what, ": unsupported dtype ", t.scalar_type());
+  }
+}
+
+// kv_cache_dtype strings: csrc/quantization/fp8/amd/quant_utils.cuh:547-573
+[[maybe_unused]] int kv_dtype_code(const std::string& s) {
+  if (s == "auto") return LVLLM_KV_AUTO;
+  if (s == "fp8" || s == "fp8_e4m3") return LVLLM_KV_FP8_E4M3;
+  TORCH_CHECK(false, "Unsupported data type of kv cache: ", s);
+}
+
+// "auto": the cache holds the query's element type; "fp8": one byte per element
+[[maybe_unused]] void check_cache_dtype(const torch::Tensor& cache, const torch::Tensor& like, int kv_code, const char* op) {
+  if (kv_code == LVLLM_KV_AUTO) {
+    TORCH_CHECK(cache.scalar_type() == like.scalar_type(), op, ": kv_cache_dtype 'auto' needs a cache of dtype ",
+                like.scalar_type(), ", got ", cache.scalar_type());
+  } else {
+    TORCH_CHECK(cache.element_size() == 1, op, ": kv_cache_dtype 'fp8' needs a one-byte cache dtype, got ",
+                cache.scalar_type());
+  }
+}
+
+// Bytes the kernels may touch behind key_cache.data_ptr() / value_cache.data_ptr() (the smaller of the two):
+// the C-ABI clamps block numbers / skips slots beyond it instead of following them out of the allocation.
+[[maybe_unused]] int64_t cache_extent_bytes(const torch::Tensor& key_cache, const torch::Tensor& value_cache) {
+  auto bytes = [](const torch::Tensor& t) {
+    return t.dim() == 0 ? (int64_t)0 : t.size(0) * t.stride(0) * (int64_t)t.element_size();
+  };
+  const int64_t k = bytes(key_cache), v = bytes(value_cache);
+  return k < v ? k : v;
+}
+
+// A paged cache as the kernels address it: every block dense ([KVH, D/x, BS, x] or [KVH, D, BS] contiguous), blocks
+// stride(0) elements apart -- the dense product, or more when the allocation pads its blocks.
+[[maybe_unused]] bool blocks_are_dense(const torch::Tensor& t) {
+  if (t.dim() < 2) return t.is_contiguous();
+  int64_t expect = 1;
+  for (int64_t d = t.dim() - 1; d >= 1; --d) {
+    if (t.size(d) != 1 && t.stride(d) != expect) return false;
+    expect *= t.size(d);
+  }
+  return t.stride(0) >= expect;
+}
+
+[[maybe_unused]] void* current_stream(const torch::Tensor& t) {
+  return (void*)c10::hip::getCurrentHIPStreamMasqueradingAsCUDA(t.device().index()).stream();
+}
+
+[[maybe_unused]] void check(int rc) { TORCH_CHECK(rc == 0, lvllm_last_error()); }
+
+#define LV_CHECK_DEVICE(t) TORCH_CHECK((t).is_cuda(), #t " must be a GPU tensor")
+
+// ---- the W8A8 decode step with activations quantised ONCE, by their producer (include/lvllm_hip.h: *_quant entries,
+// lvllm_skinny_gemm_w8a8_q): every op below is bit-identical to the op it stands for followed by / preceded by
+// static_scaled_fp8_quant
+[[maybe_unused]] void check_q_scale(const torch::Tensor& s, const char* op) {
+  TORCH_CHECK(s.is_cuda() && s.scalar_type() == at::kFloat && s.numel() == 1, op, ": one float32 scale on the device");
+}
+
+}  // namespace

@@ -43,6 +43,24 @@ class ModelConfig:
     # the projections as fp8 (bit-identical to quantising inside every projection; off = A/B runs)
     fp8_activations_once: bool = True
 
+    architecture: str = "RotaryDecoder"   # engine/registry.py
+
+    def kv_cache_specs(self):
+        """None: every layer caches num_key_value_heads x head_dim keys and values (two equal planes)."""
+        return None
+
+    def state_specs(self):
+        """Per layer the fp32 tensors a sequence carries besides its cache: none."""
+        return None
+
+    def step_activation_bytes(self, rows: int) -> int:
+        """Upper bound of the activations one captured step of `rows` tokens keeps alive, all layers: hidden / residual /
+        normed rows, qkv, attention output, SwiGLU output, the fp32 split-K partials of the o / down projections."""
+        per_layer = rows * (4 * self.hidden_size + (self.num_attention_heads + 2 * self.num_key_value_heads) * self.head_dim
+                            + self.num_attention_heads * self.head_dim + self.intermediate_size) * 2
+        per_layer += 2 * 8 * rows * self.hidden_size * 4
+        return per_layer * self.num_hidden_layers
+
     @property
     def head_dim(self) -> int:
         return self.hidden_size // self.num_attention_heads
@@ -68,6 +86,9 @@ class CacheConfig:
     num_cpu_blocks: Optional[int] = None
     sliding_window: Optional[int] = None
     enable_prefix_caching: bool = False
+    # slots of per-sequence recurrent state (models with state_specs; block_manager/state_slots.py).  None: the engine
+    # makes one for every sequence its steps in flight can hold
+    num_state_slots: Optional[int] = None
     # bytes between the end of a block and the start of the next in each K / V plane (a multiple of 16).  Blocks a power
     # of two apart (32 KiB for 8 kv heads x 128 x 16 tokens of bf16) put tile t of EVERY sequence of a freshly
     # filled cache on the same HBM channels -- sequence i's blocks start i x 2 MiB in -- and the decode attention

@@ -35,16 +35,19 @@ class DecodeGraph:
         # the five static inputs are views of one device buffer, mirrored by one pinned staging
         # buffer on the host: a step's inputs arrive with a single copy (DecodeStepArrays)
         B, W = batch_size, max_blocks_per_seq
-        o_ids, o_pos, o_slot, o_len, o_bt, o_state, total = DecodeStepArrays.layout(B, W)
+        o_ids, o_pos, o_slot, o_len, o_bt, o_state, o_rec, total = DecodeStepArrays.layout(B, W)
         self.packed = torch.zeros(total, dtype=torch.uint8, device=dev)
         self.input_ids = self.packed[o_ids:o_pos].view(torch.int64)
         self.positions = self.packed[o_pos:o_slot].view(torch.int64)
         self.slot_mapping = self.packed[o_slot:o_len].view(torch.int64)
         self.seq_lens = self.packed[o_len:o_bt].view(torch.int32)
         self.block_tables = self.packed[o_bt:o_state].view(torch.int32).view(B, W)
-        self.state_slots = self.packed[o_state:].view(torch.int32)
+        self.state_slots = self.packed[o_state:o_rec].view(torch.int32)
+        self.recurrent_slots = self.packed[o_rec:].view(torch.int32)
+        self.query_start_loc = torch.arange(B + 1, dtype=torch.int32, device=dev)
         self.slot_mapping.fill_(-1)
         self.state_slots.fill_(-1)
+        self.recurrent_slots.fill_(-1)
         self.host = torch.zeros(total, dtype=torch.uint8, pin_memory=dev.type == "cuda")
         self.staging = DecodeStepArrays(B, W, block_size, self.host.numpy())
         # pinned landing buffers of the sampled tokens: a result is read by the host right after its step
@@ -97,8 +100,9 @@ class DecodeGraph:
             slot_mapping=self.slot_mapping, seq_lens=None, seq_lens_tensor=self.seq_lens,
             max_query_len=1, max_prefill_seq_len=0,
             max_decode_seq_len=self.max_blocks_per_seq * self.block_size,
-            query_start_loc=None, seq_start_loc=None, context_lens_tensor=None,
-            block_tables=self.block_tables, use_cuda_graph=True, decode_scratch=self._scratch)
+            query_start_loc=self.query_start_loc, seq_start_loc=None, context_lens_tensor=None,
+            block_tables=self.block_tables, use_cuda_graph=True, decode_scratch=self._scratch,
+            state_slots=self.recurrent_slots)
 
     def _step(self):
         hidden = self.model.forward(self.input_ids, self.positions, self.kv_caches, self._metadata())
@@ -122,9 +126,13 @@ class DecodeGraph:
             self.hidden, self.next_tokens = self._step()
         torch.cuda.synchronize()
 
-    def load(self, input_ids, positions, slot_mapping, block_tables, seq_lens, state_slots=None) -> None:
+    def load(self, input_ids, positions, slot_mapping, block_tables, seq_lens, state_slots=None,
+             recurrent_slots=None) -> None:
         """Copy one step's inputs (device or pinned-host tensors) into the static buffers."""
         n = input_ids.shape[0]
+        self.recurrent_slots.fill_(-1)
+        if recurrent_slots is not None:
+            self.recurrent_slots[:n].copy_(recurrent_slots, non_blocking=True)
         self.state_slots.fill_(-1)
         if state_slots is not None:
             self.state_slots[:n].copy_(state_slots, non_blocking=True)

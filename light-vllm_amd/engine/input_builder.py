@@ -38,6 +38,7 @@ class InterDataForSeqGroup:
         self.context_lens = [0] * n
         self.curr_sliding_window_blocks = [0] * n
         self.prefix_cache_hit = False
+        self.state_slots: Optional[Dict[int, int]] = None  # models with recurrent state
 
 
 @dataclass
@@ -68,6 +69,7 @@ class WorkerInput:
     blocks_to_swap_in: torch.Tensor
     blocks_to_swap_out: torch.Tensor
     blocks_to_copy: torch.Tensor
+    state_copies: List[tuple] = field(default_factory=list)  # (source, destination) slots of forked sequences
 
 
 @dataclass
@@ -98,6 +100,7 @@ class ModelInputBuilder:
         d = InterDataForSeqGroup(request_id=meta.request_id, seq_ids=seq_ids, is_prompt=meta.is_prompt,
                                  block_tables=meta.block_tables,
                                  computed_block_nums=meta.computed_block_nums)
+        d.state_slots = getattr(meta, "state_slots", None)
         for i, seq_id in enumerate(seq_ids):
             data = meta.seq_data[seq_id]
             seq_len = data.get_len()
@@ -180,7 +183,7 @@ class ModelInputBuilder:
         return WorkerInput(num_seq_groups=len(out.seq_group_metadata_list),
                            blocks_to_swap_in=pairs(out.blocks_to_swap_in),
                            blocks_to_swap_out=pairs(out.blocks_to_swap_out),
-                           blocks_to_copy=pairs(out.blocks_to_copy))
+                           blocks_to_copy=pairs(out.blocks_to_copy), state_copies=out.state_copies)
 
     def __call__(self, out: SchedulerOutput) -> ExecuteInput:
         return ExecuteInput(worker_input=self.prepare_worker_input(out),
@@ -230,7 +233,7 @@ class DecodeStepArrays:
         self.nbytes = self.layout(B, W)[-1]
         buf = np.zeros(self.nbytes, dtype=np.uint8) if buffer is None else buffer
         assert buf.dtype == np.uint8 and buf.size == self.nbytes
-        o_ids, o_pos, o_slot, o_len, o_bt, o_state, _ = self.layout(B, W)
+        o_ids, o_pos, o_slot, o_len, o_bt, o_state, o_rec, _ = self.layout(B, W)
         self.buffer = buf
         self.input_ids = buf[o_ids:o_pos].view(np.int64)
         self.positions = buf[o_pos:o_slot].view(np.int64)
@@ -238,17 +241,20 @@ class DecodeStepArrays:
         self.seq_lens = buf[o_len:o_bt].view(np.int32)
         self.block_tables = buf[o_bt:o_state].view(np.int32).reshape(B, W)
         # sampler state slot of each row (device_sampler.py): -1 = plain greedy; read by the sampling kernel only
-        self.state_slots = buf[o_state:].view(np.int32)
+        self.state_slots = buf[o_state:o_rec].view(np.int32)
+        # slot of each row's recurrent state (models that have one): -1 = padding, nothing read or stored
+        self.recurrent_slots = buf[o_rec:].view(np.int32)
         self.slot_mapping[:] = -1
         self.state_slots[:] = -1
+        self.recurrent_slots[:] = -1
         self._rows: List[Optional[List[int]]] = [None] * B  # the table each row holds
         self._arange = np.arange(B)
 
     @staticmethod
     def layout(B: int, W: int):
         """Byte offsets of (input_ids i64[B], positions i64[B], slot_mapping i64[B], seq_lens i32[B],
-        block_tables i32[B, W], sampler state slots i32[B]) and the total size."""
-        return 0, 8 * B, 16 * B, 24 * B, 28 * B, 28 * B + 4 * B * W, 32 * B + 4 * B * W
+        block_tables i32[B, W], sampler state slots i32[B], recurrent state slots i32[B]) and the total size."""
+        return 0, 8 * B, 16 * B, 24 * B, 28 * B, 28 * B + 4 * B * W, 32 * B + 4 * B * W, 36 * B + 4 * B * W
 
     @staticmethod
     def eligible(metas, worker_lists_empty: bool, sliding_window) -> bool:
@@ -300,6 +306,9 @@ class DecodeStepArrays:
         self.state_slots[:] = -1
         if state_slots is not None:
             self.state_slots[:n] = state_slots
+        self.recurrent_slots[:] = -1
+        if metas and getattr(metas[0], "state_slots", None) is not None:
+            self.recurrent_slots[:n] = [m.state_slots[sid] for m, sid in zip(metas, seq_ids)]
         return seq_ids
 
 

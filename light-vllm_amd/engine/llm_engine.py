@@ -6,6 +6,7 @@ flight, legal because scheduled groups are marked busy).
 One engine = one GPU (replica).  Multi-GPU serving replicates engines, one process per GPU,
 with no collective on the kernel path.
 """
+import dataclasses
 import queue
 import threading
 import time
@@ -14,12 +15,11 @@ from typing import Dict, List, Optional, Tuple
 
 import torch
 
-from ..attention.backend import PagedAttnBackend
 from .cache_engine import CacheEngine
 from .config import CacheConfig, ModelConfig, SchedulerConfig
 from .graph_runner import DecodeGraphPool
 from .input_builder import ExecuteInput, ModelInputBuilder
-from .model import DecoderModel
+from .registry import model_entry
 from .scheduler import DecodingScheduler, SchedulerOutput
 from .sequence import Sequence, SequenceGroup, SequenceStatus
 
@@ -66,16 +66,19 @@ class Worker:
         self.model_config = model_config
         self.cache_config = cache_config
         impl_cls = attn_backend.get_impl_cls()
-        self.attn_impl = impl_cls(model_config.num_attention_heads, model_config.head_dim,
-                                  model_config.head_dim ** -0.5, model_config.num_key_value_heads,
-                                  None, cache_config.sliding_window, cache_config.cache_dtype,
-                                  decode_version=decode_version)
+        if model_config.kv_cache_specs() is not None:  # sizes differ per layer: they come with the caches
+            self.attn_impl = impl_cls()
+        else:
+            self.attn_impl = impl_cls(model_config.num_attention_heads, model_config.head_dim,
+                                      model_config.head_dim ** -0.5, model_config.num_key_value_heads,
+                                      None, cache_config.sliding_window, cache_config.cache_dtype,
+                                      decode_version=decode_version)
         if self.device.type == "cuda":  # free memory before the weights (gpu_worker.py:78-80)
             torch.cuda.empty_cache()
             self.init_gpu_memory = torch.cuda.mem_get_info(self.device)[0]
         else:
             self.init_gpu_memory = 0
-        self.model = DecoderModel(model_config, self.attn_impl, device, seed)
+        self.model = model_entry(model_config.architecture).model_cls()(model_config, self.attn_impl, device, seed)
         self.attn_backend = attn_backend
         self.cache_engine: Optional[CacheEngine] = None
         self.use_hip_graph = use_hip_graph
@@ -132,16 +135,27 @@ class Worker:
         from .sequence import SequenceData
         lens = self.profile_seq_lens(scheduler_config.max_num_batched_tokens, scheduler_config.max_num_seqs)
         metas = []
+        # a model over caches of its own kind runs the profile through a throw-away cache of just these prompts, with
+        # no state slots (nothing is stored); any other one runs without a cache
+        caches, at, bs = None, 0, self.cache_config.block_size
+        own_caches = self.model_config.kv_cache_specs() is not None
         for gid, n in enumerate(lens):
             if n == 0:
                 continue
+            nb = (n + bs - 1) // bs
             metas.append(SequenceGroupMetadata(request_id=str(gid), is_prompt=True,
-                                               seq_data={gid: SequenceData([0] * n)}, block_tables=None,
-                                               do_sample=True, token_chunk_size=n, computed_block_nums=[]))
+                                               seq_data={gid: SequenceData([0] * n)},
+                                               block_tables={gid: list(range(at, at + nb))} if own_caches else None,
+                                               do_sample=True, token_chunk_size=n, computed_block_nums=[],
+                                               state_slots={gid: -1} if own_caches else None))
+            at += nb
+        if own_caches:
+            cc = dataclasses.replace(self.cache_config, num_gpu_blocks=at, num_cpu_blocks=0, num_state_slots=1)
+            caches = CacheEngine(cc, self.model_config, self.attn_backend, self.device).model_caches()
         builder = ModelInputBuilder(scheduler_config, self.cache_config, self.attn_backend,
                                     self.cache_config.sliding_window)
         mi = builder.prepare_model_input(metas).to(self.device)
-        hidden = self.model.forward(mi.input_tokens, mi.input_positions, None, mi.attn_metadata)
+        hidden = self.model.forward(mi.input_tokens, mi.input_positions, caches, mi.attn_metadata)
         rows = torch.tensor(mi.sample_indices, dtype=torch.long, device=self.device)
         logits = self.model.compute_logits(hidden[rows]).float()
         n = logits.shape[0]
@@ -159,14 +173,16 @@ class Worker:
         capped at the 64 rows the decode path takes) twice over (a second captured size)."""
         if not self.use_hip_graph:
             return 0
-        cfg = self.model_config
         rows = min(scheduler_config.max_num_seqs, 64)
-        e = 2
-        per_layer = rows * (4 * cfg.hidden_size + (cfg.num_attention_heads + 2 * cfg.num_key_value_heads) * cfg.head_dim
-                            + cfg.num_attention_heads * cfg.head_dim + cfg.intermediate_size) * e
-        per_layer += 2 * 8 * rows * cfg.hidden_size * 4
-        step = per_layer * cfg.num_hidden_layers + rows * 4096 * 16 + (8 << 20)
+        step = self.model_config.step_activation_bytes(rows) + rows * 4096 * 16 + (8 << 20)
         return 2 * self.num_slots * step
+
+    def recurrent_state_slots(self, scheduler_config: SchedulerConfig) -> Optional[int]:
+        """Slots of recurrent state: the configured number, else one for every sequence the steps in flight can hold
+        (None: the model carries no state)."""
+        if self.model_config.state_specs() is None:
+            return None
+        return self.cache_config.num_state_slots or scheduler_config.max_num_seqs * self.num_slots
 
     def sampler_state_slots(self, scheduler_config: SchedulerConfig) -> int:
         """State slots of the device sampler: every sequence of every step in flight plus one step being built."""
@@ -200,7 +216,9 @@ class Worker:
                                           self.cache_config.gpu_memory_utilization, scheduler_config.scheduling,
                                           block_bytes, self.cache_config.swap_space_bytes,
                                           self.graph_reserve_bytes(scheduler_config)
-                                          + self.sampler_reserve_bytes(scheduler_config))
+                                          + self.sampler_reserve_bytes(scheduler_config)
+                                          + CacheEngine.get_state_bytes(self.model_config,
+                                                                        self.recurrent_state_slots(scheduler_config) or 0))
         self.profile = dict(total=total, init_free=self.init_gpu_memory, free_after_load=free_after_load,
                             free_after_profile=free_after_profile, block_bytes=block_bytes)
         import gc
@@ -214,13 +232,38 @@ class Worker:
         self.cache_engine = CacheEngine(self.cache_config, self.model_config, self.attn_backend, self.device)
         if self.use_hip_graph:
             max_blocks = (self.max_model_len + self.cache_config.block_size - 1) // self.cache_config.block_size
-            self.graph_pools = [DecodeGraphPool(self.model, self.cache_engine.gpu_cache, max_blocks,
+            self.graph_pools = [DecodeGraphPool(self.model, self.cache_engine.model_caches(), max_blocks,
                                                 self.cache_config.block_size, self.device)
                                 for _ in range(self.num_slots)]
 
     def _slots_tensor(self, slots: List[int]) -> torch.Tensor:
         t = torch.tensor(slots, dtype=torch.int32)
         return (t.pin_memory() if self.device.type == "cuda" else t).to(self.device, non_blocking=True)
+
+    def _move_cache(self, wi) -> None:
+        """Block swaps and copies, and state copies of forked sequences, that come before a step's forward."""
+        ce = self.cache_engine
+        if wi.blocks_to_swap_in.numel() > 0:
+            ce.swap_in(wi.blocks_to_swap_in)
+        if wi.blocks_to_swap_out.numel() > 0:
+            ce.swap_out(wi.blocks_to_swap_out)
+        if wi.blocks_to_copy.numel() > 0:
+            ce.copy(wi.blocks_to_copy.to(self.device, non_blocking=True))
+        if wi.state_copies:
+            ce.copy_state(wi.state_copies)
+
+    def _forward(self, mi) -> torch.Tensor:
+        mi.to(self.device)
+        return self.model.forward(mi.input_tokens, mi.input_positions, self.cache_engine.model_caches(), mi.attn_metadata)
+
+    @torch.inference_mode()
+    def execute_logits(self, execute_input: ExecuteInput, rows: List[int]) -> Optional[torch.Tensor]:
+        """The eager step without sampling: the logits of the given rows of its token batch (None: none asked for)."""
+        self._move_cache(execute_input.worker_input)
+        hidden = self._forward(execute_input.model_input)
+        if not rows:
+            return None
+        return self.model.compute_logits(hidden[torch.tensor(rows, dtype=torch.long, device=self.device)])
 
     @torch.inference_mode()
     def execute(self, execute_input: ExecuteInput, slot: int = 0, state_slots=None, logprob_rows=None) -> ExecuteOutput:
@@ -231,14 +274,8 @@ class Worker:
         log-probabilities (SamplingParams.logprobs): the step takes the general path, the adjusted logits of its
         sampled rows are restated in torch (sampling.SamplingBatch: the stages the device sampler applies) and the
         sample half of the reference's get_logprobs is read off them (sampler.py:726-990)."""
-        wi, mi = execute_input.worker_input, execute_input.model_input
-        ce = self.cache_engine
-        if wi.blocks_to_swap_in.numel() > 0:
-            ce.swap_in(wi.blocks_to_swap_in)
-        if wi.blocks_to_swap_out.numel() > 0:
-            ce.swap_out(wi.blocks_to_swap_out)
-        if wi.blocks_to_copy.numel() > 0:
-            ce.copy(wi.blocks_to_copy.to(self.device, non_blocking=True))
+        mi = execute_input.model_input
+        self._move_cache(execute_input.worker_input)
         if mi.input_tokens is None:
             return ExecuteOutput(None, [])
         md = mi.attn_metadata
@@ -255,7 +292,8 @@ class Worker:
                 for r, sl in zip(mi.sample_indices, row_slots):
                     full[r] = sl
                 per_row = self._slots_tensor(full)
-            g.load(mi.input_tokens, mi.input_positions, md.slot_mapping, md.block_tables, md.seq_lens_tensor, per_row)
+            g.load(mi.input_tokens, mi.input_positions, md.slot_mapping, md.block_tables, md.seq_lens_tensor, per_row,
+                   md.state_slots)
             tokens = g.replay()[:n]
             if len(mi.sample_indices) != n:
                 tokens = tokens[torch.tensor(mi.sample_indices, dtype=torch.long, device=self.device)]
@@ -269,8 +307,7 @@ class Worker:
                    md.query_start_loc, mi.sample_indices)
             tokens = g.replay()[:len(mi.sample_indices)]
         else:
-            mi.to(self.device)
-            hidden = self.model.forward(mi.input_tokens, mi.input_positions, ce.gpu_cache, md)
+            hidden = self._forward(mi)
             hidden_all = hidden
             if len(mi.sample_indices) != hidden.shape[0]:
                 hidden = hidden[torch.tensor(mi.sample_indices, dtype=torch.long, device=self.device)]
@@ -327,7 +364,6 @@ class Worker:
         but no penalty (sampling_metadata.py:447-456), log_softmax, then {next prompt token: (logprob, rank)} + the n
         most likely tokens per position.  `logprob_rows[seq id]["prompt_rows"]` = (first row of the chunk in the step's
         token batch, number of such positions, their next tokens)."""
-        import dataclasses
         from ..sampling import SamplingBatch, sample_logprobs
         out: Dict[int, List[dict]] = {}
         for sid, r in logprob_rows.items():
@@ -401,7 +437,12 @@ class LLMEngine:
         self.model_config, self.cache_config, self.scheduler_config = model_config, cache_config, scheduler_config
         self.device = torch.device(device)
         torch.cuda.set_device(self.device)
-        self.attn_backend = PagedAttnBackend()
+        self.attn_backend = model_entry(model_config.architecture).backend_cls()()
+        if model_config.state_specs() is not None:
+            if cache_config.enable_prefix_caching:
+                raise ValueError("prefix caching needs the state at a block's end, which a recurrent model does not keep")
+            if cache_config.cache_dtype != "auto" or cache_config.sliding_window is not None:
+                raise ValueError("hybrid decoders cache in the model's dtype, without a sliding window")
         # (multi-step decode over the prefix-caching allocator: the reference's v2 manager under lookahead is replayed
         # bit for bit -- tests/golden/block_manager_v2_cached_lookahead*.json, scheduler_lookahead_prefix_cache_v2.json)
         # steps in flight run on separate streams (a stream per task, core/executor.py:62-93), so
@@ -411,7 +452,7 @@ class LLMEngine:
         self.num_slots = (max(1, scheduler_config.max_num_on_the_fly)
                           if scheduler_config.scheduling in ("simple_async", "async", "double_buffer") else 1)
         # chunked prefill with a token budget the decode GEMM takes (<= 64 rows): mixed steps replay a graph
-        mixed = (scheduler_config.chunked_prefill_enabled and scheduler_config.max_num_batched_tokens <= 64
+        mixed = (model_config.state_specs() is None and scheduler_config.chunked_prefill_enabled and scheduler_config.max_num_batched_tokens <= 64
                  and cache_config.sliding_window is None and model_config.fuse_decode_ops
                  and cache_config.block_size in (16, 32)
                  and (cache_config.cache_dtype == "auto" or model_config.head_dim % 64 == 0))
@@ -428,6 +469,7 @@ class LLMEngine:
         gemm_wgs = scheduler_config.gemm_workgroups or (128 if concurrent else 256)
         self.gemm_workgroups = gemm_wgs
         torch.ops._C_amd.set_tuning("gemm_workgroups", gemm_wgs)
+        cache_config.num_state_slots = self.worker.recurrent_state_slots(scheduler_config)
         num_gpu, num_cpu = cache_config.num_gpu_blocks, cache_config.num_cpu_blocks
         if num_gpu is None:
             num_gpu, auto_cpu = self.worker.determine_num_available_blocks(scheduler_config)
@@ -485,6 +527,14 @@ class LLMEngine:
             with torch.cuda.stream(self.streams[slot]):
                 pool.get(batch_size)
         torch.cuda.synchronize(self.device)
+
+    @classmethod
+    def from_pretrained(cls, model_dir: str, dtype: torch.dtype = torch.bfloat16, cache_config: Optional[CacheConfig] = None,
+                        scheduler_config: Optional[SchedulerConfig] = None, **kwargs) -> "LLMEngine":
+        """An engine for a model folder (config.json, model.safetensors), by the registry's entry for its architecture."""
+        from .registry import load_model_config
+        return cls(load_model_config(model_dir, dtype), cache_config or CacheConfig(), scheduler_config or SchedulerConfig(),
+                   **kwargs)
 
     # ---- requests ----
     def add_request(self, request_id: str, prompt_token_ids: List[int], max_tokens: Optional[int] = 16,
@@ -698,7 +748,7 @@ class LLMEngine:
                                        logprob_rows=logprob_rows)
         if self.fast_decode_inputs:
             from .input_builder import DecodeStepArrays, MixedStepArrays
-            plain = not (sched.blocks_to_swap_in or sched.blocks_to_swap_out or sched.blocks_to_copy)
+            plain = not (sched.blocks_to_swap_in or sched.blocks_to_swap_out or sched.blocks_to_copy or sched.state_copies)
             metas = sched.seq_group_metadata_list
             if DecodeStepArrays.eligible(metas, plain, self.cache_config.sliding_window):
                 out = self.worker.execute_decode(metas, slot, self._burst_steps(sched), state_slots)
@@ -805,7 +855,7 @@ class LLMEngine:
             # with prefix caching (a later prompt reads blocks an earlier step is still filling; blocks are
             # marked computed at schedule time, scheduler.py:924-926) is ordered on the device instead: it waits
             # for every step in flight, and every later step waits for it.  No host wait.
-            moves = bool(sched.blocks_to_swap_in or sched.blocks_to_swap_out or sched.blocks_to_copy)
+            moves = bool(sched.blocks_to_swap_in or sched.blocks_to_swap_out or sched.blocks_to_copy or sched.state_copies)
             fence = moves or self.cache_config.enable_prefix_caching
             with torch.cuda.stream(stream):
                 if self._fence is not None:
@@ -914,6 +964,7 @@ class LLMEngine:
         from ..paged_attn import PagedAttention
         gen = torch.Generator(device=self.device).manual_seed(seed)
         cfg = self.model_config
+        own_caches = cfg.kv_cache_specs() is not None
         sched = self.scheduler
         admitted: List[SequenceGroup] = []
         while sched.waiting:
@@ -921,7 +972,7 @@ class LLMEngine:
             if sched.block_manager.can_allocate(g).name != "OK":
                 break
             sched.waiting.popleft()
-            sched.block_manager.allocate(g)
+            sched._allocate(g)
             for seq in g.get_seqs(status=SequenceStatus.WAITING):
                 seq.status = SequenceStatus.RUNNING
             sched.running.append(g)
@@ -934,7 +985,13 @@ class LLMEngine:
                                  self.cache_config.block_size, table)
         slots = torch.tensor(slot_mapping, dtype=torch.int64, device=self.device)
         T = slots.numel()
-        for kv in self.worker.cache_engine.gpu_cache:
+        if own_caches:  # every block of the cache and every state slot
+            for kv in self.worker.cache_engine.gpu_cache:
+                kv.normal_(0.0, 0.5, generator=gen)
+            for layer in self.worker.cache_engine.state:
+                for t in layer.values():
+                    t.normal_(0.0, 0.5, generator=gen)
+        for kv in () if own_caches else self.worker.cache_engine.gpu_cache:
             kc, vc = PagedAttention.split_kv_cache(kv, cfg.num_key_value_heads, cfg.head_dim)
             for s0 in range(0, T, 8192):
                 n = min(8192, T - s0)

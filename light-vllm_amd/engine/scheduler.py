@@ -20,6 +20,7 @@ from dataclasses import dataclass, field
 from typing import Deque, Dict, Iterable, List, Optional, Set, Tuple
 
 from ..block_manager.interfaces import AllocStatus, BlockSpaceManager
+from ..block_manager.state_slots import StateSlotManager
 from ..block_manager.v1 import BlockSpaceManagerV1
 from .config import CacheConfig, SchedulerConfig
 from .sequence import Sequence, SequenceData, SequenceGroup, SequenceStatus
@@ -87,6 +88,7 @@ class SequenceGroupMetadata:
     do_sample: bool
     token_chunk_size: int
     computed_block_nums: List[int]
+    state_slots: Optional[Dict[int, int]] = None  # {seq id: slot of its recurrent state} (models that have one)
 
 
 @dataclass
@@ -102,6 +104,7 @@ class SchedulerOutput:
     running_queue_size: int
     preempted: int
     seq_group_metadata_list: List[SequenceGroupMetadata] = field(default_factory=list)
+    state_copies: List[Tuple[int, int]] = field(default_factory=list)  # forked sequences: (source, destination) slot
 
     def is_empty(self) -> bool:
         return (not self.scheduled_seq_groups and not self.blocks_to_swap_in
@@ -122,6 +125,9 @@ class DecodingScheduler:
                                  num_cpu_blocks=cache_config.num_cpu_blocks or 0,
                                  sliding_window=cache_config.sliding_window,
                                  enable_caching=cache_config.enable_prefix_caching)
+        # recurrent state: one slot per admitted sequence, beside its blocks
+        self.state_slots = (StateSlotManager(cache_config.num_state_slots)
+                            if cache_config.num_state_slots is not None else None)
         self.waiting: Deque[SequenceGroup] = deque()
         self.running: Deque[SequenceGroup] = deque()
         self.swapped: Deque[SequenceGroup] = deque()
@@ -303,6 +309,8 @@ class DecodingScheduler:
                 q.popleft()
                 continue
             can_allocate = self.block_manager.can_allocate(seq_group)
+            if can_allocate == AllocStatus.OK and self.state_slots is not None:
+                can_allocate = self._can_take_state_slots(seq_group)
             if can_allocate == AllocStatus.LATER:
                 break
             if can_allocate == AllocStatus.NEVER:
@@ -316,7 +324,7 @@ class DecodingScheduler:
                                                               num_new_seqs=num_new_seqs):
                 break
             q.popleft()
-            self.block_manager.allocate(seq_group)
+            self._allocate(seq_group)
             for seq in waiting_seqs:
                 seq.status = SequenceStatus.RUNNING
             scheduled.append(ScheduledSequenceGroup(seq_group, num_new_tokens))
@@ -410,7 +418,8 @@ class DecodingScheduler:
                 metas.append(SequenceGroupMetadata(
                     request_id=g.request_id, is_prompt=False, seq_data={seq.seq_id: seq.data},
                     block_tables={seq.seq_id: bm.get_block_table(seq)}, do_sample=True,
-                    token_chunk_size=sched.token_chunk_size, computed_block_nums=[]))
+                    token_chunk_size=sched.token_chunk_size, computed_block_nums=[],
+                    state_slots=self._slots_of(seqs)))
                 continue
             seq_data: Dict[int, SequenceData] = {}
             block_tables: Dict[int, List[int]] = {}
@@ -431,19 +440,74 @@ class DecodingScheduler:
             metas.append(SequenceGroupMetadata(
                 request_id=g.request_id, is_prompt=g.is_prefill(), seq_data=seq_data,
                 block_tables=block_tables, do_sample=do_sample,
-                token_chunk_size=sched.token_chunk_size, computed_block_nums=common))
+                token_chunk_size=sched.token_chunk_size, computed_block_nums=common,
+                state_slots=self._slots_of(running)))
         if hooks:
             for sched in out.scheduled_seq_groups:
                 bm.mark_blocks_as_computed(sched.seq_group)
         out.seq_group_metadata_list = metas
+        if self.state_slots is not None:
+            out.state_copies = self.state_slots.take_copies()
         return out
+
+    def schedule_exact(self, entries: List[Tuple[SequenceGroup, int]]) -> SchedulerOutput:
+        """A step the caller composed instead of the policy (trace replay): each single-sequence group with the number of
+        its last tokens that are new.  Blocks and state slots are taken as the policies take them: on a waiting group's
+        first step, then for the tokens that were appended since.  Prompt portions come before single tokens of sequences
+        that have run (the batch order of every step), which may reorder the entries."""
+        waits = {g.request_id for g, _ in entries if g.seqs[0].status == SequenceStatus.WAITING}
+        portions = [(g, n) for g, n in entries if n > 1 or g.request_id in waits]
+        singles = [(g, n) for g, n in entries if not (n > 1 or g.request_id in waits)]
+        metas: List[SequenceGroupMetadata] = []
+        copies: List[Tuple[int, int]] = []
+        for is_prompt, group in ((True, portions), (False, singles)):
+            for g, n in group:
+                seq = g.seqs[0]
+                if g.request_id in waits:
+                    self._allocate(g)
+                    seq.status = SequenceStatus.RUNNING
+                    self.running.append(g)
+                else:
+                    copies.extend(self.block_manager.append_slots(seq, 0))
+                metas.append(SequenceGroupMetadata(
+                    request_id=g.request_id, is_prompt=is_prompt, seq_data={seq.seq_id: seq.data},
+                    block_tables={seq.seq_id: self.block_manager.get_block_table(seq)}, do_sample=True,
+                    token_chunk_size=n, computed_block_nums=[], state_slots=self._slots_of(g.seqs)))
+        return SchedulerOutput(
+            scheduled_seq_groups=[ScheduledSequenceGroup(g, n) for g, n in portions + singles],
+            num_prefill_groups=len(portions), num_batched_tokens=sum(n for _, n in entries), blocks_to_swap_in=[],
+            blocks_to_swap_out=[], blocks_to_copy=copies, ignored_seq_groups=[], num_lookahead_slots=0,
+            running_queue_size=len(self.running), preempted=0, seq_group_metadata_list=metas,
+            state_copies=self.state_slots.take_copies() if self.state_slots is not None else [])
+
+    # ---- blocks and, for models with recurrent state, the state slots that go with them ----
+    def _can_take_state_slots(self, seq_group: SequenceGroup) -> AllocStatus:
+        n = seq_group.get_max_num_running_seqs()
+        if n > self.state_slots.num_slots:
+            return AllocStatus.NEVER
+        return AllocStatus.OK if self.state_slots.can_allocate(n) else AllocStatus.LATER
+
+    def _allocate(self, seq_group: SequenceGroup) -> None:
+        self.block_manager.allocate(seq_group)
+        if self.state_slots is not None:
+            seq = seq_group.get_seqs(status=SequenceStatus.WAITING)[0]
+            self.state_slots.allocate(seq.seq_id, seq_group.get_max_num_running_seqs())
+
+    def _slots_of(self, seqs: List[Sequence]) -> Optional[Dict[int, int]]:
+        if self.state_slots is None:
+            return None
+        return {seq.seq_id: self.state_slots.slot_of(seq.seq_id) for seq in seqs}
 
     # ---- helpers shared with the output processor ----
     def fork_seq(self, parent_seq: Sequence, child_seq: Sequence) -> None:
         self.block_manager.fork(parent_seq, child_seq)
+        if self.state_slots is not None:
+            self.state_slots.fork(parent_seq.seq_id, child_seq.seq_id)
 
     def free_seq(self, seq: Sequence) -> None:
         self.block_manager.free(seq)
+        if self.state_slots is not None:
+            self.state_slots.free(seq.seq_id)
 
     def free_finished_request(self, request_ids: Iterable[str]) -> None:
         """Called once the outputs of a step were processed: finished groups leave the
