@@ -581,9 +581,6 @@ int lvllm_qk_norm_cache(void* q_out, void* key_cache, void* value_cache, const v
                         int kv_heads, int dim, int vdim, int kpad, int vpad, const int64_t* slot_mapping,
                         int64_t num_blocks, int block_size, int64_t k_block_stride, int64_t v_block_stride, int dtype,
                         void* stream);
-/* out[row, h * vdim + d] = T(attn[row, h, d] * sigmoid(gate[row, h]) * scale) */
-int lvllm_head_gate(void* out, int64_t out_stride, const void* attn, int64_t attn_head_stride, const void* gate,
-                    int64_t gate_stride, int rows, int heads, int vdim, float scale, int dtype, void* stream);
 /* out = T(o / rms(o over vdim) * weight * silu(gate) * scale) per head; o float [rows, heads, vdim]; weight float,
  * weight_head_stride apart between heads (0: shared) */
 int lvllm_head_norm_gate(void* out, int64_t out_stride, const float* o, const void* gate, int64_t gate_stride,
@@ -599,12 +596,31 @@ int lvllm_recurrent_scan(float* o, const void* q, const void* k, const void* v, 
                          int64_t v_stride, const float* log_decay, const float* bonus, float q_scale, float* state,
                          int64_t state_stride, const int32_t* state_slots, int num_slots, const int32_t* query_start_loc,
                          const int32_t* seq_lens, int num_seqs, int heads, int dk, int dv, int dtype, void* stream);
-/* Causal attention over the cache of lvllm_qk_norm_cache; q [rows, heads, kpad], out [rows, heads, vpad]. */
-int lvllm_head_attention(void* out, const void* q, const void* key_cache, const void* value_cache,
-                         const int32_t* block_tables, const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs,
-                         int rows, int heads, int kv_heads, int kpad, int vpad, int max_blocks, int block_size,
-                         int64_t num_blocks, float scale, int64_t k_block_stride, int64_t v_block_stride, int dtype,
-                         void* stream);
+/* A recurrent mixer in one call: decays (lvllm_log_decay), recurrence (lvllm_recurrent_scan), per-head norm and gate
+ * (lvllm_head_norm_gate).  max_query_len <= 1: every sequence s owns row s alone, one fused launch, no scratch.  Otherwise
+ * chunks of 16 tokens on fp32 MFMAs; o_scratch float [rows, heads, dv], workspace of
+ * lvllm_recurrent_mix_workspace_bytes. */
+int64_t lvllm_recurrent_mix_workspace_bytes(int rows, int num_seqs, int heads, int dk, int max_query_len);
+int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void* k, const void* v, int64_t q_stride,
+                        int64_t k_stride, int64_t v_stride, const void* u, int64_t u_stride, const float* a_t,
+                        const float* decay_bias, int rank, int kind, float inv_tau, const float* bonus, float q_scale,
+                        const void* gate, int64_t gate_stride, const float* norm_weight, int norm_head_stride, float eps,
+                        float out_scale, float* state, int64_t state_stride, const int32_t* state_slots, int num_slots,
+                        const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows, int heads, int dk,
+                        int dv, int max_query_len, float* o_scratch, void* workspace, int64_t workspace_bytes, int dtype,
+                        void* stream);
+/* Causal attention over the cache of lvllm_qk_norm_cache; q [rows, heads, kpad];
+ * out[row, h * vdim + d] = T(attention * sigmoid(gate[row, h]) * out_scale), gate null: no gate.  max_query_len and
+ * max_seq_len bound the step's query_len and seq_lens.  bf16 with block size 16, kpad in {64, 96, 128, 192, 256} and vpad
+ * in {32, 64, 96, 128, 192, 256} run on MFMAs; every other case on a plain fp32 body. */
+int64_t lvllm_head_attention_workspace_bytes(int rows, int num_seqs, int heads, int kv_heads, int kpad, int vpad,
+                                             int block_size, int max_seq_len, int dtype);
+int lvllm_head_attention(void* out, int64_t out_stride, const void* q, const void* key_cache, const void* value_cache,
+                         const void* gate, int64_t gate_stride, const int32_t* block_tables, const int32_t* seq_lens,
+                         const int32_t* query_start_loc, int num_seqs, int rows, int heads, int kv_heads, int kpad, int vpad,
+                         int vdim, int max_blocks, int block_size, int64_t num_blocks, float scale, float out_scale,
+                         int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len,
+                         void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -34,6 +34,8 @@ BASE_SOURCES = [
     "token_mix.hip",
     "recurrent.hip",
     "head_attention.hip",
+    "head_attention_prefill.hip",
+    "head_attention_decode.hip",
 ]
 FULL_SOURCES = [
     "layernorm.hip",

@@ -1,27 +1,10 @@
-// Causal softmax attention over a paged cache whose key and value sizes differ, without positions in the scores, for
-// gfx950.  Every sequence of a step is a chunk of query_len >= 1 new tokens that ends its context (their keys and
-// values are in the cache already); query t of a chunk sits at position seq_len - query_len + t and sees keys 0 .. there.
-//
-//   query       [rows, heads, kpad]                                (padding beyond dim is zero)
-//   key_cache   [num_blocks, kv_heads, kpad / x, block_size, x],   x = 16 / sizeof(T)
-//   value_cache [num_blocks, kv_heads, vpad, block_size]
-//   out         [rows, heads, vpad]
-//
-// Scores, softmax and accumulation are fp32.
+// Paged attention with unequal key and value sizes: the dispatcher and the body for 32-bit elements and for sizes outside
+// the MFMA bodies (see head_attention.h for the layouts).
 #include <float.h>
 
-#include "common.h"
+#include "head_attention.h"
 
 namespace lvllm {
-
-struct HeadAttnParams {
-  void* out;
-  const void *q, *k_cache, *v_cache;
-  const int32_t *block_tables, *seq_lens, *query_start_loc;
-  int num_seqs, rows, heads, kv_heads, kpad, vpad, max_blocks, block_size, max_block;
-  float scale;
-  int64_t k_block_stride, v_block_stride;
-};
 
 // One workgroup per (row, head): 256 keys per round, one per thread for the scores, then one value column per thread.
 template <typename T>
@@ -38,6 +21,11 @@ __global__ __launch_bounds__(256) void head_attention_simple_kernel(const HeadAt
   if (seq >= p.num_seqs) return;
   const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
   const int n_keys = p.seq_lens[seq] - qlen + (row - qbeg) + 1;
+  S* out = (S*)p.out + row * p.out_stride + (int64_t)head * p.vdim;
+  if (n_keys <= 0) {  // a padding row of a captured step
+    for (int d = threadIdx.x; d < p.vdim; d += 256) out[d] = T::from_float(0.f);
+    return;
+  }
   const int kvh = head / (p.heads / p.kv_heads);
   const int32_t* table = p.block_tables + (int64_t)seq * p.max_blocks;
   const S* q = (const S*)p.q + ((int64_t)row * p.heads + head) * p.kpad;
@@ -82,29 +70,78 @@ __global__ __launch_bounds__(256) void head_attention_simple_kernel(const HeadAt
     }
   }
   __syncthreads();
-  S* out = (S*)p.out + ((int64_t)row * p.heads + head) * p.vpad;
-  for (int d = threadIdx.x; d < p.vpad; d += 256) out[d] = T::from_float(sacc[d] / l);
+  const float f = gate_of<T>(p, row, head) / l;
+  for (int d = threadIdx.x; d < p.vdim; d += 256) out[d] = T::from_float(sacc[d] * f);
 }
 
 }  // namespace lvllm
 
 using namespace lvllm;
 
-extern "C" int lvllm_head_attention(void* out, const void* q, const void* key_cache, const void* value_cache,
+static bool mfma_size(int n, int least) {
+  return n == least || n == 64 || n == 96 || n == 128 || n == 192 || n == 256;
+}
+
+static bool takes_mfma(int kpad, int vpad, int block_size, int dtype) {
+  return dtype == LVLLM_BF16 && block_size == 16 && mfma_size(kpad, 64) && mfma_size(vpad, 32);
+}
+
+// Shares the keys of a sequence are cut into: enough workgroups to fill the chip, none of under 256 keys, and none at all
+// beside large prompt portions
+static int decode_shares(int rows, int num_seqs, int heads, int kv_heads, int max_seq_len) {
+  if (rows > 512) return 1;
+  const int wgs = num_seqs * kv_heads * ((heads / kv_heads + kDecodeCols - 1) / kDecodeCols);
+  int n = (1024 + wgs - 1) / wgs;
+  const int most = (max_seq_len + 255) / 256;
+  n = n < most ? n : most;
+  return n < 1 ? 1 : n > 64 ? 64 : n;
+}
+
+extern "C" int64_t lvllm_head_attention_workspace_bytes(int rows, int num_seqs, int heads, int kv_heads, int kpad, int vpad,
+                                                        int block_size, int max_seq_len, int dtype) {
+  if (heads <= 0 || kv_heads <= 0 || rows <= 0 || num_seqs <= 0 || !takes_mfma(kpad, vpad, block_size, dtype)) return 0;
+  const int n = decode_shares(rows, num_seqs, heads, kv_heads, max_seq_len);
+  return n > 1 ? (int64_t)rows * heads * n * (vpad + 2) * 4 : 0;
+}
+
+extern "C" int lvllm_head_attention(void* out, int64_t out_stride, const void* q, const void* key_cache,
+                                    const void* value_cache, const void* gate, int64_t gate_stride,
                                     const int32_t* block_tables, const int32_t* seq_lens, const int32_t* query_start_loc,
-                                    int num_seqs, int rows, int heads, int kv_heads, int kpad, int vpad, int max_blocks,
-                                    int block_size, int64_t num_blocks, float scale, int64_t k_block_stride,
-                                    int64_t v_block_stride, int dtype, void* stream) {
+                                    int num_seqs, int rows, int heads, int kv_heads, int kpad, int vpad, int vdim,
+                                    int max_blocks, int block_size, int64_t num_blocks, float scale, float out_scale,
+                                    int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len,
+                                    void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
   if (rows == 0 || num_seqs == 0) return 0;
   LV_CHECK(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "heads must be a multiple of kv_heads");
-  LV_CHECK(kpad % 8 == 0 && vpad > 0 && kpad <= 8192 && vpad <= 8192, "key rows are multiples of 8 elements");
+  LV_CHECK(kpad % 8 == 0 && vpad > 0 && vdim > 0 && vdim <= vpad && kpad <= 8192 && vpad <= 8192,
+           "key rows are multiples of 8 elements, value rows at least vdim");
   LV_CHECK(max_blocks > 0 && num_blocks > 0 && block_size > 0, "an empty cache");
-  const HeadAttnParams p{out, q, key_cache, value_cache, block_tables, seq_lens, query_start_loc, num_seqs, rows, heads,
-                         kv_heads, kpad, vpad, max_blocks, block_size, (int)(num_blocks - 1), scale, k_block_stride,
-                         v_block_stride};
+  LV_CHECK(num_seqs <= 65535 && heads <= 65535 && max_query_len > 0, "too many sequences or heads, or no query");
+  HeadAttnParams p{};
+  p.out = out; p.out_stride = out_stride; p.q = q; p.k_cache = key_cache; p.v_cache = value_cache;
+  p.gate = gate; p.gate_stride = gate_stride; p.block_tables = block_tables; p.seq_lens = seq_lens;
+  p.query_start_loc = query_start_loc; p.num_seqs = num_seqs; p.rows = rows; p.heads = heads; p.kv_heads = kv_heads;
+  p.kpad = kpad; p.vpad = vpad; p.vdim = vdim; p.max_blocks = max_blocks; p.block_size = block_size;
+  p.max_block = (int)(num_blocks - 1); p.scale = scale; p.out_scale = out_scale;
+  p.k_block_stride = k_block_stride; p.v_block_stride = v_block_stride;
+  p.max_query_len = max_query_len; p.max_seq_len = max_seq_len; p.nsplit = 1;
+  hipStream_t s = (hipStream_t)stream;
+  if (takes_mfma(kpad, vpad, block_size, dtype)) {
+    p.nsplit = decode_shares(rows, num_seqs, heads, kv_heads, max_seq_len);
+    if (p.nsplit > 1) {
+      LV_CHECK(workspace != nullptr && workspace_bytes >= (int64_t)rows * heads * p.nsplit * (vpad + 2) * 4,
+               "workspace too small (see lvllm_head_attention_workspace_bytes)");
+      p.part_o = (float*)workspace;
+      p.part_ml = p.part_o + (int64_t)rows * heads * p.nsplit * vpad;
+    }
+    if (int rc = launch_head_decode(p, s)) return rc;
+    if (max_query_len > 1)
+      if (int rc = launch_head_prefill(p, s)) return rc;
+    return 0;
+  }
   LV_DISPATCH_DTYPE(dtype, {
     hipLaunchKernelGGL((head_attention_simple_kernel<scalar_t>), dim3(rows, heads), dim3(256),
-                       (size_t)(kpad + 256 + vpad) * 4, (hipStream_t)stream, p);
+                       (size_t)(kpad + 256 + vpad) * 4, s, p);
   });
   LV_LAUNCH_CHECK();
   return 0;

@@ -8,6 +8,17 @@
 //
 //     z = A f(u_t) + bias,   ln w = logsigmoid(z) / tau   (f = identity)   or   ln w = -exp(z)   (f = tanh)
 //
+// Two bodies:
+//   * steps of single tokens (decode): ONE launch per mixer -- decay, state update, read-out, per-head RMS norm and gate --
+//     a workgroup per (sequence, head) that streams the head's state through registers once: HBM-bound;
+//   * everything else: chunks of 16 tokens on fp32 MFMAs.  A parallel pass (chunk_prepare_kernel) computes per (chunk, head)
+//     the decays and all that does not depend on the state: q scaled by the decay from the chunk's start, k scaled by the
+//     decay to its end, the masked 16 x 16 products inside the chunk.  A sequential pass (chunk_scan_kernel) then needs
+//     17 MFMAs per chunk and wave: its state tiles are MFMA accumulators AND, without a move, the B operands of the
+//     read-out (k-step r of a tile contracts rows {r, 4 + r, 8 + r, 12 + r}: accumulator register r of every lane).
+//   Inside a chunk the decay between two tokens is the product of two factors measured from the chunk's middle; a
+//   workgroup whose channels decay too fast for that (a factor would leave fp32's range) takes the products pair by pair.
+//
 // Everything but the projections' results (q, k, v, the low-rank input) is fp32: decays and their logarithms, the state,
 // the read-out.  Rows are the new tokens of `num_seqs` sequences back to back (query_start_loc); a sequence whose tokens
 // are all in this step (seq_lens == its rows) starts from a zero state, every other one from its slot.
@@ -170,6 +181,430 @@ static int launch_scan(const ScanParams& p, int num_seqs, hipStream_t s) {
   return 0;
 }
 
+
+// ---- chunks of 16 tokens ------------------------------------------------------------------------------------------
+typedef float r_f32x4_t __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ r_f32x4_t mfma_f32(float a, float b, r_f32x4_t c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+constexpr int kChunk = 16;
+constexpr float kMaxHalfDecay = 60.f;  // ln of the largest factor measured from the middle of a chunk
+
+// per (chunk, head): floats of the workspace
+__host__ __device__ constexpr int chunk_floats(int dkp) { return 2 * kChunk * dkp + kChunk * kChunk + dkp; }
+
+struct MixParams {
+  const void *q, *k, *v;  // row r, head h at r * stride + h * dk (dv)
+  int64_t q_stride, k_stride, v_stride;
+  const void* u;          // low-rank input, row stride u_stride
+  int64_t u_stride;
+  const float* a_t;       // [rank, heads * dk]
+  const float* decay_bias;
+  int kind, rank;
+  float inv_tau;
+  const float* bonus;     // [heads, dk] or null
+  float q_scale;
+  float* state;
+  int64_t state_stride;
+  const int32_t *state_slots, *query_start_loc, *seq_lens;
+  int num_seqs, num_slots, heads, dk, dv;
+  // epilogue
+  void* out;              // row r, head h at r * out_stride + h * dv
+  int64_t out_stride;
+  const void* gate;
+  int64_t gate_stride;
+  const float* norm_weight;
+  int norm_head_stride;
+  float eps, out_scale;
+  // chunked body
+  float* ws;              // [chunk slots, heads, chunk_floats(dkp)]
+  float* o;               // [rows, heads, dv]
+};
+
+// Chunk ci of sequence s has slot query_start_loc[s] / 16 + s + ci: unique, and monotonic in s.
+__device__ __forceinline__ int chunk_slot_base(const int32_t* qsl, int s) { return qsl[s] / kChunk + s; }
+
+// One workgroup (4 waves) per (chunk slot, head); wave w owns key channels [w * 16 * NT, (w + 1) * 16 * NT).
+template <typename T, int NT>
+__global__ __launch_bounds__(256) void chunk_prepare_kernel(const MixParams p) {
+  using S = typename T::store_t;
+  constexpr int DKP = 64 * NT;
+  constexpr int LD = DKP + 4;  // row stride of the LDS images (bank spread of the 16-byte reads)
+  extern __shared__ float sm[];
+  float* sq = sm;                  // [16][LD]
+  float* sk = sq + kChunk * LD;    // [16][LD]
+  float* sb = sk + kChunk * LD;    // [16][LD]: log decays (slow path), low-rank input before that
+  float* spart = sb + kChunk * LD; // [4][16][16]
+  float* sdiag = spart + 4 * 256;  // [4][16]
+  __shared__ int s_seq;
+  const int head = blockIdx.y;
+  if (threadIdx.x == 0) {  // the sequence that owns this chunk slot: the last s with base(s) <= slot
+    int lo = 0, hi = p.num_seqs;
+    while (lo < hi) {
+      const int mid = (lo + hi) >> 1;
+      if (chunk_slot_base(p.query_start_loc, mid) <= (int)blockIdx.x) lo = mid + 1;
+      else hi = mid;
+    }
+    s_seq = lo - 1;
+  }
+  __syncthreads();
+  const int seq = s_seq;
+  if (seq < 0) return;
+  const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
+  const int t0 = ((int)blockIdx.x - chunk_slot_base(p.query_start_loc, seq)) * kChunk;
+  if (t0 >= qlen) return;
+  const int nt = min(kChunk, qlen - t0);
+  const int64_t row0 = qbeg + t0;
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int g = lane >> 4, c = lane & 15;
+  float* ws = p.ws + ((int64_t)blockIdx.x * p.heads + head) * chunk_floats(DKP);
+  float* w_q = ws;                       // [16 tokens][DKP]
+  float* w_k = w_q + kChunk * DKP;       // [DKP][16 tokens]
+  float* w_a = w_k + kChunk * DKP;       // [16][16]
+  float* w_end = w_a + kChunk * kChunk;  // [DKP]
+
+  // z[token, channel] = u . a_t on MFMAs: A operand lane (token = c, k = g), B operand lane (k = g, channel = c)
+  r_f32x4_t z[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) z[i] = r_f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const bool tok_c = c < nt;
+  for (int k0 = 0; k0 < p.rank; k0 += 4) {
+    const int kk = k0 + g;
+    float a = 0.f;
+    if (tok_c && kk < p.rank) a = T::to_float(((const S*)p.u)[(row0 + c) * p.u_stride + kk]);
+    if (p.kind == kDecayNegExp) a = tanhf(a);
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const int ch = (wave * NT + i) * 16 + c;
+      const float b = (kk < p.rank && ch < p.dk) ? p.a_t[(int64_t)kk * p.heads * p.dk + head * p.dk + ch] : 0.f;
+      z[i] = mfma_f32(a, b, z[i]);
+    }
+  }
+  // lane (channel c of its tile, tokens 4g .. 4g + 3): ln w, then its running sum over the chunk's tokens
+  float cum[NT][4], excl[NT][4], mid[NT], tot[NT];
+  bool fast = true;
+#pragma unroll
+  for (int i = 0; i < NT; ++i) {
+    const int ch = (wave * NT + i) * 16 + c;
+    const float bias = ch < p.dk ? p.decay_bias[head * p.dk + ch] : 0.f;
+    float l[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      l[r] = (4 * g + r < nt && ch < p.dk) ? log_decay_of(z[i][r] + bias, p.kind, p.inv_tau) : 0.f;
+    const float s0 = l[0], s1 = s0 + l[1], s2 = s1 + l[2], s3 = s2 + l[3];
+    const float t16 = __shfl(s3, c), t32 = __shfl(s3, 16 + c), t48 = __shfl(s3, 32 + c), t64 = __shfl(s3, 48 + c);
+    const float before = g == 0 ? 0.f : g == 1 ? t16 : g == 2 ? t16 + t32 : t16 + t32 + t48;
+    mid[i] = t16 + t32;  // the sum up to the middle of the chunk
+    tot[i] = mid[i] + (t48 + t64);
+    cum[i][0] = before + s0; cum[i][1] = before + s1; cum[i][2] = before + s2; cum[i][3] = before + s3;
+    excl[i][0] = before; excl[i][1] = before + s0; excl[i][2] = before + s1; excl[i][3] = before + s2;
+    fast = fast && -mid[i] < kMaxHalfDecay && mid[i] - tot[i] < kMaxHalfDecay;
+  }
+  const bool slow = __syncthreads_or(!fast);
+  const bool has_bonus = p.bonus != nullptr;
+  float diag[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < NT; ++i) {
+    const int ch = (wave * NT + i) * 16 + c;
+    const bool ok = ch < p.dk;
+    const float bon = (has_bonus && ok) ? p.bonus[head * p.dk + ch] : 0.f;
+    float kd[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = 4 * g + r;
+      const bool live = ok && t < nt;
+      const float qv = live ? T::to_float(((const S*)p.q)[(row0 + t) * p.q_stride + head * p.dk + ch]) * p.q_scale : 0.f;
+      const float kv = live ? T::to_float(((const S*)p.k)[(row0 + t) * p.k_stride + head * p.dk + ch]) : 0.f;
+      const float eq = has_bonus ? excl[i][r] : cum[i][r];  // decay between the chunk's start and what token t reads
+      w_q[t * DKP + ch] = qv * expf(eq);
+      kd[r] = kv * expf(tot[i] - cum[i][r]);
+      if (slow) {
+        sq[t * LD + ch] = qv;
+        sk[t * LD + ch] = kv;
+        sb[t * LD + ch] = cum[i][r];
+      } else {
+        sq[t * LD + ch] = qv * expf(eq - mid[i]);
+        sk[t * LD + ch] = kv * expf(mid[i] - cum[i][r]);
+      }
+      diag[r] = fmaf(qv * bon, kv, diag[r]);
+    }
+    *reinterpret_cast<float4*>(w_k + ch * kChunk + 4 * g) = float4{kd[0], kd[1], kd[2], kd[3]};
+    if (g == 0) w_end[ch] = expf(tot[i]);
+  }
+  if (has_bonus) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+#pragma unroll
+      for (int m = 1; m < 16; m <<= 1) diag[r] += __shfl_xor(diag[r], m);
+      if (c == 0) sdiag[wave * 16 + 4 * g + r] = diag[r];
+    }
+  }
+  if (!slow) {
+    // this wave's channels only: what it wrote itself, no barrier needed for other waves' parts
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    r_f32x4_t a4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const int ch0 = (wave * NT + i) * 16 + 4 * g;
+      const float4 qa = *reinterpret_cast<const float4*>(sq + c * LD + ch0);
+      const float4 kb = *reinterpret_cast<const float4*>(sk + c * LD + ch0);
+      a4 = mfma_f32(qa.x, kb.x, a4);
+      a4 = mfma_f32(qa.y, kb.y, a4);
+      a4 = mfma_f32(qa.z, kb.z, a4);
+      a4 = mfma_f32(qa.w, kb.w, a4);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) spart[wave * 256 + (4 * g + r) * 16 + c] = a4[r];
+  }
+  __syncthreads();
+  const int ti = threadIdx.x >> 4, tj = threadIdx.x & 15;
+  const bool below = has_bonus ? tj < ti : tj <= ti;
+  float a = 0.f;
+  if (below) {
+    if (slow) {
+      for (int ch = 0; ch < p.dk; ++ch) {
+        const float b_from = sb[tj * LD + ch];
+        const float b_to = has_bonus ? (ti > 0 ? sb[(ti - 1) * LD + ch] : 0.f) : sb[ti * LD + ch];
+        a = fmaf(sq[ti * LD + ch] * expf(b_to - b_from), sk[tj * LD + ch], a);
+      }
+    } else {
+      a = (spart[threadIdx.x] + spart[256 + threadIdx.x]) + (spart[512 + threadIdx.x] + spart[768 + threadIdx.x]);
+    }
+  } else if (has_bonus && ti == tj) {
+    a = (sdiag[ti] + sdiag[16 + ti]) + (sdiag[32 + ti] + sdiag[48 + ti]);
+  }
+  w_a[threadIdx.x] = a;
+}
+
+// One workgroup per (sequence, head, 16 * NV value columns), walking the sequence's chunks in order.  Wave w holds state
+// rows [w * 16 * NT, (w + 1) * 16 * NT) as accumulator tiles; the four waves' partial read-outs meet in LDS.
+template <typename T, int NT, int NV>
+__global__ __launch_bounds__(256) void chunk_scan_kernel(const MixParams p) {
+  using S = typename T::store_t;
+  constexpr int DKP = 64 * NT;
+  __shared__ float so[2][4][kChunk][16 * NV];
+  const int head = blockIdx.x, v0 = blockIdx.y * 16 * NV, seq = blockIdx.z;
+  const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
+  if (qlen <= 0) return;
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int g = lane >> 4, c = lane & 15;
+  const int slot = p.state_slots[seq];
+  const bool live = slot >= 0 && slot < p.num_slots;
+  float* st = p.state + (int64_t)(live ? slot : 0) * p.state_stride + (int64_t)head * p.dk * p.dv;
+  const bool fresh = p.seq_lens[seq] <= qlen || !live;
+  r_f32x4_t s[NT][NV];
+#pragma unroll
+  for (int i = 0; i < NT; ++i)
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = (wave * NT + i) * 16 + 4 * g + r, col = v0 + 16 * j + c;
+        s[i][j][r] = (!fresh && row < p.dk && col < p.dv) ? st[(int64_t)row * p.dv + col] : 0.f;
+      }
+  const int nchunks = (qlen + kChunk - 1) / kChunk;
+  const float* ws0 = p.ws + ((int64_t)chunk_slot_base(p.query_start_loc, seq) * p.heads + head) * chunk_floats(DKP);
+  const int64_t ws_step = (int64_t)p.heads * chunk_floats(DKP);
+
+  struct Frag {
+    float4 q[NT], k[NT], e[NT];
+    float a;
+    float v[NV][4];
+  };
+  auto load = [&](int ci, Frag& f) __attribute__((always_inline)) {
+    const float* ws = ws0 + ci * ws_step;
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const int ch0 = (wave * NT + i) * 16;
+      f.q[i] = *reinterpret_cast<const float4*>(ws + c * DKP + ch0 + 4 * g);
+      f.k[i] = *reinterpret_cast<const float4*>(ws + kChunk * DKP + (ch0 + c) * kChunk + 4 * g);
+      f.e[i] = *reinterpret_cast<const float4*>(ws + 2 * kChunk * DKP + kChunk * kChunk + ch0 + 4 * g);
+    }
+    f.a = ws[2 * kChunk * DKP + c * kChunk + 4 * g + wave];
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = ci * kChunk + 4 * g + r, col = v0 + 16 * j + c;
+        f.v[j][r] = (t < qlen && col < p.dv)
+                        ? T::to_float(((const S*)p.v)[(int64_t)(qbeg + t) * p.v_stride + head * p.dv + col]) : 0.f;
+      }
+  };
+  auto step = [&](int ci, const Frag& f) __attribute__((always_inline)) {
+    float(*buf)[kChunk][16 * NV] = so[ci & 1];
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      r_f32x4_t o{0.f, 0.f, 0.f, 0.f};
+      // inside the chunk: this wave contracts tokens {4g + wave}
+      const float vw = wave == 0 ? f.v[j][0] : wave == 1 ? f.v[j][1] : wave == 2 ? f.v[j][2] : f.v[j][3];
+      o = mfma_f32(f.a, vw, o);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        o = mfma_f32(f.q[i].x, s[i][j][0], o);
+        o = mfma_f32(f.q[i].y, s[i][j][1], o);
+        o = mfma_f32(f.q[i].z, s[i][j][2], o);
+        o = mfma_f32(f.q[i].w, s[i][j][3], o);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) buf[wave][4 * g + r][16 * j + c] = o[r];
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        r_f32x4_t n = s[i][j];
+        n[0] *= f.e[i].x; n[1] *= f.e[i].y; n[2] *= f.e[i].z; n[3] *= f.e[i].w;
+        n = mfma_f32(f.k[i].x, f.v[j][0], n);
+        n = mfma_f32(f.k[i].y, f.v[j][1], n);
+        n = mfma_f32(f.k[i].z, f.v[j][2], n);
+        n = mfma_f32(f.k[i].w, f.v[j][3], n);
+        s[i][j] = n;
+      }
+    }
+    __syncthreads();  // (the buffer of chunk ci + 1 is the other one: it was read before this barrier)
+    for (int i = threadIdx.x; i < kChunk * 16 * NV; i += 256) {
+      const int t = i / (16 * NV), d = i - t * 16 * NV;
+      if (ci * kChunk + t < qlen && v0 + d < p.dv)
+        p.o[((int64_t)(qbeg + ci * kChunk + t) * p.heads + head) * p.dv + v0 + d] =
+            (buf[0][t][d] + buf[1][t][d]) + (buf[2][t][d] + buf[3][t][d]);
+    }
+  };
+  Frag fa, fb;
+  load(0, fa);
+  for (int ci = 0; ci < nchunks; ci += 2) {
+    if (ci + 1 < nchunks) load(ci + 1, fb);
+    step(ci, fa);
+    if (ci + 1 >= nchunks) break;
+    if (ci + 2 < nchunks) load(ci + 2, fa);
+    step(ci + 1, fb);
+  }
+  if (live) {
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int row = (wave * NT + i) * 16 + 4 * g + r, col = v0 + 16 * j + c;
+          if (row < p.dk && col < p.dv) st[(int64_t)row * p.dv + col] = s[i][j][r];
+        }
+  }
+}
+
+// ---- single tokens -------------------------------------------------------------------------------------------------
+// One workgroup per (head, sequence), sequence s owning row s.  Thread (rg, cg): state columns 4 cg .. 4 cg + 3 of rows
+// rg, rg + RG, ...
+template <typename T>
+__global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p) {
+  using S = typename T::store_t;
+  extern __shared__ float sm[];
+  const int head = blockIdx.x, seq = blockIdx.y;
+  const int row = p.query_start_loc[seq];
+  if (p.query_start_loc[seq + 1] - row != 1) return;
+  const int dk = p.dk, dv = p.dv;
+  float* sq = sm;            // [dk]
+  float* sk = sq + dk;       // [dk]
+  float* sw = sk + dk;       // [dk]
+  float* su = sw + dk;       // [rank]
+  float* sv = sm + ((3 * dk + p.rank + 3) & ~3);  // [dv], 16-byte aligned
+  float* so = sv + dv;       // [row groups][dv]
+  __shared__ float red[16];
+  __shared__ float s_bonus;
+  for (int i = threadIdx.x; i < p.rank; i += 256) {
+    const float f = T::to_float(((const S*)p.u)[(int64_t)row * p.u_stride + i]);
+    su[i] = p.kind == kDecayNegExp ? tanhf(f) : f;
+  }
+  for (int i = threadIdx.x; i < dv; i += 256) sv[i] = T::to_float(((const S*)p.v)[(int64_t)row * p.v_stride + head * dv + i]);
+  __syncthreads();
+  float bsum = 0.f;
+  for (int i = threadIdx.x; i < dk; i += 256) {
+    const float qv = T::to_float(((const S*)p.q)[(int64_t)row * p.q_stride + head * dk + i]) * p.q_scale;
+    const float kv = T::to_float(((const S*)p.k)[(int64_t)row * p.k_stride + head * dk + i]);
+    float z = 0.f;
+    for (int r = 0; r < p.rank; ++r) z = fmaf(su[r], p.a_t[(int64_t)r * p.heads * dk + head * dk + i], z);
+    sq[i] = qv;
+    sk[i] = kv;
+    sw[i] = expf(log_decay_of(z + p.decay_bias[head * dk + i], p.kind, p.inv_tau));
+    if (p.bonus != nullptr) bsum = fmaf(qv * p.bonus[head * dk + i], kv, bsum);
+  }
+  const bool has_bonus = p.bonus != nullptr;
+  const float b = block_sum(bsum, red);  // (barriers: sq / sk / sw are visible behind it)
+  if (threadIdx.x == 0) s_bonus = b;
+  const int slot = p.state_slots[seq];
+  const bool live = slot >= 0 && slot < p.num_slots;
+  const bool fresh = p.seq_lens[seq] <= 1 || !live;
+  float* st = p.state + (int64_t)(live ? slot : 0) * p.state_stride + (int64_t)head * dk * dv;
+  const bool vec = (dv & 3) == 0;
+  const int cgs = vec ? dv / 4 : dv;           // column groups
+  const int per = min(cgs, 256);               // threads along a row
+  const int rgs = 256 / per;                   // row groups
+  const int rg = threadIdx.x / per, cg0 = threadIdx.x - rg * per;
+  if (rg < rgs) {
+    for (int cg = cg0; cg < cgs; cg += per) {
+      if (vec) {
+        const float4 v = *reinterpret_cast<const float4*>(sv + 4 * cg);
+        float4 acc{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+        for (int r = rg; r < dk; r += rgs) {
+          float4 s{0.f, 0.f, 0.f, 0.f};
+          float* at = st + (int64_t)r * dv + 4 * cg;
+          if (!fresh) s = *reinterpret_cast<const float4*>(at);
+          const float w = sw[r], k = sk[r], q = sq[r];
+          float4 n{fmaf(w, s.x, k * v.x), fmaf(w, s.y, k * v.y), fmaf(w, s.z, k * v.z), fmaf(w, s.w, k * v.w)};
+          const float4 rd = has_bonus ? s : n;
+          acc.x = fmaf(q, rd.x, acc.x); acc.y = fmaf(q, rd.y, acc.y);
+          acc.z = fmaf(q, rd.z, acc.z); acc.w = fmaf(q, rd.w, acc.w);
+          if (live) *reinterpret_cast<float4*>(at) = n;
+        }
+        *reinterpret_cast<float4*>(so + rg * dv + 4 * cg) = acc;
+      } else {
+        const float v = sv[cg];
+        float acc = 0.f;
+        for (int r = rg; r < dk; r += rgs) {
+          float* at = st + (int64_t)r * dv + cg;
+          const float s = fresh ? 0.f : *at;
+          const float n = fmaf(sw[r], s, sk[r] * v);
+          acc = fmaf(sq[r], has_bonus ? s : n, acc);
+          if (live) *at = n;
+        }
+        so[rg * dv + cg] = acc;
+      }
+    }
+  }
+  __syncthreads();
+  const float bonus = s_bonus;
+  float ss = 0.f;
+  for (int d = threadIdx.x; d < dv; d += 256) {
+    float o = has_bonus ? bonus * sv[d] : 0.f;
+    for (int r = 0; r < rgs; ++r) o += so[r * dv + d];
+    so[d] = o;  // (column d is this thread's alone)
+    ss = fmaf(o, o, ss);
+  }
+  const float r = 1.f / sqrtf(block_sum(ss, red) / dv + p.eps);
+  for (int d = threadIdx.x; d < dv; d += 256) {
+    const float z = T::to_float(((const S*)p.gate)[(int64_t)row * p.gate_stride + head * dv + d]);
+    const float silu = z / (1.f + expf(-z));
+    ((S*)p.out)[(int64_t)row * p.out_stride + head * dv + d] =
+        T::from_float(so[d] * r * p.norm_weight[head * p.norm_head_stride + d] * silu * p.out_scale);
+  }
+}
+
+template <typename T, int NT>
+static void launch_chunks(const MixParams& p, int rows, hipStream_t s) {
+  constexpr int LD = 64 * NT + 4;
+  const size_t smem = (size_t)(3 * kChunk * LD + 4 * 256 + 64) * sizeof(float);
+  if (smem > 64 * 1024)
+    (void)hipFuncSetAttribute((const void*)chunk_prepare_kernel<T, NT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+  hipLaunchKernelGGL((chunk_prepare_kernel<T, NT>), dim3(rows / kChunk + p.num_seqs + 1, p.heads), dim3(256), smem, s, p);
+  const int tiles = (p.dv + 15) / 16;
+  // 16 columns per workgroup fill the chip with few (sequence, head) pairs; wider slices re-read q, k and the in-chunk
+  // products less often
+  if ((int64_t)p.heads * p.num_seqs * tiles <= 512 || tiles == 1)
+    hipLaunchKernelGGL((chunk_scan_kernel<T, NT, 1>), dim3(p.heads, tiles, p.num_seqs), dim3(256), 0, s, p);
+  else
+    hipLaunchKernelGGL((chunk_scan_kernel<T, NT, 2>), dim3(p.heads, (tiles + 1) / 2, p.num_seqs), dim3(256), 0, s, p);
+}
+
 }  // namespace lvllm
 
 using namespace lvllm;
@@ -210,4 +645,64 @@ extern "C" int lvllm_recurrent_scan(float* o, const void* q, const void* k, cons
   });
   LV_LAUNCH_CHECK();
   return 0;
+}
+
+static int padded_dk(int dk) { return (dk + 63) / 64 * 64; }
+
+extern "C" int64_t lvllm_recurrent_mix_workspace_bytes(int rows, int num_seqs, int heads, int dk, int max_query_len) {
+  if (max_query_len <= 1) return 0;
+  return ((int64_t)rows / kChunk + num_seqs + 1) * heads * chunk_floats(padded_dk(dk)) * 4;
+}
+
+extern "C" int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void* k, const void* v,
+                                   int64_t q_stride, int64_t k_stride, int64_t v_stride, const void* u, int64_t u_stride,
+                                   const float* a_t, const float* decay_bias, int rank, int kind, float inv_tau,
+                                   const float* bonus, float q_scale, const void* gate, int64_t gate_stride,
+                                   const float* norm_weight, int norm_head_stride, float eps, float out_scale, float* state,
+                                   int64_t state_stride, const int32_t* state_slots, int num_slots,
+                                   const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows,
+                                   int heads, int dk, int dv, int max_query_len, float* o_scratch, void* workspace,
+                                   int64_t workspace_bytes, int dtype, void* stream) {
+  if (num_seqs == 0 || rows == 0) return 0;
+  LV_CHECK(dk > 0 && dk <= 256 && dv > 0 && dv <= 1024, "key size must be in 1 .. 256, value size in 1 .. 1024");
+  LV_CHECK(kind == kDecayLogSigmoid || kind == kDecayNegExp, "unknown decay kind");
+  LV_CHECK(rank > 0 && rank <= 1024, "rank must be in 1 .. 1024");
+  LV_CHECK(state_stride >= (int64_t)heads * dk * dv && ((dv & 3) != 0 || (state_stride & 3) == 0),
+           "state slots overlap or are unaligned");
+  LV_CHECK(num_seqs <= 65535 && heads <= 65535, "too many sequences or heads");
+  MixParams p{};
+  p.q = q; p.k = k; p.v = v; p.q_stride = q_stride; p.k_stride = k_stride; p.v_stride = v_stride;
+  p.u = u; p.u_stride = u_stride; p.a_t = a_t; p.decay_bias = decay_bias; p.kind = kind; p.rank = rank; p.inv_tau = inv_tau;
+  p.bonus = bonus; p.q_scale = q_scale; p.state = state; p.state_stride = state_stride; p.state_slots = state_slots;
+  p.query_start_loc = query_start_loc; p.seq_lens = seq_lens; p.num_seqs = num_seqs; p.num_slots = num_slots;
+  p.heads = heads; p.dk = dk; p.dv = dv; p.out = out; p.out_stride = out_stride; p.gate = gate; p.gate_stride = gate_stride;
+  p.norm_weight = norm_weight; p.norm_head_stride = norm_head_stride; p.eps = eps; p.out_scale = out_scale;
+  hipStream_t s = (hipStream_t)stream;
+  if (max_query_len <= 1) {  // every sequence brings one token: sequence s owns row s
+    const int cgs = (dv & 3) == 0 ? dv / 4 : dv, per = cgs < 256 ? cgs : 256;
+    const size_t smem = (size_t)(3 * dk + rank + 3 + dv + (256 / per) * dv + 8) * sizeof(float);
+    LV_DISPATCH_DTYPE(dtype, {
+      if (smem > 64 * 1024)
+        (void)hipFuncSetAttribute((const void*)recurrent_decode_kernel<scalar_t>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+      hipLaunchKernelGGL((recurrent_decode_kernel<scalar_t>), dim3(heads, num_seqs), dim3(256), smem, s, p);
+    });
+    LV_LAUNCH_CHECK();
+    return 0;
+  }
+  LV_CHECK(workspace != nullptr && o_scratch != nullptr &&
+               workspace_bytes >= lvllm_recurrent_mix_workspace_bytes(rows, num_seqs, heads, dk, max_query_len),
+           "workspace too small (see lvllm_recurrent_mix_workspace_bytes)");
+  p.ws = (float*)workspace;
+  p.o = o_scratch;
+  LV_DISPATCH_DTYPE(dtype, {
+    switch (padded_dk(dk) / 64) {
+      case 1: launch_chunks<scalar_t, 1>(p, rows, s); break;
+      case 2: launch_chunks<scalar_t, 2>(p, rows, s); break;
+      case 3: launch_chunks<scalar_t, 3>(p, rows, s); break;
+      default: launch_chunks<scalar_t, 4>(p, rows, s); break;
+    }
+  });
+  LV_LAUNCH_CHECK();
+  return lvllm_head_norm_gate(out, out_stride, o_scratch, gate, gate_stride, norm_weight, norm_head_stride, eps, out_scale,
+                              rows, heads, dv, dtype, stream);
 }

@@ -227,20 +227,6 @@ __global__ void qk_norm_cache_kernel(typename T::store_t* __restrict__ q_out, ty
 
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 
-// out[row, h * vdim + d] = T(attn[row, h, d] * sigmoid(gate[row, h]) * scale): one gate number per head
-template <typename T>
-__global__ void head_gate_kernel(typename T::store_t* __restrict__ out, const int64_t out_stride,
-                                 const typename T::store_t* __restrict__ attn, const int64_t attn_head_stride,
-                                 const typename T::store_t* __restrict__ gate, const int64_t gate_stride,
-                                 const int heads, const int vdim, const float scale) {
-  const int row = blockIdx.x;
-  for (int i = threadIdx.x; i < heads * vdim; i += blockDim.x) {
-    const int h = i / vdim, d = i - h * vdim;
-    const float g = sigmoid_f(T::to_float(gate[row * gate_stride + h])) * scale;
-    out[row * out_stride + i] = T::from_float(T::to_float(attn[((int64_t)row * heads + h) * attn_head_stride + d]) * g);
-  }
-}
-
 // Per head: o / rms(o) * weight * silu(gate) * scale -> T.  o is the fp32 read-out of a recurrent state.
 // weight_head_stride: 0 (one weight of size vdim for all heads) or vdim.  A wave per (row, head).
 template <typename T>
@@ -359,18 +345,6 @@ extern "C" int lvllm_qk_norm_cache(void* q_out, void* key_cache, void* value_cac
                        (S*)key_cache, (S*)value_cache, (const S*)q, (const S*)k, (const S*)v, row_stride, q_weight,
                        k_weight, eps, heads, kv_heads, dim, vdim, kpad, vpad, slot_mapping, num_blocks * block_size,
                        block_size, k_block_stride, v_block_stride);
-  });
-  LV_LAUNCH_CHECK();
-  return 0;
-}
-
-extern "C" int lvllm_head_gate(void* out, int64_t out_stride, const void* attn, int64_t attn_head_stride, const void* gate,
-                               int64_t gate_stride, int rows, int heads, int vdim, float scale, int dtype, void* stream) {
-  if (rows == 0) return 0;
-  LV_DISPATCH_DTYPE(dtype, {
-    using S = scalar_t::store_t;
-    hipLaunchKernelGGL((head_gate_kernel<scalar_t>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (S*)out, out_stride,
-                       (const S*)attn, attn_head_stride, (const S*)gate, gate_stride, heads, vdim, scale);
   });
   LV_LAUNCH_CHECK();
   return 0;

@@ -689,42 +689,40 @@ torch::Tensor qk_norm_cache(const torch::Tensor& q, const torch::Tensor& k, cons
   return q_out;
 }
 
-torch::Tensor head_attention(const torch::Tensor& q, const torch::Tensor& key_cache, const torch::Tensor& value_cache,
-                             const torch::Tensor& block_tables, const torch::Tensor& seq_lens,
-                             const torch::Tensor& query_start_loc, double scale, int64_t max_query_len,
-                             int64_t max_seq_len) {
+void head_attention(torch::Tensor& out, const torch::Tensor& q, const torch::Tensor& key_cache,
+                    const torch::Tensor& value_cache, const torch::Tensor& block_tables, const torch::Tensor& seq_lens,
+                    const torch::Tensor& query_start_loc, const std::optional<torch::Tensor>& gate, int64_t vdim,
+                    double scale, double out_scale, int64_t max_query_len, int64_t max_seq_len) {
   const char* op = "head_attention";
   LV_CHECK_DEVICE(q);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous(), op, ": contiguous q [rows, heads, kpad]");
-  const int64_t kv_heads = key_cache.size(1);
+  const int64_t kv_heads = key_cache.size(1), rows = q.size(0), heads = q.size(1);
   const auto [kpad, vpad, bs] = head_cache_dims(key_cache, value_cache, kv_heads, q.scalar_type(), op);
-  TORCH_CHECK(q.size(2) == kpad, op, ": q and the key cache disagree on the padded key size");
+  TORCH_CHECK(q.size(2) == kpad && vdim <= vpad, op, ": q and the caches disagree on the padded sizes");
+  TORCH_CHECK(out.is_cuda() && out.dim() == 2 && out.stride(1) == 1 && out.size(0) == rows && out.size(1) == heads * vdim &&
+                  out.scalar_type() == q.scalar_type(),
+              op, ": out [rows, heads * vdim]");
+  if (gate)
+    TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 && gate->stride(1) == 1 && gate->size(0) == rows &&
+                    gate->size(1) == heads && gate->scalar_type() == q.scalar_type(),
+                op, ": gate [rows, heads]");
   check_layout(query_start_loc, seq_lens, op);
   TORCH_CHECK(block_tables.is_cuda() && block_tables.dim() == 2 && block_tables.scalar_type() == at::kInt &&
                   block_tables.is_contiguous() && block_tables.size(0) >= seq_lens.numel(),
               op, ": block_tables int32 [num_seqs, blocks]");
-  auto out = torch::empty({q.size(0), q.size(1), vpad}, q.options());
-  check(lvllm_head_attention(out.data_ptr(), q.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(),
-                             block_tables.data_ptr<int>(), seq_lens.data_ptr<int>(), query_start_loc.data_ptr<int>(),
-                             (int)seq_lens.numel(), (int)q.size(0), (int)q.size(1), (int)kv_heads, (int)kpad, (int)vpad,
-                             (int)block_tables.size(1), (int)bs, key_cache.size(0), (float)scale, key_cache.stride(0),
-                             value_cache.stride(0), dtype_code(q, op), current_stream(q)));
-  return out;
-}
-
-void head_gate(torch::Tensor& out, const torch::Tensor& attn, const torch::Tensor& gate, int64_t vdim, double scale) {
-  const char* op = "head_gate";
-  LV_CHECK_DEVICE(attn);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(attn));
-  const int64_t rows = attn.size(0), heads = attn.size(1);
-  TORCH_CHECK(attn.dim() == 3 && attn.is_contiguous() && attn.size(2) >= vdim && out.dim() == 2 && out.stride(1) == 1 &&
-                  out.size(0) == rows && out.size(1) == heads * vdim && gate.dim() == 2 && gate.stride(1) == 1 &&
-                  gate.size(0) == rows && gate.size(1) == heads && out.scalar_type() == attn.scalar_type() &&
-                  gate.scalar_type() == attn.scalar_type(),
-              op, ": attn [rows, heads, >= vdim], gate [rows, heads], out [rows, heads * vdim]");
-  check(lvllm_head_gate(out.data_ptr(), out.stride(0), attn.data_ptr(), attn.size(2), gate.data_ptr(), gate.stride(0),
-                        (int)rows, (int)heads, (int)vdim, (float)scale, dtype_code(attn, op), current_stream(attn)));
+  const int ns = (int)seq_lens.numel(), code = dtype_code(q, op);
+  const int64_t need = lvllm_head_attention_workspace_bytes((int)rows, ns, (int)heads, (int)kv_heads, (int)kpad, (int)vpad,
+                                                            (int)bs, (int)max_seq_len, code);
+  torch::Tensor ws;
+  if (need > 0) ws = torch::empty({need}, q.options().dtype(at::kByte));
+  check(lvllm_head_attention(out.data_ptr(), out.stride(0), q.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(),
+                             gate ? gate->data_ptr() : nullptr, gate ? gate->stride(0) : 0, block_tables.data_ptr<int>(),
+                             seq_lens.data_ptr<int>(), query_start_loc.data_ptr<int>(), ns, (int)rows, (int)heads,
+                             (int)kv_heads, (int)kpad, (int)vpad, (int)vdim, (int)block_tables.size(1), (int)bs,
+                             key_cache.size(0), (float)scale, (float)out_scale, key_cache.stride(0), value_cache.stride(0),
+                             (int)max_query_len, (int)max_seq_len, need > 0 ? ws.data_ptr() : nullptr, need, code,
+                             current_stream(q)));
 }
 
 void head_norm_gate(torch::Tensor& out, const torch::Tensor& o, const torch::Tensor& gate, const torch::Tensor& weight,
@@ -786,6 +784,55 @@ torch::Tensor recurrent_scan(const torch::Tensor& q, const torch::Tensor& k, con
                              (int)state.size(0), query_start_loc.data_ptr<int>(), seq_lens.data_ptr<int>(),
                              (int)seq_lens.numel(), (int)heads, (int)dk, (int)dv, dtype_code(q, op), current_stream(q)));
   return o;
+}
+
+void recurrent_mix(torch::Tensor& out, const torch::Tensor& q, const torch::Tensor& k, const torch::Tensor& v,
+                   const torch::Tensor& u, const torch::Tensor& a_t, const torch::Tensor& decay_bias, int64_t kind,
+                   double inv_tau, const std::optional<torch::Tensor>& bonus, double q_scale, const torch::Tensor& gate,
+                   const torch::Tensor& norm_weight, double eps, double out_scale, torch::Tensor& state,
+                   const torch::Tensor& state_slots, const torch::Tensor& query_start_loc, const torch::Tensor& seq_lens,
+                   int64_t max_query_len) {
+  const char* op = "recurrent_mix";
+  LV_CHECK_DEVICE(q);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
+  TORCH_CHECK(state.dim() == 4, op, ": state [slots, heads, dk, dv]");
+  const int64_t rows = q.size(0), heads = state.size(1), dk = state.size(2), dv = state.size(3), rank = u.size(1);
+  auto rows_of = [&](const torch::Tensor& t, int64_t cols, const char* what) {
+    TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == rows && t.size(1) == cols && t.stride(1) == 1 &&
+                    t.scalar_type() == q.scalar_type(),
+                op, ": ", what, " must be [rows, ", cols, "] of the compute dtype");
+  };
+  rows_of(q, heads * dk, "q");
+  rows_of(k, heads * dk, "k");
+  rows_of(v, heads * dv, "v");
+  rows_of(u, rank, "u");
+  rows_of(gate, heads * dv, "gate");
+  rows_of(out, heads * dv, "out");
+  TORCH_CHECK(a_t.dim() == 2 && a_t.size(0) == rank, op, ": a_t [rank, heads * dk]");
+  check_f32(a_t, rank * heads * dk, op, "a_t");
+  check_f32(decay_bias, heads * dk, op, "decay_bias");
+  if (bonus) check_f32(*bonus, heads * dk, op, "bonus");
+  const bool shared = norm_weight.numel() == dv;
+  check_f32(norm_weight, shared ? dv : heads * dv, op, "norm_weight");
+  check_layout(query_start_loc, seq_lens, op);
+  check_state(state, state_slots, heads * dk * dv, seq_lens.numel(), op);
+  const int ns = (int)seq_lens.numel();
+  if (max_query_len <= 1) TORCH_CHECK(ns == rows, op, ": a step of single tokens has one row per sequence");
+  const int64_t need = lvllm_recurrent_mix_workspace_bytes((int)rows, ns, (int)heads, (int)dk, (int)max_query_len);
+  torch::Tensor ws, o;
+  if (max_query_len > 1) {
+    ws = torch::empty({need}, q.options().dtype(at::kByte));
+    o = torch::empty({rows, heads, dv}, q.options().dtype(at::kFloat));
+  }
+  check(lvllm_recurrent_mix(out.data_ptr(), out.stride(0), q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0),
+                            k.stride(0), v.stride(0), u.data_ptr(), u.stride(0), a_t.data_ptr<float>(),
+                            decay_bias.data_ptr<float>(), (int)rank, (int)kind, (float)inv_tau,
+                            bonus ? bonus->data_ptr<float>() : nullptr, (float)q_scale, gate.data_ptr(), gate.stride(0),
+                            norm_weight.data_ptr<float>(), shared ? 0 : (int)dv, (float)eps, (float)out_scale,
+                            state.data_ptr<float>(), state.stride(0), state_slots.data_ptr<int>(), (int)state.size(0),
+                            query_start_loc.data_ptr<int>(), seq_lens.data_ptr<int>(), ns, (int)rows, (int)heads, (int)dk,
+                            (int)dv, (int)max_query_len, o.defined() ? o.data_ptr<float>() : nullptr,
+                            ws.defined() ? ws.data_ptr() : nullptr, need, dtype_code(q, op), current_stream(q)));
 }
 
 }  // namespace
@@ -897,11 +944,15 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, hybrid) {
   hybrid.def("qk_norm_cache(Tensor q, Tensor k, Tensor v, Tensor q_weight, Tensor k_weight, float eps, int heads, "
              "int kv_heads, Tensor(a!) key_cache, Tensor(b!) value_cache, Tensor slot_mapping) -> Tensor");
   hybrid.impl("qk_norm_cache", torch::kCUDA, &qk_norm_cache);
-  hybrid.def("head_attention(Tensor q, Tensor key_cache, Tensor value_cache, Tensor block_tables, Tensor seq_lens, "
-             "Tensor query_start_loc, float scale, int max_query_len, int max_seq_len) -> Tensor");
+  hybrid.def("head_attention(Tensor(a!) out, Tensor q, Tensor key_cache, Tensor value_cache, Tensor block_tables, "
+             "Tensor seq_lens, Tensor query_start_loc, Tensor? gate, int vdim, float scale, float out_scale, "
+             "int max_query_len, int max_seq_len) -> ()");
   hybrid.impl("head_attention", torch::kCUDA, &head_attention);
-  hybrid.def("head_gate(Tensor(a!) out, Tensor attn, Tensor gate, int vdim, float scale) -> ()");
-  hybrid.impl("head_gate", torch::kCUDA, &head_gate);
+  hybrid.def("recurrent_mix(Tensor(a!) out, Tensor q, Tensor k, Tensor v, Tensor u, Tensor a_t, Tensor decay_bias, "
+             "int kind, float inv_tau, Tensor? bonus, float q_scale, Tensor gate, Tensor norm_weight, float eps, "
+             "float out_scale, Tensor(b!) state, Tensor state_slots, Tensor query_start_loc, Tensor seq_lens, "
+             "int max_query_len) -> ()");
+  hybrid.impl("recurrent_mix", torch::kCUDA, &recurrent_mix);
   hybrid.def("head_norm_gate(Tensor(a!) out, Tensor o, Tensor gate, Tensor weight, float eps, float scale) -> ()");
   hybrid.impl("head_norm_gate", torch::kCUDA, &head_norm_gate);
   hybrid.def("log_decay(Tensor u, Tensor a_t, Tensor bias, int kind, float inv_tau) -> Tensor");

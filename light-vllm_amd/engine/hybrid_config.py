@@ -18,11 +18,16 @@ class KVSpec:
 
     @property
     def kpad(self) -> int:
-        return (self.dim + 31) // 32 * 32
+        return self._padded(self.dim, (64, 96, 128, 192, 256))
 
     @property
     def vpad(self) -> int:
-        return (self.vdim + 15) // 16 * 16
+        return self._padded(self.vdim, (32, 64, 96, 128, 192, 256))
+
+    @staticmethod
+    def _padded(n: int, sizes) -> int:
+        """The next size the MFMA bodies of the attention have (csrc/head_attention.hip); beyond them multiples of 32."""
+        return next((s for s in sizes if n <= s), (n + 31) // 32 * 32)
 
     def block_elements(self, block_size: int) -> int:
         return self.kv_heads * (self.kpad + self.vpad) * block_size
@@ -86,6 +91,8 @@ class HybridModelConfig:
     max_position_embeddings: int = 1 << 30  # no positions anywhere: unlimited
 
     def __post_init__(self) -> None:
+        if self.dtype not in (torch.bfloat16, torch.float32):
+            raise ValueError("hybrid decoders run in bfloat16 or float32")
         if self.quantization is not None:
             raise ValueError("hybrid decoders have no quantised path")
         for i, l in enumerate(self.layers):

@@ -102,6 +102,7 @@ class HybridModel:
     def _layer(self, get, name: str, l, pack: bool):
         mixer = (ParallelMixer if isinstance(l.mixer, ParallelMixerConfig) else TimeMixer)(
             get, name + ".mix", l.mixer, self.cfg.norm_eps, pack)
+        mixer.recurrence.fused = self.cfg.fuse_decode_ops
         ff = (DynTanhNorm(get, name + ".norm2"), SquaredReluMlp(get, name + ".mlp", pack)) if l.ff is not None else None
         return DynTanhNorm(get, name + ".norm1"), mixer, ff
 

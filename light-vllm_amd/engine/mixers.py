@@ -100,6 +100,25 @@ class LowRankDecay:
         return amd.log_decay(u, self.a_t, self.bias, self.kind, self.inv_tau)
 
 
+class Recurrence:
+    """A decayed matrix state with its read-out, per-head RMS norm and SiLU gate: out = norm(o) * weight * silu(g) * scale.
+    `fused`: one operator (a single launch for steps of single tokens); else decays, token-by-token recurrence, norm and
+    gate as launches of their own."""
+
+    def __init__(self, decay: LowRankDecay, bonus: Optional[torch.Tensor], eps: float):
+        self.decay, self.bonus, self.eps, self.fused = decay, bonus, eps, True
+
+    def __call__(self, out, q, k, v, u, gate, weight, out_scale: float, q_scale: float, state, step: StepLayout) -> None:
+        d = self.decay
+        if self.fused:
+            amd.recurrent_mix(out, q, k, v, u, d.a_t, d.bias, d.kind, d.inv_tau, self.bonus, q_scale, gate, weight, self.eps,
+                              out_scale, state, step.state_slots, step.query_start_loc, step.seq_lens, step.max_query_len)
+        else:
+            o = amd.recurrent_scan(q, k, v, d(u), self.bonus, q_scale, state, step.state_slots, step.query_start_loc,
+                                   step.seq_lens)
+            amd.head_norm_gate(out, o, gate, weight, self.eps, out_scale)
+
+
 class ParallelMixer:
     """left_scale * softmax heads + right_scale * gated linear attention, both reading the same normed input: ONE input
     projection (all ten weights stacked) and ONE output projection over the two concatenated results; the scales are
@@ -118,6 +137,7 @@ class ParallelMixer:
         self.q_norm, self.k_norm = get(l + ".q.norm").float(), get(l + ".k.norm").float()
         self.decay = LowRankDecay(get(rt + ".a2"), get(rt + ".a2.b"), DECAY_LOGSIGMOID, 1.0 / r.tau)
         self.out_norm = get(rt + ".norm").float()
+        self.recurrence = Recurrence(self.decay, None, eps)
         self.left_cols, self.right_cols = a.heads * a.vdim, r.heads * r.vdim
         self.out = make_weight(pad_columns(torch.cat([get(l + ".o"), get(rt + ".o")], dim=1)), pack)
         self.kv_spec = KVSpec(a.kv_heads, a.dim, a.vdim)
@@ -133,13 +153,11 @@ class ParallelMixer:
         # softmax heads
         kc, vc = attn.split_kv_cache(cache.kv, self.kv_spec, step.block_size)
         q = amd.qk_norm_cache(lq, lk, lv, self.q_norm, self.k_norm, self.eps, a.heads, a.kv_heads, kc, vc, step.slot_mapping)
-        o = amd.head_attention(q, kc, vc, step.block_tables, step.seq_lens, step.query_start_loc, a.scale,
-                               step.max_query_len, step.max_seq_len)
-        amd.head_gate(both[:, :self.left_cols], o, lg, a.vdim, self.cfg.left_scale)
+        amd.head_attention(both[:, :self.left_cols], q, kc, vc, step.block_tables, step.seq_lens, step.query_start_loc, lg,
+                           a.vdim, a.scale, self.cfg.left_scale, step.max_query_len, step.max_seq_len)
         # gated linear attention
-        s = amd.recurrent_scan(rq, rk, rv, self.decay(u), None, r.dim ** -0.5, cache.state["matrix"], step.state_slots,
-                               step.query_start_loc, step.seq_lens)
-        amd.head_norm_gate(both[:, self.left_cols:cols], s, rg, self.out_norm, self.eps, self.cfg.right_scale)
+        self.recurrence(both[:, self.left_cols:cols], rq, rk, rv, u, rg, self.out_norm, self.cfg.right_scale,
+                        r.dim ** -0.5, cache.state["matrix"], step)
         return x, project_to_residual(both, self.out)
 
 
@@ -149,7 +167,7 @@ class TimeMixer:
     MIXES = "rkvgw"
 
     def __init__(self, get, name: str, cfg: TimeMixerConfig, eps: float, pack: bool):
-        self.cfg, self.eps = cfg, eps
+        self.cfg = cfg
         self.mu = torch.stack([get(f"{name}.mu.{s}").float() for s in self.MIXES]).contiguous()
         self.rkvg = [make_weight(get(f"{name}.{s}"), pack) for s in "rkvg"]
         # the library's batched product takes the weights as [4, width, heads * dim]
@@ -158,7 +176,7 @@ class TimeMixer:
         self.rank = w1.shape[0]
         self.w1 = make_weight(stack_rows([w1])[0], pack)
         self.decay = LowRankDecay(get(name + ".w2"), get(name + ".w0"), DECAY_NEGEXP)
-        self.bonus = get(name + ".u").float().contiguous()
+        self.recurrence = Recurrence(self.decay, get(name + ".u").float().contiguous(), eps)
         self.norm = get(name + ".norm").float()
         self.out = make_weight(pad_columns(get(name + ".o")), pack)
 
@@ -169,12 +187,10 @@ class TimeMixer:
             r, k, v, g = (linear(mix[i], w) for i, w in enumerate(self.rkvg))
         else:
             r, k, v, g = torch.bmm(mix[:4], self.rkvg_t)
-        log_w = self.decay(linear(mix[4], self.w1)[:, :self.rank])
-        s = amd.recurrent_scan(r, k, v, log_w, self.bonus, 1.0, cache.state["matrix"], step.state_slots,
-                               step.query_start_loc, step.seq_lens)
+        u = linear(mix[4], self.w1)[:, :self.rank]
         cols = self.cfg.heads * self.cfg.dim
         out = (torch.empty if self.out.K == cols else torch.zeros)(rows, self.out.K, dtype=dtype, device=x.device)
-        amd.head_norm_gate(out[:, :cols], s, g, self.norm, self.eps, 1.0)
+        self.recurrence(out[:, :cols], r, k, v, u, g, self.norm, 1.0, 1.0, cache.state["matrix"], step)
         return x, project_to_residual(out, self.out)
 
 
