@@ -29,7 +29,7 @@ namespace lvllm {
 enum { kDecayLogSigmoid = 0, kDecayNegExp = 1 };
 
 __device__ __forceinline__ float log_decay_of(float z, int kind, float inv_tau) {
-  if (kind == kDecayNegExp) return -expf(z);
+  if (kind == kDecayNegExp) return -expf(fminf(z, 9.f));  // (exp(-exp(9)) is 0: a finite logarithm keeps sums finite)
   return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau;
 }
 
@@ -233,7 +233,7 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(const MixParams p) {
   extern __shared__ float sm[];
   float* sq = sm;                  // [16][LD]
   float* sk = sq + kChunk * LD;    // [16][LD]
-  float* sb = sk + kChunk * LD;    // [16][LD]: log decays (slow path), low-rank input before that
+  float* sb = sk + kChunk * LD;    // [16][LD]: ln w (slow path)
   float* spart = sb + kChunk * LD; // [4][16][16]
   float* sdiag = spart + 4 * 256;  // [4][16]
   __shared__ int s_seq;
@@ -281,28 +281,39 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(const MixParams p) {
       z[i] = mfma_f32(a, b, z[i]);
     }
   }
-  // lane (channel c of its tile, tokens 4g .. 4g + 3): ln w, then its running sum over the chunk's tokens
-  float cum[NT][4], excl[NT][4], mid[NT], tot[NT];
+  // lane (channel c of its tile, tokens 4g .. 4g + 3): ln w, then its sums over ranges of the chunk's tokens.  Every range
+  // is summed by itself: a difference of two running sums would lose the small decays behind a large one.
+  float lw[NT][4], read[NT][4], left[NT][4], tot[NT];  // read: chunk's start -> what token t reads; left: token t -> end
+  float half_q[NT][4], half_k[NT][4];                  // the middle of the chunk -> what token t reads; token t -> the middle
+  const bool has_bonus = p.bonus != nullptr;
   bool fast = true;
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
     const int ch = (wave * NT + i) * 16 + c;
     const float bias = ch < p.dk ? p.decay_bias[head * p.dk + ch] : 0.f;
-    float l[4];
+    float(&l)[4] = lw[i];
 #pragma unroll
     for (int r = 0; r < 4; ++r)
       l[r] = (4 * g + r < nt && ch < p.dk) ? log_decay_of(z[i][r] + bias, p.kind, p.inv_tau) : 0.f;
-    const float s0 = l[0], s1 = s0 + l[1], s2 = s1 + l[2], s3 = s2 + l[3];
-    const float t16 = __shfl(s3, c), t32 = __shfl(s3, 16 + c), t48 = __shfl(s3, 32 + c), t64 = __shfl(s3, 48 + c);
-    const float before = g == 0 ? 0.f : g == 1 ? t16 : g == 2 ? t16 + t32 : t16 + t32 + t48;
-    mid[i] = t16 + t32;  // the sum up to the middle of the chunk
-    tot[i] = mid[i] + (t48 + t64);
-    cum[i][0] = before + s0; cum[i][1] = before + s1; cum[i][2] = before + s2; cum[i][3] = before + s3;
-    excl[i][0] = before; excl[i][1] = before + s0; excl[i][2] = before + s1; excl[i][3] = before + s2;
-    fast = fast && -mid[i] < kMaxHalfDecay && mid[i] - tot[i] < kMaxHalfDecay;
+    const float upto[4] = {l[0], l[0] + l[1], (l[0] + l[1]) + l[2], (l[0] + l[1]) + (l[2] + l[3])};
+    const float after[4] = {l[1] + (l[2] + l[3]), l[2] + l[3], l[3], 0.f};
+    const float g0 = __shfl(upto[3], c), g1 = __shfl(upto[3], 16 + c), g2 = __shfl(upto[3], 32 + c), g3 = __shfl(upto[3], 48 + c);
+    const float before_g = g == 0 ? 0.f : g == 1 ? g0 : g == 2 ? g0 + g1 : g0 + g1 + g2;
+    const float after_g = g == 3 ? 0.f : g == 2 ? g3 : g == 1 ? g2 + g3 : g1 + (g2 + g3);
+    const float in_half = g == 0 ? g1 : g == 3 ? g2 : 0.f;  // the group of this half between this one and the middle
+    tot[i] = (g0 + g1) + (g2 + g3);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float upto_read = has_bonus ? (r == 0 ? 0.f : upto[r == 0 ? 0 : r - 1]) : upto[r];
+      const float from_read = has_bonus ? after[r] + l[r] : after[r];
+      read[i][r] = before_g + upto_read;
+      left[i][r] = after[r] + after_g;
+      half_q[i][r] = g < 2 ? -(from_read + in_half) : in_half + upto_read;
+      half_k[i][r] = g < 2 ? after[r] + in_half : -(in_half + upto[r]);
+    }
+    fast = fast && -(g0 + g1) < kMaxHalfDecay && -(g2 + g3) < kMaxHalfDecay;
   }
   const bool slow = __syncthreads_or(!fast);
-  const bool has_bonus = p.bonus != nullptr;
   float diag[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
@@ -316,16 +327,15 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(const MixParams p) {
       const bool live = ok && t < nt;
       const float qv = live ? T::to_float(((const S*)p.q)[(row0 + t) * p.q_stride + head * p.dk + ch]) * p.q_scale : 0.f;
       const float kv = live ? T::to_float(((const S*)p.k)[(row0 + t) * p.k_stride + head * p.dk + ch]) : 0.f;
-      const float eq = has_bonus ? excl[i][r] : cum[i][r];  // decay between the chunk's start and what token t reads
-      w_q[t * DKP + ch] = qv * expf(eq);
-      kd[r] = kv * expf(tot[i] - cum[i][r]);
+      w_q[t * DKP + ch] = qv * expf(read[i][r]);
+      kd[r] = kv * expf(left[i][r]);
       if (slow) {
         sq[t * LD + ch] = qv;
         sk[t * LD + ch] = kv;
-        sb[t * LD + ch] = cum[i][r];
+        sb[t * LD + ch] = lw[i][r];
       } else {
-        sq[t * LD + ch] = qv * expf(eq - mid[i]);
-        sk[t * LD + ch] = kv * expf(mid[i] - cum[i][r]);
+        sq[t * LD + ch] = qv * expf(half_q[i][r]);
+        sk[t * LD + ch] = kv * expf(half_k[i][r]);
       }
       diag[r] = fmaf(qv * bon, kv, diag[r]);
     }
@@ -365,9 +375,9 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(const MixParams p) {
   if (below) {
     if (slow) {
       for (int ch = 0; ch < p.dk; ++ch) {
-        const float b_from = sb[tj * LD + ch];
-        const float b_to = has_bonus ? (ti > 0 ? sb[(ti - 1) * LD + ch] : 0.f) : sb[ti * LD + ch];
-        a = fmaf(sq[ti * LD + ch] * expf(b_to - b_from), sk[tj * LD + ch], a);
+        float between = 0.f;
+        for (int t = tj + 1; t < (has_bonus ? ti : ti + 1); ++t) between += sb[t * LD + ch];
+        a = fmaf(sq[ti * LD + ch] * expf(between), sk[tj * LD + ch], a);
       }
     } else {
       a = (spart[threadIdx.x] + spart[256 + threadIdx.x]) + (spart[512 + threadIdx.x] + spart[768 + threadIdx.x]);
