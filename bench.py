@@ -102,6 +102,10 @@ def parse():
                          "+-1 % from run to run)")
     ap.add_argument("--no-pin", action="store_true", help="N > 1: do not pin the rank to its GPU's NUMA cores")
     ap.add_argument("--kernel-iters", type=int, default=224)  # 20 warm-up + 200 timed launches
+    ap.add_argument("--hybrid", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the hybrid decoder beside the "
+                         "rotary decoder at equal sizes (tools/bench_hybrid.py)")
+    ap.add_argument("--hybrid-only", default=None, help="with --hybrid: the cases whose name starts with this")
     ap.add_argument("--tiny", action="store_true", help="tiny model (plumbing check)")
     ap.add_argument("--replica-backend", default=None, choices=["nccl", "gloo"],
                     help="process-group backend of the barrier / clock between replicas (default: nccl = RCCL)")
@@ -836,6 +840,11 @@ def plan_steps(a):
 
 def main():
     a = parse()
+    if a.hybrid:
+        sys.path.insert(0, os.path.join(ROOT, "tools"))
+        import bench_hybrid
+        print(json.dumps({"hybrid": bench_hybrid.run("cuda:0", a.hybrid_only)}), flush=True)
+        return
     if a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(spawn_replicas(a))
     local_rank = int(os.environ.get("LOCAL_RANK", "0"))
