@@ -600,7 +600,7 @@ int lvllm_recurrent_scan(float* o, const void* q, const void* k, const void* v, 
  * (lvllm_head_norm_gate).  max_query_len <= 1: every sequence s owns row s alone, one fused launch, no scratch.  Otherwise
  * chunks of 16 tokens on fp32 MFMAs; o_scratch float [rows, heads, dv], workspace of
  * lvllm_recurrent_mix_workspace_bytes. */
-int64_t lvllm_recurrent_mix_workspace_bytes(int rows, int num_seqs, int heads, int dk, int max_query_len);
+int64_t lvllm_recurrent_mix_workspace_bytes(int rows, int num_seqs, int heads, int dk, int dv, int max_query_len);
 int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void* k, const void* v, int64_t q_stride,
                         int64_t k_stride, int64_t v_stride, const void* u, int64_t u_stride, const float* a_t,
                         const float* decay_bias, int rank, int kind, float inv_tau, const float* bonus, float q_scale,

@@ -818,7 +818,7 @@ void recurrent_mix(torch::Tensor& out, const torch::Tensor& q, const torch::Tens
   check_state(state, state_slots, heads * dk * dv, seq_lens.numel(), op);
   const int ns = (int)seq_lens.numel();
   if (max_query_len <= 1) TORCH_CHECK(ns == rows, op, ": a step of single tokens has one row per sequence");
-  const int64_t need = lvllm_recurrent_mix_workspace_bytes((int)rows, ns, (int)heads, (int)dk, (int)max_query_len);
+  const int64_t need = lvllm_recurrent_mix_workspace_bytes((int)rows, ns, (int)heads, (int)dk, (int)dv, (int)max_query_len);
   torch::Tensor ws, o;
   if (max_query_len > 1) {
     ws = torch::empty({need}, q.options().dtype(at::kByte));
