@@ -598,8 +598,7 @@ int lvllm_recurrent_scan(float* o, const void* q, const void* k, const void* v, 
                          const int32_t* seq_lens, int num_seqs, int heads, int dk, int dv, int dtype, void* stream);
 /* A recurrent mixer in one call: decays (lvllm_log_decay), recurrence (lvllm_recurrent_scan), per-head norm and gate
  * (lvllm_head_norm_gate).  max_query_len <= 1: every sequence s owns row s alone, one fused launch, no scratch.  Otherwise
- * chunks of 16 tokens on fp32 MFMAs; o_scratch float [rows, heads, dv], workspace of
- * lvllm_recurrent_mix_workspace_bytes. */
+ * chunks of 16 tokens on fp32 MFMAs (bfloat16 and float32), workspace of lvllm_recurrent_mix_workspace_bytes. */
 int64_t lvllm_recurrent_mix_workspace_bytes(int rows, int num_seqs, int heads, int dk, int dv, int max_query_len);
 int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void* k, const void* v, int64_t q_stride,
                         int64_t k_stride, int64_t v_stride, const void* u, int64_t u_stride, const float* a_t,
@@ -607,8 +606,7 @@ int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void
                         const void* gate, int64_t gate_stride, const float* norm_weight, int norm_head_stride, float eps,
                         float out_scale, float* state, int64_t state_stride, const int32_t* state_slots, int num_slots,
                         const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows, int heads, int dk,
-                        int dv, int max_query_len, float* o_scratch, void* workspace, int64_t workspace_bytes, int dtype,
-                        void* stream);
+                        int dv, int max_query_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 /* Causal attention over the cache of lvllm_qk_norm_cache; q [rows, heads, kpad];
  * out[row, h * vdim + d] = T(attention * sigmoid(gate[row, h]) * out_scale), gate null: no gate.  max_query_len and
  * max_seq_len bound the step's query_len and seq_lens.  bf16 with block size 16, kpad in {64, 96, 128, 192, 256} and vpad

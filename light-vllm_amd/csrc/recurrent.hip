@@ -11,14 +11,14 @@
 // Two bodies:
 //   * steps of single tokens (decode): ONE launch per mixer -- decay, state update, read-out, per-head RMS norm and gate --
 //     a workgroup per (sequence, head) that streams the head's state through registers once: HBM-bound;
-//   * everything else: chunks of 16 tokens on fp32 MFMAs; long sequences that alone would not fill the chip are cut into
-//     segments of chunks, whose states are found first.  A parallel pass (chunk_prepare_kernel) computes per (chunk, head)
-//     the decays and all that does not depend on the state: q scaled by the decay from the chunk's start, k scaled by the
-//     decay to its end, the masked 16 x 16 products inside the chunk.  A sequential pass (chunk_scan_kernel) then needs
-//     17 MFMAs per chunk and wave: its state tiles are MFMA accumulators AND, without a move, the B operands of the
+//   * everything else: the decays of all heads as one fp32-MFMA product, then chunks of 16 tokens on fp32 MFMAs
+//     (chunk_mix_kernel): per chunk the decay from its start is folded into q, the decay to its end into k; the masked
+//     16 x 16 products inside the chunk, the read-out of the state before it and the state update are matrix products, the
+//     per-head norm and gate its epilogue.  State tiles are MFMA accumulators AND, without a move, the B operands of the
 //     read-out (k-step r of a tile contracts rows {r, 4 + r, 8 + r, 12 + r}: accumulator register r of every lane).
-//   Inside a chunk the decay between two tokens is the product of two factors measured from the chunk's middle; a
-//   workgroup whose channels decay too fast for that (a factor would leave fp32's range) takes the products pair by pair.
+//     Sequences too few to fill the chip are cut into segments of chunks, whose states are found first.
+//   Inside a chunk the decay between two tokens is the product of two factors measured from the chunk's middle; channels
+//   that decay too fast for that (a factor would leave fp32's range) are left out and added pair by pair.
 //
 // Everything but the projections' results (q, k, v, the low-rank input) is fp32: decays and their logarithms, the state,
 // the read-out.  Rows are the new tokens of `num_seqs` sequences back to back (query_start_loc); a sequence whose tokens
@@ -42,37 +42,63 @@ __device__ __forceinline__ float exp_of(float x) {
   return fmaf(r, lo * 0.693147182f, r);
 }
 
+typedef float r_f32x4_t __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ r_f32x4_t mfma_f32(float a, float b, r_f32x4_t c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
 // ---- ln w [rows, channels] ---------------------------------------------------------------------------------------
-constexpr int kDecayRows = 8;
+// A workgroup per 64 rows x 128 channels; f(u) through LDS, a wave's two tiles of 16 channels against all four row tiles.
+constexpr int kDecayRows = 64, kDecayCols = 128;
 template <typename T>
 __global__ __launch_bounds__(256) void log_decay_kernel(float* __restrict__ out, const typename T::store_t* __restrict__ u,
                                                         const int64_t u_stride, const float* __restrict__ a_t,  // [rank, channels]
                                                         const float* __restrict__ bias, const int kind,
                                                         const float inv_tau, const int rows, const int rank,
                                                         const int channels) {
-  extern __shared__ float su[];  // [kDecayRows][rank]
-  const int row0 = blockIdx.y * kDecayRows;
-  const int nr = min(kDecayRows, rows - row0);
-  for (int i = threadIdx.x; i < kDecayRows * rank; i += blockDim.x) {
-    const int r = i / rank, c = i - r * rank;
-    float f = r < nr ? T::to_float(u[(row0 + r) * u_stride + c]) : 0.f;
-    su[i] = kind == kDecayNegExp ? tanhf(f) : f;
+  extern __shared__ float su[];  // [kDecayRows][ld]
+  const int rank4 = (rank + 3) & ~3, ld = rank4 + 1;
+  const int row0 = blockIdx.y * kDecayRows, nr = min(kDecayRows, rows - row0);
+  for (int i = threadIdx.x; i < kDecayRows * rank4; i += 256) {
+    const int r = i / rank4, k = i - r * rank4;
+    float f = 0.f;
+    if (r < nr && k < rank) f = T::to_float(u[(int64_t)(row0 + r) * u_stride + k]);
+    su[r * ld + k] = kind == kDecayNegExp ? tanhf(f) : f;
   }
   __syncthreads();
-  const int ch = blockIdx.x * blockDim.x + threadIdx.x;
-  if (ch >= channels) return;
-  float acc[kDecayRows];
+  const int lane = threadIdx.x & 63, g = lane >> 4, c = lane & 15;
+  const int ch0 = blockIdx.x * kDecayCols + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6) * 32 + c;
+  const float* b0 = a_t + min(ch0, channels - 1);
+  const float* b1 = a_t + min(ch0 + 16, channels - 1);
+  r_f32x4_t z[2][4];
 #pragma unroll
-  for (int r = 0; r < kDecayRows; ++r) acc[r] = 0.f;
-  for (int c = 0; c < rank; ++c) {
-    const float w = a_t[(int64_t)c * channels + ch];
+  for (int j = 0; j < 2; ++j)
 #pragma unroll
-    for (int r = 0; r < kDecayRows; ++r) acc[r] = fmaf(su[r * rank + c], w, acc[r]);
+    for (int i = 0; i < 4; ++i) z[j][i] = r_f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k0 = 0; k0 < rank4; k0 += 4) {
+    const int64_t at = (int64_t)min(k0 + g, rank - 1) * channels;  // (beyond the rank: f(u) is zero)
+    const float x0 = b0[at], x1 = b1[at];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float a = su[(16 * i + c) * ld + k0 + g];
+      z[0][i] = mfma_f32(a, x0, z[0][i]);
+      z[1][i] = mfma_f32(a, x1, z[1][i]);
+    }
   }
-  const float b = bias[ch];
 #pragma unroll
-  for (int r = 0; r < kDecayRows; ++r)
-    if (r < nr) out[(int64_t)(row0 + r) * channels + ch] = log_decay_of(acc[r] + b, kind, inv_tau);
+  for (int j = 0; j < 2; ++j) {
+    const int ch = ch0 + 16 * j;
+    if (ch >= channels) continue;
+    const float bb = bias[ch];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = 16 * i + 4 * g + r;
+        if (row < nr) out[(int64_t)(row0 + row) * channels + ch] = log_decay_of(z[j][i][r] + bb, kind, inv_tau);
+      }
+  }
 }
 
 // ---- token-by-token scan -----------------------------------------------------------------------------------------
@@ -192,15 +218,8 @@ static int launch_scan(const ScanParams& p, int num_seqs, hipStream_t s) {
 
 
 // ---- chunks of 16 tokens ------------------------------------------------------------------------------------------
-typedef float r_f32x4_t __attribute__((ext_vector_type(4)));
-__device__ __forceinline__ r_f32x4_t mfma_f32(float a, float b, r_f32x4_t c) {
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
-}
 constexpr int kChunk = 16;
 constexpr float kMaxHalfDecay = 60.f;  // ln of the largest factor measured from the middle of a chunk
-
-// per (chunk, head): floats of the workspace
-__host__ __device__ constexpr int chunk_floats(int dkp) { return 2 * kChunk * dkp + kChunk * kChunk + dkp; }
 
 struct MixParams {
   const void *q, *k, *v;  // row r, head h at r * stride + h * dk (dv)
@@ -225,234 +244,128 @@ struct MixParams {
   const float* norm_weight;
   int norm_head_stride;
   float eps, out_scale;
+  bool vec_in, vec_out;   // rows of v and gate take 4-element loads, rows of `out` 4-element stores
   // chunked body
-  float* ws;              // [chunk slots, heads, chunk_floats(dkp)]
-  float* o;               // [rows, heads, dv]
+  const float* log_decay; // [rows, heads, dk]
+  float* o;               // [rows, heads, dv], or null: the epilogue is applied where o is made
   int seg_chunks, max_segs;  // chunks per segment, segments of the longest sequence (1: not cut)
   float* seg_state;       // [segment slots, heads, dk, dv]
   float* seg_decay;       // [segment slots, heads, dkp]
 };
 
-// Chunk ci of sequence s has slot query_start_loc[s] / 16 + s + ci: unique, and monotonic in s.
-__device__ __forceinline__ int chunk_slot_base(const int32_t* qsl, int s) { return qsl[s] / kChunk + s; }
+// Segment k of sequence s has slot query_start_loc[s] / (tokens of a segment) + s + k: unique
 __device__ __forceinline__ int seg_slot_base(const MixParams& p, int s) {
   return p.query_start_loc[s] / (kChunk * p.seg_chunks) + s;
 }
 
-// One workgroup (4 waves) per (chunk slot, head); wave w owns key channels [w * 16 * NT, (w + 1) * 16 * NT).
-template <typename T, int NT>
-__global__ __launch_bounds__(256) void chunk_prepare_kernel(const MixParams p) {
-  using S = typename T::store_t;
-  constexpr int DKP = 64 * NT;
-  constexpr int LD = DKP + 4;  // row stride of the LDS images (bank spread of the 16-byte reads)
-  extern __shared__ float sm[];
-  float* sq = sm;                  // [16][LD]; before that the low-rank input f(u) [16][rank_ld]
-  float* sk = sq + kChunk * LD;    // [16][LD]
-  float* sb = sk + kChunk * LD;    // [16][LD]: ln w (slow path)
-  float* spart = sb + kChunk * LD; // [4][16][16]
-  float* sdiag = spart + 4 * 256;  // [4][16]
-  const int head = blockIdx.y;
-  int lo = 0, hi = p.num_seqs;  // the sequence that owns this chunk slot: the last s with base(s) <= slot
-  while (lo < hi) {
-    const int mid = (lo + hi) >> 1;
-    if (chunk_slot_base(p.query_start_loc, mid) <= (int)blockIdx.x) lo = mid + 1;
-    else hi = mid;
-  }
-  const int seq = lo - 1;
-  if (seq < 0) return;
-  const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
-  const int t0 = ((int)blockIdx.x - chunk_slot_base(p.query_start_loc, seq)) * kChunk;
-  if (t0 >= qlen) return;
-  const int nt = min(kChunk, qlen - t0);
-  const int64_t row0 = qbeg + t0;
-  const int lane = threadIdx.x & 63;
-  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int g = lane >> 4, c = lane & 15;
-  float* ws = p.ws + ((int64_t)blockIdx.x * p.heads + head) * chunk_floats(DKP);
-  float* w_q = ws;                       // [16 tokens][DKP]
-  float* w_k = w_q + kChunk * DKP;       // [DKP][16 tokens]
-  float* w_a = w_k + kChunk * DKP;       // [16][16]
-  float* w_end = w_a + kChunk * kChunk;  // [DKP]
-
-  // q and k of this lane (tokens 4g .. 4g + 3 of each channel tile), in flight while the decays are computed; addresses are
-  // clamped instead of predicated and the values masked when they are used
-  S qraw[NT][4], kraw[NT][4];
-#pragma unroll
-  for (int i = 0; i < NT; ++i) {
-    const int chc = min((wave * NT + i) * 16 + c, p.dk - 1);
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int64_t row = row0 + min(4 * g + r, nt - 1);
-      qraw[i][r] = ((const S*)p.q)[row * p.q_stride + head * p.dk + chc];
-      kraw[i][r] = ((const S*)p.k)[row * p.k_stride + head * p.dk + chc];
-    }
-  }
-  // z[token, channel] = f(u) . a_t on MFMAs: A operand lane (token = c, k = g), B operand lane (k = g, channel = c)
-  const int rank4 = (p.rank + 3) & ~3, rank_ld = rank4 + 1;
-  for (int i = threadIdx.x; i < kChunk * rank4; i += 256) {
-    const int t = i / rank4, kk = i - t * rank4;
-    float f = 0.f;
-    if (t < nt && kk < p.rank) f = T::to_float(((const S*)p.u)[(row0 + t) * p.u_stride + kk]);
-    sq[t * rank_ld + kk] = p.kind == kDecayNegExp ? tanhf(f) : f;
-  }
-  __syncthreads();
-  r_f32x4_t z[NT];
-#pragma unroll
-  for (int i = 0; i < NT; ++i) z[i] = r_f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const int64_t a_step = (int64_t)p.heads * p.dk;
-  const float* a_ch[NT];
-#pragma unroll
-  for (int i = 0; i < NT; ++i) a_ch[i] = p.a_t + head * p.dk + min((wave * NT + i) * 16 + c, p.dk - 1);
-#pragma unroll 4
-  for (int k0 = 0; k0 < rank4; k0 += 4) {
-    const float a = sq[c * rank_ld + k0 + g];
-    const int64_t at = min(k0 + g, p.rank - 1) * a_step;  // (beyond the rank: f(u) is zero)
-#pragma unroll
-    for (int i = 0; i < NT; ++i) z[i] = mfma_f32(a, a_ch[i][at], z[i]);
-  }
-  // lane (channel c of its tile, tokens 4g .. 4g + 3): ln w, then its sums over ranges of the chunk's tokens.  Every range
-  // is summed by itself: a difference of two running sums would lose the small decays behind a large one.
-  float lw[NT][4], read[NT][4], left[NT][4], h1[NT], h2[NT];  // h1, h2: the two halves; read: chunk's start -> what token t reads; left: token t -> end
-  float half_q[NT][4], half_k[NT][4];                  // the middle of the chunk -> what token t reads; token t -> the middle
-  const bool has_bonus = p.bonus != nullptr;
-  bool fast = true;
-#pragma unroll
-  for (int i = 0; i < NT; ++i) {
-    const int ch = (wave * NT + i) * 16 + c;
-    const float bias = ch < p.dk ? p.decay_bias[head * p.dk + ch] : 0.f;
-    float(&l)[4] = lw[i];
-#pragma unroll
-    for (int r = 0; r < 4; ++r)
-      l[r] = (4 * g + r < nt && ch < p.dk) ? log_decay_of(z[i][r] + bias, p.kind, p.inv_tau) : 0.f;
+// Sums of ln w over ranges of a chunk's tokens, for the lane of channel c and tokens 4g .. 4g + 3 (l).  Every range is summed
+// by itself: a difference of two running sums would lose the small decays behind a large one.
+struct ChunkSums {
+  float h1, h2;              // the chunk's two halves
+  float read[4], left[4];    // chunk's start -> what token t reads; token t -> end
+  float half_q[4], half_k[4];  // the middle of the chunk -> what token t reads; token t -> the middle
+  __device__ __forceinline__ ChunkSums(const float (&l)[4], int g, int c, bool has_bonus) {
     const float upto[4] = {l[0], l[0] + l[1], (l[0] + l[1]) + l[2], (l[0] + l[1]) + (l[2] + l[3])};
     const float after[4] = {l[1] + (l[2] + l[3]), l[2] + l[3], l[3], 0.f};
     const float g0 = __shfl(upto[3], c), g1 = __shfl(upto[3], 16 + c), g2 = __shfl(upto[3], 32 + c), g3 = __shfl(upto[3], 48 + c);
     const float before_g = g == 0 ? 0.f : g == 1 ? g0 : g == 2 ? g0 + g1 : g0 + g1 + g2;
     const float after_g = g == 3 ? 0.f : g == 2 ? g3 : g == 1 ? g2 + g3 : g1 + (g2 + g3);
     const float in_half = g == 0 ? g1 : g == 3 ? g2 : 0.f;  // the group of this half between this one and the middle
-    h1[i] = g0 + g1;
-    h2[i] = g2 + g3;
+    h1 = g0 + g1;
+    h2 = g2 + g3;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const float upto_read = has_bonus ? (r == 0 ? 0.f : upto[r == 0 ? 0 : r - 1]) : upto[r];
       const float from_read = has_bonus ? after[r] + l[r] : after[r];
-      read[i][r] = before_g + upto_read;
-      left[i][r] = after[r] + after_g;
-      half_q[i][r] = g < 2 ? -(from_read + in_half) : in_half + upto_read;
-      half_k[i][r] = g < 2 ? after[r] + in_half : -(in_half + upto[r]);
-    }
-    fast = fast && -h1[i] < kMaxHalfDecay && -h2[i] < kMaxHalfDecay;
-  }
-  const bool slow = __syncthreads_or(!fast);  // (the low-rank input in LDS has been read)
-  float diag[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-  for (int i = 0; i < NT; ++i) {
-    const int ch = (wave * NT + i) * 16 + c;
-    const bool ok = ch < p.dk;
-    const float bon = (has_bonus && ok) ? p.bonus[head * p.dk + ch] : 0.f;
-    const float to_mid = exp_of(h1[i]), from_mid = exp_of(h2[i]);
-    float kd[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = 4 * g + r;
-      const bool live = ok && t < nt;
-      const float qv = live ? T::to_float(qraw[i][r]) * p.q_scale : 0.f;
-      const float kv = live ? T::to_float(kraw[i][r]) : 0.f;
-      if (slow) {
-        w_q[t * DKP + ch] = qv * exp_of(read[i][r]);
-        kd[r] = kv * exp_of(left[i][r]);
-        sq[t * LD + ch] = qv;
-        sk[t * LD + ch] = kv;
-        sb[t * LD + ch] = lw[i][r];
-      } else {
-        const float qh = qv * exp_of(half_q[i][r]), kh = kv * exp_of(half_k[i][r]);
-        w_q[t * DKP + ch] = qh * to_mid;
-        kd[r] = kh * from_mid;
-        sq[t * LD + ch] = qh;
-        sk[t * LD + ch] = kh;
-      }
-      diag[r] = fmaf(qv * bon, kv, diag[r]);
-    }
-    *reinterpret_cast<float4*>(w_k + ch * kChunk + 4 * g) = float4{kd[0], kd[1], kd[2], kd[3]};
-    if (g == 0) w_end[ch] = exp_of(h1[i] + h2[i]);
-  }
-  if (has_bonus) {
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-#pragma unroll
-      for (int m = 1; m < 16; m <<= 1) diag[r] += __shfl_xor(diag[r], m);
-      if (c == 0) sdiag[wave * 16 + 4 * g + r] = diag[r];
+      read[r] = before_g + upto_read;
+      left[r] = after[r] + after_g;
+      half_q[r] = g < 2 ? -(from_read + in_half) : in_half + upto_read;
+      half_k[r] = g < 2 ? after[r] + in_half : -(in_half + upto[r]);
     }
   }
-  if (!slow) {
-    // this wave's channels only: what it wrote itself, no barrier needed for other waves' parts
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    r_f32x4_t a4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int ch0 = (wave * NT + i) * 16 + 4 * g;
-      const float4 qa = *reinterpret_cast<const float4*>(sq + c * LD + ch0);
-      const float4 kb = *reinterpret_cast<const float4*>(sk + c * LD + ch0);
-      a4 = mfma_f32(qa.x, kb.x, a4);
-      a4 = mfma_f32(qa.y, kb.y, a4);
-      a4 = mfma_f32(qa.z, kb.z, a4);
-      a4 = mfma_f32(qa.w, kb.w, a4);
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) spart[wave * 256 + (4 * g + r) * 16 + c] = a4[r];
-  }
-  __syncthreads();
-  const int ti = threadIdx.x >> 4, tj = threadIdx.x & 15;
-  const bool below = has_bonus ? tj < ti : tj <= ti;
-  float a = 0.f;
-  if (below) {
-    if (slow) {
-      for (int ch = 0; ch < p.dk; ++ch) {
-        float between = 0.f;
-        for (int t = tj + 1; t < (has_bonus ? ti : ti + 1); ++t) between += sb[t * LD + ch];
-        a = fmaf(sq[ti * LD + ch] * exp_of(between), sk[tj * LD + ch], a);
-      }
-    } else {
-      a = (spart[threadIdx.x] + spart[256 + threadIdx.x]) + (spart[512 + threadIdx.x] + spart[768 + threadIdx.x]);
-    }
-  } else if (has_bonus && ti == tj) {
-    a = (sdiag[ti] + sdiag[16 + ti]) + (sdiag[32 + ti] + sdiag[48 + ti]);
-  }
-  w_a[threadIdx.x] = a;
+};
+
+__host__ __device__ constexpr int mix_smem_floats(int NT, int NV) {
+  return 4 * kChunk * (64 * NT + 4) + 4 * 256 + 4 * kChunk + 5 * kChunk * (16 * NV + 4) + 4 * NT;
 }
 
-// One workgroup per (sequence, head, 16 * NV value columns), walking chunks in order.  Wave w holds state rows
-// [w * 16 * NT, (w + 1) * 16 * NT) as accumulator tiles; the four waves' partial read-outs meet in LDS.
-// Sequences too few to fill the chip are cut into segments of seg_chunks chunks:
-//   kScanWhole     no segments: the state comes from the slot and goes back there;
-//   kScanStates    each segment but the last, from a zero state: its last state and the product of its decays;
-//   (chunk_combine_kernel turns those into every segment's first state)
-//   kScanSegments  each segment from its first state; the last one stores the slot.
-enum { kScanWhole, kScanStates, kScanSegments };
-template <typename T, int NT, int NV, int MODE>
-__global__ __launch_bounds__(256) void chunk_scan_kernel(const MixParams p) {
+// N neighbouring elements as loaded
+template <typename T, int N>
+struct Packed {
+  using S = typename T::store_t;
+  static constexpr int W = sizeof(S) == 4 ? N : (N + 1) / 2;
+  uint32_t w[W];
+  // elements col .. of a row of n (beyond it the last one); `vec`: 4-element loads are aligned
+  __device__ __forceinline__ void load(const S* row, int col, int n, bool vec) {
+    if constexpr (N >= 4) {
+      if (vec && col + N <= n) {
+        constexpr int V = W * 4 / N;  // words per 4 elements
+#pragma unroll
+        for (int j = 0; j < N / 4; ++j) {
+          if constexpr (V == 2) {
+            const uint2 x = *reinterpret_cast<const uint2*>(row + col + 4 * j);
+            w[2 * j] = x.x; w[2 * j + 1] = x.y;
+          } else {
+            const uint4 x = *reinterpret_cast<const uint4*>(row + col + 4 * j);
+            w[4 * j] = x.x; w[4 * j + 1] = x.y; w[4 * j + 2] = x.z; w[4 * j + 3] = x.w;
+          }
+        }
+        return;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+      const S x = row[min(col + j, n - 1)];
+      if constexpr (sizeof(S) == 4) w[j] = __builtin_bit_cast(uint32_t, x);
+      else w[j / 2] = j % 2 == 0 ? (uint32_t)x : w[j / 2] | ((uint32_t)x << 16);
+    }
+  }
+  __device__ __forceinline__ float at(int j) const {
+    if constexpr (sizeof(S) == 4) return __builtin_bit_cast(float, w[j]);
+    else return T::to_float((uint16_t)(w[j / 2] >> (16 * (j & 1))));
+  }
+};
+
+// One workgroup per (sequence, head, slice of 16 * NV value columns, segment), walking its chunks in order.  Wave w owns key
+// channels [w * 16 * NT, (w + 1) * 16 * NT): it scales q and k there, holds those rows of the state as accumulator tiles and
+// forms partial in-chunk products and read-outs, which meet in LDS.  A lane loads channel c, tokens 4g .. 4g + 3 of a tile:
+// scaled k is then the A operand of the state update as it is; q goes through LDS.
+//   STATES: from a zero state, no read-out: a segment's last state and the product of its decays, of all segments but the
+//   last.  Otherwise the segment's first state comes from the slot (sequences that are not cut) or from chunk_combine_kernel.
+template <typename T, int NT, int NV, bool STATES>
+__global__ __launch_bounds__(256, NT == 1 && NV <= 4 ? 3 : 2) void chunk_mix_kernel(const MixParams p) {
   using S = typename T::store_t;
   constexpr int DKP = 64 * NT;
-  __shared__ float so[MODE == kScanStates ? 1 : 2][4][kChunk][16 * NV];
+  constexpr int LD = DKP + 4;       // row strides of the LDS images (bank spread of the 16-byte reads)
+  constexpr int LO = 16 * NV + 4;
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  float* sq = sm;                   // [16][LD]: q from the middle of the chunk (fast decays: q)
+  float* sk = sq + kChunk * LD;     // [16][LD]: k to the middle (fast decays: k)
+  float* sr = sk + kChunk * LD;     // [16][LD]: q from the chunk's start
+  float* sl = sr + kChunk * LD;     // [16][LD]: ln w (fast decays)
+  float* spart = sl + kChunk * LD;  // [4 waves][16][16]: in-chunk products
+  float* sdiag = spart + 4 * 256;   // [4 waves][16]: the bonus' diagonal
+  float* so = sdiag + 4 * kChunk;   // [4 waves][16][LO]: read-outs
+  float* sv = so + 4 * kChunk * LO; // [16][LO]: values
+  int* swild = reinterpret_cast<int*>(sv + kChunk * LO);  // [4 NT]: channels of a tile that decay too fast for the factors
   const int head = blockIdx.x, v0 = blockIdx.y * 16 * NV;
-  const int seq = MODE == kScanWhole ? blockIdx.z : blockIdx.z / p.max_segs;
-  const int seg = MODE == kScanWhole ? 0 : blockIdx.z - seq * p.max_segs;
+  const bool cut = p.max_segs > 1;
+  const int seq = cut ? blockIdx.z / p.max_segs : blockIdx.z, seg = cut ? blockIdx.z - seq * p.max_segs : 0;
   const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
   if (qlen <= 0) return;
   const int all_chunks = (qlen + kChunk - 1) / kChunk;
-  const int first = MODE == kScanWhole ? 0 : seg * p.seg_chunks;
-  const int last = MODE == kScanWhole ? all_chunks : min(first + p.seg_chunks, all_chunks);
-  if (first >= all_chunks || (MODE == kScanStates && last == all_chunks)) return;
+  const int first = cut ? seg * p.seg_chunks : 0;
+  const int last = cut ? min(first + p.seg_chunks, all_chunks) : all_chunks;
+  if (first >= all_chunks || (STATES && last == all_chunks)) return;
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
   const int slot = p.state_slots[seq];
   const bool live = slot >= 0 && slot < p.num_slots;
   float* st = p.state + (int64_t)(live ? slot : 0) * p.state_stride + (int64_t)head * p.dk * p.dv;
-  const bool fresh = p.seq_lens[seq] <= qlen || !live;
-  const int64_t seg_slot = MODE == kScanWhole ? 0 : seg_slot_base(p, seq) + seg;
-  float* seg_st = MODE == kScanWhole ? nullptr : p.seg_state + (seg_slot * p.heads + head) * p.dk * p.dv;
+  const int64_t seg_slot = cut ? seg_slot_base(p, seq) + seg : 0;
+  float* seg_st = cut ? p.seg_state + (seg_slot * p.heads + head) * p.dk * p.dv : nullptr;
+  const float* from = STATES ? nullptr : cut ? seg_st : (live && p.seq_lens[seq] > qlen) ? st : nullptr;
   r_f32x4_t s[NT][NV];
 #pragma unroll
   for (int i = 0; i < NT; ++i)
@@ -461,102 +374,267 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(const MixParams p) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int row = (wave * NT + i) * 16 + 4 * g + r, col = v0 + 16 * j + c;
-        const bool in = row < p.dk && col < p.dv;
-        if (MODE == kScanWhole) s[i][j][r] = (!fresh && in) ? st[(int64_t)row * p.dv + col] : 0.f;
-        else if (MODE == kScanSegments) s[i][j][r] = in ? seg_st[(int64_t)row * p.dv + col] : 0.f;
-        else s[i][j][r] = 0.f;
+        s[i][j][r] = (from != nullptr && row < p.dk && col < p.dv) ? from[(int64_t)row * p.dv + col] : 0.f;
       }
-  float4 decays[NT];  // (kScanStates) products of this lane's rows' decays
+  const bool has_bonus = p.bonus != nullptr;
+  float bon[NT], prod[NT];
 #pragma unroll
-  for (int i = 0; i < NT; ++i) decays[i] = float4{1.f, 1.f, 1.f, 1.f};
-  const float* ws0 = p.ws + ((int64_t)chunk_slot_base(p.query_start_loc, seq) * p.heads + head) * chunk_floats(DKP);
-  const int64_t ws_step = (int64_t)p.heads * chunk_floats(DKP);
-
-  struct Frag {
-    float4 q[NT], k[NT], e[NT];
-    float a;
-    float v[NV][4];
-  };
-  auto load = [&](int ci, Frag& f) __attribute__((always_inline)) {
-    const float* ws = ws0 + ci * ws_step;
-#pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int ch0 = (wave * NT + i) * 16;
-      if (MODE != kScanStates) f.q[i] = *reinterpret_cast<const float4*>(ws + c * DKP + ch0 + 4 * g);
-      f.k[i] = *reinterpret_cast<const float4*>(ws + kChunk * DKP + (ch0 + c) * kChunk + 4 * g);
-      f.e[i] = *reinterpret_cast<const float4*>(ws + 2 * kChunk * DKP + kChunk * kChunk + ch0 + 4 * g);
-    }
-    if (MODE != kScanStates) f.a = ws[2 * kChunk * DKP + c * kChunk + 4 * g + wave];
+  for (int i = 0; i < NT; ++i) {
+    const int ch = (wave * NT + i) * 16 + c;
+    bon[i] = (has_bonus && ch < p.dk) ? p.bonus[head * p.dk + ch] : 0.f;
+    prod[i] = 1.f;
+  }
+  // epilogue of this thread: token threadIdx.x / 16 of a chunk, NV columns from d0
+  const int et = threadIdx.x >> 4, d0 = v0 + (threadIdx.x & 15) * NV;
+  const bool epilogue = !STATES && p.o == nullptr;
+  float nw[NV];
+  if constexpr (!STATES) {
 #pragma unroll
     for (int j = 0; j < NV; ++j)
+      nw[j] = (epilogue && d0 + j < p.dv) ? p.norm_weight[head * p.norm_head_stride + d0 + j] * p.out_scale : 0.f;
+  }
+
+  struct Frag {
+    S q[NT][4], k[NT][4];
+    float l[NT][4];
+    S v[STATES ? NV : 1][4];       // (STATES) tokens 4g .. 4g + 3 of column c of each tile
+    Packed<T, NV> vrow, gate;      // else: this thread's NV columns of token et
+  };
+  // addresses are clamped to the sequence's rows and the head's columns; what lies beyond is masked when it is used
+  auto load = [&](int ci, Frag& f) __attribute__((always_inline)) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int64_t row = qbeg + min(ci * kChunk + 4 * g + r, qlen - 1);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        const int ch = head * p.dk + min((wave * NT + i) * 16 + c, p.dk - 1);
+        if constexpr (!STATES) f.q[i][r] = ((const S*)p.q)[row * p.q_stride + ch];
+        f.k[i][r] = ((const S*)p.k)[row * p.k_stride + ch];
+        f.l[i][r] = p.log_decay[row * p.heads * p.dk + ch];
+      }
+      if constexpr (STATES) {
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+          f.v[j][r] = ((const S*)p.v)[row * p.v_stride + head * p.dv + min(v0 + 16 * j + c, p.dv - 1)];
+      }
+    }
+    if constexpr (!STATES) {
+      const int64_t row = qbeg + min(ci * kChunk + et, qlen - 1);
+      f.vrow.load((const S*)p.v + row * p.v_stride + head * p.dv, d0, p.dv, p.vec_in);
+      if (epilogue) f.gate.load((const S*)p.gate + row * p.gate_stride + head * p.dv, d0, p.dv, p.vec_in);
+    }
+  };
+  Frag f;
+  load(first, f);
+  for (int ci = first; ci < last; ++ci) {
+    const int nt = min(kChunk, qlen - ci * kChunk);
+    if constexpr (!STATES) {
+      float* at = sv + et * LO + (d0 - v0);
+#pragma unroll
+      for (int j = 0; j < NV; ++j) at[j] = f.vrow.at(j);
+    }
+    float kd[NT][4], end[NT];  // k scaled to the chunk's end; the chunk's decay
+    bool wild = false;
+    float diag[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const int ch = (wave * NT + i) * 16 + c;
+      float l[4], kv[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int t = ci * kChunk + 4 * g + r, col = v0 + 16 * j + c;
-        f.v[j][r] = (t < qlen && col < p.dv)
-                        ? T::to_float(((const S*)p.v)[(int64_t)(qbeg + t) * p.v_stride + head * p.dv + col]) : 0.f;
+        const bool ok = 4 * g + r < nt && ch < p.dk;
+        l[r] = ok ? f.l[i][r] : 0.f;
+        kv[r] = ok ? T::to_float(f.k[i][r]) : 0.f;
       }
-  };
-  auto step = [&](int ci, const Frag& f) __attribute__((always_inline)) {
-    float(*buf)[kChunk][16 * NV] = so[MODE == kScanStates ? 0 : ci & 1];
+      const ChunkSums cs(l, g, c, has_bonus);
+      end[i] = exp_of(cs.h1 + cs.h2);
+      if constexpr (STATES) {
 #pragma unroll
-    for (int j = 0; j < NV; ++j) {
-      if (MODE != kScanStates) {
-        r_f32x4_t o{0.f, 0.f, 0.f, 0.f};
-        // inside the chunk: this wave contracts tokens {4g + wave}
-        const float vw = wave == 0 ? f.v[j][0] : wave == 1 ? f.v[j][1] : wave == 2 ? f.v[j][2] : f.v[j][3];
-        o = mfma_f32(f.a, vw, o);
+        for (int r = 0; r < 4; ++r) kd[i][r] = kv[r] * exp_of(cs.left[r]);
+        prod[i] *= end[i];
+      } else {
+        const bool mild = -cs.h1 < kMaxHalfDecay && -cs.h2 < kMaxHalfDecay;
+        wild = wild || !mild;
+        const uint64_t fast_decays = __ballot(!mild);
+        if (lane == 0) swild[wave * NT + i] = (int)(fast_decays & 0xffff);
+        const float to_mid = exp_of(cs.h1), from_mid = exp_of(cs.h2);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = 4 * g + r;
+          const float qv = t < nt && ch < p.dk ? T::to_float(f.q[i][r]) * p.q_scale : 0.f;
+          const float qh = mild ? qv * exp_of(cs.half_q[r]) : 0.f, kh = mild ? kv[r] * exp_of(cs.half_k[r]) : 0.f;
+          sq[t * LD + ch] = qh;
+          sk[t * LD + ch] = kh;
+          float qs = qh * to_mid, ks = kh * from_mid;
+          if (!mild) {
+            qs = qv * exp_of(cs.read[r]);
+            ks = kv[r] * exp_of(cs.left[r]);
+          }
+          sr[t * LD + ch] = qs;
+          kd[i][r] = ks;
+          diag[r] = fmaf(qv * bon[i], kv[r], diag[r]);
+        }
+      }
+    }
+    // the next chunk's loads are in flight during the products and the epilogue of this one
+    const Packed<T, NV> gate = f.gate;
+    S vraw[STATES ? NV : 1][4];
+    if constexpr (STATES) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) vraw[j][r] = f.v[j][r];
+    }
+    if (ci + 1 < last) load(ci + 1, f);
+    float a = 0.f;  // A operand of the in-chunk part: row c, token 4g + wave
+    if constexpr (!STATES) {
+      if (has_bonus) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+#pragma unroll
+          for (int m = 1; m < 16; m <<= 1) diag[r] += __shfl_xor(diag[r], m);
+          if (c == 0) sdiag[wave * 16 + 4 * g + r] = diag[r];
+        }
+      }
+      // this wave's channels only: what it wrote itself, no barrier needed
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+      r_f32x4_t a4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        const int ch0 = (wave * NT + i) * 16 + 4 * g;
+        const float4 qa = *reinterpret_cast<const float4*>(sq + c * LD + ch0);
+        const float4 kb = *reinterpret_cast<const float4*>(sk + c * LD + ch0);
+        a4 = mfma_f32(qa.x, kb.x, a4);
+        a4 = mfma_f32(qa.y, kb.y, a4);
+        a4 = mfma_f32(qa.z, kb.z, a4);
+        a4 = mfma_f32(qa.w, kb.w, a4);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) spart[wave * 256 + (4 * g + r) * 16 + c] = a4[r];
+      if (__syncthreads_or(wild)) {  // the products of the channels left out above, pair by pair
 #pragma unroll
         for (int i = 0; i < NT; ++i) {
-          o = mfma_f32(f.q[i].x, s[i][j][0], o);
-          o = mfma_f32(f.q[i].y, s[i][j][1], o);
-          o = mfma_f32(f.q[i].z, s[i][j][2], o);
-          o = mfma_f32(f.q[i].w, s[i][j][3], o);
+          const int ch = (wave * NT + i) * 16 + c;
+          if (swild[wave * NT + i] >> c & 1) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              const int t = 4 * g + r;
+              const bool ok = t < nt && ch < p.dk;
+              const int64_t row = qbeg + min(ci * kChunk + t, qlen - 1);
+              const int col = head * p.dk + min(ch, p.dk - 1);
+              sq[t * LD + ch] = ok ? T::to_float(((const S*)p.q)[row * p.q_stride + col]) * p.q_scale : 0.f;
+              sk[t * LD + ch] = ok ? T::to_float(((const S*)p.k)[row * p.k_stride + col]) : 0.f;
+              sl[t * LD + ch] = ok ? p.log_decay[row * p.heads * p.dk + col] : 0.f;
+            }
+          }
+        }
+        __syncthreads();
+        const int ti = threadIdx.x >> 4, tj = threadIdx.x & 15;
+        if (tj <= ti) {
+          float sum = 0.f;
+          for (int i = 0; i < 4 * NT; ++i) {
+            for (int left = swild[i]; left != 0; left &= left - 1) {
+              const int ch = i * 16 + __builtin_ctz(left);
+              float between = 0.f;
+              for (int t = tj + 1; t < (has_bonus ? ti : ti + 1); ++t) between += sl[t * LD + ch];
+              sum = fmaf(sq[ti * LD + ch] * exp_of(between), sk[tj * LD + ch], sum);
+            }
+          }
+          spart[threadIdx.x] += sum;
+        }
+        __syncthreads();
+      }
+      const int tj = 4 * g + wave, at = c * 16 + tj;
+      if (has_bonus ? tj < c : tj <= c)
+        a = (spart[at] + spart[256 + at]) + (spart[512 + at] + spart[768 + at]);
+      else if (has_bonus && tj == c)
+        a = (sdiag[c] + sdiag[16 + c]) + (sdiag[32 + c] + sdiag[48 + c]);
+    }
+    float4 qf[NT], e[NT];
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      if constexpr (!STATES) qf[i] = *reinterpret_cast<const float4*>(sr + c * LD + (wave * NT + i) * 16 + 4 * g);
+      e[i] = float4{__shfl(end[i], 4 * g), __shfl(end[i], 4 * g + 1), __shfl(end[i], 4 * g + 2), __shfl(end[i], 4 * g + 3)};
+    }
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      float v[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[r] = STATES ? T::to_float(vraw[STATES ? j : 0][r]) : sv[(4 * g + r) * LO + 16 * j + c];
+      if constexpr (!STATES) {
+        r_f32x4_t o{0.f, 0.f, 0.f, 0.f};
+        o = mfma_f32(a, wave == 0 ? v[0] : wave == 1 ? v[1] : wave == 2 ? v[2] : v[3], o);
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+          o = mfma_f32(qf[i].x, s[i][j][0], o);
+          o = mfma_f32(qf[i].y, s[i][j][1], o);
+          o = mfma_f32(qf[i].z, s[i][j][2], o);
+          o = mfma_f32(qf[i].w, s[i][j][3], o);
         }
 #pragma unroll
-        for (int r = 0; r < 4; ++r) buf[wave][4 * g + r][16 * j + c] = o[r];
+        for (int r = 0; r < 4; ++r) so[(wave * kChunk + 4 * g + r) * LO + 16 * j + c] = o[r];
       }
 #pragma unroll
       for (int i = 0; i < NT; ++i) {
         r_f32x4_t n = s[i][j];
-        n[0] *= f.e[i].x; n[1] *= f.e[i].y; n[2] *= f.e[i].z; n[3] *= f.e[i].w;
-        n = mfma_f32(f.k[i].x, f.v[j][0], n);
-        n = mfma_f32(f.k[i].y, f.v[j][1], n);
-        n = mfma_f32(f.k[i].z, f.v[j][2], n);
-        n = mfma_f32(f.k[i].w, f.v[j][3], n);
+        n[0] *= e[i].x; n[1] *= e[i].y; n[2] *= e[i].z; n[3] *= e[i].w;
+        n = mfma_f32(kd[i][0], v[0], n);
+        n = mfma_f32(kd[i][1], v[1], n);
+        n = mfma_f32(kd[i][2], v[2], n);
+        n = mfma_f32(kd[i][3], v[3], n);
         s[i][j] = n;
       }
     }
-    if (MODE == kScanStates) {
+    if constexpr (!STATES) {
+      __syncthreads();  // (`so` is written again only behind the next chunk's first barrier)
+      float o[NV], ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < NT; ++i) {
-        decays[i].x *= f.e[i].x; decays[i].y *= f.e[i].y; decays[i].z *= f.e[i].z; decays[i].w *= f.e[i].w;
+      for (int j = 0; j < NV; ++j) {
+        const float* at = so + et * LO + (d0 - v0) + j;
+        o[j] = (at[0] + at[kChunk * LO]) + (at[2 * kChunk * LO] + at[3 * kChunk * LO]);
+        if (d0 + j < p.dv) ss = fmaf(o[j], o[j], ss);
       }
-      return;
-    }
-    __syncthreads();  // (the buffer of chunk ci + 1 is the other one: it was read before this barrier)
-    for (int i = threadIdx.x; i < kChunk * 16 * NV; i += 256) {
-      const int t = i / (16 * NV), d = i - t * 16 * NV;
-      if (ci * kChunk + t < qlen && v0 + d < p.dv)
-        p.o[((int64_t)(qbeg + ci * kChunk + t) * p.heads + head) * p.dv + v0 + d] =
-            (buf[0][t][d] + buf[1][t][d]) + (buf[2][t][d] + buf[3][t][d]);
-    }
-  };
-  Frag fa, fb;
-  load(first, fa);
-  for (int ci = first; ci < last; ci += 2) {
-    if (ci + 1 < last) load(ci + 1, fb);
-    step(ci, fa);
-    if (ci + 1 >= last) break;
-    if (ci + 2 < last) load(ci + 2, fa);
-    step(ci + 1, fb);
-  }
-  if (MODE == kScanStates && blockIdx.y == 0 && c == 0) {
+      const int64_t row = qbeg + ci * kChunk + et;
+      if (!epilogue) {
+        if (et < nt)
 #pragma unroll
-    for (int i = 0; i < NT; ++i)
-      *reinterpret_cast<float4*>(p.seg_decay + (seg_slot * p.heads + head) * DKP + (wave * NT + i) * 16 + 4 * g) = decays[i];
+          for (int j = 0; j < NV; ++j)
+            if (d0 + j < p.dv) p.o[(row * p.heads + head) * p.dv + d0 + j] = o[j];
+        continue;
+      }
+#pragma unroll
+      for (int m = 8; m >= 1; m >>= 1) ss += __shfl_xor(ss, m);
+      const float rms = 1.f / sqrtf(ss / p.dv + p.eps);
+      if (et < nt) {
+        S* out = (S*)p.out + row * p.out_stride + head * p.dv + d0;
+#pragma unroll
+        for (int j = 0; j < NV; ++j) {
+          const float zg = gate.at(j);
+          o[j] = o[j] * rms * nw[j] * (zg / (1.f + expf(-zg)));
+        }
+        if constexpr (NV >= 4) {
+          if (p.vec_out && d0 + NV <= p.dv) {
+#pragma unroll
+            for (int j = 0; j < NV; j += 4) {
+              const float w[4] = {o[j], o[j + 1], o[j + 2], o[j + 3]};
+              store4<T>(out + j, w);
+            }
+            continue;
+          }
+        }
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+          if (d0 + j < p.dv) out[j] = T::from_float(o[j]);
+      }
+    }
   }
-  if (MODE == kScanStates || (live && last == all_chunks)) {
-    float* to = MODE == kScanStates ? seg_st : st;
+  if (STATES && blockIdx.y == 0 && g == 0) {
+#pragma unroll
+    for (int i = 0; i < NT; ++i) p.seg_decay[(seg_slot * p.heads + head) * DKP + (wave * NT + i) * 16 + c] = prod[i];
+  }
+  if (STATES || (live && last == all_chunks)) {
+    float* to = STATES ? seg_st : st;
 #pragma unroll
     for (int i = 0; i < NT; ++i)
 #pragma unroll
@@ -735,45 +813,59 @@ __global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p
   }
 }
 
+// 64-channel groups of the state and 16-column tiles of a value slice
+static int key_groups(int dk) { return dk <= 64 ? 1 : dk <= 128 ? 2 : 4; }
+static int value_tiles(int dk, int dv) {
+  const int most = dk <= 128 ? 8 : 4;
+  int n = 1;
+  while (n < most && n * 16 < dv) n *= 2;
+  return n;
+}
+static int value_slices(int dk, int dv) { return (dv + 16 * value_tiles(dk, dv) - 1) / (16 * value_tiles(dk, dv)); }
+
 // Chunks per segment: sequences are cut when (sequence, head, value slice) triples alone leave CUs idle
-static int segment_chunks(int rows, int heads, int dv, int max_query_len) {
+static int segment_chunks(int rows, int heads, int dk, int dv, int max_query_len) {
   const int chunks = (max_query_len + kChunk - 1) / kChunk;
   const int64_t long_seqs = (rows + max_query_len - 1) / max_query_len;
-  const int64_t wide = long_seqs * heads * ((dv + 63) / 64);  // workgroups of 64 columns
+  const int64_t wide = long_seqs * heads * value_slices(dk, dv);
   int per = chunks;
   while (per > 8 && wide * ((chunks + per - 1) / per) < 1024) per = (per + 1) / 2;
   return per < 8 ? 8 : per;
 }
-
-template <typename T, int NT, int NV>
-static void launch_scans(const MixParams& p, hipStream_t s) {
-  const int ny = ((p.dv + 15) / 16 + NV - 1) / NV;
-  if (p.max_segs <= 1) {
-    hipLaunchKernelGGL((chunk_scan_kernel<T, NT, NV, kScanWhole>), dim3(p.heads, ny, p.num_seqs), dim3(256), 0, s, p);
-    return;
-  }
-  const dim3 grid(p.heads, ny, p.num_seqs * p.max_segs);
-  hipLaunchKernelGGL((chunk_scan_kernel<T, NT, NV, kScanStates>), grid, dim3(256), 0, s, p);
-  hipLaunchKernelGGL(chunk_combine_kernel, dim3((unsigned)(((int64_t)p.dk * p.dv + 255) / 256), p.heads, p.num_seqs),
-                     dim3(256), 0, s, p, 64 * NT);
-  hipLaunchKernelGGL((chunk_scan_kernel<T, NT, NV, kScanSegments>), grid, dim3(256), 0, s, p);
+static int64_t segment_slots(int rows, int num_seqs, int per, int max_query_len) {
+  return max_query_len <= per * kChunk ? 0 : (int64_t)rows / (kChunk * per) + num_seqs + 1;
 }
 
-template <typename T, int NT>
-static void launch_chunks(const MixParams& p, int rows, hipStream_t s) {
-  constexpr int LD = 64 * NT + 4;
-  const int images = 3 * kChunk * LD + 4 * 256 + 64, low_rank = kChunk * (((p.rank + 3) & ~3) + 1);
-  const size_t smem = (size_t)(images > low_rank ? images : low_rank) * sizeof(float);
+template <typename T, int NT, int NV>
+static void launch_mix(const MixParams& p, hipStream_t s) {
+  constexpr int smem = mix_smem_floats(NT, NV) * 4;
+  const dim3 grid(p.heads, value_slices(p.dk, p.dv), p.num_seqs * p.max_segs);
+  if (p.max_segs > 1) {
+    hipLaunchKernelGGL((chunk_mix_kernel<T, NT, NV, true>), grid, dim3(256), 0, s, p);
+    hipLaunchKernelGGL(chunk_combine_kernel, dim3((unsigned)(((int64_t)p.dk * p.dv + 255) / 256), p.heads, p.num_seqs),
+                       dim3(256), 0, s, p, 64 * NT);
+  }
   if (smem > 64 * 1024)
-    (void)hipFuncSetAttribute((const void*)chunk_prepare_kernel<T, NT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
-  hipLaunchKernelGGL((chunk_prepare_kernel<T, NT>), dim3(rows / kChunk + p.num_seqs + 1, p.heads), dim3(256), smem, s, p);
-  const int tiles = (p.dv + 15) / 16;
-  // 16 columns per workgroup fill the chip with few (segment, head) pairs; wider slices re-read q, k and the in-chunk
-  // products less often
-  const int64_t wgs = (int64_t)p.heads * p.num_seqs * p.max_segs * tiles;
-  if (wgs <= 512 || tiles == 1) launch_scans<T, NT, 1>(p, s);
-  else if (wgs <= 2048 || tiles == 2 || NT > 2) launch_scans<T, NT, 2>(p, s);
-  else launch_scans<T, NT, (NT > 2 ? 2 : 4)>(p, s);
+    (void)hipFuncSetAttribute((const void*)chunk_mix_kernel<T, NT, NV, false>, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
+  hipLaunchKernelGGL((chunk_mix_kernel<T, NT, NV, false>), grid, dim3(256), smem, s, p);
+}
+
+template <typename T>
+static void launch_mix_sized(const MixParams& p, hipStream_t s) {
+  const int nv = value_tiles(p.dk, p.dv);
+  switch (key_groups(p.dk) * 16 + nv) {
+    case 17: launch_mix<T, 1, 1>(p, s); break;
+    case 18: launch_mix<T, 1, 2>(p, s); break;
+    case 20: launch_mix<T, 1, 4>(p, s); break;
+    case 24: launch_mix<T, 1, 8>(p, s); break;
+    case 33: launch_mix<T, 2, 1>(p, s); break;
+    case 34: launch_mix<T, 2, 2>(p, s); break;
+    case 36: launch_mix<T, 2, 4>(p, s); break;
+    case 40: launch_mix<T, 2, 8>(p, s); break;
+    case 65: launch_mix<T, 4, 1>(p, s); break;
+    case 66: launch_mix<T, 4, 2>(p, s); break;
+    default: launch_mix<T, 4, 4>(p, s); break;
+  }
 }
 
 }  // namespace lvllm
@@ -784,13 +876,16 @@ extern "C" int lvllm_log_decay(float* out, const void* u, int64_t u_stride, cons
                                float inv_tau, int rows, int rank, int channels, int dtype, void* stream) {
   if (rows == 0) return 0;
   LV_CHECK(kind == kDecayLogSigmoid || kind == kDecayNegExp, "unknown decay kind");
-  LV_CHECK(rank > 0 && rank <= 1024 && channels > 0, "rank must be in 1 .. 1024");
+  LV_CHECK(rank > 0 && rank <= 512 && channels > 0, "rank must be in 1 .. 512");
+  const size_t smem = (size_t)kDecayRows * (((rank + 3) & ~3) + 1) * 4;
   const int ny = (rows + kDecayRows - 1) / kDecayRows;
   LV_CHECK(ny <= 65535, "too many rows");
   LV_DISPATCH_DTYPE(dtype, {
     using S = scalar_t::store_t;
-    hipLaunchKernelGGL((log_decay_kernel<scalar_t>), dim3((channels + 255) / 256, ny), dim3(256),
-                       (size_t)kDecayRows * rank * 4, (hipStream_t)stream, out, (const S*)u, u_stride, a_t, bias, kind,
+    if (smem > 64 * 1024)
+      (void)hipFuncSetAttribute((const void*)log_decay_kernel<scalar_t>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+    hipLaunchKernelGGL((log_decay_kernel<scalar_t>), dim3((channels + kDecayCols - 1) / kDecayCols, ny), dim3(256), smem,
+                       (hipStream_t)stream, out, (const S*)u, u_stride, a_t, bias, kind,
                        inv_tau, rows, rank, channels);
   });
   LV_LAUNCH_CHECK();
@@ -818,19 +913,12 @@ extern "C" int lvllm_recurrent_scan(float* o, const void* q, const void* k, cons
   return 0;
 }
 
-static int padded_dk(int dk) { return (dk + 63) / 64 * 64; }
-
-static int64_t segment_slots(int rows, int num_seqs, int heads, int dv, int max_query_len) {
-  const int per = segment_chunks(rows, heads, dv, max_query_len);
-  if (max_query_len <= per * kChunk) return 0;
-  return (int64_t)rows / (kChunk * per) + num_seqs + 1;
-}
-
 extern "C" int64_t lvllm_recurrent_mix_workspace_bytes(int rows, int num_seqs, int heads, int dk, int dv, int max_query_len) {
   if (max_query_len <= 1) return 0;
-  const int64_t chunks = ((int64_t)rows / kChunk + num_seqs + 1) * heads * chunk_floats(padded_dk(dk));
-  const int64_t segs = segment_slots(rows, num_seqs, heads, dv, max_query_len) * heads * ((int64_t)dk * dv + padded_dk(dk));
-  return (chunks + 3 + segs) * 4;
+  const int per = segment_chunks(rows, heads, dk, dv, max_query_len);
+  const int64_t segs = segment_slots(rows, num_seqs, per, max_query_len) * heads;
+  const int64_t o = value_slices(dk, dv) > 1 ? (int64_t)rows * heads * dv : 0;
+  return ((int64_t)rows * heads * dk + segs * ((int64_t)dk * dv + 64 * key_groups(dk)) + o) * 4;
 }
 
 extern "C" int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void* k, const void* v,
@@ -840,12 +928,12 @@ extern "C" int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q,
                                    const float* norm_weight, int norm_head_stride, float eps, float out_scale, float* state,
                                    int64_t state_stride, const int32_t* state_slots, int num_slots,
                                    const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows,
-                                   int heads, int dk, int dv, int max_query_len, float* o_scratch, void* workspace,
+                                   int heads, int dk, int dv, int max_query_len, void* workspace,
                                    int64_t workspace_bytes, int dtype, void* stream) {
   if (num_seqs == 0 || rows == 0) return 0;
   LV_CHECK(dk > 0 && dk <= 256 && dv > 0 && dv <= 1024, "key size must be in 1 .. 256, value size in 1 .. 1024");
   LV_CHECK(kind == kDecayLogSigmoid || kind == kDecayNegExp, "unknown decay kind");
-  LV_CHECK(rank > 0 && rank <= 1024, "rank must be in 1 .. 1024");
+  LV_CHECK(rank > 0 && rank <= 512, "rank must be in 1 .. 512");
   LV_CHECK(state_stride >= (int64_t)heads * dk * dv && ((dv & 3) != 0 || (state_stride & 3) == 0),
            "state slots overlap or are unaligned");
   LV_CHECK(num_seqs <= 65535 && heads <= 65535, "too many sequences or heads");
@@ -872,27 +960,31 @@ extern "C" int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q,
     LV_LAUNCH_CHECK();
     return 0;
   }
-  LV_CHECK(workspace != nullptr && o_scratch != nullptr &&
+  LV_CHECK(dtype == LVLLM_BF16 || dtype == LVLLM_F32, "bfloat16 or float32");
+  LV_CHECK(workspace != nullptr &&
                workspace_bytes >= lvllm_recurrent_mix_workspace_bytes(rows, num_seqs, heads, dk, dv, max_query_len),
            "workspace too small (see lvllm_recurrent_mix_workspace_bytes)");
-  p.ws = (float*)workspace;
-  p.o = o_scratch;
-  p.seg_chunks = segment_chunks(rows, heads, dv, max_query_len);
+  float* ws = (float*)workspace;
+  p.log_decay = ws;
+  ws += (int64_t)rows * heads * dk;
+  p.seg_chunks = segment_chunks(rows, heads, dk, dv, max_query_len);
   p.max_segs = (max_query_len + kChunk * p.seg_chunks - 1) / (kChunk * p.seg_chunks);
   LV_CHECK((int64_t)num_seqs * p.max_segs <= 65535, "too many sequences or too long portions");
-  if (p.max_segs > 1) {  // (decays first: their rows are multiples of 16 bytes)
-    p.seg_decay = p.ws + ((int64_t)rows / kChunk + num_seqs + 1) * heads * chunk_floats(padded_dk(dk));
-    p.seg_state = p.seg_decay + segment_slots(rows, num_seqs, heads, dv, max_query_len) * heads * padded_dk(dk);
-  }
-  LV_DISPATCH_DTYPE(dtype, {
-    switch (padded_dk(dk) / 64) {
-      case 1: launch_chunks<scalar_t, 1>(p, rows, s); break;
-      case 2: launch_chunks<scalar_t, 2>(p, rows, s); break;
-      case 3: launch_chunks<scalar_t, 3>(p, rows, s); break;
-      default: launch_chunks<scalar_t, 4>(p, rows, s); break;
-    }
-  });
+  const int64_t segs = segment_slots(rows, num_seqs, p.seg_chunks, max_query_len) * heads;
+  p.seg_decay = ws;
+  ws += segs * 64 * key_groups(dk);
+  p.seg_state = ws;
+  ws += segs * dk * dv;
+  if (value_slices(dk, dv) > 1) p.o = ws;
+  const int esize = dtype == LVLLM_F32 ? 4 : 2;
+  p.vec_in = ((dv | v_stride | gate_stride) & 3) == 0 && (((uintptr_t)v | (uintptr_t)gate) & (4 * esize - 1)) == 0;
+  p.vec_out = ((dv | out_stride) & 3) == 0 && ((uintptr_t)out & (4 * esize - 1)) == 0;
+  if (int rc = lvllm_log_decay((float*)workspace, u, u_stride, a_t, decay_bias, kind, inv_tau, rows, rank, heads * dk, dtype, stream))
+    return rc;
+  if (dtype == LVLLM_BF16) launch_mix_sized<BF16>(p, s);
+  else launch_mix_sized<F32>(p, s);
   LV_LAUNCH_CHECK();
-  return lvllm_head_norm_gate(out, out_stride, o_scratch, gate, gate_stride, norm_weight, norm_head_stride, eps, out_scale,
-                              rows, heads, dv, dtype, stream);
+  if (p.o == nullptr) return 0;
+  return lvllm_head_norm_gate(out, out_stride, p.o, gate, gate_stride, norm_weight, norm_head_stride, eps, out_scale, rows,
+                              heads, dv, dtype, stream);
 }

@@ -819,11 +819,8 @@ void recurrent_mix(torch::Tensor& out, const torch::Tensor& q, const torch::Tens
   const int ns = (int)seq_lens.numel();
   if (max_query_len <= 1) TORCH_CHECK(ns == rows, op, ": a step of single tokens has one row per sequence");
   const int64_t need = lvllm_recurrent_mix_workspace_bytes((int)rows, ns, (int)heads, (int)dk, (int)dv, (int)max_query_len);
-  torch::Tensor ws, o;
-  if (max_query_len > 1) {
-    ws = torch::empty({need}, q.options().dtype(at::kByte));
-    o = torch::empty({rows, heads, dv}, q.options().dtype(at::kFloat));
-  }
+  torch::Tensor ws;
+  if (need > 0) ws = torch::empty({need}, q.options().dtype(at::kByte));
   check(lvllm_recurrent_mix(out.data_ptr(), out.stride(0), q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0),
                             k.stride(0), v.stride(0), u.data_ptr(), u.stride(0), a_t.data_ptr<float>(),
                             decay_bias.data_ptr<float>(), (int)rank, (int)kind, (float)inv_tau,
@@ -831,8 +828,7 @@ void recurrent_mix(torch::Tensor& out, const torch::Tensor& q, const torch::Tens
                             norm_weight.data_ptr<float>(), shared ? 0 : (int)dv, (float)eps, (float)out_scale,
                             state.data_ptr<float>(), state.stride(0), state_slots.data_ptr<int>(), (int)state.size(0),
                             query_start_loc.data_ptr<int>(), seq_lens.data_ptr<int>(), ns, (int)rows, (int)heads, (int)dk,
-                            (int)dv, (int)max_query_len, o.defined() ? o.data_ptr<float>() : nullptr,
-                            ws.defined() ? ws.data_ptr() : nullptr, need, dtype_code(q, op), current_stream(q)));
+                            (int)dv, (int)max_query_len, ws.defined() ? ws.data_ptr() : nullptr, need, dtype_code(q, op), current_stream(q)));
 }
 
 }  // namespace
