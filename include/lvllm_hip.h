@@ -270,6 +270,7 @@ int lvllm_stream_gemm(void* y, const void* x, const void* w_packed, const void* 
  * multiplies by T(T(silu(gate)) * up) (silu_and_mul fused into the down projection);
  * act = 2 -> W rows are [gate (N/2) | up (N/2)] and y is [M, N/2] = silu_and_mul of the projection,
  * applied in the epilogue (N % 32 == 0, K not split over workgroups, no partial_out);
+ * act = 5 -> y = max(X.W^T, 0)^2 (lvllm_relu_squared of the projection, bit for bit; no partial_out);
  * partial_out != 0 -> the fp32 partial sums [ksplit, M, N] stay in `workspace` (at least
  * max(ksplit,1)*M*N*4 bytes), y is not written, *ksplit_out = number of partials. */
 int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const void* bias, int M, int N,

@@ -174,6 +174,12 @@ __device__ __forceinline__ void store4(typename T::store_t* p, const float (&v)[
   }
 }
 
+// max(x, 0)^2
+__device__ __forceinline__ float relu_squared_of(float x) {
+  const float v = fmaxf(x, 0.f);
+  return v * v;
+}
+
 // The sequence that owns `row` of a step's token batch: the s with query_start_loc[s] <= row < query_start_loc[s + 1],
 // num_seqs for rows past the last sequence (padding).  Sequences without tokens own nothing.
 __device__ __forceinline__ int find_seq(const int32_t* __restrict__ query_start_loc, int num_seqs, int row) {

@@ -673,6 +673,15 @@ __global__ __launch_bounds__(256) void chunk_combine_kernel(const MixParams p, c
 }
 
 // ---- single tokens -------------------------------------------------------------------------------------------------
+// state that is not touched again before the next step: past the caches
+__device__ __forceinline__ float4 load_stream(const float* p) {
+  const r_f32x4_t v = __builtin_nontemporal_load(reinterpret_cast<const r_f32x4_t*>(p));
+  return float4{v[0], v[1], v[2], v[3]};
+}
+__device__ __forceinline__ void store_stream(float* p, float4 v) {
+  __builtin_nontemporal_store(r_f32x4_t{v.x, v.y, v.z, v.w}, reinterpret_cast<r_f32x4_t*>(p));
+}
+
 // One workgroup per (head, sequence), sequence s owning row s.  Thread (rg, cg): state columns 4 cg .. 4 cg + 3 of rows
 // rg, rg + RG, ...  With PRE > 0 the thread's PRE state rows are loaded before anything else, so that the whole state is in
 // flight while the decays are computed; PRE = 0 takes any size.
@@ -680,9 +689,7 @@ template <typename T, int PRE>
 __global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p) {
   using S = typename T::store_t;
   extern __shared__ float sm[];
-  const int head = blockIdx.x, seq = blockIdx.y;
-  const int row = p.query_start_loc[seq];
-  if (p.query_start_loc[seq + 1] - row != 1) return;
+  const int head = blockIdx.x, seq = blockIdx.y, row = seq;
   const int dk = p.dk, dv = p.dv;
   const int slot = p.state_slots[seq];
   const bool live = slot >= 0 && slot < p.num_slots;
@@ -699,7 +706,7 @@ __global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p
     for (int i = 0; i < PRE; ++i) {
       pre[i] = float4{0.f, 0.f, 0.f, 0.f};
       const int r = rg + i * rgs;
-      if (!fresh && rg < rgs && r < dk) pre[i] = *reinterpret_cast<const float4*>(st + (int64_t)r * dv + 4 * cg0);
+      if (!fresh && rg < rgs && r < dk) pre[i] = load_stream(st + (int64_t)r * dv + 4 * cg0);
     }
   }
   float* sq = sm;            // [dk]
@@ -758,7 +765,7 @@ __global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p
           const float4 rd = has_bonus ? s : n;
           acc.x = fmaf(q, rd.x, acc.x); acc.y = fmaf(q, rd.y, acc.y);
           acc.z = fmaf(q, rd.z, acc.z); acc.w = fmaf(q, rd.w, acc.w);
-          if (live) *reinterpret_cast<float4*>(st + (int64_t)r * dv + 4 * cg0) = n;
+          if (live) store_stream(st + (int64_t)r * dv + 4 * cg0, n);
         }
       }
       *reinterpret_cast<float4*>(so + rg * dv + 4 * cg0) = acc;
@@ -823,13 +830,16 @@ static int value_tiles(int dk, int dv) {
 }
 static int value_slices(int dk, int dv) { return (dv + 16 * value_tiles(dk, dv) - 1) / (16 * value_tiles(dk, dv)); }
 
-// Chunks per segment: sequences are cut when (sequence, head, value slice) triples alone leave CUs idle
+constexpr int mix_wgs_per_cu(int NT, int NV) { return NT == 1 && NV <= 4 ? 3 : 2; }  // (registers; the LDS holds as many)
+
+// Chunks per segment: sequences are cut when (sequence, head, value slice) triples alone leave CUs idle, into as many
+// segments as run at once
 static int segment_chunks(int rows, int heads, int dk, int dv, int max_query_len) {
   const int chunks = (max_query_len + kChunk - 1) / kChunk;
   const int64_t long_seqs = (rows + max_query_len - 1) / max_query_len;
   const int64_t wide = long_seqs * heads * value_slices(dk, dv);
-  int per = chunks;
-  while (per > 8 && wide * ((chunks + per - 1) / per) < 1024) per = (per + 1) / 2;
+  const int64_t segs = 256 * mix_wgs_per_cu(key_groups(dk), value_tiles(dk, dv)) / wide;
+  const int per = segs < 2 ? chunks : (int)((chunks + segs - 1) / segs);
   return per < 8 ? 8 : per;
 }
 static int64_t segment_slots(int rows, int num_seqs, int per, int max_query_len) {

@@ -18,7 +18,7 @@
 //     a small second kernel adds them (and the bias).
 // Loads outside the problem (k-steps past K, tiles past N) use an out-of-range buffer offset and
 // return zeros without touching memory, so the loop is branch-free.
-// Epilogues (act): 0 plain (+ bias); 2 SwiGLU over (gate, up) tile pairs -> [M, N/2]; 3 greedy arg-max
+// Epilogues (act): 0 plain (+ bias); 5 squared ReLU; 2 SwiGLU over (gate, up) tile pairs -> [M, N/2]; 3 greedy arg-max
 // over N -> int64 [M] (no logits written); act = 1 applies SwiGLU while loading X (kept for small shapes).
 // The same file holds the W8A8 variant (fp8 weights, X quantised while the fragments are built) and,
 // at the end, the 65..256-row kernel that moves X through LDS instead of registers.
@@ -205,6 +205,10 @@ __global__ __launch_bounds__(kGemmWaves * 64, 2) void skinny_gemm_kernel(
         if (bias != nullptr) {
 #pragma unroll
           for (int r = 0; r < 4; ++r) sum[r] += T::to_float(bias[n0 + r]);
+        }
+        if (act == 5) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) sum[r] = relu_squared_of(T::to_float(T::from_float(sum[r])));
         }
         uint2 o;
         o.x = (uint32_t)T::from_float(sum[0]) | ((uint32_t)T::from_float(sum[1]) << 16);
@@ -669,7 +673,7 @@ __global__ void skinny_gemm_reduce_kernel(typename T::store_t* __restrict__ y,
                                           const typename T::store_t* __restrict__ bias,
                                           const int64_t MN, const int N, const int ksplit,
                                           const float* __restrict__ x_scale = nullptr,
-                                          const float* __restrict__ w_scale = nullptr) {
+                                          const float* __restrict__ w_scale = nullptr, const bool relu2 = false) {
   const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * 4;
   if (i >= MN) return;
   g_f32x4_t sum = *reinterpret_cast<const g_f32x4_t*>(partial + i);
@@ -682,6 +686,10 @@ __global__ void skinny_gemm_reduce_kernel(typename T::store_t* __restrict__ y,
     const int n = (int)(i % N);
 #pragma unroll
     for (int r = 0; r < 4; ++r) sum[r] += T::to_float(bias[n + r]);
+  }
+  if (relu2) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) sum[r] = relu_squared_of(T::to_float(T::from_float(sum[r])));
   }
   uint2 o;
   o.x = (uint32_t)T::from_float(sum[0]) | ((uint32_t)T::from_float(sum[1]) << 16);
@@ -1098,7 +1106,8 @@ extern "C" int lvllm_skinny_gemm_argmax(int64_t* tokens, const void* x, const vo
 // `act` = 1: X rows are [gate (K) | up (K)] and the kernel multiplies W by silu(gate)*up
 // (the SwiGLU activation fused into the down projection); `act` = 2: W rows are [gate (N/2) | up (N/2)]
 // and y [M, N/2] = silu(X.gate^T) * (X.up^T), the activation applied in the epilogue (the gate_up
-// projection and silu_and_mul in one launch, bit-identical to the pair); `partial_out` != 0: leave the fp32
+// projection and silu_and_mul in one launch, bit-identical to the pair); `act` = 5: y = max(X.W^T, 0)^2 (bit-identical to
+// lvllm_relu_squared of the plain projection); `partial_out` != 0: leave the fp32
 // split-K partials in `workspace` ([ksplit, M, N]) and do not write y (the caller's next kernel
 // sums them: lvllm_fused_add_rms_norm_splitk).  *ksplit_out receives the number of partials.
 extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const void* bias, int M, int N,
@@ -1123,6 +1132,7 @@ extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const
     set_error("lvllm_skinny_gemm: shape outside the kernel's envelope");
     return 3;
   }
+  LV_CHECK(act >= 0 && (act <= 3 || act == 5) && !(act == 5 && partial_out), "unknown epilogue");
   const int total_steps = K / 32;
   const int cap = kGemmWaves * max_steps_per_wave(M);
   int ksplit = (total_steps + cap - 1) / cap;
@@ -1229,10 +1239,10 @@ extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const
     const int grid = (int)((MN / 4 + threads - 1) / threads);
     if (dtype == LVLLM_BF16)
       hipLaunchKernelGGL((skinny_gemm_reduce_kernel<BF16>), dim3(grid), dim3(threads), 0, s, (uint16_t*)y,
-                         partial, (const uint16_t*)bias, MN, N, ksplit);
+                         partial, (const uint16_t*)bias, MN, N, ksplit, nullptr, nullptr, act == 5);
     else
       hipLaunchKernelGGL((skinny_gemm_reduce_kernel<F16>), dim3(grid), dim3(threads), 0, s, (uint16_t*)y,
-                         partial, (const uint16_t*)bias, MN, N, ksplit);
+                         partial, (const uint16_t*)bias, MN, N, ksplit, nullptr, nullptr, act == 5);
     LV_LAUNCH_CHECK();
   }
   return 0;

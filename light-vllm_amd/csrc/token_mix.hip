@@ -86,8 +86,8 @@ __global__ void add_dyt_shift_mix_kernel(float* __restrict__ x_out, const float*
                                          const int num_slots, const int32_t* __restrict__ query_start_loc,
                                          const int32_t* __restrict__ seq_lens, const int num_seqs, const int rows,
                                          const int width) {
-  const int row = blockIdx.y;
-  const int c0 = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+  const int row = blockIdx.x;
+  const int c0 = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
   if (c0 >= width) return;
   const float a = alpha[0];
   const int64_t base = (int64_t)row * width + c0;
@@ -160,13 +160,11 @@ __global__ void relu_squared_kernel(typename T::store_t* out, const typename T::
     uint16_t* d = reinterpret_cast<uint16_t*>(&o);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      const float v = fmaxf(T::to_float(s[j]), 0.f);
-      d[j] = T::from_float(v * v);
+      d[j] = T::from_float(relu_squared_of(T::to_float(s[j])));
     }
     *reinterpret_cast<uint4*>(out + i) = o;
   } else {
-    const float v = fmaxf(T::to_float(x[i]), 0.f);
-    out[i] = T::from_float(v * v);
+    out[i] = T::from_float(relu_squared_of(T::to_float(x[i])));
   }
 }
 
@@ -389,18 +387,18 @@ extern "C" int lvllm_add_dyt_shift_mix(float* x_out, const float* x_in, const vo
                                        const int32_t* state_slots, int num_slots, const int32_t* query_start_loc,
                                        const int32_t* seq_lens, int num_seqs, int rows, int width, int dtype, void* stream) {
   if (rows == 0) return 0;
-  LV_CHECK(rows > 0 && rows <= 65535 && width > 0 && num_mix > 0, "1 .. 65535 rows, positive width and mixes");
+  LV_CHECK(rows > 0 && width > 0 && num_mix > 0, "positive rows, width and mixes");
   LV_CHECK(x_out != x_in, "x_out must not be x_in: neighbouring rows read x_in");
   LV_CHECK((y == nullptr && partials == nullptr) || x_out != nullptr, "an addend needs x_out");
   LV_DISPATCH_DTYPE(dtype, {
     using S = scalar_t::store_t;
     const auto p = proj_out<scalar_t>(y, partials, num_partials, (int64_t)rows * width);
     if (width % 4 == 0) {
-      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 4>), dim3((width / 4 + 255) / 256, rows), dim3(256), 0,
+      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 4>), dim3(rows, (width / 4 + 255) / 256), dim3(256), 0,
                          (hipStream_t)stream, x_out, x_in, p, (S*)mix, mu, num_mix, alpha, weight, bias, carried,
                          carried_stride, state_slots, num_slots, query_start_loc, seq_lens, num_seqs, rows, width);
     } else {
-      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 1>), dim3((width + 255) / 256, rows), dim3(256), 0,
+      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 1>), dim3(rows, (width + 255) / 256), dim3(256), 0,
                          (hipStream_t)stream, x_out, x_in, p, (S*)mix, mu, num_mix, alpha, weight, bias, carried,
                          carried_stride, state_slots, num_slots, query_start_loc, seq_lens, num_seqs, rows, width);
     }

@@ -217,6 +217,23 @@ torch::Tensor skinny_linear_packed_swiglu(const torch::Tensor& x, const torch::T
   return y;
 }
 
+// y = max(x . w^T, 0)^2: the squared-ReLU feed-forward's up projection in one launch, bit-identical to the two
+torch::Tensor skinny_linear_packed_relu_squared(const torch::Tensor& x, const torch::Tensor& w_packed, int64_t N, int64_t K) {
+  TORCH_CHECK(x.dim() == 2 && x.size(1) == K && w_packed.numel() == N * K, "skinny_linear_packed_relu_squared: bad shapes");
+  TORCH_CHECK(skinny_ok(x, w_packed, std::nullopt),
+              "skinny_linear_packed_relu_squared: M <= 64 rows of bf16/f16 on the GPU only");
+  const int64_t M = x.size(0);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
+  auto y = torch::empty({M, N}, x.options());
+  const int64_t ws_bytes = lvllm_skinny_gemm_workspace_bytes((int)M, (int)N, (int)K);
+  torch::Tensor ws;
+  if (ws_bytes > 0) ws = torch::empty({ws_bytes / 4}, x.options().dtype(torch::kFloat));
+  check(lvllm_skinny_gemm_ex(y.data_ptr(), x.data_ptr(), w_packed.data_ptr(), nullptr, (int)M, (int)N, (int)K, x.stride(0),
+                             dtype_code(x, "skinny_linear_packed_relu_squared"), 1, 5, 0, nullptr,
+                             ws_bytes > 0 ? ws.data_ptr() : nullptr, ws_bytes, current_stream(x)));
+  return y;
+}
+
 // A projection that leaves its fp32 split-K partials [S, M, N] for fused_add_rms_norm_splitk
 // instead of reducing them itself.  swiglu: x = [gate | up] ([M, 2K]) and the activation is applied
 // while loading x (bit-identical to silu_and_mul, but every workgroup redoes it for its K slice:
@@ -884,6 +901,8 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, amd) {
   amd.impl("pack_weight", torch::kCUDA, &pack_weight);
   amd.def("skinny_linear_packed_argmax(Tensor x, Tensor w_packed, int N, int K) -> Tensor");
   amd.impl("skinny_linear_packed_argmax", torch::kCUDA, &skinny_linear_packed_argmax);
+  amd.def("skinny_linear_packed_relu_squared(Tensor x, Tensor w_packed, int N, int K) -> Tensor");
+  amd.impl("skinny_linear_packed_relu_squared", torch::kCUDA, &skinny_linear_packed_relu_squared);
   amd.def("stream_linear_packed(Tensor x, Tensor w_packed, Tensor? bias, int N, int K) -> Tensor");
   amd.impl("stream_linear_packed", torch::kCUDA, &stream_linear_packed);
   amd.def("skinny_linear_packed_swiglu(Tensor x, Tensor w_packed, Tensor? bias, int N, int K) -> Tensor");

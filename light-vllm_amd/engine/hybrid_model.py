@@ -61,7 +61,7 @@ def random_tensor(name: str, shape: tuple, gen: torch.Generator, device) -> torc
     if ".mu." in name:
         return torch.rand(shape, generator=gen, device=device)
     if name.endswith(".w0"):
-        return -4.0 + 2.0 * t
+        return -6.0 + 5.5 * torch.rand(shape, generator=gen, device=device)
     if name.endswith(".a2.b"):
         return 2.0 + t
     if name.endswith(".u"):

@@ -203,6 +203,9 @@ class SquaredReluMlp:
         self.down = make_weight(pad_columns(get(name + ".down")), pack)
 
     def __call__(self, h: torch.Tensor) -> torch.Tensor:
-        a = linear(h, self.up)
-        amd.relu_squared(a, a)
+        if 0 < h.shape[0] <= DECODE_ROWS and self.up.packed is not None:
+            a = amd.skinny_linear_packed_relu_squared(h, self.up.packed, self.up.N, self.up.K)
+        else:
+            a = linear(h, self.up)
+            amd.relu_squared(a, a)
         return project_to_residual(a, self.down)

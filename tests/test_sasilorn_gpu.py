@@ -108,6 +108,16 @@ def test_relu_squared(amd, dtype, n):
     close(out, sasilorn.squared_relu(x.double()), 1e-6 if dtype == F32 else 8e-3)
 
 
+@pytest.mark.parametrize("m,n,k", [(1, 64, 96), (33, 160, 256), (64, 4096, 1024), (32, 512, 14336)])
+def test_relu_squared_in_the_projection(amd, m, n, k):
+    """Bit for bit the projection followed by the activation, with K inside a workgroup and split over several."""
+    x, w = rand(m, k, dtype=BF16).to(DEV), (rand(n, k, seed=1) * k ** -0.5).bfloat16().to(DEV)
+    packed = amd.pack_weight(w)
+    want = amd.skinny_linear_packed(x, packed, None, n, k)
+    amd.relu_squared(want, want)
+    assert torch.equal(amd.skinny_linear_packed_relu_squared(x, packed, n, k), want)
+
+
 # ---- recurrences ----
 def recurrence_case(kind, seqs, heads, dk, dv, rank, spread, dtype, seed=0):
     rows = sum(n for n, _ in seqs)
