@@ -29,17 +29,17 @@ namespace lvllm {
 
 enum { kDecayLogSigmoid = 0, kDecayNegExp = 1 };
 
-__device__ __forceinline__ float log_decay_of(float z, int kind, float inv_tau) {
-  if (kind == kDecayNegExp) return -expf(fminf(z, 9.f));  // (exp(-exp(9)) is 0: a finite logarithm keeps sums finite)
-  return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau;
-}
-
-// e^x for x <= 0 (and for the bounded positive factors of a chunk): 2^(x log2 e) with the product's rounding error put back
+// e^x, |x| up to a few hundred: 2^(x log2 e) with the product's rounding error put back
 __device__ __forceinline__ float exp_of(float x) {
   const float t = x * 1.44269502e+0f;
   const float lo = fmaf(x, 1.44269502e+0f, -t) + x * 1.92596299e-8f;
   const float r = __builtin_amdgcn_exp2f(t);
   return fmaf(r, lo * 0.693147182f, r);
+}
+
+__device__ __forceinline__ float log_decay_of(float z, int kind, float inv_tau) {
+  if (kind == kDecayNegExp) return -exp_of(fminf(z, 9.f));  // (exp(-exp(9)) is 0: a finite logarithm keeps sums finite)
+  return (fminf(z, 0.f) - log1pf(exp_of(-fabsf(z)))) * inv_tau;
 }
 
 typedef float r_f32x4_t __attribute__((ext_vector_type(4)));
@@ -59,11 +59,17 @@ __global__ __launch_bounds__(256) void log_decay_kernel(float* __restrict__ out,
   extern __shared__ float su[];  // [kDecayRows][ld]
   const int rank4 = (rank + 3) & ~3, ld = rank4 + 1;
   const int row0 = blockIdx.y * kDecayRows, nr = min(kDecayRows, rows - row0);
-  for (int i = threadIdx.x; i < kDecayRows * rank4; i += 256) {
-    const int r = i / rank4, k = i - r * rank4;
-    float f = 0.f;
-    if (r < nr && k < rank) f = T::to_float(u[(int64_t)(row0 + r) * u_stride + k]);
-    su[r * ld + k] = kind == kDecayNegExp ? tanhf(f) : f;
+  for (int k = threadIdx.x & 63; k < rank4; k += 64) {
+    constexpr int N = kDecayRows / 4;
+    const int r0 = threadIdx.x >> 6;
+    typename T::store_t raw[N];  // (all of a thread's loads in flight at once)
+#pragma unroll
+    for (int i = 0; i < N; ++i) raw[i] = u[(int64_t)(row0 + min(r0 + 4 * i, nr - 1)) * u_stride + min(k, rank - 1)];
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const float f = k < rank ? T::to_float(raw[i]) : 0.f;
+      su[(r0 + 4 * i) * ld + k] = kind == kDecayNegExp ? tanhf(f) : f;
+    }
   }
   __syncthreads();
   const int lane = threadIdx.x & 63, g = lane >> 4, c = lane & 15;
@@ -75,7 +81,7 @@ __global__ __launch_bounds__(256) void log_decay_kernel(float* __restrict__ out,
   for (int j = 0; j < 2; ++j)
 #pragma unroll
     for (int i = 0; i < 4; ++i) z[j][i] = r_f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll 8
   for (int k0 = 0; k0 < rank4; k0 += 4) {
     const int64_t at = (int64_t)min(k0 + g, rank - 1) * channels;  // (beyond the rank: f(u) is zero)
     const float x0 = b0[at], x1 = b1[at];
@@ -700,6 +706,27 @@ __global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p
   const int per = min(cgs, 256);               // threads along a row
   const int rgs = 256 / per;                   // row groups
   const int rg = threadIdx.x / per, cg0 = threadIdx.x - rg * per;
+  // Loads return in order: the small operands go first, the state behind them, and both are in flight while the decays are
+  // computed.  (dk <= 256: one key channel per thread; the first 256 values, low-rank inputs and columns likewise.)
+  const int tid = threadIdx.x;
+  const int kc = head * dk + min(tid, dk - 1), vc = head * dv + min(tid, dv - 1);
+  const float u0 = T::to_float(((const S*)p.u)[(int64_t)row * p.u_stride + min(tid, p.rank - 1)]);
+  const float q0 = T::to_float(((const S*)p.q)[(int64_t)row * p.q_stride + kc]) * p.q_scale;
+  const float k0 = T::to_float(((const S*)p.k)[(int64_t)row * p.k_stride + kc]);
+  const float v0 = T::to_float(((const S*)p.v)[(int64_t)row * p.v_stride + vc]);
+  const float gate0 = T::to_float(((const S*)p.gate)[(int64_t)row * p.gate_stride + vc]);
+  const float weight0 = p.norm_weight[head * p.norm_head_stride + min(tid, dv - 1)];
+  const float bias0 = p.decay_bias[kc];
+  const float bonus0 = p.bonus != nullptr ? p.bonus[kc] : 0.f;
+  // z: the rank cut into parts, thread (part, channel)
+  const int parts = 256 / dk, part_len = (p.rank + parts - 1) / parts;
+  const int part = tid / dk, part_ch = tid - part * dk;
+  const float* a = p.a_t + head * dk + part_ch;
+  const int64_t a_step = (int64_t)p.heads * dk;
+  constexpr int AR = PRE == 4 ? 16 : 32;
+  float a_pre[AR];
+#pragma unroll
+  for (int i = 0; i < AR; ++i) a_pre[i] = a[min(part * part_len + i, p.rank - 1) * a_step];
   float4 pre[PRE > 0 ? PRE : 1];
   if constexpr (PRE > 0) {
 #pragma unroll
@@ -714,39 +741,37 @@ __global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p
   float* sw = sk + dk;       // [dk]
   float* su = sw + dk;       // [rank]
   float* sv = sm + ((3 * dk + p.rank + 3) & ~3);  // [dv], 16-byte aligned
-  float* so = sv + dv;       // [row groups][dv]; before that the parts of z [max(1, 256 / dk)][dk]
+  float* so = sv + dv;       // [row groups][dv]; before that the parts of z [256 / dk][dk]
   __shared__ float red[16];
   __shared__ float s_bonus;
-  for (int i = threadIdx.x; i < p.rank; i += 256) {
+  if (tid < p.rank) su[tid] = p.kind == kDecayNegExp ? tanhf(u0) : u0;
+  for (int i = tid + 256; i < p.rank; i += 256) {
     const float f = T::to_float(((const S*)p.u)[(int64_t)row * p.u_stride + i]);
     su[i] = p.kind == kDecayNegExp ? tanhf(f) : f;
   }
-  for (int i = threadIdx.x; i < dv; i += 256) sv[i] = T::to_float(((const S*)p.v)[(int64_t)row * p.v_stride + head * dv + i]);
-  for (int i = threadIdx.x; i < dk; i += 256) {
-    sq[i] = T::to_float(((const S*)p.q)[(int64_t)row * p.q_stride + head * dk + i]) * p.q_scale;
-    sk[i] = T::to_float(((const S*)p.k)[(int64_t)row * p.k_stride + head * dk + i]);
+  if (tid < dv) sv[tid] = v0;
+  for (int i = tid + 256; i < dv; i += 256) sv[i] = T::to_float(((const S*)p.v)[(int64_t)row * p.v_stride + head * dv + i]);
+  if (tid < dk) {
+    sq[tid] = q0;
+    sk[tid] = k0;
   }
   __syncthreads();
-  const int parts = dk >= 256 ? 1 : 256 / dk, part_len = (p.rank + parts - 1) / parts;  // z: the rank cut into parts
-  {
-    const int part = threadIdx.x / dk, ch = threadIdx.x - part * dk;  // (dk <= 256)
-    if (part < parts) {
-      const int r1 = min((part + 1) * part_len, p.rank);
-      const float* a = p.a_t + head * dk + ch;
-      const int64_t a_step = (int64_t)p.heads * dk;
-      float z = 0.f;
-#pragma unroll 8
-      for (int r = part * part_len; r < r1; ++r) z = fmaf(su[r], a[r * a_step], z);
-      so[part * dk + ch] = z;
-    }
+  if (part < parts) {
+    const int r0 = part * part_len, r1 = min(r0 + part_len, p.rank);
+    float z = 0.f;
+#pragma unroll
+    for (int i = 0; i < AR; ++i)
+      if (r0 + i < r1) z = fmaf(su[r0 + i], a_pre[i], z);
+    for (int r = r0 + AR; r < r1; ++r) z = fmaf(su[r], a[r * a_step], z);
+    so[part * dk + part_ch] = z;
   }
   __syncthreads();
   float bsum = 0.f;
-  for (int i = threadIdx.x; i < dk; i += 256) {
-    float z = p.decay_bias[head * dk + i];
-    for (int q = 0; q < parts; ++q) z += so[q * dk + i];
-    sw[i] = expf(log_decay_of(z, p.kind, p.inv_tau));
-    if (p.bonus != nullptr) bsum = fmaf(sq[i] * p.bonus[head * dk + i], sk[i], bsum);
+  if (tid < dk) {
+    float z = bias0;
+    for (int q = 0; q < parts; ++q) z += so[q * dk + tid];
+    sw[tid] = expf(log_decay_of(z, p.kind, p.inv_tau));
+    bsum = q0 * bonus0 * k0;
   }
   const bool has_bonus = p.bonus != nullptr;
   const float b = block_sum(bsum, red);  // (barriers: sw is visible behind it)
@@ -813,10 +838,11 @@ __global__ __launch_bounds__(256) void recurrent_decode_kernel(const MixParams p
   }
   const float r = 1.f / sqrtf(block_sum(ss, red) / dv + p.eps);
   for (int d = threadIdx.x; d < dv; d += 256) {
-    const float z = T::to_float(((const S*)p.gate)[(int64_t)row * p.gate_stride + head * dv + d]);
+    const bool first = d == tid;
+    const float z = first ? gate0 : T::to_float(((const S*)p.gate)[(int64_t)row * p.gate_stride + head * dv + d]);
+    const float w = first ? weight0 : p.norm_weight[head * p.norm_head_stride + d];
     const float silu = z / (1.f + expf(-z));
-    ((S*)p.out)[(int64_t)row * p.out_stride + head * dv + d] =
-        T::from_float(so[d] * r * p.norm_weight[head * p.norm_head_stride + d] * silu * p.out_scale);
+    ((S*)p.out)[(int64_t)row * p.out_stride + head * dv + d] = T::from_float(so[d] * r * w * silu * p.out_scale);
   }
 }
 

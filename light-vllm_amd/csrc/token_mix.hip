@@ -86,8 +86,9 @@ __global__ void add_dyt_shift_mix_kernel(float* __restrict__ x_out, const float*
                                          const int num_slots, const int32_t* __restrict__ query_start_loc,
                                          const int32_t* __restrict__ seq_lens, const int num_seqs, const int rows,
                                          const int width) {
-  const int row = blockIdx.x;
-  const int c0 = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
+  const int per_row = (width + blockDim.x * VEC - 1) / (blockDim.x * VEC);  // workgroups of a row
+  const int row = blockIdx.x / per_row;
+  const int c0 = ((blockIdx.x - row * per_row) * blockDim.x + threadIdx.x) * VEC;
   if (c0 >= width) return;
   const float a = alpha[0];
   const int64_t base = (int64_t)row * width + c0;
@@ -171,13 +172,33 @@ __global__ void relu_squared_kernel(typename T::store_t* out, const typename T::
 // VEC consecutive elements <-> floats
 template <typename T, int VEC>
 __device__ __forceinline__ void load_vec(const typename T::store_t* p, float (&v)[VEC]) {
-  if constexpr (VEC == 4) load4<T>(p, v);
-  else v[0] = T::to_float(p[0]);
+  if constexpr (VEC == 8) {
+    static_assert(sizeof(typename T::store_t) == 2, "16-byte pieces of 16-bit elements");
+    const uint4 a = *reinterpret_cast<const uint4*>(p);
+    const uint32_t w[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      v[2 * j] = T::to_float((uint16_t)w[j]);
+      v[2 * j + 1] = T::to_float((uint16_t)(w[j] >> 16));
+    }
+  } else if constexpr (VEC == 4) {
+    load4<T>(p, v);
+  } else {
+    v[0] = T::to_float(p[0]);
+  }
 }
 template <typename T, int VEC>
 __device__ __forceinline__ void store_vec(typename T::store_t* p, const float (&v)[VEC]) {
-  if constexpr (VEC == 4) store4<T>(p, v);
-  else p[0] = T::from_float(v[0]);
+  if constexpr (VEC == 8) {
+    uint32_t w[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) w[j] = (uint32_t)T::from_float(v[2 * j]) | ((uint32_t)T::from_float(v[2 * j + 1]) << 16);
+    *reinterpret_cast<uint4*>(p) = uint4{w[0], w[1], w[2], w[3]};
+  } else if constexpr (VEC == 4) {
+    store4<T>(p, v);
+  } else {
+    p[0] = T::from_float(v[0]);
+  }
 }
 template <int L>
 __device__ __forceinline__ float group_sum(float v) {  // over L neighbouring lanes
@@ -235,11 +256,12 @@ __global__ __launch_bounds__(256) void qk_norm_cache_kernel(
 #pragma unroll
     for (int j = 0; j < VEC; ++j) ss += f[j] * f[j];
   }
+  const bool one_pass = dim <= L * VEC;  // (the values are still in registers)
   const float r = 1.f / sqrtf(group_sum<L>(ss) / dim + eps);
   for (int d = lane * VEC; d < kpad; d += L * VEC) {
     float o[VEC];
     if (d < dim) {
-      load_vec<T, VEC>(src + d, f);
+      if (!one_pass) load_vec<T, VEC>(src + d, f);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) o[j] = f[j] * r * wt[d + j];
     } else {
@@ -394,11 +416,11 @@ extern "C" int lvllm_add_dyt_shift_mix(float* x_out, const float* x_in, const vo
     using S = scalar_t::store_t;
     const auto p = proj_out<scalar_t>(y, partials, num_partials, (int64_t)rows * width);
     if (width % 4 == 0) {
-      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 4>), dim3(rows, (width / 4 + 255) / 256), dim3(256), 0,
+      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 4>), dim3((unsigned)rows * ((width + 1023) / 1024)), dim3(256), 0,
                          (hipStream_t)stream, x_out, x_in, p, (S*)mix, mu, num_mix, alpha, weight, bias, carried,
                          carried_stride, state_slots, num_slots, query_start_loc, seq_lens, num_seqs, rows, width);
     } else {
-      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 1>), dim3(rows, (width + 255) / 256), dim3(256), 0,
+      hipLaunchKernelGGL((add_dyt_shift_mix_kernel<scalar_t, 1>), dim3((unsigned)rows * ((width + 255) / 256)), dim3(256), 0,
                          (hipStream_t)stream, x_out, x_in, p, (S*)mix, mu, num_mix, alpha, weight, bias, carried,
                          carried_stride, state_slots, num_slots, query_start_loc, seq_lens, num_seqs, rows, width);
     }
@@ -444,29 +466,30 @@ extern "C" int lvllm_qk_norm_cache(void* q_out, void* key_cache, void* value_cac
                      v_block_stride * esize % 16 == 0;
   const bool vec = ((dim | row_stride) & 3) == 0 && (((uintptr_t)q | (uintptr_t)k) & (4 * esize - 1)) == 0 &&
                    (((uintptr_t)q_out | (uintptr_t)key_cache) & 15) == 0 && k_block_stride * esize % 16 == 0;
+  const bool vec8 = vec && esize == 2 && ((dim | row_stride) & 7) == 0 && (((uintptr_t)q | (uintptr_t)k) & 15) == 0;
   const int64_t items = (int64_t)rows * (heads + (tiled ? 1 : 2) * kv_heads);
   LV_CHECK(items <= INT32_MAX && kv_heads <= 65535, "too many rows");
+#define LV_QK(VEC_)                                                                                                          \
+  hipLaunchKernelGGL((qk_norm_cache_kernel<scalar_t, kL, VEC_>), grid, dim3(256), 0, (hipStream_t)stream, (S*)q_out,          \
+                     (S*)key_cache, (S*)value_cache, (const S*)q, (const S*)k, (const S*)v, row_stride, q_weight, k_weight,  \
+                     eps, rows, heads, kv_heads, dim, vdim, kpad, vpad, !tiled, slot_mapping, num_blocks * block_size,       \
+                     block_size, k_block_stride, v_block_stride)
   LV_DISPATCH_DTYPE(dtype, {
     using S = scalar_t::store_t;
-    const int lanes = lanes_for(kpad, vec ? 4 : 1);
+    constexpr int kWide = sizeof(S) == 2 ? 8 : 4;  // elements of a 16-byte piece
+    const int lanes = lanes_for(kpad, vec8 ? kWide : vec ? 4 : 1);
     const dim3 grid((unsigned)((items * lanes + 255) / 256));
     LV_LANES(lanes, {
-      if (vec)
-        hipLaunchKernelGGL((qk_norm_cache_kernel<scalar_t, kL, 4>), grid, dim3(256), 0, (hipStream_t)stream, (S*)q_out,
-                           (S*)key_cache, (S*)value_cache, (const S*)q, (const S*)k, (const S*)v, row_stride, q_weight,
-                           k_weight, eps, rows, heads, kv_heads, dim, vdim, kpad, vpad, !tiled, slot_mapping,
-                           num_blocks * block_size, block_size, k_block_stride, v_block_stride);
-      else
-        hipLaunchKernelGGL((qk_norm_cache_kernel<scalar_t, kL, 1>), grid, dim3(256), 0, (hipStream_t)stream, (S*)q_out,
-                           (S*)key_cache, (S*)value_cache, (const S*)q, (const S*)k, (const S*)v, row_stride, q_weight,
-                           k_weight, eps, rows, heads, kv_heads, dim, vdim, kpad, vpad, !tiled, slot_mapping,
-                           num_blocks * block_size, block_size, k_block_stride, v_block_stride);
+      if (vec8) LV_QK(kWide);
+      else if (vec) LV_QK(4);
+      else LV_QK(1);
     })
     if (tiled)
       hipLaunchKernelGGL((value_cache_tile_kernel<S>), dim3((rows + kValueTile - 1) / kValueTile, kv_heads), dim3(256), smem,
                          (hipStream_t)stream, (S*)value_cache, (const S*)v, row_stride, rows, vdim, vpad, slot_mapping,
                          num_blocks * block_size, block_size, v_block_stride);
   });
+#undef LV_QK
   LV_LAUNCH_CHECK();
   return 0;
 }
