@@ -15,8 +15,7 @@ def prepare(model_dir: str):
     from light_vllm_amd.engine.registry import model_entry, read_architecture
     entry = model_entry(read_architecture(model_dir))
     build.build_all(entry.native)
-    if entry.native == ("base",):
-        _native.limit_to_base()
+    _native.limit_to(entry.native)
     return entry
 
 

@@ -609,7 +609,9 @@ int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void
                         const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows, int heads, int dk,
                         int dv, int max_query_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 /* Causal attention over the cache of lvllm_qk_norm_cache; q [rows, heads, kpad];
- * out[row, h * vdim + d] = T(attention * sigmoid(gate[row, h]) * out_scale), gate null: no gate.  max_query_len and
+ * out[row, h * vdim + d] = T(attention * sigmoid(gate[row, h]) * out_scale), gate null: no gate.  A query sees the keys of the
+ * last `window` positions, its own included (window <= 0: all before it); sequences of fewer than min_query_len query tokens
+ * are left alone.  max_query_len and
  * max_seq_len bound the step's query_len and seq_lens.  bf16 with block size 16, kpad in {64, 96, 128, 192, 256} and vpad
  * in {32, 64, 96, 128, 192, 256} run on MFMAs; every other case on a plain fp32 body. */
 int64_t lvllm_head_attention_workspace_bytes(int rows, int num_seqs, int heads, int kv_heads, int kpad, int vpad,
@@ -618,8 +620,64 @@ int lvllm_head_attention(void* out, int64_t out_stride, const void* q, const voi
                          const void* gate, int64_t gate_stride, const int32_t* block_tables, const int32_t* seq_lens,
                          const int32_t* query_start_loc, int num_seqs, int rows, int heads, int kv_heads, int kpad, int vpad,
                          int vdim, int max_blocks, int block_size, int64_t num_blocks, float scale, float out_scale,
-                         int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len,
+                         int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len, int window, int min_query_len,
                          void* workspace, int64_t workspace_bytes, int dtype, void* stream);
+
+/* ---- latent decoders (csrc/latent_attention*.hip, moe*.hip, depth_mix.hip) ----
+ * Rows of a step as for the hybrid decoders.  dtype: LVLLM_F32 or LVLLM_BF16.  csrc/latent_attention.h, csrc/moe.h and
+ * csrc/depth_mix.hip give the layouts and what is computed. */
+
+/* x = table[id] * scale (fp32), h = T(x) */
+int lvllm_embed_scale(float* x, void* h, const void* table, const int64_t* ids, float scale, int rows, int vocab, int width,
+                      int dtype, void* stream);
+/* v = x_in + y * gain / sqrt(mean(y^2) + eps); x_out = v, or the average of `num_streams` streams and v by `weights`
+ * (num_streams + 1 numbers); h = T(x_out), with out_gain normed once more.  y: rows, fp32 slabs (`partials`), or slots of a
+ * mixture with their weights.  x_out, v_out may be null. */
+int lvllm_norm_add_mix(float* x_out, float* v_out, void* h, const float* x_in, const void* y, const float* partials,
+                       int num_partials, const int32_t* slots, const float* slot_weights, int num_slots, int total_slots,
+                       const float* gain, float eps, const float* streams, int64_t stream_stride, int num_streams,
+                       const float* weights, const float* out_gain, float out_eps, int rows, int width, int dtype, void* stream);
+/* cache rows [RMS norm(kv[:kv_rank]) | rotated kv[kv_rank:]] at slot_mapping (slots < 0: none); inv_freq: rot_dims / 2 */
+int lvllm_latent_cache(void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad, int rpad,
+                       const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
+                       const int64_t* positions, const double* inv_freq, int rot_dims, const int64_t* slot_mapping, int rows,
+                       int dtype, void* stream);
+/* queries into latent space: out [rows, heads, cpad + rpad] = [uk_t q | rotated | 0]; uk_t [heads, cpad, dpad], zero-padded */
+int lvllm_latent_query(void* out, const void* q, int64_t q_stride, const void* uk_t, int heads, int dim, int dpad, int cpad,
+                       int rpad, int rot_dim, int rot_dims, const int64_t* positions, const double* inv_freq,
+                       const int32_t* query_start_loc, int num_seqs, int absorbed_max, int rows, int dtype, void* stream);
+/* values out of it: out[row, h * vdim + d] = (uv o_lat)[d] * sigmoid(gate[row, h]); uv [heads, vpad, cpad], zero-padded */
+int lvllm_latent_value(void* out, int64_t out_stride, const void* o_lat, const void* uv, const void* gate, int64_t gate_stride,
+                       int heads, int vdim, int vpad, int cpad, const int32_t* query_start_loc, int num_seqs, int absorbed_max,
+                       int rows, int dtype, void* stream);
+/* out [rows, heads, cpad]: attention on the cached rows, for sequences of at most absorbed_max query tokens */
+int64_t lvllm_latent_attention_workspace_bytes(int rows, int num_seqs, int heads, int cpad, int rpad, int block_size,
+                                               int window, int absorbed_max, int max_query_len, int max_seq_len, int dtype);
+int lvllm_latent_attention(void* out, const void* q, const void* cache, int64_t block_stride, int64_t num_blocks,
+                           int block_size, int cpad, int rpad, const int32_t* block_tables, int max_blocks,
+                           const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows, int heads,
+                           float scale, int window, int absorbed_max, int max_query_len, int max_seq_len, void* workspace,
+                           int64_t workspace_bytes, int dtype, void* stream);
+/* long portions: cached rows back to back, their expanded keys / values as pages, their queries */
+int lvllm_latent_gather(void* out, const void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int row_elems,
+                        const int32_t* starts, const int32_t* first, const int32_t* seq_lens, const int32_t* block_tables,
+                        int max_blocks, int num_seqs, int n, int dtype, void* stream);
+int lvllm_latent_expand(void* key_pages, void* value_pages, const void* kv, int64_t kv_stride, const void* rows, int row_elems,
+                        int cpad, int n, int heads, int dim, int rot_dim, int vdim, int kpad, int vpad, int dtype, void* stream);
+int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_stride, int heads, int dim, int rot_dim, int kpad,
+                              const int64_t* positions, const double* inv_freq, int rot_dims, int rows, int dtype, void* stream);
+/* the `top` experts of every row and their softmax weights; with `shared` a last assignment, expert number `experts`, weighted
+ * sigmoid of the last row of w */
+int lvllm_moe_route(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
+                    int top, int rows, int width, int dtype, void* stream);
+/* assignments grouped by expert: offsets [experts + 1], token and slot [total], tiles [max_tiles, 2] of lvllm_moe_tile slots */
+int lvllm_moe_tile(int packed);
+int lvllm_moe_group(int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles, const int32_t* ids, int total, int per_row,
+                    int experts, int packed, int max_tiles, void* stream);
+/* the experts' products: up (with the activation) [rows, width] -> [slots, ff_max], down [slots, ff_max] -> [slots, width] */
+int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff, const float* limit,
+                      const int32_t* offsets, const int32_t* token, const int32_t* tiles, int experts, int slots, int rows,
+                      int width, int ff_max, int max_tiles, int up, int packed, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

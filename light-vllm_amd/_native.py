@@ -2,32 +2,31 @@
 binding is missing or fails to load, importing this module's users raises, so a product
 path can never silently run on something else.
 
-Two components (build.py): "base" -- what every model needs -- and "full" -- base plus the operators of the rotary
-decoders.  `limit_to_base()`, called before anything else of the package is imported, makes a process that serves a
-base-only model load (and need) the first alone."""
+The libraries come in components (build.py): "base" is what every model needs, "full" includes all the others.
+`limit_to(components)`, called before anything else of the package is imported, makes a process that serves one model load
+(and need) that model's components alone."""
 import ctypes
 import os
 
 import torch  # must be first: its HIP runtime (same SONAME) is the one the kernels use
 
-_LIBDIR = os.path.join(os.path.dirname(os.path.abspath(__file__)), "lib")
-BASE_LIB_PATH = os.path.join(_LIBDIR, "liblvllm_base.so")
-BASE_EXT_PATH = os.path.join(_LIBDIR, "_C_base.so")
-LIB_PATH = os.path.join(_LIBDIR, "liblvllm_hip.so")
-EXT_PATH = os.path.join(_LIBDIR, "_C.so")
+from .build import ALL, COMPONENTS, LIBDIR, with_needed
 
-_state = {"lib": None, "ext": False, "base_only": False}
+LIB_PATH = os.path.join(LIBDIR, COMPONENTS["full"][1])
+EXT_PATH = os.path.join(LIBDIR, COMPONENTS["full"][3])
+
+_state = {"lib": None, "ext": False, "components": ALL}
 
 
 class NativeLibraryError(ImportError):
     pass
 
 
-def limit_to_base() -> None:
-    """This process serves a model that the base component alone covers: nothing else is loaded or required."""
+def limit_to(components) -> None:
+    """This process serves a model that these components cover: nothing else is loaded or required."""
     if _state["lib"] is not None or _state["ext"]:
-        raise NativeLibraryError("limit_to_base() must come before the native libraries are loaded")
-    _state["base_only"] = True
+        raise NativeLibraryError("limit_to() must come before the native libraries are loaded")
+    _state["components"] = with_needed(components)
 
 
 def _require(path: str) -> str:
@@ -39,11 +38,10 @@ def _require(path: str) -> str:
 
 
 def load_hip_library() -> ctypes.CDLL:
-    """ctypes handle on the C-ABI (include/lvllm_hip.h)."""
+    """ctypes handle on the C-ABI (include/lvllm_hip.h); with fewer than all components, on the last of them."""
     if _state["lib"] is None:
-        lib = ctypes.CDLL(_require(BASE_LIB_PATH), mode=ctypes.RTLD_GLOBAL)
-        if not _state["base_only"]:
-            lib = ctypes.CDLL(_require(LIB_PATH), mode=ctypes.RTLD_GLOBAL)
+        for c in _state["components"]:
+            lib = ctypes.CDLL(_require(os.path.join(LIBDIR, COMPONENTS[c][1])), mode=ctypes.RTLD_GLOBAL)
         lib.lvllm_last_error.restype = ctypes.c_char_p
         lib.lvllm_version.restype = ctypes.c_char_p
         _state["lib"] = lib
@@ -54,12 +52,12 @@ def load_torch_ops() -> None:
     """Registers torch.ops._C / _C_cache_ops / _C_cuda_utils (reference schemas) and _C_amd."""
     if not _state["ext"]:
         load_hip_library()
-        for path in [BASE_EXT_PATH] + ([] if _state["base_only"] else [EXT_PATH]):
-            torch.ops.load_library(_require(path))
+        for c in _state["components"]:
+            torch.ops.load_library(_require(os.path.join(LIBDIR, COMPONENTS[c][3])))
         _state["ext"] = True
 
 
 def loaded_libraries():
-    full = not _state["base_only"]
-    return {"hip": (LIB_PATH if full else BASE_LIB_PATH) if _state["lib"] is not None else None,
-            "torch_ops": (EXT_PATH if full else BASE_EXT_PATH) if _state["ext"] else None}
+    last = COMPONENTS[_state["components"][-1]]
+    return {"hip": os.path.join(LIBDIR, last[1]) if _state["lib"] is not None else None,
+            "torch_ops": os.path.join(LIBDIR, last[3]) if _state["ext"] else None}

@@ -1,14 +1,18 @@
-"""Build the gfx950 native libraries in-tree (no cmake, no hipify).
+"""Build the gfx950 native libraries in-tree (no cmake, no hipify), in components:
 
-  liblvllm_base.so  what every model needs: error plumbing, cache block movement, the weight-streaming GEMMs of decode
-                    steps, step inputs, the sampler, and the kernels of the hybrid (attention + recurrent) decoders
-  liblvllm_hip.so   the rest of the C-ABI of include/lvllm_hip.h (paged and prefill attention of the rotary decoders,
-                    norms, fp8); it needs liblvllm_base.so, so a handle on it resolves every symbol of the header
-                    (hipcc --offload-arch=gfx950, one object per .hip, linked -shared)
-  _C_base.so, _C.so torch op registrations (`torch.ops._C`, `_C_cache_ops`, `_C_cuda_utils`, `_C_amd`) forwarding to
-                    the C-ABI; host-only C++, built with g++ against the torch headers.
+  base    what every model needs: error plumbing, cache block movement, the weight-streaming GEMMs of decode steps, step
+          inputs, the sampler
+  heads   softmax attention over paged caches of unequal key and value sizes (hybrid and latent decoders)
+  hybrid  row-wise operators and recurrences of the hybrid decoders
+  latent  latent attention, mixtures of experts, norms on sublayer outputs and depth averages
+  full    the rest of the C-ABI of include/lvllm_hip.h (paged and prefill attention of the rotary decoders, norms, fp8); it
+          needs all the others, so a handle on liblvllm_hip.so resolves every symbol of the header
 
-`build_all(("base",))` builds the first pair only: all that a model whose registry entry says so will load.
+Each is a kernel library (hipcc --offload-arch=gfx950, one object per .hip, linked -shared) and a torch extension: op
+registrations (`torch.ops._C`, `_C_cache_ops`, `_C_cuda_utils`, `_C_amd`) forwarding to the C-ABI; host-only C++, built with
+g++ against the torch headers.
+
+`build_all(("base", "latent"))` builds what a model whose registry entry says so will load.
 All land in light-vllm_amd/lib/.  Objects are cached under build/ keyed on the
 source mtime, so a rebuild after touching one kernel takes seconds.
 """
@@ -24,30 +28,31 @@ LIBDIR = os.path.join(PKG, "lib")
 OBJDIR = os.path.join(ROOT, "build", "obj")
 ARCH = "gfx950"
 
-BASE_SOURCES = [
-    "capi.hip",
-    "cache.hip",
-    "skinny_gemm.hip",
-    "prepare_inputs.hip",
-    "sampler.hip",
-    "activation.hip",
-    "token_mix.hip",
-    "recurrent.hip",
-    "head_attention.hip",
-    "head_attention_prefill.hip",
-    "head_attention_decode.hip",
-]
-FULL_SOURCES = [
-    "layernorm.hip",
-    "pos_encoding.hip",
-    "attention.hip",
-    "attention_bf16.hip",
-    "attention_f16.hip",
-    "prefill_attention.hip",
-    "fp8_quant.hip",
-]
-COMPONENTS = {"base": (BASE_SOURCES, "liblvllm_base.so", "torch_bindings_base.cpp", "_C_base.so"),
-              "full": (FULL_SOURCES, "liblvllm_hip.so", "torch_bindings.cpp", "_C.so")}
+SOURCES = {
+    "base": ["capi.hip", "cache.hip", "skinny_gemm.hip", "prepare_inputs.hip", "sampler.hip", "activation.hip"],
+    "heads": ["head_attention.hip", "head_attention_prefill.hip", "head_attention_decode.hip"],
+    "hybrid": ["token_mix.hip", "recurrent.hip"],
+    "latent": ["latent_attention.hip", "latent_attention_mfma.hip", "moe.hip", "moe_mfma.hip", "depth_mix.hip"],
+    "full": ["layernorm.hip", "pos_encoding.hip", "attention.hip", "attention_bf16.hip", "attention_f16.hip",
+             "prefill_attention.hip", "fp8_quant.hip"],
+}
+ALL = tuple(SOURCES)  # in link order: "base" is needed by the others, "full" needs all
+# component -> (sources, kernel library, torch registrations, torch extension)
+COMPONENTS = {c: (src,) + (("liblvllm_hip.so", "torch_bindings.cpp", "_C.so") if c == "full" else
+                           (f"liblvllm_{c}.so", f"torch_bindings_{c}.cpp", f"_C_{c}.so"))
+              for c, src in SOURCES.items()}
+
+
+def with_needed(components):
+    """The components and what they need, in link order."""
+    return ALL if "full" in components else tuple(c for c in ALL if c == "base" or c in components)
+
+
+def _links(component):
+    """Linker flags for the kernel libraries a component's own kernel library needs."""
+    need = [] if component == "base" else [c for c in ALL if c != "full"] if component == "full" else ["base"]
+    return (["-L", LIBDIR] + [f"-llvllm_{c}" for c in need] + ["-Wl,-rpath,$ORIGIN"]) if need else []
+
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # tuning experiments: e.g. LVLLM_EXTRA_HIPCC_FLAGS="-DLVLLM_ATTN_NBUF=2 -DLVLLM_ATTN_TUNE_ONLY"
@@ -83,7 +88,7 @@ def _run(cmd):
 PER_SOURCE_FLAGS = {"prefill_attention.hip": ["-fno-honor-nans"]}
 
 
-def build_kernels(components=("base", "full"), verbose=False, force=False):
+def build_kernels(components=ALL, verbose=False, force=False):
     os.makedirs(OBJDIR, exist_ok=True)
     os.makedirs(LIBDIR, exist_ok=True)
     hdrs = _headers()
@@ -110,12 +115,12 @@ def build_kernels(components=("base", "full"), verbose=False, force=False):
         if force or _newer(lib, objs[c] + [os.path.abspath(__file__)]):
             # no rpath to /opt/rocm on purpose: inside a torch process the HIP
             # runtime torch already loaded (same SONAME) must be the one used.
-            link = [] if c == "base" else ["-L", LIBDIR, "-llvllm_base", "-Wl,-rpath,$ORIGIN"]
-            _run([HIPCC, "--offload-arch=" + ARCH, "-shared", "-fPIC", "-o", lib] + objs[c] + link)
+            _run([HIPCC, "--offload-arch=" + ARCH, "-shared", "-fPIC", "-o", lib] + objs[c] +
+                 (["-Wl,--no-as-needed"] + _links(c) if c == "full" else _links(c)))
     return libs
 
 
-def build_torch_bindings(components=("base", "full"), verbose=False, force=False):
+def build_torch_bindings(components=ALL, verbose=False, force=False):
     import torch  # noqa: F401  (header + library locations)
     from torch.utils import cpp_extension as ce
     import sysconfig
@@ -140,7 +145,7 @@ def build_torch_bindings(components=("base", "full"), verbose=False, force=False
             cmd += ["-I", i]
         jobs.append(cmd + [src, "-o", out, "-L", torch_lib, "-L", LIBDIR,
                            "-ltorch", "-ltorch_cpu", "-ltorch_hip", "-lc10", "-lc10_hip"] +
-                    (["-llvllm_hip"] if c == "full" else []) + ["-llvllm_base", "-Wl,-rpath,$ORIGIN"])
+                    ["-llvllm_hip" if c == "full" else f"-llvllm_{c}", "-llvllm_base", "-Wl,-rpath,$ORIGIN"])
     if jobs:
         with ThreadPoolExecutor(max_workers=len(jobs)) as ex:
             for o in ex.map(_run, jobs):
@@ -149,9 +154,10 @@ def build_torch_bindings(components=("base", "full"), verbose=False, force=False
     return outs
 
 
-def build_all(components=("base", "full"), verbose=False, force=False):
+def build_all(components=ALL, verbose=False, force=False):
     """(kernel libraries, torch extensions) of the components, built where they are missing or older than a source
     (`force`: all of them)."""
+    components = with_needed(components)
     return build_kernels(components, verbose, force), build_torch_bindings(components, verbose, force)
 
 

@@ -234,4 +234,19 @@ __device__ inline float block_sum(float v, float* red) {
       LV_CHECK(false, "unsupported dtype");      \
   }
 
+// the two compute dtypes of decoders of listed layers
+#define LV_DISPATCH_F32_BF16(dtype, ...)         \
+  switch (dtype) {                               \
+    case LVLLM_F32: {                            \
+      using scalar_t = ::lvllm::F32;             \
+      __VA_ARGS__;                               \
+    } break;                                     \
+    case LVLLM_BF16: {                           \
+      using scalar_t = ::lvllm::BF16;            \
+      __VA_ARGS__;                               \
+    } break;                                     \
+    default:                                     \
+      LV_CHECK(false, "float32 or bfloat16");    \
+  }
+
 }  // namespace lvllm

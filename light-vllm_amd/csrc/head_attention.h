@@ -1,6 +1,8 @@
 // Causal softmax attention over a paged cache whose key and value sizes differ, without positions in the scores, for
 // gfx950.  Every sequence of a step is a chunk of query_len >= 1 new tokens that ends its context (their keys and
-// values are in the cache already); query t of a chunk sits at position seq_len - query_len + t and sees keys 0 .. there.
+// values are in the cache already); query t of a chunk sits at position pos = seq_len - query_len + t and sees keys
+// max(0, pos - window + 1) .. pos (window <= 0: keys 0 .. pos).  Sequences of fewer than min_query_len query tokens are left
+// to the caller.
 //
 //   query       [rows, heads, kpad]                                (padding beyond the key size is zero)
 //   key_cache   [num_blocks, kv_heads, kpad / x, block_size, x],   x = 16 / sizeof(T)
@@ -21,7 +23,7 @@ struct HeadAttnParams {
   const int32_t *block_tables, *seq_lens, *query_start_loc;
   float *part_o, *part_ml;  // decode shares: [rows, heads, nsplit, vpad] and [rows, heads, nsplit, 2]
   int num_seqs, rows, heads, kv_heads, kpad, vpad, vdim, max_blocks, block_size, max_block, nsplit;
-  int max_query_len, max_seq_len;
+  int max_query_len, max_seq_len, window, min_query_len;
   float scale, out_scale;
   int64_t out_stride, gate_stride, k_block_stride, v_block_stride;
 };
@@ -29,6 +31,8 @@ struct HeadAttnParams {
 // Sequences with at most this many (token, head) columns per kv head, and every sequence of one token, take the decode body.
 constexpr int kDecodeCols = 16;
 __device__ __forceinline__ bool takes_decode_body(int qlen, int group) { return qlen == 1 || qlen * group <= kDecodeCols; }
+
+__device__ __forceinline__ int first_seen(int pos, int window) { return window > 0 ? max(0, pos - window + 1) : 0; }
 
 template <typename T>
 __device__ __forceinline__ float gate_of(const HeadAttnParams& p, int64_t row, int head) {

@@ -20,6 +20,7 @@ __global__ __launch_bounds__(256) void head_attention_simple_kernel(const HeadAt
   const int seq = find_seq(p.query_start_loc, p.num_seqs, row);
   if (seq >= p.num_seqs) return;
   const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
+  if (qlen < p.min_query_len) return;
   const int n_keys = p.seq_lens[seq] - qlen + (row - qbeg) + 1;
   S* out = (S*)p.out + row * p.out_stride + (int64_t)head * p.vdim;
   if (n_keys <= 0) {  // a padding row of a captured step
@@ -33,7 +34,7 @@ __global__ __launch_bounds__(256) void head_attention_simple_kernel(const HeadAt
   for (int d = threadIdx.x; d < p.vpad; d += 256) sacc[d] = 0.f;
   float m = -FLT_MAX, l = 0.f;
   const int bs = p.block_size;
-  for (int k0 = 0; k0 < n_keys; k0 += 256) {
+  for (int k0 = first_seen(n_keys - 1, p.window); k0 < n_keys; k0 += 256) {
     __syncthreads();
     const int key = k0 + threadIdx.x;
     float score = -FLT_MAX;
@@ -110,7 +111,7 @@ extern "C" int lvllm_head_attention(void* out, int64_t out_stride, const void* q
                                     int num_seqs, int rows, int heads, int kv_heads, int kpad, int vpad, int vdim,
                                     int max_blocks, int block_size, int64_t num_blocks, float scale, float out_scale,
                                     int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len,
-                                    void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
+                                    int window, int min_query_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
   if (rows == 0 || num_seqs == 0) return 0;
   LV_CHECK(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "heads must be a multiple of kv_heads");
   LV_CHECK(kpad % 8 == 0 && vpad > 0 && vdim > 0 && vdim <= vpad && kpad <= 8192 && vpad <= 8192,
@@ -125,6 +126,7 @@ extern "C" int lvllm_head_attention(void* out, int64_t out_stride, const void* q
   p.max_block = (int)(num_blocks - 1); p.scale = scale; p.out_scale = out_scale;
   p.k_block_stride = k_block_stride; p.v_block_stride = v_block_stride;
   p.max_query_len = max_query_len; p.max_seq_len = max_seq_len; p.nsplit = 1;
+  p.window = window; p.min_query_len = min_query_len;
   hipStream_t s = (hipStream_t)stream;
   if (takes_mfma(kpad, vpad, block_size, dtype)) {
     p.nsplit = decode_shares(rows, num_seqs, heads, kv_heads, max_seq_len);
@@ -134,7 +136,8 @@ extern "C" int lvllm_head_attention(void* out, int64_t out_stride, const void* q
       p.part_o = (float*)workspace;
       p.part_ml = p.part_o + (int64_t)rows * heads * p.nsplit * vpad;
     }
-    if (int rc = launch_head_decode(p, s)) return rc;
+    if (min_query_len <= kDecodeCols)  // (longer ones all take the chunk body)
+      if (int rc = launch_head_decode(p, s)) return rc;
     if (max_query_len > 1)
       if (int rc = launch_head_prefill(p, s)) return rc;
     return 0;

@@ -26,7 +26,7 @@ __global__ __launch_bounds__(256, 2) void head_decode_kernel(const HeadAttnParam
   const int kvh = blockIdx.x / groups, cg = blockIdx.x - kvh * groups;
   const int seq = blockIdx.y, share = blockIdx.z;
   const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
-  if (qlen <= 0 || !takes_decode_body(qlen, G)) return;
+  if (qlen <= 0 || qlen < p.min_query_len || !takes_decode_body(qlen, G)) return;
   const int seq_len = p.seq_lens[seq], ctx = seq_len - qlen;
   // columns of this workgroup
   int ncols, tok, head;
@@ -43,10 +43,10 @@ __global__ __launch_bounds__(256, 2) void head_decode_kernel(const HeadAttnParam
   }
   head += kvh * G;
   const int64_t row = qbeg + tok;
-  const int pos = ctx + tok;
-  const int nblocks = (max(seq_len, 0) + 15) / 16;
-  const int per = (nblocks + p.nsplit - 1) / p.nsplit;
-  const int b0 = share * per, b1 = min(b0 + per, nblocks);
+  const int pos = ctx + tok, low = first_seen(pos, p.window);
+  const int first_block = first_seen(ctx, p.window) / 16, nblocks = (max(seq_len, 0) + 15) / 16;
+  const int per = (nblocks - first_block + p.nsplit - 1) / p.nsplit;
+  const int b0 = first_block + share * per, b1 = min(b0 + per, nblocks);
 
   h_u32x4_t qf[NK];
   {
@@ -82,7 +82,10 @@ __global__ __launch_bounds__(256, 2) void head_decode_kernel(const HeadAttnParam
       s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(h_bf16x8_t, t.k[j]),
                                                   __builtin_bit_cast(h_bf16x8_t, qf[j]), s, 0, 0, 0);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) s[r] = b * 16 + 4 * g + r <= pos ? s[r] * sl : -FLT_MAX;
+    for (int r = 0; r < 4; ++r) {
+      const int key = b * 16 + 4 * g + r;
+      s[r] = key <= pos && key >= low ? s[r] * sl : -FLT_MAX;
+    }
     float mx = fmaxf(fmaxf(s[0], s[1]), fmaxf(s[2], s[3]));
     mx = fmaxf(mx, __shfl_xor(mx, 16));
     mx = fmaxf(mx, __shfl_xor(mx, 32));
@@ -163,7 +166,7 @@ __global__ __launch_bounds__(128) void head_decode_reduce_kernel(const HeadAttnP
   const int seq = find_seq(p.query_start_loc, p.num_seqs, row);
   if (seq >= p.num_seqs) return;
   const int qlen = p.query_start_loc[seq + 1] - p.query_start_loc[seq];
-  if (!takes_decode_body(qlen, p.heads / p.kv_heads)) return;
+  if (qlen < p.min_query_len || !takes_decode_body(qlen, p.heads / p.kv_heads)) return;
   const int64_t at = ((int64_t)row * p.heads + head) * p.nsplit;
   float m = -1e30f;
   for (int s = 0; s < p.nsplit; ++s) m = fmaxf(m, p.part_ml[2 * (at + s)]);

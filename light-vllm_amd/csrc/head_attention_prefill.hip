@@ -36,7 +36,7 @@ __global__ __launch_bounds__(256, NK + NV <= 10 ? 2 : 1) void head_prefill_kerne
   const int G = p.heads / p.kv_heads;
   const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
   const int ncols = qlen * G;
-  if (qlen <= 0 || takes_decode_body(qlen, G) || tile_q * kPrefillCols >= ncols) return;
+  if (qlen <= 0 || qlen < p.min_query_len || takes_decode_body(qlen, G) || tile_q * kPrefillCols >= ncols) return;
   const int ctx = p.seq_lens[seq] - qlen;
   if (ctx < 0) return;
   const int col0 = tile_q * kPrefillCols + wave * 32;
@@ -44,11 +44,12 @@ __global__ __launch_bounds__(256, NK + NV <= 10 ? 2 : 1) void head_prefill_kerne
   const bool col_ok = col0 + lc < ncols;
   const int tok = col / G, head = kvh * G + (col - tok * G);
   const int64_t row = qbeg + tok;
-  const int pos = ctx + tok;  // the last key this lane's column sees
+  const int pos = ctx + tok, low = first_seen(pos, p.window);  // the last and the first key this lane's column sees
   const int wg_last = ctx + (min(tile_q * kPrefillCols + kPrefillCols, ncols) - 1) / G;
   const bool wave_ok = col0 < ncols;
   const int wave_first = ctx + min(col0, ncols - 1) / G, wave_last = ctx + min(col0 + 31, ncols - 1) / G;
-  const int ntiles = wg_last / 64 + 1;
+  const int wave_low = first_seen(wave_first, p.window), wave_all = first_seen(wave_last, p.window);
+  const int tile0 = first_seen(ctx + tile_q * kPrefillCols / G, p.window) / 64, ntiles = wg_last / 64 + 1;
 
   h_u32x4_t qf[2 * NK];
   {
@@ -102,14 +103,14 @@ __global__ __launch_bounds__(256, NK + NV <= 10 ? 2 : 1) void head_prefill_kerne
   const int klds = (lc >> 4) * kKBlock + (hi * 16 + key16) * 16;
   const int vlds = kImageK + lane * 16;  // (hi * 32 + lc) * 16
 
-  fetch(0);
-  put(0);
+  fetch(tile0);
+  put(tile0 & 1);
   __syncthreads();
-  for (int t = 0; t < ntiles; ++t) {
+  for (int t = tile0; t < ntiles; ++t) {
     const bool more = t + 1 < ntiles;
     if (more) fetch(t + 1);
     const int k0 = t * 64;
-    if (wave_ok && k0 <= wave_last) {
+    if (wave_ok && k0 <= wave_last && k0 + 63 >= wave_low) {
       const char* base = smem + (t & 1) * kStage;
       h_f32x16_t s[2] = {h_f32x16_t{}, h_f32x16_t{}};
 #pragma unroll
@@ -119,13 +120,13 @@ __global__ __launch_bounds__(256, NK + NV <= 10 ? 2 : 1) void head_prefill_kerne
         s[0] = mfma32(a0, qf[ks], s[0]);
         s[1] = mfma32(a1, qf[ks], s[1]);
       }
-      if (k0 + 63 > wave_first) {  // the diagonal passes through this tile for some column
+      if (k0 + 63 > wave_first || k0 < wave_all) {  // the diagonal or the window's edge passes through it for some column
 #pragma unroll
         for (int h = 0; h < 2; ++h)
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
             const int key = k0 + 32 * h + 16 * (i >> 3) + 8 * hi + (i & 7);
-            s[h][i] = key <= pos ? s[h][i] * sl : -FLT_MAX;
+            s[h][i] = key <= pos && key >= low ? s[h][i] * sl : -FLT_MAX;
           }
       } else {
 #pragma unroll

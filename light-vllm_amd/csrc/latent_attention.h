@@ -1,0 +1,44 @@
+// Latent attention for gfx950: a layer caches, per token, one latent c (kv_rank numbers) and one rotated key part (rot_dim
+// numbers) that all heads share; head h's key is [U_h c | k_rot] and its value V_h c.  A query sees the keys of the last
+// `window` positions, itself included (window <= 0: all of them).
+//
+// Two ways through, the same sums in another order:
+//   * absorbed: the query is taken into latent space once, q' = [U_h^T q | q_rot], scores and weighted sums run on the cached
+//     rows themselves (all heads on one row: bound by the cache's bytes), and V_h is applied to the summed latents.  Single
+//     tokens and portions of up to `absorbed_max` tokens;
+//   * expanded: the window's latents are gathered, keys and values of all heads made by one library product, and
+//     head_attention runs over them.  Longer portions.
+//
+//   cache  [num_blocks, block_size, cpad + rpad]: c, zeros to cpad, the rotated part, zeros to the row's end
+//   q'     [rows, heads, cpad + rpad], the same row layout
+//   o_lat  [rows, heads, cpad]: the weighted sums of the latents
+// Scores, softmax and accumulation are fp32.
+#pragma once
+#include "common.h"
+
+namespace lvllm {
+
+struct LatentAttnParams {
+  void* out;
+  const void *q, *cache;
+  const int32_t *block_tables, *seq_lens, *query_start_loc;
+  float *part_o, *part_ml;  // shares: [rows, heads, nsplit, cpad] and [rows, heads, nsplit, 2]
+  int num_seqs, rows, heads, cpad, rpad, max_blocks, block_size, max_block, nsplit, window, absorbed_max, max_query_len;
+  float scale;
+  int64_t block_stride;
+};
+
+bool latent_takes_mfma(int cpad, int rpad, int block_size, int dtype);
+int launch_latent_mfma(const LatentAttnParams& p, hipStream_t s);
+
+// The first key position `pos` sees.
+__device__ __forceinline__ int first_key(int pos, int window) { return window > 0 ? max(0, pos - window + 1) : 0; }
+
+// Rotation of pairs (2i, 2i + 1): the angle is taken in double, so that far positions keep the fp32 sine's own accuracy.
+__device__ __forceinline__ void rotation_of(int64_t position, double inv_freq, float& c, float& s) {
+  const double a = (double)position * inv_freq;
+  const double r = a - rint(a * 0.15915494309189533577) * 6.28318530717958647693;
+  sincosf((float)r, &s, &c);
+}
+
+}  // namespace lvllm

@@ -1,4 +1,4 @@
-// Helpers shared by the torch op registrations (torch_bindings_base.cpp, torch_bindings.cpp): dtype codes, argument
+// Helpers shared by the torch op registrations (torch_bindings*.cpp): dtype codes, argument
 // checks, the current stream, the C-ABI's error string as an exception.  Host-only C++.
 #pragma once
 #include <Python.h>
@@ -77,6 +77,63 @@ namespace {
 // static_scaled_fp8_quant
 [[maybe_unused]] void check_q_scale(const torch::Tensor& s, const char* op) {
   TORCH_CHECK(s.is_cuda() && s.scalar_type() == at::kFloat && s.numel() == 1, op, ": one float32 scale on the device");
+}
+
+// ---- decoders of listed layers (include/lvllm_hip.h) ----
+// a step's layout: [num_seqs + 1] / [num_seqs] int32 on the device
+[[maybe_unused]] void check_layout(const torch::Tensor& query_start_loc, const torch::Tensor& seq_lens, const char* op) {
+  TORCH_CHECK(query_start_loc.is_cuda() && seq_lens.is_cuda() && query_start_loc.scalar_type() == at::kInt &&
+                  seq_lens.scalar_type() == at::kInt && query_start_loc.is_contiguous() && seq_lens.is_contiguous() &&
+                  query_start_loc.numel() == seq_lens.numel() + 1,
+              op, ": query_start_loc int32 [num_seqs + 1] and seq_lens int32 [num_seqs] on the device");
+}
+[[maybe_unused]] void check_f32(const torch::Tensor& t, int64_t numel, const char* op, const char* what) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.is_contiguous() && t.numel() == numel, op, ": ", what,
+              " must be ", numel, " contiguous float32 elements on the device");
+}
+// [slots, ...] float32, dense behind dim 0
+[[maybe_unused]] void check_state(const torch::Tensor& t, const torch::Tensor& slots, int64_t numel, int64_t num_seqs, const char* op) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.dim() >= 2 && blocks_are_dense(t) &&
+                  t.numel() == t.size(0) * numel,
+              op, ": state must be float32 [slots, ", numel, " elements], dense behind its first dimension");
+  TORCH_CHECK(slots.is_cuda() && slots.scalar_type() == at::kInt && slots.is_contiguous() && slots.numel() >= num_seqs, op,
+              ": state_slots int32 [num_seqs] on the device");
+}
+// a projection result as an addend: [rows, width] of the compute dtype, or fp32 slabs [s, rows, width]
+struct Addend {
+  const void* y = nullptr;
+  const float* partials = nullptr;
+  int num = 0;
+};
+[[maybe_unused]] Addend addend_of(const std::optional<torch::Tensor>& y, const torch::Tensor& x, at::ScalarType dtype, const char* op) {
+  Addend a;
+  if (!y) return a;
+  TORCH_CHECK(y->is_cuda() && y->is_contiguous(), op, ": y must be contiguous on the device");
+  if (y->dim() == 3) {
+    TORCH_CHECK(y->scalar_type() == at::kFloat && y->size(1) == x.size(0) && y->size(2) == x.size(1), op,
+                ": partials must be float32 [s, rows, width]");
+    a.partials = y->data_ptr<float>();
+    a.num = (int)y->size(0);
+  } else {
+    TORCH_CHECK(y->scalar_type() == dtype && y->sizes() == x.sizes(), op, ": y must be [rows, width] of the compute dtype");
+    a.y = y->data_ptr();
+  }
+  return a;
+}
+[[maybe_unused]] void check_residual(const torch::Tensor& x, const char* op) {
+  TORCH_CHECK(x.is_cuda() && x.dim() == 2 && x.is_contiguous() && x.scalar_type() == at::kFloat, op,
+              ": the residual must be contiguous float32 [rows, width]");
+}
+
+// caches as lvllm_qk_norm_cache describes them; returns (kpad, vpad, block_size)
+[[maybe_unused]] std::tuple<int64_t, int64_t, int64_t> head_cache_dims(const torch::Tensor& kc, const torch::Tensor& vc, int64_t kv_heads,
+                                                      at::ScalarType dtype, const char* op) {
+  TORCH_CHECK(kc.is_cuda() && vc.is_cuda() && kc.dim() == 5 && vc.dim() == 4 && kc.size(0) == vc.size(0) &&
+                  kc.size(1) == kv_heads && vc.size(1) == kv_heads && kc.size(3) == vc.size(3) &&
+                  kc.scalar_type() == dtype && vc.scalar_type() == dtype && kc.size(4) * kc.element_size() == 16 &&
+                  blocks_are_dense(kc) && blocks_are_dense(vc),
+              op, ": key_cache [blocks, kv_heads, kpad/x, block_size, x] and value_cache [blocks, kv_heads, vpad, block_size]");
+  return {kc.size(2) * kc.size(4), vc.size(2), vc.size(3)};
 }
 
 }  // namespace

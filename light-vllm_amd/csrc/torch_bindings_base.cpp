@@ -570,284 +570,6 @@ int64_t get_max_shared_memory_per_block_device_attribute(int64_t device_id) {
   return lvllm_get_max_shared_memory_per_block_device_attribute(device_id);
 }
 
-// ---- hybrid decoders (include/lvllm_hip.h) ----
-// a step's layout: [num_seqs + 1] / [num_seqs] int32 on the device
-void check_layout(const torch::Tensor& query_start_loc, const torch::Tensor& seq_lens, const char* op) {
-  TORCH_CHECK(query_start_loc.is_cuda() && seq_lens.is_cuda() && query_start_loc.scalar_type() == at::kInt &&
-                  seq_lens.scalar_type() == at::kInt && query_start_loc.is_contiguous() && seq_lens.is_contiguous() &&
-                  query_start_loc.numel() == seq_lens.numel() + 1,
-              op, ": query_start_loc int32 [num_seqs + 1] and seq_lens int32 [num_seqs] on the device");
-}
-void check_f32(const torch::Tensor& t, int64_t numel, const char* op, const char* what) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.is_contiguous() && t.numel() == numel, op, ": ", what,
-              " must be ", numel, " contiguous float32 elements on the device");
-}
-// [slots, ...] float32, dense behind dim 0
-void check_state(const torch::Tensor& t, const torch::Tensor& slots, int64_t numel, int64_t num_seqs, const char* op) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.dim() >= 2 && blocks_are_dense(t) &&
-                  t.numel() == t.size(0) * numel,
-              op, ": state must be float32 [slots, ", numel, " elements], dense behind its first dimension");
-  TORCH_CHECK(slots.is_cuda() && slots.scalar_type() == at::kInt && slots.is_contiguous() && slots.numel() >= num_seqs, op,
-              ": state_slots int32 [num_seqs] on the device");
-}
-// a projection result as an addend: [rows, width] of the compute dtype, or fp32 slabs [s, rows, width]
-struct Addend {
-  const void* y = nullptr;
-  const float* partials = nullptr;
-  int num = 0;
-};
-Addend addend_of(const std::optional<torch::Tensor>& y, const torch::Tensor& x, at::ScalarType dtype, const char* op) {
-  Addend a;
-  if (!y) return a;
-  TORCH_CHECK(y->is_cuda() && y->is_contiguous(), op, ": y must be contiguous on the device");
-  if (y->dim() == 3) {
-    TORCH_CHECK(y->scalar_type() == at::kFloat && y->size(1) == x.size(0) && y->size(2) == x.size(1), op,
-                ": partials must be float32 [s, rows, width]");
-    a.partials = y->data_ptr<float>();
-    a.num = (int)y->size(0);
-  } else {
-    TORCH_CHECK(y->scalar_type() == dtype && y->sizes() == x.sizes(), op, ": y must be [rows, width] of the compute dtype");
-    a.y = y->data_ptr();
-  }
-  return a;
-}
-void check_residual(const torch::Tensor& x, const char* op) {
-  TORCH_CHECK(x.is_cuda() && x.dim() == 2 && x.is_contiguous() && x.scalar_type() == at::kFloat, op,
-              ": the residual must be contiguous float32 [rows, width]");
-}
-
-torch::Tensor add_dyt(torch::Tensor& x, const std::optional<torch::Tensor>& y, const torch::Tensor& alpha,
-                      const torch::Tensor& weight, const torch::Tensor& bias, at::ScalarType dtype) {
-  check_residual(x, "add_dyt");
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
-  check_f32(alpha, 1, "add_dyt", "alpha");
-  check_f32(weight, x.size(1), "add_dyt", "weight");
-  check_f32(bias, x.size(1), "add_dyt", "bias");
-  const Addend a = addend_of(y, x, dtype, "add_dyt");
-  auto h = torch::empty(x.sizes(), x.options().dtype(dtype));
-  float* xp = x.data_ptr<float>();
-  check(lvllm_add_dyt(y ? xp : nullptr, xp, a.y, a.partials, a.num, h.data_ptr(), alpha.data_ptr<float>(),
-                      weight.data_ptr<float>(), bias.data_ptr<float>(), (int)x.size(0), (int)x.size(1),
-                      dtype_code(h, "add_dyt"), current_stream(x)));
-  return h;
-}
-
-std::tuple<torch::Tensor, torch::Tensor> add_dyt_shift_mix(
-    const torch::Tensor& x, const std::optional<torch::Tensor>& y, const torch::Tensor& mu, const torch::Tensor& alpha,
-    const torch::Tensor& weight, const torch::Tensor& bias, torch::Tensor& carried, const torch::Tensor& state_slots,
-    const torch::Tensor& query_start_loc, const torch::Tensor& seq_lens, at::ScalarType dtype) {
-  const char* op = "add_dyt_shift_mix";
-  check_residual(x, op);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
-  const int64_t rows = x.size(0), width = x.size(1);
-  check_f32(alpha, 1, op, "alpha");
-  check_f32(weight, width, op, "weight");
-  check_f32(bias, width, op, "bias");
-  TORCH_CHECK(mu.dim() == 2, op, ": mu must be [mixes, width]");
-  check_f32(mu, mu.size(0) * width, op, "mu");
-  check_layout(query_start_loc, seq_lens, op);
-  check_state(carried, state_slots, width, seq_lens.numel(), op);
-  const Addend a = addend_of(y, x, dtype, op);
-  auto x_out = torch::empty(y ? x.sizes() : at::IntArrayRef({0, 0}), x.options());  // (nothing to add: x stays)
-  auto mix = torch::empty({mu.size(0), rows, width}, x.options().dtype(dtype));
-  check(lvllm_add_dyt_shift_mix(y ? x_out.data_ptr<float>() : nullptr, x.data_ptr<float>(), a.y, a.partials, a.num,
-                                mix.data_ptr(), mu.data_ptr<float>(), (int)mu.size(0), alpha.data_ptr<float>(),
-                                weight.data_ptr<float>(), bias.data_ptr<float>(), carried.data_ptr<float>(),
-                                carried.stride(0), state_slots.data_ptr<int>(), (int)carried.size(0),
-                                query_start_loc.data_ptr<int>(), seq_lens.data_ptr<int>(), (int)seq_lens.numel(),
-                                (int)rows, (int)width, dtype_code(mix, op), current_stream(x)));
-  return {x_out, mix};
-}
-
-void relu_squared(torch::Tensor& out, const torch::Tensor& x) {
-  LV_CHECK_DEVICE(x);
-  TORCH_CHECK(x.is_contiguous() && out.is_contiguous() && out.sizes() == x.sizes() && out.scalar_type() == x.scalar_type(),
-              "relu_squared: contiguous tensors of one shape and dtype");
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
-  check(lvllm_relu_squared(out.data_ptr(), x.data_ptr(), x.numel(), dtype_code(x, "relu_squared"), current_stream(x)));
-}
-
-// caches as lvllm_qk_norm_cache describes them; returns (kpad, vpad, block_size)
-std::tuple<int64_t, int64_t, int64_t> head_cache_dims(const torch::Tensor& kc, const torch::Tensor& vc, int64_t kv_heads,
-                                                      at::ScalarType dtype, const char* op) {
-  TORCH_CHECK(kc.is_cuda() && vc.is_cuda() && kc.dim() == 5 && vc.dim() == 4 && kc.size(0) == vc.size(0) &&
-                  kc.size(1) == kv_heads && vc.size(1) == kv_heads && kc.size(3) == vc.size(3) &&
-                  kc.scalar_type() == dtype && vc.scalar_type() == dtype && kc.size(4) * kc.element_size() == 16 &&
-                  blocks_are_dense(kc) && blocks_are_dense(vc),
-              op, ": key_cache [blocks, kv_heads, kpad/x, block_size, x] and value_cache [blocks, kv_heads, vpad, block_size]");
-  return {kc.size(2) * kc.size(4), vc.size(2), vc.size(3)};
-}
-
-torch::Tensor qk_norm_cache(const torch::Tensor& q, const torch::Tensor& k, const torch::Tensor& v,
-                            const torch::Tensor& q_weight, const torch::Tensor& k_weight, double eps, int64_t heads,
-                            int64_t kv_heads, torch::Tensor& key_cache, torch::Tensor& value_cache,
-                            const torch::Tensor& slot_mapping) {
-  const char* op = "qk_norm_cache";
-  LV_CHECK_DEVICE(q);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
-  const int64_t rows = q.size(0), dim = q.size(1) / heads, vdim = v.size(1) / kv_heads;
-  TORCH_CHECK(q.dim() == 2 && k.dim() == 2 && v.dim() == 2 && q.size(1) == heads * dim && k.size(1) == kv_heads * dim &&
-                  v.size(1) == kv_heads * vdim && k.size(0) == rows && v.size(0) == rows && q.stride(1) == 1 &&
-                  k.stride(1) == 1 && v.stride(1) == 1 && q.stride(0) == k.stride(0) && q.stride(0) == v.stride(0) &&
-                  k.scalar_type() == q.scalar_type() && v.scalar_type() == q.scalar_type(),
-              op, ": q [rows, heads * dim], k [rows, kv_heads * dim], v [rows, kv_heads * vdim] with one row stride");
-  check_f32(q_weight, dim, op, "q_weight");
-  check_f32(k_weight, dim, op, "k_weight");
-  const auto [kpad, vpad, bs] = head_cache_dims(key_cache, value_cache, kv_heads, q.scalar_type(), op);
-  TORCH_CHECK(slot_mapping.is_cuda() && slot_mapping.scalar_type() == at::kLong && slot_mapping.is_contiguous() &&
-                  slot_mapping.numel() >= rows,
-              op, ": slot_mapping int64 [rows]");
-  auto q_out = torch::empty({rows, heads, kpad}, q.options());
-  check(lvllm_qk_norm_cache(q_out.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(), q.data_ptr(), k.data_ptr(),
-                            v.data_ptr(), q.stride(0), q_weight.data_ptr<float>(), k_weight.data_ptr<float>(), (float)eps,
-                            (int)rows, (int)heads, (int)kv_heads, (int)dim, (int)vdim, (int)kpad, (int)vpad,
-                            slot_mapping.data_ptr<int64_t>(), key_cache.size(0), (int)bs, key_cache.stride(0),
-                            value_cache.stride(0), dtype_code(q, op), current_stream(q)));
-  return q_out;
-}
-
-void head_attention(torch::Tensor& out, const torch::Tensor& q, const torch::Tensor& key_cache,
-                    const torch::Tensor& value_cache, const torch::Tensor& block_tables, const torch::Tensor& seq_lens,
-                    const torch::Tensor& query_start_loc, const std::optional<torch::Tensor>& gate, int64_t vdim,
-                    double scale, double out_scale, int64_t max_query_len, int64_t max_seq_len) {
-  const char* op = "head_attention";
-  LV_CHECK_DEVICE(q);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
-  TORCH_CHECK(q.dim() == 3 && q.is_contiguous(), op, ": contiguous q [rows, heads, kpad]");
-  const int64_t kv_heads = key_cache.size(1), rows = q.size(0), heads = q.size(1);
-  const auto [kpad, vpad, bs] = head_cache_dims(key_cache, value_cache, kv_heads, q.scalar_type(), op);
-  TORCH_CHECK(q.size(2) == kpad && vdim <= vpad, op, ": q and the caches disagree on the padded sizes");
-  TORCH_CHECK(out.is_cuda() && out.dim() == 2 && out.stride(1) == 1 && out.size(0) == rows && out.size(1) == heads * vdim &&
-                  out.scalar_type() == q.scalar_type(),
-              op, ": out [rows, heads * vdim]");
-  if (gate)
-    TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 && gate->stride(1) == 1 && gate->size(0) == rows &&
-                    gate->size(1) == heads && gate->scalar_type() == q.scalar_type(),
-                op, ": gate [rows, heads]");
-  check_layout(query_start_loc, seq_lens, op);
-  TORCH_CHECK(block_tables.is_cuda() && block_tables.dim() == 2 && block_tables.scalar_type() == at::kInt &&
-                  block_tables.is_contiguous() && block_tables.size(0) >= seq_lens.numel(),
-              op, ": block_tables int32 [num_seqs, blocks]");
-  const int ns = (int)seq_lens.numel(), code = dtype_code(q, op);
-  const int64_t need = lvllm_head_attention_workspace_bytes((int)rows, ns, (int)heads, (int)kv_heads, (int)kpad, (int)vpad,
-                                                            (int)bs, (int)max_seq_len, code);
-  torch::Tensor ws;
-  if (need > 0) ws = torch::empty({need}, q.options().dtype(at::kByte));
-  check(lvllm_head_attention(out.data_ptr(), out.stride(0), q.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(),
-                             gate ? gate->data_ptr() : nullptr, gate ? gate->stride(0) : 0, block_tables.data_ptr<int>(),
-                             seq_lens.data_ptr<int>(), query_start_loc.data_ptr<int>(), ns, (int)rows, (int)heads,
-                             (int)kv_heads, (int)kpad, (int)vpad, (int)vdim, (int)block_tables.size(1), (int)bs,
-                             key_cache.size(0), (float)scale, (float)out_scale, key_cache.stride(0), value_cache.stride(0),
-                             (int)max_query_len, (int)max_seq_len, need > 0 ? ws.data_ptr() : nullptr, need, code,
-                             current_stream(q)));
-}
-
-void head_norm_gate(torch::Tensor& out, const torch::Tensor& o, const torch::Tensor& gate, const torch::Tensor& weight,
-                    double eps, double scale) {
-  const char* op = "head_norm_gate";
-  LV_CHECK_DEVICE(o);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(o));
-  TORCH_CHECK(o.dim() == 3 && o.is_contiguous() && o.scalar_type() == at::kFloat, op, ": o float32 [rows, heads, vdim]");
-  const int64_t rows = o.size(0), heads = o.size(1), vdim = o.size(2);
-  TORCH_CHECK(out.dim() == 2 && out.stride(1) == 1 && out.size(0) == rows && out.size(1) == heads * vdim &&
-                  gate.dim() == 2 && gate.stride(1) == 1 && gate.size(0) == rows && gate.size(1) == heads * vdim &&
-                  gate.scalar_type() == out.scalar_type(),
-              op, ": out and gate [rows, heads * vdim]");
-  const bool shared = weight.numel() == vdim;
-  check_f32(weight, shared ? vdim : heads * vdim, op, "weight");
-  check(lvllm_head_norm_gate(out.data_ptr(), out.stride(0), o.data_ptr<float>(), gate.data_ptr(), gate.stride(0),
-                             weight.data_ptr<float>(), shared ? 0 : (int)vdim, (float)eps, (float)scale, (int)rows,
-                             (int)heads, (int)vdim, dtype_code(out, op), current_stream(o)));
-}
-
-torch::Tensor log_decay(const torch::Tensor& u, const torch::Tensor& a_t, const torch::Tensor& bias, int64_t kind,
-                        double inv_tau) {
-  const char* op = "log_decay";
-  LV_CHECK_DEVICE(u);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(u));
-  TORCH_CHECK(u.dim() == 2 && u.stride(1) == 1 && a_t.dim() == 2 && a_t.size(0) == u.size(1), op,
-              ": u [rows, rank], a_t [rank, channels]");
-  check_f32(a_t, a_t.size(0) * a_t.size(1), op, "a_t");
-  check_f32(bias, a_t.size(1), op, "bias");
-  auto out = torch::empty({u.size(0), a_t.size(1)}, u.options().dtype(at::kFloat));
-  check(lvllm_log_decay(out.data_ptr<float>(), u.data_ptr(), u.stride(0), a_t.data_ptr<float>(), bias.data_ptr<float>(),
-                        (int)kind, (float)inv_tau, (int)u.size(0), (int)u.size(1), (int)a_t.size(1), dtype_code(u, op),
-                        current_stream(u)));
-  return out;
-}
-
-torch::Tensor recurrent_scan(const torch::Tensor& q, const torch::Tensor& k, const torch::Tensor& v,
-                             const torch::Tensor& log_decay, const std::optional<torch::Tensor>& bonus, double q_scale,
-                             torch::Tensor& state, const torch::Tensor& state_slots, const torch::Tensor& query_start_loc,
-                             const torch::Tensor& seq_lens) {
-  const char* op = "recurrent_scan";
-  LV_CHECK_DEVICE(q);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
-  TORCH_CHECK(state.dim() == 4, op, ": state [slots, heads, dk, dv]");
-  const int64_t rows = q.size(0), heads = state.size(1), dk = state.size(2), dv = state.size(3);
-  TORCH_CHECK(q.dim() == 2 && k.dim() == 2 && v.dim() == 2 && q.size(1) == heads * dk && k.size(1) == heads * dk &&
-                  v.size(1) == heads * dv && k.size(0) == rows && v.size(0) == rows && q.stride(1) == 1 &&
-                  k.stride(1) == 1 && v.stride(1) == 1 && k.scalar_type() == q.scalar_type() &&
-                  v.scalar_type() == q.scalar_type(),
-              op, ": q, k [rows, heads * dk], v [rows, heads * dv]");
-  check_f32(log_decay, rows * heads * dk, op, "log_decay");
-  if (bonus) check_f32(*bonus, heads * dk, op, "bonus");
-  check_layout(query_start_loc, seq_lens, op);
-  check_state(state, state_slots, heads * dk * dv, seq_lens.numel(), op);
-  auto o = torch::empty({rows, heads, dv}, q.options().dtype(at::kFloat));
-  check(lvllm_recurrent_scan(o.data_ptr<float>(), q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0),
-                             v.stride(0), log_decay.data_ptr<float>(), bonus ? bonus->data_ptr<float>() : nullptr,
-                             (float)q_scale, state.data_ptr<float>(), state.stride(0), state_slots.data_ptr<int>(),
-                             (int)state.size(0), query_start_loc.data_ptr<int>(), seq_lens.data_ptr<int>(),
-                             (int)seq_lens.numel(), (int)heads, (int)dk, (int)dv, dtype_code(q, op), current_stream(q)));
-  return o;
-}
-
-void recurrent_mix(torch::Tensor& out, const torch::Tensor& q, const torch::Tensor& k, const torch::Tensor& v,
-                   const torch::Tensor& u, const torch::Tensor& a_t, const torch::Tensor& decay_bias, int64_t kind,
-                   double inv_tau, const std::optional<torch::Tensor>& bonus, double q_scale, const torch::Tensor& gate,
-                   const torch::Tensor& norm_weight, double eps, double out_scale, torch::Tensor& state,
-                   const torch::Tensor& state_slots, const torch::Tensor& query_start_loc, const torch::Tensor& seq_lens,
-                   int64_t max_query_len) {
-  const char* op = "recurrent_mix";
-  LV_CHECK_DEVICE(q);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
-  TORCH_CHECK(state.dim() == 4, op, ": state [slots, heads, dk, dv]");
-  const int64_t rows = q.size(0), heads = state.size(1), dk = state.size(2), dv = state.size(3), rank = u.size(1);
-  auto rows_of = [&](const torch::Tensor& t, int64_t cols, const char* what) {
-    TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == rows && t.size(1) == cols && t.stride(1) == 1 &&
-                    t.scalar_type() == q.scalar_type(),
-                op, ": ", what, " must be [rows, ", cols, "] of the compute dtype");
-  };
-  rows_of(q, heads * dk, "q");
-  rows_of(k, heads * dk, "k");
-  rows_of(v, heads * dv, "v");
-  rows_of(u, rank, "u");
-  rows_of(gate, heads * dv, "gate");
-  rows_of(out, heads * dv, "out");
-  TORCH_CHECK(a_t.dim() == 2 && a_t.size(0) == rank, op, ": a_t [rank, heads * dk]");
-  check_f32(a_t, rank * heads * dk, op, "a_t");
-  check_f32(decay_bias, heads * dk, op, "decay_bias");
-  if (bonus) check_f32(*bonus, heads * dk, op, "bonus");
-  const bool shared = norm_weight.numel() == dv;
-  check_f32(norm_weight, shared ? dv : heads * dv, op, "norm_weight");
-  check_layout(query_start_loc, seq_lens, op);
-  check_state(state, state_slots, heads * dk * dv, seq_lens.numel(), op);
-  const int ns = (int)seq_lens.numel();
-  if (max_query_len <= 1) TORCH_CHECK(ns == rows, op, ": a step of single tokens has one row per sequence");
-  const int64_t need = lvllm_recurrent_mix_workspace_bytes((int)rows, ns, (int)heads, (int)dk, (int)dv, (int)max_query_len);
-  torch::Tensor ws;
-  if (need > 0) ws = torch::empty({need}, q.options().dtype(at::kByte));
-  check(lvllm_recurrent_mix(out.data_ptr(), out.stride(0), q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0),
-                            k.stride(0), v.stride(0), u.data_ptr(), u.stride(0), a_t.data_ptr<float>(),
-                            decay_bias.data_ptr<float>(), (int)rank, (int)kind, (float)inv_tau,
-                            bonus ? bonus->data_ptr<float>() : nullptr, (float)q_scale, gate.data_ptr(), gate.stride(0),
-                            norm_weight.data_ptr<float>(), shared ? 0 : (int)dv, (float)eps, (float)out_scale,
-                            state.data_ptr<float>(), state.stride(0), state_slots.data_ptr<int>(), (int)state.size(0),
-                            query_start_loc.data_ptr<int>(), seq_lens.data_ptr<int>(), ns, (int)rows, (int)heads, (int)dk,
-                            (int)dv, (int)max_query_len, ws.defined() ? ws.data_ptr() : nullptr, need, dtype_code(q, op), current_stream(q)));
-}
-
 }  // namespace
 
 TORCH_LIBRARY_FRAGMENT(_C, ops) {
@@ -945,36 +667,6 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, amd) {
     check(lvllm_get_tuning(key.c_str(), &v));
     return (int64_t)v;
   });
-}
-
-TORCH_LIBRARY_FRAGMENT(_C_amd, hybrid) {
-  hybrid.def("add_dyt(Tensor(a!) x, Tensor? y, Tensor alpha, Tensor weight, Tensor bias, ScalarType dtype) -> Tensor");
-  hybrid.impl("add_dyt", torch::kCUDA, &add_dyt);
-  hybrid.def("add_dyt_shift_mix(Tensor x, Tensor? y, Tensor mu, Tensor alpha, Tensor weight, Tensor bias, "
-             "Tensor(a!) carried, Tensor state_slots, Tensor query_start_loc, Tensor seq_lens, ScalarType dtype) "
-             "-> (Tensor, Tensor)");
-  hybrid.impl("add_dyt_shift_mix", torch::kCUDA, &add_dyt_shift_mix);
-  hybrid.def("relu_squared(Tensor(a!) out, Tensor x) -> ()");
-  hybrid.impl("relu_squared", torch::kCUDA, &relu_squared);
-  hybrid.def("qk_norm_cache(Tensor q, Tensor k, Tensor v, Tensor q_weight, Tensor k_weight, float eps, int heads, "
-             "int kv_heads, Tensor(a!) key_cache, Tensor(b!) value_cache, Tensor slot_mapping) -> Tensor");
-  hybrid.impl("qk_norm_cache", torch::kCUDA, &qk_norm_cache);
-  hybrid.def("head_attention(Tensor(a!) out, Tensor q, Tensor key_cache, Tensor value_cache, Tensor block_tables, "
-             "Tensor seq_lens, Tensor query_start_loc, Tensor? gate, int vdim, float scale, float out_scale, "
-             "int max_query_len, int max_seq_len) -> ()");
-  hybrid.impl("head_attention", torch::kCUDA, &head_attention);
-  hybrid.def("recurrent_mix(Tensor(a!) out, Tensor q, Tensor k, Tensor v, Tensor u, Tensor a_t, Tensor decay_bias, "
-             "int kind, float inv_tau, Tensor? bonus, float q_scale, Tensor gate, Tensor norm_weight, float eps, "
-             "float out_scale, Tensor(b!) state, Tensor state_slots, Tensor query_start_loc, Tensor seq_lens, "
-             "int max_query_len) -> ()");
-  hybrid.impl("recurrent_mix", torch::kCUDA, &recurrent_mix);
-  hybrid.def("head_norm_gate(Tensor(a!) out, Tensor o, Tensor gate, Tensor weight, float eps, float scale) -> ()");
-  hybrid.impl("head_norm_gate", torch::kCUDA, &head_norm_gate);
-  hybrid.def("log_decay(Tensor u, Tensor a_t, Tensor bias, int kind, float inv_tau) -> Tensor");
-  hybrid.impl("log_decay", torch::kCUDA, &log_decay);
-  hybrid.def("recurrent_scan(Tensor q, Tensor k, Tensor v, Tensor log_decay, Tensor? bonus, float q_scale, "
-             "Tensor(a!) state, Tensor state_slots, Tensor query_start_loc, Tensor seq_lens) -> Tensor");
-  hybrid.impl("recurrent_scan", torch::kCUDA, &recurrent_scan);
 }
 
 TORCH_LIBRARY_FRAGMENT(_C_cuda_utils, cuda_utils) {

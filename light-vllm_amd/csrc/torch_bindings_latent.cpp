@@ -1,0 +1,339 @@
+// torch op registrations of the latent library: latent attention, mixtures of experts, norms on sublayer outputs with depth
+// averages.
+#include "torch_bindings.h"
+
+namespace {
+
+void check_rot(const torch::Tensor& positions, const torch::Tensor& inv_freq, int64_t rows, const char* op) {
+  TORCH_CHECK(positions.is_cuda() && positions.scalar_type() == at::kLong && positions.is_contiguous() &&
+                  positions.numel() >= rows && inv_freq.is_cuda() && inv_freq.scalar_type() == at::kDouble &&
+                  inv_freq.is_contiguous(),
+              op, ": positions int64 [rows] and inv_freq float64 [rot_dims / 2] on the device");
+}
+void check_latent_rows(const torch::Tensor& cache, int64_t cpad, int64_t rpad, const char* op) {
+  TORCH_CHECK(cache.is_cuda() && cache.dim() == 3 && cache.size(2) == cpad + rpad && blocks_are_dense(cache), op,
+              ": cache [blocks, block_size, cpad + rpad], blocks dense");
+}
+void check_rows2d(const torch::Tensor& t, int64_t rows, int64_t cols, at::ScalarType dtype, const char* op, const char* what) {
+  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == rows && t.size(1) == cols && t.stride(1) == 1 &&
+                  t.scalar_type() == dtype,
+              op, ": ", what, " must be [", rows, ", ", cols, "] rows of the compute dtype");
+}
+void check_i32(const torch::Tensor& t, int64_t least, const char* op, const char* what) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kInt && t.is_contiguous() && t.numel() >= least, op, ": ", what,
+              " must be ", least, " or more contiguous int32 elements on the device");
+}
+void check_tables(const torch::Tensor& block_tables, int64_t num_seqs, const char* op) {
+  TORCH_CHECK(block_tables.is_cuda() && block_tables.dim() == 2 && block_tables.scalar_type() == at::kInt &&
+                  block_tables.is_contiguous() && block_tables.size(0) >= num_seqs,
+              op, ": block_tables int32 [num_seqs, blocks]");
+}
+
+void latent_cache(torch::Tensor& cache, const torch::Tensor& kv, const torch::Tensor& weight, double eps, int64_t cpad,
+                  const torch::Tensor& positions, const torch::Tensor& inv_freq, const torch::Tensor& slot_mapping) {
+  const char* op = "latent_cache";
+  LV_CHECK_DEVICE(kv);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(kv));
+  const int64_t rows = kv.size(0), rank = weight.numel(), rpad = cache.size(2) - cpad;
+  check_latent_rows(cache, cpad, rpad, op);
+  check_rows2d(kv, rows, kv.size(1), cache.scalar_type(), op, "kv");
+  check_f32(weight, rank, op, "weight");
+  check_rot(positions, inv_freq, rows, op);
+  TORCH_CHECK(kv.size(1) >= rank && slot_mapping.is_cuda() && slot_mapping.scalar_type() == at::kLong &&
+                  slot_mapping.is_contiguous() && slot_mapping.numel() >= rows,
+              op, ": slot_mapping int64 [rows]");
+  check(lvllm_latent_cache(cache.data_ptr(), cache.stride(0), cache.size(0), (int)cache.size(1), (int)cpad, (int)rpad,
+                           kv.data_ptr(), kv.stride(0), (int)rank, (int)(kv.size(1) - rank), weight.data_ptr<float>(),
+                           (float)eps, positions.data_ptr<int64_t>(), inv_freq.data_ptr<double>(), (int)inv_freq.numel() * 2,
+                           slot_mapping.data_ptr<int64_t>(), (int)rows, dtype_code(kv, op), current_stream(kv)));
+}
+
+torch::Tensor latent_query(const torch::Tensor& q, const torch::Tensor& uk_t, int64_t dim, int64_t rpad,
+                           const torch::Tensor& positions, const torch::Tensor& inv_freq,
+                           const torch::Tensor& query_start_loc, int64_t absorbed_max) {
+  const char* op = "latent_query";
+  LV_CHECK_DEVICE(q);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
+  TORCH_CHECK(uk_t.is_cuda() && uk_t.dim() == 3 && uk_t.is_contiguous() && uk_t.scalar_type() == q.scalar_type(), op,
+              ": uk_t [heads, cpad, dpad]");
+  const int64_t rows = q.size(0), heads = uk_t.size(0), cpad = uk_t.size(1);
+  TORCH_CHECK(q.dim() == 2 && q.size(1) % heads == 0 && q.size(1) / heads >= dim, op, ": q [rows, heads * (dim + rot_dim)]");
+  check_rows2d(q, rows, q.size(1), q.scalar_type(), op, "q");
+  check_rot(positions, inv_freq, rows, op);
+  check_i32(query_start_loc, 1, op, "query_start_loc");
+  auto out = torch::empty({rows, heads, cpad + rpad}, q.options());
+  check(lvllm_latent_query(out.data_ptr(), q.data_ptr(), q.stride(0), uk_t.data_ptr(), (int)heads, (int)dim,
+                           (int)uk_t.size(2), (int)cpad, (int)rpad, (int)(q.size(1) / heads - dim),
+                           (int)inv_freq.numel() * 2, positions.data_ptr<int64_t>(), inv_freq.data_ptr<double>(),
+                           query_start_loc.data_ptr<int>(), (int)query_start_loc.numel() - 1, (int)absorbed_max, (int)rows,
+                           dtype_code(q, op), current_stream(q)));
+  return out;
+}
+
+torch::Tensor latent_attention(const torch::Tensor& q, const torch::Tensor& cache, int64_t cpad,
+                               const torch::Tensor& block_tables, const torch::Tensor& seq_lens,
+                               const torch::Tensor& query_start_loc, double scale, int64_t window, int64_t absorbed_max,
+                               int64_t max_query_len, int64_t max_seq_len) {
+  const char* op = "latent_attention";
+  LV_CHECK_DEVICE(q);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
+  TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.scalar_type() == cache.scalar_type(), op, ": contiguous q [rows, heads, row]");
+  const int64_t rows = q.size(0), heads = q.size(1), rpad = q.size(2) - cpad;
+  check_latent_rows(cache, cpad, rpad, op);
+  check_layout(query_start_loc, seq_lens, op);
+  check_tables(block_tables, seq_lens.numel(), op);
+  const int ns = (int)seq_lens.numel(), code = dtype_code(q, op), bs = (int)cache.size(1);
+  const int64_t need = lvllm_latent_attention_workspace_bytes((int)rows, ns, (int)heads, (int)cpad, (int)rpad, bs, (int)window,
+                                                              (int)absorbed_max, (int)max_query_len, (int)max_seq_len, code);
+  torch::Tensor ws;
+  if (need > 0) ws = torch::empty({need}, q.options().dtype(at::kByte));
+  auto out = torch::empty({rows, heads, cpad}, q.options());
+  check(lvllm_latent_attention(out.data_ptr(), q.data_ptr(), cache.data_ptr(), cache.stride(0), cache.size(0), bs, (int)cpad,
+                               (int)rpad, block_tables.data_ptr<int>(), (int)block_tables.size(1), seq_lens.data_ptr<int>(),
+                               query_start_loc.data_ptr<int>(), ns, (int)rows, (int)heads, (float)scale, (int)window,
+                               (int)absorbed_max, (int)max_query_len, (int)max_seq_len, need > 0 ? ws.data_ptr() : nullptr,
+                               need, code, current_stream(q)));
+  return out;
+}
+
+void latent_value(torch::Tensor& out, const torch::Tensor& o_lat, const torch::Tensor& uv,
+                  const std::optional<torch::Tensor>& gate, int64_t vdim, const torch::Tensor& query_start_loc,
+                  int64_t absorbed_max) {
+  const char* op = "latent_value";
+  LV_CHECK_DEVICE(o_lat);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(o_lat));
+  TORCH_CHECK(o_lat.dim() == 3 && o_lat.is_contiguous(), op, ": contiguous o_lat [rows, heads, cpad]");
+  const int64_t rows = o_lat.size(0), heads = o_lat.size(1), cpad = o_lat.size(2);
+  TORCH_CHECK(uv.is_cuda() && uv.dim() == 3 && uv.is_contiguous() && uv.size(0) == heads && uv.size(2) == cpad &&
+                  uv.scalar_type() == o_lat.scalar_type(),
+              op, ": uv [heads, vpad, cpad]");
+  check_rows2d(out, rows, heads * vdim, o_lat.scalar_type(), op, "out");
+  if (gate) check_rows2d(*gate, rows, heads, o_lat.scalar_type(), op, "gate");
+  check_i32(query_start_loc, 1, op, "query_start_loc");
+  check(lvllm_latent_value(out.data_ptr(), out.stride(0), o_lat.data_ptr(), uv.data_ptr(), gate ? gate->data_ptr() : nullptr,
+                           gate ? gate->stride(0) : 0, (int)heads, (int)vdim, (int)uv.size(1), (int)cpad,
+                           query_start_loc.data_ptr<int>(), (int)query_start_loc.numel() - 1, (int)absorbed_max, (int)rows,
+                           dtype_code(o_lat, op), current_stream(o_lat)));
+}
+
+torch::Tensor latent_gather(const torch::Tensor& cache, const torch::Tensor& starts, const torch::Tensor& first,
+                            const torch::Tensor& seq_lens, const torch::Tensor& block_tables, int64_t n) {
+  const char* op = "latent_gather";
+  LV_CHECK_DEVICE(cache);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(cache));
+  check_latent_rows(cache, cache.size(2), 0, op);
+  const int64_t ns = seq_lens.numel();
+  check_i32(seq_lens, ns, op, "seq_lens");
+  check_i32(starts, ns + 1, op, "starts");
+  check_i32(first, ns, op, "first");
+  check_tables(block_tables, ns, op);
+  auto out = torch::empty({n, cache.size(2)}, cache.options());
+  check(lvllm_latent_gather(out.data_ptr(), cache.data_ptr(), cache.stride(0), cache.size(0), (int)cache.size(1),
+                            (int)cache.size(2), starts.data_ptr<int>(), first.data_ptr<int>(), seq_lens.data_ptr<int>(),
+                            block_tables.data_ptr<int>(), (int)block_tables.size(1), (int)ns, (int)n, dtype_code(cache, op),
+                            current_stream(cache)));
+  return out;
+}
+
+std::tuple<torch::Tensor, torch::Tensor> latent_expand(const torch::Tensor& kv, const torch::Tensor& rows, int64_t cpad,
+                                                       int64_t heads, int64_t dim, int64_t rot_dim, int64_t vdim, int64_t kpad,
+                                                       int64_t vpad) {
+  const char* op = "latent_expand";
+  LV_CHECK_DEVICE(kv);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(kv));
+  const int64_t n = rows.size(0);
+  TORCH_CHECK(rows.dim() == 2 && rows.is_contiguous() && rows.scalar_type() == kv.scalar_type() && cpad + rot_dim <= rows.size(1) &&
+                  n % 16 == 0,
+              op, ": gathered rows [16 n, cpad + rpad]");
+  check_rows2d(kv, n, heads * (dim + vdim), rows.scalar_type(), op, "kv");
+  auto k = torch::empty({n / 16, heads, kpad / 8, 16, 8}, kv.options());
+  auto v = torch::empty({n / 16, heads, vpad, 16}, kv.options());
+  check(lvllm_latent_expand(k.data_ptr(), v.data_ptr(), kv.data_ptr(), kv.stride(0), rows.data_ptr(), (int)rows.size(1),
+                            (int)cpad, (int)n, (int)heads, (int)dim, (int)rot_dim, (int)vdim, (int)kpad, (int)vpad,
+                            dtype_code(kv, op), current_stream(kv)));
+  return {k, v};
+}
+
+torch::Tensor latent_rotate_query(const torch::Tensor& q, int64_t heads, int64_t dim, int64_t kpad,
+                                  const torch::Tensor& positions, const torch::Tensor& inv_freq) {
+  const char* op = "latent_rotate_query";
+  LV_CHECK_DEVICE(q);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
+  const int64_t rows = q.size(0);
+  TORCH_CHECK(heads > 0 && q.dim() == 2 && q.size(1) % heads == 0 && q.size(1) / heads >= dim, op, ": q [rows, heads * (dim + rot_dim)]");
+  check_rows2d(q, rows, q.size(1), q.scalar_type(), op, "q");
+  check_rot(positions, inv_freq, rows, op);
+  auto out = torch::empty({rows, heads, kpad}, q.options());
+  check(lvllm_latent_rotate_query(out.data_ptr(), q.data_ptr(), q.stride(0), (int)heads, (int)dim,
+                                  (int)(q.size(1) / heads - dim), (int)kpad, positions.data_ptr<int64_t>(),
+                                  inv_freq.data_ptr<double>(), (int)inv_freq.numel() * 2, (int)rows, dtype_code(q, op),
+                                  current_stream(q)));
+  return out;
+}
+
+std::tuple<torch::Tensor, torch::Tensor> moe_route(const torch::Tensor& h, const torch::Tensor& w, const torch::Tensor& bias,
+                                                   int64_t top) {
+  const char* op = "moe_route";
+  LV_CHECK_DEVICE(h);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(h));
+  const int64_t rows = h.size(0), width = h.size(1), experts = bias.numel(), shared = w.size(0) - experts;
+  TORCH_CHECK(h.dim() == 2 && h.is_contiguous() && w.is_cuda() && w.dim() == 2 && w.is_contiguous() && w.size(1) == width &&
+                  w.scalar_type() == h.scalar_type() && (shared == 0 || shared == 1),
+              op, ": h [rows, width], w [experts (+ 1), width]");
+  check_f32(bias, experts, op, "bias");
+  auto ids = torch::empty({rows, top + shared}, h.options().dtype(at::kInt));
+  auto weights = torch::empty({rows, top + shared}, h.options().dtype(at::kFloat));
+  check(lvllm_moe_route(ids.data_ptr<int>(), weights.data_ptr<float>(), h.data_ptr(), w.data_ptr(), bias.data_ptr<float>(),
+                        (int)experts, (int)shared, (int)top, (int)rows, (int)width, dtype_code(h, op), current_stream(h)));
+  return {ids, weights};
+}
+
+std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_group(const torch::Tensor& ids, int64_t experts,
+                                                                                 bool packed) {
+  const char* op = "moe_group";
+  TORCH_CHECK(ids.dim() == 2, op, ": ids [rows, assignments]");
+  check_i32(ids, ids.numel(), op, "ids");
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(ids));
+  const int64_t total = ids.numel(), tile = lvllm_moe_tile(packed);
+  const int64_t max_tiles = std::min(total, total / tile + experts);
+  auto offsets = torch::empty({experts + 1}, ids.options()), token = torch::empty({total}, ids.options());
+  auto slot = torch::empty_like(ids), tiles = torch::empty({max_tiles, 2}, ids.options());
+  check(lvllm_moe_group(offsets.data_ptr<int>(), token.data_ptr<int>(), slot.data_ptr<int>(), tiles.data_ptr<int>(),
+                        ids.data_ptr<int>(), (int)total, (int)ids.size(1), (int)experts, packed, (int)max_tiles,
+                        current_stream(ids)));
+  return {offsets, token, slot, tiles};
+}
+
+torch::Tensor moe_experts(const torch::Tensor& x, const torch::Tensor& w, const torch::Tensor& w_offset,
+                          const torch::Tensor& ff, const torch::Tensor& limit, const torch::Tensor& offsets,
+                          const torch::Tensor& token, const torch::Tensor& tiles, int64_t rows, int64_t width, int64_t ff_max,
+                          bool up, bool packed) {
+  const char* op = "moe_experts";
+  LV_CHECK_DEVICE(x);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
+  const int64_t experts = ff.numel(), slots = token.numel();
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.size(0) == (up ? rows : slots) && x.size(1) == (up ? width : ff_max), op,
+              ": x must be [rows, width] going up, [slots, ff_max] going down");
+  TORCH_CHECK(w.is_cuda() && w.is_contiguous() && w.scalar_type() == x.scalar_type() && w_offset.is_cuda() &&
+                  w_offset.scalar_type() == at::kLong && w_offset.numel() == experts,
+              op, ": one weight buffer and int64 offsets [experts]");
+  check_i32(ff, experts, op, "ff");
+  check_f32(limit, experts, op, "limit");
+  check_i32(offsets, experts + 1, op, "offsets");
+  check_i32(token, slots, op, "token");
+  check_i32(tiles, 2, op, "tiles");
+  auto out = torch::empty({slots, up ? ff_max : width}, x.options());
+  check(lvllm_moe_experts(out.data_ptr(), x.data_ptr(), w.data_ptr(), w_offset.data_ptr<int64_t>(), ff.data_ptr<int>(),
+                          limit.data_ptr<float>(), offsets.data_ptr<int>(), token.data_ptr<int>(), tiles.data_ptr<int>(),
+                          (int)experts, (int)slots, (int)rows, (int)width, (int)ff_max, (int)tiles.size(0), up, packed,
+                          dtype_code(x, op), current_stream(x)));
+  return out;
+}
+
+torch::Tensor embed_scale(torch::Tensor& x, const torch::Tensor& table, const torch::Tensor& ids, double scale) {
+  const char* op = "embed_scale";
+  check_residual(x, op);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
+  TORCH_CHECK(table.is_cuda() && table.dim() == 2 && table.is_contiguous() && table.size(1) == x.size(1) && ids.is_cuda() &&
+                  ids.scalar_type() == at::kLong && ids.is_contiguous() && ids.numel() == x.size(0),
+              op, ": table [vocab, width], ids int64 [rows]");
+  auto h = torch::empty(x.sizes(), table.options());
+  check(lvllm_embed_scale(x.data_ptr<float>(), h.data_ptr(), table.data_ptr(), ids.data_ptr<int64_t>(), (float)scale,
+                          (int)x.size(0), (int)table.size(0), (int)x.size(1), dtype_code(table, op), current_stream(x)));
+  return h;
+}
+
+// y: rows of the compute dtype, fp32 slabs [s, rows, width], or (with slots and weights) the slots of a mixture
+torch::Tensor norm_add_mix(const std::optional<torch::Tensor>& x_out, const std::optional<torch::Tensor>& v_out,
+                           const torch::Tensor& x, const torch::Tensor& y, const std::optional<torch::Tensor>& slots,
+                           const std::optional<torch::Tensor>& slot_weights, const torch::Tensor& gain, double eps,
+                           const std::optional<torch::Tensor>& streams, const std::optional<torch::Tensor>& weights,
+                           const std::optional<torch::Tensor>& out_gain, at::ScalarType dtype) {
+  const char* op = "norm_add_mix";
+  check_residual(x, op);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
+  const int64_t rows = x.size(0), width = x.size(1);
+  check_f32(gain, 1, op, "gain");
+  if (out_gain) check_f32(*out_gain, 1, op, "out_gain");
+  for (const auto* t : {&x_out, &v_out})
+    if (*t) {
+      check_residual(**t, op);
+      TORCH_CHECK((*t)->sizes() == x.sizes(), op, ": outputs of the residual's shape");
+    }
+  Addend a;
+  int per_row = 0, total = 0;
+  if (slots) {
+    TORCH_CHECK(slot_weights && slots->dim() == 2 && slots->size(0) == rows && y.is_cuda() && y.dim() == 2 && y.is_contiguous() &&
+                    y.size(1) == width && y.scalar_type() == dtype,
+                op, ": slots int32 [rows, n] of y [slots, width], with their weights");
+    check_i32(*slots, slots->numel(), op, "slots");
+    check_f32(*slot_weights, slots->numel(), op, "slot_weights");
+    a.y = y.data_ptr();
+    per_row = (int)slots->size(1);
+    total = (int)y.size(0);
+  } else {
+    a = addend_of(y, x, dtype, op);
+  }
+  int num_streams = 0;
+  int64_t stream_stride = 0;
+  TORCH_CHECK(!streams || weights, op, ": streams need weights");
+  if (weights) {
+    num_streams = streams ? (int)streams->size(0) : 0;
+    check_f32(*weights, num_streams + 1, op, "weights");
+    if (streams) {
+      TORCH_CHECK(streams->is_cuda() && streams->dim() == 3 && streams->scalar_type() == at::kFloat && streams->size(1) == rows &&
+                      streams->size(2) == width && (rows == 0 || (*streams)[0].is_contiguous()),
+                  op, ": streams float32 [n, rows, width], each contiguous");
+      stream_stride = streams->stride(0);
+    }
+  }
+  auto h = torch::empty(x.sizes(), x.options().dtype(dtype));
+  check(lvllm_norm_add_mix(x_out ? x_out->data_ptr<float>() : nullptr, v_out ? v_out->data_ptr<float>() : nullptr, h.data_ptr(),
+                           x.data_ptr<float>(), a.y, a.partials, a.num, slots ? slots->data_ptr<int>() : nullptr,
+                           slots ? slot_weights->data_ptr<float>() : nullptr, per_row, total, gain.data_ptr<float>(), (float)eps,
+                           streams ? streams->data_ptr<float>() : nullptr, stream_stride, num_streams,
+                           weights ? weights->data_ptr<float>() : nullptr, out_gain ? out_gain->data_ptr<float>() : nullptr,
+                           (float)eps, (int)rows, (int)width, dtype_code(h, op), current_stream(x)));
+  return h;
+}
+
+}  // namespace
+
+TORCH_LIBRARY_FRAGMENT(_C_amd, latent) {
+  latent.def("latent_cache(Tensor(a!) cache, Tensor kv, Tensor weight, float eps, int cpad, Tensor positions, Tensor inv_freq, "
+             "Tensor slot_mapping) -> ()");
+  latent.impl("latent_cache", torch::kCUDA, &latent_cache);
+  latent.def("latent_query(Tensor q, Tensor uk_t, int dim, int rpad, Tensor positions, Tensor inv_freq, "
+             "Tensor query_start_loc, int absorbed_max) -> Tensor");
+  latent.impl("latent_query", torch::kCUDA, &latent_query);
+  latent.def("latent_attention(Tensor q, Tensor cache, int cpad, Tensor block_tables, Tensor seq_lens, "
+             "Tensor query_start_loc, float scale, int window, int absorbed_max, int max_query_len, int max_seq_len) -> Tensor");
+  latent.impl("latent_attention", torch::kCUDA, &latent_attention);
+  latent.def("latent_value(Tensor(a!) out, Tensor o_lat, Tensor uv, Tensor? gate, int vdim, Tensor query_start_loc, "
+             "int absorbed_max) -> ()");
+  latent.impl("latent_value", torch::kCUDA, &latent_value);
+  latent.def("latent_gather(Tensor cache, Tensor starts, Tensor first, Tensor seq_lens, Tensor block_tables, int n) -> Tensor");
+  latent.impl("latent_gather", torch::kCUDA, &latent_gather);
+  latent.def("latent_expand(Tensor kv, Tensor rows, int cpad, int heads, int dim, int rot_dim, int vdim, int kpad, int vpad) "
+             "-> (Tensor, Tensor)");
+  latent.impl("latent_expand", torch::kCUDA, &latent_expand);
+  latent.def("latent_rotate_query(Tensor q, int heads, int dim, int kpad, Tensor positions, Tensor inv_freq) -> Tensor");
+  latent.impl("latent_rotate_query", torch::kCUDA, &latent_rotate_query);
+  latent.def("moe_route(Tensor h, Tensor w, Tensor bias, int top) -> (Tensor, Tensor)");
+  latent.impl("moe_route", torch::kCUDA, &moe_route);
+  latent.def("moe_group(Tensor ids, int experts, bool packed) -> (Tensor, Tensor, Tensor, Tensor)");
+  latent.impl("moe_group", torch::kCUDA, &moe_group);
+  latent.def("moe_experts(Tensor x, Tensor w, Tensor w_offset, Tensor ff, Tensor limit, Tensor offsets, Tensor token, "
+             "Tensor tiles, int rows, int width, int ff_max, bool up, bool packed) -> Tensor");
+  latent.impl("moe_experts", torch::kCUDA, &moe_experts);
+  latent.def("embed_scale(Tensor(a!) x, Tensor table, Tensor ids, float scale) -> Tensor");
+  latent.impl("embed_scale", torch::kCUDA, &embed_scale);
+  latent.def("norm_add_mix(Tensor(a!)? x_out, Tensor(b!)? v_out, Tensor x, Tensor y, Tensor? slots, Tensor? slot_weights, "
+             "Tensor gain, float eps, Tensor? streams, Tensor? weights, Tensor? out_gain, ScalarType dtype) -> Tensor");
+  latent.impl("norm_add_mix", torch::kCUDA, &norm_add_mix);
+}
+
+PyMODINIT_FUNC PyInit__C_latent(void) {
+  static struct PyModuleDef module = {PyModuleDef_HEAD_INIT, "_C_latent", nullptr, 0, nullptr};
+  return PyModule_Create(&module);
+}

@@ -59,7 +59,7 @@ class CacheEngine:
         from .mixers import LayerCache
         kv = iter(self.gpu_cache)
         return ModelCaches([LayerCache(next(kv) if spec is not None else None, state)
-                            for spec, state in zip(self.kv_specs, self.state)], self.block_size)
+                            for spec, state in zip(self.kv_specs, self.state or [{}] * len(self.kv_specs))], self.block_size)
 
     def copy_state(self, pairs: List[Tuple[int, int]]) -> None:
         """Forked sequences: [(source slot, destination slot)] of every layer's state."""

@@ -7,9 +7,8 @@ import torch
 import torch.nn.functional as F
 
 from .hybrid_config import HybridModelConfig, ParallelMixerConfig
-from .mixers import DynTanhNorm, LayerCache, ParallelMixer, SquaredReluMlp, StepLayout, TimeMixer
-from .model import Weight, linear
-from .weights import load_checkpoint
+from .layered_model import LayeredModel
+from .mixers import DynTanhNorm, LayerCache, ParallelMixer, SquaredReluMlp, TimeMixer
 
 
 def tensor_shapes(cfg: HybridModelConfig) -> Dict[str, tuple]:
@@ -71,23 +70,12 @@ def random_tensor(name: str, shape: tuple, gen: torch.Generator, device) -> torc
     return t * shape[-1] ** -0.5
 
 
-class HybridModel:
-    """forward(input_ids, positions, caches, attn_metadata) -> normed hidden states [rows, width]."""
+class HybridModel(LayeredModel):
 
-    def __init__(self, cfg: HybridModelConfig, attn_impl, device="cuda:0", seed: int = 0, tensors=None):
-        """Weights come from `tensors` (name -> tensor), else from cfg.weights_dir, else from the seed."""
-        self.cfg, self.device, self.attn = cfg, torch.device(device), attn_impl
-        if tensors is None and cfg.weights_dir is not None:
-            tensors = load_checkpoint(cfg.weights_dir)
-        if tensors is None:
-            gen, shapes = torch.Generator(device=self.device).manual_seed(seed), tensor_shapes(cfg)
+    tensor_shapes, random_tensor = staticmethod(tensor_shapes), staticmethod(random_tensor)
 
-            def get(name):
-                return random_tensor(name, shapes[name], gen, self.device).to(cfg.dtype)
-        else:
-            def get(name):
-                return tensors[name].to(self.device).to(cfg.dtype)
-        pack = cfg.pack_weights and self.device.type == "cuda"
+    def load(self, get, pack: bool) -> None:
+        cfg = self.cfg
         self.embed = get("embed").float()
         self.layers: List[tuple] = []
         for i, l in enumerate(cfg.layers):
@@ -97,7 +85,6 @@ class HybridModel:
             else:
                 self.layers.append(self._layer(get, f"l{j}", l, pack))
         self.final_norm = DynTanhNorm(get, "final.norm")
-        self.head = Weight(get("head").contiguous(), pack and cfg.dtype != torch.float32)
 
     def _layer(self, get, name: str, l, pack: bool):
         mixer = (ParallelMixer if isinstance(l.mixer, ParallelMixerConfig) else TimeMixer)(
@@ -106,15 +93,11 @@ class HybridModel:
         ff = (DynTanhNorm(get, name + ".norm2"), SquaredReluMlp(get, name + ".mlp", pack)) if l.ff is not None else None
         return DynTanhNorm(get, name + ".norm1"), mixer, ff
 
-    def step_layout(self, md, block_size: int) -> StepLayout:
-        return StepLayout(md.query_start_loc, md.seq_lens_tensor, md.block_tables, md.slot_mapping, md.state_slots,
-                          md.max_query_len or 1, max(md.max_prefill_seq_len or 0, md.max_decode_seq_len or 0), block_size)
-
     def forward(self, input_ids: torch.Tensor, positions: torch.Tensor, caches: List[LayerCache], attn_metadata,
                 on_layer=None) -> torch.Tensor:
         """`on_layer(i, x)`: called with the residual stream after every layer (tests)."""
         dtype = self.cfg.dtype
-        step = self.step_layout(attn_metadata, caches.block_size)
+        step = self.step_layout(attn_metadata, positions, caches.block_size)
         x, y = F.embedding(input_ids, self.embed), None
         for i, ((norm1, mixer, ff), cache) in enumerate(zip(self.layers, caches.layers)):
             x, y = mixer(x, y, norm1, cache, step, self.attn, dtype)
@@ -124,15 +107,6 @@ class HybridModel:
             if on_layer is not None:
                 on_layer(i, x + (y.sum(0) if y.dim() == 3 else y).float())
         return self.final_norm(x, y, dtype)
-
-    def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
-        return linear(hidden, self.head)
-
-    def greedy_tokens(self, hidden: torch.Tensor) -> torch.Tensor:
-        w = self.head
-        if 0 < hidden.shape[0] <= 64 and w.packed is not None:
-            return torch.ops._C_amd.skinny_linear_packed_argmax(hidden, w.packed, w.N, w.K)
-        return torch.argmax(self.compute_logits(hidden), dim=-1)
 
     def weight_bytes(self) -> int:
         n, seen = self.head.numel(), set()

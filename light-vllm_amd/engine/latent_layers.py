@@ -1,0 +1,222 @@
+"""Sublayers of latent decoders on the gfx950 operators: latent attention, the mixture of experts, and the norm on a
+sublayer's output with the residual add and the average over the depth.
+
+A mixer takes the rows h it reads (compute dtype) and returns its projection: [rows, width], or the fp32 split-K slabs of a
+decode-size step; the mixture returns its assignments' rows, which the norm's launch sums.  Constants come from the
+configuration; nothing here knows a model's sizes."""
+from dataclasses import dataclass
+from typing import Dict, List, NamedTuple, Optional
+
+import numpy as np
+import torch
+import torch.nn.functional as F
+
+from .hybrid_config import KVSpec
+from .latent_config import LatentAttentionConfig, MixtureConfig, RotationConfig
+from .mixers import StepLayout, ceil_to, make_weight, pad_columns, project_to_residual, stack_rows
+from .model import linear
+
+amd = torch.ops._C_amd
+ABSORBED_MAX = 64      # portions of up to this many tokens attend in latent space (csrc/latent_attention.h)
+UNBOUNDED = 1 << 30
+
+
+class SublayerOutput(NamedTuple):
+    """What a sublayer adds to the stream: rows (or split-K slabs), or the rows of a mixture's slots."""
+    y: torch.Tensor
+    slots: Optional[torch.Tensor] = None      # int32 [rows, assignments]
+    weights: Optional[torch.Tensor] = None    # float32 [rows, assignments]
+
+
+class OutputNorm:
+    """RMS norm of a sublayer's output with one gain for all coordinates, added to the stream; then, after a layer, the
+    average over the depth, and after the last one the model's norm."""
+
+    def __init__(self, get, name: str, eps: float):
+        self.gain, self.eps = get(name).float().reshape(1), eps
+
+    def __call__(self, out: SublayerOutput, x: torch.Tensor, dtype, *, x_out=None, v_out=None, streams=None, depth=None,
+                 final: Optional["OutputNorm"] = None) -> torch.Tensor:
+        return amd.norm_add_mix(x_out, v_out, x, out.y, out.slots, out.weights, self.gain, self.eps, streams, depth,
+                                final.gain if final is not None else None, dtype)
+
+
+class Rotation:
+    """Frequencies in double: angles are taken in double and reduced before the fp32 sine and cosine."""
+
+    def __init__(self, cfg: RotationConfig, device):
+        i = torch.arange(0, cfg.dims, 2, dtype=torch.float64, device=device)
+        self.inv_freq = float(cfg.base) ** (-i / max(cfg.dims, 1))
+
+
+@dataclass
+class LongPortions:
+    """A step's sequences that attend over expanded keys, for one window: where their keys lie, back to back."""
+    n: int                       # gathered rows, every sequence from a multiple of 16
+    starts: torch.Tensor         # int32 [num_seqs + 1]
+    first: torch.Tensor          # int32 [num_seqs]: the first key taken (a multiple of the page size)
+    seq_lens: torch.Tensor       # int32 [num_seqs], counted from the first key taken
+    tables: torch.Tensor         # int32 [num_seqs, pages]
+    max_seq_len: int
+
+
+def plan_long_portions(query_lens: List[int], context_lens: List[int], window: int, longest_short: int, page: int, device):
+    """None when every sequence is short."""
+    q, c = np.asarray(query_lens, np.int64), np.asarray(context_lens, np.int64)
+    long = q > longest_short
+    if not long.any():
+        return None
+    first = np.maximum(c - window + 1, 0) // page * page
+    keys = np.where(long, c + q - first, 0)
+    starts = np.zeros(len(q) + 1, np.int64)
+    np.cumsum(-(-keys // page) * page, out=starts[1:])
+    pages = int(-(-keys.max() // page))
+    tables = starts[:-1, None] // page + np.arange(pages)[None]
+    tables = np.minimum(tables, starts[-1] // page - 1)
+    seq_lens = np.where(long, keys, q)
+    flat = torch.from_numpy(np.concatenate([starts, first, seq_lens, tables.reshape(-1)]).astype(np.int32))
+    if torch.device(device).type == "cuda":
+        flat = flat.pin_memory().to(device, non_blocking=True)
+    ns = len(q)
+    # (pieces begin anywhere: the kernels read single int32s)
+    return LongPortions(int(starts[-1]), flat[:ns + 1], flat[ns + 1:2 * ns + 1], flat[2 * ns + 1:3 * ns + 1],
+                        flat[3 * ns + 1:].view(ns, pages), int(keys.max()))
+
+
+class LatentStep:
+    """A step's layout and what its layers share: the plans of long portions per window, gathered latents per cache."""
+
+    def __init__(self, layout: StepLayout):
+        self.layout = layout
+        self._plans: Dict[int, Optional[LongPortions]] = {}
+        self._gathered: Dict[tuple, torch.Tensor] = {}
+
+    def long_portions(self, window: int) -> Optional[LongPortions]:
+        l = self.layout
+        if l.query_lens is None or l.max_query_len <= ABSORBED_MAX:
+            return None
+        if window not in self._plans:
+            self._plans[window] = plan_long_portions(l.query_lens, l.context_lens, window, ABSORBED_MAX, l.block_size,
+                                                     l.seq_lens.device)
+        return self._plans[window]
+
+    def gathered(self, layer: int, window: int, rows_view: torch.Tensor, plan: LongPortions) -> torch.Tensor:
+        key = (layer, window)
+        if key not in self._gathered:
+            l = self.layout
+            self._gathered[key] = amd.latent_gather(rows_view, plan.starts, plan.first, l.seq_lens, l.block_tables, plan.n)
+        return self._gathered[key]
+
+
+class LatentAttention:
+
+    def __init__(self, get, name: str, cfg: LatentAttentionConfig, eps: float, pack: bool):
+        self.cfg, self.eps, self.spec = cfg, eps, cfg.spec
+        H = cfg.heads
+        parts = [get(name + ".q"), get(name + ".g")]
+        if cfg.kv_from is None:
+            parts.append(get(name + ".dkv"))
+            self.norm = get(name + ".dkv.norm").float()
+        stack, self.at = stack_rows(parts)
+        self.sizes = [p.shape[0] for p in parts]
+        self.proj = make_weight(stack, pack)
+        uk, uv = get(name + ".uk"), get(name + ".uv")
+        dpad, vpad, cpad = ceil_to(cfg.dim, 32), ceil_to(cfg.vdim, 16), self.spec.cpad
+        self.uk_t = uk.new_zeros(H, cpad, dpad)
+        self.uk_t[:, :cfg.kv_rank, :cfg.dim] = uk.view(H, cfg.dim, cfg.kv_rank).transpose(1, 2)
+        self.uv = uv.new_zeros(H, vpad, cpad)
+        self.uv[:, :cfg.vdim, :cfg.kv_rank] = uv.view(H, cfg.vdim, cfg.kv_rank)
+        self.pages = KVSpec(H, cfg.dim + cfg.rot_dim, cfg.vdim)  # of expanded keys and values
+        # long portions take the expanded way where head_attention has a matrix-core body
+        self.expands = uk.dtype == torch.bfloat16 and uk.is_cuda and self.pages.kpad <= 256 and self.pages.vpad <= 256
+        self.expand = F.pad(torch.cat([uk, uv]), (0, cpad - cfg.kv_rank)).contiguous() if self.expands else None
+        self.rotation = Rotation(cfg.rot, uk.device)
+        self.out_cols = H * cfg.vdim
+        self.out = make_weight(pad_columns(get(name + ".o")), pack)
+
+    def weights(self):
+        return [self.proj, self.out]
+
+    def __call__(self, h: torch.Tensor, kv: torch.Tensor, layer: int, step: LatentStep, attn) -> SublayerOutput:
+        """`kv`: the cache of layer number `layer`, this one's own or the one it reads."""
+        c, l, spec, inv_freq = self.cfg, step.layout, self.spec, self.rotation.inv_freq
+        proj = linear(h, self.proj)
+        q, gate, *dkv = (proj[:, o:o + n] for o, n in zip(self.at, self.sizes))
+        cache = attn.rows_view(kv, spec, l.block_size)
+        if dkv:
+            amd.latent_cache(cache, dkv[0], self.norm, self.eps, spec.cpad, l.positions, inv_freq, l.slot_mapping)
+        rows = h.shape[0]
+        heads_out = (torch.empty if self.out.K == self.out_cols else torch.zeros)(rows, self.out.K, dtype=h.dtype, device=h.device)
+        out = heads_out[:, :self.out_cols]
+        plan = step.long_portions(c.window) if self.expands and l.block_size == 16 else None
+        longest = ABSORBED_MAX if plan is not None else UNBOUNDED
+        if plan is None or min(l.query_lens) <= ABSORBED_MAX:
+            qa = amd.latent_query(q, self.uk_t, c.dim, spec.rpad, l.positions, inv_freq, l.query_start_loc, longest)
+            o = amd.latent_attention(qa, cache, spec.cpad, l.block_tables, l.seq_lens, l.query_start_loc, c.scale, c.window,
+                                     longest, l.max_query_len, l.max_seq_len)
+            amd.latent_value(out, o, self.uv, gate, c.vdim, l.query_start_loc, longest)
+        if plan is not None:
+            self._long(out, q, gate, cache, layer, plan, step)
+        return SublayerOutput(project_to_residual(heads_out, self.out))
+
+    def _long(self, out, q, gate, cache, layer: int, plan: LongPortions, step: LatentStep) -> None:
+        c, l, spec, p = self.cfg, step.layout, self.spec, self.pages
+        lat = step.gathered(layer, c.window, cache, plan)
+        kv = F.linear(lat[:, :spec.cpad], self.expand)
+        keys, values = amd.latent_expand(kv, lat, spec.cpad, c.heads, c.dim, c.rot_dim, c.vdim, p.kpad, p.vpad)
+        qr = amd.latent_rotate_query(q, c.heads, c.dim, p.kpad, l.positions, self.rotation.inv_freq)
+        amd.head_attention(out, qr, keys, values, plan.tables, plan.seq_lens, l.query_start_loc, gate, c.vdim, c.scale, 1.0,
+                           l.max_query_len, plan.max_seq_len, c.window, ABSORBED_MAX + 1)
+
+
+def interleave_16(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+    """[ff, k] twice -> [2 ffp, k]: 16 rows of one, 16 of the other, ...; ffp: ff up to a multiple of 32 with zero rows."""
+    pad = ceil_to(gate.shape[0], 32) - gate.shape[0]
+    g, u = (F.pad(t, (0, 0, 0, pad)).view(-1, 1, 16, t.shape[1]) for t in (gate, up))
+    return torch.cat([g, u], 1).reshape(-1, gate.shape[1])
+
+
+class MixtureOfExperts:
+    """The shared expert is one more expert of the grouped products, with sizes and a limit of its own."""
+
+    def __init__(self, get, name: str, cfg: MixtureConfig, pack: bool):
+        self.cfg = cfg
+        router, self.bias = get(name + ".router"), get(name + ".router.b").float().contiguous()
+        names, ff = [f"{name}.e{i}" for i in range(cfg.experts)], [cfg.expert.ff] * cfg.experts
+        limits = [cfg.expert.limit] * cfg.experts
+        if cfg.shared is not None:
+            names.append(name + ".shared")
+            ff.append(cfg.shared.ff)
+            limits.append(cfg.shared.limit)
+            router = torch.cat([router, get(name + ".shared.sg")])
+        self.router = router.contiguous()
+        self.width, dev = router.shape[1], router.device
+        self.packed = pack and router.dtype == torch.bfloat16 and self.width % 32 == 0
+        ffp = [ceil_to(n, 32) for n in ff]
+        self.ff_max, self.experts = max(ffp), len(names)
+        up_at, down_at = ([0] + np.cumsum([k * n * self.width for n in ffp]).tolist() for k in (2, 1))
+        self.up = torch.empty(up_at[-1], dtype=router.dtype, device=dev)
+        self.down = torch.empty(down_at[-1], dtype=router.dtype, device=dev)
+        for i, s in enumerate(names):
+            up = interleave_16(get(s + ".gate"), get(s + ".up"))
+            down = pad_columns(get(s + ".down")).contiguous()
+            if self.packed:
+                up, down = amd.pack_weight(up), amd.pack_weight(down)
+            self.up[up_at[i]:up_at[i + 1]] = up.reshape(-1)
+            self.down[down_at[i]:down_at[i + 1]] = down.reshape(-1)
+        self.up_at, self.down_at = (torch.tensor(a[:-1], dtype=torch.int64, device=dev) for a in (up_at, down_at))
+        self.ff = torch.tensor(ffp, dtype=torch.int32, device=dev)
+        self.limits = torch.tensor(limits, dtype=torch.float32, device=dev)
+
+    def numel(self) -> int:
+        return self.up.numel() + self.down.numel()
+
+    def __call__(self, h: torch.Tensor) -> SublayerOutput:
+        ids, weights = amd.moe_route(h, self.router, self.bias, self.cfg.top)
+        offsets, token, slots, tiles = amd.moe_group(ids, self.experts, self.packed)
+        rows = h.shape[0]
+        a = amd.moe_experts(h, self.up, self.up_at, self.ff, self.limits, offsets, token, tiles, rows, self.width, self.ff_max,
+                            True, self.packed)
+        y = amd.moe_experts(a, self.down, self.down_at, self.ff, self.limits, offsets, token, tiles, rows, self.width,
+                            self.ff_max, False, self.packed)
+        return SublayerOutput(y, slots, weights)

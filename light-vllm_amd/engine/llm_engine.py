@@ -438,11 +438,11 @@ class LLMEngine:
         self.device = torch.device(device)
         torch.cuda.set_device(self.device)
         self.attn_backend = model_entry(model_config.architecture).backend_cls()()
-        if model_config.state_specs() is not None:
-            if cache_config.enable_prefix_caching:
-                raise ValueError("prefix caching needs the state at a block's end, which a recurrent model does not keep")
-            if cache_config.cache_dtype != "auto" or cache_config.sliding_window is not None:
-                raise ValueError("hybrid decoders cache in the model's dtype, without a sliding window")
+        if model_config.state_specs() is not None and cache_config.enable_prefix_caching:
+            raise ValueError("prefix caching needs the state at a block's end, which a recurrent model does not keep")
+        if model_config.kv_cache_specs() is not None and (cache_config.cache_dtype != "auto"
+                                                          or cache_config.sliding_window is not None):
+            raise ValueError("decoders of listed layers cache in the model's dtype, without a sliding window of the cache")
         # (multi-step decode over the prefix-caching allocator: the reference's v2 manager under lookahead is replayed
         # bit for bit -- tests/golden/block_manager_v2_cached_lookahead*.json, scheduler_lookahead_prefix_cache_v2.json)
         # steps in flight run on separate streams (a stream per task, core/executor.py:62-93), so
@@ -988,7 +988,7 @@ class LLMEngine:
         if own_caches:  # every block of the cache and every state slot
             for kv in self.worker.cache_engine.gpu_cache:
                 kv.normal_(0.0, 0.5, generator=gen)
-            for layer in self.worker.cache_engine.state:
+            for layer in self.worker.cache_engine.state or ():
                 for t in layer.values():
                     t.normal_(0.0, 0.5, generator=gen)
         for kv in () if own_caches else self.worker.cache_engine.gpu_cache:

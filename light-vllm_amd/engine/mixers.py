@@ -29,6 +29,10 @@ class StepLayout:
     max_query_len: int
     max_seq_len: int
     block_size: int
+    positions: Optional[torch.Tensor] = None    # int64 [rows]
+    # host copies of the sequences' new tokens and of what came before (None: a captured step)
+    query_lens: Optional[List[int]] = None
+    context_lens: Optional[List[int]] = None
 
 
 @dataclass

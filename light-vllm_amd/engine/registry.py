@@ -35,9 +35,11 @@ class ModelEntry:
 MODELS = {
     # Llama / Qwen2-shaped decoders (random weights: engine/config.py ModelConfig)
     "RotaryDecoder": ModelEntry(".config:ModelConfig", ".model:DecoderModel", "..attention.backend:PagedAttnBackend",
-                                ("base", "full")),
+                                ("full",)),
     "Sasilorn": ModelEntry(".hybrid_config:HybridModelConfig", ".hybrid_model:HybridModel",
-                           "..attention.head_backend:HeadAttnBackend", ("base",)),
+                           "..attention.head_backend:HeadAttnBackend", ("heads", "hybrid")),
+    "Lepalorn": ModelEntry(".latent_config:LatentModelConfig", ".latent_model:LatentModel",
+                           "..attention.latent_backend:LatentAttnBackend", ("heads", "latent")),
 }
 
 
