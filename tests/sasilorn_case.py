@@ -1,11 +1,10 @@
 """Small Sasilorn models for the tests: configurations, random weights (every projection scaled so that single keys,
-decays and tokens stand out in the logits), model folders, and schedules played through the framework's trace replay."""
+decays and tokens stand out in the logits)."""
 import functools
-import json
-import os
 
 import torch
 
+from layered_case import error, play, portions, replay, tokens, write_model  # noqa: F401
 from oracle import sasilorn
 
 
@@ -103,27 +102,6 @@ def random_weights(cfg, seed=0, rank=12):
     return out
 
 
-def write_model(folder, cfg, weights):
-    """A model folder; the safetensors file is written here, byte by byte as the format says."""
-    os.makedirs(folder, exist_ok=True)
-    with open(os.path.join(folder, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    header, blobs, at = {}, [], 0
-    for name, t in weights.items():
-        raw = t.bfloat16().contiguous().view(torch.int16).numpy().tobytes()
-        header[name] = {"dtype": "BF16", "shape": list(t.shape), "data_offsets": [at, at + len(raw)]}
-        blobs.append(raw)
-        at += len(raw)
-    head = json.dumps(header).encode()
-    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
-        f.write(len(head).to_bytes(8, "little") + head + b"".join(blobs))
-    return str(folder)
-
-
-def tokens(cfg, n, seed):
-    return torch.randint(0, cfg["vocab"], (n,), generator=torch.Generator().manual_seed(1000 + seed)).tolist()
-
-
 @functools.lru_cache(maxsize=None)
 def case(name, seed=0):
     cfg = CONFIGS[name]
@@ -136,46 +114,3 @@ def expected(name, n, seed):
     cfg, w = case(name)
     t = tokens(cfg, n, seed)
     return t, sasilorn.forward(cfg, w, t)
-
-
-def error(got, want):
-    """RMS over the vocabulary of the difference (means taken off) per row, in units of the expected logits' spread."""
-    d = got.double() - want
-    d = d - d.mean(1, keepdim=True)
-    return d.pow(2).mean(1).sqrt() / want.std()
-
-
-def replay(folder, dtype, max_tokens):
-    from light_vllm_amd.engine.registry import load_model_config
-    from light_vllm_amd.engine.trace import TraceReplay
-    return TraceReplay(load_model_config(folder, dtype), max_tokens)
-
-
-def play(rp, requests, steps):
-    """requests {id: tokens}; steps [[(id, n), ...], ...] -> {id: logits of all its tokens}.  A request ends with its last
-    token."""
-    at, out = {}, {rid: [] for rid in requests}
-    for step in steps:
-        entries = []
-        for rid, n in step:
-            a = at.get(rid, 0)
-            entries.append((rid, requests[rid][a:a + n], list(range(n))))
-            at[rid] = a + n
-        logits = rp.step(entries)
-        row = 0
-        for rid, n in step:
-            out[rid].append(logits[row:row + n])
-            row += n
-            if at[rid] == len(requests[rid]):
-                rp.end(rid)
-    return {rid: torch.cat(o) for rid, o in out.items()}
-
-
-def portions(n, sizes):
-    """n cut into portions of the given sizes in turn."""
-    out, i = [], 0
-    while n > 0:
-        k = min(n, sizes[i % len(sizes)])
-        out.append(k)
-        n, i = n - k, i + 1
-    return out

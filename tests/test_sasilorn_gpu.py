@@ -8,7 +8,9 @@ import sys
 import pytest
 import torch
 
+import layered_case
 import sasilorn_case as sc
+from layered_case import engine, generate
 from oracle import sasilorn
 
 pytestmark = pytest.mark.gpu
@@ -384,35 +386,7 @@ def test_long_decoding(folders):
 
 
 def greedy(cfg, w, prompt, n):
-    t, rows = list(prompt), []
-    for _ in range(n):
-        rows.append(sasilorn.forward(cfg, w, t)[-1])
-        t.append(int(rows[-1].argmax()))
-    return t[len(prompt):]
-
-
-def engine(folder, dtype, graph=True, num_blocks=64, max_seqs=8, chunked=False, budget=512, **kw):
-    from light_vllm_amd.engine.config import CacheConfig, SchedulerConfig
-    from light_vllm_amd.engine.llm_engine import LLMEngine
-    return LLMEngine.from_pretrained(
-        folder, dtype, CacheConfig(num_gpu_blocks=num_blocks, num_cpu_blocks=32),
-        SchedulerConfig(max_num_batched_tokens=budget, max_num_seqs=max_seqs, max_model_len=256,
-                        chunked_prefill_enabled=chunked, **kw), use_hip_graph=graph)
-
-
-def generate(eng, prompts, n, use_async=False):
-    for i, p in enumerate(prompts):
-        eng.add_request(str(i), p, max_tokens=n)
-    done = {}
-    step = eng.async_step if use_async else eng.step
-    for _ in range(2000):
-        for out in step():
-            if out.finished:
-                done[int(out.request_id)] = out.token_ids
-        if not eng.has_unfinished_requests() and eng.num_on_the_fly == 0:
-            break
-    eng.shutdown()
-    return [done[i] for i in range(len(prompts))]
+    return layered_case.greedy(lambda t: sasilorn.forward(cfg, w, t), prompt, n)
 
 
 @pytest.mark.parametrize("name", sorted(sc.CONFIGS))
