@@ -106,6 +106,10 @@ def parse():
                     help="instead of the headline workload: prefill and decode throughput of the hybrid decoder beside the "
                          "rotary decoder at equal sizes (tools/bench_hybrid.py)")
     ap.add_argument("--hybrid-only", default=None, help="with --hybrid: the cases whose name starts with this")
+    ap.add_argument("--latent", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the latent decoder beside the "
+                         "rotary decoder at equal sizes (tools/bench_latent.py)")
+    ap.add_argument("--latent-only", default=None, help="with --latent: the cases whose name starts with this")
     ap.add_argument("--tiny", action="store_true", help="tiny model (plumbing check)")
     ap.add_argument("--replica-backend", default=None, choices=["nccl", "gloo"],
                     help="process-group backend of the barrier / clock between replicas (default: nccl = RCCL)")
@@ -844,6 +848,11 @@ def main():
         sys.path.insert(0, os.path.join(ROOT, "tools"))
         import bench_hybrid
         print(json.dumps({"hybrid": bench_hybrid.run("cuda:0", a.hybrid_only)}), flush=True)
+        return
+    if a.latent:
+        sys.path.insert(0, os.path.join(ROOT, "tools"))
+        import bench_latent
+        print(json.dumps({"latent": bench_latent.run("cuda:0", a.latent_only)}), flush=True)
         return
     if a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(spawn_replicas(a))

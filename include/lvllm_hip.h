@@ -637,24 +637,26 @@ int lvllm_norm_add_mix(float* x_out, float* v_out, void* h, const float* x_in, c
                        int num_partials, const int32_t* slots, const float* slot_weights, int num_slots, int total_slots,
                        const float* gain, float eps, const float* streams, int64_t stream_stride, int num_streams,
                        const float* weights, const float* out_gain, float out_eps, int rows, int width, int dtype, void* stream);
-/* cache rows [RMS norm(kv[:kv_rank]) | rotated kv[kv_rank:]] at slot_mapping (slots < 0: none); inv_freq: rot_dims / 2 */
+/* cache rows [RMS norm(kv[:kv_rank]) | rotated kv[kv_rank:]] at slot_mapping (slots < 0: none).  turns: rot_dims / 2 numbers,
+ * the full turns a pair makes per position */
 int lvllm_latent_cache(void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad, int rpad,
                        const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
-                       const int64_t* positions, const double* inv_freq, int rot_dims, const int64_t* slot_mapping, int rows,
+                       const int64_t* positions, const double* turns, int rot_dims, const int64_t* slot_mapping, int rows,
                        int dtype, void* stream);
-/* queries into latent space: out [rows, heads, cpad + rpad] = [uk_t q | rotated | 0]; uk_t [heads, cpad, dpad], zero-padded */
+/* queries into latent space: out [rows, heads, cpad + rpad] = [uk_t q | rotated | 0]; uk_t [heads, cpad, dpad], zero-padded.
+ * kv not null: the same launch writes the rows' cache entries, as lvllm_latent_cache does */
 int lvllm_latent_query(void* out, const void* q, int64_t q_stride, const void* uk_t, int heads, int dim, int dpad, int cpad,
-                       int rpad, int rot_dim, int rot_dims, const int64_t* positions, const double* inv_freq,
-                       const int32_t* query_start_loc, int num_seqs, int absorbed_max, int rows, int dtype, void* stream);
-/* values out of it: out[row, h * vdim + d] = (uv o_lat)[d] * sigmoid(gate[row, h]); uv [heads, vpad, cpad], zero-padded */
-int lvllm_latent_value(void* out, int64_t out_stride, const void* o_lat, const void* uv, const void* gate, int64_t gate_stride,
-                       int heads, int vdim, int vpad, int cpad, const int32_t* query_start_loc, int num_seqs, int absorbed_max,
-                       int rows, int dtype, void* stream);
-/* out [rows, heads, cpad]: attention on the cached rows, for sequences of at most absorbed_max query tokens */
+                       int rpad, int rot_dim, int rot_dims, const int64_t* positions, const double* turns,
+                       const int32_t* query_start_loc, int num_seqs, int absorbed_max, void* cache, int64_t block_stride,
+                       int64_t num_blocks, int block_size, const void* kv, int64_t kv_stride, int kv_rank, const float* weight,
+                       float eps, const int64_t* slot_mapping, int rows, int dtype, void* stream);
+/* attention on the cached rows, for sequences of at most absorbed_max query tokens, and its values out of latent space:
+ * out[row, h * vdim + d] = (uv_h sum)[d] * sigmoid(gate[row, h]); uv [heads, vpad, cpad], zero-padded; gate null: none */
 int64_t lvllm_latent_attention_workspace_bytes(int rows, int num_seqs, int heads, int cpad, int rpad, int block_size,
                                                int window, int absorbed_max, int max_query_len, int max_seq_len, int dtype);
-int lvllm_latent_attention(void* out, const void* q, const void* cache, int64_t block_stride, int64_t num_blocks,
-                           int block_size, int cpad, int rpad, const int32_t* block_tables, int max_blocks,
+int lvllm_latent_attention(void* out, int64_t out_stride, const void* q, const void* cache, int64_t block_stride,
+                           int64_t num_blocks, int block_size, int cpad, int rpad, const void* uv, int vdim, int vpad,
+                           const void* gate, int64_t gate_stride, const int32_t* block_tables, int max_blocks,
                            const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows, int heads,
                            float scale, int window, int absorbed_max, int max_query_len, int max_seq_len, void* workspace,
                            int64_t workspace_bytes, int dtype, void* stream);
@@ -665,19 +667,20 @@ int lvllm_latent_gather(void* out, const void* cache, int64_t block_stride, int6
 int lvllm_latent_expand(void* key_pages, void* value_pages, const void* kv, int64_t kv_stride, const void* rows, int row_elems,
                         int cpad, int n, int heads, int dim, int rot_dim, int vdim, int kpad, int vpad, int dtype, void* stream);
 int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_stride, int heads, int dim, int rot_dim, int kpad,
-                              const int64_t* positions, const double* inv_freq, int rot_dims, int rows, int dtype, void* stream);
+                              const int64_t* positions, const double* turns, int rot_dims, int rows, int dtype, void* stream);
 /* the `top` experts of every row and their softmax weights; with `shared` a last assignment, expert number `experts`, weighted
- * sigmoid of the last row of w */
+ * sigmoid of the last row of w.  `packed`: w as lvllm_pack_weight leaves it, rows padded to a multiple of 16 */
 int lvllm_moe_route(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
-                    int top, int rows, int width, int dtype, void* stream);
-/* assignments grouped by expert: offsets [experts + 1], token and slot [total], tiles [max_tiles, 2] of lvllm_moe_tile slots */
+                    int top, int rows, int width, int packed, int dtype, void* stream);
+/* assignments grouped by expert: offsets [experts + 1], token and slot [total], tiles [max_tiles + 1, 2] of lvllm_moe_tile slots */
 int lvllm_moe_tile(int packed);
 int lvllm_moe_group(int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles, const int32_t* ids, int total, int per_row,
                     int experts, int packed, int max_tiles, void* stream);
 /* the experts' products: up (with the activation) [rows, width] -> [slots, ff_max], down [slots, ff_max] -> [slots, width] */
 int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff, const float* limit,
                       const int32_t* offsets, const int32_t* token, const int32_t* tiles, int experts, int slots, int rows,
-                      int width, int ff_max, int max_tiles, int up, int packed, int dtype, void* stream);
+                      int width, int ff_max, int ff_first, int ff_last, int max_tiles, int up, int packed, int dtype,
+                      void* stream);
 
 #ifdef __cplusplus
 }

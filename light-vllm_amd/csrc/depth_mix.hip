@@ -41,70 +41,84 @@ __device__ __forceinline__ void store_items(typename T::store_t* p, const float 
   else p[0] = T::from_float(v[0]);
 }
 
-// A workgroup per row; a thread keeps its ITEMS groups of VEC columns in registers.
+// A workgroup per row; a thread keeps its ITEMS groups of VEC columns in registers.  Everything that does not depend on the
+// norm -- the sublayer's output, the stream, the earlier streams -- is read before the reduction, several rows at a time.
 template <typename T, int VEC, int ITEMS>
-__global__ __launch_bounds__(256) void norm_add_mix_kernel(const DepthMixParams p) {
+__global__ __launch_bounds__(1024) void norm_add_mix_kernel(const DepthMixParams p) {
   using S = typename T::store_t;
+  constexpr int B = ITEMS <= 2 ? 8 : 4;  // rows in flight
   __shared__ float red[16];
   const int row = blockIdx.x;
   const int64_t base = (int64_t)row * p.width;
-  float v[ITEMS][VEC];
-  float ss = 0.f;
+  auto column = [&](int it) { return (it * (int)blockDim.x + (int)threadIdx.x) * VEC; };
+  float v[ITEMS][VEC], x[ITEMS][VEC], mix[ITEMS][VEC];
 #pragma unroll
   for (int it = 0; it < ITEMS; ++it) {
-    const int c = (it * 256 + threadIdx.x) * VEC;
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) v[it][j] = 0.f;
-    if (c >= p.width) continue;
-    if (p.slots != nullptr) {
-      for (int i = 0; i < p.num_slots; ++i) {
-        const int s = min(max(p.slots[(int64_t)row * p.num_slots + i], 0), p.total_slots - 1);
-        const float w = p.slot_weights[(int64_t)row * p.num_slots + i];
-        float t[VEC];
-        load_items<T, VEC>((const S*)p.y + (int64_t)s * p.width + c, t);
+    for (int j = 0; j < VEC; ++j) v[it][j] = x[it][j] = mix[it][j] = 0.f;
+    if (column(it) < p.width) load_f32<VEC>(p.x_in + base + column(it), x[it]);
+  }
+  auto add_rows = [&](float (&acc)[ITEMS][VEC], int n, auto weight_of, auto load) __attribute__((always_inline)) {
+    for (int i0 = 0; i0 < n; i0 += B) {
+      float w[B];
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) v[it][j] = fmaf(w, t[j], v[it][j]);
+      for (int i = 0; i < B; ++i) w[i] = i0 + i < n ? weight_of(i0 + i) : 0.f;
+#pragma unroll
+      for (int it = 0; it < ITEMS; ++it) {
+        if (column(it) >= p.width) continue;
+        float t[B][VEC];
+#pragma unroll
+        for (int i = 0; i < B; ++i)
+          if (i0 + i < n) load(i0 + i, column(it), t[i]);
+#pragma unroll
+        for (int i = 0; i < B; ++i)
+          if (i0 + i < n) {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) acc[it][j] = fmaf(w[i], t[i][j], acc[it][j]);
+          }
       }
-    } else if (p.partials != nullptr) {
-      for (int s = 0; s < p.num_partials; ++s) {
-        float t[VEC];
-        load_f32<VEC>(p.partials + (int64_t)s * p.rows * p.width + base + c, t);
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) v[it][j] += t[j];
-      }
-    } else {
-      load_items<T, VEC>((const S*)p.y + base + c, v[it]);
     }
+  };
+  if (p.slots != nullptr) {
+    const int32_t* slots = p.slots + (int64_t)row * p.num_slots;
+    const float* weights = p.slot_weights + (int64_t)row * p.num_slots;
+    add_rows(v, p.num_slots, [&](int i) { return weights[i]; }, [&](int i, int c, float (&t)[VEC]) {
+      load_items<T, VEC>((const S*)p.y + (int64_t)min(max(slots[i], 0), p.total_slots - 1) * p.width + c, t);
+    });
+  } else if (p.partials != nullptr) {
+    add_rows(v, p.num_partials, [](int) { return 1.f; }, [&](int i, int c, float (&t)[VEC]) {
+      load_f32<VEC>(p.partials + (int64_t)i * p.rows * p.width + base + c, t);
+    });
+  } else {
+#pragma unroll
+    for (int it = 0; it < ITEMS; ++it)
+      if (column(it) < p.width) load_items<T, VEC>((const S*)p.y + base + column(it), v[it]);
+  }
+  if (p.weights != nullptr)
+    add_rows(mix, p.num_streams, [&](int i) { return p.weights[i]; }, [&](int i, int c, float (&t)[VEC]) {
+      load_f32<VEC>(p.streams + i * p.stream_stride + base + c, t);
+    });
+  float ss = 0.f;
+#pragma unroll
+  for (int it = 0; it < ITEMS; ++it)
 #pragma unroll
     for (int j = 0; j < VEC; ++j) ss = fmaf(v[it][j], v[it][j], ss);
-  }
   ss = block_sum(ss, red);
   const float f = p.gain[0] / sqrtf(ss / (float)p.width + p.eps);
   const float wv = p.weights != nullptr ? p.weights[p.num_streams] : 1.f;
   float so = 0.f;
 #pragma unroll
   for (int it = 0; it < ITEMS; ++it) {
-    const int c = (it * 256 + threadIdx.x) * VEC;
-    if (c >= p.width) continue;
-    float x[VEC];
-    load_f32<VEC>(p.x_in + base + c, x);
+    if (column(it) >= p.width) continue;
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) x[j] = fmaf(v[it][j], f, x[j]);
-    if (p.v_out != nullptr) store_items<F32, VEC>(p.v_out + base + c, x);
+    for (int j = 0; j < VEC; ++j) x[it][j] = fmaf(v[it][j], f, x[it][j]);
+    if (p.v_out != nullptr) store_items<F32, VEC>(p.v_out + base + column(it), x[it]);
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) v[it][j] = x[j] * wv;
-    if (p.weights != nullptr) {
-      for (int s = 0; s < p.num_streams; ++s) {
-        float t[VEC];
-        load_f32<VEC>(p.streams + s * p.stream_stride + base + c, t);
-        const float w = p.weights[s];
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) v[it][j] = fmaf(w, t[j], v[it][j]);
-      }
+    for (int j = 0; j < VEC; ++j) {
+      v[it][j] = fmaf(wv, x[it][j], mix[it][j]);
+      so = fmaf(v[it][j], v[it][j], so);
     }
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) so = fmaf(v[it][j], v[it][j], so);
-    if (p.x_out != nullptr) store_items<F32, VEC>(p.x_out + base + c, v[it]);
+    if (p.x_out != nullptr) store_items<F32, VEC>(p.x_out + base + column(it), v[it]);
   }
   float fo = 1.f;
   if (p.out_gain != nullptr) {
@@ -113,26 +127,29 @@ __global__ __launch_bounds__(256) void norm_add_mix_kernel(const DepthMixParams 
   }
 #pragma unroll
   for (int it = 0; it < ITEMS; ++it) {
-    const int c = (it * 256 + threadIdx.x) * VEC;
-    if (c >= p.width) continue;
+    if (column(it) >= p.width) continue;
 #pragma unroll
     for (int j = 0; j < VEC; ++j) v[it][j] *= fo;
-    store_items<T, VEC>((S*)p.h + base + c, v[it]);
+    store_items<T, VEC>((S*)p.h + base + column(it), v[it]);
   }
 }
 
 // x = table[id] * scale, h = T(x)
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void embed_scale_kernel(float* __restrict__ x, typename T::store_t* __restrict__ h,
                                                           const typename T::store_t* __restrict__ table,
                                                           const int64_t* __restrict__ ids, const float scale, const int vocab,
                                                           const int width) {
   const int row = blockIdx.x;
   const int64_t id = ids[row] < 0 ? 0 : ids[row] >= vocab ? vocab - 1 : ids[row];
-  for (int c = threadIdx.x; c < width; c += 256) {
-    const float v = T::to_float(table[id * width + c]) * scale;
-    x[(int64_t)row * width + c] = v;
-    h[(int64_t)row * width + c] = T::from_float(v);
+  const int64_t base = (int64_t)row * width;
+  for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
+    float v[VEC];
+    load_items<T, VEC>(table + id * width + c, v);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] *= scale;
+    store_items<F32, VEC>(x + base + c, v);
+    store_items<T, VEC>(h + base + c, v);
   }
 }
 
@@ -146,8 +163,12 @@ extern "C" int lvllm_embed_scale(float* x, void* h, const void* table, const int
   LV_CHECK(vocab > 0 && width > 0, "an empty table");
   LV_DISPATCH_F32_BF16(dtype, {
     using S = typename scalar_t::store_t;
-    hipLaunchKernelGGL((embed_scale_kernel<scalar_t>), dim3(rows), dim3(256), 0, (hipStream_t)stream, x, (S*)h,
-                       (const S*)table, ids, scale, vocab, width);
+    if (width % 4 == 0)
+      hipLaunchKernelGGL((embed_scale_kernel<scalar_t, 4>), dim3(rows), dim3(256), 0, (hipStream_t)stream, x, (S*)h,
+                         (const S*)table, ids, scale, vocab, width);
+    else
+      hipLaunchKernelGGL((embed_scale_kernel<scalar_t, 1>), dim3(rows), dim3(256), 0, (hipStream_t)stream, x, (S*)h,
+                         (const S*)table, ids, scale, vocab, width);
   });
   LV_LAUNCH_CHECK();
   return 0;
@@ -167,24 +188,25 @@ extern "C" int lvllm_norm_add_mix(float* x_out, float* v_out, void* h, const flo
   p.eps = eps; p.streams = streams; p.stream_stride = stream_stride; p.num_streams = num_streams; p.weights = weights;
   p.out_gain = out_gain; p.out_eps = out_eps; p.rows = rows; p.width = width;
   hipStream_t s = (hipStream_t)stream;
+  // few rows: as many threads as a row has groups of columns; many: 256, several groups each
+  const int vec = width % 4 == 0 ? 4 : 1, groups = width / vec;
+  int threads = 256;
+  while (threads < 1024 && (rows <= 256 ? threads < groups : threads * 4 < groups)) threads *= 2;
+  const int items = (groups + threads - 1) / threads;
 #define LV_GO(VEC_, ITEMS_)                                                                                        \
-  LV_DISPATCH_F32_BF16(dtype, {                                                                                       \
-    hipLaunchKernelGGL((norm_add_mix_kernel<scalar_t, VEC_, ITEMS_>), dim3(rows), dim3(256), 0, s, p);             \
+  LV_DISPATCH_F32_BF16(dtype, {                                                                                    \
+    hipLaunchKernelGGL((norm_add_mix_kernel<scalar_t, VEC_, ITEMS_>), dim3(rows), dim3(threads), 0, s, p);         \
   })
-  if (width % 4 == 0) {
-    const int items = (width + 1023) / 1024;
+  if (vec == 4) {
     if (items <= 1) { LV_GO(4, 1); }
     else if (items <= 2) { LV_GO(4, 2); }
-    else if (items <= 4) { LV_GO(4, 4); }
-    else if (items <= 8) { LV_GO(4, 8); }
     else {
-      LV_CHECK(items <= 16, "rows of at most 16384");
-      LV_GO(4, 16);
+      LV_CHECK(items <= 4, "rows of at most 16384");
+      LV_GO(4, 4);
     }
   } else {
     LV_CHECK(width <= 4096, "rows that are no multiple of 4: at most 4096");
-    if (width <= 1024) { LV_GO(1, 4); }
-    else { LV_GO(1, 16); }
+    LV_GO(1, 4);
   }
 #undef LV_GO
   LV_LAUNCH_CHECK();

@@ -11,7 +11,6 @@
 //
 //   cache  [num_blocks, block_size, cpad + rpad]: c, zeros to cpad, the rotated part, zeros to the row's end
 //   q'     [rows, heads, cpad + rpad], the same row layout
-//   o_lat  [rows, heads, cpad]: the weighted sums of the latents
 // Scores, softmax and accumulation are fp32.
 #pragma once
 #include "common.h"
@@ -19,13 +18,15 @@
 namespace lvllm {
 
 struct LatentAttnParams {
-  void* out;
+  void* out;               // row r, head h at r * out_stride + h * vdim
   const void *q, *cache;
+  const void *uv, *gate;   // [heads, vpad, cpad], zero-padded; gate [rows, heads] (gate_stride apart) or null
   const int32_t *block_tables, *seq_lens, *query_start_loc;
   float *part_o, *part_ml;  // shares: [rows, heads, nsplit, cpad] and [rows, heads, nsplit, 2]
   int num_seqs, rows, heads, cpad, rpad, max_blocks, block_size, max_block, nsplit, window, absorbed_max, max_query_len;
+  int vdim, vpad;
   float scale;
-  int64_t block_stride;
+  int64_t block_stride, out_stride, gate_stride;
 };
 
 bool latent_takes_mfma(int cpad, int rpad, int block_size, int dtype);
@@ -34,11 +35,11 @@ int launch_latent_mfma(const LatentAttnParams& p, hipStream_t s);
 // The first key position `pos` sees.
 __device__ __forceinline__ int first_key(int pos, int window) { return window > 0 ? max(0, pos - window + 1) : 0; }
 
-// Rotation of pairs (2i, 2i + 1): the angle is taken in double, so that far positions keep the fp32 sine's own accuracy.
-__device__ __forceinline__ void rotation_of(int64_t position, double inv_freq, float& c, float& s) {
-  const double a = (double)position * inv_freq;
-  const double r = a - rint(a * 0.15915494309189533577) * 6.28318530717958647693;
-  sincosf((float)r, &s, &c);
+// Rotation of pairs (2i, 2i + 1) by position * turns full turns: the product is taken in double, so that far positions keep
+// the fp32 sine's own accuracy.
+__device__ __forceinline__ void rotation_of(int64_t position, double turns, float& c, float& s) {
+  const double t = (double)position * turns;
+  sincospif((float)(2.0 * (t - rint(t))), &s, &c);
 }
 
 }  // namespace lvllm

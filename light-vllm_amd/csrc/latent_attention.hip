@@ -1,5 +1,5 @@
-// Latent attention: the cache write, queries into and values out of latent space, the gather and the expansion for long
-// portions, and the plain attention body (see latent_attention.h for the layouts).
+// Latent attention: the cache write, queries into latent space, the gather and the expansion for long portions, and the plain
+// attention body with its values' way out of latent space (see latent_attention.h for the layouts).
 #include <float.h>
 
 #include "latent_attention.h"
@@ -9,55 +9,79 @@ namespace lvllm {
 typedef __bf16 l_bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float l_f32x4_t __attribute__((ext_vector_type(4)));
 
-// RMS-normed latent and rotated key part of every row -> its cache slot.  A wave per row.
+struct LatentCacheParams {
+  void* cache;
+  const void* kv;          // null: nothing to write
+  const float* weight;
+  const int64_t *positions, *slot_mapping;
+  const double* turns;
+  int64_t block_stride, num_slots, kv_stride;
+  int block_size, cpad, rpad, kv_rank, rot_dim, rot_dims, rows;
+  float eps;
+};
+
+// RMS-normed latent and rotated key part of a row -> its cache slot; one wave, 16 bytes a lane where the sizes allow it
 template <typename T>
-__global__ __launch_bounds__(256) void latent_cache_kernel(typename T::store_t* __restrict__ cache, const int64_t block_stride,
-                                                           const int64_t num_slots, const int block_size, const int cpad,
-                                                           const int rpad, const typename T::store_t* __restrict__ kv,
-                                                           const int64_t kv_stride, const int kv_rank, const int rot_dim,
-                                                           const float* __restrict__ weight, const float eps,
-                                                           const int64_t* __restrict__ positions,
-                                                           const double* __restrict__ inv_freq, const int rot_dims,
-                                                           const int64_t* __restrict__ slot_mapping, const int rows) {
+__device__ __forceinline__ void write_latent_row(const LatentCacheParams& p, int row) {
   using S = typename T::store_t;
-  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (row >= rows) return;
-  const int64_t slot = slot_mapping[row];
-  if (slot < 0 || slot >= num_slots) return;
-  const S* z = kv + row * kv_stride;
-  S* out = cache + (slot / block_size) * block_stride + (slot % block_size) * (int64_t)(cpad + rpad);
+  constexpr int X = 16 / sizeof(S);
+  const int lane = threadIdx.x & 63;
+  const int64_t slot = p.slot_mapping[row];
+  if (slot < 0 || slot >= p.num_slots) return;
+  const S* z = (const S*)p.kv + row * p.kv_stride;
+  S* out = (S*)p.cache + (slot / p.block_size) * p.block_stride + (slot % p.block_size) * (int64_t)(p.cpad + p.rpad);
+  const int64_t pos = p.positions[row];
+  const bool vec = p.kv_rank % X == 0 && p.kv_rank <= 64 * X && ((uintptr_t)z & 15) == 0;
   float ss = 0.f;
-  for (int i = lane; i < kv_rank; i += 64) {
-    const float v = T::to_float(z[i]);
-    ss = fmaf(v, v, ss);
-  }
-  const float f = 1.f / sqrtf(wave_sum(ss) / (float)kv_rank + eps);
-  for (int i = lane; i < cpad; i += 64) out[i] = T::from_float(i < kv_rank ? T::to_float(z[i]) * f * weight[i] : 0.f);
-  const int64_t pos = positions[row];
-  for (int i = lane; i < rpad; i += 64) {
-    float v = 0.f;
-    if (i < rot_dims) {
-      float c, s;
-      rotation_of(pos, inv_freq[i >> 1], c, s);
-      const float a = T::to_float(z[kv_rank + i]), b = T::to_float(z[kv_rank + (i ^ 1)]);
-      v = i & 1 ? a * c + b * s : a * c - b * s;
-    } else if (i < rot_dim) {
-      v = T::to_float(z[kv_rank + i]);
+  if (vec) {
+    const int i = lane * X;
+    Vec16<T> raw;
+    float v[X];
+#pragma unroll
+    for (int j = 0; j < X; ++j) v[j] = 0.f;
+    if (i < p.kv_rank) {
+      raw = *reinterpret_cast<const Vec16<T>*>(z + i);
+#pragma unroll
+      for (int j = 0; j < X; ++j) {
+        v[j] = T::to_float(raw.v[j]);
+        ss = fmaf(v[j], v[j], ss);
+      }
     }
-    out[cpad + i] = T::from_float(v);
+    const float f = 1.f / sqrtf(wave_sum(ss) / (float)p.kv_rank + p.eps);
+    if (i < p.cpad) {
+#pragma unroll
+      for (int j = 0; j < X; ++j) raw.v[j] = T::from_float(i < p.kv_rank ? v[j] * f * p.weight[i + j] : 0.f);
+      *reinterpret_cast<Vec16<T>*>(out + i) = raw;
+    }
+    for (int d = 64 * X + lane; d < p.cpad; d += 64) out[d] = T::from_float(0.f);
+  } else {
+    for (int i = lane; i < p.kv_rank; i += 64) {
+      const float v = T::to_float(z[i]);
+      ss = fmaf(v, v, ss);
+    }
+    const float f = 1.f / sqrtf(wave_sum(ss) / (float)p.kv_rank + p.eps);
+    for (int i = lane; i < p.cpad; i += 64) out[i] = T::from_float(i < p.kv_rank ? T::to_float(z[i]) * f * p.weight[i] : 0.f);
+  }
+  z += p.kv_rank;
+  out += p.cpad;
+  for (int i = lane * 2; i < p.rpad; i += 128) {
+    float u = i < p.rot_dim ? T::to_float(z[i]) : 0.f, v = i + 1 < p.rot_dim ? T::to_float(z[i + 1]) : 0.f;
+    if (i < p.rot_dims) {
+      float c, s;
+      rotation_of(pos, p.turns[i >> 1], c, s);
+      const float t = u * c - v * s;
+      v = v * c + u * s;
+      u = t;
+    }
+    out[i] = T::from_float(u);
+    out[i + 1] = T::from_float(v);
   }
 }
 
-// entry i of a query head's rotated part
 template <typename T>
-__device__ __forceinline__ float rotated_entry(const typename T::store_t* z, int i, int rot_dim, int rot_dims, int64_t pos,
-                                               const double* inv_freq) {
-  if (i >= rot_dim) return 0.f;
-  if (i >= rot_dims) return T::to_float(z[i]);
-  float c, s;
-  rotation_of(pos, inv_freq[i >> 1], c, s);
-  const float a = T::to_float(z[i]), b = T::to_float(z[i ^ 1]);
-  return i & 1 ? a * c + b * s : a * c - b * s;
+__global__ __launch_bounds__(256) void latent_cache_kernel(const LatentCacheParams p) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row < p.rows) write_latent_row<T>(p, row);
 }
 
 // Rows of a 16-row tile that all belong to one long portion need nothing in latent space.
@@ -76,7 +100,8 @@ struct HeadProjectParams {
   // the tail of a query row: its rotated part at entry n .. n + tail - 1 of y, from x's entries k .. k + rot_dim - 1
   int tail, rot_dim, rot_dims;
   const int64_t* positions;
-  const double* inv_freq;
+  const double* turns;
+  LatentCacheParams cache;  // the rows' own latents, written by the launch that takes their queries to latent space
 };
 
 template <typename T>
@@ -88,13 +113,36 @@ __device__ __forceinline__ float project_gate(const HeadProjectParams& p, int ro
 template <typename T>
 __device__ __forceinline__ void project_tail(const HeadProjectParams& p, int row0, int head) {
   using S = typename T::store_t;
-  for (int i = threadIdx.x; i < 16 * p.tail; i += 256) {
-    const int row = row0 + i / p.tail, e = i % p.tail;
+  const int pairs = p.tail >> 1;
+  for (int i = threadIdx.x; i < 16 * pairs; i += 256) {
+    const int row = row0 + i / pairs, e = 2 * (i % pairs);
     if (row >= p.rows) break;
     const S* z = (const S*)p.x + row * p.x_stride + (int64_t)head * p.x_head + p.k;
-    ((S*)p.y)[row * p.y_stride + (int64_t)head * p.y_head + p.n + e] =
-        T::from_float(rotated_entry<T>(z, e, p.rot_dim, p.rot_dims, p.positions[row], p.inv_freq));
+    float u = e < p.rot_dim ? T::to_float(z[e]) : 0.f, v = e + 1 < p.rot_dim ? T::to_float(z[e + 1]) : 0.f;
+    if (e < p.rot_dims) {
+      float c, s;
+      rotation_of(p.positions[row], p.turns[e >> 1], c, s);
+      const float t = u * c - v * s;
+      v = v * c + u * s;
+      u = t;
+    }
+    S* y = (S*)p.y + row * p.y_stride + (int64_t)head * p.y_head + p.n + e;
+    y[0] = T::from_float(u);
+    y[1] = T::from_float(v);
   }
+}
+
+// What a workgroup does besides products; true: nothing else is left to do.
+template <typename T>
+__device__ __forceinline__ bool beside_products(const HeadProjectParams& p, int row0, int head) {
+  const bool last = p.tail > 0 && blockIdx.x == gridDim.x - 1;
+  if (last && head == 0 && p.cache.kv != nullptr)
+    for (int i = threadIdx.x >> 6; i < 16 && row0 + i < p.rows; i += 4) write_latent_row<T>(p.cache, row0 + i);
+  if (p.query_start_loc != nullptr &&
+      tile_is_expanded(p.query_start_loc, p.num_seqs, row0, min(row0 + 15, p.rows - 1), p.absorbed_max))
+    return true;
+  if (last) project_tail<T>(p, row0, head);
+  return last;
 }
 
 // y[r, h, :] = W_h x[r, h, :] (* sigmoid(gate[r, h])).  grid (n tiles (+ 1 for the tail), heads, 16-row tiles)
@@ -102,10 +150,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void head_project_simple_kernel(const HeadProjectParams p) {
   using S = typename T::store_t;
   const int head = blockIdx.y, row0 = blockIdx.z * 16;
-  if (p.query_start_loc != nullptr &&
-      tile_is_expanded(p.query_start_loc, p.num_seqs, row0, min(row0 + 15, p.rows - 1), p.absorbed_max))
-    return;
-  if (p.tail > 0 && blockIdx.x == gridDim.x - 1) return project_tail<T>(p, row0, head);
+  if (beside_products<T>(p, row0, head)) return;
   const int row = row0 + (threadIdx.x >> 4), n = blockIdx.x * 16 + (threadIdx.x & 15);
   if (row >= p.rows || n >= p.n) return;
   const S* x = (const S*)p.x + row * p.x_stride + (int64_t)head * p.x_head;
@@ -118,10 +163,7 @@ __global__ __launch_bounds__(256) void head_project_simple_kernel(const HeadProj
 // The same on 16x16x32 MFMAs: W rows are the A operand, the 16 rows' x the B operand; a wave per 16 outputs.
 __global__ __launch_bounds__(256) void head_project_mfma_kernel(const HeadProjectParams p) {
   const int head = blockIdx.y, row0 = blockIdx.z * 16;
-  if (p.query_start_loc != nullptr &&
-      tile_is_expanded(p.query_start_loc, p.num_seqs, row0, min(row0 + 15, p.rows - 1), p.absorbed_max))
-    return;
-  if (p.tail > 0 && blockIdx.x == gridDim.x - 1) return project_tail<BF16>(p, row0, head);
+  if (beside_products<BF16>(p, row0, head)) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
   const int n0 = (blockIdx.x * 4 + wave) * 16;
   if (n0 >= p.npad) return;
@@ -129,13 +171,20 @@ __global__ __launch_bounds__(256) void head_project_mfma_kernel(const HeadProjec
   const uint16_t* x = (const uint16_t*)p.x + row * p.x_stride + (int64_t)head * p.x_head + 8 * g;
   const uint16_t* w = (const uint16_t*)p.w + ((int64_t)head * p.npad + n0 + c) * p.kpad + 8 * g;
   l_f32x4_t acc{0.f, 0.f, 0.f, 0.f};
-  const uint4 zero{0, 0, 0, 0};
-#pragma unroll 4
-  for (int k = 0; k < p.kpad; k += 32) {
-    const uint4 a = *reinterpret_cast<const uint4*>(w + k);
-    const uint4 b = k + 8 * g < p.k ? *reinterpret_cast<const uint4*>(x + k) : zero;
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(l_bf16x8_t, a), __builtin_bit_cast(l_bf16x8_t, b), acc,
-                                                  0, 0, 0);
+  constexpr int B = 4;  // k-steps in flight
+  for (int k0 = 0; k0 < p.kpad; k0 += 32 * B) {
+    uint4 a[B], b[B];
+#pragma unroll
+    for (int j = 0; j < B; ++j) {
+      const int k = k0 + 32 * j;
+      a[j] = b[j] = uint4{0, 0, 0, 0};
+      if (k < p.kpad) a[j] = *reinterpret_cast<const uint4*>(w + k);
+      if (k + 8 * g < p.k) b[j] = *reinterpret_cast<const uint4*>(x + k);
+    }
+#pragma unroll
+    for (int j = 0; j < B; ++j)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(l_bf16x8_t, a[j]), __builtin_bit_cast(l_bf16x8_t, b[j]),
+                                                    acc, 0, 0, 0);
   }
   if (row0 + c >= p.rows) return;
   const float f = project_gate<BF16>(p, row, head);
@@ -163,8 +212,9 @@ static int head_project(const HeadProjectParams& p, int dtype, hipStream_t s) {
 }
 
 // The plain body, for 32-bit elements and sizes without an MFMA instantiation: a workgroup per (row, head), 256 keys a round.
+// Its result, [rows, heads, cpad], is the weighted sum in latent space.
 template <typename T>
-__global__ __launch_bounds__(256) void latent_attention_simple_kernel(const LatentAttnParams p) {
+__global__ __launch_bounds__(256) void latent_attention_simple_kernel(const LatentAttnParams p, void* o_lat) {
   using S = typename T::store_t;
   constexpr int x = 16 / sizeof(S);
   extern __shared__ float sm[];
@@ -176,13 +226,13 @@ __global__ __launch_bounds__(256) void latent_attention_simple_kernel(const Late
   const int row = blockIdx.x, head = blockIdx.y;
   const int seq = find_seq(p.query_start_loc, p.num_seqs, row);
   if (seq >= p.num_seqs) {  // padding rows: whatever is read afterwards is finite
-    for (int d = threadIdx.x; d < p.cpad; d += 256) ((S*)p.out)[((int64_t)row * p.heads + head) * p.cpad + d] = T::from_float(0.f);
+    for (int d = threadIdx.x; d < p.cpad; d += 256) ((S*)o_lat)[((int64_t)row * p.heads + head) * p.cpad + d] = T::from_float(0.f);
     return;
   }
   const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
   if (qlen > p.absorbed_max) return;
   const int pos = p.seq_lens[seq] - qlen + (row - qbeg);
-  S* out = (S*)p.out + ((int64_t)row * p.heads + head) * p.cpad;
+  S* out = (S*)o_lat + ((int64_t)row * p.heads + head) * p.cpad;
   if (pos < 0) {  // a padding row of a captured step
     for (int d = threadIdx.x; d < p.cpad; d += 256) out[d] = T::from_float(0.f);
     return;
@@ -302,37 +352,53 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(uint16_t* __restrict
   }
 }
 
-// Queries of long portions as head_attention takes them: [rows, heads, kpad] = [q | rotated | 0].
-template <typename T>
+// Queries of long portions as head_attention takes them: [rows, heads, kpad] = [q | rotated | 0].  A thread takes E entries.
+template <typename T, int E>
 __global__ __launch_bounds__(256) void latent_rotate_query_kernel(typename T::store_t* __restrict__ out,
                                                                   const typename T::store_t* __restrict__ q,
                                                                   const int64_t q_stride, const int heads, const int dim,
                                                                   const int rot_dim, const int kpad,
                                                                   const int64_t* __restrict__ positions,
-                                                                  const double* __restrict__ inv_freq, const int rot_dims) {
+                                                                  const double* __restrict__ turns, const int rot_dims) {
+  using S = typename T::store_t;
+  struct alignas(E * sizeof(S)) Piece { S v[E]; };
   extern __shared__ float cs[];  // [rot_dims / 2][2]
   const int row = blockIdx.x;
-  for (int i = threadIdx.x; i < rot_dims / 2; i += 256) rotation_of(positions[row], inv_freq[i], cs[2 * i], cs[2 * i + 1]);
+  for (int i = threadIdx.x; i < rot_dims / 2; i += 256) rotation_of(positions[row], turns[i], cs[2 * i], cs[2 * i + 1]);
   __syncthreads();
-  const typename T::store_t* x = q + row * q_stride;
-  typename T::store_t* y = out + (int64_t)row * heads * kpad;
-  const int qd = dim + rot_dim;
-  for (int i = threadIdx.x; i < heads * kpad / 2; i += 256) {
-    const int h = 2 * i / kpad, d = 2 * i - h * kpad;
-#pragma unroll
-    for (int e = 0; e < 2; ++e) {
-      const int dd = d + e, r = dd - dim;
-      float v = 0.f;
-      if (dd < qd) {
-        const typename T::store_t* xh = x + (int64_t)h * qd;
-        v = T::to_float(xh[dd]);
-        if (r >= 0 && r < rot_dims) {
-          const float w = T::to_float(xh[dim + (r ^ 1)]), c = cs[r & ~1], s = cs[r | 1];
-          v = r & 1 ? v * c + w * s : v * c - w * s;
-        }
+  const S* x = q + row * q_stride;
+  S* y = out + (int64_t)row * heads * kpad;
+  const int qd = dim + rot_dim, per = kpad / E;
+  for (int i = threadIdx.x; i < heads * per; i += 256) {
+    const int h = i / per, d = (i - h * per) * E;
+    const S* xh = x + (int64_t)h * qd;
+    Piece t;
+    if constexpr (E == 1) {
+      float v = d < qd ? T::to_float(xh[d]) : 0.f;
+      const int r = d - dim;
+      if (r >= 0 && r < rot_dims) {
+        const float w = T::to_float(xh[dim + (r ^ 1)]), c = cs[r & ~1], s = cs[r | 1];
+        v = r & 1 ? v * c + w * s : v * c - w * s;
       }
-      y[2 * i + e] = T::from_float(v);
+      t.v[0] = T::from_float(v);
+    } else {  // (dim, rot_dim and rot_dims are multiples of E)
+      if (d < qd) {
+        t = *reinterpret_cast<const Piece*>(xh + d);
+        const int r = d - dim;
+        if (r >= 0 && r < rot_dims) {
+#pragma unroll
+          for (int e = 0; e < E; e += 2) {
+            const float u = T::to_float(t.v[e]), v = T::to_float(t.v[e + 1]), c = cs[r + e], s = cs[r + e + 1];
+            t.v[e] = T::from_float(u * c - v * s);
+            t.v[e + 1] = T::from_float(v * c + u * s);
+          }
+        }
+      } else {
+#pragma unroll
+        for (int e = 0; e < E; ++e) t.v[e] = T::from_float(0.f);
+      }
     }
+    *reinterpret_cast<Piece*>(y + (int64_t)i * E) = t;
   }
 }
 
@@ -340,18 +406,28 @@ __global__ __launch_bounds__(256) void latent_rotate_query_kernel(typename T::st
 
 using namespace lvllm;
 
+static int cache_params(LatentCacheParams& p, void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad,
+                        int rpad, const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
+                        const int64_t* positions, const double* turns, int rot_dims, const int64_t* slot_mapping, int rows) {
+  LV_CHECK(kv_rank > 0 && kv_rank <= cpad && cpad % 8 == 0 && rot_dim >= 0 && rot_dim <= rpad && rpad % 8 == 0 &&
+               rot_dims <= rot_dim && rot_dims % 2 == 0, "latent sizes");
+  p.cache = cache; p.block_stride = block_stride; p.num_slots = num_blocks * block_size; p.block_size = block_size;
+  p.cpad = cpad; p.rpad = rpad; p.kv = kv; p.kv_stride = kv_stride; p.kv_rank = kv_rank; p.rot_dim = rot_dim;
+  p.weight = weight; p.eps = eps; p.positions = positions; p.turns = turns; p.rot_dims = rot_dims;
+  p.slot_mapping = slot_mapping; p.rows = rows;
+  return 0;
+}
+
 extern "C" int lvllm_latent_cache(void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad, int rpad,
                                   const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
-                                  const int64_t* positions, const double* inv_freq, int rot_dims,
+                                  const int64_t* positions, const double* turns, int rot_dims,
                                   const int64_t* slot_mapping, int rows, int dtype, void* stream) {
   if (rows == 0) return 0;
-  LV_CHECK(kv_rank > 0 && kv_rank <= cpad && rot_dim >= 0 && rot_dim <= rpad && rot_dims <= rot_dim && rot_dims % 2 == 0,
-           "latent sizes");
+  LatentCacheParams p{};
+  if (int rc = cache_params(p, cache, block_stride, num_blocks, block_size, cpad, rpad, kv, kv_stride, kv_rank, rot_dim, weight,
+                            eps, positions, turns, rot_dims, slot_mapping, rows)) return rc;
   LV_DISPATCH_F32_BF16(dtype, {
-    using S = typename scalar_t::store_t;
-    hipLaunchKernelGGL((latent_cache_kernel<scalar_t>), dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, (S*)cache,
-                       block_stride, num_blocks * block_size, block_size, cpad, rpad, (const S*)kv, kv_stride, kv_rank, rot_dim,
-                       weight, eps, positions, inv_freq, rot_dims, slot_mapping, rows);
+    hipLaunchKernelGGL((latent_cache_kernel<scalar_t>), dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, p);
   });
   LV_LAUNCH_CHECK();
   return 0;
@@ -359,39 +435,32 @@ extern "C" int lvllm_latent_cache(void* cache, int64_t block_stride, int64_t num
 
 extern "C" int lvllm_latent_query(void* out, const void* q, int64_t q_stride, const void* uk_t, int heads, int dim, int dpad,
                                   int cpad, int rpad, int rot_dim, int rot_dims, const int64_t* positions,
-                                  const double* inv_freq, const int32_t* query_start_loc, int num_seqs, int absorbed_max,
-                                  int rows, int dtype, void* stream) {
-  LV_CHECK(dim > 0 && dim <= dpad && rot_dim <= rpad && rot_dims <= rot_dim && rot_dims % 2 == 0 && cpad % 16 == 0,
-           "latent sizes");
+                                  const double* turns, const int32_t* query_start_loc, int num_seqs, int absorbed_max,
+                                  void* cache, int64_t block_stride, int64_t num_blocks, int block_size, const void* kv,
+                                  int64_t kv_stride, int kv_rank, const float* weight, float eps,
+                                  const int64_t* slot_mapping, int rows, int dtype, void* stream) {
+  LV_CHECK(dim > 0 && dim <= dpad && rot_dim <= rpad && rot_dims <= rot_dim && rot_dims % 2 == 0 && cpad % 16 == 0 &&
+               rpad > 0 && rpad % 2 == 0, "latent sizes");
   HeadProjectParams p{};
   p.y = out; p.y_stride = (int64_t)heads * (cpad + rpad); p.y_head = cpad + rpad; p.n = cpad; p.npad = cpad;
   p.x = q; p.x_stride = q_stride; p.x_head = dim + rot_dim; p.k = dim; p.kpad = dpad; p.w = uk_t;
   p.rows = rows; p.heads = heads; p.query_start_loc = query_start_loc; p.num_seqs = num_seqs; p.absorbed_max = absorbed_max;
-  p.tail = rpad; p.rot_dim = rot_dim; p.rot_dims = rot_dims; p.positions = positions; p.inv_freq = inv_freq;
+  p.tail = rpad; p.rot_dim = rot_dim; p.rot_dims = rot_dims; p.positions = positions; p.turns = turns;
+  if (kv != nullptr)
+    if (int rc = cache_params(p.cache, cache, block_stride, num_blocks, block_size, cpad, rpad, kv, kv_stride, kv_rank, rot_dim,
+                              weight, eps, positions, turns, rot_dims, slot_mapping, rows)) return rc;
   return head_project(p, dtype, (hipStream_t)stream);
 }
 
-extern "C" int lvllm_latent_value(void* out, int64_t out_stride, const void* o_lat, const void* uv, const void* gate,
-                                  int64_t gate_stride, int heads, int vdim, int vpad, int cpad,
-                                  const int32_t* query_start_loc, int num_seqs, int absorbed_max, int rows, int dtype,
-                                  void* stream) {
-  LV_CHECK(vdim > 0 && vdim <= vpad && vpad % 16 == 0, "latent sizes");
-  HeadProjectParams p{};
-  p.y = out; p.y_stride = out_stride; p.y_head = vdim; p.n = vdim; p.npad = vpad;
-  p.x = o_lat; p.x_stride = (int64_t)heads * cpad; p.x_head = cpad; p.k = cpad; p.kpad = cpad; p.w = uv;
-  p.gate = gate; p.gate_stride = gate_stride;
-  p.rows = rows; p.heads = heads; p.query_start_loc = query_start_loc; p.num_seqs = num_seqs; p.absorbed_max = absorbed_max;
-  return head_project(p, dtype, (hipStream_t)stream);
-}
-
-// Shares the keys of a sequence are cut into: enough workgroups to fill the chip, none of under 128 keys
-static int latent_shares(int rows, int num_seqs, int heads, int max_query_len, int max_keys) {
+// Shares the keys of a sequence are cut into: a workgroup per CU (two where their tiles fit its LDS), none of under 128 keys
+static int latent_shares(int rows, int num_seqs, int heads, int cpad, int rpad, int max_query_len, int max_keys) {
   const int64_t cols = (int64_t)heads * max_query_len;
-  const int64_t wgs = num_seqs * ((cols + 31) / 32);
-  int64_t n = (512 + wgs - 1) / wgs;
-  const int64_t most = (max_keys + 127) / 128, room = ((int64_t)64 << 20) / ((int64_t)rows * heads) + 1;
+  const int64_t wgs = num_seqs * (cols <= 16 ? 1 : (cols + 31) / 32);
+  const int64_t room = 2 * 128 * (cpad + rpad) * 2 <= 150 * 1024 ? 512 : 256;
+  int64_t n = (room + wgs - 1) / wgs;
+  const int64_t most = (max_keys + 127) / 128, part = ((int64_t)64 << 20) / ((int64_t)rows * heads) + 1;
   n = n < most ? n : most;
-  n = n < room ? n : room;
+  n = n < part ? n : part;
   return n < 1 ? 1 : n > 64 ? 64 : (int)n;
 }
 
@@ -403,14 +472,16 @@ static int latent_max_keys(int max_seq_len, int window, int max_query_len) {
 extern "C" int64_t lvllm_latent_attention_workspace_bytes(int rows, int num_seqs, int heads, int cpad, int rpad,
                                                           int block_size, int window, int absorbed_max, int max_query_len,
                                                           int max_seq_len, int dtype) {
-  if (rows <= 0 || num_seqs <= 0 || heads <= 0 || !latent_takes_mfma(cpad, rpad, block_size, dtype)) return 0;
+  if (rows <= 0 || num_seqs <= 0 || heads <= 0) return 0;
+  if (!latent_takes_mfma(cpad, rpad, block_size, dtype)) return (int64_t)rows * heads * cpad * (dtype == LVLLM_F32 ? 4 : 2);
   const int q = max_query_len < absorbed_max ? max_query_len : absorbed_max;
-  const int n = latent_shares(rows, num_seqs, heads, q, latent_max_keys(max_seq_len, window, q));
-  return n > 1 ? (int64_t)rows * heads * n * (cpad + 2) * 4 : 0;
+  const int n = latent_shares(rows, num_seqs, heads, cpad, rpad, q, latent_max_keys(max_seq_len, window, q));
+  return (int64_t)rows * heads * n * (cpad + 2) * 4;
 }
 
-extern "C" int lvllm_latent_attention(void* out, const void* q, const void* cache, int64_t block_stride, int64_t num_blocks,
-                                      int block_size, int cpad, int rpad, const int32_t* block_tables, int max_blocks,
+extern "C" int lvllm_latent_attention(void* out, int64_t out_stride, const void* q, const void* cache, int64_t block_stride,
+                                      int64_t num_blocks, int block_size, int cpad, int rpad, const void* uv, int vdim, int vpad,
+                                      const void* gate, int64_t gate_stride, const int32_t* block_tables, int max_blocks,
                                       const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows,
                                       int heads, float scale, int window, int absorbed_max, int max_query_len,
                                       int max_seq_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
@@ -418,29 +489,37 @@ extern "C" int lvllm_latent_attention(void* out, const void* q, const void* cach
   LV_CHECK(heads > 0 && heads <= 65535 && num_seqs <= 65535 && max_query_len > 0, "too many heads or sequences, or no query");
   LV_CHECK(cpad > 0 && cpad % 16 == 0 && rpad % 16 == 0 && cpad <= 8192 && rpad <= 2048, "rows are multiples of 16 elements");
   LV_CHECK(max_blocks > 0 && num_blocks > 0 && block_size > 0, "an empty cache");
+  LV_CHECK(vdim > 0 && vdim <= vpad && vpad % 16 == 0, "value sizes");
+  LV_CHECK(workspace != nullptr &&
+               workspace_bytes >= lvllm_latent_attention_workspace_bytes(rows, num_seqs, heads, cpad, rpad, block_size, window,
+                                                                         absorbed_max, max_query_len, max_seq_len, dtype),
+           "workspace too small (see lvllm_latent_attention_workspace_bytes)");
   LatentAttnParams p{};
-  p.out = out; p.q = q; p.cache = cache; p.block_tables = block_tables; p.seq_lens = seq_lens;
+  p.out = out; p.out_stride = out_stride; p.q = q; p.cache = cache; p.block_tables = block_tables; p.seq_lens = seq_lens;
   p.query_start_loc = query_start_loc; p.num_seqs = num_seqs; p.rows = rows; p.heads = heads; p.cpad = cpad; p.rpad = rpad;
   p.max_blocks = max_blocks; p.block_size = block_size; p.max_block = (int)(num_blocks - 1); p.nsplit = 1; p.window = window;
-  p.absorbed_max = absorbed_max; p.scale = scale; p.block_stride = block_stride;
+  p.absorbed_max = absorbed_max; p.scale = scale; p.block_stride = block_stride; p.uv = uv; p.vdim = vdim; p.vpad = vpad;
+  p.gate = gate; p.gate_stride = gate_stride;
   p.max_query_len = max_query_len < absorbed_max ? max_query_len : absorbed_max;
   hipStream_t s = (hipStream_t)stream;
   if (latent_takes_mfma(cpad, rpad, block_size, dtype)) {
-    p.nsplit = latent_shares(rows, num_seqs, heads, p.max_query_len, latent_max_keys(max_seq_len, window, p.max_query_len));
-    if (p.nsplit > 1) {
-      LV_CHECK(workspace != nullptr && workspace_bytes >= (int64_t)rows * heads * p.nsplit * (cpad + 2) * 4,
-               "workspace too small (see lvllm_latent_attention_workspace_bytes)");
-      p.part_o = (float*)workspace;
-      p.part_ml = p.part_o + (int64_t)rows * heads * p.nsplit * cpad;
-    }
+    p.nsplit = latent_shares(rows, num_seqs, heads, cpad, rpad, p.max_query_len,
+                             latent_max_keys(max_seq_len, window, p.max_query_len));
+    p.part_o = (float*)workspace;
+    p.part_ml = p.part_o + (int64_t)rows * heads * p.nsplit * cpad;
     return launch_latent_mfma(p, s);
   }
   LV_DISPATCH_F32_BF16(dtype, {
     hipLaunchKernelGGL((latent_attention_simple_kernel<scalar_t>), dim3(rows, heads), dim3(256),
-                       (size_t)(2 * cpad + rpad + 256) * 4, s, p);
+                       (size_t)(2 * cpad + rpad + 256) * 4, s, p, workspace);
   });
   LV_LAUNCH_CHECK();
-  return 0;
+  HeadProjectParams v{};
+  v.y = out; v.y_stride = out_stride; v.y_head = vdim; v.n = vdim; v.npad = vpad;
+  v.x = workspace; v.x_stride = (int64_t)heads * cpad; v.x_head = cpad; v.k = cpad; v.kpad = cpad; v.w = uv;
+  v.gate = gate; v.gate_stride = gate_stride;
+  v.rows = rows; v.heads = heads; v.query_start_loc = query_start_loc; v.num_seqs = num_seqs; v.absorbed_max = absorbed_max;
+  return head_project(v, dtype, s);
 }
 
 extern "C" int lvllm_latent_gather(void* out, const void* cache, int64_t block_stride, int64_t num_blocks, int block_size,
@@ -470,15 +549,22 @@ extern "C" int lvllm_latent_expand(void* key_pages, void* value_pages, const voi
 }
 
 extern "C" int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_stride, int heads, int dim, int rot_dim, int kpad,
-                                         const int64_t* positions, const double* inv_freq, int rot_dims, int rows, int dtype,
+                                         const int64_t* positions, const double* turns, int rot_dims, int rows, int dtype,
                                          void* stream) {
   if (rows == 0) return 0;
-  LV_CHECK(dim + rot_dim <= kpad && kpad % 2 == 0 && rot_dims <= rot_dim && rot_dims % 2 == 0 && rot_dims <= 4096, "query sizes");
+  LV_CHECK(dim + rot_dim <= kpad && rot_dims <= rot_dim && rot_dims % 2 == 0 && rot_dims <= 4096, "query sizes");
+  const int e = dtype == LVLLM_F32 ? 4 : 8;
+  const bool vec = ((dim | rot_dim | rot_dims | kpad) % e == 0) && q_stride % e == 0 && ((uintptr_t)q & 15) == 0;
   LV_DISPATCH_F32_BF16(dtype, {
     using S = typename scalar_t::store_t;
-    hipLaunchKernelGGL((latent_rotate_query_kernel<scalar_t>), dim3(rows), dim3(256), (size_t)rot_dims * 4 + 8,
-                       (hipStream_t)stream, (S*)out, (const S*)q, q_stride, heads, dim, rot_dim, kpad, positions, inv_freq,
-                       rot_dims);
+    if (vec)
+      hipLaunchKernelGGL((latent_rotate_query_kernel<scalar_t, 16 / sizeof(S)>), dim3(rows), dim3(256),
+                         (size_t)rot_dims * 4 + 8, (hipStream_t)stream, (S*)out, (const S*)q, q_stride, heads, dim, rot_dim,
+                         kpad, positions, turns, rot_dims);
+    else
+      hipLaunchKernelGGL((latent_rotate_query_kernel<scalar_t, 1>), dim3(rows), dim3(256), (size_t)rot_dims * 4 + 8,
+                         (hipStream_t)stream, (S*)out, (const S*)q, q_stride, heads, dim, rot_dim, kpad, positions, turns,
+                         rot_dims);
   });
   LV_LAUNCH_CHECK();
   return 0;

@@ -1,13 +1,14 @@
 // The absorbed body of latent_attention.h on bf16 MFMAs: scores and weighted sums on the cached rows themselves.
 //
 // A workgroup serves 16 CT (token, head) columns of one sequence and one share of the keys; the columns' window is walked in
-// tiles of 64 keys = 4 pages.  Pages are contiguous in memory and go to LDS row by row (16 bytes of padding between rows: row
-// reads and transposed reads are free of bank conflicts), the next tile's loads in flight in registers meanwhile.  Four
+// tiles of 64 keys = 4 pages.  Pages are contiguous in memory and go straight to LDS (two stages: the next tile's copies are
+// in flight while one is used), the 16-byte chunks of a row exchanged so that row reads are free of bank conflicts.  Four
 // waves work on 16 columns:
 //   * S^T = rows x q'^T: wave w scores the tile's page w; the columns' maxima meet in LDS;
 //   * the probabilities go through LDS (64 keys x 16 columns of bf16);
 //   * O^T += rows^T x P: wave w sums a quarter of the latent's entries; rows^T is read with the transposing LDS read.
-// One read of a row serves both products and all 16 CT columns.  Shares meet in a second small launch.
+// One read of a row serves both products and all 16 CT columns.  A second launch adds the shares, takes the sums out of
+// latent space (V_h) and applies the gate.
 #include <float.h>
 
 #include "latent_attention.h"
@@ -25,21 +26,30 @@ __device__ __forceinline__ m_f32x4_t mfma16(m_u32x4_t a, m_u32x4_t b, m_f32x4_t 
                                                  0);
 }
 
+// What chunk numbers of row r of a page are exchanged by (an exclusive or): rows whose first bank is the same differ.
+template <int NK>
+__device__ __forceinline__ int exchange(int r) {
+  return NK % 4 == 0 ? r & 15 : NK % 2 == 0 ? (r >> 1) & 7 : (r >> 2) & 3;
+}
+
+// everything written to LDS so far is seen by the workgroup; copies in flight stay in flight
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 // NC, NR: latent and rotated part in units of 32 entries
 template <int NC, int NR, int CT>
-__global__ __launch_bounds__(256 * CT, CT == 1 ? 2 : 1) void latent_attention_mfma_kernel(const LatentAttnParams p) {
+__global__ __launch_bounds__(256 * CT, 1) void latent_attention_mfma_kernel(const LatentAttnParams p) {
   constexpr int NK = NC + NR, RE = 32 * NK, CP = 32 * NC;
-  constexpr int RC = 4 * NK;               // 16-byte chunks of a row
-  constexpr int PITCH = RE * 2 + 16;       // bytes between rows in LDS
-  constexpr int LOADS = CT == 1 ? NK : (NK + 1) / 2;  // of 64 chunks, per wave: a page is 64 NK chunks
+  constexpr int RC = 4 * NK, RB = 64 * NK;  // 16-byte chunks and bytes of a row
+  constexpr int kStage = 64 * RB;
+  constexpr int COPIES = (NK + CT - 1) / CT;  // of 1 KiB, per wave and tile: a page is NK KiB
   constexpr int NT = NC / 2;               // 16-entry tiles of O a wave owns
   constexpr int PP = 72;                   // elements between columns of P
-  extern __shared__ __attribute__((aligned(16))) char tile[];  // [64][PITCH]
+  extern __shared__ __attribute__((aligned(16))) char tile[];  // [2][64][RB]
   __shared__ __attribute__((aligned(16))) uint16_t sp[CT][16 * PP];
   __shared__ float sm[CT][4][16];
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int kg = wave & 3, ct = wave >> 2;
+  const int kg = CT == 1 ? wave : wave & 3, ct = CT == 1 ? 0 : wave >> 2;
   const int g = lane >> 4, c = lane & 15;
   const int seq = blockIdx.y, share = blockIdx.z;
   const int qbeg = p.query_start_loc[seq], qlen = p.query_start_loc[seq + 1] - qbeg;
@@ -58,48 +68,65 @@ __global__ __launch_bounds__(256 * CT, CT == 1 ? 2 : 1) void latent_attention_mf
   const int per = (ntiles + p.nsplit - 1) / p.nsplit;
   const int t0 = share * per, t1 = min(t0 + per, ntiles);
 
+  const int32_t* table = p.block_tables + (int64_t)seq * p.max_blocks;
+  int from[COPIES];  // elements from the page's start that this lane copies
+#pragma unroll
+  for (int j = 0; j < COPIES; ++j) {
+    const int i = (j * CT + ct) * 64 + lane, r = i / RC;
+    from[j] = r * RE + ((i - r * RC) ^ exchange<NK>(r)) * 8;
+  }
+  auto page_of = [&](int t) { return table[min(lo / 16 + 4 * t + kg, p.max_blocks - 1)]; };
+  auto copy = [&](int t, int page) __attribute__((always_inline)) {
+    const int64_t blk = min(max(page, 0), p.max_block);
+    const uint16_t* src = (const uint16_t*)p.cache + blk * p.block_stride;
+    char* dst = tile + ((t - t0) & 1) * kStage + kg * 16 * RB;
+#pragma unroll
+    for (int j = 0; j < COPIES; ++j)
+      if (j * CT + ct < NK)
+        __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + from[j]),
+                                         (__attribute__((address_space(3))) void*)(dst + (j * CT + ct) * 1024), 16, 0, 0);
+  };
+  if (t0 < t1) copy(t0, page_of(t0));
+  int page = page_of(t0 + 1);  // (looked up a tile ahead)
   m_u32x4_t qf[NK];
   {
     const uint16_t* q = (const uint16_t*)p.q + at * RE + 8 * g;
 #pragma unroll
     for (int j = 0; j < NK; ++j) qf[j] = *reinterpret_cast<const m_u32x4_t*>(q + 32 * j);
   }
-  const int32_t* table = p.block_tables + (int64_t)seq * p.max_blocks;
-  m_u32x4_t st[LOADS];
-  auto fetch = [&](int t) __attribute__((always_inline)) {
-    const int64_t blk = min(max(table[min(lo / 16 + 4 * t + kg, p.max_blocks - 1)], 0), p.max_block);
-    const uint16_t* src = (const uint16_t*)p.cache + blk * p.block_stride;
-#pragma unroll
-    for (int j = 0; j < LOADS; ++j) {
-      const int i = (ct * LOADS + j) * 64 + lane;
-      if (CT == 1 || ct * LOADS + j < NK) st[j] = *reinterpret_cast<const m_u32x4_t*>(src + i * 8);
-    }
-  };
-  auto put = [&]() __attribute__((always_inline)) {
-#pragma unroll
-    for (int j = 0; j < LOADS; ++j) {
-      const int i = (ct * LOADS + j) * 64 + lane;
-      if (CT == 1 || ct * LOADS + j < NK)
-        *reinterpret_cast<m_u32x4_t*>(tile + (kg * 16 + i / RC) * PITCH + (i % RC) * 16) = st[j];
-    }
-  };
+  __builtin_amdgcn_s_waitcnt(0 | (7 << 4) | (15 << 8));  // (q has landed: nothing in the loop waits for it)
   const float sl = p.scale * 1.4426950408889634f;
   float m = -1e30f, l = 0.f;
   m_f32x4_t o[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) o[i] = m_f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const char* krow = tile + (kg * 16 + c) * PITCH + 16 * g;
-  const char* vrow = tile + (8 * g + (c >> 2)) * PITCH + (kg * NT * 16 + 4 * (c & 3)) * 2;
+  const int kx = exchange<NK>(c), krow = (kg * 16 + c) * RB;
+  const int vr = 8 * g + (c >> 2), vx0 = exchange<NK>(vr & 15), vx1 = exchange<NK>((vr + 4) & 15);
+  const int vc = kg * NT * 2 + ((c & 3) >> 1), vb = (c & 1) * 8;
   typedef __attribute__((address_space(3))) m_i16x4_t* lds_tr_t;
 
-  if (t0 < t1) fetch(t0);
   for (int t = t0; t < t1; ++t) {
-    put();
-    __syncthreads();
-    if (t + 1 < t1) fetch(t + 1);
-    m_f32x4_t s{0.f, 0.f, 0.f, 0.f};
+    // the copies of this tile have landed, for every wave; everyone is done with the tile before
+    __builtin_amdgcn_s_waitcnt(0 | (7 << 4) | (15 << 8));
+    asm volatile("s_barrier" ::: "memory");
+    if (t + 1 < t1) copy(t + 1, page);
+    page = page_of(t + 2);
+    const char* st = tile + ((t - t0) & 1) * kStage;
+    m_f32x4_t s{0.f, 0.f, 0.f, 0.f}, s2{0.f, 0.f, 0.f, 0.f};
+    constexpr int W = NK < 6 ? NK : 6;  // fragments read ahead
+    m_u32x4_t k[W];
+    auto kread = [&](int j) { return *reinterpret_cast<const m_u32x4_t*>(st + krow + (((4 * j + g) ^ kx) * 16)); };
 #pragma unroll
-    for (int j = 0; j < NK; ++j) s = mfma16(*reinterpret_cast<const m_u32x4_t*>(krow + 64 * j), qf[j], s);
+    for (int j = 0; j < W; ++j) k[j] = kread(j);
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int j = 0; j < NK; ++j) {
+      if (j & 1) s2 = mfma16(k[j % W], qf[j], s2);
+      else s = mfma16(k[j % W], qf[j], s);
+      if (j + W < NK) k[j % W] = kread(j + W);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    s += s2;
     const int key0 = lo + 64 * t + 16 * kg + 4 * g;
 #pragma unroll
     for (int r = 0; r < 4; ++r) s[r] = key0 + r <= pos && key0 + r >= low ? s[r] * sl : -FLT_MAX;
@@ -107,7 +134,7 @@ __global__ __launch_bounds__(256 * CT, CT == 1 ? 2 : 1) void latent_attention_mf
     mx = fmaxf(mx, __shfl_xor(mx, 16));
     mx = fmaxf(mx, __shfl_xor(mx, 32));
     if (g == 0) sm[ct][kg][c] = mx;
-    __syncthreads();
+    lds_barrier();
     mx = fmaxf(fmaxf(sm[ct][0][c], sm[ct][1][c]), fmaxf(sm[ct][2][c], sm[ct][3][c]));
     if (__any(mx > m)) {
       const float mn = fmaxf(m, mx), corr = exp2f(m - mn);
@@ -125,73 +152,122 @@ __global__ __launch_bounds__(256 * CT, CT == 1 ? 2 : 1) void latent_attention_mf
       w.y = (uint32_t)BF16::from_float(s[2]) | ((uint32_t)BF16::from_float(s[3]) << 16);
       *reinterpret_cast<uint2*>(&sp[ct][c * PP + 16 * kg + 4 * g]) = w;
     }
-    __syncthreads();
+    lds_barrier();
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
       const m_u32x4_t pf = *reinterpret_cast<const m_u32x4_t*>(&sp[ct][c * PP + 32 * ks + 8 * g]);
+      const char* v = st + (32 * ks + vr) * RB + vb;
+      m_i16x4_t a[NT], b[NT];
 #pragma unroll
       for (int i = 0; i < NT; ++i) {
-        const char* v = vrow + 32 * ks * PITCH + 32 * i;
-        const m_i16x4_t a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_t)v);
-        const m_i16x4_t b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_t)(v + 4 * PITCH));
-        const m_u32x2_t ua = __builtin_bit_cast(m_u32x2_t, a), ub = __builtin_bit_cast(m_u32x2_t, b);
+        a[i] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_t)(v + (((vc + 2 * i) ^ vx0) * 16)));
+        b[i] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_t)(v + 4 * RB + (((vc + 2 * i) ^ vx1) * 16)));
+      }
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        const m_u32x2_t ua = __builtin_bit_cast(m_u32x2_t, a[i]), ub = __builtin_bit_cast(m_u32x2_t, b[i]);
         o[i] = mfma16(m_u32x4_t{ua.x, ua.y, ub.x, ub.y}, pf, o[i]);
       }
     }
-    __syncthreads();
   }
   l += __shfl_xor(l, 16);
   l += __shfl_xor(l, 32);
+  __syncthreads();
   if (g == 0) sm[ct][kg][c] = l;
   __syncthreads();
-  l = (sm[ct][0][c] + sm[ct][1][c]) + (sm[ct][2][c] + sm[ct][3][c]);
   if (!col_ok) return;
-  if (p.nsplit > 1) {
-    const int64_t part = at * p.nsplit + share;
-    float* out = p.part_o + part * CP + kg * NT * 16 + 4 * g;
+  const int64_t part = at * p.nsplit + share;
+  float* out = p.part_o + part * CP + kg * NT * 16 + 4 * g;
 #pragma unroll
-    for (int i = 0; i < NT; ++i) *reinterpret_cast<m_f32x4_t*>(out + 16 * i) = o[i];
-    if (kg == 0 && g == 0) {
-      p.part_ml[2 * part] = m;
-      p.part_ml[2 * part + 1] = l;
-    }
-  } else {
-    const float f = l > 0.f ? 1.f / l : 0.f;
-    uint16_t* out = (uint16_t*)p.out + at * CP + kg * NT * 16 + 4 * g;
-#pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const float v[4] = {o[i][0] * f, o[i][1] * f, o[i][2] * f, o[i][3] * f};
-      store4<BF16>(out + 16 * i, v);
-    }
+  for (int i = 0; i < NT; ++i) *reinterpret_cast<m_f32x4_t*>(out + 16 * i) = o[i];
+  if (kg == 0 && g == 0) {
+    p.part_ml[2 * part] = m;
+    p.part_ml[2 * part + 1] = (sm[ct][0][c] + sm[ct][1][c]) + (sm[ct][2][c] + sm[ct][3][c]);
   }
 }
 
-// Shares of one (row, head) -> out
-__global__ __launch_bounds__(128) void latent_reduce_kernel(const LatentAttnParams p) {
-  const int row = blockIdx.x, head = blockIdx.y;
-  const int seq = find_seq(p.query_start_loc, p.num_seqs, row);
-  if (seq >= p.num_seqs) return;
-  if (p.query_start_loc[seq + 1] - p.query_start_loc[seq] > p.absorbed_max) return;
-  const int64_t at = ((int64_t)row * p.heads + head) * p.nsplit;
-  float m = -1e30f;
-  for (int s = 0; s < p.nsplit; ++s) m = fmaxf(m, p.part_ml[2 * (at + s)]);
-  float l = 0.f;
-  for (int s = 0; s < p.nsplit; ++s) l += p.part_ml[2 * (at + s) + 1] * exp2f(p.part_ml[2 * (at + s)] - m);
-  const float f = l > 0.f ? 1.f / l : 0.f;
-  for (int d = threadIdx.x * 4; d < p.cpad; d += 512) {
-    float v[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < p.nsplit; ++s) {
-      const float w = exp2f(p.part_ml[2 * (at + s)] - m) * f;
-      const float4 t = *reinterpret_cast<const float4*>(p.part_o + (at + s) * p.cpad + d);
-      v[0] = fmaf(t.x, w, v[0]); v[1] = fmaf(t.y, w, v[1]); v[2] = fmaf(t.z, w, v[2]); v[3] = fmaf(t.w, w, v[3]);
+// The shares of R rows of one head -> their weighted sum o in latent space (bf16, as W's product reads it) -> out = V_h o * gate.
+// grid (heads, rows / R); a wave adds the shares of R / 4 rows, then takes every fourth 16-row tile of V_h.
+template <int R>
+__global__ __launch_bounds__(256) void latent_value_kernel(const LatentAttnParams p) {
+  extern __shared__ __attribute__((aligned(16))) uint16_t so[];  // [R][cpad + 8]
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int g = lane >> 4, c = lane & 15;
+  const int head = blockIdx.x, row0 = blockIdx.y * R, ld = p.cpad + 8;
+  constexpr int B = 8;  // k-steps in flight
+  const int steps = p.cpad >> 5;
+  const uint16_t* uv = (const uint16_t*)p.uv + ((int64_t)head * p.vpad + c) * p.cpad + 8 * g;
+  m_u32x4_t w[B];
+  auto fetch = [&](int n, int k0) __attribute__((always_inline)) {
+#pragma unroll
+    for (int j = 0; j < B; ++j)
+      w[j] = *reinterpret_cast<const m_u32x4_t*>(uv + (int64_t)n * 16 * p.cpad + 32 * min(k0 + j, steps - 1));
+  };
+  if (wave * 16 < p.vpad) fetch(wave, 0);
+  for (int i = wave; i < R; i += 4) {
+    const int row = row0 + i;
+    const int seq = row < p.rows ? find_seq(p.query_start_loc, p.num_seqs, row) : p.num_seqs;
+    const bool ok = seq < p.num_seqs && p.query_start_loc[seq + 1] - p.query_start_loc[seq] <= p.absorbed_max;
+    if (!ok) {
+      for (int d = lane; d < p.cpad; d += 64) so[i * ld + d] = 0;
+      continue;
     }
-    store4<BF16>((uint16_t*)p.out + ((int64_t)row * p.heads + head) * p.cpad + d, v);
+    const int64_t at = ((int64_t)row * p.heads + head) * p.nsplit;
+    const float ms = lane < p.nsplit ? p.part_ml[2 * (at + lane)] : -1e30f;
+    const float ls = lane < p.nsplit ? p.part_ml[2 * (at + lane) + 1] : 0.f;
+    const float m = wave_max(ms);
+    const float e = exp2f(ms - m), l = wave_sum(ls * e);
+    const float ws = l > 0.f ? e / l : 0.f;
+    for (int d = lane * 4; d < p.cpad; d += 256) {
+      float v[4] = {0.f, 0.f, 0.f, 0.f};
+      for (int s0 = 0; s0 < p.nsplit; s0 += 4) {
+        float4 t[4];
+#pragma unroll
+        for (int s = 0; s < 4; ++s) t[s] = *reinterpret_cast<const float4*>(p.part_o + (at + min(s0 + s, p.nsplit - 1)) * p.cpad + d);
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+          const float f = s0 + s < p.nsplit ? __shfl(ws, s0 + s) : 0.f;
+          v[0] = fmaf(t[s].x, f, v[0]); v[1] = fmaf(t[s].y, f, v[1]); v[2] = fmaf(t[s].z, f, v[2]); v[3] = fmaf(t[s].w, f, v[3]);
+        }
+      }
+      store4<BF16>(so + i * ld + d, v);
+    }
+  }
+  __syncthreads();
+  const int row = row0 + c;
+  bool mine = c < R && row < p.rows;
+  if (mine) {
+    const int seq = find_seq(p.query_start_loc, p.num_seqs, row);  // (padding rows get zeros)
+    mine = seq >= p.num_seqs || p.query_start_loc[seq + 1] - p.query_start_loc[seq] <= p.absorbed_max;
+  }
+  float f = 1.f;
+  if (mine && p.gate != nullptr)
+    f = 1.f / (1.f + expf(-BF16::to_float(((const uint16_t*)p.gate)[row * p.gate_stride + head])));
+  for (int n = wave; n * 16 < p.vpad; n += 4) {
+    m_f32x4_t acc{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < steps; k0 += B) {
+      if (n != wave || k0 > 0) fetch(n, k0);
+#pragma unroll
+      for (int j = 0; j < B; ++j) {
+        const int k = 32 * (k0 + j) + 8 * g;
+        m_u32x4_t x{0, 0, 0, 0};
+        if (k0 + j < steps && c < R) x = *reinterpret_cast<const m_u32x4_t*>(so + c * ld + k);
+        acc = mfma16(w[j], x, acc);
+      }
+    }
+    if (!mine) continue;
+    uint16_t* out = (uint16_t*)p.out + row * p.out_stride + (int64_t)head * p.vdim + 16 * n + 4 * g;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (16 * n + 4 * g + r < p.vdim) out[r] = BF16::from_float(acc[r] * f);
   }
 }
 
 template <int NC, int NR, int CT>
 static void go(const LatentAttnParams& p, hipStream_t s) {
-  constexpr int smem = 64 * (64 * (NC + NR) + 16);
+  constexpr int smem = 2 * 64 * 64 * (NC + NR);
   if (smem > 64 * 1024)
     (void)hipFuncSetAttribute((const void*)latent_attention_mfma_kernel<NC, NR, CT>,
                               hipFuncAttributeMaxDynamicSharedMemorySize, smem);
@@ -225,10 +301,12 @@ int launch_latent_mfma(const LatentAttnParams& p, hipStream_t s) {
   }
 #undef LV_LATENT_R
   LV_LAUNCH_CHECK();
-  if (p.nsplit > 1) {
-    hipLaunchKernelGGL(latent_reduce_kernel, dim3(p.rows, p.heads), dim3(128), 0, s, p);
-    LV_LAUNCH_CHECK();
-  }
+  LV_CHECK((p.rows + 3) / 4 <= 65535, "too many rows");
+  if (p.rows <= 256)
+    hipLaunchKernelGGL((latent_value_kernel<4>), dim3(p.heads, (p.rows + 3) / 4), dim3(256), 4 * (p.cpad + 8) * 2, s, p);
+  else
+    hipLaunchKernelGGL((latent_value_kernel<16>), dim3(p.heads, (p.rows + 15) / 16), dim3(256), 16 * (p.cpad + 8) * 2, s, p);
+  LV_LAUNCH_CHECK();
   return 0;
 }
 

@@ -1,52 +1,8 @@
 // Mixture of experts: the router, the grouping of a step's assignments, and the plain products (moe.h; the matrix-core
 // bodies are in moe_mfma.hip).
-#include <float.h>
-
 #include "moe.h"
 
 namespace lvllm {
-
-constexpr int kMaxExperts = 1024;
-
-// The `top` largest of z[0 .. experts) (LDS; ties: the smaller index) by one wave, their softmax, and the shared expert.
-// Any z gives indices in range.
-__device__ __forceinline__ void choose_experts(float* z, int experts, int top, bool shared, int32_t* ids, float* weights) {
-  const int lane = threadIdx.x & 63;
-  float first = 0.f, sum = 0.f, mine = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float best = -INFINITY;
-    int at = kMaxExperts;
-    for (int e = lane; e < experts; e += 64) {
-      const float v = z[e];
-      if (v > best || (at == kMaxExperts && v == v && v != -INFINITY)) { best = v; at = e; }
-    }
-#pragma unroll
-    for (int m = 32; m >= 1; m >>= 1) {
-      const float ob = __shfl_xor(best, m);
-      const int oa = __shfl_xor(at, m);
-      if (oa < kMaxExperts && (at == kMaxExperts || ob > best || (ob == best && oa < at))) { best = ob; at = oa; }
-    }
-    if (at >= kMaxExperts) {  // nothing comparable left: the first one not taken (marked by -inf) or, among NaNs, the k-th
-      at = k;
-      best = first;
-    }
-    if (k == 0) first = best;
-    const float e = expf(best - first);
-    sum += e;
-    if (lane == k) mine = e;
-    if (lane == 0) {
-      ids[k] = at;
-      z[at] = -INFINITY;
-    }
-    __builtin_amdgcn_wave_barrier();
-    __threadfence_block();
-  }
-  if (lane < top) weights[lane] = mine / sum;
-  if (shared && lane == 0) {
-    ids[top] = experts;
-    weights[top] = 1.f / (1.f + expf(-z[experts]));
-  }
-}
 
 // A workgroup per row: a wave takes one expert after the other.  Logits are fp32 sums of exact products.
 template <typename T, int VEC>
@@ -87,7 +43,18 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(int32_t* __restrict__ o
   __shared__ int count[kMaxExperts + 1], first[kMaxExperts + 2], tile0[kMaxExperts + 2];
   for (int e = threadIdx.x; e < experts; e += 1024) count[e] = 0;
   __syncthreads();
-  for (int i = threadIdx.x; i < total; i += 1024) slot[i] = atomicAdd(&count[min(max(ids[i], 0), experts - 1)], 1);
+  constexpr int B = 8;  // loads in flight
+  for (int i0 = threadIdx.x; i0 < total; i0 += 1024 * B) {
+    int e[B];
+#pragma unroll
+    for (int j = 0; j < B; ++j) e[j] = i0 + 1024 * j < total ? min(max(ids[i0 + 1024 * j], 0), experts - 1) : -1;
+#pragma unroll
+    for (int j = 0; j < B; ++j)
+      if (e[j] >= 0) e[j] = atomicAdd(&count[e[j]], 1);
+#pragma unroll
+    for (int j = 0; j < B; ++j)
+      if (i0 + 1024 * j < total) slot[i0 + 1024 * j] = e[j];
+  }
   __syncthreads();
   if (threadIdx.x < 64) {  // running sums, 64 experts a turn
     int base = 0, tbase = 0;
@@ -108,10 +75,21 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(int32_t* __restrict__ o
   }
   __syncthreads();
   for (int e = threadIdx.x; e <= experts; e += 1024) offsets[e] = first[e];
-  for (int i = threadIdx.x; i < total; i += 1024) {
-    const int s = first[min(max(ids[i], 0), experts - 1)] + slot[i];
-    slot[i] = s;
-    token[s] = i / per_row;
+  for (int i0 = threadIdx.x; i0 < total; i0 += 1024 * B) {
+    int e[B], s[B];
+#pragma unroll
+    for (int j = 0; j < B; ++j) {
+      const int i = min(i0 + 1024 * j, total - 1);
+      e[j] = min(max(ids[i], 0), experts - 1);
+      s[j] = slot[i];
+    }
+#pragma unroll
+    for (int j = 0; j < B; ++j) {
+      const int i = i0 + 1024 * j;
+      if (i >= total) break;
+      slot[i] = first[e[j]] + s[j];
+      token[first[e[j]] + s[j]] = i / per_row;
+    }
   }
   for (int e = threadIdx.x; e < experts; e += 1024)
     for (int t = tile0[e]; t < tile0[e + 1] && t < max_tiles; ++t) {
@@ -119,6 +97,10 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(int32_t* __restrict__ o
       tiles[2 * t + 1] = first[e] + (t - tile0[e]) * tile;
     }
   for (int t = tile0[experts] + threadIdx.x; t < max_tiles; t += 1024) tiles[2 * t] = -1;
+  if (threadIdx.x == 0) {
+    tiles[2 * max_tiles] = min(tile0[experts - 1], max_tiles);
+    tiles[2 * max_tiles + 1] = min(tile0[experts], max_tiles);
+  }
 }
 
 // 16 slots x 16 outputs a workgroup, row-major weights, 32 of K a turn through LDS.
@@ -166,17 +148,22 @@ __global__ __launch_bounds__(256) void moe_simple_kernel(const MoeParams p) {
 using namespace lvllm;
 
 extern "C" int lvllm_moe_route(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts,
-                               int shared, int top, int rows, int width, int dtype, void* stream) {
+                               int shared, int top, int rows, int width, int packed, int dtype, void* stream) {
   if (rows == 0) return 0;
   LV_CHECK(experts > 0 && experts < kMaxExperts && top > 0 && top <= experts && top <= 64, "experts (fewer than 1024) or top (at most 64)");
+  hipStream_t s = (hipStream_t)stream;
+  if (packed) {
+    LV_CHECK(moe_takes_mfma(width, dtype), "packed router: bf16, a width that is a multiple of 32");
+    return launch_moe_route_mfma(ids, weights, h, w, bias, experts, shared != 0, top, rows, width, s);
+  }
   LV_DISPATCH_F32_BF16(dtype, {
     using S = typename scalar_t::store_t;
     if (width % 4 == 0)
-      hipLaunchKernelGGL((moe_route_kernel<scalar_t, 4>), dim3(rows), dim3(256), 0, (hipStream_t)stream, ids, weights,
-                         (const S*)h, (const S*)w, bias, experts, shared != 0, top, width);
+      hipLaunchKernelGGL((moe_route_kernel<scalar_t, 4>), dim3(rows), dim3(256), 0, s, ids, weights, (const S*)h, (const S*)w,
+                         bias, experts, shared != 0, top, width);
     else
-      hipLaunchKernelGGL((moe_route_kernel<scalar_t, 1>), dim3(rows), dim3(256), 0, (hipStream_t)stream, ids, weights,
-                         (const S*)h, (const S*)w, bias, experts, shared != 0, top, width);
+      hipLaunchKernelGGL((moe_route_kernel<scalar_t, 1>), dim3(rows), dim3(256), 0, s, ids, weights, (const S*)h, (const S*)w,
+                         bias, experts, shared != 0, top, width);
   });
   LV_LAUNCH_CHECK();
   return 0;
@@ -196,14 +183,14 @@ extern "C" int lvllm_moe_group(int32_t* offsets, int32_t* token, int32_t* slot, 
 
 extern "C" int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff,
                                  const float* limit, const int32_t* offsets, const int32_t* token, const int32_t* tiles,
-                                 int experts, int slots, int rows, int width, int ff_max, int max_tiles, int up, int packed,
-                                 int dtype, void* stream) {
+                                 int experts, int slots, int rows, int width, int ff_max, int ff_first, int ff_last, int max_tiles, int up,
+                                 int packed, int dtype, void* stream) {
   if (slots == 0) return 0;
   LV_CHECK(experts > 0 && ff_max > 0 && ff_max % 32 == 0 && width > 0 && max_tiles > 0 && max_tiles <= 65535, "sizes of the experts");
   MoeParams p{};
   p.out = out; p.x = x; p.w = w; p.w_offset = w_offset; p.ff = ff; p.limit = limit; p.offsets = offsets; p.token = token;
   p.tiles = tiles; p.experts = experts; p.slots = slots; p.rows = rows; p.width = width; p.ff_max = ff_max;
-  p.max_tiles = max_tiles;
+  p.max_tiles = max_tiles; p.ff_first = ff_first; p.ff_last = ff_last;
   hipStream_t s = (hipStream_t)stream;
   if (packed) {
     LV_CHECK(moe_takes_mfma(width, dtype), "packed experts: bf16, a width that is a multiple of 32");

@@ -2,10 +2,12 @@
 // lane ends up with consecutive outputs of one slot, and gate and value of an activation in the same register of two tiles.
 //
 //   * few slots per expert (decode steps): bound by the weights' bytes.  A workgroup takes 16 slots of one expert and a share
-//     of its outputs; the slots' rows sit in LDS in fragment order, every wave streams W tiles of its own (1 KiB a load, eight
-//     k-steps in flight behind the eight in use) and needs no other wave;
-//   * prompts: 128 slots x 256 W rows a workgroup, a wave 128 x 64.  The slots' rows go through LDS (two stages of 64 k,
-//     XOR-swizzled), W comes from global memory straight into the operand registers of the one wave that uses it.
+//     of its outputs; the slots' rows sit in LDS in fragment order (2048 of K at a time), every wave streams the two W tiles
+//     of its own (1 KiB a load, eight k-steps in flight behind the eight in use) and needs no other wave;
+//   * prompts: 256 W rows x 128 slots a workgroup, a wave 128 x 64.  Both operands go straight from memory to LDS, 32 of K a
+//     stage, two stages in flight behind the one in use.  Packed W tiles are LDS images as they are; a slot's 64 bytes are
+//     four chunks, exchanged so that a fragment read is free of bank conflicts.  The work is dealt so that an XCD walks
+//     consecutive tiles with all their W blocks: its L2 sees a tile's rows and an expert's weights once.
 #include "moe.h"
 
 namespace lvllm {
@@ -19,13 +21,12 @@ __device__ __forceinline__ e_f32x4_t moe_mfma(e_u32x4_t a, e_u32x4_t b, e_f32x4_
                                                  0);
 }
 
-constexpr int kStreamMaxRows = 64, kStreamMaxK = 4096, kStreamBatch = 8;
+constexpr int kStreamMaxRows = 64, kStreamBatch = 8, kStreamChunk = 64;  // rows of a step; k-steps per batch, per LDS chunk
 
-// grid (shares of the outputs, experts, groups of 16 slots)
+// grid (shares of the outputs, experts, groups of 16 slots); a wave computes W tiles 2 u and 2 u + 1
 template <bool UP>
 __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
-  extern __shared__ __attribute__((aligned(16))) char sx[];  // [K / 32][4][16][8]
-  constexpr int NW = UP ? 2 : 1;  // W tiles of a unit: gate and value
+  extern __shared__ __attribute__((aligned(16))) char sx[];  // [k-steps of a chunk][4][16][8]
   const int e = blockIdx.y;
   const int s0 = p.offsets[e] + 16 * blockIdx.z, s1 = min(p.offsets[e + 1], p.slots);
   if (s0 >= s1) return;
@@ -33,156 +34,169 @@ __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
   const int ff = p.ff[e], K = UP ? p.width : ff, steps = K >> 5;
-  const int units = UP ? ff >> 4 : p.width >> 4;
-  const uint16_t* w = (const uint16_t*)p.w + p.w_offset[e] + lane * 8;
-  e_u32x4_t a[2][NW][kStreamBatch];
-  auto fetch = [&](int u, int b, e_u32x4_t (&t)[NW][kStreamBatch]) __attribute__((always_inline)) {
+  const int units = UP ? ff >> 4 : p.width >> 5;
+  if ((int)blockIdx.x * 4 >= units) return;
+  const int u = min((int)blockIdx.x * 4 + wave, units - 1);  // (a wave too many repeats the last unit)
+  const uint16_t* w = (const uint16_t*)p.w + p.w_offset[e] + (int64_t)2 * u * steps * 512 + lane * 8;
+  e_u32x4_t a[2][2][kStreamBatch];
+  auto fetch = [&](int b, e_u32x4_t (&t)[2][kStreamBatch]) __attribute__((always_inline)) {
 #pragma unroll
     for (int j = 0; j < kStreamBatch; ++j)
 #pragma unroll
-      for (int i = 0; i < NW; ++i)
-        if (b + j < steps) t[i][j] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)(NW * u + i) * steps + b + j) * 512);
+      for (int i = 0; i < 2; ++i)
+        if (b + j < steps) t[i][j] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)i * steps + b + j) * 512);
   };
-  int u = blockIdx.x * 4 + wave;
-  if (u < units) fetch(u, 0, a[0]);
-  {
-    const int64_t ld = UP ? p.width : p.ff_max;
-    const int slot = s0 + (threadIdx.x & 15);
-    const int64_t row = slot >= s1 ? -1 : UP ? min(max(p.token[slot], 0), p.rows - 1) : slot;
-    const uint16_t* x = (const uint16_t*)p.x + (row < 0 ? 0 : row) * ld;
-    for (int i = threadIdx.x; i < K * 2; i += 256) {  // 16-byte chunk i: slot i % 16, entries 8 (i / 16) ..
+  fetch(0, a[0]);
+  const int64_t ld = UP ? p.width : p.ff_max;
+  const int my_slot = s0 + (threadIdx.x & 15);
+  const int64_t row = my_slot >= s1 ? -1 : UP ? min(max(p.token[my_slot], 0), p.rows - 1) : my_slot;
+  const uint16_t* x = (const uint16_t*)p.x + (row < 0 ? 0 : row) * ld;
+  auto stage = [&](int step0) __attribute__((always_inline)) {
+    const int n = min(kStreamChunk, steps - step0) * 64;
+    for (int i = threadIdx.x; i < n; i += 256) {  // 16-byte chunk i: slot i % 16, entries 8 (i / 16) ..
       e_u32x4_t v{0, 0, 0, 0};
-      if (row >= 0) v = *reinterpret_cast<const e_u32x4_t*>(x + (i >> 4) * 8);
+      if (row >= 0) v = *reinterpret_cast<const e_u32x4_t*>(x + step0 * 32 + (i >> 4) * 8);
       *reinterpret_cast<e_u32x4_t*>(sx + i * 16) = v;
     }
-  }
-  __syncthreads();
+    __syncthreads();
+  };
   const char* xf = sx + lane * 16;
-  for (; u < units; u += gridDim.x * 4) {
-    const int un = u + gridDim.x * 4;
-    e_f32x4_t acc[NW];
+  e_f32x4_t acc[2] = {e_f32x4_t{0.f, 0.f, 0.f, 0.f}, e_f32x4_t{0.f, 0.f, 0.f, 0.f}};
+  auto use = [&](int b, const e_u32x4_t (&t)[2][kStreamBatch]) __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < NW; ++i) acc[i] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
-    auto use = [&](int b, const e_u32x4_t (&t)[NW][kStreamBatch]) __attribute__((always_inline)) {
-#pragma unroll
-      for (int j = 0; j < kStreamBatch; ++j)
-        if (b + j < steps) {
-          const e_u32x4_t x = *reinterpret_cast<const e_u32x4_t*>(xf + (b + j) * 1024);
-#pragma unroll
-          for (int i = 0; i < NW; ++i) acc[i] = moe_mfma(t[i][j], x, acc[i]);
-        }
-    };
-    for (int b = 0; b < steps; b += 2 * kStreamBatch) {
-      const bool two = b + kStreamBatch < steps;
-      if (two) fetch(u, b + kStreamBatch, a[1]);
-      use(b, a[0]);
-      if (b + 2 * kStreamBatch < steps) fetch(u, b + 2 * kStreamBatch, a[0]);
-      else if (un < units) fetch(un, 0, a[0]);
-      if (two) use(b + kStreamBatch, a[1]);
+    for (int j = 0; j < kStreamBatch; ++j)
+      if (b + j < steps) {
+        const e_u32x4_t xv = *reinterpret_cast<const e_u32x4_t*>(xf + ((b + j) % kStreamChunk) * 1024);
+        acc[0] = moe_mfma(t[0][j], xv, acc[0]);
+        acc[1] = moe_mfma(t[1][j], xv, acc[1]);
+      }
+  };
+  stage(0);
+  for (int b = 0; b < steps; b += 2 * kStreamBatch) {
+    const bool two = b + kStreamBatch < steps;
+    if (two) fetch(b + kStreamBatch, a[1]);
+    if (b > 0 && b % kStreamChunk == 0) {
+      __syncthreads();
+      stage(b);
     }
-    const int slot = s0 + c;
-    if (slot >= s1) continue;
-    float v[4];
-    if constexpr (UP) {
-      const float limit = p.limit[e];
+    use(b, a[0]);
+    if (b + 2 * kStreamBatch < steps) fetch(b + 2 * kStreamBatch, a[0]);
+    if (two) use(b + kStreamBatch, a[1]);
+  }
+  const int slot = s0 + c;
+  if (slot >= s1) return;
+  float v[4];
+  if constexpr (UP) {
+    const float limit = p.limit[e];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) v[r] = clamped_gate(acc[0][r], acc[1][r], limit);
-      store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.ff_max + 16 * u + 4 * g, v);
-    } else {
+    for (int r = 0; r < 4; ++r) v[r] = clamped_gate(acc[0][r], acc[1][r], limit);
+    store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.ff_max + 16 * u + 4 * g, v);
+  } else {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) v[r] = acc[0][r];
-      store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.width + 16 * u + 4 * g, v);
+    for (int i = 0; i < 2; ++i) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[r] = acc[i][r];
+      store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.width + 32 * u + 16 * i + 4 * g, v);
     }
   }
 }
 
-// grid (blocks of 256 W rows, tiles of 128 slots)
+constexpr int kTileW = 16;                                 // W tiles of a workgroup
+constexpr int kStageBytes = (kTileW + kMoeTile / 16) * 1024;  // 32 of K: W tiles, then 16-slot groups
+constexpr int kStages = 3;
+
+__device__ __forceinline__ void to_lds(const uint16_t* src, char* dst) {  // 16 bytes a lane, 1 KiB a wave
+  __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
+                                   (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
+}
+
 template <bool UP>
-__global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p) {
-  constexpr int MT = kMoeTile / 16;
-  __shared__ __attribute__((aligned(16))) char sx[2][kMoeTile * 128];
-  const int e = p.tiles[2 * blockIdx.y];
+__global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, const int blocks_first, const int blocks_last) {
+  extern __shared__ __attribute__((aligned(16))) char ring[];  // [kStages][kStageBytes]
+  // the tiles of all experts but the last one, then the last one's (the shared expert may be larger): an eighth of each to
+  // every XCD
+  const int tiles_first = p.tiles[2 * p.max_tiles], tiles_all = p.tiles[2 * p.max_tiles + 1];
+  const int xcd = blockIdx.x & 7, turn = blockIdx.x >> 3;
+  const int all_first = tiles_first * blocks_first, all_last = (tiles_all - tiles_first) * blocks_last;
+  const int per_first = (all_first + 7) / 8, per_last = (all_last + 7) / 8;
+  int tile, block;
+  if (turn < per_first) {
+    const int i = xcd * per_first + turn;
+    if (i >= all_first) return;
+    tile = i / blocks_first;
+    block = i - tile * blocks_first;
+  } else {
+    const int t = turn - per_first, i = xcd * per_last + t;
+    if (t >= per_last || i >= all_last) return;
+    tile = i / blocks_last;
+    block = i - tile * blocks_last;
+    tile += tiles_first;
+  }
+  const int e = p.tiles[2 * tile];
   if (e < 0 || e >= p.experts) return;
-  const int s0 = p.tiles[2 * blockIdx.y + 1], s1 = min(min(p.offsets[e + 1], s0 + kMoeTile), p.slots);
-  const int ff = p.ff[e], K = UP ? p.width : ff, steps = K >> 5;
+  const int s0 = p.tiles[2 * tile + 1], s1 = min(min(p.offsets[e + 1], s0 + kMoeTile), p.slots);
+  const int ff = p.ff[e], steps = (UP ? p.width : ff) >> 5;
   const int ntiles = UP ? ff >> 3 : p.width >> 4;  // of 16 W rows
-  if ((int)blockIdx.x * 16 >= ntiles || s0 >= s1) return;
+  if (block * kTileW >= ntiles || s0 >= s1) return;
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
-  const int nt0 = blockIdx.x * 16 + wave * 4;
   const int64_t ld = UP ? p.width : p.ff_max;
-  // chunks this thread moves: row 32 i + tid / 8 of the tile, 16 bytes tid % 8 of its 128
-  const int q = threadIdx.x & 7, r0 = threadIdx.x >> 3;
-  const uint16_t* xrow[4];
-  char* xdst[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int r = 32 * i + r0, slot = min(s0 + r, s1 - 1);
-    const int64_t row = UP ? min(max(p.token[slot], 0), p.rows - 1) : slot;
-    xrow[i] = (const uint16_t*)p.x + row * ld + q * 8;
-    xdst[i] = sx[0] + r * 128 + ((q ^ (r & 7)) * 16);
-  }
+  // what this wave moves: W tiles 4 wave .. and 16-slot groups 2 wave ..; lane l of a group: slot l / 4, chunk l % 4 of it
+  // exchanged by the slot's number / 4
+  const uint16_t *wsrc[4], *xsrc[2];
   const uint16_t* w = (const uint16_t*)p.w + p.w_offset[e] + lane * 8;
-  e_u32x4_t xs[4], a[2][4][2];
-  const e_u32x4_t zero{0, 0, 0, 0};
-  auto fetch_x = [&](int s) __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      xs[i] = s * 32 + q * 8 < K ? *reinterpret_cast<const e_u32x4_t*>(xrow[i] + s * 32) : zero;
+  for (int j = 0; j < 4; ++j) wsrc[j] = w + (int64_t)min(block * kTileW + wave * 4 + j, ntiles - 1) * steps * 512;
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int slot = min(s0 + (wave * 2 + j) * 16 + (lane >> 2), s1 - 1);
+    const int64_t row = UP ? min(max(p.token[slot], 0), p.rows - 1) : slot;
+    xsrc[j] = (const uint16_t*)p.x + row * ld + ((lane & 3) ^ (lane >> 4)) * 8;
+  }
+  auto issue = [&](int k, char* st) __attribute__((always_inline)) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) to_lds(wsrc[j] + k * 512, st + (wave * 4 + j) * 1024);
+#pragma unroll
+    for (int j = 0; j < 2; ++j) to_lds(xsrc[j] + k * 32, st + (kTileW + wave * 2 + j) * 1024);
   };
-  auto put_x = [&](int stage) __attribute__((always_inline)) {
+  const int wn = wave & 1, wm = wave >> 1;
+  const int woff = wn * 8 * 1024 + lane * 16, xoff = (kTileW + wm * 4) * 1024 + c * 64 + ((g ^ (c >> 2)) * 16);
+  e_f32x4_t acc[8][4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) *reinterpret_cast<e_u32x4_t*>(xdst[i] + stage * kMoeTile * 128) = xs[i];
-  };
-  auto fetch_w = [&](int s, e_u32x4_t (&t)[4][2]) __attribute__((always_inline)) {
+  for (int n = 0; n < 8; ++n)
 #pragma unroll
-    for (int n = 0; n < 4; ++n)
+    for (int m = 0; m < 4; ++m) acc[n][m] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
+  issue(0, ring);
+  if (steps > 1) issue(1, ring + kStageBytes);
+  char *cur = ring, *nxt = ring + 2 * kStageBytes;
+  for (int k = 0; k < steps; ++k) {
+    // loads retire in order: with only the next stage's six outstanding, this one's have landed
+    if (k + 1 < steps) asm volatile("s_waitcnt vmcnt(6)" ::: "memory");
+    else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    asm volatile("s_barrier" ::: "memory");  // ... for every wave; and everyone is done with the stage that is filled next
+    if (k + 2 < steps) issue(k + 2, nxt);
+    e_u32x4_t x[4], a[8];
 #pragma unroll
-      for (int k = 0; k < 2; ++k)
-        t[n][k] = s + k < steps && nt0 + n < ntiles
-                      ? *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)(nt0 + n) * steps + s + k) * 512) : zero;
-  };
-  e_f32x4_t acc[4][MT];
+    for (int m = 0; m < 4; ++m) x[m] = *reinterpret_cast<const e_u32x4_t*>(cur + xoff + m * 1024);
 #pragma unroll
-  for (int n = 0; n < 4; ++n)
+    for (int n = 0; n < 8; ++n) a[n] = *reinterpret_cast<const e_u32x4_t*>(cur + woff + n * 1024);
+    __builtin_amdgcn_sched_barrier(0);  // (the reads first: they return while the first products run)
 #pragma unroll
-    for (int m = 0; m < MT; ++m) acc[n][m] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
-  auto use = [&](int stage, const e_u32x4_t (&t)[4][2]) __attribute__((always_inline)) {
-    const char* base = sx[stage] + c * 128;
+    for (int n = 0; n < 8; ++n)
 #pragma unroll
-    for (int k = 0; k < 2; ++k)
-#pragma unroll
-      for (int m = 0; m < MT; ++m) {
-        const e_u32x4_t x = *reinterpret_cast<const e_u32x4_t*>(base + m * 2048 + (((4 * k + g) ^ (c & 7)) * 16));
-#pragma unroll
-        for (int n = 0; n < 4; ++n) acc[n][m] = moe_mfma(t[n][k], x, acc[n][m]);
-      }
-  };
-  fetch_x(0);
-  fetch_w(0, a[0]);
-  put_x(0);
-  __syncthreads();
-  for (int s = 0; s < steps; s += 4) {  // two stages a turn
-    const bool second = s + 2 < steps;
-    if (second) { fetch_x(s + 2); fetch_w(s + 2, a[1]); }
-    use(0, a[0]);
-    if (second) put_x(1);
-    __syncthreads();
-    if (!second) break;
-    const bool third = s + 4 < steps;
-    if (third) { fetch_x(s + 4); fetch_w(s + 4, a[0]); }
-    use(1, a[1]);
-    if (third) put_x(0);
-    __syncthreads();
+      for (int m = 0; m < 4; ++m) acc[n][m] = moe_mfma(a[n], x[m], acc[n][m]);
+    cur = cur == ring + 2 * kStageBytes ? ring : cur + kStageBytes;
+    nxt = nxt == ring + 2 * kStageBytes ? ring : nxt + kStageBytes;
   }
   const float limit = UP ? p.limit[e] : 0.f;
+  const int nt0 = block * kTileW + wn * 8;
 #pragma unroll
-  for (int m = 0; m < MT; ++m) {
-    const int slot = s0 + 16 * m + c;
+  for (int m = 0; m < 4; ++m) {
+    const int slot = s0 + (wm * 4 + m) * 16 + c;
     if (slot >= s1) continue;
 #pragma unroll
-    for (int n = 0; n < 4; n += UP ? 2 : 1) {
+    for (int n = 0; n < 8; n += UP ? 2 : 1) {
       if (nt0 + n >= ntiles) continue;
       float v[4];
       if constexpr (UP) {
@@ -198,25 +212,92 @@ __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p) {
   }
 }
 
+// The router on packed weights (experts and the shared gate, up to a multiple of 16 rows): 16 rows of h a workgroup, its 8
+// waves take every eighth k-step, the logits meet in LDS in wave order, a wave chooses for two rows.
+__global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
+                                                             const uint16_t* __restrict__ h, const uint16_t* __restrict__ w,
+                                                             const float* __restrict__ bias, const int experts,
+                                                             const int shared, const int top, const int rows, const int width) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  e_f32x4_t* red = reinterpret_cast<e_f32x4_t*>(smem);      // [8 waves][4 tiles][64 lanes]
+  float* z = reinterpret_cast<float*>(smem + 8 * 4 * 1024);  // [16][ld]
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int g = lane >> 4, c = lane & 15;
+  const int steps = width >> 5, ntiles = (experts + shared + 15) >> 4, ld = ntiles * 16 + 1;
+  const int row0 = blockIdx.x * 16;
+  const uint16_t* x = h + (int64_t)min(row0 + c, rows - 1) * width + 8 * g;
+  for (int t0 = 0; t0 < ntiles; t0 += 4) {
+    e_f32x4_t acc[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
+    constexpr int B = 4;  // k-steps in flight
+    for (int k0 = wave; k0 < steps; k0 += 8 * B) {
+      e_u32x4_t xv[B], wv[B][4];
+#pragma unroll
+      for (int j = 0; j < B; ++j) {
+        const int k = min(k0 + 8 * j, steps - 1);
+        xv[j] = k0 + 8 * j < steps ? *reinterpret_cast<const e_u32x4_t*>(x + 32 * k) : e_u32x4_t{0, 0, 0, 0};
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          wv[j][i] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)min(t0 + i, ntiles - 1) * steps + k) * 512 + lane * 8);
+      }
+#pragma unroll
+      for (int j = 0; j < B; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[i] = moe_mfma(wv[j][i], xv[j], acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) red[(wave * 4 + i) * 64 + lane] = acc[i];
+    __syncthreads();
+    if (threadIdx.x < 256 && t0 + wave < ntiles) {  // wave i sums tile i
+      e_f32x4_t s = red[threadIdx.x];
+#pragma unroll
+      for (int v = 1; v < 8; ++v) s += red[v * 256 + threadIdx.x];
+      const int n = (t0 + wave) * 16 + 4 * g;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) z[c * ld + n + r] = s[r] + (n + r < experts ? bias[n + r] : 0.f);
+    }
+    __syncthreads();
+  }
+  const int n = top + shared;
+  for (int r = wave; r < 16 && row0 + r < rows; r += 8)
+    choose_experts(z + r * ld, experts, top, shared != 0, ids + (int64_t)(row0 + r) * n, weights + (int64_t)(row0 + r) * n);
+}
+
+int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
+                          int top, int rows, int width, hipStream_t s) {
+  const int smem = 8 * 4 * 1024 + 16 * ((experts + shared + 15) / 16 * 16 + 1) * 4;
+  if (smem > 64 * 1024)
+    (void)hipFuncSetAttribute((const void*)moe_route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
+  hipLaunchKernelGGL(moe_route_mfma_kernel, dim3((rows + 15) / 16), dim3(512), smem, s, ids, weights, (const uint16_t*)h,
+                     (const uint16_t*)w, bias, experts, shared, top, rows, width);
+  LV_LAUNCH_CHECK();
+  return 0;
+}
+
 bool moe_takes_mfma(int width, int dtype) { return dtype == LVLLM_BF16 && width % 32 == 0; }
 
 template <bool UP>
 static void go(const MoeParams& p, hipStream_t s) {
-  const int K = UP ? p.width : p.ff_max, n = UP ? p.ff_max : p.width;  // of the largest expert
-  if (p.rows <= kStreamMaxRows && K <= kStreamMaxK) {
-    const int smem = K * 32;
-    if (smem > 64 * 1024)
-      (void)hipFuncSetAttribute((const void*)moe_stream_kernel<UP>, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
-    const int units = n / 16;
-    int shares = (units + 3) / 4;
-    hipLaunchKernelGGL((moe_stream_kernel<UP>), dim3(shares, p.experts, (p.rows + 15) / 16), dim3(256), smem, s, p);
+  if (p.rows <= kStreamMaxRows) {
+    const int steps = (UP ? p.width : p.ff_max) / 32, units = UP ? p.ff_max / 16 : p.width / 32;  // of the largest expert
+    const int smem = (steps < kStreamChunk ? steps : kStreamChunk) * 1024;
+    hipLaunchKernelGGL((moe_stream_kernel<UP>), dim3((units + 3) / 4, p.experts, (p.rows + 15) / 16), dim3(256), smem, s, p);
   } else {
-    hipLaunchKernelGGL((moe_tile_kernel<UP>), dim3((n * (UP ? 2 : 1) + 255) / 256, p.max_tiles), dim3(256), 0, s, p);
+    constexpr int smem = kStages * kStageBytes;
+    (void)hipFuncSetAttribute((const void*)moe_tile_kernel<UP>, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
+    auto blocks = [&](int ff) { return ((UP ? ff / 8 : p.width / 16) + kTileW - 1) / kTileW; };
+    const int first = blocks(p.ff_first), last = blocks(p.ff_last);
+    const int64_t last_tiles = (p.rows + kMoeTile - 1) / kMoeTile;  // a token takes an expert once
+    const int64_t wgs = 8 * (((int64_t)p.max_tiles * first + 7) / 8 + (last_tiles * last + 7) / 8);
+    hipLaunchKernelGGL((moe_tile_kernel<UP>), dim3((unsigned)wgs), dim3(256), smem, s, p, first, last);
   }
 }
 
 int launch_moe_mfma(const MoeParams& p, bool up, hipStream_t s) {
-  LV_CHECK(p.experts <= 65535 && p.max_tiles <= 65535, "too many experts or tiles");
+  LV_CHECK(p.experts <= 65535 && p.ff_first > 0 && p.ff_last > 0 && p.ff_first <= p.ff_max && p.ff_last <= p.ff_max,
+           "sizes of the experts");
   if (up) go<true>(p, s);
   else go<false>(p, s);
   LV_LAUNCH_CHECK();

@@ -4,11 +4,11 @@
 
 namespace {
 
-void check_rot(const torch::Tensor& positions, const torch::Tensor& inv_freq, int64_t rows, const char* op) {
+void check_rot(const torch::Tensor& positions, const torch::Tensor& turns, int64_t rows, const char* op) {
   TORCH_CHECK(positions.is_cuda() && positions.scalar_type() == at::kLong && positions.is_contiguous() &&
-                  positions.numel() >= rows && inv_freq.is_cuda() && inv_freq.scalar_type() == at::kDouble &&
-                  inv_freq.is_contiguous(),
-              op, ": positions int64 [rows] and inv_freq float64 [rot_dims / 2] on the device");
+                  positions.numel() >= rows && turns.is_cuda() && turns.scalar_type() == at::kDouble &&
+                  turns.is_contiguous(),
+              op, ": positions int64 [rows] and turns float64 [rot_dims / 2] on the device");
 }
 void check_latent_rows(const torch::Tensor& cache, int64_t cpad, int64_t rpad, const char* op) {
   TORCH_CHECK(cache.is_cuda() && cache.dim() == 3 && cache.size(2) == cpad + rpad && blocks_are_dense(cache), op,
@@ -30,7 +30,7 @@ void check_tables(const torch::Tensor& block_tables, int64_t num_seqs, const cha
 }
 
 void latent_cache(torch::Tensor& cache, const torch::Tensor& kv, const torch::Tensor& weight, double eps, int64_t cpad,
-                  const torch::Tensor& positions, const torch::Tensor& inv_freq, const torch::Tensor& slot_mapping) {
+                  const torch::Tensor& positions, const torch::Tensor& turns, const torch::Tensor& slot_mapping) {
   const char* op = "latent_cache";
   LV_CHECK_DEVICE(kv);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(kv));
@@ -38,82 +38,80 @@ void latent_cache(torch::Tensor& cache, const torch::Tensor& kv, const torch::Te
   check_latent_rows(cache, cpad, rpad, op);
   check_rows2d(kv, rows, kv.size(1), cache.scalar_type(), op, "kv");
   check_f32(weight, rank, op, "weight");
-  check_rot(positions, inv_freq, rows, op);
+  check_rot(positions, turns, rows, op);
   TORCH_CHECK(kv.size(1) >= rank && slot_mapping.is_cuda() && slot_mapping.scalar_type() == at::kLong &&
                   slot_mapping.is_contiguous() && slot_mapping.numel() >= rows,
               op, ": slot_mapping int64 [rows]");
   check(lvllm_latent_cache(cache.data_ptr(), cache.stride(0), cache.size(0), (int)cache.size(1), (int)cpad, (int)rpad,
                            kv.data_ptr(), kv.stride(0), (int)rank, (int)(kv.size(1) - rank), weight.data_ptr<float>(),
-                           (float)eps, positions.data_ptr<int64_t>(), inv_freq.data_ptr<double>(), (int)inv_freq.numel() * 2,
+                           (float)eps, positions.data_ptr<int64_t>(), turns.data_ptr<double>(), (int)turns.numel() * 2,
                            slot_mapping.data_ptr<int64_t>(), (int)rows, dtype_code(kv, op), current_stream(kv)));
 }
 
-torch::Tensor latent_query(const torch::Tensor& q, const torch::Tensor& uk_t, int64_t dim, int64_t rpad,
-                           const torch::Tensor& positions, const torch::Tensor& inv_freq,
-                           const torch::Tensor& query_start_loc, int64_t absorbed_max) {
+// kv, weight, slot_mapping: the rows' own latents, written to the cache by the same launch
+torch::Tensor latent_query(const torch::Tensor& q, const torch::Tensor& uk_t, int64_t dim, const torch::Tensor& positions,
+                           const torch::Tensor& turns, const torch::Tensor& query_start_loc, int64_t absorbed_max,
+                           torch::Tensor& cache, const std::optional<torch::Tensor>& kv,
+                           const std::optional<torch::Tensor>& weight, double eps, const torch::Tensor& slot_mapping) {
   const char* op = "latent_query";
   LV_CHECK_DEVICE(q);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
-  TORCH_CHECK(uk_t.is_cuda() && uk_t.dim() == 3 && uk_t.is_contiguous() && uk_t.scalar_type() == q.scalar_type(), op,
-              ": uk_t [heads, cpad, dpad]");
-  const int64_t rows = q.size(0), heads = uk_t.size(0), cpad = uk_t.size(1);
+  TORCH_CHECK(uk_t.is_cuda() && uk_t.dim() == 3 && uk_t.is_contiguous() && uk_t.scalar_type() == q.scalar_type() &&
+                  cache.scalar_type() == q.scalar_type(),
+              op, ": uk_t [heads, cpad, dpad]");
+  const int64_t rows = q.size(0), heads = uk_t.size(0), cpad = uk_t.size(1), rpad = cache.size(2) - cpad;
+  check_latent_rows(cache, cpad, rpad, op);
   TORCH_CHECK(q.dim() == 2 && q.size(1) % heads == 0 && q.size(1) / heads >= dim, op, ": q [rows, heads * (dim + rot_dim)]");
   check_rows2d(q, rows, q.size(1), q.scalar_type(), op, "q");
-  check_rot(positions, inv_freq, rows, op);
+  check_rot(positions, turns, rows, op);
   check_i32(query_start_loc, 1, op, "query_start_loc");
+  const int64_t rot_dim = q.size(1) / heads - dim;
+  if (kv) {
+    TORCH_CHECK(weight.has_value(), op, ": kv needs its norm's weight");
+    check_rows2d(*kv, rows, weight->numel() + rot_dim, q.scalar_type(), op, "kv");
+    check_f32(*weight, weight->numel(), op, "weight");
+    TORCH_CHECK(slot_mapping.is_cuda() && slot_mapping.scalar_type() == at::kLong && slot_mapping.is_contiguous() &&
+                    slot_mapping.numel() >= rows,
+                op, ": slot_mapping int64 [rows]");
+  }
   auto out = torch::empty({rows, heads, cpad + rpad}, q.options());
   check(lvllm_latent_query(out.data_ptr(), q.data_ptr(), q.stride(0), uk_t.data_ptr(), (int)heads, (int)dim,
-                           (int)uk_t.size(2), (int)cpad, (int)rpad, (int)(q.size(1) / heads - dim),
-                           (int)inv_freq.numel() * 2, positions.data_ptr<int64_t>(), inv_freq.data_ptr<double>(),
-                           query_start_loc.data_ptr<int>(), (int)query_start_loc.numel() - 1, (int)absorbed_max, (int)rows,
-                           dtype_code(q, op), current_stream(q)));
+                           (int)uk_t.size(2), (int)cpad, (int)rpad, (int)rot_dim, (int)turns.numel() * 2,
+                           positions.data_ptr<int64_t>(), turns.data_ptr<double>(), query_start_loc.data_ptr<int>(),
+                           (int)query_start_loc.numel() - 1, (int)absorbed_max, cache.data_ptr(), cache.stride(0),
+                           cache.size(0), (int)cache.size(1), kv ? kv->data_ptr() : nullptr, kv ? kv->stride(0) : 0,
+                           kv ? (int)weight->numel() : 0, kv ? weight->data_ptr<float>() : nullptr, (float)eps,
+                           slot_mapping.data_ptr<int64_t>(), (int)rows, dtype_code(q, op), current_stream(q)));
   return out;
 }
 
-torch::Tensor latent_attention(const torch::Tensor& q, const torch::Tensor& cache, int64_t cpad,
-                               const torch::Tensor& block_tables, const torch::Tensor& seq_lens,
-                               const torch::Tensor& query_start_loc, double scale, int64_t window, int64_t absorbed_max,
-                               int64_t max_query_len, int64_t max_seq_len) {
+void latent_attention(torch::Tensor& out, const torch::Tensor& q, const torch::Tensor& cache, const torch::Tensor& uv,
+                      const std::optional<torch::Tensor>& gate, int64_t vdim, const torch::Tensor& block_tables,
+                      const torch::Tensor& seq_lens, const torch::Tensor& query_start_loc, double scale, int64_t window,
+                      int64_t absorbed_max, int64_t max_query_len, int64_t max_seq_len) {
   const char* op = "latent_attention";
   LV_CHECK_DEVICE(q);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.scalar_type() == cache.scalar_type(), op, ": contiguous q [rows, heads, row]");
-  const int64_t rows = q.size(0), heads = q.size(1), rpad = q.size(2) - cpad;
+  const int64_t rows = q.size(0), heads = q.size(1);
+  TORCH_CHECK(uv.is_cuda() && uv.dim() == 3 && uv.is_contiguous() && uv.size(0) == heads && uv.scalar_type() == q.scalar_type(), op,
+              ": uv [heads, vpad, cpad]");
+  const int64_t cpad = uv.size(2), rpad = q.size(2) - cpad;
   check_latent_rows(cache, cpad, rpad, op);
   check_layout(query_start_loc, seq_lens, op);
   check_tables(block_tables, seq_lens.numel(), op);
+  check_rows2d(out, rows, heads * vdim, q.scalar_type(), op, "out");
+  if (gate) check_rows2d(*gate, rows, heads, q.scalar_type(), op, "gate");
   const int ns = (int)seq_lens.numel(), code = dtype_code(q, op), bs = (int)cache.size(1);
   const int64_t need = lvllm_latent_attention_workspace_bytes((int)rows, ns, (int)heads, (int)cpad, (int)rpad, bs, (int)window,
                                                               (int)absorbed_max, (int)max_query_len, (int)max_seq_len, code);
-  torch::Tensor ws;
-  if (need > 0) ws = torch::empty({need}, q.options().dtype(at::kByte));
-  auto out = torch::empty({rows, heads, cpad}, q.options());
-  check(lvllm_latent_attention(out.data_ptr(), q.data_ptr(), cache.data_ptr(), cache.stride(0), cache.size(0), bs, (int)cpad,
-                               (int)rpad, block_tables.data_ptr<int>(), (int)block_tables.size(1), seq_lens.data_ptr<int>(),
-                               query_start_loc.data_ptr<int>(), ns, (int)rows, (int)heads, (float)scale, (int)window,
-                               (int)absorbed_max, (int)max_query_len, (int)max_seq_len, need > 0 ? ws.data_ptr() : nullptr,
-                               need, code, current_stream(q)));
-  return out;
-}
-
-void latent_value(torch::Tensor& out, const torch::Tensor& o_lat, const torch::Tensor& uv,
-                  const std::optional<torch::Tensor>& gate, int64_t vdim, const torch::Tensor& query_start_loc,
-                  int64_t absorbed_max) {
-  const char* op = "latent_value";
-  LV_CHECK_DEVICE(o_lat);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(o_lat));
-  TORCH_CHECK(o_lat.dim() == 3 && o_lat.is_contiguous(), op, ": contiguous o_lat [rows, heads, cpad]");
-  const int64_t rows = o_lat.size(0), heads = o_lat.size(1), cpad = o_lat.size(2);
-  TORCH_CHECK(uv.is_cuda() && uv.dim() == 3 && uv.is_contiguous() && uv.size(0) == heads && uv.size(2) == cpad &&
-                  uv.scalar_type() == o_lat.scalar_type(),
-              op, ": uv [heads, vpad, cpad]");
-  check_rows2d(out, rows, heads * vdim, o_lat.scalar_type(), op, "out");
-  if (gate) check_rows2d(*gate, rows, heads, o_lat.scalar_type(), op, "gate");
-  check_i32(query_start_loc, 1, op, "query_start_loc");
-  check(lvllm_latent_value(out.data_ptr(), out.stride(0), o_lat.data_ptr(), uv.data_ptr(), gate ? gate->data_ptr() : nullptr,
-                           gate ? gate->stride(0) : 0, (int)heads, (int)vdim, (int)uv.size(1), (int)cpad,
-                           query_start_loc.data_ptr<int>(), (int)query_start_loc.numel() - 1, (int)absorbed_max, (int)rows,
-                           dtype_code(o_lat, op), current_stream(o_lat)));
+  auto ws = torch::empty({need}, q.options().dtype(at::kByte));
+  check(lvllm_latent_attention(out.data_ptr(), out.stride(0), q.data_ptr(), cache.data_ptr(), cache.stride(0), cache.size(0), bs,
+                               (int)cpad, (int)rpad, uv.data_ptr(), (int)vdim, (int)uv.size(1),
+                               gate ? gate->data_ptr() : nullptr, gate ? gate->stride(0) : 0, block_tables.data_ptr<int>(),
+                               (int)block_tables.size(1), seq_lens.data_ptr<int>(), query_start_loc.data_ptr<int>(), ns,
+                               (int)rows, (int)heads, (float)scale, (int)window, (int)absorbed_max, (int)max_query_len,
+                               (int)max_seq_len, ws.data_ptr(), need, code, current_stream(q)));
 }
 
 torch::Tensor latent_gather(const torch::Tensor& cache, const torch::Tensor& starts, const torch::Tensor& first,
@@ -155,36 +153,38 @@ std::tuple<torch::Tensor, torch::Tensor> latent_expand(const torch::Tensor& kv, 
 }
 
 torch::Tensor latent_rotate_query(const torch::Tensor& q, int64_t heads, int64_t dim, int64_t kpad,
-                                  const torch::Tensor& positions, const torch::Tensor& inv_freq) {
+                                  const torch::Tensor& positions, const torch::Tensor& turns) {
   const char* op = "latent_rotate_query";
   LV_CHECK_DEVICE(q);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
   const int64_t rows = q.size(0);
   TORCH_CHECK(heads > 0 && q.dim() == 2 && q.size(1) % heads == 0 && q.size(1) / heads >= dim, op, ": q [rows, heads * (dim + rot_dim)]");
   check_rows2d(q, rows, q.size(1), q.scalar_type(), op, "q");
-  check_rot(positions, inv_freq, rows, op);
+  check_rot(positions, turns, rows, op);
   auto out = torch::empty({rows, heads, kpad}, q.options());
   check(lvllm_latent_rotate_query(out.data_ptr(), q.data_ptr(), q.stride(0), (int)heads, (int)dim,
                                   (int)(q.size(1) / heads - dim), (int)kpad, positions.data_ptr<int64_t>(),
-                                  inv_freq.data_ptr<double>(), (int)inv_freq.numel() * 2, (int)rows, dtype_code(q, op),
+                                  turns.data_ptr<double>(), (int)turns.numel() * 2, (int)rows, dtype_code(q, op),
                                   current_stream(q)));
   return out;
 }
 
 std::tuple<torch::Tensor, torch::Tensor> moe_route(const torch::Tensor& h, const torch::Tensor& w, const torch::Tensor& bias,
-                                                   int64_t top) {
+                                                   int64_t top, bool shared, bool packed) {
   const char* op = "moe_route";
   LV_CHECK_DEVICE(h);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(h));
-  const int64_t rows = h.size(0), width = h.size(1), experts = bias.numel(), shared = w.size(0) - experts;
+  const int64_t rows = h.size(0), width = h.size(1), experts = bias.numel();
   TORCH_CHECK(h.dim() == 2 && h.is_contiguous() && w.is_cuda() && w.dim() == 2 && w.is_contiguous() && w.size(1) == width &&
-                  w.scalar_type() == h.scalar_type() && (shared == 0 || shared == 1),
-              op, ": h [rows, width], w [experts (+ 1), width]");
+                  w.scalar_type() == h.scalar_type() &&
+                  w.size(0) == (packed ? (experts + shared + 15) / 16 * 16 : experts + shared),
+              op, ": h [rows, width], w [experts (+ 1), width], packed: rows up to a multiple of 16");
   check_f32(bias, experts, op, "bias");
   auto ids = torch::empty({rows, top + shared}, h.options().dtype(at::kInt));
   auto weights = torch::empty({rows, top + shared}, h.options().dtype(at::kFloat));
   check(lvllm_moe_route(ids.data_ptr<int>(), weights.data_ptr<float>(), h.data_ptr(), w.data_ptr(), bias.data_ptr<float>(),
-                        (int)experts, (int)shared, (int)top, (int)rows, (int)width, dtype_code(h, op), current_stream(h)));
+                        (int)experts, (int)shared, (int)top, (int)rows, (int)width, packed, dtype_code(h, op),
+                        current_stream(h)));
   return {ids, weights};
 }
 
@@ -197,7 +197,7 @@ std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_group
   const int64_t total = ids.numel(), tile = lvllm_moe_tile(packed);
   const int64_t max_tiles = std::min(total, total / tile + experts);
   auto offsets = torch::empty({experts + 1}, ids.options()), token = torch::empty({total}, ids.options());
-  auto slot = torch::empty_like(ids), tiles = torch::empty({max_tiles, 2}, ids.options());
+  auto slot = torch::empty_like(ids), tiles = torch::empty({max_tiles + 1, 2}, ids.options());
   check(lvllm_moe_group(offsets.data_ptr<int>(), token.data_ptr<int>(), slot.data_ptr<int>(), tiles.data_ptr<int>(),
                         ids.data_ptr<int>(), (int)total, (int)ids.size(1), (int)experts, packed, (int)max_tiles,
                         current_stream(ids)));
@@ -207,7 +207,7 @@ std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_group
 torch::Tensor moe_experts(const torch::Tensor& x, const torch::Tensor& w, const torch::Tensor& w_offset,
                           const torch::Tensor& ff, const torch::Tensor& limit, const torch::Tensor& offsets,
                           const torch::Tensor& token, const torch::Tensor& tiles, int64_t rows, int64_t width, int64_t ff_max,
-                          bool up, bool packed) {
+                          int64_t ff_first, int64_t ff_last, bool up, bool packed) {
   const char* op = "moe_experts";
   LV_CHECK_DEVICE(x);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
@@ -221,11 +221,12 @@ torch::Tensor moe_experts(const torch::Tensor& x, const torch::Tensor& w, const 
   check_f32(limit, experts, op, "limit");
   check_i32(offsets, experts + 1, op, "offsets");
   check_i32(token, slots, op, "token");
-  check_i32(tiles, 2, op, "tiles");
+  check_i32(tiles, 4, op, "tiles");
   auto out = torch::empty({slots, up ? ff_max : width}, x.options());
   check(lvllm_moe_experts(out.data_ptr(), x.data_ptr(), w.data_ptr(), w_offset.data_ptr<int64_t>(), ff.data_ptr<int>(),
                           limit.data_ptr<float>(), offsets.data_ptr<int>(), token.data_ptr<int>(), tiles.data_ptr<int>(),
-                          (int)experts, (int)slots, (int)rows, (int)width, (int)ff_max, (int)tiles.size(0), up, packed,
+                          (int)experts, (int)slots, (int)rows, (int)width, (int)ff_max, (int)ff_first, (int)ff_last,
+                          (int)tiles.size(0) - 1, up, packed,
                           dtype_code(x, op), current_stream(x)));
   return out;
 }
@@ -300,31 +301,30 @@ torch::Tensor norm_add_mix(const std::optional<torch::Tensor>& x_out, const std:
 }  // namespace
 
 TORCH_LIBRARY_FRAGMENT(_C_amd, latent) {
-  latent.def("latent_cache(Tensor(a!) cache, Tensor kv, Tensor weight, float eps, int cpad, Tensor positions, Tensor inv_freq, "
+  latent.def("latent_cache(Tensor(a!) cache, Tensor kv, Tensor weight, float eps, int cpad, Tensor positions, Tensor turns, "
              "Tensor slot_mapping) -> ()");
   latent.impl("latent_cache", torch::kCUDA, &latent_cache);
-  latent.def("latent_query(Tensor q, Tensor uk_t, int dim, int rpad, Tensor positions, Tensor inv_freq, "
-             "Tensor query_start_loc, int absorbed_max) -> Tensor");
+  latent.def("latent_query(Tensor q, Tensor uk_t, int dim, Tensor positions, Tensor turns, Tensor query_start_loc, "
+             "int absorbed_max, Tensor(a!) cache, Tensor? kv, Tensor? weight, float eps, Tensor slot_mapping) -> Tensor");
   latent.impl("latent_query", torch::kCUDA, &latent_query);
-  latent.def("latent_attention(Tensor q, Tensor cache, int cpad, Tensor block_tables, Tensor seq_lens, "
-             "Tensor query_start_loc, float scale, int window, int absorbed_max, int max_query_len, int max_seq_len) -> Tensor");
+  latent.def("latent_attention(Tensor(a!) out, Tensor q, Tensor cache, Tensor uv, Tensor? gate, int vdim, Tensor block_tables, "
+             "Tensor seq_lens, Tensor query_start_loc, float scale, int window, int absorbed_max, int max_query_len, "
+             "int max_seq_len) -> ()");
   latent.impl("latent_attention", torch::kCUDA, &latent_attention);
-  latent.def("latent_value(Tensor(a!) out, Tensor o_lat, Tensor uv, Tensor? gate, int vdim, Tensor query_start_loc, "
-             "int absorbed_max) -> ()");
-  latent.impl("latent_value", torch::kCUDA, &latent_value);
   latent.def("latent_gather(Tensor cache, Tensor starts, Tensor first, Tensor seq_lens, Tensor block_tables, int n) -> Tensor");
   latent.impl("latent_gather", torch::kCUDA, &latent_gather);
   latent.def("latent_expand(Tensor kv, Tensor rows, int cpad, int heads, int dim, int rot_dim, int vdim, int kpad, int vpad) "
              "-> (Tensor, Tensor)");
   latent.impl("latent_expand", torch::kCUDA, &latent_expand);
-  latent.def("latent_rotate_query(Tensor q, int heads, int dim, int kpad, Tensor positions, Tensor inv_freq) -> Tensor");
+  latent.def("latent_rotate_query(Tensor q, int heads, int dim, int kpad, Tensor positions, Tensor turns) -> Tensor");
   latent.impl("latent_rotate_query", torch::kCUDA, &latent_rotate_query);
-  latent.def("moe_route(Tensor h, Tensor w, Tensor bias, int top) -> (Tensor, Tensor)");
+  latent.def("moe_route(Tensor h, Tensor w, Tensor bias, int top, bool shared, bool packed) -> (Tensor, Tensor)");
   latent.impl("moe_route", torch::kCUDA, &moe_route);
   latent.def("moe_group(Tensor ids, int experts, bool packed) -> (Tensor, Tensor, Tensor, Tensor)");
   latent.impl("moe_group", torch::kCUDA, &moe_group);
   latent.def("moe_experts(Tensor x, Tensor w, Tensor w_offset, Tensor ff, Tensor limit, Tensor offsets, Tensor token, "
-             "Tensor tiles, int rows, int width, int ff_max, bool up, bool packed) -> Tensor");
+             "Tensor tiles, int rows, int width, int ff_max, int ff_first, int ff_last, bool up, bool packed) "
+             "-> Tensor");
   latent.impl("moe_experts", torch::kCUDA, &moe_experts);
   latent.def("embed_scale(Tensor(a!) x, Tensor table, Tensor ids, float scale) -> Tensor");
   latent.impl("embed_scale", torch::kCUDA, &embed_scale);

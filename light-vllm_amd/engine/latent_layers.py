@@ -42,11 +42,11 @@ class OutputNorm:
 
 
 class Rotation:
-    """Frequencies in double: angles are taken in double and reduced before the fp32 sine and cosine."""
+    """Full turns per position of every pair, in double: angles are reduced in double before the fp32 sine and cosine."""
 
     def __init__(self, cfg: RotationConfig, device):
         i = torch.arange(0, cfg.dims, 2, dtype=torch.float64, device=device)
-        self.inv_freq = float(cfg.base) ** (-i / max(cfg.dims, 1))
+        self.turns = float(cfg.base) ** (-i / max(cfg.dims, 1)) / (2 * np.pi)
 
 
 @dataclass
@@ -139,22 +139,23 @@ class LatentAttention:
 
     def __call__(self, h: torch.Tensor, kv: torch.Tensor, layer: int, step: LatentStep, attn) -> SublayerOutput:
         """`kv`: the cache of layer number `layer`, this one's own or the one it reads."""
-        c, l, spec, inv_freq = self.cfg, step.layout, self.spec, self.rotation.inv_freq
+        c, l, spec, turns = self.cfg, step.layout, self.spec, self.rotation.turns
         proj = linear(h, self.proj)
         q, gate, *dkv = (proj[:, o:o + n] for o, n in zip(self.at, self.sizes))
         cache = attn.rows_view(kv, spec, l.block_size)
-        if dkv:
-            amd.latent_cache(cache, dkv[0], self.norm, self.eps, spec.cpad, l.positions, inv_freq, l.slot_mapping)
         rows = h.shape[0]
         heads_out = (torch.empty if self.out.K == self.out_cols else torch.zeros)(rows, self.out.K, dtype=h.dtype, device=h.device)
         out = heads_out[:, :self.out_cols]
         plan = step.long_portions(c.window) if self.expands and l.block_size == 16 else None
-        longest = ABSORBED_MAX if plan is not None else UNBOUNDED
+        if plan is not None and dkv:
+            amd.latent_cache(cache, dkv[0], self.norm, self.eps, spec.cpad, l.positions, turns, l.slot_mapping)
         if plan is None or min(l.query_lens) <= ABSORBED_MAX:
-            qa = amd.latent_query(q, self.uk_t, c.dim, spec.rpad, l.positions, inv_freq, l.query_start_loc, longest)
-            o = amd.latent_attention(qa, cache, spec.cpad, l.block_tables, l.seq_lens, l.query_start_loc, c.scale, c.window,
-                                     longest, l.max_query_len, l.max_seq_len)
-            amd.latent_value(out, o, self.uv, gate, c.vdim, l.query_start_loc, longest)
+            longest = ABSORBED_MAX if plan is not None else UNBOUNDED
+            own = (dkv[0], self.norm) if dkv and plan is None else (None, None)  # (written by the same launch)
+            qa = amd.latent_query(q, self.uk_t, c.dim, l.positions, turns, l.query_start_loc, longest, cache, *own, self.eps,
+                                  l.slot_mapping)
+            amd.latent_attention(out, qa, cache, self.uv, gate, c.vdim, l.block_tables, l.seq_lens, l.query_start_loc, c.scale,
+                                 c.window, longest, l.max_query_len, l.max_seq_len)
         if plan is not None:
             self._long(out, q, gate, cache, layer, plan, step)
         return SublayerOutput(project_to_residual(heads_out, self.out))
@@ -164,7 +165,7 @@ class LatentAttention:
         lat = step.gathered(layer, c.window, cache, plan)
         kv = F.linear(lat[:, :spec.cpad], self.expand)
         keys, values = amd.latent_expand(kv, lat, spec.cpad, c.heads, c.dim, c.rot_dim, c.vdim, p.kpad, p.vpad)
-        qr = amd.latent_rotate_query(q, c.heads, c.dim, p.kpad, l.positions, self.rotation.inv_freq)
+        qr = amd.latent_rotate_query(q, c.heads, c.dim, p.kpad, l.positions, self.rotation.turns)
         amd.head_attention(out, qr, keys, values, plan.tables, plan.seq_lens, l.query_start_loc, gate, c.vdim, c.scale, 1.0,
                            l.max_query_len, plan.max_seq_len, c.window, ABSORBED_MAX + 1)
 
@@ -189,11 +190,11 @@ class MixtureOfExperts:
             ff.append(cfg.shared.ff)
             limits.append(cfg.shared.limit)
             router = torch.cat([router, get(name + ".shared.sg")])
-        self.router = router.contiguous()
         self.width, dev = router.shape[1], router.device
         self.packed = pack and router.dtype == torch.bfloat16 and self.width % 32 == 0
+        self.router = amd.pack_weight(stack_rows([router])[0]) if self.packed else router.contiguous()
         ffp = [ceil_to(n, 32) for n in ff]
-        self.ff_max, self.experts = max(ffp), len(names)
+        self.ff_max, self.ff_first, self.ff_last, self.experts = max(ffp), max(ffp[:-1] or ffp), ffp[-1], len(names)
         up_at, down_at = ([0] + np.cumsum([k * n * self.width for n in ffp]).tolist() for k in (2, 1))
         self.up = torch.empty(up_at[-1], dtype=router.dtype, device=dev)
         self.down = torch.empty(down_at[-1], dtype=router.dtype, device=dev)
@@ -212,11 +213,10 @@ class MixtureOfExperts:
         return self.up.numel() + self.down.numel()
 
     def __call__(self, h: torch.Tensor) -> SublayerOutput:
-        ids, weights = amd.moe_route(h, self.router, self.bias, self.cfg.top)
+        ids, weights = amd.moe_route(h, self.router, self.bias, self.cfg.top, self.cfg.shared is not None, self.packed)
         offsets, token, slots, tiles = amd.moe_group(ids, self.experts, self.packed)
         rows = h.shape[0]
-        a = amd.moe_experts(h, self.up, self.up_at, self.ff, self.limits, offsets, token, tiles, rows, self.width, self.ff_max,
-                            True, self.packed)
-        y = amd.moe_experts(a, self.down, self.down_at, self.ff, self.limits, offsets, token, tiles, rows, self.width,
-                            self.ff_max, False, self.packed)
+        sizes = rows, self.width, self.ff_max, self.ff_first, self.ff_last
+        a = amd.moe_experts(h, self.up, self.up_at, self.ff, self.limits, offsets, token, tiles, *sizes, True, self.packed)
+        y = amd.moe_experts(a, self.down, self.down_at, self.ff, self.limits, offsets, token, tiles, *sizes, False, self.packed)
         return SublayerOutput(y, slots, weights)

@@ -224,7 +224,7 @@ def test_rotation_far_from_the_start(amd, dtype):
     from light_vllm_amd.engine.latent_layers import Rotation
     pos = [0, 1, 17, 4095, 131071, 1000003]
     heads, dim, rot, rank, dims, base = 3, 16, 24, 40, 20, 5e4
-    inv = Rotation(RotationConfig(dims, base), DEV).inv_freq
+    inv = Rotation(RotationConfig(dims, base), DEV).turns
     kv, q = rand(6, rank + rot, seed=1, dtype=dtype), rand(6, heads * (dim + rot), seed=2, dtype=dtype)
     cache = torch.zeros(2, 16, 96, dtype=dtype, device=DEV)
     p = torch.tensor(pos, device=DEV)
@@ -294,6 +294,10 @@ def F_pad(t, n):
     return torch.nn.functional.pad(t, (0, n - t.shape[-1]))
 
 
+def F_rows(t, n):
+    return torch.nn.functional.pad(t, (0, 0, 0, -t.shape[0] % n))
+
+
 # ---- mixture of experts ----
 def mixture_case(experts, top, width, ff, shared_ff, seed=0, bias=1.0):
     mlp = lc.moe(experts, top, ff, 1.3, shared_ff, 0.8)
@@ -333,14 +337,16 @@ def test_router(amd, dtype, experts, width):
     for rows in (1, 33, 200):
         h, w, b = rand(rows, width, seed=1, dtype=dtype), rand(experts + 1, width, seed=2, dtype=dtype), rand(experts, seed=3)
         z = h.double() @ w.double().T
+        packed = dtype == BF16 and width % 32 == 0
+        wd = amd.pack_weight(F_rows(w, 16).to(DEV)) if packed else w.to(DEV)
         for top in (1, 3, 5):
-            ids, weights = amd.moe_route(h.to(DEV), w.to(DEV), b.to(DEV), top)
+            ids, weights = amd.moe_route(h.to(DEV), wd, b.to(DEV), top, True, packed)
             want_ids, want_w = lepalorn.route(z[:, :experts] + b.double(), top)
             assert torch.equal(ids[:, :top].long().cpu(), want_ids) and (ids[:, top] == experts).all()
             close(weights[:, :top], want_w, 1e-5)
             close(weights[:, top], torch.sigmoid(z[:, experts]), 1e-5)
     # equal logits: the smaller numbers
-    ids, weights = amd.moe_route(torch.zeros(2, width, dtype=dtype, device=DEV), w.to(DEV), torch.zeros(experts, device=DEV), 4)
+    ids, weights = amd.moe_route(torch.zeros(2, width, dtype=dtype, device=DEV), wd, torch.zeros(experts, device=DEV), 4, True, packed)
     assert ids[:, :4].tolist() == [[0, 1, 2, 3]] * 2 and (weights == torch.tensor([0.25] * 4 + [0.5], device=DEV)).all()
 
 
