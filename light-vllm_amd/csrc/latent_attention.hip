@@ -26,10 +26,11 @@ __device__ __forceinline__ void write_latent_row(const LatentCacheParams& p, int
   using S = typename T::store_t;
   constexpr int X = 16 / sizeof(S);
   const int lane = threadIdx.x & 63;
-  const int64_t slot = p.slot_mapping[row];
-  if (slot < 0 || slot >= p.num_slots) return;
+  const int64_t wide = p.slot_mapping[row];
+  if (wide < 0 || wide >= p.num_slots) return;
+  const unsigned slot = (unsigned)wide, block = slot / (unsigned)p.block_size;
   const S* z = (const S*)p.kv + row * p.kv_stride;
-  S* out = (S*)p.cache + (slot / p.block_size) * p.block_stride + (slot % p.block_size) * (int64_t)(p.cpad + p.rpad);
+  S* out = (S*)p.cache + block * p.block_stride + (slot - block * p.block_size) * (int64_t)(p.cpad + p.rpad);
   const int64_t pos = p.positions[row];
   const bool vec = p.kv_rank % X == 0 && p.kv_rank <= 64 * X && ((uintptr_t)z & 15) == 0;
   float ss = 0.f;
@@ -136,8 +137,8 @@ __device__ __forceinline__ void project_tail(const HeadProjectParams& p, int row
 template <typename T>
 __device__ __forceinline__ bool beside_products(const HeadProjectParams& p, int row0, int head) {
   const bool last = p.tail > 0 && blockIdx.x == gridDim.x - 1;
-  if (last && head == 0 && p.cache.kv != nullptr)
-    for (int i = threadIdx.x >> 6; i < 16 && row0 + i < p.rows; i += 4) write_latent_row<T>(p.cache, row0 + i);
+  if (last && p.cache.kv != nullptr)  // (the tile's rows are dealt to the heads' workgroups)
+    for (int i = 4 * head + (threadIdx.x >> 6); i < 16 && row0 + i < p.rows; i += 4 * p.heads) write_latent_row<T>(p.cache, row0 + i);
   if (p.query_start_loc != nullptr &&
       tile_is_expanded(p.query_start_loc, p.num_seqs, row0, min(row0 + 15, p.rows - 1), p.absorbed_max))
     return true;
@@ -409,6 +410,7 @@ using namespace lvllm;
 static int cache_params(LatentCacheParams& p, void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad,
                         int rpad, const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
                         const int64_t* positions, const double* turns, int rot_dims, const int64_t* slot_mapping, int rows) {
+  LV_CHECK(num_blocks * block_size < ((int64_t)1 << 32), "too many slots");
   LV_CHECK(kv_rank > 0 && kv_rank <= cpad && cpad % 8 == 0 && rot_dim >= 0 && rot_dim <= rpad && rpad % 8 == 0 &&
                rot_dims <= rot_dim && rot_dims % 2 == 0, "latent sizes");
   p.cache = cache; p.block_stride = block_stride; p.num_slots = num_blocks * block_size; p.block_size = block_size;
@@ -444,7 +446,8 @@ extern "C" int lvllm_latent_query(void* out, const void* q, int64_t q_stride, co
   HeadProjectParams p{};
   p.y = out; p.y_stride = (int64_t)heads * (cpad + rpad); p.y_head = cpad + rpad; p.n = cpad; p.npad = cpad;
   p.x = q; p.x_stride = q_stride; p.x_head = dim + rot_dim; p.k = dim; p.kpad = dpad; p.w = uk_t;
-  p.rows = rows; p.heads = heads; p.query_start_loc = query_start_loc; p.num_seqs = num_seqs; p.absorbed_max = absorbed_max;
+  p.rows = rows; p.heads = heads; p.num_seqs = num_seqs; p.absorbed_max = absorbed_max;
+  p.query_start_loc = absorbed_max < rows ? query_start_loc : nullptr;  // (no portion can be longer)
   p.tail = rpad; p.rot_dim = rot_dim; p.rot_dims = rot_dims; p.positions = positions; p.turns = turns;
   if (kv != nullptr)
     if (int rc = cache_params(p.cache, cache, block_stride, num_blocks, block_size, cpad, rpad, kv, kv_stride, kv_rank, rot_dim,
@@ -518,7 +521,8 @@ extern "C" int lvllm_latent_attention(void* out, int64_t out_stride, const void*
   v.y = out; v.y_stride = out_stride; v.y_head = vdim; v.n = vdim; v.npad = vpad;
   v.x = workspace; v.x_stride = (int64_t)heads * cpad; v.x_head = cpad; v.k = cpad; v.kpad = cpad; v.w = uv;
   v.gate = gate; v.gate_stride = gate_stride;
-  v.rows = rows; v.heads = heads; v.query_start_loc = query_start_loc; v.num_seqs = num_seqs; v.absorbed_max = absorbed_max;
+  v.rows = rows; v.heads = heads; v.num_seqs = num_seqs; v.absorbed_max = absorbed_max;
+  v.query_start_loc = absorbed_max < rows ? query_start_loc : nullptr;  // (no portion can be longer)
   return head_project(v, dtype, s);
 }
 

@@ -188,74 +188,87 @@ __global__ __launch_bounds__(256 * CT, 1) void latent_attention_mfma_kernel(cons
 }
 
 // The shares of R rows of one head -> their weighted sum o in latent space (bf16, as W's product reads it) -> out = V_h o * gate.
-// grid (heads, rows / R); a wave adds the shares of R / 4 rows, then takes every fourth 16-row tile of V_h.
+// grid (heads, rows / R); 8 waves add the shares of R rows' halves, then take every eighth 16-row tile of V_h.
 template <int R>
-__global__ __launch_bounds__(256) void latent_value_kernel(const LatentAttnParams p) {
+__global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnParams p) {
   extern __shared__ __attribute__((aligned(16))) uint16_t so[];  // [R][cpad + 8]
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
   const int head = blockIdx.x, row0 = blockIdx.y * R, ld = p.cpad + 8;
-  constexpr int B = 8;  // k-steps in flight
+  constexpr int B = 16, S = 8;  // k-steps and shares in flight
   const int steps = p.cpad >> 5;
   const uint16_t* uv = (const uint16_t*)p.uv + ((int64_t)head * p.vpad + c) * p.cpad + 8 * g;
   m_u32x4_t w[B];
   auto fetch = [&](int n, int k0) __attribute__((always_inline)) {
 #pragma unroll
     for (int j = 0; j < B; ++j)
-      w[j] = *reinterpret_cast<const m_u32x4_t*>(uv + (int64_t)n * 16 * p.cpad + 32 * min(k0 + j, steps - 1));
+      if (k0 + j < steps) w[j] = *reinterpret_cast<const m_u32x4_t*>(uv + (int64_t)n * 16 * p.cpad + 32 * (k0 + j));
+  };
+  // steps of single tokens: row i is sequence i; else the row's sequence tells whether it is in latent space at all
+  const bool single = p.max_query_len == 1 && p.rows == p.num_seqs;
+  auto absorbed = [&](int row) {
+    if (single) return true;
+    const int seq = find_seq(p.query_start_loc, p.num_seqs, row);
+    return seq < p.num_seqs && p.query_start_loc[seq + 1] - p.query_start_loc[seq] <= p.absorbed_max;
   };
   if (wave * 16 < p.vpad) fetch(wave, 0);
-  for (int i = wave; i < R; i += 4) {
-    const int row = row0 + i;
-    const int seq = row < p.rows ? find_seq(p.query_start_loc, p.num_seqs, row) : p.num_seqs;
-    const bool ok = seq < p.num_seqs && p.query_start_loc[seq + 1] - p.query_start_loc[seq] <= p.absorbed_max;
-    if (!ok) {
-      for (int d = lane; d < p.cpad; d += 64) so[i * ld + d] = 0;
+  const int half = (p.cpad >> 1) >= 256 ? 2 : 1, part = p.cpad / half;  // (a lane takes 4 entries a turn)
+  for (int i = wave; i < R * half; i += 8) {
+    const int r = i / half, row = row0 + r, d0 = (i - r * half) * part;
+    if (row >= p.rows || !absorbed(row)) {
+      for (int d = d0 + lane; d < d0 + part; d += 64) so[r * ld + d] = 0;
       continue;
     }
     const int64_t at = ((int64_t)row * p.heads + head) * p.nsplit;
     const float ms = lane < p.nsplit ? p.part_ml[2 * (at + lane)] : -1e30f;
     const float ls = lane < p.nsplit ? p.part_ml[2 * (at + lane) + 1] : 0.f;
+    float4 t[S];
+    auto load = [&](int d, int s0) __attribute__((always_inline)) {
+#pragma unroll
+      for (int s = 0; s < S; ++s)
+        if (s0 + s < p.nsplit) t[s] = *reinterpret_cast<const float4*>(p.part_o + (at + s0 + s) * p.cpad + d);
+    };
+    int d = d0 + lane * 4;
+    if (d < d0 + part) load(d, 0);
     const float m = wave_max(ms);
     const float e = exp2f(ms - m), l = wave_sum(ls * e);
     const float ws = l > 0.f ? e / l : 0.f;
-    for (int d = lane * 4; d < p.cpad; d += 256) {
+    for (; d < d0 + part; d += 256) {
       float v[4] = {0.f, 0.f, 0.f, 0.f};
-      for (int s0 = 0; s0 < p.nsplit; s0 += 4) {
-        float4 t[4];
+      for (int s0 = 0; s0 < p.nsplit; s0 += S) {
+        if (s0 > 0 || d >= d0 + 256) load(d, s0);
 #pragma unroll
-        for (int s = 0; s < 4; ++s) t[s] = *reinterpret_cast<const float4*>(p.part_o + (at + min(s0 + s, p.nsplit - 1)) * p.cpad + d);
-#pragma unroll
-        for (int s = 0; s < 4; ++s) {
-          const float f = s0 + s < p.nsplit ? __shfl(ws, s0 + s) : 0.f;
-          v[0] = fmaf(t[s].x, f, v[0]); v[1] = fmaf(t[s].y, f, v[1]); v[2] = fmaf(t[s].z, f, v[2]); v[3] = fmaf(t[s].w, f, v[3]);
-        }
+        for (int s = 0; s < S; ++s)
+          if (s0 + s < p.nsplit) {
+            const float f = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, ws), s0 + s));
+            v[0] = fmaf(t[s].x, f, v[0]); v[1] = fmaf(t[s].y, f, v[1]); v[2] = fmaf(t[s].z, f, v[2]); v[3] = fmaf(t[s].w, f, v[3]);
+          }
       }
-      store4<BF16>(so + i * ld + d, v);
+      store4<BF16>(so + r * ld + d, v);
     }
   }
-  __syncthreads();
   const int row = row0 + c;
   bool mine = c < R && row < p.rows;
-  if (mine) {
-    const int seq = find_seq(p.query_start_loc, p.num_seqs, row);  // (padding rows get zeros)
-    mine = seq >= p.num_seqs || p.query_start_loc[seq + 1] - p.query_start_loc[seq] <= p.absorbed_max;
-  }
   float f = 1.f;
   if (mine && p.gate != nullptr)
     f = 1.f / (1.f + expf(-BF16::to_float(((const uint16_t*)p.gate)[row * p.gate_stride + head])));
-  for (int n = wave; n * 16 < p.vpad; n += 4) {
+  if (mine && !single) {
+    const int seq = find_seq(p.query_start_loc, p.num_seqs, row);  // (padding rows get zeros)
+    mine = seq >= p.num_seqs || p.query_start_loc[seq + 1] - p.query_start_loc[seq] <= p.absorbed_max;
+  }
+  __syncthreads();
+  for (int n = wave; n * 16 < p.vpad; n += 8) {
     m_f32x4_t acc{0.f, 0.f, 0.f, 0.f};
     for (int k0 = 0; k0 < steps; k0 += B) {
       if (n != wave || k0 > 0) fetch(n, k0);
 #pragma unroll
-      for (int j = 0; j < B; ++j) {
-        const int k = 32 * (k0 + j) + 8 * g;
-        m_u32x4_t x{0, 0, 0, 0};
-        if (k0 + j < steps && c < R) x = *reinterpret_cast<const m_u32x4_t*>(so + c * ld + k);
-        acc = mfma16(w[j], x, acc);
-      }
+      for (int j = 0; j < B; ++j)
+        if (k0 + j < steps) {
+          m_u32x4_t x{0, 0, 0, 0};
+          if (c < R) x = *reinterpret_cast<const m_u32x4_t*>(so + c * ld + 32 * (k0 + j) + 8 * g);
+          acc = mfma16(w[j], x, acc);
+        }
     }
     if (!mine) continue;
     uint16_t* out = (uint16_t*)p.out + row * p.out_stride + (int64_t)head * p.vdim + 16 * n + 4 * g;
@@ -303,9 +316,9 @@ int launch_latent_mfma(const LatentAttnParams& p, hipStream_t s) {
   LV_LAUNCH_CHECK();
   LV_CHECK((p.rows + 3) / 4 <= 65535, "too many rows");
   if (p.rows <= 256)
-    hipLaunchKernelGGL((latent_value_kernel<4>), dim3(p.heads, (p.rows + 3) / 4), dim3(256), 4 * (p.cpad + 8) * 2, s, p);
+    hipLaunchKernelGGL((latent_value_kernel<4>), dim3(p.heads, (p.rows + 3) / 4), dim3(512), 4 * (p.cpad + 8) * 2, s, p);
   else
-    hipLaunchKernelGGL((latent_value_kernel<16>), dim3(p.heads, (p.rows + 15) / 16), dim3(256), 16 * (p.cpad + 8) * 2, s, p);
+    hipLaunchKernelGGL((latent_value_kernel<16>), dim3(p.heads, (p.rows + 15) / 16), dim3(512), 16 * (p.cpad + 8) * 2, s, p);
   LV_LAUNCH_CHECK();
   return 0;
 }

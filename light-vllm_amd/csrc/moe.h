@@ -19,7 +19,9 @@ struct MoeParams {
   const int32_t *ff;      // [experts] ffp
   const float* limit;     // [experts]
   const int32_t *offsets, *token;
-  const int32_t* tiles;   // [max_tiles + 1][2]: expert, first slot (expert < 0: none); last: tiles of all but the last expert, of all
+  // [max_tiles + 1][4]: expert (< 0: none), first slot, the expert's first tile and its number of tiles; the last entry: tiles
+  // of all experts but the last one, tiles of all
+  const int32_t* tiles;
   int experts, slots, rows, width, ff_max, max_tiles;
   int ff_first, ff_last;  // largest ffp of all experts but the last, the last one's
 };
@@ -32,40 +34,36 @@ __device__ __forceinline__ float clamped_gate(float g, float u, float limit) {
 
 constexpr int kMaxExperts = 1024;
 
-// The `top` largest of z[0 .. experts) (LDS; ties: the smaller index) by one wave, their softmax, and the shared expert.
-// Any z gives indices in range.
-__device__ __forceinline__ void choose_experts(float* z, int experts, int top, bool shared, int32_t* ids, float* weights) {
+// The `top` largest of z[0 .. experts) (LDS; ties: the smaller index) by one wave, their softmax, and the shared expert.  Every
+// logit's place is the number of logits ahead of it; NaNs come last, so that any z gives distinct indices in range.
+__device__ __forceinline__ void choose_experts(const float* z, int experts, int top, bool shared, int32_t* ids, float* weights) {
   const int lane = threadIdx.x & 63;
-  float first = 0.f, sum = 0.f, mine = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float best = -INFINITY;
-    int at = kMaxExperts;
+  auto value = [&](int e) { return z[e] == z[e] ? z[e] : -INFINITY; };
+  float mx = -INFINITY;
+  for (int e = lane; e < experts; e += 64) mx = fmaxf(mx, value(e));
+  mx = wave_max(mx);
+  if (mx == -INFINITY) mx = 0.f;  // (nothing to compare)
+  float sum = 0.f;
+  for (int pass = 0; pass < 2; ++pass) {  // the chosen ones' sum, then their weights
     for (int e = lane; e < experts; e += 64) {
-      const float v = z[e];
-      if (v > best || (at == kMaxExperts && v == v && v != -INFINITY)) { best = v; at = e; }
+      const float v = value(e);
+      int place = 0;
+#pragma unroll 8
+      for (int j = 0; j < experts; ++j) {
+        const float o = value(j);
+        place += o > v || (o == v && j < e);
+      }
+      if (place >= top) continue;
+      const float w = v == -INFINITY ? 1e-30f : expf(v - mx);
+      if (pass == 0) {
+        sum += w;
+      } else {
+        ids[place] = e;
+        weights[place] = w / sum;
+      }
     }
-#pragma unroll
-    for (int m = 32; m >= 1; m >>= 1) {
-      const float ob = __shfl_xor(best, m);
-      const int oa = __shfl_xor(at, m);
-      if (oa < kMaxExperts && (at == kMaxExperts || ob > best || (ob == best && oa < at))) { best = ob; at = oa; }
-    }
-    if (at >= kMaxExperts) {  // nothing comparable left: the first one not taken (marked by -inf) or, among NaNs, the k-th
-      at = k;
-      best = first;
-    }
-    if (k == 0) first = best;
-    const float e = expf(best - first);
-    sum += e;
-    if (lane == k) mine = e;
-    if (lane == 0) {
-      ids[k] = at;
-      z[at] = -INFINITY;
-    }
-    __builtin_amdgcn_wave_barrier();
-    __threadfence_block();
+    if (pass == 0) sum = wave_sum(sum);
   }
-  if (lane < top) weights[lane] = mine / sum;
   if (shared && lane == 0) {
     ids[top] = experts;
     weights[top] = 1.f / (1.f + expf(-z[experts]));

@@ -35,13 +35,14 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int32_t* __restrict__ id
   if (threadIdx.x < 64) choose_experts(z, experts, top, shared != 0, ids + (int64_t)row * n, weights + (int64_t)row * n);
 }
 
-// Counts, offsets, slots and tiles of `total` assignments; one workgroup.
+// Counts, offsets, slots and tiles of `total` assignments; one workgroup.  `shared`: the last assignment of every row is the
+// last expert's, in row order.
 __global__ __launch_bounds__(1024) void moe_group_kernel(int32_t* __restrict__ offsets, int32_t* __restrict__ token,
                                                          int32_t* __restrict__ slot, int32_t* __restrict__ tiles,
                                                          const int32_t* __restrict__ ids, const int total, const int per_row,
-                                                         const int experts, const int tile, const int max_tiles) {
+                                                         const int experts, const int shared, const int tile, const int max_tiles) {
   __shared__ int count[kMaxExperts + 1], first[kMaxExperts + 2], tile0[kMaxExperts + 2];
-  for (int e = threadIdx.x; e < experts; e += 1024) count[e] = 0;
+  for (int e = threadIdx.x; e < experts; e += 1024) count[e] = shared && e == experts - 1 ? total / per_row : 0;
   __syncthreads();
   constexpr int B = 8;  // loads in flight
   for (int i0 = threadIdx.x; i0 < total; i0 += 1024 * B) {
@@ -50,7 +51,7 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(int32_t* __restrict__ o
     for (int j = 0; j < B; ++j) e[j] = i0 + 1024 * j < total ? min(max(ids[i0 + 1024 * j], 0), experts - 1) : -1;
 #pragma unroll
     for (int j = 0; j < B; ++j)
-      if (e[j] >= 0) e[j] = atomicAdd(&count[e[j]], 1);
+      if (e[j] >= 0) e[j] = shared && e[j] == experts - 1 ? (i0 + 1024 * j) / per_row : atomicAdd(&count[e[j]], 1);
 #pragma unroll
     for (int j = 0; j < B; ++j)
       if (i0 + 1024 * j < total) slot[i0 + 1024 * j] = e[j];
@@ -93,13 +94,15 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(int32_t* __restrict__ o
   }
   for (int e = threadIdx.x; e < experts; e += 1024)
     for (int t = tile0[e]; t < tile0[e + 1] && t < max_tiles; ++t) {
-      tiles[2 * t] = e;
-      tiles[2 * t + 1] = first[e] + (t - tile0[e]) * tile;
+      tiles[4 * t] = e;
+      tiles[4 * t + 1] = first[e] + (t - tile0[e]) * tile;
+      tiles[4 * t + 2] = tile0[e];
+      tiles[4 * t + 3] = tile0[e + 1] - tile0[e];
     }
-  for (int t = tile0[experts] + threadIdx.x; t < max_tiles; t += 1024) tiles[2 * t] = -1;
+  for (int t = tile0[experts] + threadIdx.x; t < max_tiles; t += 1024) tiles[4 * t] = -1;
   if (threadIdx.x == 0) {
-    tiles[2 * max_tiles] = min(tile0[experts - 1], max_tiles);
-    tiles[2 * max_tiles + 1] = min(tile0[experts], max_tiles);
+    tiles[4 * max_tiles] = min(tile0[experts - 1], max_tiles);
+    tiles[4 * max_tiles + 1] = min(tile0[experts], max_tiles);
   }
 }
 
@@ -108,9 +111,9 @@ template <typename T, bool UP>
 __global__ __launch_bounds__(256) void moe_simple_kernel(const MoeParams p) {
   using S = typename T::store_t;
   __shared__ float sx[16][33], sg[16][33], su[UP ? 16 : 1][33];
-  const int e = p.tiles[2 * blockIdx.y];
+  const int e = p.tiles[4 * blockIdx.y];
   if (e < 0 || e >= p.experts) return;
-  const int s0 = p.tiles[2 * blockIdx.y + 1], s1 = min(min(p.offsets[e + 1], s0 + 16), p.slots);
+  const int s0 = p.tiles[4 * blockIdx.y + 1], s1 = min(min(p.offsets[e + 1], s0 + 16), p.slots);
   const int ff = p.ff[e], K = UP ? p.width : ff, n0 = blockIdx.x * 16;
   if (n0 >= (UP ? ff : p.width)) return;
   const S* w = (const S*)p.w + p.w_offset[e];
@@ -172,11 +175,11 @@ extern "C" int lvllm_moe_route(int32_t* ids, float* weights, const void* h, cons
 extern "C" int lvllm_moe_tile(int packed) { return packed ? kMoeTile : kMoeSimpleTile; }
 
 extern "C" int lvllm_moe_group(int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles, const int32_t* ids, int total,
-                               int per_row, int experts, int packed, int max_tiles, void* stream) {
+                               int per_row, int experts, int shared, int packed, int max_tiles, void* stream) {
   if (total == 0) return 0;
   LV_CHECK(experts > 0 && experts <= kMaxExperts && per_row > 0, "experts (shared one included): at most 1024");
   hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, (hipStream_t)stream, offsets, token, slot, tiles, ids, total,
-                     per_row, experts, lvllm_moe_tile(packed), max_tiles);
+                     per_row, experts, shared != 0, lvllm_moe_tile(packed), max_tiles);
   LV_LAUNCH_CHECK();
   return 0;
 }

@@ -4,10 +4,11 @@
 //   * few slots per expert (decode steps): bound by the weights' bytes.  A workgroup takes 16 slots of one expert and a share
 //     of its outputs; the slots' rows sit in LDS in fragment order (2048 of K at a time), every wave streams the two W tiles
 //     of its own (1 KiB a load, eight k-steps in flight behind the eight in use) and needs no other wave;
-//   * prompts: 256 W rows x 128 slots a workgroup, a wave 128 x 64.  Both operands go straight from memory to LDS, 32 of K a
-//     stage, two stages in flight behind the one in use.  Packed W tiles are LDS images as they are; a slot's 64 bytes are
-//     four chunks, exchanged so that a fragment read is free of bank conflicts.  The work is dealt so that an XCD walks
-//     consecutive tiles with all their W blocks: its L2 sees a tile's rows and an expert's weights once.
+//   * prompts: 256 W rows x 128 slots a workgroup, a wave 64 x 128.  W goes from memory straight into the operand registers
+//     of the one wave that uses it, the slots' rows straight to LDS, 32 of K a step, three steps in flight behind the one in
+//     use (through LDS, W would take more of its bandwidth than there is).  A slot's 64 bytes are four chunks, exchanged so
+//     that a fragment read is free of bank conflicts.  An XCD gets consecutive work: up to eight tiles of an expert side by
+//     side, W block after W block, so that its L2 serves a W block to all of them and their rows to the next blocks.
 #include "moe.h"
 
 namespace lvllm {
@@ -102,8 +103,7 @@ __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
 }
 
 constexpr int kTileW = 16;                                 // W tiles of a workgroup
-constexpr int kStageBytes = (kTileW + kMoeTile / 16) * 1024;  // 32 of K: W tiles, then 16-slot groups
-constexpr int kStages = 3;
+constexpr int kStages = 4, kStageBytes = kMoeTile * 64;    // of 32 of K: 16-slot groups of 1 KiB
 
 __device__ __forceinline__ void to_lds(const uint16_t* src, char* dst) {  // 16 bytes a lane, 1 KiB a wave
   __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
@@ -112,29 +112,35 @@ __device__ __forceinline__ void to_lds(const uint16_t* src, char* dst) {  // 16 
 
 template <bool UP>
 __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, const int blocks_first, const int blocks_last) {
-  extern __shared__ __attribute__((aligned(16))) char ring[];  // [kStages][kStageBytes]
+  __shared__ __attribute__((aligned(16))) char ring[kStages][kStageBytes];
   // the tiles of all experts but the last one, then the last one's (the shared expert may be larger): an eighth of each to
   // every XCD
-  const int tiles_first = p.tiles[2 * p.max_tiles], tiles_all = p.tiles[2 * p.max_tiles + 1];
+  const int tiles_first = p.tiles[4 * p.max_tiles], tiles_all = p.tiles[4 * p.max_tiles + 1];
   const int xcd = blockIdx.x & 7, turn = blockIdx.x >> 3;
   const int all_first = tiles_first * blocks_first, all_last = (tiles_all - tiles_first) * blocks_last;
   const int per_first = (all_first + 7) / 8, per_last = (all_last + 7) / 8;
-  int tile, block;
+  int unit, blocks, tile;
   if (turn < per_first) {
-    const int i = xcd * per_first + turn;
-    if (i >= all_first) return;
-    tile = i / blocks_first;
-    block = i - tile * blocks_first;
+    unit = xcd * per_first + turn;
+    if (unit >= all_first) return;
+    blocks = blocks_first;
+    tile = unit / blocks;
   } else {
-    const int t = turn - per_first, i = xcd * per_last + t;
-    if (t >= per_last || i >= all_last) return;
-    tile = i / blocks_last;
-    block = i - tile * blocks_last;
-    tile += tiles_first;
+    unit = xcd * per_last + turn - per_first;
+    if (turn - per_first >= per_last || unit >= all_last) return;
+    blocks = blocks_last;
+    tile = tiles_first + unit / blocks;
+    unit += tiles_first * blocks;
   }
-  const int e = p.tiles[2 * tile];
-  if (e < 0 || e >= p.experts) return;
-  const int s0 = p.tiles[2 * tile + 1], s1 = min(min(p.offsets[e + 1], s0 + kMoeTile), p.slots);
+  constexpr int kSide = 8;
+  const int e = p.tiles[4 * tile], tile0 = p.tiles[4 * tile + 2], count = p.tiles[4 * tile + 3];
+  if (e < 0 || e >= p.experts || count <= 0) return;
+  unit -= tile0 * blocks;  // of this expert's
+  const int group = unit / (kSide * blocks), side = min(kSide, count - group * kSide);
+  unit -= group * kSide * blocks;
+  const int block = unit / side;
+  tile = tile0 + group * kSide + unit - block * side;
+  const int s0 = p.tiles[4 * tile + 1], s1 = min(min(p.offsets[e + 1], s0 + kMoeTile), p.slots);
   const int ff = p.ff[e], steps = (UP ? p.width : ff) >> 5;
   const int ntiles = UP ? ff >> 3 : p.width >> 4;  // of 16 W rows
   if (block * kTileW >= ntiles || s0 >= s1) return;
@@ -142,61 +148,68 @@ __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, con
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
   const int64_t ld = UP ? p.width : p.ff_max;
-  // what this wave moves: W tiles 4 wave .. and 16-slot groups 2 wave ..; lane l of a group: slot l / 4, chunk l % 4 of it
-  // exchanged by the slot's number / 4
+  const int nt0 = block * kTileW + wave * 4;
+  // this wave's W tiles, and the two 16-slot groups it copies: lane l moves chunk l % 4, exchanged by slot / 4, of slot l / 4
   const uint16_t *wsrc[4], *xsrc[2];
   const uint16_t* w = (const uint16_t*)p.w + p.w_offset[e] + lane * 8;
 #pragma unroll
-  for (int j = 0; j < 4; ++j) wsrc[j] = w + (int64_t)min(block * kTileW + wave * 4 + j, ntiles - 1) * steps * 512;
+  for (int j = 0; j < 4; ++j) wsrc[j] = w + (int64_t)min(nt0 + j, ntiles - 1) * steps * 512;
 #pragma unroll
   for (int j = 0; j < 2; ++j) {
     const int slot = min(s0 + (wave * 2 + j) * 16 + (lane >> 2), s1 - 1);
     const int64_t row = UP ? min(max(p.token[slot], 0), p.rows - 1) : slot;
     xsrc[j] = (const uint16_t*)p.x + row * ld + ((lane & 3) ^ (lane >> 4)) * 8;
   }
-  auto issue = [&](int k, char* st) __attribute__((always_inline)) {
+  e_u32x4_t a[kStages][4];
+  auto issue = [&](int k, int stage) __attribute__((always_inline)) {  // (past the end: the last step once more)
+    k = min(k, steps - 1);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) to_lds(wsrc[j] + k * 512, st + (wave * 4 + j) * 1024);
+    for (int j = 0; j < 2; ++j) to_lds(xsrc[j] + k * 32, ring[stage] + (wave * 2 + j) * 1024);
 #pragma unroll
-    for (int j = 0; j < 2; ++j) to_lds(xsrc[j] + k * 32, st + (kTileW + wave * 2 + j) * 1024);
+    for (int j = 0; j < 4; ++j) a[stage][j] = *reinterpret_cast<const e_u32x4_t*>(wsrc[j] + k * 512);
   };
-  const int wn = wave & 1, wm = wave >> 1;
-  const int woff = wn * 8 * 1024 + lane * 16, xoff = (kTileW + wm * 4) * 1024 + c * 64 + ((g ^ (c >> 2)) * 16);
-  e_f32x4_t acc[8][4];
+  constexpr int MT = kMoeTile / 16;
+  const int xoff = c * 64 + ((g ^ (c >> 2)) * 16);
+  e_f32x4_t acc[4][MT];
 #pragma unroll
-  for (int n = 0; n < 8; ++n)
+  for (int n = 0; n < 4; ++n)
 #pragma unroll
-    for (int m = 0; m < 4; ++m) acc[n][m] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
-  issue(0, ring);
-  if (steps > 1) issue(1, ring + kStageBytes);
-  char *cur = ring, *nxt = ring + 2 * kStageBytes;
-  for (int k = 0; k < steps; ++k) {
-    // loads retire in order: with only the next stage's six outstanding, this one's have landed
-    if (k + 1 < steps) asm volatile("s_waitcnt vmcnt(6)" ::: "memory");
-    else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    for (int m = 0; m < MT; ++m) acc[n][m] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
+  auto step = [&](int k, int stage) __attribute__((always_inline)) {
+    // loads retire in order: with only the two younger steps' six each outstanding, this one's have landed
+    __builtin_amdgcn_s_waitcnt(12 | (7 << 4) | (15 << 8));
     asm volatile("s_barrier" ::: "memory");  // ... for every wave; and everyone is done with the stage that is filled next
-    if (k + 2 < steps) issue(k + 2, nxt);
-    e_u32x4_t x[4], a[8];
+    issue(k + 3, (stage + 3) % kStages);
+    e_u32x4_t x[MT];
 #pragma unroll
-    for (int m = 0; m < 4; ++m) x[m] = *reinterpret_cast<const e_u32x4_t*>(cur + xoff + m * 1024);
+    for (int m = 0; m < MT; ++m) x[m] = *reinterpret_cast<const e_u32x4_t*>(ring[stage] + xoff + m * 1024);
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int n = 0; n < 8; ++n) a[n] = *reinterpret_cast<const e_u32x4_t*>(cur + woff + n * 1024);
-    __builtin_amdgcn_sched_barrier(0);  // (the reads first: they return while the first products run)
+    for (int m = 0; m < MT; ++m)
 #pragma unroll
-    for (int n = 0; n < 8; ++n)
-#pragma unroll
-      for (int m = 0; m < 4; ++m) acc[n][m] = moe_mfma(a[n], x[m], acc[n][m]);
-    cur = cur == ring + 2 * kStageBytes ? ring : cur + kStageBytes;
-    nxt = nxt == ring + 2 * kStageBytes ? ring : nxt + kStageBytes;
+      for (int n = 0; n < 4; ++n) acc[n][m] = moe_mfma(a[stage][n], x[m], acc[n][m]);
+  };
+  issue(0, 0);
+  issue(1, 1);
+  issue(2, 2);
+  int k = 0;
+  for (; k + 4 <= steps; k += 4) {
+    step(k, 0);
+    step(k + 1, 1);
+    step(k + 2, 2);
+    step(k + 3, 3);
   }
+  if (k < steps) step(k, 0);
+  if (k + 1 < steps) step(k + 1, 1);
+  if (k + 2 < steps) step(k + 2, 2);
+  __builtin_amdgcn_s_waitcnt(0 | (7 << 4) | (15 << 8));  // (no copy to LDS outlives the workgroup)
   const float limit = UP ? p.limit[e] : 0.f;
-  const int nt0 = block * kTileW + wn * 8;
 #pragma unroll
-  for (int m = 0; m < 4; ++m) {
-    const int slot = s0 + (wm * 4 + m) * 16 + c;
+  for (int m = 0; m < MT; ++m) {
+    const int slot = s0 + 16 * m + c;
     if (slot >= s1) continue;
 #pragma unroll
-    for (int n = 0; n < 8; n += UP ? 2 : 1) {
+    for (int n = 0; n < 4; n += UP ? 2 : 1) {
       if (nt0 + n >= ntiles) continue;
       float v[4];
       if constexpr (UP) {
@@ -213,47 +226,49 @@ __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, con
 }
 
 // The router on packed weights (experts and the shared gate, up to a multiple of 16 rows): 16 rows of h a workgroup, its 8
-// waves take every eighth k-step, the logits meet in LDS in wave order, a wave chooses for two rows.
+// waves take every eighth k-step of eight tiles of weights, the logits meet in LDS in wave order, a wave chooses for two rows.
 __global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
                                                              const uint16_t* __restrict__ h, const uint16_t* __restrict__ w,
                                                              const float* __restrict__ bias, const int experts,
                                                              const int shared, const int top, const int rows, const int width) {
+  constexpr int TG = 8, B = 4;  // tiles and k-steps in flight
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  e_f32x4_t* red = reinterpret_cast<e_f32x4_t*>(smem);      // [8 waves][4 tiles][64 lanes]
-  float* z = reinterpret_cast<float*>(smem + 8 * 4 * 1024);  // [16][ld]
+  e_f32x4_t* red = reinterpret_cast<e_f32x4_t*>(smem);       // [8 waves][TG tiles][64 lanes]
+  float* z = reinterpret_cast<float*>(smem + 8 * TG * 1024);  // [16][ld]
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
   const int steps = width >> 5, ntiles = (experts + shared + 15) >> 4, ld = ntiles * 16 + 1;
   const int row0 = blockIdx.x * 16;
   const uint16_t* x = h + (int64_t)min(row0 + c, rows - 1) * width + 8 * g;
-  for (int t0 = 0; t0 < ntiles; t0 += 4) {
-    e_f32x4_t acc[4];
+  for (int t0 = 0; t0 < ntiles; t0 += TG) {
+    e_f32x4_t acc[TG];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
-    constexpr int B = 4;  // k-steps in flight
+    for (int i = 0; i < TG; ++i) acc[i] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
     for (int k0 = wave; k0 < steps; k0 += 8 * B) {
-      e_u32x4_t xv[B], wv[B][4];
+      e_u32x4_t xv[B], wv[B][TG];
 #pragma unroll
       for (int j = 0; j < B; ++j) {
         const int k = min(k0 + 8 * j, steps - 1);
         xv[j] = k0 + 8 * j < steps ? *reinterpret_cast<const e_u32x4_t*>(x + 32 * k) : e_u32x4_t{0, 0, 0, 0};
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          wv[j][i] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)min(t0 + i, ntiles - 1) * steps + k) * 512 + lane * 8);
+        for (int i = 0; i < TG; ++i)
+          if (t0 + i < ntiles) wv[j][i] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)(t0 + i) * steps + k) * 512 + lane * 8);
       }
 #pragma unroll
-      for (int j = 0; j < B; ++j)
+      for (int i = 0; i < TG; ++i)
+        if (t0 + i < ntiles) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) acc[i] = moe_mfma(wv[j][i], xv[j], acc[i]);
+          for (int j = 0; j < B; ++j) acc[i] = moe_mfma(wv[j][i], xv[j], acc[i]);
+        }
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) red[(wave * 4 + i) * 64 + lane] = acc[i];
+    for (int i = 0; i < TG; ++i) red[(wave * TG + i) * 64 + lane] = acc[i];
     __syncthreads();
-    if (threadIdx.x < 256 && t0 + wave < ntiles) {  // wave i sums tile i
+    if (t0 + wave < ntiles) {  // wave i sums tile i
       e_f32x4_t s = red[threadIdx.x];
 #pragma unroll
-      for (int v = 1; v < 8; ++v) s += red[v * 256 + threadIdx.x];
+      for (int v = 1; v < 8; ++v) s += red[v * TG * 64 + threadIdx.x];
       const int n = (t0 + wave) * 16 + 4 * g;
 #pragma unroll
       for (int r = 0; r < 4; ++r) z[c * ld + n + r] = s[r] + (n + r < experts ? bias[n + r] : 0.f);
@@ -267,9 +282,8 @@ __global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict
 
 int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
                           int top, int rows, int width, hipStream_t s) {
-  const int smem = 8 * 4 * 1024 + 16 * ((experts + shared + 15) / 16 * 16 + 1) * 4;
-  if (smem > 64 * 1024)
-    (void)hipFuncSetAttribute((const void*)moe_route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
+  const int smem = 8 * 8 * 1024 + 16 * ((experts + shared + 15) / 16 * 16 + 1) * 4;
+  (void)hipFuncSetAttribute((const void*)moe_route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
   hipLaunchKernelGGL(moe_route_mfma_kernel, dim3((rows + 15) / 16), dim3(512), smem, s, ids, weights, (const uint16_t*)h,
                      (const uint16_t*)w, bias, experts, shared, top, rows, width);
   LV_LAUNCH_CHECK();
@@ -285,13 +299,11 @@ static void go(const MoeParams& p, hipStream_t s) {
     const int smem = (steps < kStreamChunk ? steps : kStreamChunk) * 1024;
     hipLaunchKernelGGL((moe_stream_kernel<UP>), dim3((units + 3) / 4, p.experts, (p.rows + 15) / 16), dim3(256), smem, s, p);
   } else {
-    constexpr int smem = kStages * kStageBytes;
-    (void)hipFuncSetAttribute((const void*)moe_tile_kernel<UP>, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
     auto blocks = [&](int ff) { return ((UP ? ff / 8 : p.width / 16) + kTileW - 1) / kTileW; };
     const int first = blocks(p.ff_first), last = blocks(p.ff_last);
     const int64_t last_tiles = (p.rows + kMoeTile - 1) / kMoeTile;  // a token takes an expert once
     const int64_t wgs = 8 * (((int64_t)p.max_tiles * first + 7) / 8 + (last_tiles * last + 7) / 8);
-    hipLaunchKernelGGL((moe_tile_kernel<UP>), dim3((unsigned)wgs), dim3(256), smem, s, p, first, last);
+    hipLaunchKernelGGL((moe_tile_kernel<UP>), dim3((unsigned)wgs), dim3(256), 0, s, p, first, last);
   }
 }
 

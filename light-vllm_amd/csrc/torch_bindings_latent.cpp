@@ -188,7 +188,7 @@ std::tuple<torch::Tensor, torch::Tensor> moe_route(const torch::Tensor& h, const
   return {ids, weights};
 }
 
-std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_group(const torch::Tensor& ids, int64_t experts,
+std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_group(const torch::Tensor& ids, int64_t experts, bool shared,
                                                                                  bool packed) {
   const char* op = "moe_group";
   TORCH_CHECK(ids.dim() == 2, op, ": ids [rows, assignments]");
@@ -197,9 +197,9 @@ std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_group
   const int64_t total = ids.numel(), tile = lvllm_moe_tile(packed);
   const int64_t max_tiles = std::min(total, total / tile + experts);
   auto offsets = torch::empty({experts + 1}, ids.options()), token = torch::empty({total}, ids.options());
-  auto slot = torch::empty_like(ids), tiles = torch::empty({max_tiles + 1, 2}, ids.options());
+  auto slot = torch::empty_like(ids), tiles = torch::empty({max_tiles + 1, 4}, ids.options());
   check(lvllm_moe_group(offsets.data_ptr<int>(), token.data_ptr<int>(), slot.data_ptr<int>(), tiles.data_ptr<int>(),
-                        ids.data_ptr<int>(), (int)total, (int)ids.size(1), (int)experts, packed, (int)max_tiles,
+                        ids.data_ptr<int>(), (int)total, (int)ids.size(1), (int)experts, shared, packed, (int)max_tiles,
                         current_stream(ids)));
   return {offsets, token, slot, tiles};
 }
@@ -221,7 +221,7 @@ torch::Tensor moe_experts(const torch::Tensor& x, const torch::Tensor& w, const 
   check_f32(limit, experts, op, "limit");
   check_i32(offsets, experts + 1, op, "offsets");
   check_i32(token, slots, op, "token");
-  check_i32(tiles, 4, op, "tiles");
+  check_i32(tiles, 8, op, "tiles");
   auto out = torch::empty({slots, up ? ff_max : width}, x.options());
   check(lvllm_moe_experts(out.data_ptr(), x.data_ptr(), w.data_ptr(), w_offset.data_ptr<int64_t>(), ff.data_ptr<int>(),
                           limit.data_ptr<float>(), offsets.data_ptr<int>(), token.data_ptr<int>(), tiles.data_ptr<int>(),
@@ -320,7 +320,7 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, latent) {
   latent.impl("latent_rotate_query", torch::kCUDA, &latent_rotate_query);
   latent.def("moe_route(Tensor h, Tensor w, Tensor bias, int top, bool shared, bool packed) -> (Tensor, Tensor)");
   latent.impl("moe_route", torch::kCUDA, &moe_route);
-  latent.def("moe_group(Tensor ids, int experts, bool packed) -> (Tensor, Tensor, Tensor, Tensor)");
+  latent.def("moe_group(Tensor ids, int experts, bool shared, bool packed) -> (Tensor, Tensor, Tensor, Tensor)");
   latent.impl("moe_group", torch::kCUDA, &moe_group);
   latent.def("moe_experts(Tensor x, Tensor w, Tensor w_offset, Tensor ff, Tensor limit, Tensor offsets, Tensor token, "
              "Tensor tiles, int rows, int width, int ff_max, int ff_first, int ff_last, bool up, bool packed) "
