@@ -669,13 +669,14 @@ int lvllm_latent_expand(void* key_pages, void* value_pages, const void* kv, int6
 int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_stride, int heads, int dim, int rot_dim, int kpad,
                               const int64_t* positions, const double* turns, int rot_dims, int rows, int dtype, void* stream);
 /* the `top` experts of every row and their softmax weights; with `shared` a last assignment, expert number `experts`, weighted
- * sigmoid of the last row of w.  `packed`: w as lvllm_pack_weight leaves it, rows padded to a multiple of 16 */
-int lvllm_moe_route(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
-                    int top, int rows, int width, int packed, int dtype, void* stream);
-/* assignments grouped by expert: offsets [experts + 1], token and slot [total], tiles [max_tiles + 1, 4] of lvllm_moe_tile slots */
-int lvllm_moe_tile(int packed);
-int lvllm_moe_group(int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles, const int32_t* ids, int total, int per_row,
-                    int experts, int shared, int packed, int max_tiles, void* stream);
+ * sigmoid of the last row of w.  The assignments come grouped by expert: offsets [experts + shared + 1], token and slot
+ * [assignments], tiles [max_tiles + 1, 4] of lvllm_moe_tile slots.  `packed`: w as lvllm_pack_weight leaves it, rows padded to a
+ * multiple of 16 */
+int lvllm_moe_tile(int packed, int rows);
+int64_t lvllm_moe_route_workspace_bytes(int experts, int shared, int rows, int width, int packed);
+int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles, int max_tiles,
+                    const void* h, const void* w, const float* bias, int experts, int shared, int top, int rows, int width,
+                    int packed, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 /* the experts' products: up (with the activation) [rows, width] -> [slots, ff_max], down [slots, ff_max] -> [slots, width] */
 int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff, const float* limit,
                       const int32_t* offsets, const int32_t* token, const int32_t* tiles, int experts, int slots, int rows,

@@ -35,75 +35,15 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int32_t* __restrict__ id
   if (threadIdx.x < 64) choose_experts(z, experts, top, shared != 0, ids + (int64_t)row * n, weights + (int64_t)row * n);
 }
 
-// Counts, offsets, slots and tiles of `total` assignments; one workgroup.  `shared`: the last assignment of every row is the
-// last expert's, in row order.
-__global__ __launch_bounds__(1024) void moe_group_kernel(int32_t* __restrict__ offsets, int32_t* __restrict__ token,
-                                                         int32_t* __restrict__ slot, int32_t* __restrict__ tiles,
-                                                         const int32_t* __restrict__ ids, const int total, const int per_row,
-                                                         const int experts, const int shared, const int tile, const int max_tiles) {
-  __shared__ int count[kMaxExperts + 1], first[kMaxExperts + 2], tile0[kMaxExperts + 2];
-  for (int e = threadIdx.x; e < experts; e += 1024) count[e] = shared && e == experts - 1 ? total / per_row : 0;
-  __syncthreads();
-  constexpr int B = 8;  // loads in flight
-  for (int i0 = threadIdx.x; i0 < total; i0 += 1024 * B) {
-    int e[B];
-#pragma unroll
-    for (int j = 0; j < B; ++j) e[j] = i0 + 1024 * j < total ? min(max(ids[i0 + 1024 * j], 0), experts - 1) : -1;
-#pragma unroll
-    for (int j = 0; j < B; ++j)
-      if (e[j] >= 0) e[j] = shared && e[j] == experts - 1 ? (i0 + 1024 * j) / per_row : atomicAdd(&count[e[j]], 1);
-#pragma unroll
-    for (int j = 0; j < B; ++j)
-      if (i0 + 1024 * j < total) slot[i0 + 1024 * j] = e[j];
-  }
-  __syncthreads();
-  if (threadIdx.x < 64) {  // running sums, 64 experts a turn
-    int base = 0, tbase = 0;
-    for (int e0 = 0; e0 < experts; e0 += 64) {
-      const int e = e0 + threadIdx.x;
-      const int c = e < experts ? count[e] : 0, t = (c + tile - 1) / tile;
-      int s = c, ts = t;
-#pragma unroll
-      for (int d = 1; d < 64; d <<= 1) {
-        const int a = __shfl_up(s, d), b = __shfl_up(ts, d);
-        if ((int)threadIdx.x >= d) { s += a; ts += b; }
-      }
-      if (e < experts) { first[e] = base + s - c; tile0[e] = tbase + ts - t; }
-      base += __shfl(s, 63);
-      tbase += __shfl(ts, 63);
-    }
-    if (threadIdx.x == 0) { first[experts] = base; tile0[experts] = tbase; }
-  }
-  __syncthreads();
-  for (int e = threadIdx.x; e <= experts; e += 1024) offsets[e] = first[e];
-  for (int i0 = threadIdx.x; i0 < total; i0 += 1024 * B) {
-    int e[B], s[B];
-#pragma unroll
-    for (int j = 0; j < B; ++j) {
-      const int i = min(i0 + 1024 * j, total - 1);
-      e[j] = min(max(ids[i], 0), experts - 1);
-      s[j] = slot[i];
-    }
-#pragma unroll
-    for (int j = 0; j < B; ++j) {
-      const int i = i0 + 1024 * j;
-      if (i >= total) break;
-      slot[i] = first[e[j]] + s[j];
-      token[first[e[j]] + s[j]] = i / per_row;
-    }
-  }
-  for (int e = threadIdx.x; e < experts; e += 1024)
-    for (int t = tile0[e]; t < tile0[e + 1] && t < max_tiles; ++t) {
-      tiles[4 * t] = e;
-      tiles[4 * t + 1] = first[e] + (t - tile0[e]) * tile;
-      tiles[4 * t + 2] = tile0[e];
-      tiles[4 * t + 3] = tile0[e + 1] - tile0[e];
-    }
-  for (int t = tile0[experts] + threadIdx.x; t < max_tiles; t += 1024) tiles[4 * t] = -1;
-  if (threadIdx.x == 0) {
-    tiles[4 * max_tiles] = min(tile0[experts - 1], max_tiles);
-    tiles[4 * max_tiles + 1] = min(tile0[experts], max_tiles);
-  }
+__global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t* ids, const int total, const int per_row,
+                                                         const int experts, const int shared, const MoeGroups groups) {
+  group_assignments(ids, total, per_row, experts, shared, groups);
+}
+
+int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, const MoeGroups& groups, hipStream_t s) {
+  hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, s, ids, total, per_row, experts, shared, groups);
+  LV_LAUNCH_CHECK();
+  return 0;
 }
 
 // 16 slots x 16 outputs a workgroup, row-major weights, 32 of K a turn through LDS.
@@ -150,38 +90,38 @@ __global__ __launch_bounds__(256) void moe_simple_kernel(const MoeParams p) {
 
 using namespace lvllm;
 
-extern "C" int lvllm_moe_route(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts,
-                               int shared, int top, int rows, int width, int packed, int dtype, void* stream) {
+extern "C" int lvllm_moe_tile(int packed, int rows) { return moe_tile(packed != 0, rows); }
+
+extern "C" int64_t lvllm_moe_route_workspace_bytes(int experts, int shared, int rows, int width, int packed) {
+  return packed ? moe_route_mfma_workspace(experts, shared != 0, rows, width) : 0;
+}
+
+extern "C" int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles,
+                               int max_tiles, const void* h, const void* w, const float* bias, int experts, int shared, int top,
+                               int rows, int width, int packed, void* workspace, int64_t workspace_bytes, int dtype,
+                               void* stream) {
   if (rows == 0) return 0;
-  LV_CHECK(experts > 0 && experts < kMaxExperts && top > 0 && top <= experts && top <= 64, "experts (fewer than 1024) or top (at most 64)");
+  LV_CHECK(experts > 0 && experts < kMaxExperts && top > 0 && top <= experts, "experts: fewer than 1024, top of them");
+  LV_CHECK((int64_t)rows * (top + 1) < ((int64_t)1 << 31) && max_tiles > 0, "too many assignments");
+  LV_CHECK(workspace_bytes >= lvllm_moe_route_workspace_bytes(experts, shared, rows, width, packed), "workspace too small");
   hipStream_t s = (hipStream_t)stream;
+  shared = shared != 0;
+  const MoeGroups groups{offsets, token, slot, tiles, lvllm_moe_tile(packed, rows), max_tiles};
   if (packed) {
     LV_CHECK(moe_takes_mfma(width, dtype), "packed router: bf16, a width that is a multiple of 32");
-    return launch_moe_route_mfma(ids, weights, h, w, bias, experts, shared != 0, top, rows, width, s);
+    return launch_moe_route_mfma(ids, weights, h, w, bias, experts, shared, top, rows, width, groups, (float*)workspace, s);
   }
   LV_DISPATCH_F32_BF16(dtype, {
     using S = typename scalar_t::store_t;
     if (width % 4 == 0)
       hipLaunchKernelGGL((moe_route_kernel<scalar_t, 4>), dim3(rows), dim3(256), 0, s, ids, weights, (const S*)h, (const S*)w,
-                         bias, experts, shared != 0, top, width);
+                         bias, experts, shared, top, width);
     else
       hipLaunchKernelGGL((moe_route_kernel<scalar_t, 1>), dim3(rows), dim3(256), 0, s, ids, weights, (const S*)h, (const S*)w,
-                         bias, experts, shared != 0, top, width);
+                         bias, experts, shared, top, width);
   });
   LV_LAUNCH_CHECK();
-  return 0;
-}
-
-extern "C" int lvllm_moe_tile(int packed) { return packed ? kMoeTile : kMoeSimpleTile; }
-
-extern "C" int lvllm_moe_group(int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles, const int32_t* ids, int total,
-                               int per_row, int experts, int shared, int packed, int max_tiles, void* stream) {
-  if (total == 0) return 0;
-  LV_CHECK(experts > 0 && experts <= kMaxExperts && per_row > 0, "experts (shared one included): at most 1024");
-  hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, (hipStream_t)stream, offsets, token, slot, tiles, ids, total,
-                     per_row, experts, shared != 0, lvllm_moe_tile(packed), max_tiles);
-  LV_LAUNCH_CHECK();
-  return 0;
+  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, groups, s);
 }
 
 extern "C" int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff,

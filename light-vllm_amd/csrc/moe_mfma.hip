@@ -22,30 +22,39 @@ __device__ __forceinline__ e_f32x4_t moe_mfma(e_u32x4_t a, e_u32x4_t b, e_f32x4_
                                                  0);
 }
 
-constexpr int kStreamMaxRows = 64, kStreamBatch = 8, kStreamChunk = 64;  // rows of a step; k-steps per batch, per LDS chunk
+constexpr int kStreamBatch = 8, kStreamChunk = 64;  // k-steps per batch, per LDS chunk
 
-// grid (shares of the outputs, experts, groups of 16 slots); a wave computes W tiles 2 u and 2 u + 1
-template <bool UP>
+// grid (shares of the outputs, tiles of 16 slots); a wave computes W tiles 2 u and 2 u + 1, or (KS > 1, when few
+// experts have work) a KS-th of their k-steps, 64 / KS of every LDS chunk
+template <bool UP, int KS>
 __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
   extern __shared__ __attribute__((aligned(16))) char sx[];  // [k-steps of a chunk][4][16][8]
-  const int e = blockIdx.y;
-  const int s0 = p.offsets[e] + 16 * blockIdx.z, s1 = min(p.offsets[e + 1], p.slots);
+  __shared__ e_f32x4_t red[KS > 1 ? 4 : 1][2][64];
+  const int e = p.tiles[4 * blockIdx.y];
+  if (e < 0 || e >= p.experts) return;
+  const int s0 = p.tiles[4 * blockIdx.y + 1], s1 = min(min(p.offsets[e + 1], s0 + 16), p.slots);
   if (s0 >= s1) return;
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
   const int ff = p.ff[e], K = UP ? p.width : ff, steps = K >> 5;
   const int units = UP ? ff >> 4 : p.width >> 5;
-  if ((int)blockIdx.x * 4 >= units) return;
-  const int u = min((int)blockIdx.x * 4 + wave, units - 1);  // (a wave too many repeats the last unit)
+  constexpr int U = 4 / KS, P = kStreamChunk / KS;  // units of a workgroup; this wave's k-steps of a chunk
+  if ((int)blockIdx.x * U >= units) return;
+  const int u = min((int)blockIdx.x * U + wave / KS, units - 1), kq = wave % KS;  // (a wave too many repeats the last unit)
+  // k-steps, some missing ones of the last chunk included
+  const int mine = KS == 1 ? (steps + 2 * kStreamBatch - 1) / (2 * kStreamBatch) * (2 * kStreamBatch)
+                           : (steps + kStreamChunk - 1) / kStreamChunk * P;
+  auto step_of = [&](int v) { return KS == 1 ? v : v / P * kStreamChunk + kq * P + v % P; };  // of batch v, a multiple of 8
   const uint16_t* w = (const uint16_t*)p.w + p.w_offset[e] + (int64_t)2 * u * steps * 512 + lane * 8;
   e_u32x4_t a[2][2][kStreamBatch];
-  auto fetch = [&](int b, e_u32x4_t (&t)[2][kStreamBatch]) __attribute__((always_inline)) {
+  auto fetch = [&](int v, e_u32x4_t (&t)[2][kStreamBatch]) __attribute__((always_inline)) {
+    const int b = step_of(v);
 #pragma unroll
     for (int j = 0; j < kStreamBatch; ++j)
 #pragma unroll
-      for (int i = 0; i < 2; ++i)
-        if (b + j < steps) t[i][j] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)i * steps + b + j) * 512);
+      for (int i = 0; i < 2; ++i)  // (a missing step: the last one again)
+        t[i][j] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)i * steps + min(b + j, steps - 1)) * 512);
   };
   fetch(0, a[0]);
   const int64_t ld = UP ? p.width : p.ff_max;
@@ -63,26 +72,42 @@ __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
   };
   const char* xf = sx + lane * 16;
   e_f32x4_t acc[2] = {e_f32x4_t{0.f, 0.f, 0.f, 0.f}, e_f32x4_t{0.f, 0.f, 0.f, 0.f}};
-  auto use = [&](int b, const e_u32x4_t (&t)[2][kStreamBatch]) __attribute__((always_inline)) {
+  auto use = [&](int v, const e_u32x4_t (&t)[2][kStreamBatch]) __attribute__((always_inline)) {
+    const int b = step_of(v), at = b % kStreamChunk;
+    auto one = [&](int j) __attribute__((always_inline)) {
+      const e_u32x4_t xv = *reinterpret_cast<const e_u32x4_t*>(xf + (at + j) * 1024);
+      acc[0] = moe_mfma(t[0][j], xv, acc[0]);
+      acc[1] = moe_mfma(t[1][j], xv, acc[1]);
+    };
+    if (b + kStreamBatch <= steps) {
 #pragma unroll
-    for (int j = 0; j < kStreamBatch; ++j)
-      if (b + j < steps) {
-        const e_u32x4_t xv = *reinterpret_cast<const e_u32x4_t*>(xf + ((b + j) % kStreamChunk) * 1024);
-        acc[0] = moe_mfma(t[0][j], xv, acc[0]);
-        acc[1] = moe_mfma(t[1][j], xv, acc[1]);
-      }
+      for (int j = 0; j < kStreamBatch; ++j) one(j);
+    } else {
+#pragma unroll
+      for (int j = 0; j < kStreamBatch; ++j)
+        if (b + j < steps) one(j);
+    }
   };
   stage(0);
-  for (int b = 0; b < steps; b += 2 * kStreamBatch) {
-    const bool two = b + kStreamBatch < steps;
-    if (two) fetch(b + kStreamBatch, a[1]);
-    if (b > 0 && b % kStreamChunk == 0) {
+  for (int v = 0; v < mine; v += 2 * kStreamBatch) {
+    fetch(v + kStreamBatch, a[1]);
+    if (v > 0 && v % P == 0) {
       __syncthreads();
-      stage(b);
+      stage(v / P * kStreamChunk);
     }
-    use(b, a[0]);
-    if (b + 2 * kStreamBatch < steps) fetch(b + 2 * kStreamBatch, a[0]);
-    if (two) use(b + kStreamBatch, a[1]);
+    use(v, a[0]);
+    fetch(v + 2 * kStreamBatch, a[0]);
+    use(v + kStreamBatch, a[1]);
+  }
+  if constexpr (KS > 1) {
+    red[wave][0][lane] = acc[0];
+    red[wave][1][lane] = acc[1];
+    __syncthreads();
+    if (kq != 0 || (int)blockIdx.x * U + wave / KS >= units) return;
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int q = 1; q < KS; ++q) acc[i] += red[wave + q][i][lane];
   }
   const int slot = s0 + c;
   if (slot >= s1) return;
@@ -225,32 +250,30 @@ __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, con
   }
 }
 
-// The router on packed weights (experts and the shared gate, up to a multiple of 16 rows): 16 rows of h a workgroup, its 8
-// waves take every eighth k-step of eight tiles of weights, the logits meet in LDS in wave order, a wave chooses for two rows.
-__global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
-                                                             const uint16_t* __restrict__ h, const uint16_t* __restrict__ w,
-                                                             const float* __restrict__ bias, const int experts,
-                                                             const int shared, const int top, const int rows, const int width) {
-  constexpr int TG = 8, B = 4;  // tiles and k-steps in flight
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  e_f32x4_t* red = reinterpret_cast<e_f32x4_t*>(smem);       // [8 waves][TG tiles][64 lanes]
-  float* z = reinterpret_cast<float*>(smem + 8 * TG * 1024);  // [16][ld]
+// The router's logits on packed weights (experts and the shared gate, up to a multiple of 16 rows): 16 rows of h and a share
+// of the k-steps a workgroup; its 8 waves take every eighth step of eight tiles of weights and meet in LDS in wave order.
+// z [rows 16 at a time][ld] in LDS, without the bias.
+constexpr int kRouteTiles = 8, kRouteBatch = 4;  // tiles and k-steps in flight
+constexpr int kRouteShares = 16;              // most shares of the k-steps
+constexpr int kRouteLds = 8 * kRouteTiles * 1024;
+
+__device__ __forceinline__ void route_logits(float* z, int ld, e_f32x4_t* red, const uint16_t* h, const uint16_t* w, int row0,
+                                             int rows, int width, int ntiles, int step0, int step1) {
+  constexpr int TG = kRouteTiles, B = kRouteBatch;
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int g = lane >> 4, c = lane & 15;
-  const int steps = width >> 5, ntiles = (experts + shared + 15) >> 4, ld = ntiles * 16 + 1;
-  const int row0 = blockIdx.x * 16;
+  const int g = lane >> 4, c = lane & 15, steps = width >> 5;
   const uint16_t* x = h + (int64_t)min(row0 + c, rows - 1) * width + 8 * g;
   for (int t0 = 0; t0 < ntiles; t0 += TG) {
     e_f32x4_t acc[TG];
 #pragma unroll
     for (int i = 0; i < TG; ++i) acc[i] = e_f32x4_t{0.f, 0.f, 0.f, 0.f};
-    for (int k0 = wave; k0 < steps; k0 += 8 * B) {
+    for (int k0 = step0 + wave; k0 < step1; k0 += 8 * B) {
       e_u32x4_t xv[B], wv[B][TG];
 #pragma unroll
       for (int j = 0; j < B; ++j) {
-        const int k = min(k0 + 8 * j, steps - 1);
-        xv[j] = k0 + 8 * j < steps ? *reinterpret_cast<const e_u32x4_t*>(x + 32 * k) : e_u32x4_t{0, 0, 0, 0};
+        const int k = min(k0 + 8 * j, step1 - 1);
+        xv[j] = k0 + 8 * j < step1 ? *reinterpret_cast<const e_u32x4_t*>(x + 32 * k) : e_u32x4_t{0, 0, 0, 0};
 #pragma unroll
         for (int i = 0; i < TG; ++i)
           if (t0 + i < ntiles) wv[j][i] = *reinterpret_cast<const e_u32x4_t*>(w + ((int64_t)(t0 + i) * steps + k) * 512 + lane * 8);
@@ -269,35 +292,114 @@ __global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict
       e_f32x4_t s = red[threadIdx.x];
 #pragma unroll
       for (int v = 1; v < 8; ++v) s += red[v * TG * 64 + threadIdx.x];
-      const int n = (t0 + wave) * 16 + 4 * g;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) z[c * ld + n + r] = s[r] + (n + r < experts ? bias[n + r] : 0.f);
+      for (int r = 0; r < 4; ++r) z[c * ld + (t0 + wave) * 16 + 4 * g + r] = s[r];
     }
     __syncthreads();
   }
-  const int n = top + shared;
-  for (int r = wave; r < 16 && row0 + r < rows; r += 8)
+}
+
+// many rows: logits and choice in one launch, a wave chooses for two rows
+__global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
+                                                             const uint16_t* __restrict__ h, const uint16_t* __restrict__ w,
+                                                             const float* __restrict__ bias, const int experts,
+                                                             const int shared, const int top, const int rows, const int width) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  float* z = reinterpret_cast<float*>(smem + kRouteLds);
+  const int ntiles = (experts + shared + 15) >> 4, ld = ntiles * 16 + 1, row0 = blockIdx.x * 16, n = top + shared;
+  route_logits(z, ld, reinterpret_cast<e_f32x4_t*>(smem), h, w, row0, rows, width, ntiles, 0, width >> 5);
+  const int lane = threadIdx.x & 63;
+  for (int r = threadIdx.x >> 6; r < 16 && row0 + r < rows; r += 8) {
+    for (int e = lane; e < experts; e += 64) z[r * ld + e] += bias[e];
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (the wave's own next reads see it)
     choose_experts(z + r * ld, experts, top, shared != 0, ids + (int64_t)(row0 + r) * n, weights + (int64_t)(row0 + r) * n);
+  }
+}
+
+// few rows: the k-steps are dealt to workgroups as well (grid.y), whose logits leave as part [share][16-row tiles][16][ld]
+__global__ __launch_bounds__(512) void moe_logits_kernel(float* __restrict__ part, const uint16_t* __restrict__ h,
+                                                         const uint16_t* __restrict__ w, const int ntiles, const int rows,
+                                                         const int width, const int per) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  float* z = reinterpret_cast<float*>(smem + kRouteLds);
+  const int ld = ntiles * 16, step0 = blockIdx.y * per, step1 = min(step0 + per, width >> 5);
+  route_logits(z, ld, reinterpret_cast<e_f32x4_t*>(smem), h, w, blockIdx.x * 16, rows, width, ntiles, step0, step1);
+  float* out = part + ((int64_t)blockIdx.y * gridDim.x + blockIdx.x) * 16 * ld;
+  for (int i = threadIdx.x; i < 16 * ld; i += 512) out[i] = z[i];
+}
+
+// ... and one workgroup adds them, chooses (a wave per row) and groups the assignments
+__global__ __launch_bounds__(1024) void moe_choose_group_kernel(int32_t* ids, float* weights, const float* __restrict__ part,
+                                                                const float* __restrict__ bias, const int shares,
+                                                                const int row_tiles, const int ld, const int experts,
+                                                                const int shared, const int top, const int rows,
+                                                                const MoeGroups groups) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = top + shared;
+  float* z = reinterpret_cast<float*>(smem) + wave * ld;
+  for (int row = wave; row < rows; row += 16) {
+    for (int e = lane; e < experts + shared; e += 64) {
+      float v = e < experts ? bias[e] : 0.f, t[kRouteShares];
+#pragma unroll
+      for (int s = 0; s < kRouteShares; ++s) t[s] = part[((int64_t)min(s, shares - 1) * row_tiles * 16 + row) * ld + e];
+#pragma unroll
+      for (int s = 0; s < kRouteShares; ++s) v += s < shares ? t[s] : 0.f;
+      z[e] = v;
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (the wave's own next reads see it)
+    choose_experts(z, experts, top, shared != 0, ids + (int64_t)row * n, weights + (int64_t)row * n);
+  }
+  __syncthreads();
+  group_assignments(ids, rows * n, n, experts + shared, shared, groups);
+}
+
+static int route_shares(int width) {
+  const int steps = width / 32;
+  return steps < 16 ? 1 : steps / 16 > kRouteShares ? kRouteShares : steps / 16;  // (at least two k-steps a wave)
+}
+
+int64_t moe_route_mfma_workspace(int experts, int shared, int rows, int width) {
+  if (rows > kMoeFewRows) return 0;
+  return (int64_t)route_shares(width) * ((rows + 15) / 16) * 16 * ((experts + shared + 15) / 16 * 16) * 4;
 }
 
 int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
-                          int top, int rows, int width, hipStream_t s) {
-  const int smem = 8 * 8 * 1024 + 16 * ((experts + shared + 15) / 16 * 16 + 1) * 4;
-  (void)hipFuncSetAttribute((const void*)moe_route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, smem);
-  hipLaunchKernelGGL(moe_route_mfma_kernel, dim3((rows + 15) / 16), dim3(512), smem, s, ids, weights, (const uint16_t*)h,
+                          int top, int rows, int width, const MoeGroups& groups, float* workspace, hipStream_t s) {
+  const int ntiles = (experts + shared + 15) / 16, row_tiles = (rows + 15) / 16;
+  if (rows <= kMoeFewRows) {
+    const int shares = route_shares(width), per = (width / 32 + shares - 1) / shares, ld = ntiles * 16;
+    const int lds = kRouteLds + 16 * ld * 4, lds_choose = 16 * ld * 4;
+    (void)hipFuncSetAttribute((const void*)moe_logits_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    (void)hipFuncSetAttribute((const void*)moe_choose_group_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds_choose);
+    hipLaunchKernelGGL(moe_logits_kernel, dim3(row_tiles, shares), dim3(512), lds, s, workspace, (const uint16_t*)h,
+                       (const uint16_t*)w, ntiles, rows, width, per);
+    LV_LAUNCH_CHECK();
+    hipLaunchKernelGGL(moe_choose_group_kernel, dim3(1), dim3(1024), lds_choose, s, ids, weights, workspace, bias, shares,
+                       row_tiles, ld, experts, shared, top, rows, groups);
+    LV_LAUNCH_CHECK();
+    return 0;
+  }
+  const int lds = kRouteLds + 16 * (ntiles * 16 + 1) * 4;
+  (void)hipFuncSetAttribute((const void*)moe_route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+  hipLaunchKernelGGL(moe_route_mfma_kernel, dim3(row_tiles), dim3(512), lds, s, ids, weights, (const uint16_t*)h,
                      (const uint16_t*)w, bias, experts, shared, top, rows, width);
   LV_LAUNCH_CHECK();
-  return 0;
+  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, groups, s);
 }
 
 bool moe_takes_mfma(int width, int dtype) { return dtype == LVLLM_BF16 && width % 32 == 0; }
 
 template <bool UP>
 static void go(const MoeParams& p, hipStream_t s) {
-  if (p.rows <= kStreamMaxRows) {
+  if (p.rows <= kMoeFewRows) {
     const int steps = (UP ? p.width : p.ff_max) / 32, units = UP ? p.ff_max / 16 : p.width / 32;  // of the largest expert
     const int smem = (steps < kStreamChunk ? steps : kStreamChunk) * 1024;
-    hipLaunchKernelGGL((moe_stream_kernel<UP>), dim3((units + 3) / 4, p.experts, (p.rows + 15) / 16), dim3(256), smem, s, p);
+    // workgroups with work, were every wave to take whole units
+    const int64_t wgs = (int64_t)p.max_tiles * (((UP ? p.ff_first / 16 : units) + 3) / 4);
+    const unsigned t = p.max_tiles;
+    if (wgs <= 256) hipLaunchKernelGGL((moe_stream_kernel<UP, 4>), dim3(units, t), dim3(256), smem, s, p);
+    else if (wgs <= 512) hipLaunchKernelGGL((moe_stream_kernel<UP, 2>), dim3((units + 1) / 2, t), dim3(256), smem, s, p);
+    else hipLaunchKernelGGL((moe_stream_kernel<UP, 1>), dim3((units + 3) / 4, t), dim3(256), smem, s, p);
   } else {
     auto blocks = [&](int ff) { return ((UP ? ff / 8 : p.width / 16) + kTileW - 1) / kTileW; };
     const int first = blocks(p.ff_first), last = blocks(p.ff_last);

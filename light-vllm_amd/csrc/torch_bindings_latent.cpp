@@ -169,8 +169,9 @@ torch::Tensor latent_rotate_query(const torch::Tensor& q, int64_t heads, int64_t
   return out;
 }
 
-std::tuple<torch::Tensor, torch::Tensor> moe_route(const torch::Tensor& h, const torch::Tensor& w, const torch::Tensor& bias,
-                                                   int64_t top, bool shared, bool packed) {
+// (ids, weights, offsets, token, slots, tiles)
+std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_route(
+    const torch::Tensor& h, const torch::Tensor& w, const torch::Tensor& bias, int64_t top, bool shared, bool packed) {
   const char* op = "moe_route";
   LV_CHECK_DEVICE(h);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(h));
@@ -180,28 +181,19 @@ std::tuple<torch::Tensor, torch::Tensor> moe_route(const torch::Tensor& h, const
                   w.size(0) == (packed ? (experts + shared + 15) / 16 * 16 : experts + shared),
               op, ": h [rows, width], w [experts (+ 1), width], packed: rows up to a multiple of 16");
   check_f32(bias, experts, op, "bias");
-  auto ids = torch::empty({rows, top + shared}, h.options().dtype(at::kInt));
-  auto weights = torch::empty({rows, top + shared}, h.options().dtype(at::kFloat));
-  check(lvllm_moe_route(ids.data_ptr<int>(), weights.data_ptr<float>(), h.data_ptr(), w.data_ptr(), bias.data_ptr<float>(),
-                        (int)experts, (int)shared, (int)top, (int)rows, (int)width, packed, dtype_code(h, op),
-                        current_stream(h)));
-  return {ids, weights};
-}
-
-std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_group(const torch::Tensor& ids, int64_t experts, bool shared,
-                                                                                 bool packed) {
-  const char* op = "moe_group";
-  TORCH_CHECK(ids.dim() == 2, op, ": ids [rows, assignments]");
-  check_i32(ids, ids.numel(), op, "ids");
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(ids));
-  const int64_t total = ids.numel(), tile = lvllm_moe_tile(packed);
-  const int64_t max_tiles = std::min(total, total / tile + experts);
-  auto offsets = torch::empty({experts + 1}, ids.options()), token = torch::empty({total}, ids.options());
-  auto slot = torch::empty_like(ids), tiles = torch::empty({max_tiles + 1, 4}, ids.options());
-  check(lvllm_moe_group(offsets.data_ptr<int>(), token.data_ptr<int>(), slot.data_ptr<int>(), tiles.data_ptr<int>(),
-                        ids.data_ptr<int>(), (int)total, (int)ids.size(1), (int)experts, shared, packed, (int)max_tiles,
-                        current_stream(ids)));
-  return {offsets, token, slot, tiles};
+  const auto ints = h.options().dtype(at::kInt);
+  const int64_t n = top + shared, total = rows * n, tile = lvllm_moe_tile(packed, (int)rows);
+  const int64_t max_tiles = std::max<int64_t>(1, std::min(total, total / tile + experts + shared));
+  auto ids = torch::empty({rows, n}, ints), slot = torch::empty({rows, n}, ints), token = torch::empty({total}, ints);
+  auto offsets = torch::empty({experts + shared + 1}, ints), tiles = torch::empty({max_tiles + 1, 4}, ints);
+  auto weights = torch::empty({rows, n}, h.options().dtype(at::kFloat));
+  const int64_t need = lvllm_moe_route_workspace_bytes((int)experts, shared, (int)rows, (int)width, packed);
+  auto ws = torch::empty({need}, h.options().dtype(at::kByte));
+  check(lvllm_moe_route(ids.data_ptr<int>(), weights.data_ptr<float>(), offsets.data_ptr<int>(), token.data_ptr<int>(),
+                        slot.data_ptr<int>(), tiles.data_ptr<int>(), (int)max_tiles, h.data_ptr(), w.data_ptr(),
+                        bias.data_ptr<float>(), (int)experts, shared, (int)top, (int)rows, (int)width, packed, ws.data_ptr(),
+                        need, dtype_code(h, op), current_stream(h)));
+  return {ids, weights, offsets, token, slot, tiles};
 }
 
 torch::Tensor moe_experts(const torch::Tensor& x, const torch::Tensor& w, const torch::Tensor& w_offset,
@@ -318,10 +310,9 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, latent) {
   latent.impl("latent_expand", torch::kCUDA, &latent_expand);
   latent.def("latent_rotate_query(Tensor q, int heads, int dim, int kpad, Tensor positions, Tensor turns) -> Tensor");
   latent.impl("latent_rotate_query", torch::kCUDA, &latent_rotate_query);
-  latent.def("moe_route(Tensor h, Tensor w, Tensor bias, int top, bool shared, bool packed) -> (Tensor, Tensor)");
+  latent.def("moe_route(Tensor h, Tensor w, Tensor bias, int top, bool shared, bool packed) "
+             "-> (Tensor, Tensor, Tensor, Tensor, Tensor, Tensor)");
   latent.impl("moe_route", torch::kCUDA, &moe_route);
-  latent.def("moe_group(Tensor ids, int experts, bool shared, bool packed) -> (Tensor, Tensor, Tensor, Tensor)");
-  latent.impl("moe_group", torch::kCUDA, &moe_group);
   latent.def("moe_experts(Tensor x, Tensor w, Tensor w_offset, Tensor ff, Tensor limit, Tensor offsets, Tensor token, "
              "Tensor tiles, int rows, int width, int ff_max, int ff_first, int ff_last, bool up, bool packed) "
              "-> Tensor");

@@ -213,9 +213,8 @@ class MixtureOfExperts:
         return self.up.numel() + self.down.numel()
 
     def __call__(self, h: torch.Tensor) -> SublayerOutput:
-        shared = self.cfg.shared is not None
-        ids, weights = amd.moe_route(h, self.router, self.bias, self.cfg.top, shared, self.packed)
-        offsets, token, slots, tiles = amd.moe_group(ids, self.experts, shared, self.packed)
+        _, weights, offsets, token, slots, tiles = amd.moe_route(h, self.router, self.bias, self.cfg.top,
+                                                                 self.cfg.shared is not None, self.packed)
         rows = h.shape[0]
         sizes = rows, self.width, self.ff_max, self.ff_first, self.ff_last
         a = amd.moe_experts(h, self.up, self.up_at, self.ff, self.limits, offsets, token, tiles, *sizes, True, self.packed)

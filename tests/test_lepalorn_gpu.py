@@ -340,13 +340,13 @@ def test_router(amd, dtype, experts, width):
         packed = dtype == BF16 and width % 32 == 0
         wd = amd.pack_weight(F_rows(w, 16).to(DEV)) if packed else w.to(DEV)
         for top in (1, 3, 5):
-            ids, weights = amd.moe_route(h.to(DEV), wd, b.to(DEV), top, True, packed)
+            ids, weights, *_ = amd.moe_route(h.to(DEV), wd, b.to(DEV), top, True, packed)
             want_ids, want_w = lepalorn.route(z[:, :experts] + b.double(), top)
             assert torch.equal(ids[:, :top].long().cpu(), want_ids) and (ids[:, top] == experts).all()
             close(weights[:, :top], want_w, 1e-5)
             close(weights[:, top], torch.sigmoid(z[:, experts]), 1e-5)
     # equal logits: the smaller numbers
-    ids, weights = amd.moe_route(torch.zeros(2, width, dtype=dtype, device=DEV), wd, torch.zeros(experts, device=DEV), 4, True, packed)
+    ids, weights, *_ = amd.moe_route(torch.zeros(2, width, dtype=dtype, device=DEV), wd, torch.zeros(experts, device=DEV), 4, True, packed)
     assert ids[:, :4].tolist() == [[0, 1, 2, 3]] * 2 and (weights == torch.tensor([0.25] * 4 + [0.5], device=DEV)).all()
 
 
