@@ -26,33 +26,34 @@ __device__ __forceinline__ void write_latent_row(const LatentCacheParams& p, int
   using S = typename T::store_t;
   constexpr int X = 16 / sizeof(S);
   const int lane = threadIdx.x & 63;
-  const int64_t wide = p.slot_mapping[row];
+  const S* z = (const S*)p.kv + row * p.kv_stride;
+  const bool vec = p.kv_rank % X == 0 && p.kv_rank <= 64 * X && ((uintptr_t)z & 15) == 0;
+  const int64_t wide = p.slot_mapping[row], pos = p.positions[row];
+  Vec16<T> raw{};
+  float weight[X];
+#pragma unroll
+  for (int j = 0; j < X; ++j) weight[j] = 0.f;
+  if (vec && lane * X < p.kv_rank) {  // (asked for before the slot is known)
+    raw = *reinterpret_cast<const Vec16<T>*>(z + lane * X);
+#pragma unroll
+    for (int j = 0; j < X; ++j) weight[j] = p.weight[lane * X + j];
+  }
   if (wide < 0 || wide >= p.num_slots) return;
   const unsigned slot = (unsigned)wide, block = slot / (unsigned)p.block_size;
-  const S* z = (const S*)p.kv + row * p.kv_stride;
   S* out = (S*)p.cache + block * p.block_stride + (slot - block * p.block_size) * (int64_t)(p.cpad + p.rpad);
-  const int64_t pos = p.positions[row];
-  const bool vec = p.kv_rank % X == 0 && p.kv_rank <= 64 * X && ((uintptr_t)z & 15) == 0;
   float ss = 0.f;
   if (vec) {
-    const int i = lane * X;
-    Vec16<T> raw;
     float v[X];
 #pragma unroll
-    for (int j = 0; j < X; ++j) v[j] = 0.f;
-    if (i < p.kv_rank) {
-      raw = *reinterpret_cast<const Vec16<T>*>(z + i);
-#pragma unroll
-      for (int j = 0; j < X; ++j) {
-        v[j] = T::to_float(raw.v[j]);
-        ss = fmaf(v[j], v[j], ss);
-      }
+    for (int j = 0; j < X; ++j) {
+      v[j] = T::to_float(raw.v[j]);
+      ss = fmaf(v[j], v[j], ss);
     }
     const float f = 1.f / sqrtf(wave_sum(ss) / (float)p.kv_rank + p.eps);
-    if (i < p.cpad) {
+    if (lane * X < p.cpad) {
 #pragma unroll
-      for (int j = 0; j < X; ++j) raw.v[j] = T::from_float(i < p.kv_rank ? v[j] * f * p.weight[i + j] : 0.f);
-      *reinterpret_cast<Vec16<T>*>(out + i) = raw;
+      for (int j = 0; j < X; ++j) raw.v[j] = T::from_float(v[j] * f * weight[j]);
+      *reinterpret_cast<Vec16<T>*>(out + lane * X) = raw;
     }
     for (int d = 64 * X + lane; d < p.cpad; d += 64) out[d] = T::from_float(0.f);
   } else {

@@ -94,80 +94,94 @@ __device__ __forceinline__ void choose_experts(const float* z, int experts, int 
   }
 }
 
-// Where the grouped assignments go: offsets [experts + 1], token and slot [assignments], tiles of `tile` slots.
+// Where the grouped assignments go: offsets [experts + 1], token and slot [assignments], tiles of `tile` slots.  count
+// [experts], zeroed: only for rows that count their own assignments (moe_count_assignments).
 struct MoeGroups {
-  int32_t *offsets, *token, *slot, *tiles;
+  int32_t *offsets, *token, *slot, *tiles, *count;
   int tile, max_tiles;
 };
 
-// Counts, offsets, slots and tiles of `total` assignments, by one workgroup of 1024.  `shared`: the last assignment of every
-// row is the last expert's, in row order.
-__device__ __forceinline__ void group_assignments(const int32_t* ids, const int total, const int per_row, const int experts,
-                                                  const int shared, const MoeGroups& out) {
-  int32_t *offsets = out.offsets, *token = out.token, *slot = out.slot, *tiles = out.tiles;
-  const int tile = out.tile, max_tiles = out.max_tiles;
-  __shared__ int count[kMaxExperts + 1], first[kMaxExperts + 2], tile0[kMaxExperts + 2];
-  for (int e = threadIdx.x; e < experts; e += 1024) count[e] = shared && e == experts - 1 ? total / per_row : 0;
-  __syncthreads();
-  constexpr int B = 8;  // loads in flight
-  for (int i0 = threadIdx.x; i0 < total; i0 += 1024 * B) {
-    int e[B];
+// Running sums of the experts' slots and tiles, 64 experts a turn, by the first wave; count, first [experts + 1] and tile0
+// [experts + 1] in LDS.
+__device__ __forceinline__ void moe_running_sums(const int* count, int* first, int* tile0, int experts, int tile) {
+  if (threadIdx.x >= 64) return;
+  int base = 0, tbase = 0;
+  for (int e0 = 0; e0 < experts; e0 += 64) {
+    const int e = e0 + threadIdx.x;
+    const int c = e < experts ? count[e] : 0, t = (c + tile - 1) / tile;
+    int s = c, ts = t;
 #pragma unroll
-    for (int j = 0; j < B; ++j) e[j] = i0 + 1024 * j < total ? min(max(ids[i0 + 1024 * j], 0), experts - 1) : -1;
-#pragma unroll
-    for (int j = 0; j < B; ++j)
-      if (e[j] >= 0) e[j] = shared && e[j] == experts - 1 ? (i0 + 1024 * j) / per_row : atomicAdd(&count[e[j]], 1);
-#pragma unroll
-    for (int j = 0; j < B; ++j)
-      if (i0 + 1024 * j < total) slot[i0 + 1024 * j] = e[j];
-  }
-  __syncthreads();
-  if (threadIdx.x < 64) {  // running sums, 64 experts a turn
-    int base = 0, tbase = 0;
-    for (int e0 = 0; e0 < experts; e0 += 64) {
-      const int e = e0 + threadIdx.x;
-      const int c = e < experts ? count[e] : 0, t = (c + tile - 1) / tile;
-      int s = c, ts = t;
-#pragma unroll
-      for (int d = 1; d < 64; d <<= 1) {
-        const int a = __shfl_up(s, d), b = __shfl_up(ts, d);
-        if ((int)threadIdx.x >= d) { s += a; ts += b; }
-      }
-      if (e < experts) { first[e] = base + s - c; tile0[e] = tbase + ts - t; }
-      base += __shfl(s, 63);
-      tbase += __shfl(ts, 63);
+    for (int d = 1; d < 64; d <<= 1) {
+      const int a = __shfl_up(s, d), b = __shfl_up(ts, d);
+      if ((int)threadIdx.x >= d) { s += a; ts += b; }
     }
-    if (threadIdx.x == 0) { first[experts] = base; tile0[experts] = tbase; }
+    if (e < experts) { first[e] = base + s - c; tile0[e] = tbase + ts - t; }
+    base += __shfl(s, 63);
+    tbase += __shfl(ts, 63);
   }
-  __syncthreads();
-  for (int e = threadIdx.x; e <= experts; e += 1024) offsets[e] = first[e];
-  for (int i0 = threadIdx.x; i0 < total; i0 += 1024 * B) {
-    int e[B], s[B];
-#pragma unroll
-    for (int j = 0; j < B; ++j) {
-      const int i = min(i0 + 1024 * j, total - 1);
-      e[j] = min(max(ids[i], 0), experts - 1);
-      s[j] = slot[i];
-    }
-#pragma unroll
-    for (int j = 0; j < B; ++j) {
-      const int i = i0 + 1024 * j;
-      if (i >= total) break;
-      slot[i] = first[e[j]] + s[j];
-      token[first[e[j]] + s[j]] = i / per_row;
-    }
-  }
-  for (int e = threadIdx.x; e < experts; e += 1024)
-    for (int t = tile0[e]; t < tile0[e + 1] && t < max_tiles; ++t) {
+  if (threadIdx.x == 0) { first[experts] = base; tile0[experts] = tbase; }
+}
+
+// offsets and tiles, by the whole workgroup
+__device__ __forceinline__ void moe_write_tiles(const int* first, const int* tile0, int experts, const MoeGroups& out) {
+  int32_t* tiles = out.tiles;
+  for (int e = threadIdx.x; e <= experts; e += blockDim.x) out.offsets[e] = first[e];
+  for (int e = threadIdx.x; e < experts; e += blockDim.x)
+    for (int t = tile0[e]; t < tile0[e + 1] && t < out.max_tiles; ++t) {
       tiles[4 * t] = e;
-      tiles[4 * t + 1] = first[e] + (t - tile0[e]) * tile;
+      tiles[4 * t + 1] = first[e] + (t - tile0[e]) * out.tile;
       tiles[4 * t + 2] = tile0[e];
       tiles[4 * t + 3] = tile0[e + 1] - tile0[e];
     }
-  for (int t = tile0[experts] + threadIdx.x; t < max_tiles; t += 1024) tiles[4 * t] = -1;
+  for (int t = tile0[experts] + threadIdx.x; t < out.max_tiles; t += blockDim.x) tiles[4 * t] = -1;
   if (threadIdx.x == 0) {
-    tiles[4 * max_tiles] = min(tile0[experts - 1], max_tiles);
-    tiles[4 * max_tiles + 1] = min(tile0[experts], max_tiles);
+    tiles[4 * out.max_tiles] = min(tile0[experts - 1], out.max_tiles);
+    tiles[4 * out.max_tiles + 1] = min(tile0[experts], out.max_tiles);
+  }
+}
+
+// Everything of `total` assignments, by one workgroup of 1024.  `shared`: the last assignment of every row is the last
+// expert's, in row order.
+__device__ __forceinline__ void group_assignments(const int32_t* ids, const int total, const int per_row, const int experts,
+                                                  const int shared, const MoeGroups& out) {
+  __shared__ int count[kMaxExperts + 1], first[kMaxExperts + 2], tile0[kMaxExperts + 2];
+  for (int e = threadIdx.x; e < experts; e += 1024) count[e] = shared && e == experts - 1 ? total / per_row : 0;
+  __syncthreads();
+  for (int i = threadIdx.x; i < total; i += 1024) {
+    const int e = min(max(ids[i], 0), experts - 1);
+    out.slot[i] = shared && e == experts - 1 ? i / per_row : atomicAdd(&count[e], 1);
+  }
+  __syncthreads();
+  moe_running_sums(count, first, tile0, experts, out.tile);
+  __syncthreads();
+  for (int i = threadIdx.x; i < total; i += 1024) {
+    const int s = first[min(max(ids[i], 0), experts - 1)] + out.slot[i];
+    out.slot[i] = s;
+    out.token[s] = i / per_row;
+  }
+  moe_write_tiles(first, tile0, experts, out);
+}
+
+// Many rows: a workgroup that has chosen for rows row0 .. row0 + n - 1 counts their assignments -- in LDS (`local`, experts
+// long), then once per expert in memory -- and leaves every assignment's rank among its expert's in `slot`; the running sums
+// and the final slots are a launch each (launch_moe_group).
+__device__ __forceinline__ void moe_count_assignments(const int32_t* ids, int row0, int n, int per_row, int experts, int shared,
+                                                      int* local, const MoeGroups& out) {
+  for (int e = threadIdx.x; e < experts; e += blockDim.x) local[e] = 0;
+  __syncthreads();
+  const int total = n * per_row;
+  for (int i = threadIdx.x; i < total; i += blockDim.x) {
+    const int at = row0 * per_row + i, e = min(max(ids[at], 0), experts - 1);
+    const bool last = shared && e == experts - 1;
+    out.slot[at] = last ? row0 + i / per_row : atomicAdd(&local[e], 1);
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < experts; e += blockDim.x)
+    if (local[e] > 0) local[e] = atomicAdd(&out.count[e], local[e]);
+  __syncthreads();
+  for (int i = threadIdx.x; i < total; i += blockDim.x) {
+    const int at = row0 * per_row + i, e = min(max(ids[at], 0), experts - 1);
+    if (!(shared && e == experts - 1)) out.slot[at] += local[e];
   }
 }
 
@@ -177,7 +191,9 @@ inline int moe_tile(bool packed, int rows) { return packed && rows > kMoeFewRows
 
 bool moe_takes_mfma(int width, int dtype);
 int launch_moe_mfma(const MoeParams& p, bool up, hipStream_t s);
-int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, const MoeGroups& groups, hipStream_t s);
+// `counted`: the rows have counted their assignments
+int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, bool counted, const MoeGroups& groups,
+                     hipStream_t s);
 int64_t moe_route_mfma_workspace(int experts, int shared, int rows, int width);
 int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
                           int top, int rows, int width, const MoeGroups& groups, float* workspace, hipStream_t s);

@@ -40,8 +40,33 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t* ids, con
   group_assignments(ids, total, per_row, experts, shared, groups);
 }
 
-int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, const MoeGroups& groups, hipStream_t s) {
-  hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, s, ids, total, per_row, experts, shared, groups);
+__global__ __launch_bounds__(256) void moe_tiles_kernel(const int experts, const int shared, const int rows, const MoeGroups groups) {
+  __shared__ int count[kMaxExperts + 1], first[kMaxExperts + 2], tile0[kMaxExperts + 2];
+  for (int e = threadIdx.x; e < experts; e += 256) count[e] = shared && e == experts - 1 ? rows : groups.count[e];
+  __syncthreads();
+  moe_running_sums(count, first, tile0, experts, groups.tile);
+  __syncthreads();
+  moe_write_tiles(first, tile0, experts, groups);
+}
+
+__global__ __launch_bounds__(256) void moe_slots_kernel(const int32_t* __restrict__ ids, const int total, const int per_row,
+                                                        const int experts, const MoeGroups groups) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int s = min(max(groups.offsets[min(max(ids[i], 0), experts - 1)] + groups.slot[i], 0), total - 1);
+  groups.slot[i] = s;
+  groups.token[s] = i / per_row;
+}
+
+int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, bool counted, const MoeGroups& groups,
+                     hipStream_t s) {
+  if (counted) {
+    hipLaunchKernelGGL(moe_tiles_kernel, dim3(1), dim3(256), 0, s, experts, shared, total / per_row, groups);
+    LV_LAUNCH_CHECK();
+    hipLaunchKernelGGL(moe_slots_kernel, dim3((total + 255) / 256), dim3(256), 0, s, ids, total, per_row, experts, groups);
+  } else {
+    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, s, ids, total, per_row, experts, shared, groups);
+  }
   LV_LAUNCH_CHECK();
   return 0;
 }
@@ -106,7 +131,7 @@ extern "C" int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, i
   LV_CHECK(workspace_bytes >= lvllm_moe_route_workspace_bytes(experts, shared, rows, width, packed), "workspace too small");
   hipStream_t s = (hipStream_t)stream;
   shared = shared != 0;
-  const MoeGroups groups{offsets, token, slot, tiles, lvllm_moe_tile(packed, rows), max_tiles};
+  const MoeGroups groups{offsets, token, slot, tiles, (int32_t*)workspace, moe_tile(packed != 0, rows), max_tiles};
   if (packed) {
     LV_CHECK(moe_takes_mfma(width, dtype), "packed router: bf16, a width that is a multiple of 32");
     return launch_moe_route_mfma(ids, weights, h, w, bias, experts, shared, top, rows, width, groups, (float*)workspace, s);
@@ -121,7 +146,7 @@ extern "C" int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, i
                          bias, experts, shared, top, width);
   });
   LV_LAUNCH_CHECK();
-  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, groups, s);
+  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, false, groups, s);
 }
 
 extern "C" int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff,

@@ -300,10 +300,11 @@ __device__ __forceinline__ void route_logits(float* z, int ld, e_f32x4_t* red, c
 }
 
 // many rows: logits and choice in one launch, a wave chooses for two rows
-__global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
+__global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* ids, float* __restrict__ weights,
                                                              const uint16_t* __restrict__ h, const uint16_t* __restrict__ w,
                                                              const float* __restrict__ bias, const int experts,
-                                                             const int shared, const int top, const int rows, const int width) {
+                                                             const int shared, const int top, const int rows, const int width,
+                                                             const MoeGroups groups) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   float* z = reinterpret_cast<float*>(smem + kRouteLds);
   const int ntiles = (experts + shared + 15) >> 4, ld = ntiles * 16 + 1, row0 = blockIdx.x * 16, n = top + shared;
@@ -314,6 +315,12 @@ __global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* __restrict
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (the wave's own next reads see it)
     choose_experts(z + r * ld, experts, top, shared != 0, ids + (int64_t)(row0 + r) * n, weights + (int64_t)(row0 + r) * n);
   }
+  __syncthreads();  // (the logits' partial sums make room for the counts)
+  moe_count_assignments(ids, row0, min(16, rows - row0), n, experts + shared, shared, reinterpret_cast<int*>(smem), groups);
+}
+
+__global__ __launch_bounds__(256) void moe_zero_kernel(int32_t* __restrict__ p, const int n) {
+  for (int i = threadIdx.x; i < n; i += 256) p[i] = 0;
 }
 
 // few rows: the k-steps are dealt to workgroups as well (grid.y), whose logits leave as part [share][16-row tiles][16][ld]
@@ -359,7 +366,7 @@ static int route_shares(int width) {
 }
 
 int64_t moe_route_mfma_workspace(int experts, int shared, int rows, int width) {
-  if (rows > kMoeFewRows) return 0;
+  if (rows > kMoeFewRows) return (int64_t)(experts + shared) * 4;  // (the experts' counts)
   return (int64_t)route_shares(width) * ((rows + 15) / 16) * 16 * ((experts + shared + 15) / 16 * 16) * 4;
 }
 
@@ -381,10 +388,12 @@ int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const voi
   }
   const int lds = kRouteLds + 16 * (ntiles * 16 + 1) * 4;
   (void)hipFuncSetAttribute((const void*)moe_route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  hipLaunchKernelGGL(moe_route_mfma_kernel, dim3(row_tiles), dim3(512), lds, s, ids, weights, (const uint16_t*)h,
-                     (const uint16_t*)w, bias, experts, shared, top, rows, width);
+  hipLaunchKernelGGL(moe_zero_kernel, dim3(1), dim3(256), 0, s, groups.count, experts + shared);
   LV_LAUNCH_CHECK();
-  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, groups, s);
+  hipLaunchKernelGGL(moe_route_mfma_kernel, dim3(row_tiles), dim3(512), lds, s, ids, weights, (const uint16_t*)h,
+                     (const uint16_t*)w, bias, experts, shared, top, rows, width, groups);
+  LV_LAUNCH_CHECK();
+  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, true, groups, s);
 }
 
 bool moe_takes_mfma(int width, int dtype) { return dtype == LVLLM_BF16 && width % 32 == 0; }

@@ -140,7 +140,8 @@ class LatentModelConfig:
         total = (len(self.layers) + 1) * rows * w * 4
         for l in self.layers:
             m = l.mixer
-            total += rows * (m.heads * (m.dim + m.rot_dim + m.vdim + m.spec.row + 66 * m.spec.cpad) + m.spec.row + 4 * w) * 4
+            total += rows * (m.heads * (m.dim + m.rot_dim + m.vdim + m.spec.row) + m.spec.row + 4 * w) * 4
+            total += (rows * m.heads + 512 * 32) * (m.spec.cpad + 2) * 4  # shares of the attention
             if l.mlp is not None:
                 n = l.mlp.top + 1
                 ff = max(l.mlp.expert.ff, l.mlp.shared.ff if l.mlp.shared is not None else 0)

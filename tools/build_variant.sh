@@ -10,7 +10,7 @@ d=build/$name; mkdir -p $d
 objs=$(ls build/obj/*.o | grep -v "/$stem.o")
 extra=""
 [ "$stem" = "prefill_attention" ] && extra="-fno-honor-nans"
-/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off $extra "$@" \
+/opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -Xclang -target-feature -Xclang -packed-fp32-ops $extra "$@" \
   -c light-vllm_amd/csrc/$src -o $d/$stem.o
 /opt/rocm/bin/hipcc --offload-arch=gfx950 -shared -fPIC -o $d/liblvllm_hip.so $objs $d/$stem.o
 echo $d/liblvllm_hip.so
