@@ -2,6 +2,7 @@
 most of a softmax row; gains, limits and depth averages of their own in every layer)."""
 import functools
 
+import pytest
 import torch
 
 from layered_case import tokens
@@ -106,3 +107,57 @@ def expected(name, n, seed):
     cfg, w = case(name)
     t = tokens(cfg, n, seed)
     return t, lepalorn.forward(cfg, w, t)
+
+
+def rand(*shape, seed=0):
+    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed))
+
+
+def mixer_case(sizes, seed=0):
+    """(configuration of one mixer, its weights by name)"""
+    heads, dim, rot, dims, vdim, rank = sizes
+    cfg = layer(heads, dim, rot, vdim, rank, 0, 2.5 * (dim + rot) ** -0.5, 3e3, rot_dims=dims)["mixer"]
+    width = 64
+    w = {"q": rand(heads * (dim + rot), width, seed=seed + 1) / 8, "g": rand(heads, width, seed=seed + 2) / 16,
+         "dkv": rand(rank + rot, width, seed=seed + 3) / 8, "dkv.norm": 1 + 0.2 * rand(rank, seed=seed + 4),
+         "uk": rand(heads * dim, rank, seed=seed + 5) * rank ** -0.5, "uv": rand(heads * vdim, rank, seed=seed + 6) * rank ** -0.5,
+         "o": rand(width, heads * vdim, seed=seed + 7) * (heads * vdim) ** -0.5}
+    return cfg, {k: t.bfloat16().float() for k, t in w.items()}
+
+
+def edge_inputs(cfg, w, n, window, seed):
+    """Rows of one sequence whose last token's first head looks for two keys: the first its window has and the one before
+    that.  Their latents point along the query (and differ in what is left), so that each would carry most of the softmax."""
+    x = rand(n, w["q"].shape[1], seed=seed).double()
+    x[-1] *= 2  # (latents are normed: the query alone decides how far the best key is ahead)
+    q = w["q"][:cfg["dim"]].double() @ x[-1]
+    latent = (w["uk"][:cfg["dim"]].double() * w["dkv.norm"].double()).T @ q
+    want = torch.linalg.lstsq(w["dkv"][:cfg["kv_rank"]].double(), latent[:, None]).solution[:, 0]
+    want = want / want.norm() * x.shape[1] ** 0.5
+    for j, other in ((n - window, 0.8), (n - 1 - window, 0.1)):  # (the one outside would win)
+        if 0 <= j < n - 1:
+            x[j] = want + other * x[j]
+    return x.bfloat16().float()
+
+
+def dense_mixer(h, m, w, lat, window):
+    """lepalorn.latent_attention with the softmax over a masked matrix (its own loop takes every row and head)."""
+    def attention(q, k, v, scale, size):
+        i = torch.arange(q.shape[0])
+        seen = (i[:, None] >= i[None]) & (i[:, None] - i[None] < size)
+        s = (q.transpose(0, 1) @ k.permute(1, 2, 0) * scale).masked_fill(~seen, float("-inf"))
+        return (s.softmax(-1) @ v.transpose(0, 1)).transpose(0, 1)
+    with pytest.MonkeyPatch.context() as mp:
+        mp.setattr(lepalorn, "window_attention", attention)
+        mp.setattr(lepalorn, "rotate", fast_rotate)
+        return lepalorn.latent_attention(h, dict(m, mask={"size": window}), lambda s: w[s].double(), lat)
+
+
+def fast_rotate(x, positions, dims, base):
+    p = torch.tensor(list(positions), dtype=torch.float64)
+    a = p[:, None] * base ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims)
+    a = a.view(x.shape[0], *[1] * (x.dim() - 2), -1)
+    out = x.clone()
+    u, v = x[..., 0:dims:2], x[..., 1:dims:2]
+    out[..., 0:dims:2], out[..., 1:dims:2] = u * a.cos() - v * a.sin(), v * a.cos() + u * a.sin()
+    return out

@@ -202,3 +202,19 @@ def test_planted_mistakes_show():
         assert changed(patch=patch) > 1e-2, patch.__name__
     assert changed(lambda c: c["layers"][4]["mixer"].update(kv_from=2) or c["embedding"].update(scale=3.1)) > 1e-3
     assert changed(lambda c: c["norm"].update(eps=1e-2)) > 1e-4
+
+
+@pytest.mark.parametrize("window", [1, 16, 50])
+@pytest.mark.parametrize("sizes", [(3, 24, 16, 16, 40, 48), (16, 128, 64, 64, 128, 512)])
+def test_edge_inputs_show_both_sides_of_a_window(sizes, window):
+    """The inputs the operator tests use: a window one token longer or shorter changes the last row by far more than they
+    allow."""
+    cfg, w = lc.mixer_case(sizes)
+    h = lc.edge_inputs(cfg, w, 90, window, 5).double()
+    lat = lepalorn.latent_parts(h, cfg, lambda s: w[s].double(), 1e-5)
+    want = lc.dense_mixer(h, cfg, w, lat, window)[-1]
+    assert torch.allclose(want, lepalorn.latent_attention(h, dict(cfg, mask={"size": window}), lambda s: w[s].double(), lat)[-1])
+    for other in (window - 1, window + 1):
+        if other > 0:
+            got = lc.dense_mixer(h, cfg, w, lat, other)[-1]
+            assert (got - want).abs().max() > 0.12 * want.abs().max(), other
