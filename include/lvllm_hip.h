@@ -609,19 +609,29 @@ int lvllm_recurrent_mix(void* out, int64_t out_stride, const void* q, const void
                         const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows, int heads, int dk,
                         int dv, int max_query_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 /* Causal attention over the cache of lvllm_qk_norm_cache; q [rows, heads, kpad];
- * out[row, h * vdim + d] = T(attention * sigmoid(gate[row, h]) * out_scale), gate null: no gate.  A query sees the keys of the
- * last `window` positions, its own included (window <= 0: all before it); sequences of fewer than min_query_len query tokens
- * are left alone.  max_query_len and
- * max_seq_len bound the step's query_len and seq_lens.  bf16 with block size 16, kpad in {64, 96, 128, 192, 256} and vpad
- * in {32, 64, 96, 128, 192, 256} run on MFMAs; every other case on a plain fp32 body. */
+ * out[row, h * vdim + d] = T(attention * sigmoid(gate[row, h]) * out_scale), gate null: no gate.  Options (csrc/head_attention.h):
+ *   window, chunk  a query sees the last `window` positions, its own included, and of those the ones in its own aligned run of
+ *                  `chunk` positions (<= 0: not limited)
+ *   keep_first     the first keys of a sequence, seen by all queries behind them
+ *   maps           2: queries and keys hold two vectors of kpad / 2, whose softmaxes' results a, b become the per-head RMS
+ *                  normed a - map_weight * b
+ *   min_query_len  sequences of fewer query tokens are left alone
+ *   softcap        > 0: score = softcap * tanh(score / softcap);  sink [heads], fp32 (null: none): a score without a key
+ * max_query_len and max_seq_len bound the step's query_len and seq_lens.  bf16 with block size 16, kpad in {64, 96 (one map),
+ * 128, 192, 256} and vpad in {32, 64, 96, 128, 192, 256} run on MFMAs; every other case on a plain fp32 body. */
+typedef struct lvllm_head_options {
+  int window, chunk, keep_first, maps, min_query_len;
+  float softcap, map_weight, map_eps;
+  const float* sink;
+} lvllm_head_options;
 int64_t lvllm_head_attention_workspace_bytes(int rows, int num_seqs, int heads, int kv_heads, int kpad, int vpad,
-                                             int block_size, int max_seq_len, int dtype);
+                                             int block_size, int max_seq_len, const lvllm_head_options* options, int dtype);
 int lvllm_head_attention(void* out, int64_t out_stride, const void* q, const void* key_cache, const void* value_cache,
                          const void* gate, int64_t gate_stride, const int32_t* block_tables, const int32_t* seq_lens,
                          const int32_t* query_start_loc, int num_seqs, int rows, int heads, int kv_heads, int kpad, int vpad,
                          int vdim, int max_blocks, int block_size, int64_t num_blocks, float scale, float out_scale,
-                         int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len, int window, int min_query_len,
-                         void* workspace, int64_t workspace_bytes, int dtype, void* stream);
+                         int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len,
+                         const lvllm_head_options* options, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 
 /* ---- latent decoders (csrc/latent_attention*.hip, moe*.hip, depth_mix.hip) ----
  * Rows of a step as for the hybrid decoders.  dtype: LVLLM_F32 or LVLLM_BF16.  csrc/latent_attention.h, csrc/moe.h and
@@ -668,20 +678,74 @@ int lvllm_latent_expand(void* key_pages, void* value_pages, const void* kv, int6
                         int cpad, int n, int heads, int dim, int rot_dim, int vdim, int kpad, int vpad, int dtype, void* stream);
 int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_stride, int heads, int dim, int rot_dim, int kpad,
                               const int64_t* positions, const double* turns, int rot_dims, int rows, int dtype, void* stream);
-/* the `top` experts of every row and their softmax weights; with `shared` a last assignment, expert number `experts`, weighted
- * sigmoid of the last row of w.  The assignments come grouped by expert: offsets [experts + shared + 1], token and slot
- * [assignments], tiles [max_tiles + 1, 4] of lvllm_moe_tile slots.  `packed`: w as lvllm_pack_weight leaves it, rows padded to a
- * multiple of 16 */
+/* ---- mixtures of experts (csrc/moe*.hip, moe.h) ---- */
+enum { LVLLM_MOE_SOFTMAX = 0, LVLLM_MOE_SIGMOID = 1 };  /* weights: softmax over the chosen logits, or each logit's sigmoid */
+enum { LVLLM_MOE_NO_SHARED = 0, LVLLM_MOE_GATED_SHARED = 1, LVLLM_MOE_PLAIN_SHARED = 2 };
+enum { LVLLM_MOE_CLAMPED = 0, LVLLM_MOE_SILU = 1 };     /* activations */
+typedef struct lvllm_moe_routing {
+  int experts, top, scoring, shared;
+} lvllm_moe_routing;
+/* the `top` experts of every row and their weights; with a shared one a last assignment, expert number `experts`, weighted by the
+ * sigmoid of the last row of w (GATED) or 1 (PLAIN).  bias null: none.  The assignments come grouped by expert: offsets [experts +
+ * shared + 1], token and slot [assignments], tiles [max_tiles + 1, 4] of lvllm_moe_tile slots, slot_weight [assignments] (null:
+ * not kept).  `packed`: w as lvllm_pack_weight leaves it, rows padded to a multiple of 16 */
 int lvllm_moe_tile(int packed, int rows);
-int64_t lvllm_moe_route_workspace_bytes(int experts, int shared, int rows, int width, int packed);
-int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles, int max_tiles,
-                    const void* h, const void* w, const float* bias, int experts, int shared, int top, int rows, int width,
-                    int packed, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
-/* the experts' products: up (with the activation) [rows, width] -> [slots, ff_max], down [slots, ff_max] -> [slots, width] */
+int64_t lvllm_moe_route_workspace_bytes(const lvllm_moe_routing* routing, int rows, int width, int packed);
+int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, int32_t* token, int32_t* slot, float* slot_weight,
+                    int32_t* tiles, int max_tiles, const void* h, const void* w, const float* bias,
+                    const lvllm_moe_routing* routing, int rows, int width, int packed, void* workspace, int64_t workspace_bytes,
+                    int dtype, void* stream);
+/* the experts' products: up (with the activation) [rows, width] -> [slots, ff_max], down [slots, ff_max] -> [slots, width].
+ * slot_weight not null: it scales what the experts read.  limit: of LVLLM_MOE_CLAMPED */
 int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff, const float* limit,
-                      const int32_t* offsets, const int32_t* token, const int32_t* tiles, int experts, int slots, int rows,
-                      int width, int ff_max, int ff_first, int ff_last, int max_tiles, int up, int packed, int dtype,
-                      void* stream);
+                      const float* slot_weight, int act, const int32_t* offsets, const int32_t* token, const int32_t* tiles,
+                      int experts, int slots, int rows, int width, int ff_max, int ff_first, int ff_last, int max_tiles, int up,
+                      int packed, int dtype, void* stream);
+
+/* ---- local decoders (csrc/head_cache.hip, retention.hip, sandwich_norm.hip) ----
+ * Rows of a step as for the hybrid decoders.  dtype: LVLLM_F32 or LVLLM_BF16. */
+
+/* as lvllm_qk_norm_cache, with rotary positions (entry i of a vector with entry i + rot_dims / 2, turns [rot_dims / 2] full turns
+ * per position) and RMS norms over all of a row's queries and keys at once (weights [heads * maps * dim] and
+ * [kv_heads * maps * dim], null: none).  maps: vectors per head, each padded to kpad / maps.  v may be k: the keys as projected */
+int lvllm_rotary_cache(void* q_out, void* key_cache, void* value_cache, const void* q, const void* k, const void* v,
+                       int64_t row_stride, const float* q_weight, const float* k_weight, float eps, int rows, int heads,
+                       int kv_heads, int maps, int dim, int vdim, int kpad, int vpad, const int64_t* positions,
+                       const double* turns, int rot_dims, const int64_t* slot_mapping, int64_t num_blocks, int block_size,
+                       int64_t k_block_stride, int64_t v_block_stride, int dtype, void* stream);
+/* lvllm_recurrent_mix with one decay per head (head_decay [2, heads]: the decays and their logarithms) over queries and keys
+ * that are rotated as above, in fp32.  norm_weight null: none */
+int64_t lvllm_retention_workspace_bytes(int rows, int num_seqs, int heads, int dk, int dv, int max_query_len);
+int lvllm_retention(void* out, int64_t out_stride, const void* q, const void* k, const void* v, int64_t q_stride,
+                    int64_t k_stride, int64_t v_stride, const int64_t* positions, const double* turns, int rot_dims,
+                    const float* head_decay, float q_scale, const void* gate, int64_t gate_stride, const float* norm_weight,
+                    int norm_head_stride, float eps, float out_scale, float* state, int64_t state_stride,
+                    const int32_t* state_slots, int num_slots, const int32_t* query_start_loc, const int32_t* seq_lens,
+                    int num_seqs, int rows, int heads, int dk, int dv, int max_query_len, void* workspace,
+                    int64_t workspace_bytes, int dtype, void* stream);
+/* what a sublayer returned: rows y, fp32 slabs `partials`, or the slots of a mixture, with an optional bias */
+typedef struct lvllm_sandwich_branch {
+  const void* y;
+  const float* partials;
+  const int32_t* slots;
+  const float *bias, *weight;
+  int num_partials, num_slots, total_slots;
+} lvllm_sandwich_branch;
+/* x += RMS norm(v) * weight, h = T(RMS norm(x) * next_weight); v: the branch, or half the sum of two branches' weighted norms */
+int lvllm_sandwich_norm(float* x, void* h, const lvllm_sandwich_branch* branches, int num_branches, const float* weight,
+                        const float* next_weight, float eps, int rows, int width, int dtype, void* stream);
+/* x = table[id] + pairs[(previous * mul_previous + id * mul_current) mod buckets], a sequence's first token: row `buckets`;
+ * h = T(RMS norm(x) * weight).  previous [slots]: the sequences' last tokens, read and updated.  pairs null: none */
+int lvllm_pair_embed(float* x, void* h, const void* table, const void* pairs, const int64_t* ids, int32_t* previous,
+                     const int32_t* state_slots, int num_slots, const int32_t* query_start_loc, const int32_t* seq_lens,
+                     int num_seqs, int64_t mul_previous, int64_t mul_current, int buckets, const float* weight, float eps,
+                     int rows, int vocab, int width, int dtype, void* stream);
+/* out[r, i] = g * sigmoid(1.702 g) * (u + 1), g = min(in[r, i], limit), u = clamp(in[r, d + i], -limit, limit) */
+int lvllm_clamped_unit(void* out, const void* in, int64_t rows, int d, float limit, int dtype, void* stream);
+/* ... of a decode projection's result, in its epilogue: w [gate rows | up rows] (N rows, packed or not), y [M, N / 2], gate and up
+ * rounded to T first.  The envelope of lvllm_skinny_gemm, N a multiple of 32 */
+int lvllm_skinny_gemm_clamped_unit(void* y, const void* x, const void* w, int M, int N, int K, int64_t ldx, int dtype,
+                                   int packed, float limit, void* workspace, int64_t workspace_bytes, void* stream);
 
 #ifdef __cplusplus
 }

@@ -2,9 +2,11 @@
 
   base    what every model needs: error plumbing, cache block movement, the weight-streaming GEMMs of decode steps, step
           inputs, the sampler
-  heads   softmax attention over paged caches of unequal key and value sizes (hybrid and latent decoders)
+  heads   softmax attention over paged caches of unequal key and value sizes, and what goes into them
+  moe     routers and grouped products of mixtures of experts
   hybrid  row-wise operators and recurrences of the hybrid decoders
-  latent  latent attention, mixtures of experts, norms on sublayer outputs and depth averages
+  latent  latent attention, norms on sublayer outputs and depth averages
+  local   retention, norms around sublayers, embeddings of token pairs (local decoders)
   full    the rest of the C-ABI of include/lvllm_hip.h (paged and prefill attention of the rotary decoders, norms, fp8); it
           needs all the others, so a handle on liblvllm_hip.so resolves every symbol of the header
 
@@ -30,9 +32,12 @@ ARCH = "gfx950"
 
 SOURCES = {
     "base": ["capi.hip", "cache.hip", "skinny_gemm.hip", "prepare_inputs.hip", "sampler.hip", "activation.hip"],
-    "heads": ["head_attention.hip", "head_attention_prefill.hip", "head_attention_decode.hip"],
+    "heads": ["head_attention.hip", "head_attention_prefill.hip", "head_attention_decode.hip", "head_attention_maps.hip",
+              "head_cache.hip"],
+    "moe": ["moe.hip", "moe_mfma.hip"],
     "hybrid": ["token_mix.hip", "recurrent.hip"],
-    "latent": ["latent_attention.hip", "latent_attention_mfma.hip", "moe.hip", "moe_mfma.hip", "depth_mix.hip"],
+    "latent": ["latent_attention.hip", "latent_attention_mfma.hip", "depth_mix.hip"],
+    "local": ["retention.hip", "sandwich_norm.hip"],
     "full": ["layernorm.hip", "pos_encoding.hip", "attention.hip", "attention_bf16.hip", "attention_f16.hip",
              "prefill_attention.hip", "fp8_quant.hip"],
 }

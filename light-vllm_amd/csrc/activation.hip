@@ -6,7 +6,7 @@
 //   before the T x T multiply).
 // Launch: flat grid over 16-byte chunks (not one block per token): at decode
 // batch sizes a per-token grid leaves most of the 256 CUs idle.
-#include "common.h"
+#include "row_ops.h"
 
 namespace lvllm {
 
@@ -118,6 +118,43 @@ extern "C" int lvllm_gelu(void* out, const void* x, int64_t numel, int dtype, vo
   else
     hipLaunchKernelGGL((lvllm::gelu_vec_kernel<lvllm::F16>), dim3(grid), dim3(threads), 0, (hipStream_t)stream,
                        (uint16_t*)out, (const uint16_t*)x, chunks);
+  LV_LAUNCH_CHECK();
+  return 0;
+}
+
+// The clamped unit of a feed-forward: out[r, i] = clamped_unit_of(in[r, i], in[r, d + i])
+namespace lvllm {
+template <typename T, int VEC>
+__global__ void clamped_unit_kernel(typename T::store_t* __restrict__ out, const typename T::store_t* __restrict__ in,
+                                    const int64_t pieces, const int per_row, const float limit) {
+  for (int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; idx < pieces; idx += (int64_t)gridDim.x * blockDim.x) {
+    const int64_t r = idx / per_row, at = 2 * r * per_row + (idx - r * per_row);
+    float g[VEC], u[VEC];
+    load_vec<T, VEC>(in + at * VEC, g);
+    load_vec<T, VEC>(in + (at + per_row) * VEC, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) g[j] = clamped_unit_of(g[j], u[j], limit);
+    store_vec<T, VEC>(out + idx * VEC, g);
+  }
+}
+}  // namespace lvllm
+
+extern "C" int lvllm_clamped_unit(void* out, const void* in, int64_t rows, int d, float limit, int dtype, void* stream) {
+  if (rows == 0 || d == 0) return 0;
+  const bool aligned = (((uintptr_t)out | (uintptr_t)in) & 15) == 0;
+  LV_DISPATCH_F32_BF16(dtype, {
+    using S = typename scalar_t::store_t;
+    constexpr int kWide = sizeof(S) == 2 ? 8 : 4;
+    const bool vec = aligned && d % kWide == 0;
+    const int64_t pieces = rows * (int64_t)(vec ? d / kWide : d), want = (pieces + 255) / 256;
+    const dim3 grid((unsigned)(want < 16384 ? want : 16384));
+    if (vec)
+      hipLaunchKernelGGL((lvllm::clamped_unit_kernel<scalar_t, kWide>), grid, dim3(256), 0, (hipStream_t)stream, (S*)out,
+                         (const S*)in, pieces, d / kWide, limit);
+    else
+      hipLaunchKernelGGL((lvllm::clamped_unit_kernel<scalar_t, 1>), grid, dim3(256), 0, (hipStream_t)stream, (S*)out,
+                         (const S*)in, pieces, d, limit);
+  });
   LV_LAUNCH_CHECK();
   return 0;
 }

@@ -180,6 +180,13 @@ __device__ __forceinline__ float relu_squared_of(float x) {
   return v * v;
 }
 
+// A sigmoid-gated linear unit whose gate is bounded above and whose value on both sides
+__device__ __forceinline__ float clamped_unit_of(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+}
+
 // The sequence that owns `row` of a step's token batch: the s with query_start_loc[s] <= row < query_start_loc[s + 1],
 // num_seqs for rows past the last sequence (padding).  Sequences without tokens own nothing.
 __device__ __forceinline__ int find_seq(const int32_t* __restrict__ query_start_loc, int num_seqs, int row) {

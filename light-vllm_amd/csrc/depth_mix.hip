@@ -7,7 +7,7 @@
 //
 // y comes as rows of T, as the fp32 split-K slabs of a decode GEMM, or as the slots of a mixture of experts: row r is
 // sum_i slot_weight[r, i] * y[slot[r, i]].
-#include "common.h"
+#include "row_ops.h"
 
 namespace lvllm {
 
@@ -26,21 +26,6 @@ struct DepthMixParams {
   float eps, out_eps;
 };
 
-template <typename T, int VEC>
-__device__ __forceinline__ void load_items(const typename T::store_t* p, float (&v)[VEC]) {
-  if constexpr (VEC == 4) load4<T>(p, v);
-  else v[0] = T::to_float(p[0]);
-}
-template <int VEC>
-__device__ __forceinline__ void load_f32(const float* p, float (&v)[VEC]) {
-  load_items<F32, VEC>(p, v);
-}
-template <typename T, int VEC>
-__device__ __forceinline__ void store_items(typename T::store_t* p, const float (&v)[VEC]) {
-  if constexpr (VEC == 4) store4<T>(p, v);
-  else p[0] = T::from_float(v[0]);
-}
-
 // A workgroup per row; a thread keeps its ITEMS groups of VEC columns in registers.  Everything that does not depend on the
 // norm -- the sublayer's output, the stream, the earlier streams -- is read before the reduction, several rows at a time.
 template <typename T, int VEC, int ITEMS>
@@ -56,7 +41,7 @@ __global__ __launch_bounds__(1024) void norm_add_mix_kernel(const DepthMixParams
   for (int it = 0; it < ITEMS; ++it) {
 #pragma unroll
     for (int j = 0; j < VEC; ++j) v[it][j] = x[it][j] = mix[it][j] = 0.f;
-    if (column(it) < p.width) load_f32<VEC>(p.x_in + base + column(it), x[it]);
+    if (column(it) < p.width) load_vec<F32, VEC>(p.x_in + base + column(it), x[it]);
   }
   auto add_rows = [&](float (&acc)[ITEMS][VEC], int n, auto weight_of, auto load) __attribute__((always_inline)) {
     for (int i0 = 0; i0 < n; i0 += B) {
@@ -83,20 +68,20 @@ __global__ __launch_bounds__(1024) void norm_add_mix_kernel(const DepthMixParams
     const int32_t* slots = p.slots + (int64_t)row * p.num_slots;
     const float* weights = p.slot_weights + (int64_t)row * p.num_slots;
     add_rows(v, p.num_slots, [&](int i) { return weights[i]; }, [&](int i, int c, float (&t)[VEC]) {
-      load_items<T, VEC>((const S*)p.y + (int64_t)min(max(slots[i], 0), p.total_slots - 1) * p.width + c, t);
+      load_vec<T, VEC>((const S*)p.y + (int64_t)min(max(slots[i], 0), p.total_slots - 1) * p.width + c, t);
     });
   } else if (p.partials != nullptr) {
     add_rows(v, p.num_partials, [](int) { return 1.f; }, [&](int i, int c, float (&t)[VEC]) {
-      load_f32<VEC>(p.partials + (int64_t)i * p.rows * p.width + base + c, t);
+      load_vec<F32, VEC>(p.partials + (int64_t)i * p.rows * p.width + base + c, t);
     });
   } else {
 #pragma unroll
     for (int it = 0; it < ITEMS; ++it)
-      if (column(it) < p.width) load_items<T, VEC>((const S*)p.y + base + column(it), v[it]);
+      if (column(it) < p.width) load_vec<T, VEC>((const S*)p.y + base + column(it), v[it]);
   }
   if (p.weights != nullptr)
     add_rows(mix, p.num_streams, [&](int i) { return p.weights[i]; }, [&](int i, int c, float (&t)[VEC]) {
-      load_f32<VEC>(p.streams + i * p.stream_stride + base + c, t);
+      load_vec<F32, VEC>(p.streams + i * p.stream_stride + base + c, t);
     });
   float ss = 0.f;
 #pragma unroll
@@ -112,13 +97,13 @@ __global__ __launch_bounds__(1024) void norm_add_mix_kernel(const DepthMixParams
     if (column(it) >= p.width) continue;
 #pragma unroll
     for (int j = 0; j < VEC; ++j) x[it][j] = fmaf(v[it][j], f, x[it][j]);
-    if (p.v_out != nullptr) store_items<F32, VEC>(p.v_out + base + column(it), x[it]);
+    if (p.v_out != nullptr) store_vec<F32, VEC>(p.v_out + base + column(it), x[it]);
 #pragma unroll
     for (int j = 0; j < VEC; ++j) {
       v[it][j] = fmaf(wv, x[it][j], mix[it][j]);
       so = fmaf(v[it][j], v[it][j], so);
     }
-    if (p.x_out != nullptr) store_items<F32, VEC>(p.x_out + base + column(it), v[it]);
+    if (p.x_out != nullptr) store_vec<F32, VEC>(p.x_out + base + column(it), v[it]);
   }
   float fo = 1.f;
   if (p.out_gain != nullptr) {
@@ -130,7 +115,7 @@ __global__ __launch_bounds__(1024) void norm_add_mix_kernel(const DepthMixParams
     if (column(it) >= p.width) continue;
 #pragma unroll
     for (int j = 0; j < VEC; ++j) v[it][j] *= fo;
-    store_items<T, VEC>((S*)p.h + base + column(it), v[it]);
+    store_vec<T, VEC>((S*)p.h + base + column(it), v[it]);
   }
 }
 
@@ -145,11 +130,11 @@ __global__ __launch_bounds__(256) void embed_scale_kernel(float* __restrict__ x,
   const int64_t base = (int64_t)row * width;
   for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
     float v[VEC];
-    load_items<T, VEC>(table + id * width + c, v);
+    load_vec<T, VEC>(table + id * width + c, v);
 #pragma unroll
     for (int j = 0; j < VEC; ++j) v[j] *= scale;
-    store_items<F32, VEC>(x + base + c, v);
-    store_items<T, VEC>(h + base + c, v);
+    store_vec<F32, VEC>(x + base + c, v);
+    store_vec<T, VEC>(h + base + c, v);
   }
 }
 

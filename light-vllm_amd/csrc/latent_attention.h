@@ -13,7 +13,7 @@
 //   q'     [rows, heads, cpad + rpad], the same row layout
 // Scores, softmax and accumulation are fp32.
 #pragma once
-#include "common.h"
+#include "rotation.h"
 
 namespace lvllm {
 
@@ -34,12 +34,5 @@ int launch_latent_mfma(const LatentAttnParams& p, hipStream_t s);
 
 // The first key position `pos` sees.
 __device__ __forceinline__ int first_key(int pos, int window) { return window > 0 ? max(0, pos - window + 1) : 0; }
-
-// Rotation of pairs (2i, 2i + 1) by position * turns full turns: the product is taken in double, so that far positions keep
-// the fp32 sine's own accuracy.
-__device__ __forceinline__ void rotation_of(int64_t position, double turns, float& c, float& s) {
-  const double t = (double)position * turns;
-  sincospif((float)(2.0 * (t - rint(t))), &s, &c);
-}
 
 }  // namespace lvllm

@@ -1,12 +1,15 @@
-// Mixture of experts for gfx950.  A token takes its `top` experts (softmax over the chosen logits) and, as one more
-// assignment, the shared expert with a gate of its own.  The step's assignments are grouped by expert: slot s of the grouped
-// order belongs to row token[s]; expert e owns slots offsets[e] .. offsets[e + 1].
+// Mixture of experts for gfx950.  A token takes the `top` experts of the largest logits, weighted by the softmax over the chosen
+// ones or each by its own sigmoid, and, as one more assignment, the shared expert, with a gate of its own or the weight 1.  The
+// step's assignments are grouped by expert: slot s of the grouped order belongs to row token[s]; expert e owns slots
+// offsets[e] .. offsets[e + 1].
 //
 // Expert weights are two matrices per expert in one buffer:
 //   up    [2 ffp, width]: 16 gate rows, 16 value rows, 16 gate rows, ... (ffp: the inner size, zero rows up to a multiple of 32)
 //   down  [width, ffp]
 // row-major or, where the matrix-core bodies run, packed as lvllm_pack_weight does.  The activation is
-//   g = min(gate, limit), u = clamp(value, -limit, limit), a = g * sigmoid(1.702 g) * (u + 1).
+//   g = min(gate, limit), u = clamp(value, -limit, limit), a = g * sigmoid(1.702 g) * (u + 1)   (LVLLM_MOE_CLAMPED), or
+//   a = gate * sigmoid(gate) * value                                                        (LVLLM_MOE_SILU)
+// where an assignment's weight may scale the expert's input, that is gate and value, instead of its output (slot_weight).
 #pragma once
 #include "common.h"
 
@@ -22,27 +25,51 @@ struct MoeParams {
   // [max_tiles + 1][4]: expert (< 0: none), first slot, the expert's first tile and its number of tiles; the last entry: tiles
   // of all experts but the last one, tiles of all
   const int32_t* tiles;
+  const float* slot_weight;  // [slots] or null
+  int act;                // LVLLM_MOE_CLAMPED or LVLLM_MOE_SILU
   int experts, slots, rows, width, ff_max, max_tiles;
   int ff_first, ff_last;  // largest ffp of all experts but the last, the last one's
 };
 
-__device__ __forceinline__ float clamped_gate(float g, float u, float limit) {
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+// gate and value of slot `slot` of expert e -> its activation
+struct MoeActivation {
+  float limit;
+  bool silu;
+  __device__ __forceinline__ MoeActivation(const MoeParams& p, int e) : limit(0.f), silu(p.act == LVLLM_MOE_SILU) {
+    if (!silu) limit = p.limit[e];
+  }
+  __device__ __forceinline__ float operator()(float g, float u) const {
+    return silu ? g / (1.f + expf(-g)) * u : clamped_unit_of(g, u, limit);
+  }
+};
+__device__ __forceinline__ float slot_weight_of(const MoeParams& p, int slot) {
+  return p.slot_weight != nullptr ? p.slot_weight[slot] : 1.f;
 }
+
+// How a token's assignments are found: experts and a last shared one (`gated`: weighted by its own logit's sigmoid)
+struct MoeRouting {
+  int experts, top, scoring;
+  bool shared, gated;
+  __host__ __device__ __forceinline__ int logits() const { return experts + gated; }
+  __host__ __device__ __forceinline__ int all() const { return experts + shared; }
+  __host__ __device__ __forceinline__ int per_row() const { return top + shared; }
+};
 
 constexpr int kMaxExperts = 1024;
 
-// The `top` largest of z[0 .. experts) (LDS; ties: the smaller index) by one wave, their softmax, and the shared expert.  NaNs
+// The `top` largest of z[0 .. experts) (LDS; ties: the smaller index) by one wave, their weights, and the shared expert.  NaNs
 // come last; any z gives distinct indices in range.
-__device__ __forceinline__ void choose_experts(const float* z, int experts, int top, bool shared, int32_t* ids, float* weights) {
+__device__ __forceinline__ void choose_experts(const float* z, const MoeRouting& r, int32_t* ids, float* weights) {
+  const int experts = r.experts, top = r.top;
+  const bool sigmoid = r.scoring == LVLLM_MOE_SIGMOID;
   const int lane = threadIdx.x & 63;
   auto value = [&](int e) {
     const float v = z[e];
     return v == v ? v : -INFINITY;
   };
-  auto weight_of = [](float v, float mx) { return v == -INFINITY ? 1e-30f : expf(v - mx); };
+  auto weight_of = [&](float v, float mx) {
+    return v == -INFINITY ? 1e-30f : sigmoid ? 1.f / (1.f + expf(-v)) : expf(v - mx);
+  };
   if (experts <= 64) {  // a logit's place is the number of logits ahead of it
     const float v = lane < experts ? value(lane) : -INFINITY;
     int place = 0;
@@ -53,7 +80,7 @@ __device__ __forceinline__ void choose_experts(const float* z, int experts, int 
     const bool chosen = lane < experts && place < top;
     const float mx = wave_max(v);  // (by all lanes)
     const float w = chosen ? weight_of(v, mx) : 0.f;
-    const float sum = wave_sum(w);
+    const float sum = sigmoid ? 1.f : wave_sum(w);
     if (chosen) {
       ids[place] = lane;
       weights[place] = w / sum;
@@ -83,23 +110,31 @@ __device__ __forceinline__ void choose_experts(const float* z, int experts, int 
           sum += w;
         } else if (lane == 0) {
           ids[k] = at;
-          weights[k] = w / sum;
+          weights[k] = sigmoid ? w : w / sum;
         }
       }
     }
   }
-  if (shared && lane == 0) {
+  if (r.shared && lane == 0) {
     ids[top] = experts;
-    weights[top] = 1.f / (1.f + expf(-z[experts]));
+    weights[top] = r.gated ? 1.f / (1.f + expf(-z[experts])) : 1.f;
   }
 }
 
-// Where the grouped assignments go: offsets [experts + 1], token and slot [assignments], tiles of `tile` slots.  count
-// [experts], zeroed: only for rows that count their own assignments (moe_count_assignments).
+// Where the grouped assignments go: offsets [experts + 1], token and slot [assignments], tiles of `tile` slots, and (null: not
+// kept) the assignments' weights in the order of the slots.  count [experts], zeroed: only for rows that count their own
+// assignments (moe_count_assignments).
 struct MoeGroups {
   int32_t *offsets, *token, *slot, *tiles, *count;
   int tile, max_tiles;
+  const float* weights;  // [rows, per row]
+  float* slot_weight;    // [assignments] or null
 };
+__device__ __forceinline__ void moe_place(const MoeGroups& out, int i, int per_row, int s) {
+  out.slot[i] = s;
+  out.token[s] = i / per_row;
+  if (out.slot_weight != nullptr) out.slot_weight[s] = out.weights[i];
+}
 
 // Running sums of the experts' slots and tiles, 64 experts a turn, by the first wave; count, first [experts + 1] and tile0
 // [experts + 1] in LDS.
@@ -155,9 +190,7 @@ __device__ __forceinline__ void group_assignments(const int32_t* ids, const int 
   moe_running_sums(count, first, tile0, experts, out.tile);
   __syncthreads();
   for (int i = threadIdx.x; i < total; i += 1024) {
-    const int s = first[min(max(ids[i], 0), experts - 1)] + out.slot[i];
-    out.slot[i] = s;
-    out.token[s] = i / per_row;
+    moe_place(out, i, per_row, first[min(max(ids[i], 0), experts - 1)] + out.slot[i]);
   }
   moe_write_tiles(first, tile0, experts, out);
 }
@@ -194,8 +227,8 @@ int launch_moe_mfma(const MoeParams& p, bool up, hipStream_t s);
 // `counted`: the rows have counted their assignments
 int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, bool counted, const MoeGroups& groups,
                      hipStream_t s);
-int64_t moe_route_mfma_workspace(int experts, int shared, int rows, int width);
-int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
-                          int top, int rows, int width, const MoeGroups& groups, float* workspace, hipStream_t s);
+int64_t moe_route_mfma_workspace(const MoeRouting& r, int rows, int width);
+int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, const MoeRouting& r,
+                          int rows, int width, const MoeGroups& groups, float* workspace, hipStream_t s);
 
 }  // namespace lvllm

@@ -9,12 +9,11 @@ template <typename T, int VEC>
 __global__ __launch_bounds__(256) void moe_route_kernel(int32_t* __restrict__ ids, float* __restrict__ weights,
                                                         const typename T::store_t* __restrict__ h,
                                                         const typename T::store_t* __restrict__ w,
-                                                        const float* __restrict__ bias, const int experts, const int shared,
-                                                        const int top, const int width) {
+                                                        const float* __restrict__ bias, const MoeRouting r, const int width) {
   __shared__ float z[kMaxExperts + 1];
-  const int row = blockIdx.x, lane = threadIdx.x & 63, n = top + shared;
+  const int row = blockIdx.x, lane = threadIdx.x & 63, n = r.per_row();
   const typename T::store_t* x = h + (int64_t)row * width;
-  for (int e = threadIdx.x >> 6; e < experts + shared; e += 4) {
+  for (int e = threadIdx.x >> 6; e < r.logits(); e += 4) {
     const typename T::store_t* we = w + (int64_t)e * width;
     float acc = 0.f;
     for (int i = lane * VEC; i < width; i += 64 * VEC) {
@@ -29,10 +28,10 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int32_t* __restrict__ id
       }
     }
     acc = wave_sum(acc);
-    if (lane == 0) z[e] = e < experts ? acc + bias[e] : acc;
+    if (lane == 0) z[e] = e < r.experts && bias != nullptr ? acc + bias[e] : acc;
   }
   __syncthreads();
-  if (threadIdx.x < 64) choose_experts(z, experts, top, shared != 0, ids + (int64_t)row * n, weights + (int64_t)row * n);
+  if (threadIdx.x < 64) choose_experts(z, r, ids + (int64_t)row * n, weights + (int64_t)row * n);
 }
 
 __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t* ids, const int total, const int per_row,
@@ -54,8 +53,7 @@ __global__ __launch_bounds__(256) void moe_slots_kernel(const int32_t* __restric
   const int i = blockIdx.x * 256 + threadIdx.x;
   if (i >= total) return;
   const int s = min(max(groups.offsets[min(max(ids[i], 0), experts - 1)] + groups.slot[i], 0), total - 1);
-  groups.slot[i] = s;
-  groups.token[s] = i / per_row;
+  moe_place(groups, i, per_row, s);
 }
 
 int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, bool counted, const MoeGroups& groups,
@@ -107,8 +105,10 @@ __global__ __launch_bounds__(256) void moe_simple_kernel(const MoeParams p) {
   }
   const int s = s0 + a, n = n0 + b;
   if (s >= s1) return;
-  if constexpr (UP) ((S*)p.out)[(int64_t)s * p.ff_max + n] = T::from_float(clamped_gate(accg, accu, p.limit[e]));
-  else if (n < p.width) ((S*)p.out)[(int64_t)s * p.width + n] = T::from_float(accg);
+  if constexpr (UP) {
+    const float f = slot_weight_of(p, s);
+    ((S*)p.out)[(int64_t)s * p.ff_max + n] = T::from_float(MoeActivation(p, e)(accg * f, accu * f));
+  } else if (n < p.width) ((S*)p.out)[(int64_t)s * p.width + n] = T::from_float(accg);
 }
 
 }  // namespace lvllm
@@ -117,48 +117,56 @@ using namespace lvllm;
 
 extern "C" int lvllm_moe_tile(int packed, int rows) { return moe_tile(packed != 0, rows); }
 
-extern "C" int64_t lvllm_moe_route_workspace_bytes(int experts, int shared, int rows, int width, int packed) {
-  return packed ? moe_route_mfma_workspace(experts, shared != 0, rows, width) : 0;
+static MoeRouting routing_of(const lvllm_moe_routing& r) {
+  return MoeRouting{r.experts, r.top, r.scoring, r.shared != LVLLM_MOE_NO_SHARED, r.shared == LVLLM_MOE_GATED_SHARED};
 }
 
-extern "C" int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, int32_t* token, int32_t* slot, int32_t* tiles,
-                               int max_tiles, const void* h, const void* w, const float* bias, int experts, int shared, int top,
-                               int rows, int width, int packed, void* workspace, int64_t workspace_bytes, int dtype,
-                               void* stream) {
+extern "C" int64_t lvllm_moe_route_workspace_bytes(const lvllm_moe_routing* routing, int rows, int width, int packed) {
+  return packed ? moe_route_mfma_workspace(routing_of(*routing), rows, width) : 0;
+}
+
+extern "C" int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, int32_t* token, int32_t* slot,
+                               float* slot_weight, int32_t* tiles, int max_tiles, const void* h, const void* w,
+                               const float* bias, const lvllm_moe_routing* routing, int rows, int width, int packed,
+                               void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
   if (rows == 0) return 0;
-  LV_CHECK(experts > 0 && experts < kMaxExperts && top > 0 && top <= experts, "experts: fewer than 1024, top of them");
-  LV_CHECK((int64_t)rows * (top + 1) < ((int64_t)1 << 31) && max_tiles > 0, "too many assignments");
-  LV_CHECK(workspace_bytes >= lvllm_moe_route_workspace_bytes(experts, shared, rows, width, packed), "workspace too small");
+  const MoeRouting r = routing_of(*routing);
+  LV_CHECK(r.experts > 0 && r.experts < kMaxExperts && r.top > 0 && r.top <= r.experts, "experts: fewer than 1024, top of them");
+  LV_CHECK(r.scoring == LVLLM_MOE_SOFTMAX || r.scoring == LVLLM_MOE_SIGMOID, "unknown scores");
+  LV_CHECK((int64_t)rows * (r.top + 1) < ((int64_t)1 << 31) && max_tiles > 0, "too many assignments");
+  LV_CHECK(workspace_bytes >= lvllm_moe_route_workspace_bytes(routing, rows, width, packed), "workspace too small");
   hipStream_t s = (hipStream_t)stream;
-  shared = shared != 0;
-  const MoeGroups groups{offsets, token, slot, tiles, (int32_t*)workspace, moe_tile(packed != 0, rows), max_tiles};
+  const MoeGroups groups{offsets, token, slot, tiles, (int32_t*)workspace, moe_tile(packed != 0, rows), max_tiles, weights,
+                         slot_weight};
   if (packed) {
     LV_CHECK(moe_takes_mfma(width, dtype), "packed router: bf16, a width that is a multiple of 32");
-    return launch_moe_route_mfma(ids, weights, h, w, bias, experts, shared, top, rows, width, groups, (float*)workspace, s);
+    return launch_moe_route_mfma(ids, weights, h, w, bias, r, rows, width, groups, (float*)workspace, s);
   }
   LV_DISPATCH_F32_BF16(dtype, {
     using S = typename scalar_t::store_t;
     if (width % 4 == 0)
       hipLaunchKernelGGL((moe_route_kernel<scalar_t, 4>), dim3(rows), dim3(256), 0, s, ids, weights, (const S*)h, (const S*)w,
-                         bias, experts, shared, top, width);
+                         bias, r, width);
     else
       hipLaunchKernelGGL((moe_route_kernel<scalar_t, 1>), dim3(rows), dim3(256), 0, s, ids, weights, (const S*)h, (const S*)w,
-                         bias, experts, shared, top, width);
+                         bias, r, width);
   });
   LV_LAUNCH_CHECK();
-  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, false, groups, s);
+  return launch_moe_group(ids, rows * r.per_row(), r.per_row(), r.all(), r.shared, false, groups, s);
 }
 
 extern "C" int lvllm_moe_experts(void* out, const void* x, const void* w, const int64_t* w_offset, const int32_t* ff,
-                                 const float* limit, const int32_t* offsets, const int32_t* token, const int32_t* tiles,
-                                 int experts, int slots, int rows, int width, int ff_max, int ff_first, int ff_last, int max_tiles, int up,
-                                 int packed, int dtype, void* stream) {
+                                 const float* limit, const float* slot_weight, int act, const int32_t* offsets,
+                                 const int32_t* token, const int32_t* tiles, int experts, int slots, int rows, int width,
+                                 int ff_max, int ff_first, int ff_last, int max_tiles, int up, int packed, int dtype,
+                                 void* stream) {
   if (slots == 0) return 0;
   LV_CHECK(experts > 0 && ff_max > 0 && ff_max % 32 == 0 && width > 0 && max_tiles > 0 && max_tiles <= 65535, "sizes of the experts");
+  LV_CHECK(!up || act == LVLLM_MOE_SILU || (act == LVLLM_MOE_CLAMPED && limit != nullptr), "unknown activation");
   MoeParams p{};
   p.out = out; p.x = x; p.w = w; p.w_offset = w_offset; p.ff = ff; p.limit = limit; p.offsets = offsets; p.token = token;
   p.tiles = tiles; p.experts = experts; p.slots = slots; p.rows = rows; p.width = width; p.ff_max = ff_max;
-  p.max_tiles = max_tiles; p.ff_first = ff_first; p.ff_last = ff_last;
+  p.max_tiles = max_tiles; p.ff_first = ff_first; p.ff_last = ff_last; p.slot_weight = slot_weight; p.act = act;
   hipStream_t s = (hipStream_t)stream;
   if (packed) {
     LV_CHECK(moe_takes_mfma(width, dtype), "packed experts: bf16, a width that is a multiple of 32");

@@ -113,9 +113,10 @@ __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
   if (slot >= s1) return;
   float v[4];
   if constexpr (UP) {
-    const float limit = p.limit[e];
+    const MoeActivation act(p, e);
+    const float f = slot_weight_of(p, slot);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = clamped_gate(acc[0][r], acc[1][r], limit);
+    for (int r = 0; r < 4; ++r) v[r] = act(acc[0][r] * f, acc[1][r] * f);
     store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.ff_max + 16 * u + 4 * g, v);
   } else {
 #pragma unroll
@@ -228,18 +229,19 @@ __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, con
   if (k + 1 < steps) step(k + 1, 1);
   if (k + 2 < steps) step(k + 2, 2);
   __builtin_amdgcn_s_waitcnt(0 | (7 << 4) | (15 << 8));  // (no copy to LDS outlives the workgroup)
-  const float limit = UP ? p.limit[e] : 0.f;
+  const MoeActivation act(p, UP ? e : 0);
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
     const int slot = s0 + 16 * m + c;
     if (slot >= s1) continue;
+    const float f = UP ? slot_weight_of(p, slot) : 1.f;
 #pragma unroll
     for (int n = 0; n < 4; n += UP ? 2 : 1) {
       if (nt0 + n >= ntiles) continue;
       float v[4];
       if constexpr (UP) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] = clamped_gate(acc[n][m][r], acc[n + 1][m][r], limit);
+        for (int r = 0; r < 4; ++r) v[r] = act(acc[n][m][r] * f, acc[n + 1][m][r] * f);
         store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.ff_max + (nt0 + n) * 8 + 4 * g, v);
       } else {
 #pragma unroll
@@ -302,21 +304,21 @@ __device__ __forceinline__ void route_logits(float* z, int ld, e_f32x4_t* red, c
 // many rows: logits and choice in one launch, a wave chooses for two rows
 __global__ __launch_bounds__(512) void moe_route_mfma_kernel(int32_t* ids, float* __restrict__ weights,
                                                              const uint16_t* __restrict__ h, const uint16_t* __restrict__ w,
-                                                             const float* __restrict__ bias, const int experts,
-                                                             const int shared, const int top, const int rows, const int width,
-                                                             const MoeGroups groups) {
+                                                             const float* __restrict__ bias, const MoeRouting r,
+                                                             const int rows, const int width, const MoeGroups groups) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   float* z = reinterpret_cast<float*>(smem + kRouteLds);
-  const int ntiles = (experts + shared + 15) >> 4, ld = ntiles * 16 + 1, row0 = blockIdx.x * 16, n = top + shared;
+  const int ntiles = (r.logits() + 15) >> 4, ld = ntiles * 16 + 1, row0 = blockIdx.x * 16, n = r.per_row();
   route_logits(z, ld, reinterpret_cast<e_f32x4_t*>(smem), h, w, row0, rows, width, ntiles, 0, width >> 5);
   const int lane = threadIdx.x & 63;
-  for (int r = threadIdx.x >> 6; r < 16 && row0 + r < rows; r += 8) {
-    for (int e = lane; e < experts; e += 64) z[r * ld + e] += bias[e];
+  for (int i = threadIdx.x >> 6; i < 16 && row0 + i < rows; i += 8) {
+    if (bias != nullptr)
+      for (int e = lane; e < r.experts; e += 64) z[i * ld + e] += bias[e];
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (the wave's own next reads see it)
-    choose_experts(z + r * ld, experts, top, shared != 0, ids + (int64_t)(row0 + r) * n, weights + (int64_t)(row0 + r) * n);
+    choose_experts(z + i * ld, r, ids + (int64_t)(row0 + i) * n, weights + (int64_t)(row0 + i) * n);
   }
   __syncthreads();  // (the logits' partial sums make room for the counts)
-  moe_count_assignments(ids, row0, min(16, rows - row0), n, experts + shared, shared, reinterpret_cast<int*>(smem), groups);
+  moe_count_assignments(ids, row0, min(16, rows - row0), n, r.all(), r.shared, reinterpret_cast<int*>(smem), groups);
 }
 
 __global__ __launch_bounds__(256) void moe_zero_kernel(int32_t* __restrict__ p, const int n) {
@@ -338,15 +340,14 @@ __global__ __launch_bounds__(512) void moe_logits_kernel(float* __restrict__ par
 // ... and one workgroup adds them, chooses (a wave per row) and groups the assignments
 __global__ __launch_bounds__(1024) void moe_choose_group_kernel(int32_t* ids, float* weights, const float* __restrict__ part,
                                                                 const float* __restrict__ bias, const int shares,
-                                                                const int row_tiles, const int ld, const int experts,
-                                                                const int shared, const int top, const int rows,
-                                                                const MoeGroups groups) {
+                                                                const int row_tiles, const int ld, const MoeRouting r,
+                                                                const int rows, const MoeGroups groups) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = top + shared;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = r.per_row();
   float* z = reinterpret_cast<float*>(smem) + wave * ld;
   for (int row = wave; row < rows; row += 16) {
-    for (int e = lane; e < experts + shared; e += 64) {
-      float v = e < experts ? bias[e] : 0.f, t[kRouteShares];
+    for (int e = lane; e < r.logits(); e += 64) {
+      float v = e < r.experts && bias != nullptr ? bias[e] : 0.f, t[kRouteShares];
 #pragma unroll
       for (int s = 0; s < kRouteShares; ++s) t[s] = part[((int64_t)min(s, shares - 1) * row_tiles * 16 + row) * ld + e];
 #pragma unroll
@@ -354,10 +355,10 @@ __global__ __launch_bounds__(1024) void moe_choose_group_kernel(int32_t* ids, fl
       z[e] = v;
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (the wave's own next reads see it)
-    choose_experts(z, experts, top, shared != 0, ids + (int64_t)row * n, weights + (int64_t)row * n);
+    choose_experts(z, r, ids + (int64_t)row * n, weights + (int64_t)row * n);
   }
   __syncthreads();
-  group_assignments(ids, rows * n, n, experts + shared, shared, groups);
+  group_assignments(ids, rows * n, n, r.all(), r.shared, groups);
 }
 
 static int route_shares(int width) {
@@ -365,14 +366,14 @@ static int route_shares(int width) {
   return steps < 16 ? 1 : steps / 16 > kRouteShares ? kRouteShares : steps / 16;  // (at least two k-steps a wave)
 }
 
-int64_t moe_route_mfma_workspace(int experts, int shared, int rows, int width) {
-  if (rows > kMoeFewRows) return (int64_t)(experts + shared) * 4;  // (the experts' counts)
-  return (int64_t)route_shares(width) * ((rows + 15) / 16) * 16 * ((experts + shared + 15) / 16 * 16) * 4;
+int64_t moe_route_mfma_workspace(const MoeRouting& r, int rows, int width) {
+  if (rows > kMoeFewRows) return (int64_t)r.all() * 4;  // (the experts' counts)
+  return (int64_t)route_shares(width) * ((rows + 15) / 16) * 16 * ((r.logits() + 15) / 16 * 16) * 4;
 }
 
-int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, int experts, int shared,
-                          int top, int rows, int width, const MoeGroups& groups, float* workspace, hipStream_t s) {
-  const int ntiles = (experts + shared + 15) / 16, row_tiles = (rows + 15) / 16;
+int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const void* w, const float* bias, const MoeRouting& r,
+                          int rows, int width, const MoeGroups& groups, float* workspace, hipStream_t s) {
+  const int ntiles = (r.logits() + 15) / 16, row_tiles = (rows + 15) / 16;
   if (rows <= kMoeFewRows) {
     const int shares = route_shares(width), per = (width / 32 + shares - 1) / shares, ld = ntiles * 16;
     const int lds = kRouteLds + 16 * ld * 4, lds_choose = 16 * ld * 4;
@@ -382,18 +383,18 @@ int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const voi
                        (const uint16_t*)w, ntiles, rows, width, per);
     LV_LAUNCH_CHECK();
     hipLaunchKernelGGL(moe_choose_group_kernel, dim3(1), dim3(1024), lds_choose, s, ids, weights, workspace, bias, shares,
-                       row_tiles, ld, experts, shared, top, rows, groups);
+                       row_tiles, ld, r, rows, groups);
     LV_LAUNCH_CHECK();
     return 0;
   }
   const int lds = kRouteLds + 16 * (ntiles * 16 + 1) * 4;
   (void)hipFuncSetAttribute((const void*)moe_route_mfma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  hipLaunchKernelGGL(moe_zero_kernel, dim3(1), dim3(256), 0, s, groups.count, experts + shared);
+  hipLaunchKernelGGL(moe_zero_kernel, dim3(1), dim3(256), 0, s, groups.count, r.all());
   LV_LAUNCH_CHECK();
   hipLaunchKernelGGL(moe_route_mfma_kernel, dim3(row_tiles), dim3(512), lds, s, ids, weights, (const uint16_t*)h,
-                     (const uint16_t*)w, bias, experts, shared, top, rows, width, groups);
+                     (const uint16_t*)w, bias, r, rows, width, groups);
   LV_LAUNCH_CHECK();
-  return launch_moe_group(ids, rows * (top + shared), top + shared, experts + shared, shared, true, groups, s);
+  return launch_moe_group(ids, rows * r.per_row(), r.per_row(), r.all(), r.shared, true, groups, s);
 }
 
 bool moe_takes_mfma(int width, int dtype) { return dtype == LVLLM_BF16 && width % 32 == 0; }

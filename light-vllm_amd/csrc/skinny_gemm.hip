@@ -19,7 +19,7 @@
 // Loads outside the problem (k-steps past K, tiles past N) use an out-of-range buffer offset and
 // return zeros without touching memory, so the loop is branch-free.
 // Epilogues (act): 0 plain (+ bias); 5 squared ReLU; 2 SwiGLU over (gate, up) tile pairs -> [M, N/2]; 3 greedy arg-max
-// over N -> int64 [M] (no logits written); act = 1 applies SwiGLU while loading X (kept for small shapes).
+// over N -> int64 [M] (no logits written); 6 as 2 with the clamped unit (clamped_unit_of) for silu(gate) * up; act = 1 applies SwiGLU while loading X (kept for small shapes).
 // The same file holds the W8A8 variant (fp8 weights, X quantised while the fragments are built) and,
 // at the end, the 65..256-row kernel that moves X through LDS instead of registers.
 //
@@ -104,7 +104,7 @@ __global__ __launch_bounds__(kGemmWaves * 64, 2) void skinny_gemm_kernel(
     const typename T::store_t* __restrict__ bias, const int M, const int N, const int K,
     const int64_t ldx, const int steps_per_wave, const int ntiles, const int act, const int stage_tiles,
     const float* __restrict__ x_scale, const float* __restrict__ w_scale, uint8_t* __restrict__ y8 = nullptr,
-    const float* __restrict__ y8_scale = nullptr) {
+    const float* __restrict__ y8_scale = nullptr, const float limit = 0.f) {
   using S = typename T::store_t;
   static_assert(!XQ || (W8 && KSTEPS == 8 && MT <= 2), "pre-quantised activations: the W8A8 variants of <= 32 rows");
   LVLLM_TRACE_BEGIN();
@@ -136,7 +136,7 @@ __global__ __launch_bounds__(kGemmWaves * 64, 2) void skinny_gemm_kernel(
   // glu (act == 2, W = [gate rows | up rows]): the workgroup owns PAIRS -- local tiles 2j and 2j+1
   // are the gate tile and the up tile of pair blockIdx.x + j * gridDim.x -- so that the epilogue
   // can apply silu(gate) * up before anything is written (no [M, N] intermediate, no second kernel).
-  const bool glu = act == 2;
+  const bool glu = act == 2 || act == 6;
   const int nunits = glu ? ntiles >> 1 : ntiles;  // tiles or pairs handed out round-robin
   const int my_units = nunits > (int)blockIdx.x ? (nunits - blockIdx.x + gridDim.x - 1) / gridDim.x : 0;
   const int my_tiles_ld = glu ? 2 * my_units : my_units;
@@ -237,9 +237,13 @@ __global__ __launch_bounds__(kGemmWaves * 64, 2) void skinny_gemm_kernel(
       S o[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const float gf = T::to_float(T::from_float(gs[r]));
-        const S a = T::from_float(gf / (1.0f + expf(-gf)));
-        o[r] = T::from_float(T::to_float(a) * T::to_float(T::from_float(us[r])));
+        const float gf = T::to_float(T::from_float(gs[r])), uf = T::to_float(T::from_float(us[r]));
+        if (act == 6) {
+          o[r] = T::from_float(clamped_unit_of(gf, uf, limit));
+        } else {
+          const S a = T::from_float(gf / (1.0f + expf(-gf)));
+          o[r] = T::from_float(T::to_float(a) * uf);
+        }
       }
       if (y != nullptr) {
         uint2 ov;
@@ -737,7 +741,7 @@ __global__ void skinny_argmax_reduce_kernel(int64_t* __restrict__ tokens, const 
 template <typename T>
 __global__ void skinny_gemm_reduce_swiglu_kernel(typename T::store_t* __restrict__ y, const float* __restrict__ partial,
                                                  const typename T::store_t* __restrict__ bias, const int M,
-                                                 const int N, const int ksplit) {
+                                                 const int N, const int ksplit, const bool clamped, const float limit) {
   using S = typename T::store_t;
   const int half_n = N >> 1;
   const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x) * 4;  // index into [M, N/2]
@@ -762,9 +766,9 @@ __global__ void skinny_gemm_reduce_swiglu_kernel(typename T::store_t* __restrict
   S o[4];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
-    const float gf = T::to_float(T::from_float(gs[r]));
+    const float gf = T::to_float(T::from_float(gs[r])), uf = T::to_float(T::from_float(us[r]));
     const S a = T::from_float(gf / (1.0f + expf(-gf)));
-    o[r] = T::from_float(T::to_float(a) * T::to_float(T::from_float(us[r])));
+    o[r] = clamped ? T::from_float(clamped_unit_of(gf, uf, limit)) : T::from_float(T::to_float(a) * uf);
   }
   uint2 ov;
   ov.x = (uint32_t)o[0] | ((uint32_t)o[1] << 16);
@@ -826,12 +830,13 @@ template <typename T, int MT, int KSTEPS, bool W8 = false, bool XQ = false>
 static void launch_skinny(void* y, float* partial, const void* x, const void* w, const void* bias, int M,
                           int N, int K, int64_t ldx, int steps_per_wave, int ntiles, int groups, int ksplit,
                           bool packed, int act, hipStream_t stream, const float* x_scale = nullptr,
-                          const float* w_scale = nullptr, uint8_t* y8 = nullptr, const float* y8_scale = nullptr) {
+                          const float* w_scale = nullptr, uint8_t* y8 = nullptr, const float* y8_scale = nullptr,
+                          float limit = 0.f) {
   using S = typename T::store_t;
   constexpr int NT = LVLLM_GEMM_NT / MT > 0 ? LVLLM_GEMM_NT / MT : 1;  // NT * MT slabs per meeting
   const size_t red_bytes = (size_t)2 * kGemmWaves * NT * MT * 64 * sizeof(g_f32x4_t);
   // output stage: as many tiles as the workgroup owns, capped by what is left of the 160 KiB LDS
-  const bool glu = act == 2;  // tiles are handed out in (gate, up) pairs
+  const bool glu = act == 2 || act == 6;  // tiles are handed out in (gate, up) pairs
   const int tiles_per_wg = glu ? 2 * ((ntiles / 2 + groups - 1) / groups) : (ntiles + groups - 1) / groups;
   int stage_tiles = ((tiles_per_wg + NT - 1) / NT) * NT;
   // wave-private scratch that turns row-order activation loads into fragments (16-bit path only)
@@ -847,7 +852,7 @@ static void launch_skinny(void* y, float* partial, const void* x, const void* w,
       (void)hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
     hipLaunchKernelGGL(kern, dim3(groups, ksplit), dim3(kGemmWaves * 64), smem, stream, (S*)y, partial,
                        (const S*)x, (const S*)w, (const S*)bias, M, N, K, ldx, steps_per_wave, ntiles, act,
-                       stage_tiles, x_scale, w_scale, y8, y8_scale);
+                       stage_tiles, x_scale, w_scale, y8, y8_scale, limit);
   };
   if constexpr (W8 && XQ) {
     go(skinny_gemm_kernel<T, MT, KSTEPS, true, NT, true, true>);
@@ -1121,9 +1126,9 @@ extern "C" int lvllm_skinny_gemm(void* y, const void* x, const void* w, const vo
                               workspace_bytes, stream);
 }
 
-extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const void* bias, int M, int N,
-                                    int K, int64_t ldx, int dtype, int packed, int act, int partial_out,
-                                    int* ksplit_out, void* workspace, int64_t workspace_bytes, void* stream) {
+static int skinny_gemm(void* y, const void* x, const void* w, const void* bias, int M, int N, int K, int64_t ldx, int dtype,
+                       int packed, int act, float limit, int partial_out, int* ksplit_out, void* workspace,
+                       int64_t workspace_bytes, void* stream) {
   if (M <= 0 || N <= 0) return 0;
   if (!(dtype == LVLLM_BF16 || dtype == LVLLM_F16) || M > 64 || (K % 32) != 0 || (N % 16) != 0 ||
       (int64_t)N * K * 2 >= ((int64_t)1 << 32) - 16 || (ldx % 8) != 0 ||
@@ -1132,7 +1137,8 @@ extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const
     set_error("lvllm_skinny_gemm: shape outside the kernel's envelope");
     return 3;
   }
-  LV_CHECK(act >= 0 && (act <= 3 || act == 5) && !(act == 5 && partial_out), "unknown epilogue");
+  LV_CHECK(act >= 0 && (act <= 3 || act == 5 || act == 6) && !(act == 5 && partial_out), "unknown epilogue");
+  const bool glu = act == 2 || act == 6, clamped = act == 6;
   const int total_steps = K / 32;
   const int cap = kGemmWaves * max_steps_per_wave(M);
   int ksplit = (total_steps + cap - 1) / cap;
@@ -1150,12 +1156,12 @@ extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const
                                                                             : tuning().gemm_workgroups;
   int groups = gemm_cus / ksplit;
   if (groups < 1) groups = 1;
-  const bool glu_reduce = act == 2 && ksplit > 1;  // K split over workgroups: SwiGLU inside the reduce pass
-  if (act == 2) {  // SwiGLU: y is [M, N / 2]
+  const bool glu_reduce = glu && ksplit > 1;  // K split over workgroups: SwiGLU inside the reduce pass
+  if (glu) {  // SwiGLU: y is [M, N / 2]
     LV_CHECK(N % 32 == 0 && !partial_out, "the SwiGLU epilogue needs N % 32 == 0 and writes y itself");
     if (glu_reduce) act = 0;  // plain tiles into the fp32 partials
   }
-  groups = balanced_groups(act == 2 ? ntiles / 2 : ntiles, groups);  // (SwiGLU: (gate, up) pairs are handed out)
+  groups = balanced_groups(glu && !glu_reduce ? ntiles / 2 : ntiles, groups);  // (SwiGLU: (gate, up) pairs are handed out)
   void* const tokens_out = y;
   const bool amax_reduce = act == 3 && ksplit > 1;  // K split over workgroups: arg-max inside a reduce pass
   float* amax_cand = nullptr;
@@ -1187,17 +1193,17 @@ extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const
   do {                                                                                              \
     if (k8)                                                                                         \
       launch_skinny<T_, MT_, 8>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, \
-                                ksplit, packed != 0, act, s);                                       \
+                                ksplit, packed != 0, act, s, nullptr, nullptr, nullptr, nullptr, limit);                                       \
     else                                                                                            \
       launch_skinny<T_, MT_, 16>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, \
-                                 ksplit, packed != 0, act, s);                                      \
+                                 ksplit, packed != 0, act, s, nullptr, nullptr, nullptr, nullptr, limit);                                      \
   } while (0)
 #define LV_SG_MT(T_)                           \
   switch (MT) {                                \
     case 1: LV_SG(T_, 1); break;               \
     case 2: LV_SG(T_, 2); break;               \
     default:                                   \
-      launch_skinny<T_, 4, 8>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, ksplit, packed != 0, act, s); \
+      launch_skinny<T_, 4, 8>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, ksplit, packed != 0, act, s, nullptr, nullptr, nullptr, nullptr, limit); \
       break;                                   \
   }
   if (dtype == LVLLM_BF16) { LV_SG_MT(BF16) } else { LV_SG_MT(F16) }
@@ -1226,10 +1232,10 @@ extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const
     const int grid = (int)(((int64_t)M * (N / 2) / 4 + 255) / 256);
     if (dtype == LVLLM_BF16)
       hipLaunchKernelGGL((skinny_gemm_reduce_swiglu_kernel<BF16>), dim3(grid), dim3(256), 0, s, (uint16_t*)y, partial,
-                         (const uint16_t*)bias, M, N, ksplit);
+                         (const uint16_t*)bias, M, N, ksplit, clamped, limit);
     else
       hipLaunchKernelGGL((skinny_gemm_reduce_swiglu_kernel<F16>), dim3(grid), dim3(256), 0, s, (uint16_t*)y, partial,
-                         (const uint16_t*)bias, M, N, ksplit);
+                         (const uint16_t*)bias, M, N, ksplit, clamped, limit);
     LV_LAUNCH_CHECK();
     return 0;
   }
@@ -1246,6 +1252,19 @@ extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const
     LV_LAUNCH_CHECK();
   }
   return 0;
+}
+
+extern "C" int lvllm_skinny_gemm_ex(void* y, const void* x, const void* w, const void* bias, int M, int N,
+                                    int K, int64_t ldx, int dtype, int packed, int act, int partial_out,
+                                    int* ksplit_out, void* workspace, int64_t workspace_bytes, void* stream) {
+  LV_CHECK(act != 6, "the clamped unit has an entry of its own");
+  return skinny_gemm(y, x, w, bias, M, N, K, ldx, dtype, packed, act, 0.f, partial_out, ksplit_out, workspace, workspace_bytes,
+                     stream);
+}
+
+extern "C" int lvllm_skinny_gemm_clamped_unit(void* y, const void* x, const void* w, int M, int N, int K, int64_t ldx, int dtype,
+                                              int packed, float limit, void* workspace, int64_t workspace_bytes, void* stream) {
+  return skinny_gemm(y, x, w, nullptr, M, N, K, ldx, dtype, packed, 6, limit, 0, nullptr, workspace, workspace_bytes, stream);
 }
 
 // W8A8: Y[M,N] = T((fp8(X / x_scale) . W8^T) * x_scale * w_scale + bias).  X [M, K] in T (ldx apart),

@@ -1,11 +1,10 @@
 // Row-wise operators of hybrid decoders for gfx950: the fp32 residual add with a Dynamic-Tanh norm, the token shift with
-// its per-projection mixes, squared ReLU, per-head query/key RMS norms with the paged-cache write, and the gates in
-// front of an output projection.
+// its per-projection mixes, and squared ReLU.
 //
-// The residual stream, the norms and every gate are fp32; what a projection reads is rounded to its element type T once,
+// The residual stream and the norms are fp32; what a projection reads is rounded to its element type T once,
 // when it is stored.  A step's rows are the new tokens of `num_seqs` sequences back to back (query_start_loc), sequence
 // s ending at position seq_lens[s] - 1; rows past the last sequence are padding of a captured step.
-#include "common.h"
+#include "row_ops.h"
 
 namespace lvllm {
 
@@ -169,210 +168,6 @@ __global__ void relu_squared_kernel(typename T::store_t* out, const typename T::
   }
 }
 
-// VEC consecutive elements <-> floats
-template <typename T, int VEC>
-__device__ __forceinline__ void load_vec(const typename T::store_t* p, float (&v)[VEC]) {
-  if constexpr (VEC == 8) {
-    static_assert(sizeof(typename T::store_t) == 2, "16-byte pieces of 16-bit elements");
-    const uint4 a = *reinterpret_cast<const uint4*>(p);
-    const uint32_t w[4] = {a.x, a.y, a.z, a.w};
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      v[2 * j] = T::to_float((uint16_t)w[j]);
-      v[2 * j + 1] = T::to_float((uint16_t)(w[j] >> 16));
-    }
-  } else if constexpr (VEC == 4) {
-    load4<T>(p, v);
-  } else {
-    v[0] = T::to_float(p[0]);
-  }
-}
-template <typename T, int VEC>
-__device__ __forceinline__ void store_vec(typename T::store_t* p, const float (&v)[VEC]) {
-  if constexpr (VEC == 8) {
-    uint32_t w[4];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) w[j] = (uint32_t)T::from_float(v[2 * j]) | ((uint32_t)T::from_float(v[2 * j + 1]) << 16);
-    *reinterpret_cast<uint4*>(p) = uint4{w[0], w[1], w[2], w[3]};
-  } else if constexpr (VEC == 4) {
-    store4<T>(p, v);
-  } else {
-    p[0] = T::from_float(v[0]);
-  }
-}
-template <int L>
-__device__ __forceinline__ float group_sum(float v) {  // over L neighbouring lanes
-#pragma unroll
-  for (int m = L / 2; m >= 1; m >>= 1) v += __shfl_xor(v, m);
-  return v;
-}
-
-// Per-head RMS norm of queries and keys (weights [dim], shared by the heads) and the write of the normed keys and the
-// values into a paged cache whose key and value sizes differ:
-//   key_cache   [num_blocks, kv_heads, kpad / x, block_size, x],  x = 16 / sizeof(T), kpad >= dim (rest zeroed)
-//   value_cache [num_blocks, kv_heads, vpad, block_size],         vpad >= vdim (rest zeroed)
-// q_out [rows, heads, kpad] (padding zeroed).  L lanes per (row, head); the values of few rows ride along as further
-// "heads" (with_values), those of many go through value_cache_tile_kernel.
-template <typename T, int L, int VEC>
-__global__ __launch_bounds__(256) void qk_norm_cache_kernel(
-    typename T::store_t* __restrict__ q_out, typename T::store_t* __restrict__ key_cache,
-    typename T::store_t* __restrict__ value_cache, const typename T::store_t* __restrict__ q,
-    const typename T::store_t* __restrict__ k, const typename T::store_t* __restrict__ v, const int64_t row_stride,
-    const float* __restrict__ q_weight, const float* __restrict__ k_weight, const float eps, const int rows, const int heads,
-    const int kv_heads, const int dim, const int vdim, const int kpad, const int vpad, const bool with_values,
-    const int64_t* __restrict__ slot_mapping, const int64_t num_slots, const int block_size, const int64_t k_block_stride,
-    const int64_t v_block_stride) {
-  using S = typename T::store_t;
-  constexpr int x = 16 / sizeof(S);
-  const int lane = threadIdx.x % L;
-  const int per_row = heads + (with_values ? 2 : 1) * kv_heads;
-  const unsigned item = blockIdx.x * (256 / L) + threadIdx.x / L;
-  const int row = (int)(item / (unsigned)per_row), h = (int)(item - (unsigned)row * per_row);
-  if (row >= rows) return;
-  int64_t block = 0;
-  int off = 0;
-  if (h >= heads) {
-    const int64_t slot = slot_mapping[row];
-    if (slot < 0 || slot >= num_slots) return;
-    block = slot / block_size;
-    off = (int)(slot - block * block_size);
-  }
-  if (h >= heads + kv_heads) {
-    const int g = h - heads - kv_heads;
-    const S* src = v + row * row_stride + (int64_t)g * vdim;
-    S* dst = value_cache + block * v_block_stride + (int64_t)g * vpad * block_size + off;
-    for (int d = lane; d < vpad; d += L) dst[(int64_t)d * block_size] = d < vdim ? src[d] : T::from_float(0.f);
-    return;
-  }
-  const bool is_q = h < heads;
-  const S* src = (is_q ? q + (int64_t)h * dim : k + (int64_t)(h - heads) * dim) + row * row_stride;
-  const float* wt = is_q ? q_weight : k_weight;
-  S* dst = is_q ? q_out + ((int64_t)row * heads + h) * kpad
-                : key_cache + block * k_block_stride + (int64_t)(h - heads) * kpad * block_size + (int64_t)off * x;
-  float f[VEC];
-  float ss = 0.f;
-  for (int d = lane * VEC; d < dim; d += L * VEC) {
-    load_vec<T, VEC>(src + d, f);
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) ss += f[j] * f[j];
-  }
-  const bool one_pass = dim <= L * VEC;  // (the values are still in registers)
-  const float r = 1.f / sqrtf(group_sum<L>(ss) / dim + eps);
-  for (int d = lane * VEC; d < kpad; d += L * VEC) {
-    float o[VEC];
-    if (d < dim) {
-      if (!one_pass) load_vec<T, VEC>(src + d, f);
-#pragma unroll
-      for (int j = 0; j < VEC; ++j) o[j] = f[j] * r * wt[d + j];
-    } else {
-#pragma unroll
-      for (int j = 0; j < VEC; ++j) o[j] = 0.f;
-    }
-    store_vec<T, VEC>(is_q ? dst + d : dst + (int64_t)(d / x) * block_size * x + d % x, o);
-  }
-}
-
-// Values of many rows: a workgroup takes 64 rows of one kv head through LDS.  Its rows are cut into groups of consecutive
-// slots inside one aligned 8-slot window; a thread stores a (d, group) as one piece when the group is full.
-constexpr int kValueTile = 64;
-template <typename S>
-__global__ __launch_bounds__(256) void value_cache_tile_kernel(S* __restrict__ value_cache, const S* __restrict__ v,
-                                                               const int64_t row_stride, const int rows, const int vdim,
-                                                               const int vpad, const int64_t* __restrict__ slot_mapping,
-                                                               const int64_t num_slots, const int block_size,
-                                                               const int64_t v_block_stride) {
-  struct alignas(16) Eight { S e[8]; };
-  constexpr int LD = kValueTile + 2;
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  S* tile = reinterpret_cast<S*>(smem);  // [vdim][LD]
-  __shared__ int64_t slots[kValueTile];
-  __shared__ int groups[kValueTile], num_groups;  // first row | length << 8
-  const int row0 = blockIdx.x * kValueTile, head = blockIdx.y, nt = min(kValueTile, rows - row0), tid = threadIdx.x;
-  if (tid < kValueTile) {
-    int64_t s = tid < nt ? slot_mapping[row0 + tid] : -1;
-    if (s >= num_slots) s = -1;
-    slots[tid] = s;
-    const int64_t prev = (int64_t)__shfl_up((long long)s, 1);
-    const bool first = s >= 0 && (tid == 0 || prev < 0 || s != prev + 1 || (s & 7) == 0);
-    const uint64_t starts = __ballot(first), used = __ballot(s >= 0);
-    if (first) {
-      const uint64_t above = tid == 63 ? 0 : (starts | ~used) >> (tid + 1);
-      const int len = above ? __builtin_ctzll(above) + 1 : 64 - tid;
-      groups[__builtin_popcountll(starts & ((1ull << tid) - 1))] = tid | (len << 8);
-    }
-    if (tid == 0) num_groups = __builtin_popcountll(starts);
-  }
-  const S* src = v + (int64_t)row0 * row_stride + (int64_t)head * vdim;
-  for (int i = tid; i < nt * vdim; i += 256) {
-    const int t = i / vdim, d = i - t * vdim;
-    tile[d * LD + t] = src[t * row_stride + d];
-  }
-  __syncthreads();
-  const int ng = num_groups;
-  for (int i = tid; i < vpad * ng; i += 256) {
-    const int d = i / ng, gr = groups[i - d * ng], t = gr & 0xff, len = gr >> 8;
-    const int64_t s = slots[t], b = s / block_size;
-    S* dst = value_cache + b * v_block_stride + ((int64_t)head * vpad + d) * block_size + (s - b * block_size);
-    Eight e;
-#pragma unroll
-    for (int j = 0; j < 8; ++j) e.e[j] = (d < vdim && j < len) ? tile[d * LD + t + j] : (S)0;
-    if (len == 8) {
-      *reinterpret_cast<Eight*>(dst) = e;
-    } else {
-#pragma unroll
-      for (int j = 0; j < 8; ++j)
-        if (j < len) dst[j] = e.e[j];
-    }
-  }
-}
-
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-
-// Per head: o / rms(o) * weight * silu(gate) * scale -> T.  o is the fp32 read-out of a recurrent state.
-// weight_head_stride: 0 (one weight of size vdim for all heads) or vdim.  L lanes per (row, head).
-template <typename T, int L, int VEC>
-__global__ __launch_bounds__(256) void head_norm_gate_kernel(
-    typename T::store_t* __restrict__ out, const int64_t out_stride, const float* __restrict__ o,
-    const typename T::store_t* __restrict__ gate, const int64_t gate_stride, const float* __restrict__ weight,
-    const int weight_head_stride, const float eps, const float scale, const int rows, const int heads, const int vdim) {
-  const int lane = threadIdx.x % L;
-  const int64_t item = (int64_t)blockIdx.x * (256 / L) + threadIdx.x / L;
-  if (item >= (int64_t)rows * heads) return;
-  const int64_t row = item / heads;
-  const int h = (int)(item - row * heads);
-  const float* src = o + item * vdim;
-  float f[VEC], z[VEC];
-  float ss = 0.f;
-  for (int d = lane * VEC; d < vdim; d += L * VEC) {
-    load_vec<F32, VEC>(src + d, f);
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) ss += f[j] * f[j];
-  }
-  const float r = 1.f / sqrtf(group_sum<L>(ss) / vdim + eps);
-  for (int d = lane * VEC; d < vdim; d += L * VEC) {
-    load_vec<F32, VEC>(src + d, f);
-    load_vec<T, VEC>(gate + row * gate_stride + h * vdim + d, z);
-#pragma unroll
-    for (int j = 0; j < VEC; ++j)
-      f[j] = f[j] * r * weight[h * weight_head_stride + d + j] * (z[j] * sigmoid_f(z[j])) * scale;
-    store_vec<T, VEC>(out + row * out_stride + h * vdim + d, f);
-  }
-}
-
-// lanes that cover n elements in one pass of VEC each: 8, 16, 32 or 64
-static int lanes_for(int n, int vec) {
-  int l = 8;
-  while (l < 64 && l * vec < n) l *= 2;
-  return l;
-}
-#define LV_LANES(LANES_, ...)                         \
-  switch (LANES_) {                                   \
-    case 8: { constexpr int kL = 8; __VA_ARGS__ } break;   \
-    case 16: { constexpr int kL = 16; __VA_ARGS__ } break; \
-    case 32: { constexpr int kL = 32; __VA_ARGS__ } break; \
-    default: { constexpr int kL = 64; __VA_ARGS__ } break; \
-  }
-
 template <typename T>
 static ProjOut<T> proj_out(const void* y, const float* partials, int num_partials, int64_t n) {
   return ProjOut<T>{(const typename T::store_t*)y, partials, num_partials, n};
@@ -446,75 +241,6 @@ extern "C" int lvllm_relu_squared(void* out, const void* x, int64_t n, int dtype
                          (const S*)x, n);
     });
   }
-  LV_LAUNCH_CHECK();
-  return 0;
-}
-
-extern "C" int lvllm_qk_norm_cache(void* q_out, void* key_cache, void* value_cache, const void* q, const void* k,
-                                   const void* v, int64_t row_stride, const float* q_weight, const float* k_weight,
-                                   float eps, int rows, int heads, int kv_heads, int dim, int vdim, int kpad, int vpad,
-                                   const int64_t* slot_mapping, int64_t num_blocks, int block_size,
-                                   int64_t k_block_stride, int64_t v_block_stride, int dtype, void* stream) {
-  if (rows == 0) return 0;
-  LV_CHECK(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "heads must be a multiple of kv_heads");
-  LV_CHECK(dim <= kpad && vdim <= vpad && kpad % 8 == 0, "padded sizes must hold the real ones");
-  LV_CHECK(k_block_stride >= (int64_t)kv_heads * kpad * block_size && v_block_stride >= (int64_t)kv_heads * vpad * block_size,
-           "cache blocks overlap");
-  const int esize = dtype == LVLLM_F32 ? 4 : 2;
-  const size_t smem = (size_t)vdim * (kValueTile + 2) * esize;
-  const bool tiled = rows > 64 && smem <= 64 * 1024 && block_size % 8 == 0 && ((uintptr_t)value_cache & 15) == 0 &&
-                     v_block_stride * esize % 16 == 0;
-  const bool vec = ((dim | row_stride) & 3) == 0 && (((uintptr_t)q | (uintptr_t)k) & (4 * esize - 1)) == 0 &&
-                   (((uintptr_t)q_out | (uintptr_t)key_cache) & 15) == 0 && k_block_stride * esize % 16 == 0;
-  const bool vec8 = vec && esize == 2 && ((dim | row_stride) & 7) == 0 && (((uintptr_t)q | (uintptr_t)k) & 15) == 0;
-  const int64_t items = (int64_t)rows * (heads + (tiled ? 1 : 2) * kv_heads);
-  LV_CHECK(items <= INT32_MAX && kv_heads <= 65535, "too many rows");
-#define LV_QK(VEC_)                                                                                                          \
-  hipLaunchKernelGGL((qk_norm_cache_kernel<scalar_t, kL, VEC_>), grid, dim3(256), 0, (hipStream_t)stream, (S*)q_out,          \
-                     (S*)key_cache, (S*)value_cache, (const S*)q, (const S*)k, (const S*)v, row_stride, q_weight, k_weight,  \
-                     eps, rows, heads, kv_heads, dim, vdim, kpad, vpad, !tiled, slot_mapping, num_blocks * block_size,       \
-                     block_size, k_block_stride, v_block_stride)
-  LV_DISPATCH_DTYPE(dtype, {
-    using S = scalar_t::store_t;
-    constexpr int kWide = sizeof(S) == 2 ? 8 : 4;  // elements of a 16-byte piece
-    const int lanes = lanes_for(kpad, vec8 ? kWide : vec ? 4 : 1);
-    const dim3 grid((unsigned)((items * lanes + 255) / 256));
-    LV_LANES(lanes, {
-      if (vec8) LV_QK(kWide);
-      else if (vec) LV_QK(4);
-      else LV_QK(1);
-    })
-    if (tiled)
-      hipLaunchKernelGGL((value_cache_tile_kernel<S>), dim3((rows + kValueTile - 1) / kValueTile, kv_heads), dim3(256), smem,
-                         (hipStream_t)stream, (S*)value_cache, (const S*)v, row_stride, rows, vdim, vpad, slot_mapping,
-                         num_blocks * block_size, block_size, v_block_stride);
-  });
-#undef LV_QK
-  LV_LAUNCH_CHECK();
-  return 0;
-}
-
-extern "C" int lvllm_head_norm_gate(void* out, int64_t out_stride, const float* o, const void* gate, int64_t gate_stride,
-                                    const float* weight, int weight_head_stride, float eps, float scale, int rows,
-                                    int heads, int vdim, int dtype, void* stream) {
-  if (rows == 0) return 0;
-  const int64_t items = (int64_t)rows * heads;
-  const int esize = dtype == LVLLM_F32 ? 4 : 2;
-  const bool vec = ((vdim | out_stride | gate_stride) & 3) == 0 && ((uintptr_t)o & 15) == 0 &&
-                   (((uintptr_t)out | (uintptr_t)gate) & (4 * esize - 1)) == 0;
-  const int lanes = lanes_for(vdim, vec ? 4 : 1);
-  const dim3 grid((unsigned)((items * lanes + 255) / 256));
-  LV_DISPATCH_DTYPE(dtype, {
-    using S = scalar_t::store_t;
-    LV_LANES(lanes, {
-      if (vec)
-        hipLaunchKernelGGL((head_norm_gate_kernel<scalar_t, kL, 4>), grid, dim3(256), 0, (hipStream_t)stream, (S*)out,
-                           out_stride, o, (const S*)gate, gate_stride, weight, weight_head_stride, eps, scale, rows, heads, vdim);
-      else
-        hipLaunchKernelGGL((head_norm_gate_kernel<scalar_t, kL, 1>), grid, dim3(256), 0, (hipStream_t)stream, (S*)out,
-                           out_stride, o, (const S*)gate, gate_stride, weight, weight_head_stride, eps, scale, rows, heads, vdim);
-    })
-  });
   LV_LAUNCH_CHECK();
   return 0;
 }

@@ -136,4 +136,31 @@ struct Addend {
   return {kc.size(2) * kc.size(4), vc.size(2), vc.size(3)};
 }
 
+// rotary positions, rows of projections, integer tables, block tables
+[[maybe_unused]] void check_rot(const torch::Tensor& positions, const torch::Tensor& turns, int64_t rows, const char* op) {
+  TORCH_CHECK(positions.is_cuda() && positions.scalar_type() == at::kLong && positions.is_contiguous() &&
+                  positions.numel() >= rows && turns.is_cuda() && turns.scalar_type() == at::kDouble &&
+                  turns.is_contiguous(),
+              op, ": positions int64 [rows] and turns float64 [rot_dims / 2] on the device");
+}
+[[maybe_unused]] void check_rows2d(const torch::Tensor& t, int64_t rows, int64_t cols, at::ScalarType dtype, const char* op, const char* what) {
+  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == rows && t.size(1) == cols && t.stride(1) == 1 &&
+                  t.scalar_type() == dtype,
+              op, ": ", what, " must be [", rows, ", ", cols, "] rows of the compute dtype");
+}
+[[maybe_unused]] void check_i32(const torch::Tensor& t, int64_t least, const char* op, const char* what) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kInt && t.is_contiguous() && t.numel() >= least, op, ": ", what,
+              " must be ", least, " or more contiguous int32 elements on the device");
+}
+[[maybe_unused]] void check_tables(const torch::Tensor& block_tables, int64_t num_seqs, const char* op) {
+  TORCH_CHECK(block_tables.is_cuda() && block_tables.dim() == 2 && block_tables.scalar_type() == at::kInt &&
+                  block_tables.is_contiguous() && block_tables.size(0) >= num_seqs,
+              op, ": block_tables int32 [num_seqs, blocks]");
+}
+[[maybe_unused]] void check_slots(const torch::Tensor& slot_mapping, int64_t rows, const char* op) {
+  TORCH_CHECK(slot_mapping.is_cuda() && slot_mapping.scalar_type() == at::kLong && slot_mapping.is_contiguous() &&
+                  slot_mapping.numel() >= rows,
+              op, ": slot_mapping int64 [rows]");
+}
+
 }  // namespace

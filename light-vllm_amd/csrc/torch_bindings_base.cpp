@@ -234,6 +234,36 @@ torch::Tensor skinny_linear_packed_relu_squared(const torch::Tensor& x, const to
   return y;
 }
 
+// The clamped unit of a feed-forward's gate and up projection, [gate rows | up rows], in one launch: clamped_unit of the plain
+// projection
+torch::Tensor skinny_linear_packed_clamped_unit(const torch::Tensor& x, const torch::Tensor& w_packed, int64_t N, int64_t K,
+                                                double limit) {
+  const char* op = "skinny_linear_packed_clamped_unit";
+  TORCH_CHECK(x.dim() == 2 && x.size(1) == K && w_packed.numel() == N * K && N % 32 == 0, op, ": bad shapes");
+  TORCH_CHECK(skinny_ok(x, w_packed, std::nullopt), op, ": M <= 64 rows of bf16/f16 on the GPU only");
+  const int64_t M = x.size(0);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
+  auto y = torch::empty({M, N / 2}, x.options());
+  const int64_t ws_bytes = lvllm_skinny_gemm_workspace_bytes((int)M, (int)N, (int)K);
+  torch::Tensor ws;
+  if (ws_bytes > 0) ws = torch::empty({ws_bytes / 4}, x.options().dtype(torch::kFloat));
+  check(lvllm_skinny_gemm_clamped_unit(y.data_ptr(), x.data_ptr(), w_packed.data_ptr(), (int)M, (int)N, (int)K, x.stride(0),
+                                       dtype_code(x, op), 1, (float)limit, ws_bytes > 0 ? ws.data_ptr() : nullptr, ws_bytes,
+                                       current_stream(x)));
+  return y;
+}
+
+torch::Tensor clamped_unit(const torch::Tensor& x, double limit) {
+  const char* op = "clamped_unit";
+  LV_CHECK_DEVICE(x);
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.size(1) % 2 == 0, op, ": contiguous [rows, gate | up]");
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
+  auto y = torch::empty({x.size(0), x.size(1) / 2}, x.options());
+  check(lvllm_clamped_unit(y.data_ptr(), x.data_ptr(), x.size(0), (int)y.size(1), (float)limit, dtype_code(x, op),
+                           current_stream(x)));
+  return y;
+}
+
 // A projection that leaves its fp32 split-K partials [S, M, N] for fused_add_rms_norm_splitk
 // instead of reducing them itself.  swiglu: x = [gate | up] ([M, 2K]) and the activation is applied
 // while loading x (bit-identical to silu_and_mul, but every workgroup redoes it for its K slice:
@@ -623,6 +653,10 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, amd) {
   amd.impl("pack_weight", torch::kCUDA, &pack_weight);
   amd.def("skinny_linear_packed_argmax(Tensor x, Tensor w_packed, int N, int K) -> Tensor");
   amd.impl("skinny_linear_packed_argmax", torch::kCUDA, &skinny_linear_packed_argmax);
+  amd.def("skinny_linear_packed_clamped_unit(Tensor x, Tensor w_packed, int N, int K, float limit) -> Tensor");
+  amd.impl("skinny_linear_packed_clamped_unit", torch::kCUDA, &skinny_linear_packed_clamped_unit);
+  amd.def("clamped_unit(Tensor x, float limit) -> Tensor");
+  amd.impl("clamped_unit", torch::kCUDA, &clamped_unit);
   amd.def("skinny_linear_packed_relu_squared(Tensor x, Tensor w_packed, int N, int K) -> Tensor");
   amd.impl("skinny_linear_packed_relu_squared", torch::kCUDA, &skinny_linear_packed_relu_squared);
   amd.def("stream_linear_packed(Tensor x, Tensor w_packed, Tensor? bias, int N, int K) -> Tensor");

@@ -54,34 +54,6 @@ void relu_squared(torch::Tensor& out, const torch::Tensor& x) {
   check(lvllm_relu_squared(out.data_ptr(), x.data_ptr(), x.numel(), dtype_code(x, "relu_squared"), current_stream(x)));
 }
 
-torch::Tensor qk_norm_cache(const torch::Tensor& q, const torch::Tensor& k, const torch::Tensor& v,
-                            const torch::Tensor& q_weight, const torch::Tensor& k_weight, double eps, int64_t heads,
-                            int64_t kv_heads, torch::Tensor& key_cache, torch::Tensor& value_cache,
-                            const torch::Tensor& slot_mapping) {
-  const char* op = "qk_norm_cache";
-  LV_CHECK_DEVICE(q);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
-  const int64_t rows = q.size(0), dim = q.size(1) / heads, vdim = v.size(1) / kv_heads;
-  TORCH_CHECK(q.dim() == 2 && k.dim() == 2 && v.dim() == 2 && q.size(1) == heads * dim && k.size(1) == kv_heads * dim &&
-                  v.size(1) == kv_heads * vdim && k.size(0) == rows && v.size(0) == rows && q.stride(1) == 1 &&
-                  k.stride(1) == 1 && v.stride(1) == 1 && q.stride(0) == k.stride(0) && q.stride(0) == v.stride(0) &&
-                  k.scalar_type() == q.scalar_type() && v.scalar_type() == q.scalar_type(),
-              op, ": q [rows, heads * dim], k [rows, kv_heads * dim], v [rows, kv_heads * vdim] with one row stride");
-  check_f32(q_weight, dim, op, "q_weight");
-  check_f32(k_weight, dim, op, "k_weight");
-  const auto [kpad, vpad, bs] = head_cache_dims(key_cache, value_cache, kv_heads, q.scalar_type(), op);
-  TORCH_CHECK(slot_mapping.is_cuda() && slot_mapping.scalar_type() == at::kLong && slot_mapping.is_contiguous() &&
-                  slot_mapping.numel() >= rows,
-              op, ": slot_mapping int64 [rows]");
-  auto q_out = torch::empty({rows, heads, kpad}, q.options());
-  check(lvllm_qk_norm_cache(q_out.data_ptr(), key_cache.data_ptr(), value_cache.data_ptr(), q.data_ptr(), k.data_ptr(),
-                            v.data_ptr(), q.stride(0), q_weight.data_ptr<float>(), k_weight.data_ptr<float>(), (float)eps,
-                            (int)rows, (int)heads, (int)kv_heads, (int)dim, (int)vdim, (int)kpad, (int)vpad,
-                            slot_mapping.data_ptr<int64_t>(), key_cache.size(0), (int)bs, key_cache.stride(0),
-                            value_cache.stride(0), dtype_code(q, op), current_stream(q)));
-  return q_out;
-}
-
 void head_norm_gate(torch::Tensor& out, const torch::Tensor& o, const torch::Tensor& gate, const torch::Tensor& weight,
                     double eps, double scale) {
   const char* op = "head_norm_gate";
@@ -199,9 +171,6 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, hybrid) {
   hybrid.impl("add_dyt_shift_mix", torch::kCUDA, &add_dyt_shift_mix);
   hybrid.def("relu_squared(Tensor(a!) out, Tensor x) -> ()");
   hybrid.impl("relu_squared", torch::kCUDA, &relu_squared);
-  hybrid.def("qk_norm_cache(Tensor q, Tensor k, Tensor v, Tensor q_weight, Tensor k_weight, float eps, int heads, "
-             "int kv_heads, Tensor(a!) key_cache, Tensor(b!) value_cache, Tensor slot_mapping) -> Tensor");
-  hybrid.impl("qk_norm_cache", torch::kCUDA, &qk_norm_cache);
   hybrid.def("recurrent_mix(Tensor(a!) out, Tensor q, Tensor k, Tensor v, Tensor u, Tensor a_t, Tensor decay_bias, "
              "int kind, float inv_tau, Tensor? bonus, float q_scale, Tensor gate, Tensor norm_weight, float eps, "
              "float out_scale, Tensor(b!) state, Tensor state_slots, Tensor query_start_loc, Tensor seq_lens, "

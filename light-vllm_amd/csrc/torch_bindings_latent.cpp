@@ -1,34 +1,12 @@
-// torch op registrations of the latent library: latent attention, mixtures of experts, norms on sublayer outputs with depth
-// averages.
+// torch op registrations of the latent library: latent attention, norms on sublayer outputs with depth averages.
 #include "torch_bindings.h"
 
 namespace {
 
-void check_rot(const torch::Tensor& positions, const torch::Tensor& turns, int64_t rows, const char* op) {
-  TORCH_CHECK(positions.is_cuda() && positions.scalar_type() == at::kLong && positions.is_contiguous() &&
-                  positions.numel() >= rows && turns.is_cuda() && turns.scalar_type() == at::kDouble &&
-                  turns.is_contiguous(),
-              op, ": positions int64 [rows] and turns float64 [rot_dims / 2] on the device");
-}
 void check_latent_rows(const torch::Tensor& cache, int64_t cpad, int64_t rpad, const char* op) {
   TORCH_CHECK(cache.is_cuda() && cache.dim() == 3 && cache.size(2) == cpad + rpad && blocks_are_dense(cache), op,
               ": cache [blocks, block_size, cpad + rpad], blocks dense");
 }
-void check_rows2d(const torch::Tensor& t, int64_t rows, int64_t cols, at::ScalarType dtype, const char* op, const char* what) {
-  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == rows && t.size(1) == cols && t.stride(1) == 1 &&
-                  t.scalar_type() == dtype,
-              op, ": ", what, " must be [", rows, ", ", cols, "] rows of the compute dtype");
-}
-void check_i32(const torch::Tensor& t, int64_t least, const char* op, const char* what) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kInt && t.is_contiguous() && t.numel() >= least, op, ": ", what,
-              " must be ", least, " or more contiguous int32 elements on the device");
-}
-void check_tables(const torch::Tensor& block_tables, int64_t num_seqs, const char* op) {
-  TORCH_CHECK(block_tables.is_cuda() && block_tables.dim() == 2 && block_tables.scalar_type() == at::kInt &&
-                  block_tables.is_contiguous() && block_tables.size(0) >= num_seqs,
-              op, ": block_tables int32 [num_seqs, blocks]");
-}
-
 void latent_cache(torch::Tensor& cache, const torch::Tensor& kv, const torch::Tensor& weight, double eps, int64_t cpad,
                   const torch::Tensor& positions, const torch::Tensor& turns, const torch::Tensor& slot_mapping) {
   const char* op = "latent_cache";
@@ -169,60 +147,6 @@ torch::Tensor latent_rotate_query(const torch::Tensor& q, int64_t heads, int64_t
   return out;
 }
 
-// (ids, weights, offsets, token, slots, tiles)
-std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_route(
-    const torch::Tensor& h, const torch::Tensor& w, const torch::Tensor& bias, int64_t top, bool shared, bool packed) {
-  const char* op = "moe_route";
-  LV_CHECK_DEVICE(h);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(h));
-  const int64_t rows = h.size(0), width = h.size(1), experts = bias.numel();
-  TORCH_CHECK(h.dim() == 2 && h.is_contiguous() && w.is_cuda() && w.dim() == 2 && w.is_contiguous() && w.size(1) == width &&
-                  w.scalar_type() == h.scalar_type() &&
-                  w.size(0) == (packed ? (experts + shared + 15) / 16 * 16 : experts + shared),
-              op, ": h [rows, width], w [experts (+ 1), width], packed: rows up to a multiple of 16");
-  check_f32(bias, experts, op, "bias");
-  const auto ints = h.options().dtype(at::kInt);
-  const int64_t n = top + shared, total = rows * n, tile = lvllm_moe_tile(packed, (int)rows);
-  const int64_t max_tiles = std::max<int64_t>(1, std::min(total, total / tile + experts + shared));
-  auto ids = torch::empty({rows, n}, ints), slot = torch::empty({rows, n}, ints), token = torch::empty({total}, ints);
-  auto offsets = torch::empty({experts + shared + 1}, ints), tiles = torch::empty({max_tiles + 1, 4}, ints);
-  auto weights = torch::empty({rows, n}, h.options().dtype(at::kFloat));
-  const int64_t need = lvllm_moe_route_workspace_bytes((int)experts, shared, (int)rows, (int)width, packed);
-  auto ws = torch::empty({need}, h.options().dtype(at::kByte));
-  check(lvllm_moe_route(ids.data_ptr<int>(), weights.data_ptr<float>(), offsets.data_ptr<int>(), token.data_ptr<int>(),
-                        slot.data_ptr<int>(), tiles.data_ptr<int>(), (int)max_tiles, h.data_ptr(), w.data_ptr(),
-                        bias.data_ptr<float>(), (int)experts, shared, (int)top, (int)rows, (int)width, packed, ws.data_ptr(),
-                        need, dtype_code(h, op), current_stream(h)));
-  return {ids, weights, offsets, token, slot, tiles};
-}
-
-torch::Tensor moe_experts(const torch::Tensor& x, const torch::Tensor& w, const torch::Tensor& w_offset,
-                          const torch::Tensor& ff, const torch::Tensor& limit, const torch::Tensor& offsets,
-                          const torch::Tensor& token, const torch::Tensor& tiles, int64_t rows, int64_t width, int64_t ff_max,
-                          int64_t ff_first, int64_t ff_last, bool up, bool packed) {
-  const char* op = "moe_experts";
-  LV_CHECK_DEVICE(x);
-  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
-  const int64_t experts = ff.numel(), slots = token.numel();
-  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.size(0) == (up ? rows : slots) && x.size(1) == (up ? width : ff_max), op,
-              ": x must be [rows, width] going up, [slots, ff_max] going down");
-  TORCH_CHECK(w.is_cuda() && w.is_contiguous() && w.scalar_type() == x.scalar_type() && w_offset.is_cuda() &&
-                  w_offset.scalar_type() == at::kLong && w_offset.numel() == experts,
-              op, ": one weight buffer and int64 offsets [experts]");
-  check_i32(ff, experts, op, "ff");
-  check_f32(limit, experts, op, "limit");
-  check_i32(offsets, experts + 1, op, "offsets");
-  check_i32(token, slots, op, "token");
-  check_i32(tiles, 8, op, "tiles");
-  auto out = torch::empty({slots, up ? ff_max : width}, x.options());
-  check(lvllm_moe_experts(out.data_ptr(), x.data_ptr(), w.data_ptr(), w_offset.data_ptr<int64_t>(), ff.data_ptr<int>(),
-                          limit.data_ptr<float>(), offsets.data_ptr<int>(), token.data_ptr<int>(), tiles.data_ptr<int>(),
-                          (int)experts, (int)slots, (int)rows, (int)width, (int)ff_max, (int)ff_first, (int)ff_last,
-                          (int)tiles.size(0) - 1, up, packed,
-                          dtype_code(x, op), current_stream(x)));
-  return out;
-}
-
 torch::Tensor embed_scale(torch::Tensor& x, const torch::Tensor& table, const torch::Tensor& ids, double scale) {
   const char* op = "embed_scale";
   check_residual(x, op);
@@ -310,13 +234,6 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, latent) {
   latent.impl("latent_expand", torch::kCUDA, &latent_expand);
   latent.def("latent_rotate_query(Tensor q, int heads, int dim, int kpad, Tensor positions, Tensor turns) -> Tensor");
   latent.impl("latent_rotate_query", torch::kCUDA, &latent_rotate_query);
-  latent.def("moe_route(Tensor h, Tensor w, Tensor bias, int top, bool shared, bool packed) "
-             "-> (Tensor, Tensor, Tensor, Tensor, Tensor, Tensor)");
-  latent.impl("moe_route", torch::kCUDA, &moe_route);
-  latent.def("moe_experts(Tensor x, Tensor w, Tensor w_offset, Tensor ff, Tensor limit, Tensor offsets, Tensor token, "
-             "Tensor tiles, int rows, int width, int ff_max, int ff_first, int ff_last, bool up, bool packed) "
-             "-> Tensor");
-  latent.impl("moe_experts", torch::kCUDA, &moe_experts);
   latent.def("embed_scale(Tensor(a!) x, Tensor table, Tensor ids, float scale) -> Tensor");
   latent.impl("embed_scale", torch::kCUDA, &embed_scale);
   latent.def("norm_add_mix(Tensor(a!)? x_out, Tensor(b!)? v_out, Tensor x, Tensor y, Tensor? slots, Tensor? slot_weights, "

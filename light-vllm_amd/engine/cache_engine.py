@@ -7,6 +7,7 @@ Behaviour of light_vllm/decoding/worker/cache_engine.py:15-103: zero-initialised
 (:33-36), `block bytes = 2 * L * block_size * kv_heads * head_size * sizeof(element)`, swaps layer
 by layer through the backend, copy-on-write copies in one fused call.
 """
+import math
 from typing import List, Optional, Tuple
 
 import torch
@@ -17,10 +18,11 @@ _FP8_NAMES = ("fp8", "fp8_e4m3")
 
 
 class ModelCaches:
-    """One LayerCache per layer (engine/mixers.py) and the block size they are paged in."""
+    """One LayerCache per layer (engine/mixers.py), the block size they are paged in, and what a sequence carries besides its
+    layers' states (name -> [slots, ...])."""
 
-    def __init__(self, layers, block_size: int) -> None:
-        self.layers, self.block_size = layers, block_size
+    def __init__(self, layers, block_size: int, sequence=None) -> None:
+        self.layers, self.block_size, self.sequence = layers, block_size, sequence or {}
 
 
 class CacheEngine:
@@ -39,6 +41,14 @@ class CacheEngine:
         self.gpu_cache = self._allocate(self.num_gpu_blocks, self.device)
         self.cpu_cache = self._allocate(self.num_cpu_blocks, torch.device("cpu"))
         self.state = self._allocate_state(model_config, cache_config.num_state_slots, self.device)
+        self.sequence_state = {name: torch.zeros(cache_config.num_state_slots, *shape, dtype=dtype, device=self.device)
+                               for name, (shape, dtype) in self.sequence_state_specs(model_config).items()}
+
+    @staticmethod
+    def sequence_state_specs(model_config):
+        """name -> (shape, dtype) of a model with recurrent state, {} for the others."""
+        specs = getattr(model_config, "sequence_state_specs", None)
+        return specs() if specs is not None else {}
 
     @staticmethod
     def _allocate_state(model_config, num_slots: Optional[int], where: torch.device):
@@ -59,12 +69,13 @@ class CacheEngine:
         from .mixers import LayerCache
         kv = iter(self.gpu_cache)
         return ModelCaches([LayerCache(next(kv) if spec is not None else None, state)
-                            for spec, state in zip(self.kv_specs, self.state or [{}] * len(self.kv_specs))], self.block_size)
+                            for spec, state in zip(self.kv_specs, self.state or [{}] * len(self.kv_specs))], self.block_size,
+                           self.sequence_state)
 
     def copy_state(self, pairs: List[Tuple[int, int]]) -> None:
         """Forked sequences: [(source slot, destination slot)] of every layer's state."""
         idx = torch.tensor(pairs, dtype=torch.long, device=self.device)
-        for layer in self.state:
+        for layer in (*self.state, self.sequence_state):
             for t in layer.values():
                 t.index_copy_(0, idx[:, 1], t.index_select(0, idx[:, 0]))
 
@@ -176,11 +187,7 @@ class CacheEngine:
         specs = model_config.state_specs()
         if specs is None:
             return 0
-        n = 0
-        for s in specs:
-            for shape in s.values():
-                k = 1
-                for d in shape:
-                    k *= d
-                n += k
-        return 4 * n * num_slots
+        n = sum(4 * math.prod(shape) for s in specs for shape in s.values())
+        n += sum(math.prod(shape) * torch.empty((), dtype=dtype).element_size()
+                 for shape, dtype in CacheEngine.sequence_state_specs(model_config).values())
+        return n * num_slots

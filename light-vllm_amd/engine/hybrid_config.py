@@ -15,9 +15,12 @@ class KVSpec:
     kv_heads: int
     dim: int
     vdim: int
+    maps: int = 1    # key vectors per kv head (csrc/head_attention.h), each padded by itself
 
     @property
     def kpad(self) -> int:
+        if self.maps == 2:
+            return 2 * self._padded(self.dim, (32, 64, 96, 128))
         return self._padded(self.dim, (64, 96, 128, 192, 256))
 
     @property

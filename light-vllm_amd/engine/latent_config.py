@@ -8,6 +8,8 @@ from typing import List, Optional
 
 import torch
 
+from .moe import ExpertConfig, MixtureConfig
+
 
 @dataclass(frozen=True)
 class RotationConfig:
@@ -58,21 +60,6 @@ class LatentAttentionConfig:
     @property
     def spec(self) -> LatentKVSpec:
         return LatentKVSpec(self.kv_rank, self.rot_dim)
-
-
-@dataclass(frozen=True)
-class ExpertConfig:
-    ff: int
-    limit: float
-
-
-@dataclass(frozen=True)
-class MixtureConfig:
-    """`top` of `experts` small feed-forwards per token, and one that every token takes."""
-    experts: int
-    top: int
-    expert: ExpertConfig
-    shared: Optional[ExpertConfig]
 
 
 @dataclass(frozen=True)

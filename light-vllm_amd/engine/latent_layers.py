@@ -1,31 +1,25 @@
-"""Sublayers of latent decoders on the gfx950 operators: latent attention, the mixture of experts, and the norm on a
-sublayer's output with the residual add and the average over the depth.
+"""Sublayers of latent decoders on the gfx950 operators: latent attention, and the norm on a sublayer's output with the
+residual add and the average over the depth (the mixture of experts: engine/moe.py).
 
 A mixer takes the rows h it reads (compute dtype) and returns its projection: [rows, width], or the fp32 split-K slabs of a
 decode-size step; the mixture returns its assignments' rows, which the norm's launch sums.  Constants come from the
 configuration; nothing here knows a model's sizes."""
 from dataclasses import dataclass
-from typing import Dict, List, NamedTuple, Optional
+from typing import Dict, List, Optional
 
 import numpy as np
 import torch
 import torch.nn.functional as F
 
 from .hybrid_config import KVSpec
-from .latent_config import LatentAttentionConfig, MixtureConfig, RotationConfig
+from .latent_config import LatentAttentionConfig, RotationConfig
 from .mixers import StepLayout, ceil_to, make_weight, pad_columns, project_to_residual, stack_rows
 from .model import linear
+from .moe import MixtureOfExperts, SublayerOutput, interleave_16  # noqa: F401
 
 amd = torch.ops._C_amd
 ABSORBED_MAX = 64      # portions of up to this many tokens attend in latent space (csrc/latent_attention.h)
 UNBOUNDED = 1 << 30
-
-
-class SublayerOutput(NamedTuple):
-    """What a sublayer adds to the stream: rows (or split-K slabs), or the rows of a mixture's slots."""
-    y: torch.Tensor
-    slots: Optional[torch.Tensor] = None      # int32 [rows, assignments]
-    weights: Optional[torch.Tensor] = None    # float32 [rows, assignments]
 
 
 class OutputNorm:
@@ -168,55 +162,3 @@ class LatentAttention:
         qr = amd.latent_rotate_query(q, c.heads, c.dim, p.kpad, l.positions, self.rotation.turns)
         amd.head_attention(out, qr, keys, values, plan.tables, plan.seq_lens, l.query_start_loc, gate, c.vdim, c.scale, 1.0,
                            l.max_query_len, plan.max_seq_len, c.window, ABSORBED_MAX + 1)
-
-
-def interleave_16(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
-    """[ff, k] twice -> [2 ffp, k]: 16 rows of one, 16 of the other, ...; ffp: ff up to a multiple of 32 with zero rows."""
-    pad = ceil_to(gate.shape[0], 32) - gate.shape[0]
-    g, u = (F.pad(t, (0, 0, 0, pad)).view(-1, 1, 16, t.shape[1]) for t in (gate, up))
-    return torch.cat([g, u], 1).reshape(-1, gate.shape[1])
-
-
-class MixtureOfExperts:
-    """The shared expert is one more expert of the grouped products, with sizes and a limit of its own."""
-
-    def __init__(self, get, name: str, cfg: MixtureConfig, pack: bool):
-        self.cfg = cfg
-        router, self.bias = get(name + ".router"), get(name + ".router.b").float().contiguous()
-        names, ff = [f"{name}.e{i}" for i in range(cfg.experts)], [cfg.expert.ff] * cfg.experts
-        limits = [cfg.expert.limit] * cfg.experts
-        if cfg.shared is not None:
-            names.append(name + ".shared")
-            ff.append(cfg.shared.ff)
-            limits.append(cfg.shared.limit)
-            router = torch.cat([router, get(name + ".shared.sg")])
-        self.width, dev = router.shape[1], router.device
-        self.packed = pack and router.dtype == torch.bfloat16 and self.width % 32 == 0
-        self.router = amd.pack_weight(stack_rows([router])[0]) if self.packed else router.contiguous()
-        ffp = [ceil_to(n, 32) for n in ff]
-        self.ff_max, self.ff_first, self.ff_last, self.experts = max(ffp), max(ffp[:-1] or ffp), ffp[-1], len(names)
-        up_at, down_at = ([0] + np.cumsum([k * n * self.width for n in ffp]).tolist() for k in (2, 1))
-        self.up = torch.empty(up_at[-1], dtype=router.dtype, device=dev)
-        self.down = torch.empty(down_at[-1], dtype=router.dtype, device=dev)
-        for i, s in enumerate(names):
-            up = interleave_16(get(s + ".gate"), get(s + ".up"))
-            down = pad_columns(get(s + ".down")).contiguous()
-            if self.packed:
-                up, down = amd.pack_weight(up), amd.pack_weight(down)
-            self.up[up_at[i]:up_at[i + 1]] = up.reshape(-1)
-            self.down[down_at[i]:down_at[i + 1]] = down.reshape(-1)
-        self.up_at, self.down_at = (torch.tensor(a[:-1], dtype=torch.int64, device=dev) for a in (up_at, down_at))
-        self.ff = torch.tensor(ffp, dtype=torch.int32, device=dev)
-        self.limits = torch.tensor(limits, dtype=torch.float32, device=dev)
-
-    def numel(self) -> int:
-        return self.up.numel() + self.down.numel()
-
-    def __call__(self, h: torch.Tensor) -> SublayerOutput:
-        _, weights, offsets, token, slots, tiles = amd.moe_route(h, self.router, self.bias, self.cfg.top,
-                                                                 self.cfg.shared is not None, self.packed)
-        rows = h.shape[0]
-        sizes = rows, self.width, self.ff_max, self.ff_first, self.ff_last
-        a = amd.moe_experts(h, self.up, self.up_at, self.ff, self.limits, offsets, token, tiles, *sizes, True, self.packed)
-        y = amd.moe_experts(a, self.down, self.down_at, self.ff, self.limits, offsets, token, tiles, *sizes, False, self.packed)
-        return SublayerOutput(y, slots, weights)

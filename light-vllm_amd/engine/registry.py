@@ -39,7 +39,9 @@ MODELS = {
     "Sasilorn": ModelEntry(".hybrid_config:HybridModelConfig", ".hybrid_model:HybridModel",
                            "..attention.head_backend:HeadAttnBackend", ("heads", "hybrid")),
     "Lepalorn": ModelEntry(".latent_config:LatentModelConfig", ".latent_model:LatentModel",
-                           "..attention.latent_backend:LatentAttnBackend", ("heads", "latent")),
+                           "..attention.latent_backend:LatentAttnBackend", ("heads", "moe", "latent")),
+    "Lizazen": ModelEntry(".local_config:LocalModelConfig", ".local_model:LocalModel",
+                          "..attention.head_backend:HeadAttnBackend", ("heads", "moe", "local")),
 }
 
 
