@@ -110,6 +110,10 @@ def parse():
                     help="instead of the headline workload: prefill and decode throughput of the latent decoder beside the "
                          "rotary decoder at equal sizes (tools/bench_latent.py)")
     ap.add_argument("--latent-only", default=None, help="with --latent: the cases whose name starts with this")
+    ap.add_argument("--local", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the local decoder beside the "
+                         "hybrid decoder at equal sizes (tools/bench_local.py)")
+    ap.add_argument("--local-only", default=None, help="with --local: the cases whose name starts with this")
     ap.add_argument("--tiny", action="store_true", help="tiny model (plumbing check)")
     ap.add_argument("--replica-backend", default=None, choices=["nccl", "gloo"],
                     help="process-group backend of the barrier / clock between replicas (default: nccl = RCCL)")
@@ -853,6 +857,11 @@ def main():
         sys.path.insert(0, os.path.join(ROOT, "tools"))
         import bench_latent
         print(json.dumps({"latent": bench_latent.run("cuda:0", a.latent_only)}), flush=True)
+        return
+    if a.local:
+        sys.path.insert(0, os.path.join(ROOT, "tools"))
+        import bench_local
+        print(json.dumps({"local": bench_local.run("cuda:0", a.local_only)}), flush=True)
         return
     if a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(spawn_replicas(a))
