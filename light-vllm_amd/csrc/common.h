@@ -223,6 +223,23 @@ __device__ inline float block_sum(float v, float* red) {
   return r;
 }
 
+// ... of two values at once; `red` is 32 floats.
+__device__ inline float2 block_sum2(float a, float b, float* red) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int nw = (blockDim.x + 63) >> 6;
+  a = wave_sum(a);
+  b = wave_sum(b);
+  if (lane == 0) {
+    red[wave] = a;
+    red[16 + wave] = b;
+  }
+  __syncthreads();
+  a = wave_sum(lane < nw ? red[lane] : 0.f);
+  b = wave_sum(lane < nw ? red[16 + lane] : 0.f);
+  __syncthreads();
+  return float2{a, b};
+}
+
 #define LV_DISPATCH_DTYPE(dtype, ...)            \
   switch (dtype) {                               \
     case LVLLM_F32: {                            \

@@ -153,24 +153,28 @@ __global__ __launch_bounds__(256) void rotary_cache_kernel(const RotaryCachePara
   using S = typename T::store_t;
   constexpr int x = 16 / sizeof(S);
   extern __shared__ float cs[];  // [rot_dims / 2] cosines, then sines
-  __shared__ float red[16];
+  __shared__ float red[32];
   const int row = blockIdx.x, half = p.rot_dims / 2;
   const S* q = (const S*)p.q + row * p.row_stride;
   const S* k = (const S*)p.k + row * p.row_stride;
   const int64_t pos = p.positions[row], slot = p.slot_mapping[row];
   for (int i = threadIdx.x; i < half; i += 256) rotation_of(pos, p.turns[i], cs[i], cs[half + i]);
-  auto norm_of = [&](const S* src, int n) {
-    float ss = 0.f, f[VEC];
-    for (int d = threadIdx.x * VEC; d < n; d += 256 * VEC) {
-      load_vec<T, VEC>(src + d, f);
-#pragma unroll
-      for (int j = 0; j < VEC; ++j) ss = fmaf(f[j], f[j], ss);
-    }
-    return 1.f / sqrtf(block_sum(ss, red) / (float)n + p.eps);
-  };
   const int nq = p.heads * p.maps, nk = p.kv_heads * p.maps;
-  const float fq = p.q_weight != nullptr ? norm_of(q, nq * p.dim) : 1.f;
-  const float fk = p.k_weight != nullptr ? norm_of(k, nk * p.dim) : 1.f;
+  float fq = 1.f, fk = 1.f;
+  if (p.q_weight != nullptr || p.k_weight != nullptr) {
+    auto squares = [&](const S* src, int n) __attribute__((always_inline)) {
+      float ss = 0.f, f[VEC];
+      for (int d = threadIdx.x * VEC; d < n; d += 256 * VEC) {
+        load_vec<T, VEC>(src + d, f);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss = fmaf(f[j], f[j], ss);
+      }
+      return ss;
+    };
+    const float2 ss = block_sum2(squares(q, nq * p.dim), squares(k, nk * p.dim), red);
+    fq = 1.f / sqrtf(ss.x / (float)(nq * p.dim) + p.eps);
+    fk = 1.f / sqrtf(ss.y / (float)(nk * p.dim) + p.eps);
+  }
   __syncthreads();
   const bool stored = slot >= 0 && slot < p.num_slots;
   const int64_t block = stored ? slot / p.block_size : 0;

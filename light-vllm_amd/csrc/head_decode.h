@@ -179,22 +179,30 @@ __global__ __launch_bounds__(128) void head_decode_reduce_kernel(const HeadAttnP
   if (seq >= p.num_seqs) return;
   const int qlen = p.query_start_loc[seq + 1] - p.query_start_loc[seq];
   if (qlen < p.min_query_len || !takes_decode_body(qlen, p.heads / p.kv_heads * MAPS)) return;
+  // the shares' weights, one share per lane (nsplit <= 64), through LDS
+  __shared__ float weight[MAPS][64];
   const int64_t at = ((int64_t)row * p.heads + head) * MAPS * p.nsplit;
-  float m[MAPS], f[MAPS];
+  const int lane = threadIdx.x & 63;
 #pragma unroll
   for (int i = 0; i < MAPS; ++i) {
-    const float* ml = p.part_ml + 2 * (at + i * p.nsplit);
-    m[i] = -1e30f;
-    for (int s = 0; s < p.nsplit; ++s) m[i] = fmaxf(m[i], ml[2 * s]);
-    float l = 0.f;
-    for (int s = 0; s < p.nsplit; ++s) l += ml[2 * s + 1] * exp2f(ml[2 * s] - m[i]);
-    f[i] = l > 0.f ? 1.f / (l + sink_term(p, head, m[i])) : 0.f;
+    const float2 ml = lane < p.nsplit ? *reinterpret_cast<const float2*>(p.part_ml + 2 * (at + i * p.nsplit + lane)) : float2{-1e30f, 0.f};
+    const float m = wave_max(ml.x), w = lane < p.nsplit ? exp2f(ml.x - m) : 0.f, l = wave_sum(ml.y * w);
+    weight[i][lane] = l > 0.f ? w / (l + sink_term(p, head, m)) : 0.f;
   }
-  auto sum_of = [&](int i, int d) {
-    const int64_t first = at + i * p.nsplit;
+  __syncthreads();
+  auto sum_of = [&](int i, int d) __attribute__((always_inline)) {
+    constexpr int B = 8;  // loads in flight
+    const float* part = p.part_o + (at + i * p.nsplit) * p.vpad + d;
     float v = 0.f;
-    for (int s = 0; s < p.nsplit; ++s) v += p.part_o[(first + s) * p.vpad + d] * exp2f(p.part_ml[2 * (first + s)] - m[i]);
-    return v * f[i];
+    for (int s0 = 0; s0 < p.nsplit; s0 += B) {
+      float t[B];
+#pragma unroll
+      for (int s = 0; s < B; ++s) t[s] = part[(int64_t)min(s0 + s, p.nsplit - 1) * p.vpad];
+#pragma unroll
+      for (int s = 0; s < B; ++s)
+        if (s0 + s < p.nsplit) v = fmaf(t[s], weight[i][s0 + s], v);
+    }
+    return v;
   };
   uint16_t* out = (uint16_t*)p.out + row * p.out_stride + (int64_t)head * p.vdim;
   const float gate = gate_of<BF16>(p, row, head);

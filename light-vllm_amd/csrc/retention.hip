@@ -4,8 +4,8 @@
 
 namespace lvllm {
 
-// A workgroup per row: the row's angles once, through LDS.
-template <typename T>
+// A workgroup per row: the row's angles once, through LDS; a thread takes VEC neighbouring entries and their partners.
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void rotate_rows_kernel(float* __restrict__ q_out, float* __restrict__ k_out,
                                                           const typename T::store_t* __restrict__ q,
                                                           const typename T::store_t* __restrict__ k, const int64_t q_stride,
@@ -13,21 +13,24 @@ __global__ __launch_bounds__(256) void rotate_rows_kernel(float* __restrict__ q_
                                                           const double* __restrict__ turns, const int rot_dims, const int heads,
                                                           const int dk) {
   extern __shared__ float cs[];  // [rot_dims / 2] cosines, then sines
-  const int row = blockIdx.x, half = rot_dims / 2, n = heads * dk;
+  const int row = blockIdx.x, half = rot_dims / 2, n = heads * dk / VEC;
   for (int i = threadIdx.x; i < half; i += 256) rotation_of(positions[row], turns[i], cs[i], cs[half + i]);
   __syncthreads();
   for (int i = threadIdx.x; i < 2 * n; i += 256) {
     const bool is_q = i < n;
-    const int at = is_q ? i : i - n, h = at / dk, d = at - h * dk;
+    const int at = (is_q ? i : i - n) * VEC, d = at % dk;
     const typename T::store_t* src = is_q ? q + row * q_stride : k + row * k_stride;
-    float v = T::to_float(src[at]);
+    float v[VEC];
+    load_vec<T, VEC>(src + at, v);
     if (d < rot_dims) {
       const bool first = d < half;
       const int pair = first ? d : d - half;
-      const float t = T::to_float(src[first ? at + half : at - half]);
-      v = v * cs[pair] + (first ? -t : t) * cs[half + pair];
+      float t[VEC];
+      load_vec<T, VEC>(src + (first ? at + half : at - half), t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] = v[j] * cs[pair + j] + (first ? -t[j] : t[j]) * cs[half + pair + j];
     }
-    (is_q ? q_out : k_out)[(int64_t)row * n + at] = v;
+    store_vec<F32, VEC>((is_q ? q_out : k_out) + (int64_t)row * heads * dk + at, v);
   }
 }
 
@@ -72,8 +75,15 @@ extern "C" int lvllm_retention(void* out, int64_t out_stride, const void* q, con
   LV_CHECK((int64_t)num_seqs * p.max_segs <= 65535, "too many sequences or too long portions");
   LV_DISPATCH_F32_BF16(dtype, {
     using S = typename scalar_t::store_t;
-    hipLaunchKernelGGL((rotate_rows_kernel<scalar_t>), dim3(rows), dim3(256), (size_t)rot_dims * sizeof(float), s, qr, kr,
-                       (const S*)q, (const S*)k, q_stride, k_stride, positions, turns, rot_dims, heads, dk);
+    const bool vec = ((dk | (rot_dims / 2)) & 3) == 0 && ((q_stride | k_stride) & 3) == 0 &&
+                     (((uintptr_t)q | (uintptr_t)k) & (4 * sizeof(S) - 1)) == 0 && ((uintptr_t)qr & 15) == 0;
+    const size_t smem = (size_t)rot_dims * sizeof(float);
+    if (vec)
+      hipLaunchKernelGGL((rotate_rows_kernel<scalar_t, 4>), dim3(rows), dim3(256), smem, s, qr, kr, (const S*)q, (const S*)k,
+                         q_stride, k_stride, positions, turns, rot_dims, heads, dk);
+    else
+      hipLaunchKernelGGL((rotate_rows_kernel<scalar_t, 1>), dim3(rows), dim3(256), smem, s, qr, kr, (const S*)q, (const S*)k,
+                         q_stride, k_stride, positions, turns, rot_dims, heads, dk);
   });
   LV_LAUNCH_CHECK();
   p.q = qr; p.k = kr; p.q_stride = p.k_stride = (int64_t)heads * dk;

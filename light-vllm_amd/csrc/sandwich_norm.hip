@@ -34,7 +34,7 @@ template <typename T, int VEC, int ITEMS, int BRANCHES>
 __global__ __launch_bounds__(1024) void sandwich_norm_kernel(const SandwichParams p) {
   using S = typename T::store_t;
   constexpr int B = ITEMS <= 2 ? 8 : 4;  // rows in flight
-  __shared__ float red[BRANCHES == 2 ? 2 : 1][16];
+  __shared__ float red[BRANCHES * 16];
   const int row = blockIdx.x;
   const int64_t base = (int64_t)row * p.width;
   auto column = [&](int it) { return (it * (int)blockDim.x + (int)threadIdx.x) * VEC; };
@@ -96,7 +96,8 @@ __global__ __launch_bounds__(1024) void sandwich_norm_kernel(const SandwichParam
   };
   auto inv_rms = [&](float ss) { return 1.f / sqrtf(ss / (float)p.width + p.eps); };
   if constexpr (BRANCHES == 2) {
-    const float f0 = 0.5f * inv_rms(block_sum(squares(v[0]), red[0])), f1 = 0.5f * inv_rms(block_sum(squares(v[1]), red[1]));
+    const float2 ss = block_sum2(squares(v[0]), squares(v[1]), red);
+    const float f0 = 0.5f * inv_rms(ss.x), f1 = 0.5f * inv_rms(ss.y);
 #pragma unroll
     for (int it = 0; it < ITEMS; ++it) {
       if (column(it) >= p.width) continue;
@@ -107,7 +108,7 @@ __global__ __launch_bounds__(1024) void sandwich_norm_kernel(const SandwichParam
       for (int j = 0; j < VEC; ++j) v[0][it][j] = v[0][it][j] * f0 * w0[j] + v[1][it][j] * f1 * w1[j];
     }
   }
-  const float f = inv_rms(block_sum(squares(v[0]), red[0]));
+  const float f = inv_rms(block_sum(squares(v[0]), red));
 #pragma unroll
   for (int it = 0; it < ITEMS; ++it) {
     if (column(it) >= p.width) continue;
@@ -117,7 +118,7 @@ __global__ __launch_bounds__(1024) void sandwich_norm_kernel(const SandwichParam
     for (int j = 0; j < VEC; ++j) x[it][j] = fmaf(v[0][it][j] * f, w[j], x[it][j]);
     store_vec<F32, VEC>(p.x + base + column(it), x[it]);
   }
-  const float g = inv_rms(block_sum(squares(x), red[0]));
+  const float g = inv_rms(block_sum(squares(x), red));
 #pragma unroll
   for (int it = 0; it < ITEMS; ++it) {
     if (column(it) >= p.width) continue;
@@ -199,10 +200,10 @@ __global__ __launch_bounds__(1024) void pair_embed_kernel(const PairEmbedParams 
   }
 }
 
-// few rows: as many threads as a row has groups of columns; many: 256, several groups each
+// few or short rows: as many threads as a row has groups of columns; many long ones: 256, several groups each
 static int threads_of(int rows, int groups) {
   int threads = 256;
-  while (threads < 1024 && (rows <= 256 ? threads < groups : threads * 4 < groups)) threads *= 2;
+  while (threads < 1024 && (rows <= 256 || groups <= 512 ? threads < groups : threads * 4 < groups)) threads *= 2;
   return threads;
 }
 

@@ -19,7 +19,8 @@
 // Loads outside the problem (k-steps past K, tiles past N) use an out-of-range buffer offset and
 // return zeros without touching memory, so the loop is branch-free.
 // Epilogues (act): 0 plain (+ bias); 5 squared ReLU; 2 SwiGLU over (gate, up) tile pairs -> [M, N/2]; 3 greedy arg-max
-// over N -> int64 [M] (no logits written); 6 as 2 with the clamped unit (clamped_unit_of) for silu(gate) * up; act = 1 applies SwiGLU while loading X (kept for small shapes).
+// over N -> int64 [M] (no logits written); 6 as 2 with the clamped unit (clamped_unit_of) for silu(gate) * up; act = 1 applies
+// SwiGLU while loading X (kept for small shapes).
 // The same file holds the W8A8 variant (fp8 weights, X quantised while the fragments are built) and,
 // at the end, the 65..256-row kernel that moves X through LDS instead of registers.
 //
@@ -1189,26 +1190,26 @@ static int skinny_gemm(void* y, const void* x, const void* w, const void* bias, 
   hipStream_t s = (hipStream_t)stream;
   const int MT = (M + 15) / 16;
   const bool k8 = steps_per_wave <= 8;
-#define LV_SG(T_, MT_)                                                                              \
-  do {                                                                                              \
-    if (k8)                                                                                         \
-      launch_skinny<T_, MT_, 8>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, \
-                                ksplit, packed != 0, act, s, nullptr, nullptr, nullptr, nullptr, limit);                                       \
-    else                                                                                            \
-      launch_skinny<T_, MT_, 16>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, \
-                                 ksplit, packed != 0, act, s, nullptr, nullptr, nullptr, nullptr, limit);                                      \
+#define LV_SG_GO(T_, MT_, KS_)                                                                                             \
+  launch_skinny<T_, MT_, KS_>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, ksplit, packed != 0, act, s, \
+                              nullptr, nullptr, nullptr, nullptr, limit)
+#define LV_SG(T_, MT_)             \
+  do {                             \
+    if (k8) LV_SG_GO(T_, MT_, 8);  \
+    else LV_SG_GO(T_, MT_, 16);    \
   } while (0)
-#define LV_SG_MT(T_)                           \
-  switch (MT) {                                \
-    case 1: LV_SG(T_, 1); break;               \
-    case 2: LV_SG(T_, 2); break;               \
-    default:                                   \
-      launch_skinny<T_, 4, 8>(y, partial, x, w, bias, M, N, K, ldx, steps_per_wave, ntiles, groups, ksplit, packed != 0, act, s, nullptr, nullptr, nullptr, nullptr, limit); \
-      break;                                   \
+#define LV_SG_MT(T_)               \
+  switch (MT) {                    \
+    case 1: LV_SG(T_, 1); break;   \
+    case 2: LV_SG(T_, 2); break;   \
+    default:                       \
+      LV_SG_GO(T_, 4, 8);          \
+      break;                       \
   }
   if (dtype == LVLLM_BF16) { LV_SG_MT(BF16) } else { LV_SG_MT(F16) }
 #undef LV_SG_MT
 #undef LV_SG
+#undef LV_SG_GO
   LV_LAUNCH_CHECK();
   if (amax_reduce) {
     if (dtype == LVLLM_BF16)

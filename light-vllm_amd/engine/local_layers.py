@@ -107,8 +107,9 @@ class RotaryHeads:
         rot = amd.rotary_cache(q, k, v, self.q_norm, self.k_norm, self.eps, c.heads, c.kv_heads, c.maps, step.positions,
                                self.turns, kc, vc, step.slot_mapping)
         rows = self.out.rows(q)
+        shortest = min(step.query_lens) if step.query_lens else 0  # (no short portions: no launch for them)
         amd.head_attention(rows[:, :self.out.cols], rot, kc, vc, step.block_tables, step.seq_lens, step.query_start_loc, None,
-                           c.vdim, c.scale, self.out_scale, step.max_query_len, step.max_seq_len, c.sees.window, 0,
+                           c.vdim, c.scale, self.out_scale, step.max_query_len, step.max_seq_len, c.sees.window, shortest,
                            c.sees.chunk, c.sees.keep_first, c.softcap, self.sink, c.maps, self.map_weight, self.eps)
         return self.out(rows)
 
