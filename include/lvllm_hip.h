@@ -633,8 +633,8 @@ int lvllm_head_attention(void* out, int64_t out_stride, const void* q, const voi
                          int64_t k_block_stride, int64_t v_block_stride, int max_query_len, int max_seq_len,
                          const lvllm_head_options* options, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 
-/* ---- latent decoders (csrc/latent_attention*.hip, moe*.hip, depth_mix.hip) ----
- * Rows of a step as for the hybrid decoders.  dtype: LVLLM_F32 or LVLLM_BF16.  csrc/latent_attention.h, csrc/moe.h and
+/* ---- latent decoders (csrc/latent_attention*.hip, depth_mix.hip) ----
+ * Rows of a step as for the hybrid decoders.  dtype: LVLLM_F32 or LVLLM_BF16.  csrc/latent_attention.h and
  * csrc/depth_mix.hip give the layouts and what is computed. */
 
 /* x = table[id] * scale (fp32), h = T(x) */
