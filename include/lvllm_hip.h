@@ -648,28 +648,35 @@ int lvllm_norm_add_mix(float* x_out, float* v_out, void* h, const float* x_in, c
                        const float* gain, float eps, const float* streams, int64_t stream_stride, int num_streams,
                        const float* weights, const float* out_gain, float out_eps, int rows, int width, int dtype, void* stream);
 /* cache rows [RMS norm(kv[:kv_rank]) | rotated kv[kv_rank:]] at slot_mapping (slots < 0: none).  turns: rot_dims / 2 numbers,
- * the full turns a pair makes per position */
+ * the full turns a pair makes per position; grow: what a rotated vector's length is multiplied by */
 int lvllm_latent_cache(void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad, int rpad,
                        const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
-                       const int64_t* positions, const double* turns, int rot_dims, const int64_t* slot_mapping, int rows,
-                       int dtype, void* stream);
+                       const int64_t* positions, const double* turns, int rot_dims, float grow, const int64_t* slot_mapping,
+                       int rows, int dtype, void* stream);
+/* the same in one launch with out [rows, q_pad] = RMS norm(q [rows, q_rank]) * q_weight, zeros behind q_rank */
+int lvllm_latent_down(void* out, const void* q, int64_t q_stride, int q_rank, int q_pad, const float* q_weight, void* cache,
+                      int64_t block_stride, int64_t num_blocks, int block_size, int cpad, int rpad, const void* kv,
+                      int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps, const int64_t* positions,
+                      const double* turns, int rot_dims, float grow, const int64_t* slot_mapping, int rows, int dtype,
+                      void* stream);
 /* queries into latent space: out [rows, heads, cpad + rpad] = [uk_t q | rotated | 0]; uk_t [heads, cpad, dpad], zero-padded.
  * kv not null: the same launch writes the rows' cache entries, as lvllm_latent_cache does */
 int lvllm_latent_query(void* out, const void* q, int64_t q_stride, const void* uk_t, int heads, int dim, int dpad, int cpad,
-                       int rpad, int rot_dim, int rot_dims, const int64_t* positions, const double* turns,
+                       int rpad, int rot_dim, int rot_dims, const int64_t* positions, const double* turns, float grow,
                        const int32_t* query_start_loc, int num_seqs, int absorbed_max, void* cache, int64_t block_stride,
                        int64_t num_blocks, int block_size, const void* kv, int64_t kv_stride, int kv_rank, const float* weight,
                        float eps, const int64_t* slot_mapping, int rows, int dtype, void* stream);
 /* attention on the cached rows, for sequences of at most absorbed_max query tokens, and its values out of latent space:
- * out[row, h * vdim + d] = (uv_h sum)[d] * sigmoid(gate[row, h]); uv [heads, vpad, cpad], zero-padded; gate null: none */
+ * out[row, h * vdim + d] = (uv_h sum)[d] * sigmoid(gate[row, h]); uv [heads, vpad, cpad], zero-padded; gate null: none;
+ * sink [heads], fp32 (null: none): one more score of a head's softmax, without a key */
 int64_t lvllm_latent_attention_workspace_bytes(int rows, int num_seqs, int heads, int cpad, int rpad, int block_size,
                                                int window, int absorbed_max, int max_query_len, int max_seq_len, int dtype);
 int lvllm_latent_attention(void* out, int64_t out_stride, const void* q, const void* cache, int64_t block_stride,
                            int64_t num_blocks, int block_size, int cpad, int rpad, const void* uv, int vdim, int vpad,
-                           const void* gate, int64_t gate_stride, const int32_t* block_tables, int max_blocks,
-                           const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows, int heads,
-                           float scale, int window, int absorbed_max, int max_query_len, int max_seq_len, void* workspace,
-                           int64_t workspace_bytes, int dtype, void* stream);
+                           const void* gate, int64_t gate_stride, const float* sink, const int32_t* block_tables,
+                           int max_blocks, const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows,
+                           int heads, float scale, int window, int absorbed_max, int max_query_len, int max_seq_len,
+                           void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 /* long portions: cached rows back to back, their expanded keys / values as pages, their queries */
 int lvllm_latent_gather(void* out, const void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int row_elems,
                         const int32_t* starts, const int32_t* first, const int32_t* seq_lens, const int32_t* block_tables,
@@ -677,13 +684,16 @@ int lvllm_latent_gather(void* out, const void* cache, int64_t block_stride, int6
 int lvllm_latent_expand(void* key_pages, void* value_pages, const void* kv, int64_t kv_stride, const void* rows, int row_elems,
                         int cpad, int n, int heads, int dim, int rot_dim, int vdim, int kpad, int vpad, int dtype, void* stream);
 int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_stride, int heads, int dim, int rot_dim, int kpad,
-                              const int64_t* positions, const double* turns, int rot_dims, int rows, int dtype, void* stream);
+                              const int64_t* positions, const double* turns, int rot_dims, float grow, int rows, int dtype,
+                              void* stream);
 /* ---- mixtures of experts (csrc/moe*.hip, moe.h) ---- */
 enum { LVLLM_MOE_SOFTMAX = 0, LVLLM_MOE_SIGMOID = 1 };  /* weights: softmax over the chosen logits, or each logit's sigmoid */
 enum { LVLLM_MOE_NO_SHARED = 0, LVLLM_MOE_GATED_SHARED = 1, LVLLM_MOE_PLAIN_SHARED = 2 };
-enum { LVLLM_MOE_CLAMPED = 0, LVLLM_MOE_SILU = 1 };     /* activations */
+enum { LVLLM_MOE_CLAMPED = 0, LVLLM_MOE_SILU = 1, LVLLM_MOE_RELU_SQUARED = 2 };  /* activations; the last one has no gate rows */
 typedef struct lvllm_moe_routing {
   int experts, top, scoring, shared;
+  int groups, keep;  /* groups > 1: experts of the `keep` groups with the largest best logits only */
+  float scale;       /* of the chosen experts' weights */
 } lvllm_moe_routing;
 /* the `top` experts of every row and their weights; with a shared one a last assignment, expert number `experts`, weighted by the
  * sigmoid of the last row of w (GATED) or 1 (PLAIN).  bias null: none.  The assignments come grouped by expert: offsets [experts +
@@ -746,6 +756,49 @@ int lvllm_clamped_unit(void* out, const void* in, int64_t rows, int d, float lim
  * rounded to T first.  The envelope of lvllm_skinny_gemm, N a multiple of 32 */
 int lvllm_skinny_gemm_clamped_unit(void* y, const void* x, const void* w, int M, int N, int K, int64_t ldx, int dtype,
                                    int packed, float limit, void* workspace, int64_t workspace_bytes, void* stream);
+
+/* ---- decoders with residual streams and delta-rule layers (csrc/stream_mix.hip, short_conv.h, delta_rule.h) ----
+ * Rows of a step as for the hybrid decoders.  dtype: LVLLM_F32 or LVLLM_BF16. */
+
+/* x_t = sum_s mix[s, t] x_s + out[t] y for all streams at once, h = T(RMS norm(sum_t in[t] x_t) * weight).  Streams are
+ * in_stride (0: all the same rows) and out_stride apart; x_out null: not kept.  y: rows, fp32 slabs (`partials`), or slots of a
+ * mixture with their weights */
+int lvllm_stream_mix(float* x_out, int64_t out_stride, const float* x_in, int64_t in_stride, void* h, const void* y,
+                     const float* partials, int num_partials, const int32_t* slots, const float* slot_weights, int num_slots,
+                     int total_slots, const float* mix, const float* out, const float* in, int streams, const float* weight,
+                     float eps, int rows, int width, int dtype, void* stream);
+/* x = table[id] (every stream's start), h = T(RMS norm(x * sum(in)) * weight) */
+int lvllm_stream_embed(float* x, void* h, const void* table, const int64_t* ids, const float* in, int streams,
+                       const float* weight, float eps, int rows, int vocab, int width, int dtype, void* stream);
+/* y[t, c] = silu(sum_j weight[taps - 1 - j, c] x[t - j, c]); weight [taps, channels], state [slots, taps, channels] (slots
+ * state_stride apart): the input of position p in row p mod taps */
+int lvllm_short_conv(void* out, int64_t out_stride, const void* x, int64_t x_stride, const float* weight, int taps, int channels,
+                     float* state, int64_t state_stride, const int32_t* state_slots, int num_slots,
+                     const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int max_query_len, int dtype,
+                     void* stream);
+/* q [kv_heads, dk] at column 0 of a row, k likewise at k_at, v [heads, dv] at v_at */
+typedef struct lvllm_delta_sizes {
+  int heads, kv_heads, dk, dv, k_at, v_at;
+  float q_scale;
+} lvllm_delta_sizes;
+/* a step of single tokens (sequence s owns row s): convolutions of the rows x, decays, delta rule, norm, gate.  decay_w
+ * [pieces, heads * dk, 16 bytes], gate_w [pieces, heads * dv, 16 bytes]: a row's low-rank weights in pieces of 16 bytes, zeros
+ * behind the rank; u, z their inputs, beta [heads] logits, all x_stride apart */
+int lvllm_delta_step(void* out, int64_t out_stride, const void* x, int64_t x_stride, const void* u, const void* z,
+                     const void* beta, const float* conv_weight, int taps, int channels, float* conv_state, int64_t conv_stride,
+                     const void* decay_w, int decay_rank, const void* gate_w, int gate_rank, const float* decay_scale,
+                     const float* decay_bias, const float* norm_weight, float eps, const lvllm_delta_sizes* sizes, float* state,
+                     int64_t state_stride, const int32_t* state_slots, int num_slots, const int32_t* seq_lens, int num_seqs,
+                     int dtype, void* stream);
+/* portions: y are rows behind lvllm_short_conv, a_t float [decay_rank, heads * dk], gate [rows, heads * dv] before its sigmoid;
+ * u and beta are u_stride apart */
+int64_t lvllm_delta_chunks_workspace_bytes(const lvllm_delta_sizes* sizes, int rows, int num_seqs);
+int lvllm_delta_chunks(void* out, int64_t out_stride, const void* y, int64_t y_stride, const void* u, const void* beta,
+                       int64_t u_stride, const float* a_t, int decay_rank, const float* decay_scale, const float* decay_bias,
+                       const void* gate, int64_t gate_stride, const float* norm_weight, float eps,
+                       const lvllm_delta_sizes* sizes, float* state, int64_t state_stride, const int32_t* state_slots,
+                       int num_slots, const int32_t* query_start_loc, const int32_t* seq_lens, int num_seqs, int rows,
+                       int max_query_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

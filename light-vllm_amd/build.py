@@ -7,6 +7,7 @@
   hybrid  row-wise operators and recurrences of the hybrid decoders
   latent  latent attention, norms on sublayer outputs and depth averages
   local   retention, norms around sublayers, embeddings of token pairs (local decoders)
+  delta   residual streams, short convolutions, the gated delta rule (stream decoders)
   full    the rest of the C-ABI of include/lvllm_hip.h (paged and prefill attention of the rotary decoders, norms, fp8); it
           needs all the others, so a handle on liblvllm_hip.so resolves every symbol of the header
 
@@ -38,6 +39,7 @@ SOURCES = {
     "hybrid": ["token_mix.hip", "recurrent.hip"],
     "latent": ["latent_attention.hip", "latent_attention_mfma.hip", "depth_mix.hip"],
     "local": ["retention.hip", "sandwich_norm.hip"],
+    "delta": ["delta_rule.hip", "short_conv.hip", "stream_mix.hip"],
     "full": ["layernorm.hip", "pos_encoding.hip", "attention.hip", "attention_bf16.hip", "attention_f16.hip",
              "prefill_attention.hip", "fp8_quant.hip"],
 }

@@ -9,6 +9,8 @@
 //   * expanded: the window's latents are gathered, keys and values of all heads made by one library product, and
 //     head_attention runs over them.  Longer portions.
 //
+// sink[h], where given, is one more score of head h's softmax, without a key.
+//
 //   cache  [num_blocks, block_size, cpad + rpad]: c, zeros to cpad, the rotated part, zeros to the row's end
 //   q'     [rows, heads, cpad + rpad], the same row layout
 // Scores, softmax and accumulation are fp32.
@@ -21,6 +23,7 @@ struct LatentAttnParams {
   void* out;               // row r, head h at r * out_stride + h * vdim
   const void *q, *cache;
   const void *uv, *gate;   // [heads, vpad, cpad], zero-padded; gate [rows, heads] (gate_stride apart) or null
+  const float* sink;       // [heads] or null
   const int32_t *block_tables, *seq_lens, *query_start_loc;
   float *part_o, *part_ml;  // shares: [rows, heads, nsplit, cpad] and [rows, heads, nsplit, 2]
   int num_seqs, rows, heads, cpad, rpad, max_blocks, block_size, max_block, nsplit, window, absorbed_max, max_query_len;

@@ -17,7 +17,7 @@ struct LatentCacheParams {
   const double* turns;
   int64_t block_stride, num_slots, kv_stride;
   int block_size, cpad, rpad, kv_rank, rot_dim, rot_dims, rows;
-  float eps;
+  float eps, grow;  // grow: of the rotation
 };
 
 // RMS-normed latent and rotated key part of a row -> its cache slot; one wave, 16 bytes a lane where the sizes allow it
@@ -70,7 +70,7 @@ __device__ __forceinline__ void write_latent_row(const LatentCacheParams& p, int
     float u = i < p.rot_dim ? T::to_float(z[i]) : 0.f, v = i + 1 < p.rot_dim ? T::to_float(z[i + 1]) : 0.f;
     if (i < p.rot_dims) {
       float c, s;
-      rotation_of(pos, p.turns[i >> 1], c, s);
+      rotation_of(pos, p.turns[i >> 1], p.grow, c, s);
       const float t = u * c - v * s;
       v = v * c + u * s;
       u = t;
@@ -84,6 +84,62 @@ template <typename T>
 __global__ __launch_bounds__(256) void latent_cache_kernel(const LatentCacheParams p) {
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row < p.rows) write_latent_row<T>(p, row);
+}
+
+// A layer whose queries come out of a latent of their own: RMS-normed query latents [rows, q_pad] (zeros behind q_rank), and
+// in the same launch the rows' cache entries.  A wave per row; grid.y: 0 the cache, 1 the queries.
+struct QueryLatentParams {
+  void* out;
+  const void* q;
+  const float* weight;
+  int64_t q_stride;
+  int q_rank, q_pad;
+};
+template <typename T>
+__global__ __launch_bounds__(256) void latent_down_kernel(const LatentCacheParams p, const QueryLatentParams z) {
+  using S = typename T::store_t;
+  constexpr int X = 16 / sizeof(S), N = 4;  // pieces of X a lane keeps
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (row >= p.rows) return;
+  if (blockIdx.y == 0) {
+    write_latent_row<T>(p, row);
+    return;
+  }
+  const S* q = (const S*)z.q + row * z.q_stride;
+  S* out = (S*)z.out + (int64_t)row * z.q_pad;
+  float ss = 0.f;
+  if (z.q_rank % X == 0 && z.q_rank <= 64 * X * N && ((uintptr_t)q & 15) == 0) {
+    float v[N][X];
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int d = (i * 64 + lane) * X;
+      if (d >= z.q_rank) continue;
+      const Vec16<T> raw = *reinterpret_cast<const Vec16<T>*>(q + d);
+#pragma unroll
+      for (int j = 0; j < X; ++j) {
+        v[i][j] = T::to_float(raw.v[j]);
+        ss = fmaf(v[i][j], v[i][j], ss);
+      }
+    }
+    const float f = 1.f / sqrtf(wave_sum(ss) / (float)z.q_rank + p.eps);
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int d = (i * 64 + lane) * X;
+      if (d >= z.q_rank) continue;
+      Vec16<T> y;
+#pragma unroll
+      for (int j = 0; j < X; ++j) y.v[j] = T::from_float(v[i][j] * f * z.weight[d + j]);
+      *reinterpret_cast<Vec16<T>*>(out + d) = y;
+    }
+    for (int d = z.q_rank + lane; d < z.q_pad; d += 64) out[d] = T::from_float(0.f);
+    return;
+  }
+  for (int d = lane; d < z.q_rank; d += 64) {
+    const float v = T::to_float(q[d]);
+    ss = fmaf(v, v, ss);
+  }
+  const float f = 1.f / sqrtf(wave_sum(ss) / (float)z.q_rank + p.eps);
+  for (int d = lane; d < z.q_pad; d += 64) out[d] = T::from_float(d < z.q_rank ? T::to_float(q[d]) * f * z.weight[d] : 0.f);
 }
 
 // Rows of a 16-row tile that all belong to one long portion need nothing in latent space.
@@ -101,6 +157,7 @@ struct HeadProjectParams {
   int num_seqs, absorbed_max;
   // the tail of a query row: its rotated part at entry n .. n + tail - 1 of y, from x's entries k .. k + rot_dim - 1
   int tail, rot_dim, rot_dims;
+  float grow;
   const int64_t* positions;
   const double* turns;
   LatentCacheParams cache;  // the rows' own latents, written by the launch that takes their queries to latent space
@@ -123,7 +180,7 @@ __device__ __forceinline__ void project_tail(const HeadProjectParams& p, int row
     float u = e < p.rot_dim ? T::to_float(z[e]) : 0.f, v = e + 1 < p.rot_dim ? T::to_float(z[e + 1]) : 0.f;
     if (e < p.rot_dims) {
       float c, s;
-      rotation_of(p.positions[row], p.turns[e >> 1], c, s);
+      rotation_of(p.positions[row], p.turns[e >> 1], p.grow, c, s);
       const float t = u * c - v * s;
       v = v * c + u * s;
       u = t;
@@ -281,7 +338,12 @@ __global__ __launch_bounds__(256) void latent_attention_simple_kernel(const Late
       sacc[d] = acc;
     }
   }
-  for (int d = threadIdx.x; d < p.cpad; d += 256) out[d] = T::from_float(sacc[d] / l);
+  float f = 1.f / l;
+  if (p.sink != nullptr) {
+    const float sink = p.sink[head], top = fmaxf(m, sink), own = expf(m - top);
+    f = own / (l * own + expf(sink - top));
+  }
+  for (int d = threadIdx.x; d < p.cpad; d += 256) out[d] = T::from_float(sacc[d] * f);
 }
 
 // Rows first[s] .. of every long sequence, back to back (padded to 16 rows a sequence): out[starts[s] + i] = key first[s] + i.
@@ -361,12 +423,13 @@ __global__ __launch_bounds__(256) void latent_rotate_query_kernel(typename T::st
                                                                   const int64_t q_stride, const int heads, const int dim,
                                                                   const int rot_dim, const int kpad,
                                                                   const int64_t* __restrict__ positions,
-                                                                  const double* __restrict__ turns, const int rot_dims) {
+                                                                  const double* __restrict__ turns, const int rot_dims,
+                                                                  const float grow) {
   using S = typename T::store_t;
   struct alignas(E * sizeof(S)) Piece { S v[E]; };
   extern __shared__ float cs[];  // [rot_dims / 2][2]
   const int row = blockIdx.x;
-  for (int i = threadIdx.x; i < rot_dims / 2; i += 256) rotation_of(positions[row], turns[i], cs[2 * i], cs[2 * i + 1]);
+  for (int i = threadIdx.x; i < rot_dims / 2; i += 256) rotation_of(positions[row], turns[i], grow, cs[2 * i], cs[2 * i + 1]);
   __syncthreads();
   const S* x = q + row * q_stride;
   S* y = out + (int64_t)row * heads * kpad;
@@ -410,25 +473,26 @@ using namespace lvllm;
 
 static int cache_params(LatentCacheParams& p, void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad,
                         int rpad, const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
-                        const int64_t* positions, const double* turns, int rot_dims, const int64_t* slot_mapping, int rows) {
+                        const int64_t* positions, const double* turns, int rot_dims, float grow, const int64_t* slot_mapping,
+                        int rows) {
   LV_CHECK(num_blocks * block_size < ((int64_t)1 << 32), "too many slots");
   LV_CHECK(kv_rank > 0 && kv_rank <= cpad && cpad % 8 == 0 && rot_dim >= 0 && rot_dim <= rpad && rpad % 8 == 0 &&
                rot_dims <= rot_dim && rot_dims % 2 == 0, "latent sizes");
   p.cache = cache; p.block_stride = block_stride; p.num_slots = num_blocks * block_size; p.block_size = block_size;
   p.cpad = cpad; p.rpad = rpad; p.kv = kv; p.kv_stride = kv_stride; p.kv_rank = kv_rank; p.rot_dim = rot_dim;
   p.weight = weight; p.eps = eps; p.positions = positions; p.turns = turns; p.rot_dims = rot_dims;
-  p.slot_mapping = slot_mapping; p.rows = rows;
+  p.grow = grow; p.slot_mapping = slot_mapping; p.rows = rows;
   return 0;
 }
 
 extern "C" int lvllm_latent_cache(void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad, int rpad,
                                   const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
-                                  const int64_t* positions, const double* turns, int rot_dims,
+                                  const int64_t* positions, const double* turns, int rot_dims, float grow,
                                   const int64_t* slot_mapping, int rows, int dtype, void* stream) {
   if (rows == 0) return 0;
   LatentCacheParams p{};
   if (int rc = cache_params(p, cache, block_stride, num_blocks, block_size, cpad, rpad, kv, kv_stride, kv_rank, rot_dim, weight,
-                            eps, positions, turns, rot_dims, slot_mapping, rows)) return rc;
+                            eps, positions, turns, rot_dims, grow, slot_mapping, rows)) return rc;
   LV_DISPATCH_F32_BF16(dtype, {
     hipLaunchKernelGGL((latent_cache_kernel<scalar_t>), dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, p);
   });
@@ -436,10 +500,28 @@ extern "C" int lvllm_latent_cache(void* cache, int64_t block_stride, int64_t num
   return 0;
 }
 
+extern "C" int lvllm_latent_down(void* out, const void* q, int64_t q_stride, int q_rank, int q_pad, const float* q_weight,
+                                 void* cache, int64_t block_stride, int64_t num_blocks, int block_size, int cpad, int rpad,
+                                 const void* kv, int64_t kv_stride, int kv_rank, int rot_dim, const float* weight, float eps,
+                                 const int64_t* positions, const double* turns, int rot_dims, float grow,
+                                 const int64_t* slot_mapping, int rows, int dtype, void* stream) {
+  if (rows == 0) return 0;
+  LV_CHECK(q_rank > 0 && q_rank <= q_pad && q_pad % 8 == 0, "query latents of zero or of more than the padded size");
+  LatentCacheParams p{};
+  if (int rc = cache_params(p, cache, block_stride, num_blocks, block_size, cpad, rpad, kv, kv_stride, kv_rank, rot_dim, weight,
+                            eps, positions, turns, rot_dims, grow, slot_mapping, rows)) return rc;
+  const QueryLatentParams z{out, q, q_weight, q_stride, q_rank, q_pad};
+  LV_DISPATCH_F32_BF16(dtype, {
+    hipLaunchKernelGGL((latent_down_kernel<scalar_t>), dim3((rows + 3) / 4, 2), dim3(256), 0, (hipStream_t)stream, p, z);
+  });
+  LV_LAUNCH_CHECK();
+  return 0;
+}
+
 extern "C" int lvllm_latent_query(void* out, const void* q, int64_t q_stride, const void* uk_t, int heads, int dim, int dpad,
                                   int cpad, int rpad, int rot_dim, int rot_dims, const int64_t* positions,
-                                  const double* turns, const int32_t* query_start_loc, int num_seqs, int absorbed_max,
-                                  void* cache, int64_t block_stride, int64_t num_blocks, int block_size, const void* kv,
+                                  const double* turns, float grow, const int32_t* query_start_loc, int num_seqs,
+                                  int absorbed_max, void* cache, int64_t block_stride, int64_t num_blocks, int block_size, const void* kv,
                                   int64_t kv_stride, int kv_rank, const float* weight, float eps,
                                   const int64_t* slot_mapping, int rows, int dtype, void* stream) {
   LV_CHECK(dim > 0 && dim <= dpad && rot_dim <= rpad && rot_dims <= rot_dim && rot_dims % 2 == 0 && cpad % 16 == 0 &&
@@ -449,10 +531,11 @@ extern "C" int lvllm_latent_query(void* out, const void* q, int64_t q_stride, co
   p.x = q; p.x_stride = q_stride; p.x_head = dim + rot_dim; p.k = dim; p.kpad = dpad; p.w = uk_t;
   p.rows = rows; p.heads = heads; p.num_seqs = num_seqs; p.absorbed_max = absorbed_max;
   p.query_start_loc = absorbed_max < rows ? query_start_loc : nullptr;  // (no portion can be longer)
-  p.tail = rpad; p.rot_dim = rot_dim; p.rot_dims = rot_dims; p.positions = positions; p.turns = turns;
+  p.tail = rpad; p.rot_dim = rot_dim; p.rot_dims = rot_dims; p.grow = grow; p.positions = positions;
+  p.turns = turns;
   if (kv != nullptr)
     if (int rc = cache_params(p.cache, cache, block_stride, num_blocks, block_size, cpad, rpad, kv, kv_stride, kv_rank, rot_dim,
-                              weight, eps, positions, turns, rot_dims, slot_mapping, rows)) return rc;
+                              weight, eps, positions, turns, rot_dims, grow, slot_mapping, rows)) return rc;
   return head_project(p, dtype, (hipStream_t)stream);
 }
 
@@ -485,8 +568,8 @@ extern "C" int64_t lvllm_latent_attention_workspace_bytes(int rows, int num_seqs
 
 extern "C" int lvllm_latent_attention(void* out, int64_t out_stride, const void* q, const void* cache, int64_t block_stride,
                                       int64_t num_blocks, int block_size, int cpad, int rpad, const void* uv, int vdim, int vpad,
-                                      const void* gate, int64_t gate_stride, const int32_t* block_tables, int max_blocks,
-                                      const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows,
+                                      const void* gate, int64_t gate_stride, const float* sink,
+                                      const int32_t* block_tables, int max_blocks, const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows,
                                       int heads, float scale, int window, int absorbed_max, int max_query_len,
                                       int max_seq_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
   if (rows == 0 || num_seqs == 0) return 0;
@@ -503,7 +586,7 @@ extern "C" int lvllm_latent_attention(void* out, int64_t out_stride, const void*
   p.query_start_loc = query_start_loc; p.num_seqs = num_seqs; p.rows = rows; p.heads = heads; p.cpad = cpad; p.rpad = rpad;
   p.max_blocks = max_blocks; p.block_size = block_size; p.max_block = (int)(num_blocks - 1); p.nsplit = 1; p.window = window;
   p.absorbed_max = absorbed_max; p.scale = scale; p.block_stride = block_stride; p.uv = uv; p.vdim = vdim; p.vpad = vpad;
-  p.gate = gate; p.gate_stride = gate_stride;
+  p.gate = gate; p.gate_stride = gate_stride; p.sink = sink;
   p.max_query_len = max_query_len < absorbed_max ? max_query_len : absorbed_max;
   hipStream_t s = (hipStream_t)stream;
   if (latent_takes_mfma(cpad, rpad, block_size, dtype)) {
@@ -554,8 +637,8 @@ extern "C" int lvllm_latent_expand(void* key_pages, void* value_pages, const voi
 }
 
 extern "C" int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_stride, int heads, int dim, int rot_dim, int kpad,
-                                         const int64_t* positions, const double* turns, int rot_dims, int rows, int dtype,
-                                         void* stream) {
+                                         const int64_t* positions, const double* turns, int rot_dims, float grow, int rows,
+                                         int dtype, void* stream) {
   if (rows == 0) return 0;
   LV_CHECK(dim + rot_dim <= kpad && rot_dims <= rot_dim && rot_dims % 2 == 0 && rot_dims <= 4096, "query sizes");
   const int e = dtype == LVLLM_F32 ? 4 : 8;
@@ -565,11 +648,11 @@ extern "C" int lvllm_latent_rotate_query(void* out, const void* q, int64_t q_str
     if (vec)
       hipLaunchKernelGGL((latent_rotate_query_kernel<scalar_t, 16 / sizeof(S)>), dim3(rows), dim3(256),
                          (size_t)rot_dims * 4 + 8, (hipStream_t)stream, (S*)out, (const S*)q, q_stride, heads, dim, rot_dim,
-                         kpad, positions, turns, rot_dims);
+                         kpad, positions, turns, rot_dims, grow);
     else
       hipLaunchKernelGGL((latent_rotate_query_kernel<scalar_t, 1>), dim3(rows), dim3(256), (size_t)rot_dims * 4 + 8,
                          (hipStream_t)stream, (S*)out, (const S*)q, q_stride, heads, dim, rot_dim, kpad, positions, turns,
-                         rot_dims);
+                         rot_dims, grow);
   });
   LV_LAUNCH_CHECK();
   return 0;

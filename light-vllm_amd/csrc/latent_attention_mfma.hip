@@ -231,8 +231,11 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const LatentAttnParam
     };
     int d = d0 + lane * 4;
     if (d < d0 + part) load(d, 0);
-    const float m = wave_max(ms);
-    const float e = exp2f(ms - m), l = wave_sum(ls * e);
+    const float sink = p.sink != nullptr ? p.sink[head] * 1.4426950408889634f : -1e30f;
+    const float m = fmaxf(wave_max(ms), sink);
+    const float e = exp2f(ms - m);
+    float l = wave_sum(ls * e);
+    if (p.sink != nullptr) l += exp2f(sink - m);
     const float ws = l > 0.f ? e / l : 0.f;
     for (; d < d0 + part; d += 256) {
       float v[4] = {0.f, 0.f, 0.f, 0.f};

@@ -1,6 +1,7 @@
 // Mixture of experts for gfx950.  A token takes the `top` experts of the largest logits, weighted by the softmax over the chosen
-// ones or each by its own sigmoid, and, as one more assignment, the shared expert, with a gate of its own or the weight 1.  The
-// step's assignments are grouped by expert: slot s of the grouped order belongs to row token[s]; expert e owns slots
+// ones or each by its own sigmoid, times `scale`, and, as one more assignment, the shared expert, with a gate of its own or the
+// weight 1.  With groups (equal runs of neighbouring experts) only the experts of the `keep` groups whose best logits are the
+// largest can be chosen.  The step's assignments are grouped by expert: slot s of the grouped order belongs to row token[s]; expert e owns slots
 // offsets[e] .. offsets[e + 1].
 //
 // Expert weights are two matrices per expert in one buffer:
@@ -9,11 +10,16 @@
 // row-major or, where the matrix-core bodies run, packed as lvllm_pack_weight does.  The activation is
 //   g = min(gate, limit), u = clamp(value, -limit, limit), a = g * sigmoid(1.702 g) * (u + 1)   (LVLLM_MOE_CLAMPED), or
 //   a = gate * sigmoid(gate) * value                                                        (LVLLM_MOE_SILU)
+// or, without gate rows (up [ffp, width]),
+//   a = max(value, 0)^2                                                                     (LVLLM_MOE_RELU_SQUARED)
 // where an assignment's weight may scale the expert's input, that is gate and value, instead of its output (slot_weight).
 #pragma once
 #include "common.h"
 
 namespace lvllm {
+
+// The products of an expert: up with gate rows, up without, down
+enum { kMoeGated = 0, kMoePlain = 1, kMoeDown = 2 };
 
 struct MoeParams {
   void* out;              // up: a [slots, ff_max]; down: y [slots, width]
@@ -26,17 +32,17 @@ struct MoeParams {
   // of all experts but the last one, tiles of all
   const int32_t* tiles;
   const float* slot_weight;  // [slots] or null
-  int act;                // LVLLM_MOE_CLAMPED or LVLLM_MOE_SILU
+  int act;                // LVLLM_MOE_CLAMPED, LVLLM_MOE_SILU or LVLLM_MOE_RELU_SQUARED
   int experts, slots, rows, width, ff_max, max_tiles;
   int ff_first, ff_last;  // largest ffp of all experts but the last, the last one's
 };
 
-// gate and value of slot `slot` of expert e -> its activation
+// gate and value of a slot of expert e -> its activation
 struct MoeActivation {
   float limit;
   bool silu;
   __device__ __forceinline__ MoeActivation(const MoeParams& p, int e) : limit(0.f), silu(p.act == LVLLM_MOE_SILU) {
-    if (!silu) limit = p.limit[e];
+    if (!silu && e >= 0) limit = p.limit[e];
   }
   __device__ __forceinline__ float operator()(float g, float u) const {
     return silu ? g / (1.f + expf(-g)) * u : clamped_unit_of(g, u, limit);
@@ -50,17 +56,37 @@ __device__ __forceinline__ float slot_weight_of(const MoeParams& p, int slot) {
 struct MoeRouting {
   int experts, top, scoring;
   bool shared, gated;
+  int groups, keep;  // groups <= 1: none
+  float scale;
   __host__ __device__ __forceinline__ int logits() const { return experts + gated; }
   __host__ __device__ __forceinline__ int all() const { return experts + shared; }
   __host__ __device__ __forceinline__ int per_row() const { return top + shared; }
 };
 
-constexpr int kMaxExperts = 1024;
+constexpr int kMaxExperts = 1024, kMaxGroups = 64;
+
+// Logits of groups that are not among the `keep` best (ties: the earlier group) become -INFINITY; by one wave, a lane per group.
+__device__ __forceinline__ void close_groups(float* z, const MoeRouting& r) {
+  const int lane = threadIdx.x & 63, size = r.experts / r.groups;
+  float best = -INFINITY;
+  if (lane < r.groups)
+    for (int e = lane * size; e < (lane + 1) * size; ++e) best = fmaxf(best, z[e]);
+  int place = 0;
+  for (int j = 0; j < r.groups; ++j) {
+    const float o = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, best), j));
+    place += o > best || (o == best && j < lane);
+  }
+  const uint64_t open = __ballot(lane < r.groups && place < r.keep);
+  for (int e = lane; e < r.experts; e += 64)
+    if (!(open >> (e / size) & 1)) z[e] = -INFINITY;
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (the wave's own next reads see it)
+}
 
 // The `top` largest of z[0 .. experts) (LDS; ties: the smaller index) by one wave, their weights, and the shared expert.  NaNs
 // come last; any z gives distinct indices in range.
-__device__ __forceinline__ void choose_experts(const float* z, const MoeRouting& r, int32_t* ids, float* weights) {
+__device__ __forceinline__ void choose_experts(float* z, const MoeRouting& r, int32_t* ids, float* weights) {
   const int experts = r.experts, top = r.top;
+  if (r.groups > 1) close_groups(z, r);
   const bool sigmoid = r.scoring == LVLLM_MOE_SIGMOID;
   const int lane = threadIdx.x & 63;
   auto value = [&](int e) {
@@ -83,7 +109,7 @@ __device__ __forceinline__ void choose_experts(const float* z, const MoeRouting&
     const float sum = sigmoid ? 1.f : wave_sum(w);
     if (chosen) {
       ids[place] = lane;
-      weights[place] = w / sum;
+      weights[place] = w / sum * r.scale;
     }
   } else {  // one after the other; `taken`: which of this lane's logits are gone
     uint32_t taken = 0;
@@ -110,7 +136,7 @@ __device__ __forceinline__ void choose_experts(const float* z, const MoeRouting&
           sum += w;
         } else if (lane == 0) {
           ids[k] = at;
-          weights[k] = sigmoid ? w : w / sum;
+          weights[k] = (sigmoid ? w : w / sum) * r.scale;
         }
       }
     }
@@ -223,7 +249,7 @@ constexpr int kMoeTile = 128, kMoeSmallTile = 16, kMoeFewRows = 64;
 inline int moe_tile(bool packed, int rows) { return packed && rows > kMoeFewRows ? kMoeTile : kMoeSmallTile; }
 
 bool moe_takes_mfma(int width, int dtype);
-int launch_moe_mfma(const MoeParams& p, bool up, hipStream_t s);
+int launch_moe_mfma(const MoeParams& p, int product, hipStream_t s);
 // `counted`: the rows have counted their assignments
 int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, int shared, bool counted, const MoeGroups& groups,
                      hipStream_t s);

@@ -70,10 +70,11 @@ int launch_moe_group(const int32_t* ids, int total, int per_row, int experts, in
 }
 
 // 16 slots x 16 outputs a workgroup, row-major weights, 32 of K a turn through LDS.
-template <typename T, bool UP>
+template <typename T, int PRODUCT>
 __global__ __launch_bounds__(256) void moe_simple_kernel(const MoeParams p) {
   using S = typename T::store_t;
-  __shared__ float sx[16][33], sg[16][33], su[UP ? 16 : 1][33];
+  constexpr bool UP = PRODUCT != kMoeDown, GATED = PRODUCT == kMoeGated;
+  __shared__ float sx[16][33], sg[16][33], su[GATED ? 16 : 1][33];
   const int e = p.tiles[4 * blockIdx.y];
   if (e < 0 || e >= p.experts) return;
   const int s0 = p.tiles[4 * blockIdx.y + 1], s1 = min(min(p.offsets[e + 1], s0 + 16), p.slots);
@@ -92,22 +93,24 @@ __global__ __launch_bounds__(256) void moe_simple_kernel(const MoeParams p) {
         v = T::to_float(((const S*)p.x)[row * (UP ? p.width : p.ff_max) + k]);
       }
       sx[r][i & 31] = v;
-      const int n = UP ? 2 * n0 + r : n0 + r;  // UP: 16 gate rows, then 16 value rows
+      const int n = GATED ? 2 * n0 + r : n0 + r;  // GATED: 16 gate rows, then 16 value rows
       sg[r][i & 31] = k < K && (UP || n < p.width) ? T::to_float(w[(int64_t)n * K + k]) : 0.f;
-      if constexpr (UP) su[r][i & 31] = k < K ? T::to_float(w[(int64_t)(n + 16) * K + k]) : 0.f;
+      if constexpr (GATED) su[r][i & 31] = k < K ? T::to_float(w[(int64_t)(n + 16) * K + k]) : 0.f;
     }
     __syncthreads();
 #pragma unroll 8
     for (int k = 0; k < 32; ++k) {
       accg = fmaf(sx[a][k], sg[b][k], accg);
-      if constexpr (UP) accu = fmaf(sx[a][k], su[b][k], accu);
+      if constexpr (GATED) accu = fmaf(sx[a][k], su[b][k], accu);
     }
   }
   const int s = s0 + a, n = n0 + b;
   if (s >= s1) return;
-  if constexpr (UP) {
+  if constexpr (GATED) {
     const float f = slot_weight_of(p, s);
     ((S*)p.out)[(int64_t)s * p.ff_max + n] = T::from_float(MoeActivation(p, e)(accg * f, accu * f));
+  } else if constexpr (UP) {
+    ((S*)p.out)[(int64_t)s * p.ff_max + n] = T::from_float(relu_squared_of(accg * slot_weight_of(p, s)));
   } else if (n < p.width) ((S*)p.out)[(int64_t)s * p.width + n] = T::from_float(accg);
 }
 
@@ -118,7 +121,8 @@ using namespace lvllm;
 extern "C" int lvllm_moe_tile(int packed, int rows) { return moe_tile(packed != 0, rows); }
 
 static MoeRouting routing_of(const lvllm_moe_routing& r) {
-  return MoeRouting{r.experts, r.top, r.scoring, r.shared != LVLLM_MOE_NO_SHARED, r.shared == LVLLM_MOE_GATED_SHARED};
+  return MoeRouting{r.experts, r.top, r.scoring, r.shared != LVLLM_MOE_NO_SHARED, r.shared == LVLLM_MOE_GATED_SHARED,
+                    r.groups, r.keep, r.scale};
 }
 
 extern "C" int64_t lvllm_moe_route_workspace_bytes(const lvllm_moe_routing* routing, int rows, int width, int packed) {
@@ -132,6 +136,9 @@ extern "C" int lvllm_moe_route(int32_t* ids, float* weights, int32_t* offsets, i
   if (rows == 0) return 0;
   const MoeRouting r = routing_of(*routing);
   LV_CHECK(r.experts > 0 && r.experts < kMaxExperts && r.top > 0 && r.top <= r.experts, "experts: fewer than 1024, top of them");
+  LV_CHECK(r.groups <= 1 || (r.groups <= kMaxGroups && r.experts % r.groups == 0 && r.keep > 0 && r.keep <= r.groups &&
+                             r.keep * (r.experts / r.groups) >= r.top),
+           "groups: at most 64 of equal size, as many kept as the chosen experts need");
   LV_CHECK(r.scoring == LVLLM_MOE_SOFTMAX || r.scoring == LVLLM_MOE_SIGMOID, "unknown scores");
   LV_CHECK((int64_t)rows * (r.top + 1) < ((int64_t)1 << 31) && max_tiles > 0, "too many assignments");
   LV_CHECK(workspace_bytes >= lvllm_moe_route_workspace_bytes(routing, rows, width, packed), "workspace too small");
@@ -162,20 +169,22 @@ extern "C" int lvllm_moe_experts(void* out, const void* x, const void* w, const 
                                  void* stream) {
   if (slots == 0) return 0;
   LV_CHECK(experts > 0 && ff_max > 0 && ff_max % 32 == 0 && width > 0 && max_tiles > 0 && max_tiles <= 65535, "sizes of the experts");
-  LV_CHECK(!up || act == LVLLM_MOE_SILU || (act == LVLLM_MOE_CLAMPED && limit != nullptr), "unknown activation");
+  LV_CHECK(!up || act == LVLLM_MOE_SILU || act == LVLLM_MOE_RELU_SQUARED || (act == LVLLM_MOE_CLAMPED && limit != nullptr), "unknown activation");
   MoeParams p{};
   p.out = out; p.x = x; p.w = w; p.w_offset = w_offset; p.ff = ff; p.limit = limit; p.offsets = offsets; p.token = token;
   p.tiles = tiles; p.experts = experts; p.slots = slots; p.rows = rows; p.width = width; p.ff_max = ff_max;
   p.max_tiles = max_tiles; p.ff_first = ff_first; p.ff_last = ff_last; p.slot_weight = slot_weight; p.act = act;
   hipStream_t s = (hipStream_t)stream;
+  const int product = !up ? kMoeDown : act == LVLLM_MOE_RELU_SQUARED ? kMoePlain : kMoeGated;
   if (packed) {
     LV_CHECK(moe_takes_mfma(width, dtype), "packed experts: bf16, a width that is a multiple of 32");
-    return launch_moe_mfma(p, up != 0, s);
+    return launch_moe_mfma(p, product, s);
   }
   const dim3 grid(((up ? ff_max : width) + 15) / 16, max_tiles);
   LV_DISPATCH_F32_BF16(dtype, {
-    if (up) hipLaunchKernelGGL((moe_simple_kernel<scalar_t, true>), grid, dim3(256), 0, s, p);
-    else hipLaunchKernelGGL((moe_simple_kernel<scalar_t, false>), grid, dim3(256), 0, s, p);
+    if (product == kMoeGated) hipLaunchKernelGGL((moe_simple_kernel<scalar_t, kMoeGated>), grid, dim3(256), 0, s, p);
+    else if (product == kMoePlain) hipLaunchKernelGGL((moe_simple_kernel<scalar_t, kMoePlain>), grid, dim3(256), 0, s, p);
+    else hipLaunchKernelGGL((moe_simple_kernel<scalar_t, kMoeDown>), grid, dim3(256), 0, s, p);
   });
   LV_LAUNCH_CHECK();
   return 0;

@@ -26,8 +26,9 @@ constexpr int kStreamBatch = 8, kStreamChunk = 64;  // k-steps per batch, per LD
 
 // grid (shares of the outputs, tiles of 16 slots); a wave computes W tiles 2 u and 2 u + 1, or (KS > 1, when few
 // experts have work) a KS-th of their k-steps, 64 / KS of every LDS chunk
-template <bool UP, int KS>
+template <int PRODUCT, int KS>
 __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
+  constexpr bool UP = PRODUCT != kMoeDown, GATED = PRODUCT == kMoeGated;
   extern __shared__ __attribute__((aligned(16))) char sx[];  // [k-steps of a chunk][4][16][8]
   __shared__ e_f32x4_t red[KS > 1 ? 4 : 1][2][64];
   const int e = p.tiles[4 * blockIdx.y];
@@ -38,7 +39,7 @@ __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
   const int ff = p.ff[e], K = UP ? p.width : ff, steps = K >> 5;
-  const int units = UP ? ff >> 4 : p.width >> 5;
+  const int units = GATED ? ff >> 4 : (UP ? ff : p.width) >> 5;
   constexpr int U = 4 / KS, P = kStreamChunk / KS;  // units of a workgroup; this wave's k-steps of a chunk
   if ((int)blockIdx.x * U >= units) return;
   const int u = min((int)blockIdx.x * U + wave / KS, units - 1), kq = wave % KS;  // (a wave too many repeats the last unit)
@@ -112,9 +113,9 @@ __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
   const int slot = s0 + c;
   if (slot >= s1) return;
   float v[4];
-  if constexpr (UP) {
+  const float f = UP ? slot_weight_of(p, slot) : 1.f;
+  if constexpr (GATED) {
     const MoeActivation act(p, e);
-    const float f = slot_weight_of(p, slot);
 #pragma unroll
     for (int r = 0; r < 4; ++r) v[r] = act(acc[0][r] * f, acc[1][r] * f);
     store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.ff_max + 16 * u + 4 * g, v);
@@ -122,8 +123,8 @@ __global__ __launch_bounds__(256, 2) void moe_stream_kernel(const MoeParams p) {
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) v[r] = acc[i][r];
-      store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.width + 32 * u + 16 * i + 4 * g, v);
+      for (int r = 0; r < 4; ++r) v[r] = UP ? relu_squared_of(acc[i][r] * f) : acc[i][r];
+      store4<BF16>((uint16_t*)p.out + (int64_t)slot * (UP ? p.ff_max : p.width) + 32 * u + 16 * i + 4 * g, v);
     }
   }
 }
@@ -136,8 +137,9 @@ __device__ __forceinline__ void to_lds(const uint16_t* src, char* dst) {  // 16 
                                    (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
 }
 
-template <bool UP>
+template <int PRODUCT>
 __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, const int blocks_first, const int blocks_last) {
+  constexpr bool UP = PRODUCT != kMoeDown, GATED = PRODUCT == kMoeGated;
   __shared__ __attribute__((aligned(16))) char ring[kStages][kStageBytes];
   // the tiles of all experts but the last one, then the last one's (the shared expert may be larger): an eighth of each to
   // every XCD
@@ -168,7 +170,7 @@ __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, con
   tile = tile0 + group * kSide + unit - block * side;
   const int s0 = p.tiles[4 * tile + 1], s1 = min(min(p.offsets[e + 1], s0 + kMoeTile), p.slots);
   const int ff = p.ff[e], steps = (UP ? p.width : ff) >> 5;
-  const int ntiles = UP ? ff >> 3 : p.width >> 4;  // of 16 W rows
+  const int ntiles = GATED ? ff >> 3 : (UP ? ff : p.width) >> 4;  // of 16 W rows
   if (block * kTileW >= ntiles || s0 >= s1) return;
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -229,24 +231,24 @@ __global__ __launch_bounds__(256, 2) void moe_tile_kernel(const MoeParams p, con
   if (k + 1 < steps) step(k + 1, 1);
   if (k + 2 < steps) step(k + 2, 2);
   __builtin_amdgcn_s_waitcnt(0 | (7 << 4) | (15 << 8));  // (no copy to LDS outlives the workgroup)
-  const MoeActivation act(p, UP ? e : 0);
+  [[maybe_unused]] const MoeActivation act(p, GATED ? e : -1);
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
     const int slot = s0 + 16 * m + c;
     if (slot >= s1) continue;
     const float f = UP ? slot_weight_of(p, slot) : 1.f;
 #pragma unroll
-    for (int n = 0; n < 4; n += UP ? 2 : 1) {
+    for (int n = 0; n < 4; n += GATED ? 2 : 1) {
       if (nt0 + n >= ntiles) continue;
       float v[4];
-      if constexpr (UP) {
+      if constexpr (GATED) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) v[r] = act(acc[n][m][r] * f, acc[n + 1][m][r] * f);
         store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.ff_max + (nt0 + n) * 8 + 4 * g, v);
       } else {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] = acc[n][m][r];
-        store4<BF16>((uint16_t*)p.out + (int64_t)slot * p.width + (nt0 + n) * 16 + 4 * g, v);
+        for (int r = 0; r < 4; ++r) v[r] = UP ? relu_squared_of(acc[n][m][r] * f) : acc[n][m][r];
+        store4<BF16>((uint16_t*)p.out + (int64_t)slot * (UP ? p.ff_max : p.width) + (nt0 + n) * 16 + 4 * g, v);
       }
     }
   }
@@ -399,31 +401,33 @@ int launch_moe_route_mfma(int32_t* ids, float* weights, const void* h, const voi
 
 bool moe_takes_mfma(int width, int dtype) { return dtype == LVLLM_BF16 && width % 32 == 0; }
 
-template <bool UP>
+template <int PRODUCT>
 static void go(const MoeParams& p, hipStream_t s) {
+  constexpr bool UP = PRODUCT != kMoeDown, GATED = PRODUCT == kMoeGated;
   if (p.rows <= kMoeFewRows) {
-    const int steps = (UP ? p.width : p.ff_max) / 32, units = UP ? p.ff_max / 16 : p.width / 32;  // of the largest expert
+    const int steps = (UP ? p.width : p.ff_max) / 32, units = GATED ? p.ff_max / 16 : (UP ? p.ff_max : p.width) / 32;  // of the largest expert
     const int smem = (steps < kStreamChunk ? steps : kStreamChunk) * 1024;
     // workgroups with work, were every wave to take whole units
-    const int64_t wgs = (int64_t)p.max_tiles * (((UP ? p.ff_first / 16 : units) + 3) / 4);
+    const int64_t wgs = (int64_t)p.max_tiles * (((GATED ? p.ff_first / 16 : UP ? p.ff_first / 32 : units) + 3) / 4);
     const unsigned t = p.max_tiles;
-    if (wgs <= 256) hipLaunchKernelGGL((moe_stream_kernel<UP, 4>), dim3(units, t), dim3(256), smem, s, p);
-    else if (wgs <= 512) hipLaunchKernelGGL((moe_stream_kernel<UP, 2>), dim3((units + 1) / 2, t), dim3(256), smem, s, p);
-    else hipLaunchKernelGGL((moe_stream_kernel<UP, 1>), dim3((units + 3) / 4, t), dim3(256), smem, s, p);
+    if (wgs <= 256) hipLaunchKernelGGL((moe_stream_kernel<PRODUCT, 4>), dim3(units, t), dim3(256), smem, s, p);
+    else if (wgs <= 512) hipLaunchKernelGGL((moe_stream_kernel<PRODUCT, 2>), dim3((units + 1) / 2, t), dim3(256), smem, s, p);
+    else hipLaunchKernelGGL((moe_stream_kernel<PRODUCT, 1>), dim3((units + 3) / 4, t), dim3(256), smem, s, p);
   } else {
-    auto blocks = [&](int ff) { return ((UP ? ff / 8 : p.width / 16) + kTileW - 1) / kTileW; };
+    auto blocks = [&](int ff) { return ((GATED ? ff / 8 : (UP ? ff : p.width) / 16) + kTileW - 1) / kTileW; };
     const int first = blocks(p.ff_first), last = blocks(p.ff_last);
     const int64_t last_tiles = (p.rows + kMoeTile - 1) / kMoeTile;  // a token takes an expert once
     const int64_t wgs = 8 * (((int64_t)p.max_tiles * first + 7) / 8 + (last_tiles * last + 7) / 8);
-    hipLaunchKernelGGL((moe_tile_kernel<UP>), dim3((unsigned)wgs), dim3(256), 0, s, p, first, last);
+    hipLaunchKernelGGL((moe_tile_kernel<PRODUCT>), dim3((unsigned)wgs), dim3(256), 0, s, p, first, last);
   }
 }
 
-int launch_moe_mfma(const MoeParams& p, bool up, hipStream_t s) {
+int launch_moe_mfma(const MoeParams& p, int product, hipStream_t s) {
   LV_CHECK(p.experts <= 65535 && p.ff_first > 0 && p.ff_last > 0 && p.ff_first <= p.ff_max && p.ff_last <= p.ff_max,
            "sizes of the experts");
-  if (up) go<true>(p, s);
-  else go<false>(p, s);
+  if (product == kMoeGated) go<kMoeGated>(p, s);
+  else if (product == kMoePlain) go<kMoePlain>(p, s);
+  else go<kMoeDown>(p, s);
   LV_LAUNCH_CHECK();
   return 0;
 }

@@ -8,7 +8,7 @@
 //
 //     z = A f(u_t) + bias,   ln w = logsigmoid(z) / tau   (f = identity)   or   ln w = -exp(z)   (f = tanh)
 //
-// or one fixed decay per head (FIXED), and then rotary positions on q and k, in fp32, where asked for.
+// (log_decay.h), or one fixed decay per head (FIXED), and then rotary positions on q and k, in fp32, where asked for.
 //
 // Two bodies:
 //   * steps of single tokens (decode): ONE launch per mixer -- decay, state update, read-out, per-head RMS norm and gate --
@@ -27,35 +27,14 @@
 // the read-out.  Rows are the new tokens of `num_seqs` sequences back to back (query_start_loc); a sequence whose tokens
 // are all in this step (seq_lens == its rows) starts from a zero state, every other one from its slot.
 #pragma once
+#include "head_norm_gate.h"
+#include "log_decay.h"
 #include "rotation.h"
 #include "row_ops.h"
 
 namespace lvllm {
 
-enum { kDecayLogSigmoid = 0, kDecayNegExp = 1 };
-
-// e^x, |x| up to a few hundred: 2^(x log2 e) with the product's rounding error put back
-__device__ __forceinline__ float exp_of(float x) {
-  const float t = x * 1.44269502e+0f;
-  const float lo = fmaf(x, 1.44269502e+0f, -t) + x * 1.92596299e-8f;
-  const float r = __builtin_amdgcn_exp2f(t);
-  return fmaf(r, lo * 0.693147182f, r);
-}
-
-__device__ __forceinline__ float log_decay_of(float z, int kind, float inv_tau) {
-  if (kind == kDecayNegExp) return -exp_of(fminf(z, 9.f));  // (exp(-exp(9)) is 0: a finite logarithm keeps sums finite)
-  return (fminf(z, 0.f) - log1pf(exp_of(-fabsf(z)))) * inv_tau;
-}
-
-typedef float r_f32x4_t __attribute__((ext_vector_type(4)));
-__device__ __forceinline__ r_f32x4_t mfma_f32(float a, float b, r_f32x4_t c) {
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
-}
-
 // ---- chunks of 16 tokens ------------------------------------------------------------------------------------------
-constexpr int kChunk = 16;
-constexpr float kMaxHalfDecay = 60.f;  // ln of the largest factor measured from the middle of a chunk
-
 struct MixParams {
   const void *q, *k, *v;  // row r, head h at r * stride + h * dk (dv)
   int64_t q_stride, k_stride, v_stride;
@@ -96,33 +75,6 @@ struct MixParams {
 __device__ __forceinline__ int seg_slot_base(const MixParams& p, int s) {
   return p.query_start_loc[s] / (kChunk * p.seg_chunks) + s;
 }
-
-// Sums of ln w over ranges of a chunk's tokens, for the lane of channel c and tokens 4g .. 4g + 3 (l).  Every range is summed
-// by itself: a difference of two running sums would lose the small decays behind a large one.
-struct ChunkSums {
-  float h1, h2;              // the chunk's two halves
-  float read[4], left[4];    // chunk's start -> what token t reads; token t -> end
-  float half_q[4], half_k[4];  // the middle of the chunk -> what token t reads; token t -> the middle
-  __device__ __forceinline__ ChunkSums(const float (&l)[4], int g, int c, bool has_bonus) {
-    const float upto[4] = {l[0], l[0] + l[1], (l[0] + l[1]) + l[2], (l[0] + l[1]) + (l[2] + l[3])};
-    const float after[4] = {l[1] + (l[2] + l[3]), l[2] + l[3], l[3], 0.f};
-    const float g0 = __shfl(upto[3], c), g1 = __shfl(upto[3], 16 + c), g2 = __shfl(upto[3], 32 + c), g3 = __shfl(upto[3], 48 + c);
-    const float before_g = g == 0 ? 0.f : g == 1 ? g0 : g == 2 ? g0 + g1 : g0 + g1 + g2;
-    const float after_g = g == 3 ? 0.f : g == 2 ? g3 : g == 1 ? g2 + g3 : g1 + (g2 + g3);
-    const float in_half = g == 0 ? g1 : g == 3 ? g2 : 0.f;  // the group of this half between this one and the middle
-    h1 = g0 + g1;
-    h2 = g2 + g3;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float upto_read = has_bonus ? (r == 0 ? 0.f : upto[r == 0 ? 0 : r - 1]) : upto[r];
-      const float from_read = has_bonus ? after[r] + l[r] : after[r];
-      read[r] = before_g + upto_read;
-      left[r] = after[r] + after_g;
-      half_q[r] = g < 2 ? -(from_read + in_half) : in_half + upto_read;
-      half_k[r] = g < 2 ? after[r] + in_half : -(in_half + upto[r]);
-    }
-  }
-};
 
 __host__ __device__ constexpr int mix_smem_floats(int NT, int NV) {
   return 4 * kChunk * (64 * NT + 4) + 4 * 256 + 4 * kChunk + 5 * kChunk * (16 * NV + 4) + 4 * NT;
@@ -767,64 +719,6 @@ static void launch_mix_sized(const MixParams& p, hipStream_t s) {
     case 66: launch_mix<T, QT, 4, 2, FIXED>(p, s); break;
     default: launch_mix<T, QT, 4, 4, FIXED>(p, s); break;
   }
-}
-
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-
-// Per head: o / rms(o) * weight * silu(gate) * scale -> T.  o is the fp32 read-out of a recurrent state.
-// weight_head_stride: 0 (one weight of size vdim for all heads) or vdim; weight null: none.  L lanes per (row, head).
-template <typename T, int L, int VEC>
-static __global__ __launch_bounds__(256) void head_norm_gate_kernel(
-    typename T::store_t* __restrict__ out, const int64_t out_stride, const float* __restrict__ o,
-    const typename T::store_t* __restrict__ gate, const int64_t gate_stride, const float* __restrict__ weight,
-    const int weight_head_stride, const float eps, const float scale, const int rows, const int heads, const int vdim) {
-  const int lane = threadIdx.x % L;
-  const int64_t item = (int64_t)blockIdx.x * (256 / L) + threadIdx.x / L;
-  if (item >= (int64_t)rows * heads) return;
-  const int64_t row = item / heads;
-  const int h = (int)(item - row * heads);
-  const float* src = o + item * vdim;
-  float f[VEC], z[VEC];
-  float ss = 0.f;
-  for (int d = lane * VEC; d < vdim; d += L * VEC) {
-    load_vec<F32, VEC>(src + d, f);
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) ss += f[j] * f[j];
-  }
-  const float r = 1.f / sqrtf(group_sum<L>(ss) / vdim + eps);
-  for (int d = lane * VEC; d < vdim; d += L * VEC) {
-    load_vec<F32, VEC>(src + d, f);
-    load_vec<T, VEC>(gate + row * gate_stride + h * vdim + d, z);
-#pragma unroll
-    for (int j = 0; j < VEC; ++j)
-      f[j] = f[j] * r * (weight != nullptr ? weight[h * weight_head_stride + d + j] : 1.f) * (z[j] * sigmoid_f(z[j])) * scale;
-    store_vec<T, VEC>(out + row * out_stride + h * vdim + d, f);
-  }
-}
-
-static int launch_head_norm_gate(void* out, int64_t out_stride, const float* o, const void* gate, int64_t gate_stride,
-                                 const float* weight, int weight_head_stride, float eps, float scale, int rows,
-                                 int heads, int vdim, int dtype, hipStream_t stream) {
-  if (rows == 0) return 0;
-  const int64_t items = (int64_t)rows * heads;
-  const int esize = dtype == LVLLM_F32 ? 4 : 2;
-  const bool vec = ((vdim | out_stride | gate_stride) & 3) == 0 && ((uintptr_t)o & 15) == 0 &&
-                   (((uintptr_t)out | (uintptr_t)gate) & (4 * esize - 1)) == 0;
-  const int lanes = lanes_for(vdim, vec ? 4 : 1);
-  const dim3 grid((unsigned)((items * lanes + 255) / 256));
-  LV_DISPATCH_DTYPE(dtype, {
-    using S = scalar_t::store_t;
-    LV_LANES(lanes, {
-      if (vec)
-        hipLaunchKernelGGL((head_norm_gate_kernel<scalar_t, kL, 4>), grid, dim3(256), 0, stream, (S*)out,
-                           out_stride, o, (const S*)gate, gate_stride, weight, weight_head_stride, eps, scale, rows, heads, vdim);
-      else
-        hipLaunchKernelGGL((head_norm_gate_kernel<scalar_t, kL, 1>), grid, dim3(256), 0, stream, (S*)out,
-                           out_stride, o, (const S*)gate, gate_stride, weight, weight_head_stride, eps, scale, rows, heads, vdim);
-    })
-  });
-  LV_LAUNCH_CHECK();
-  return 0;
 }
 
 // every sequence brings one token: sequence s owns row s

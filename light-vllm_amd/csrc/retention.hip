@@ -94,6 +94,6 @@ extern "C" int lvllm_retention(void* out, int64_t out_stride, const void* q, con
   else launch_mix_sized<F32, F32, true>(p, s);
   LV_LAUNCH_CHECK();
   if (p.o == nullptr) return 0;
-  return launch_head_norm_gate(out, out_stride, p.o, gate, gate_stride, norm_weight, norm_head_stride, eps, out_scale, rows,
+  return launch_head_norm_gate<true>(out, out_stride, p.o, gate, gate_stride, norm_weight, norm_head_stride, eps, out_scale, rows,
                                heads, dv, dtype, s);
 }

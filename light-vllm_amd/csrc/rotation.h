@@ -9,5 +9,11 @@ __device__ __forceinline__ void rotation_of(int64_t position, double turns, floa
   const double t = (double)position * turns;
   sincospif((float)(2.0 * (t - rint(t))), &s, &c);
 }
+// ... of a rotation that also makes vectors `grow` times as long
+__device__ __forceinline__ void rotation_of(int64_t position, double turns, float grow, float& c, float& s) {
+  rotation_of(position, turns, c, s);
+  c *= grow;
+  s *= grow;
+}
 
 }  // namespace lvllm

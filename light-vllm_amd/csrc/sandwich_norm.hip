@@ -200,26 +200,6 @@ __global__ __launch_bounds__(1024) void pair_embed_kernel(const PairEmbedParams 
   }
 }
 
-// few or short rows: as many threads as a row has groups of columns; many long ones: 256, several groups each
-static int threads_of(int rows, int groups) {
-  int threads = 256;
-  while (threads < 1024 && (rows <= 256 || groups <= 512 ? threads < groups : threads * 4 < groups)) threads *= 2;
-  return threads;
-}
-
-// vectors of 4 up to rows of 16384, single columns up to 4096
-#define LV_ROWS(WIDTH_, THREADS_, GO_)                                       \
-  if ((WIDTH_) % 4 == 0) {                                                   \
-    const int items = ((WIDTH_) / 4 + (THREADS_) - 1) / (THREADS_);          \
-    LV_CHECK(items <= 4, "rows of at most 16384");                           \
-    if (items <= 1) { GO_(4, 1); }                                           \
-    else if (items <= 2) { GO_(4, 2); }                                      \
-    else { GO_(4, 4); }                                                      \
-  } else {                                                                   \
-    LV_CHECK((WIDTH_) <= 4 * (THREADS_), "rows that are no multiple of 4: at most 4096"); \
-    GO_(1, 4);                                                               \
-  }
-
 }  // namespace lvllm
 
 using namespace lvllm;

@@ -253,6 +253,17 @@ torch::Tensor skinny_linear_packed_clamped_unit(const torch::Tensor& x, const to
   return y;
 }
 
+// silu(gate) * up of [rows, gate | up]
+torch::Tensor silu_unit(const torch::Tensor& x) {
+  const char* op = "silu_unit";
+  LV_CHECK_DEVICE(x);
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.size(1) % 2 == 0, op, ": contiguous [rows, gate | up]");
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(x));
+  auto y = torch::empty({x.size(0), x.size(1) / 2}, x.options());
+  check(lvllm_silu_and_mul(y.data_ptr(), x.data_ptr(), x.size(0), (int)y.size(1), dtype_code(x, op), current_stream(x)));
+  return y;
+}
+
 torch::Tensor clamped_unit(const torch::Tensor& x, double limit) {
   const char* op = "clamped_unit";
   LV_CHECK_DEVICE(x);
@@ -657,6 +668,8 @@ TORCH_LIBRARY_FRAGMENT(_C_amd, amd) {
   amd.impl("skinny_linear_packed_clamped_unit", torch::kCUDA, &skinny_linear_packed_clamped_unit);
   amd.def("clamped_unit(Tensor x, float limit) -> Tensor");
   amd.impl("clamped_unit", torch::kCUDA, &clamped_unit);
+  amd.def("silu_unit(Tensor x) -> Tensor");
+  amd.impl("silu_unit", torch::kCUDA, &silu_unit);
   amd.def("skinny_linear_packed_relu_squared(Tensor x, Tensor w_packed, int N, int K) -> Tensor");
   amd.impl("skinny_linear_packed_relu_squared", torch::kCUDA, &skinny_linear_packed_relu_squared);
   amd.def("stream_linear_packed(Tensor x, Tensor w_packed, Tensor? bias, int N, int K) -> Tensor");

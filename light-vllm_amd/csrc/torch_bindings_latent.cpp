@@ -8,7 +8,7 @@ void check_latent_rows(const torch::Tensor& cache, int64_t cpad, int64_t rpad, c
               ": cache [blocks, block_size, cpad + rpad], blocks dense");
 }
 void latent_cache(torch::Tensor& cache, const torch::Tensor& kv, const torch::Tensor& weight, double eps, int64_t cpad,
-                  const torch::Tensor& positions, const torch::Tensor& turns, const torch::Tensor& slot_mapping) {
+                  const torch::Tensor& positions, const torch::Tensor& turns, const torch::Tensor& slot_mapping, double grow) {
   const char* op = "latent_cache";
   LV_CHECK_DEVICE(kv);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(kv));
@@ -23,14 +23,40 @@ void latent_cache(torch::Tensor& cache, const torch::Tensor& kv, const torch::Te
   check(lvllm_latent_cache(cache.data_ptr(), cache.stride(0), cache.size(0), (int)cache.size(1), (int)cpad, (int)rpad,
                            kv.data_ptr(), kv.stride(0), (int)rank, (int)(kv.size(1) - rank), weight.data_ptr<float>(),
                            (float)eps, positions.data_ptr<int64_t>(), turns.data_ptr<double>(), (int)turns.numel() * 2,
-                           slot_mapping.data_ptr<int64_t>(), (int)rows, dtype_code(kv, op), current_stream(kv)));
+                           (float)grow, slot_mapping.data_ptr<int64_t>(), (int)rows, dtype_code(kv, op), current_stream(kv)));
+}
+
+// q [rows, q_rank] -> its RMS norm, [rows, q_pad]; the rows' cache entries as latent_cache writes them
+torch::Tensor latent_down(const torch::Tensor& q, const torch::Tensor& q_weight, int64_t q_pad, torch::Tensor& cache,
+                          const torch::Tensor& kv, const torch::Tensor& weight, double eps, int64_t cpad,
+                          const torch::Tensor& positions, const torch::Tensor& turns, const torch::Tensor& slot_mapping,
+                          double grow) {
+  const char* op = "latent_down";
+  LV_CHECK_DEVICE(q);
+  const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
+  const int64_t rows = q.size(0), q_rank = q_weight.numel(), rank = weight.numel(), rpad = cache.size(2) - cpad;
+  check_latent_rows(cache, cpad, rpad, op);
+  check_rows2d(q, rows, q_rank, cache.scalar_type(), op, "q");
+  check_rows2d(kv, rows, kv.size(1), cache.scalar_type(), op, "kv");
+  check_f32(q_weight, q_rank, op, "q_weight");
+  check_f32(weight, rank, op, "weight");
+  check_rot(positions, turns, rows, op);
+  check_slots(slot_mapping, rows, op);
+  TORCH_CHECK(kv.size(1) >= rank, op, ": kv [rows, kv_rank + rot_dim]");
+  auto out = torch::empty({rows, q_pad}, q.options());
+  check(lvllm_latent_down(out.data_ptr(), q.data_ptr(), q.stride(0), (int)q_rank, (int)q_pad, q_weight.data_ptr<float>(),
+                          cache.data_ptr(), cache.stride(0), cache.size(0), (int)cache.size(1), (int)cpad, (int)rpad,
+                          kv.data_ptr(), kv.stride(0), (int)rank, (int)(kv.size(1) - rank), weight.data_ptr<float>(),
+                          (float)eps, positions.data_ptr<int64_t>(), turns.data_ptr<double>(), (int)turns.numel() * 2,
+                          (float)grow, slot_mapping.data_ptr<int64_t>(), (int)rows, dtype_code(q, op), current_stream(q)));
+  return out;
 }
 
 // kv, weight, slot_mapping: the rows' own latents, written to the cache by the same launch
 torch::Tensor latent_query(const torch::Tensor& q, const torch::Tensor& uk_t, int64_t dim, const torch::Tensor& positions,
                            const torch::Tensor& turns, const torch::Tensor& query_start_loc, int64_t absorbed_max,
                            torch::Tensor& cache, const std::optional<torch::Tensor>& kv,
-                           const std::optional<torch::Tensor>& weight, double eps, const torch::Tensor& slot_mapping) {
+                           const std::optional<torch::Tensor>& weight, double eps, const torch::Tensor& slot_mapping, double grow) {
   const char* op = "latent_query";
   LV_CHECK_DEVICE(q);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
@@ -55,7 +81,7 @@ torch::Tensor latent_query(const torch::Tensor& q, const torch::Tensor& uk_t, in
   auto out = torch::empty({rows, heads, cpad + rpad}, q.options());
   check(lvllm_latent_query(out.data_ptr(), q.data_ptr(), q.stride(0), uk_t.data_ptr(), (int)heads, (int)dim,
                            (int)uk_t.size(2), (int)cpad, (int)rpad, (int)rot_dim, (int)turns.numel() * 2,
-                           positions.data_ptr<int64_t>(), turns.data_ptr<double>(), query_start_loc.data_ptr<int>(),
+                           positions.data_ptr<int64_t>(), turns.data_ptr<double>(), (float)grow, query_start_loc.data_ptr<int>(),
                            (int)query_start_loc.numel() - 1, (int)absorbed_max, cache.data_ptr(), cache.stride(0),
                            cache.size(0), (int)cache.size(1), kv ? kv->data_ptr() : nullptr, kv ? kv->stride(0) : 0,
                            kv ? (int)weight->numel() : 0, kv ? weight->data_ptr<float>() : nullptr, (float)eps,
@@ -66,7 +92,7 @@ torch::Tensor latent_query(const torch::Tensor& q, const torch::Tensor& uk_t, in
 void latent_attention(torch::Tensor& out, const torch::Tensor& q, const torch::Tensor& cache, const torch::Tensor& uv,
                       const std::optional<torch::Tensor>& gate, int64_t vdim, const torch::Tensor& block_tables,
                       const torch::Tensor& seq_lens, const torch::Tensor& query_start_loc, double scale, int64_t window,
-                      int64_t absorbed_max, int64_t max_query_len, int64_t max_seq_len) {
+                      int64_t absorbed_max, int64_t max_query_len, int64_t max_seq_len, const std::optional<torch::Tensor>& sink) {
   const char* op = "latent_attention";
   LV_CHECK_DEVICE(q);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
@@ -80,13 +106,15 @@ void latent_attention(torch::Tensor& out, const torch::Tensor& q, const torch::T
   check_tables(block_tables, seq_lens.numel(), op);
   check_rows2d(out, rows, heads * vdim, q.scalar_type(), op, "out");
   if (gate) check_rows2d(*gate, rows, heads, q.scalar_type(), op, "gate");
+  if (sink) check_f32(*sink, heads, op, "sink");
   const int ns = (int)seq_lens.numel(), code = dtype_code(q, op), bs = (int)cache.size(1);
   const int64_t need = lvllm_latent_attention_workspace_bytes((int)rows, ns, (int)heads, (int)cpad, (int)rpad, bs, (int)window,
                                                               (int)absorbed_max, (int)max_query_len, (int)max_seq_len, code);
   auto ws = torch::empty({need}, q.options().dtype(at::kByte));
   check(lvllm_latent_attention(out.data_ptr(), out.stride(0), q.data_ptr(), cache.data_ptr(), cache.stride(0), cache.size(0), bs,
                                (int)cpad, (int)rpad, uv.data_ptr(), (int)vdim, (int)uv.size(1),
-                               gate ? gate->data_ptr() : nullptr, gate ? gate->stride(0) : 0, block_tables.data_ptr<int>(),
+                               gate ? gate->data_ptr() : nullptr, gate ? gate->stride(0) : 0,
+                               sink ? sink->data_ptr<float>() : nullptr, block_tables.data_ptr<int>(),
                                (int)block_tables.size(1), seq_lens.data_ptr<int>(), query_start_loc.data_ptr<int>(), ns,
                                (int)rows, (int)heads, (float)scale, (int)window, (int)absorbed_max, (int)max_query_len,
                                (int)max_seq_len, ws.data_ptr(), need, code, current_stream(q)));
@@ -131,7 +159,7 @@ std::tuple<torch::Tensor, torch::Tensor> latent_expand(const torch::Tensor& kv, 
 }
 
 torch::Tensor latent_rotate_query(const torch::Tensor& q, int64_t heads, int64_t dim, int64_t kpad,
-                                  const torch::Tensor& positions, const torch::Tensor& turns) {
+                                  const torch::Tensor& positions, const torch::Tensor& turns, double grow) {
   const char* op = "latent_rotate_query";
   LV_CHECK_DEVICE(q);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(q));
@@ -142,7 +170,7 @@ torch::Tensor latent_rotate_query(const torch::Tensor& q, int64_t heads, int64_t
   auto out = torch::empty({rows, heads, kpad}, q.options());
   check(lvllm_latent_rotate_query(out.data_ptr(), q.data_ptr(), q.stride(0), (int)heads, (int)dim,
                                   (int)(q.size(1) / heads - dim), (int)kpad, positions.data_ptr<int64_t>(),
-                                  turns.data_ptr<double>(), (int)turns.numel() * 2, (int)rows, dtype_code(q, op),
+                                  turns.data_ptr<double>(), (int)turns.numel() * 2, (float)grow, (int)rows, dtype_code(q, op),
                                   current_stream(q)));
   return out;
 }
@@ -218,21 +246,26 @@ torch::Tensor norm_add_mix(const std::optional<torch::Tensor>& x_out, const std:
 
 TORCH_LIBRARY_FRAGMENT(_C_amd, latent) {
   latent.def("latent_cache(Tensor(a!) cache, Tensor kv, Tensor weight, float eps, int cpad, Tensor positions, Tensor turns, "
-             "Tensor slot_mapping) -> ()");
+             "Tensor slot_mapping, float grow=1.) -> ()");
   latent.impl("latent_cache", torch::kCUDA, &latent_cache);
+  latent.def("latent_down(Tensor q, Tensor q_weight, int q_pad, Tensor(a!) cache, Tensor kv, Tensor weight, float eps, int cpad, "
+             "Tensor positions, Tensor turns, Tensor slot_mapping, float grow=1.) -> Tensor");
+  latent.impl("latent_down", torch::kCUDA, &latent_down);
   latent.def("latent_query(Tensor q, Tensor uk_t, int dim, Tensor positions, Tensor turns, Tensor query_start_loc, "
-             "int absorbed_max, Tensor(a!) cache, Tensor? kv, Tensor? weight, float eps, Tensor slot_mapping) -> Tensor");
+             "int absorbed_max, Tensor(a!) cache, Tensor? kv, Tensor? weight, float eps, Tensor slot_mapping, "
+             "float grow=1.) -> Tensor");
   latent.impl("latent_query", torch::kCUDA, &latent_query);
   latent.def("latent_attention(Tensor(a!) out, Tensor q, Tensor cache, Tensor uv, Tensor? gate, int vdim, Tensor block_tables, "
              "Tensor seq_lens, Tensor query_start_loc, float scale, int window, int absorbed_max, int max_query_len, "
-             "int max_seq_len) -> ()");
+             "int max_seq_len, Tensor? sink=None) -> ()");
   latent.impl("latent_attention", torch::kCUDA, &latent_attention);
   latent.def("latent_gather(Tensor cache, Tensor starts, Tensor first, Tensor seq_lens, Tensor block_tables, int n) -> Tensor");
   latent.impl("latent_gather", torch::kCUDA, &latent_gather);
   latent.def("latent_expand(Tensor kv, Tensor rows, int cpad, int heads, int dim, int rot_dim, int vdim, int kpad, int vpad) "
              "-> (Tensor, Tensor)");
   latent.impl("latent_expand", torch::kCUDA, &latent_expand);
-  latent.def("latent_rotate_query(Tensor q, int heads, int dim, int kpad, Tensor positions, Tensor turns) -> Tensor");
+  latent.def("latent_rotate_query(Tensor q, int heads, int dim, int kpad, Tensor positions, Tensor turns, "
+             "float grow=1.) -> Tensor");
   latent.impl("latent_rotate_query", torch::kCUDA, &latent_rotate_query);
   latent.def("embed_scale(Tensor(a!) x, Tensor table, Tensor ids, float scale) -> Tensor");
   latent.impl("embed_scale", torch::kCUDA, &embed_scale);

@@ -6,7 +6,7 @@ namespace {
 // (ids, weights, offsets, token, slots, tiles, slot_weight); w has a row per expert and, `gated`, one for the shared expert
 std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor> moe_route(
     const torch::Tensor& h, const torch::Tensor& w, const std::optional<torch::Tensor>& bias, int64_t top, bool shared,
-    bool packed, int64_t experts, bool gated, int64_t scoring, bool by_slot) {
+    bool packed, int64_t experts, bool gated, int64_t scoring, bool by_slot, int64_t groups, int64_t keep, double scale) {
   const char* op = "moe_route";
   LV_CHECK_DEVICE(h);
   const c10::hip::OptionalHIPGuardMasqueradingAsCUDA guard(device_of(h));
@@ -18,7 +18,8 @@ std::tuple<torch::Tensor, torch::Tensor, torch::Tensor, torch::Tensor, torch::Te
               op, ": h [rows, width], w [logits, width], packed: rows up to a multiple of 16");
   if (bias) check_f32(*bias, experts, op, "bias");
   const lvllm_moe_routing routing{(int)experts, (int)top, (int)scoring,
-                                  !shared ? LVLLM_MOE_NO_SHARED : gated ? LVLLM_MOE_GATED_SHARED : LVLLM_MOE_PLAIN_SHARED};
+                                  !shared ? LVLLM_MOE_NO_SHARED : gated ? LVLLM_MOE_GATED_SHARED : LVLLM_MOE_PLAIN_SHARED,
+                                  (int)groups, (int)keep, (float)scale};
   const auto ints = h.options().dtype(at::kInt), floats = h.options().dtype(at::kFloat);
   const int64_t n = top + shared, total = rows * n, tile = lvllm_moe_tile(packed, (int)rows);
   const int64_t max_tiles = std::max<int64_t>(1, std::min(total, total / tile + experts + shared));
@@ -67,7 +68,7 @@ torch::Tensor moe_experts(const torch::Tensor& x, const torch::Tensor& w, const 
 
 TORCH_LIBRARY_FRAGMENT(_C_amd, moe) {
   moe.def("moe_route(Tensor h, Tensor w, Tensor? bias, int top, bool shared, bool packed, int experts=0, bool gated=True, "
-          "int scoring=0, bool by_slot=False) -> (Tensor, Tensor, Tensor, Tensor, Tensor, Tensor, Tensor)");
+          "int scoring=0, bool by_slot=False, int groups=1, int keep=1, float scale=1.) -> (Tensor, Tensor, Tensor, Tensor, Tensor, Tensor, Tensor)");
   moe.impl("moe_route", torch::kCUDA, &moe_route);
   moe.def("moe_experts(Tensor x, Tensor w, Tensor w_offset, Tensor ff, Tensor? limit, Tensor offsets, Tensor token, "
           "Tensor tiles, int rows, int width, int ff_max, int ff_first, int ff_last, bool up, bool packed, "

@@ -3,6 +3,7 @@ part per token for all heads) and an optional mixture of experts, norms on what 
 the depth after every layer.  A layer may read an earlier layer's cache instead of having one.
 
 The engine asks for what it has to provide (`kv_cache_specs`, `state_specs`, `step_activation_bytes`), as for every model."""
+import math
 from dataclasses import dataclass
 from typing import List, Optional
 
@@ -12,10 +13,44 @@ from .moe import ExpertConfig, MixtureConfig
 
 
 @dataclass(frozen=True)
+class RampScaling:
+    """Pairs that turn `fast` times or more within `original` positions keep their frequency, those that turn `slow` times or
+    less are slowed down by `factor`, a linear ramp over the pairs lies between.  Vectors grow with the logarithm of the factor."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+    def __call__(self, frequencies: List[float], dims: int, base: float) -> List[float]:
+        def pair(turns):  # the (fractional) pair that turns so often
+            return dims * math.log(self.original / (2 * math.pi * turns)) / (2 * math.log(base))
+        first, last = max(math.floor(pair(self.fast)), 0), min(math.ceil(pair(self.slow)), dims - 1)
+        slowed = [min(max((i - first) / max(last - first, 1e-3), 0.0), 1.0) for i in range(len(frequencies))]
+        return [f / self.factor * s + f * (1.0 - s) for f, s in zip(frequencies, slowed)]
+
+    @property
+    def grow(self) -> float:
+        return 0.1 * math.log(self.factor) + 1.0
+
+
+@dataclass(frozen=True)
 class RotationConfig:
-    """Pairs (2i, 2i + 1) of the first `dims` entries turn by position * base^(-2i / dims)."""
+    """Pairs of the first `dims` entries -- (2i, 2i + 1), or (i, i + dims / 2) with `halves` -- turn by
+    position * base^(-2i / dims), scaled."""
     dims: int
     base: float
+    halves: bool = False
+    scaling: Optional[RampScaling] = None
+
+    def frequencies(self) -> List[float]:
+        """Radians per position of every pair."""
+        out = [self.base ** (-2.0 * i / self.dims) for i in range(self.dims // 2)]
+        return out if self.scaling is None else self.scaling(out, self.dims, self.base)
+
+    @property
+    def grow(self) -> float:
+        """What a rotated vector's length is multiplied by."""
+        return 1.0 if self.scaling is None else self.scaling.grow
 
 
 @dataclass(frozen=True)
@@ -54,8 +89,11 @@ class LatentAttentionConfig:
     kv_rank: int
     rot: RotationConfig
     scale: float
-    window: int                    # keys a query sees, its own included
+    window: int                    # keys a query sees, its own included (0: all up to its own)
     kv_from: Optional[int] = None  # the layer whose cache this one reads
+    q_rank: Optional[int] = None   # queries come out of a normed latent of this size
+    gate: bool = True              # a logit per head whose sigmoid scales the head's result
+    sink: bool = False             # one more score per head, without a key
 
     @property
     def spec(self) -> LatentKVSpec:

@@ -36,11 +36,22 @@ class OutputNorm:
 
 
 class Rotation:
-    """Full turns per position of every pair, in double: angles are reduced in double before the fp32 sine and cosine."""
+    """Full turns per position of every pair, in double: angles are reduced in double before the fp32 sine and cosine.
+
+    The kernels turn entries 2i and 2i + 1.  Rotated entries meet in a dot product only, so that other pairs are an order of the
+    rows that project queries and keys (`ordered`)."""
 
     def __init__(self, cfg: RotationConfig, device):
-        i = torch.arange(0, cfg.dims, 2, dtype=torch.float64, device=device)
-        self.turns = float(cfg.base) ** (-i / max(cfg.dims, 1)) / (2 * np.pi)
+        self.cfg, self.grow = cfg, cfg.grow
+        self.turns = torch.tensor(np.asarray(cfg.frequencies(), np.float64) / (2 * np.pi), dtype=torch.float64, device=device)
+
+    def ordered(self, rows: torch.Tensor) -> torch.Tensor:
+        """rows [..., rot_dim, k], of the rotated entries."""
+        if not self.cfg.halves:
+            return rows
+        half = self.cfg.dims // 2
+        at = [j for i in range(half) for j in (i, i + half)] + list(range(self.cfg.dims, rows.shape[-2]))
+        return rows.index_select(-2, torch.tensor(at, device=rows.device))
 
 
 @dataclass
@@ -60,7 +71,7 @@ def plan_long_portions(query_lens: List[int], context_lens: List[int], window: i
     long = q > longest_short
     if not long.any():
         return None
-    first = np.maximum(c - window + 1, 0) // page * page
+    first = np.maximum(c - (window or UNBOUNDED) + 1, 0) // page * page
     keys = np.where(long, c + q - first, 0)
     starts = np.zeros(len(q) + 1, np.int64)
     np.cumsum(-(-keys // page) * page, out=starts[1:])
@@ -107,14 +118,28 @@ class LatentAttention:
     def __init__(self, get, name: str, cfg: LatentAttentionConfig, eps: float, pack: bool):
         self.cfg, self.eps, self.spec = cfg, eps, cfg.spec
         H = cfg.heads
-        parts = [get(name + ".q"), get(name + ".g")]
-        if cfg.kv_from is None:
-            parts.append(get(name + ".dkv"))
-            self.norm = get(name + ".dkv.norm").float()
-        stack, self.at = stack_rows(parts)
-        self.sizes = [p.shape[0] for p in parts]
-        self.proj = make_weight(stack, pack)
         uk, uv = get(name + ".uk"), get(name + ".uv")
+        self.rotation = Rotation(cfg.rot, uk.device)
+
+        def queries(w):
+            w = w.view(H, cfg.dim + cfg.rot_dim, -1)
+            return torch.cat([w[:, :cfg.dim], self.rotation.ordered(w[:, cfg.dim:])], 1).reshape(H * w.shape[1], -1)
+        parts = {}
+        if cfg.q_rank is None:
+            parts["q"], self.up = queries(get(name + ".q")), None
+        else:
+            parts["q"], self.q_norm = get(name + ".dq"), get(name + ".dq.norm").float()
+            self.up = make_weight(stack_rows([pad_columns(queries(get(name + ".uq")))])[0], pack)
+        if cfg.gate:
+            parts["gate"] = get(name + ".g")
+        if cfg.kv_from is None:
+            dkv = get(name + ".dkv")
+            parts["dkv"] = torch.cat([dkv[:cfg.kv_rank], self.rotation.ordered(dkv[cfg.kv_rank:])])
+            self.norm = get(name + ".dkv.norm").float()
+        stack, at = stack_rows(list(parts.values()))
+        self.columns = {s: slice(o, o + p.shape[0]) for (s, p), o in zip(parts.items(), at)}
+        self.proj = make_weight(stack, pack)
+        self.sink = get(name + ".sink").float().contiguous() if cfg.sink else None
         dpad, vpad, cpad = ceil_to(cfg.dim, 32), ceil_to(cfg.vdim, 16), self.spec.cpad
         self.uk_t = uk.new_zeros(H, cpad, dpad)
         self.uk_t[:, :cfg.kv_rank, :cfg.dim] = uk.view(H, cfg.dim, cfg.kv_rank).transpose(1, 2)
@@ -124,32 +149,40 @@ class LatentAttention:
         # long portions take the expanded way where head_attention has a matrix-core body
         self.expands = uk.dtype == torch.bfloat16 and uk.is_cuda and self.pages.kpad <= 256 and self.pages.vpad <= 256
         self.expand = F.pad(torch.cat([uk, uv]), (0, cpad - cfg.kv_rank)).contiguous() if self.expands else None
-        self.rotation = Rotation(cfg.rot, uk.device)
         self.out_cols = H * cfg.vdim
         self.out = make_weight(pad_columns(get(name + ".o")), pack)
 
     def weights(self):
-        return [self.proj, self.out]
+        return [self.proj, self.out] + ([self.up] if self.up is not None else [])
+
+    def numel(self) -> int:
+        """What a decode step reads of them."""
+        return sum(w.numel() for w in self.weights()) + self.uk_t.numel() + self.uv.numel()
 
     def __call__(self, h: torch.Tensor, kv: torch.Tensor, layer: int, step: LatentStep, attn) -> SublayerOutput:
         """`kv`: the cache of layer number `layer`, this one's own or the one it reads."""
-        c, l, spec, turns = self.cfg, step.layout, self.spec, self.rotation.turns
+        c, l, spec, turns, grow = self.cfg, step.layout, self.spec, self.rotation.turns, self.rotation.grow
         proj = linear(h, self.proj)
-        q, gate, *dkv = (proj[:, o:o + n] for o, n in zip(self.at, self.sizes))
+        q, gate, dkv = (proj[:, self.columns[s]] if s in self.columns else None for s in ("q", "gate", "dkv"))
         cache = attn.rows_view(kv, spec, l.block_size)
         rows = h.shape[0]
         heads_out = (torch.empty if self.out.K == self.out_cols else torch.zeros)(rows, self.out.K, dtype=h.dtype, device=h.device)
         out = heads_out[:, :self.out_cols]
         plan = step.long_portions(c.window) if self.expands and l.block_size == 16 else None
-        if plan is not None and dkv:
-            amd.latent_cache(cache, dkv[0], self.norm, self.eps, spec.cpad, l.positions, turns, l.slot_mapping)
+        if self.up is not None:  # the query latents' norm; the rows' own latents go to the cache beside it
+            q = amd.latent_down(q, self.q_norm, self.up.K, cache, dkv, self.norm, self.eps, spec.cpad, l.positions, turns,
+                                l.slot_mapping, grow)
+            q, dkv = linear(q, self.up)[:, :c.heads * (c.dim + c.rot_dim)], None
+        elif plan is not None and dkv is not None:
+            amd.latent_cache(cache, dkv, self.norm, self.eps, spec.cpad, l.positions, turns, l.slot_mapping, grow)
+            dkv = None
         if plan is None or min(l.query_lens) <= ABSORBED_MAX:
             longest = ABSORBED_MAX if plan is not None else UNBOUNDED
-            own = (dkv[0], self.norm) if dkv and plan is None else (None, None)  # (written by the same launch)
+            own = (dkv, self.norm) if dkv is not None else (None, None)  # (written by the same launch)
             qa = amd.latent_query(q, self.uk_t, c.dim, l.positions, turns, l.query_start_loc, longest, cache, *own, self.eps,
-                                  l.slot_mapping)
+                                  l.slot_mapping, grow)
             amd.latent_attention(out, qa, cache, self.uv, gate, c.vdim, l.block_tables, l.seq_lens, l.query_start_loc, c.scale,
-                                 c.window, longest, l.max_query_len, l.max_seq_len)
+                                 c.window, longest, l.max_query_len, l.max_seq_len, self.sink)
         if plan is not None:
             self._long(out, q, gate, cache, layer, plan, step)
         return SublayerOutput(project_to_residual(heads_out, self.out))
@@ -159,6 +192,7 @@ class LatentAttention:
         lat = step.gathered(layer, c.window, cache, plan)
         kv = F.linear(lat[:, :spec.cpad], self.expand)
         keys, values = amd.latent_expand(kv, lat, spec.cpad, c.heads, c.dim, c.rot_dim, c.vdim, p.kpad, p.vpad)
-        qr = amd.latent_rotate_query(q, c.heads, c.dim, p.kpad, l.positions, self.rotation.turns)
+        qr = amd.latent_rotate_query(q, c.heads, c.dim, p.kpad, l.positions, self.rotation.turns,
+                                     self.rotation.grow)
         amd.head_attention(out, qr, keys, values, plan.tables, plan.seq_lens, l.query_start_loc, gate, c.vdim, c.scale, 1.0,
-                           l.max_query_len, plan.max_seq_len, c.window, ABSORBED_MAX + 1)
+                           l.max_query_len, plan.max_seq_len, c.window, ABSORBED_MAX + 1, sink=self.sink)

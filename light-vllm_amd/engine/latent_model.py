@@ -97,7 +97,7 @@ class LatentModel(LayeredModel):
         """Bytes of the projections and of all experts (a decode step reads the experts its tokens take)."""
         n = self.head.numel()
         for _, mixer, ff, _ in self.layers:
-            n += sum(w.numel() for w in mixer.weights()) + mixer.uk_t.numel() + mixer.uv.numel()
+            n += mixer.numel()
             if ff is not None:
                 n += ff[1].numel()
         return n * torch.empty((), dtype=self.cfg.dtype).element_size()

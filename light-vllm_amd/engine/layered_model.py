@@ -28,7 +28,7 @@ class LayeredModel:
                 return tensors[name].to(self.device).to(cfg.dtype)
         pack = cfg.pack_weights and self.device.type == "cuda"
         self.load(get, pack)
-        self.head = Weight(get("head").contiguous(), pack and cfg.dtype != torch.float32)
+        self.head = Weight(self.head_rows(get).contiguous(), pack and cfg.dtype != torch.float32)
 
     @staticmethod
     def tensor_shapes(cfg) -> Dict[str, tuple]:
@@ -41,6 +41,10 @@ class LayeredModel:
     def load(self, get: Callable[[str], torch.Tensor], pack: bool) -> None:
         """Everything but the head."""
         raise NotImplementedError
+
+    def head_rows(self, get: Callable[[str], torch.Tensor]) -> torch.Tensor:
+        """[vocab, width]"""
+        return get("head")
 
     def step_layout(self, md, positions: torch.Tensor, block_size: int, unified: Optional[tuple] = None) -> StepLayout:
         """`unified`: the device tensors of a captured mixed step (graph_runner.MixedGraph) in place of metadata."""

@@ -198,6 +198,25 @@ class TimeMixer:
         return x, project_to_residual(out, self.out)
 
 
+class SiluMlp:
+    """W_down (silu(W_gate h) * (W_up h))."""
+
+    def __init__(self, get, name: str, pack: bool):
+        # zero rows of gate and up give zero activations: all sizes may be padded for the weight-streaming kernel
+        self.up = make_weight(stack_rows([get(name + ".gate"), get(name + ".up")], 32)[0], pack)
+        self.down = make_weight(pad_columns(get(name + ".down")), pack)
+
+    def numel(self) -> int:
+        return self.up.numel() + self.down.numel()
+
+    def __call__(self, h: torch.Tensor) -> torch.Tensor:
+        if 0 < h.shape[0] <= DECODE_ROWS and self.up.packed is not None:
+            a = amd.skinny_linear_packed_swiglu(h, self.up.packed, None, self.up.N, self.up.K)
+        else:
+            a = amd.silu_unit(linear(h, self.up))
+        return project_to_residual(a, self.down)
+
+
 class SquaredReluMlp:
 
     def __init__(self, get, name: str, pack: bool):

@@ -11,7 +11,7 @@ from .mixers import ceil_to, pad_columns, stack_rows
 
 amd = torch.ops._C_amd
 SCORES = {"softmax": 0, "sigmoid": 1}     # include/lvllm_hip.h LVLLM_MOE_*
-ACTIVATIONS = {"clamped": 0, "silu": 1}
+ACTIVATIONS = {"clamped": 0, "silu": 1, "relu_squared": 2}
 
 
 class SublayerOutput(NamedTuple):
@@ -35,10 +35,22 @@ class MixtureConfig:
     expert: ExpertConfig
     shared: Optional[ExpertConfig]
     scores: str = "softmax"                   # weights: softmax over the chosen logits, or each logit's sigmoid
-    activation: str = "clamped"               # g sigmoid(1.702 g) (u + 1) of clamped g, u; "silu": g sigmoid(g) u
+    activation: str = "clamped"               # g sigmoid(1.702 g) (u + 1) of clamped g, u; "silu": g sigmoid(g) u;
+                                              # "relu_squared": max(u, 0)^2, without gate rows
     router_bias: bool = True
     shared_gate: bool = True                  # the shared expert is weighted by a logit of its own; else by 1
     weigh_input: bool = False                 # a weight scales what its expert reads, not what it returns
+    groups: int = 1                           # equal runs of neighbouring experts, of which a token may choose from the
+    keep: int = 1                             # `keep` with the largest best scores
+    weight_scale: float = 1.0                 # of the chosen experts' weights
+
+    def check(self, where: str) -> None:
+        if not 1 <= self.top <= self.experts:
+            raise ValueError(f"{where}: {self.top} of {self.experts} experts")
+        if self.groups < 1 or self.groups > 64 or self.experts % self.groups or not 1 <= self.keep <= self.groups:
+            raise ValueError(f"{where}: {self.keep} of {self.groups} groups of {self.experts} experts")
+        if self.top > self.keep * (self.experts // self.groups):
+            raise ValueError(f"{where}: {self.top} experts out of {self.keep} groups of {self.experts // self.groups}")
 
 
 def interleave_16(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
@@ -68,11 +80,12 @@ class MixtureOfExperts:
         self.router = amd.pack_weight(stack_rows([router])[0]) if self.packed else router.contiguous()
         ffp = [ceil_to(n, 32) for n in ff]
         self.ff_max, self.ff_first, self.ff_last, self.experts = max(ffp), max(ffp[:-1] or ffp), ffp[-1], len(names)
-        up_at, down_at = ([0] + np.cumsum([k * n * self.width for n in ffp]).tolist() for k in (2, 1))
+        gated = cfg.activation != "relu_squared"
+        up_at, down_at = ([0] + np.cumsum([k * n * self.width for n in ffp]).tolist() for k in (1 + gated, 1))
         self.up = torch.empty(up_at[-1], dtype=router.dtype, device=dev)
         self.down = torch.empty(down_at[-1], dtype=router.dtype, device=dev)
         for i, s in enumerate(names):
-            up = interleave_16(get(s + ".gate"), get(s + ".up"))
+            up = interleave_16(get(s + ".gate"), get(s + ".up")) if gated else stack_rows([get(s + ".up")], 32)[0]
             down = pad_columns(get(s + ".down")).contiguous()
             if self.packed:
                 up, down = amd.pack_weight(up), amd.pack_weight(down)
@@ -90,7 +103,7 @@ class MixtureOfExperts:
         c = self.cfg
         _, weights, offsets, token, slots, tiles, by_slot = amd.moe_route(
             h, self.router, self.bias, c.top, c.shared is not None, self.packed, c.experts, c.shared_gate, SCORES[c.scores],
-            c.weigh_input)
+            c.weigh_input, c.groups, c.keep, c.weight_scale)
         rows = h.shape[0]
         sizes = rows, self.width, self.ff_max, self.ff_first, self.ff_last
         a = amd.moe_experts(h, self.up, self.up_at, self.ff, self.limits, offsets, token, tiles, *sizes, True, self.packed,

@@ -42,6 +42,8 @@ MODELS = {
                            "..attention.latent_backend:LatentAttnBackend", ("heads", "moe", "latent")),
     "Lizazen": ModelEntry(".local_config:LocalModelConfig", ".local_model:LocalModel",
                           "..attention.head_backend:HeadAttnBackend", ("heads", "moe", "local")),
+    "Susalorn": ModelEntry(".stream_config:StreamModelConfig", ".stream_model:StreamModel",
+                           "..attention.latent_backend:LatentAttnBackend", ("heads", "moe", "latent", "delta")),
 }
 
 
