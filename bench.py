@@ -114,6 +114,10 @@ def parse():
                     help="instead of the headline workload: prefill and decode throughput of the local decoder beside the "
                          "hybrid decoder at equal sizes (tools/bench_local.py)")
     ap.add_argument("--local-only", default=None, help="with --local: the cases whose name starts with this")
+    ap.add_argument("--stream", action="store_true",
+                    help="instead of the headline workload: prefill and decode throughput of the stream decoder beside the "
+                         "latent decoder at equal sizes (tools/bench_stream.py)")
+    ap.add_argument("--stream-only", default=None, help="with --stream: the cases whose name starts with this")
     ap.add_argument("--tiny", action="store_true", help="tiny model (plumbing check)")
     ap.add_argument("--replica-backend", default=None, choices=["nccl", "gloo"],
                     help="process-group backend of the barrier / clock between replicas (default: nccl = RCCL)")
@@ -862,6 +866,11 @@ def main():
         sys.path.insert(0, os.path.join(ROOT, "tools"))
         import bench_local
         print(json.dumps({"local": bench_local.run("cuda:0", a.local_only)}), flush=True)
+        return
+    if a.stream:
+        sys.path.insert(0, os.path.join(ROOT, "tools"))
+        import bench_stream
+        print(json.dumps({"stream": bench_stream.run("cuda:0", a.stream_only)}), flush=True)
         return
     if a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(spawn_replicas(a))
