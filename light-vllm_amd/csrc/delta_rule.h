@@ -47,9 +47,10 @@ struct DeltaStepParams {
   float q_scale, eps;
 };
 
-// Pieces of one (chunk, head) in the workspace, in floats.  Fragments: 16-byte piece `lane` of a tile of 16 key channels (W, Q: row
-// lane % 16, channels 4 (lane / 16) ..; K: channel lane % 16, rows 4 (lane / 16) ..), of 16 value columns (U: column lane % 16,
-// rows 4 (lane / 16) ..), or of P (row lane % 16, columns 4 (lane / 16) ..).
+// Pieces of one (chunk, head) in the workspace, in floats.  W, q and k: 16-byte piece `lane` of a tile of 16 key channels (W, q:
+// row lane % 16, channels 4 (lane / 16) ..; k: channel lane % 16, rows 4 (lane / 16) ..).  U, per tile of 16 value columns, and P:
+// four runs of 64, entry `lane` of run r being row 4 (lane / 16) + r, column lane % 16 (P: row lane % 16, column
+// 4 (lane / 16) + r).
 struct ChunkLayout {
   int dkp, dvp;  // multiples of 64 and 16
   __host__ __device__ __forceinline__ int w() const { return 0; }

@@ -450,7 +450,7 @@ __global__ __launch_bounds__(256, NT <= 2 ? 2 : 1) void delta_prepare_kernel(con
     const int at = threadIdx.x;  // token ti, token tj
     const float pq = (spart[at] + spart[256 + at]) + (spart[512 + at] + spart[768 + at]) + extra_q;
     const float pk = (spart[1024 + at] + spart[1280 + at]) + (spart[1536 + at] + spart[1792 + at]) + extra_k;
-    ws[p.layout.p() + ((tj >> 2) * 16 + ti) * 4 + (tj & 3)] = tj <= ti ? pq : 0.f;
+    ws[p.layout.p() + (tj & 3) * 64 + (tj >> 2) * 16 + ti] = tj <= ti ? pq : 0.f;
     sa[ti * LA + tj] = tj < ti ? sb[ti] * pk : 0.f;
   }
   __syncthreads();
@@ -487,10 +487,9 @@ __global__ __launch_bounds__(256, NT <= 2 ? 2 : 1) void delta_prepare_kernel(con
 #pragma unroll
       for (int t = 0; t < 16; ++t) sks[t * LD + col] = x[t];
     } else {
-      float* u = ws + p.layout.u() + (d >> 4) * 256 + (d & 15) * 4;
+      float* u = ws + p.layout.u() + (d >> 4) * 256 + (d & 15);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        *reinterpret_cast<float4*>(u + j * 64) = float4{x[4 * j], x[4 * j + 1], x[4 * j + 2], x[4 * j + 3]};
+      for (int t = 0; t < 16; ++t) u[(t & 3) * 64 + (t >> 2) * 16] = x[t];
     }
   }
   __syncthreads();
@@ -533,102 +532,134 @@ __global__ __launch_bounds__(256, NT * NV <= 4 ? 2 : 1) void delta_scan_kernel(c
   const int64_t step = (int64_t)p.heads * p.layout.size();
   const float* ws = p.chunks + ((int64_t)chunk_slot_base(p.query_start_loc, seq) * p.heads + head) * p.layout.size();
   struct Frag {
-    float4 w[NT], q[NT], k[NT], end[NT], u[NV], pr;
+    float4 w[NT], q[NT], k[NT], end[NT];
+    float u[NV], pr;  // this wave's rows 4 g + wave of U, and columns 4 g + wave of P
   };
-  auto load = [&](int ci, Frag& f) __attribute__((always_inline)) {
-    const float* at = ws + ci * step;
+  const int tile_at = wave * NT * 256 + lane * 4;
+  auto load_tiles = [&](int ci, int piece, float4 (&to)[NT]) __attribute__((always_inline)) {
+    const float* at = ws + min(ci, chunks - 1) * step + piece + tile_at;
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int o = ((wave * NT + i) * 64 + lane) * 4;
-      f.w[i] = *reinterpret_cast<const float4*>(at + p.layout.w() + o);
-      f.q[i] = *reinterpret_cast<const float4*>(at + p.layout.q() + o);
-      f.k[i] = *reinterpret_cast<const float4*>(at + p.layout.k() + o);
-      f.end[i] = *reinterpret_cast<const float4*>(at + p.layout.end() + (wave * NT + i) * 16 + 4 * g);
-    }
+    for (int i = 0; i < NT; ++i) to[i] = *reinterpret_cast<const float4*>(at + i * 256);
+  };
+  auto load_rest = [&](int ci, Frag& f) __attribute__((always_inline)) {
+    const float* at = ws + min(ci, chunks - 1) * step;
 #pragma unroll
-    for (int j = 0; j < NV; ++j)
-      f.u[j] = *reinterpret_cast<const float4*>(at + p.layout.u() + (min(tile0 + j, tiles - 1) * 64 + lane) * 4);
-    f.pr = *reinterpret_cast<const float4*>(at + p.layout.p() + lane * 4);
+    for (int i = 0; i < NT; ++i) f.end[i] = *reinterpret_cast<const float4*>(at + p.layout.end() + (wave * NT + i) * 16 + 4 * g);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) f.u[j] = at[p.layout.u() + min(tile0 + j, tiles - 1) * 256 + wave * 64 + lane];
+    f.pr = at[p.layout.p() + wave * 64 + lane];
+  };
+  // (conditions per lane: selects, no branches)
+  const bool odd_wave = (threadIdx.x >> 6) & 1, high_wave = (threadIdx.x >> 7) & 1;
+  auto of_wave = [&](float x, float y, float z, float w) {
+    const float lo = odd_wave ? y : x, hi = odd_wave ? w : z;
+    return high_wave ? hi : lo;
   };
   // token et, column ec of a tile: where the accumulator layout has it
   const int et = threadIdx.x >> 4, ec = threadIdx.x & 15, eat = ((et >> 2) * 16 + ec) * 4 + (et & 3);
-  auto read_out = [&](int ci) __attribute__((always_inline)) {
-    const int t = ci * kChunk + et;
-    if (t >= qlen) return;
+  float* out = p.o + ((int64_t)(qbeg + et) * p.heads + head) * dv + tile0 * 16 + ec;  // of the chunk read out next
+  const int64_t out_step = (int64_t)kChunk * p.heads * dv;
+  auto read_out = [&](int ci, const float (&o)[NV][4]) __attribute__((always_inline)) {
 #pragma unroll
-    for (int j = 0; j < NV; ++j) {
-      const int col = (tile0 + j) * 16 + ec;
-      const float o = (so[ci & 1][0][j][eat] + so[ci & 1][1][j][eat]) + (so[ci & 1][2][j][eat] + so[ci & 1][3][j][eat]);
-      if (col < dv) p.o[((int64_t)(qbeg + t) * p.heads + head) * dv + col] = o;
-    }
+    for (int j = 0; j < NV; ++j)
+      if (ci * kChunk + et < qlen && (tile0 + j) * 16 + ec < dv) out[16 * j] = (o[j][0] + o[j][1]) + (o[j][2] + o[j][3]);
+    out += out_step;
   };
-  auto chunk = [&](int ci, const Frag& f) __attribute__((always_inline)) {
-    const int par = ci & 1;
-    r_f32x4_t o[NV];
+  auto shares_of = [&](int par, float (&o)[NV][4]) __attribute__((always_inline)) {
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int w = 0; w < 4; ++w) o[j][w] = so[par][w][j][eat];
+  };
+  // par: ci & 1.  The waves' shares of W S - U meet in LDS; half of (G q) S is computed while they are written, half while they
+  // are read.  What a later chunk needs is asked for as soon as its registers are free.
+  auto chunk = [&](int ci, int ahead, int par, Frag& f) __attribute__((always_inline)) {
+    r_f32x4_t a[NV], o[NV];
+    auto times_state = [&](int j, const float4 (&x)[NT], int r, r_f32x4_t acc) __attribute__((always_inline)) {
+#pragma unroll
+      for (int i = 0; i < NT; ++i)
+        acc = mfma_f32(r == 0 ? x[i].x : r == 1 ? x[i].y : r == 2 ? x[i].z : x[i].w, s[i][j][r], acc);
+      return acc;
+    };
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
-      r_f32x4_t a{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int i = 0; i < NT; ++i) {
-        a = mfma_f32(f.w[i].x, s[i][j][0], a);
-        a = mfma_f32(f.w[i].y, s[i][j][1], a);
-        a = mfma_f32(f.w[i].z, s[i][j][2], a);
-        a = mfma_f32(f.w[i].w, s[i][j][3], a);
-      }
-      *reinterpret_cast<r_f32x4_t*>(&swu[par][wave][j][lane * 4]) = a;
-    }
-#pragma unroll
-    for (int j = 0; j < NV; ++j) {
+      const float u = -f.u[j];
+      a[j] = r_f32x4_t{odd_wave || high_wave ? 0.f : u, !odd_wave || high_wave ? 0.f : u, odd_wave || !high_wave ? 0.f : u,
+                       odd_wave && high_wave ? u : 0.f};
       o[j] = r_f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int i = 0; i < NT; ++i) {
-        o[j] = mfma_f32(f.q[i].x, s[i][j][0], o[j]);
-        o[j] = mfma_f32(f.q[i].y, s[i][j][1], o[j]);
-        o[j] = mfma_f32(f.q[i].z, s[i][j][2], o[j]);
-        o[j] = mfma_f32(f.q[i].w, s[i][j][3], o[j]);
-      }
     }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int j = 0; j < NV; ++j) a[j] = times_state(j, f.w, r, a[j]);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) o[j] = times_state(j, f.q, 0, o[j]);
+    __builtin_amdgcn_sched_barrier(0);
+    load_tiles(ci + ahead, p.layout.w(), f.w);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) *reinterpret_cast<r_f32x4_t*>(&swu[par][wave][j][lane * 4]) = a[j];
+#pragma unroll
+    for (int j = 0; j < NV; ++j) o[j] = times_state(j, f.q, 1, o[j]);
+    __builtin_amdgcn_sched_barrier(0);
     delta_barrier();
+    r_f32x4_t t[NV][4];
+    float before[NV][4];  // the chunk before's read-out is complete
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int w = 0; w < 4; ++w) t[j][w] = *reinterpret_cast<const r_f32x4_t*>(&swu[par][w][j][lane * 4]);
+    shares_of(par ^ 1, before);
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int r = 2; r < 4; ++r)
+#pragma unroll
+      for (int j = 0; j < NV; ++j) o[j] = times_state(j, f.q, r, o[j]);
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        s[i][j][0] *= f.end[i].x; s[i][j][1] *= f.end[i].y; s[i][j][2] *= f.end[i].z; s[i][j][3] *= f.end[i].w;
+      }
+    __builtin_amdgcn_sched_barrier(0);
+    load_tiles(ci + ahead, p.layout.q(), f.q);
+    const float pr = f.pr;
+    load_rest(ci + ahead, f);
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
-      r_f32x4_t u{f.u[j].x, f.u[j].y, f.u[j].z, f.u[j].w};
-      {
-        r_f32x4_t t[4];
+      r_f32x4_t u;
 #pragma unroll
-        for (int w = 0; w < 4; ++w) t[w] = *reinterpret_cast<const r_f32x4_t*>(&swu[par][w][j][lane * 4]);
+      for (int r = 0; r < 4; ++r) u[r] = -((t[j][0][r] + t[j][1][r]) + (t[j][2][r] + t[j][3][r]));
+      o[j] = mfma_f32(pr, of_wave(u[0], u[1], u[2], u[3]), o[j]);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) u[r] -= (t[0][r] + t[1][r]) + (t[2][r] + t[3][r]);
-      }
+      for (int r = 0; r < 4; ++r)
 #pragma unroll
-      for (int i = 0; i < NT; ++i) {
-        r_f32x4_t n = s[i][j];
-        n[0] *= f.end[i].x; n[1] *= f.end[i].y; n[2] *= f.end[i].z; n[3] *= f.end[i].w;
-        n = mfma_f32(f.k[i].x, u[0], n);
-        n = mfma_f32(f.k[i].y, u[1], n);
-        n = mfma_f32(f.k[i].z, u[2], n);
-        n = mfma_f32(f.k[i].w, u[3], n);
-        s[i][j] = n;
-      }
-      // a wave takes a quarter of P's columns
-      o[j] = mfma_f32(wave == 0 ? f.pr.x : wave == 1 ? f.pr.y : wave == 2 ? f.pr.z : f.pr.w,
-                      wave == 0 ? u[0] : wave == 1 ? u[1] : wave == 2 ? u[2] : u[3], o[j]);
-      *reinterpret_cast<r_f32x4_t*>(&so[par][wave][j][lane * 4]) = o[j];
+        for (int i = 0; i < NT; ++i)
+          s[i][j] = mfma_f32(r == 0 ? f.k[i].x : r == 1 ? f.k[i].y : r == 2 ? f.k[i].z : f.k[i].w, u[r], s[i][j]);
     }
-    if (ci > 0) read_out(ci - 1);  // (complete since this chunk's barrier)
+    __builtin_amdgcn_sched_barrier(0);
+    load_tiles(ci + ahead, p.layout.k(), f.k);
+    if (ci > 0) read_out(ci - 1, before);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) *reinterpret_cast<r_f32x4_t*>(&so[par][wave][j][lane * 4]) = o[j];
   };
-  Frag f0, f1;
-  load(0, f0);
-  load(min(1, chunks - 1), f1);
-  for (int ci = 0; ci < chunks; ci += 2) {
-    chunk(ci, f0);
-    load(min(ci + 2, chunks - 1), f0);
-    if (ci + 1 < chunks) {
-      chunk(ci + 1, f1);
-      load(min(ci + 3, chunks - 1), f1);
-    }
+  constexpr int kDepth = NT * NV <= 2 ? 4 : 2;  // chunks asked for ahead
+  Frag f[kDepth];
+#pragma unroll
+  for (int d = 0; d < kDepth; ++d) {
+    load_tiles(d, p.layout.w(), f[d].w);
+    load_tiles(d, p.layout.q(), f[d].q);
+    load_rest(d, f[d]);
+    load_tiles(d, p.layout.k(), f[d].k);
+  }
+  for (int ci = 0; ci < chunks; ci += kDepth) {
+#pragma unroll
+    for (int d = 0; d < kDepth; ++d)
+      if (ci + d < chunks) chunk(ci + d, kDepth, d & 1, f[d]);
   }
   delta_barrier();
-  read_out(chunks - 1);
+  float last[NV][4];
+  shares_of((chunks - 1) & 1, last);
+  read_out(chunks - 1, last);
   if (!live) return;
 #pragma unroll
   for (int i = 0; i < NT; ++i)

@@ -214,11 +214,14 @@ class Worker:
         block_bytes = CacheEngine.get_cache_block_footprint(self.cache_config, self.model_config)
         out = self.kv_blocks_from_profile(total, self.init_gpu_memory, free_after_load, free_after_profile,
                                           self.cache_config.gpu_memory_utilization, scheduler_config.scheduling,
-                                          block_bytes, self.cache_config.swap_space_bytes,
+                                          max(block_bytes, 1), self.cache_config.swap_space_bytes,
                                           self.graph_reserve_bytes(scheduler_config)
                                           + self.sampler_reserve_bytes(scheduler_config)
                                           + CacheEngine.get_state_bytes(self.model_config,
                                                                         self.recurrent_state_slots(scheduler_config) or 0))
+        if block_bytes == 0:  # (no layer has a cache: blocks are numbers, as many as full sequences hold)
+            per_seq = -(-scheduler_config.max_model_len // self.cache_config.block_size)
+            out = (self.num_slots * scheduler_config.max_num_seqs * per_seq,) * 2
         self.profile = dict(total=total, init_free=self.init_gpu_memory, free_after_load=free_after_load,
                             free_after_profile=free_after_profile, block_bytes=block_bytes)
         import gc

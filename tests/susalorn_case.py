@@ -66,6 +66,10 @@ CONFIGS = {
         (latent(16, 128, 64, 128, 512, 320, 0.08), None),
         (delta(1, 1, 256, 264, 4), dense(160)),
         (delta(3, 3, 128, 96, 16), None)]),
+    # one kind of layer alone: states without a cache, caches without a state
+    "states": model(120, 64, 1e-4, 3, (0, 1, 2), [(delta(4, 4, 16, 32, 4), dense(48)), (delta(2, 1, 32, 16, 3), None)]),
+    "caches": model(120, 64, 1e-4, 3, (0, 2, 2), [
+        (latent(2, 16, 16, 24, 32, 24, 0.25), None), (latent(4, 24, 8, 16, 64, 40, 0.2, 5e3, None), moe(4, 1, 48, 2, 1, 1.3))]),
 }
 
 

@@ -540,6 +540,13 @@ def test_refuses_what_it_does_not_keep(folders):
         engine(folders["odd"], BF16, cache=dict(enable_prefix_caching=True))
 
 
+def test_sizing_without_a_cache(folders):
+    """Blocks cost nothing where no layer has a cache: the engine still finds a number of them."""
+    cfg, w = sc.case("states")
+    p = tokens(cfg, 20, 3)
+    assert generate(engine(folders["states"], F32, num_blocks=None), [p], 6) == [greedy(cfg, w, p, 6)]
+
+
 def test_programs(folders, tmp_path):
     """bin/generate and bin/trace_run as a user starts them."""
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
