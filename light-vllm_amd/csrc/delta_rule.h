@@ -20,7 +20,7 @@
 //       k to its end;
 //     - delta_scan_kernel, chunk after chunk: u = U - W S,  o = (G q)^T S + P u,  S <- G_end S + (k to the end)^T u.  The state's
 //       columns are independent: a workgroup takes 16 NV of them, its four waves a quarter of the key channels each.  What it
-//       reads is in fragment order, one 16-byte piece a lane, and asked for a chunk ahead;
+//       reads is in fragment order and asked for several chunks ahead;
 //     - head_norm_gate.h.
 //
 // Everything but the projections' results, the convolutions' and the gate is fp32.  Rows, sequences and slots as in recurrent.h.

@@ -103,7 +103,8 @@ __global__ __launch_bounds__(256) void delta_step_kernel(const DeltaStepParams p
     for (int j = 1; j < kAhead; ++j) y = fmaf(h.w[j], h.old[j], y);
     for (int j = kAhead; j < p.taps && j <= pos && live; ++j) {
       const int r = ring_row - j;
-      y = fmaf(p.conv_weight[(int64_t)(p.taps - 1 - j) * p.channels + c], ring[(int64_t)(r < 0 ? r + p.taps : r) * p.channels + c], y);
+      const float old = ring[(int64_t)(r < 0 ? r + p.taps : r) * p.channels + c];
+      y = fmaf(p.conv_weight[(int64_t)(p.taps - 1 - j) * p.channels + c], old, y);
     }
     if (keep && live) ring[(int64_t)ring_row * p.channels + c] = h.now;  // (read by nobody in this step)
     return silu_of(y);

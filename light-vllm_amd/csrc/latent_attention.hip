@@ -521,8 +521,8 @@ extern "C" int lvllm_latent_down(void* out, const void* q, int64_t q_stride, int
 extern "C" int lvllm_latent_query(void* out, const void* q, int64_t q_stride, const void* uk_t, int heads, int dim, int dpad,
                                   int cpad, int rpad, int rot_dim, int rot_dims, const int64_t* positions,
                                   const double* turns, float grow, const int32_t* query_start_loc, int num_seqs,
-                                  int absorbed_max, void* cache, int64_t block_stride, int64_t num_blocks, int block_size, const void* kv,
-                                  int64_t kv_stride, int kv_rank, const float* weight, float eps,
+                                  int absorbed_max, void* cache, int64_t block_stride, int64_t num_blocks, int block_size,
+                                  const void* kv, int64_t kv_stride, int kv_rank, const float* weight, float eps,
                                   const int64_t* slot_mapping, int rows, int dtype, void* stream) {
   LV_CHECK(dim > 0 && dim <= dpad && rot_dim <= rpad && rot_dims <= rot_dim && rot_dims % 2 == 0 && cpad % 16 == 0 &&
                rpad > 0 && rpad % 2 == 0, "latent sizes");
@@ -569,9 +569,10 @@ extern "C" int64_t lvllm_latent_attention_workspace_bytes(int rows, int num_seqs
 extern "C" int lvllm_latent_attention(void* out, int64_t out_stride, const void* q, const void* cache, int64_t block_stride,
                                       int64_t num_blocks, int block_size, int cpad, int rpad, const void* uv, int vdim, int vpad,
                                       const void* gate, int64_t gate_stride, const float* sink,
-                                      const int32_t* block_tables, int max_blocks, const int32_t* seq_lens, const int32_t* query_start_loc, int num_seqs, int rows,
-                                      int heads, float scale, int window, int absorbed_max, int max_query_len,
-                                      int max_seq_len, void* workspace, int64_t workspace_bytes, int dtype, void* stream) {
+                                      const int32_t* block_tables, int max_blocks, const int32_t* seq_lens,
+                                      const int32_t* query_start_loc, int num_seqs, int rows, int heads, float scale,
+                                      int window, int absorbed_max, int max_query_len, int max_seq_len, void* workspace,
+                                      int64_t workspace_bytes, int dtype, void* stream) {
   if (rows == 0 || num_seqs == 0) return 0;
   LV_CHECK(heads > 0 && heads <= 65535 && num_seqs <= 65535 && max_query_len > 0, "too many heads or sequences, or no query");
   LV_CHECK(cpad > 0 && cpad % 16 == 0 && rpad % 16 == 0 && cpad <= 8192 && rpad <= 2048, "rows are multiples of 16 elements");

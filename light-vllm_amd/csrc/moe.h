@@ -1,8 +1,8 @@
 // Mixture of experts for gfx950.  A token takes the `top` experts of the largest logits, weighted by the softmax over the chosen
 // ones or each by its own sigmoid, times `scale`, and, as one more assignment, the shared expert, with a gate of its own or the
 // weight 1.  With groups (equal runs of neighbouring experts) only the experts of the `keep` groups whose best logits are the
-// largest can be chosen.  The step's assignments are grouped by expert: slot s of the grouped order belongs to row token[s]; expert e owns slots
-// offsets[e] .. offsets[e + 1].
+// largest can be chosen.  The step's assignments are grouped by expert: slot s of the grouped order belongs to row token[s]; expert
+// e owns slots offsets[e] .. offsets[e + 1].
 //
 // Expert weights are two matrices per expert in one buffer:
 //   up    [2 ffp, width]: 16 gate rows, 16 value rows, 16 gate rows, ... (ffp: the inner size, zero rows up to a multiple of 32)

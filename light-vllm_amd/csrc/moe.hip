@@ -169,7 +169,8 @@ extern "C" int lvllm_moe_experts(void* out, const void* x, const void* w, const 
                                  void* stream) {
   if (slots == 0) return 0;
   LV_CHECK(experts > 0 && ff_max > 0 && ff_max % 32 == 0 && width > 0 && max_tiles > 0 && max_tiles <= 65535, "sizes of the experts");
-  LV_CHECK(!up || act == LVLLM_MOE_SILU || act == LVLLM_MOE_RELU_SQUARED || (act == LVLLM_MOE_CLAMPED && limit != nullptr), "unknown activation");
+  LV_CHECK(!up || act == LVLLM_MOE_SILU || act == LVLLM_MOE_RELU_SQUARED || (act == LVLLM_MOE_CLAMPED && limit != nullptr),
+           "unknown activation");
   MoeParams p{};
   p.out = out; p.x = x; p.w = w; p.w_offset = w_offset; p.ff = ff; p.limit = limit; p.offsets = offsets; p.token = token;
   p.tiles = tiles; p.experts = experts; p.slots = slots; p.rows = rows; p.width = width; p.ff_max = ff_max;

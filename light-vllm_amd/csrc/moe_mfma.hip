@@ -405,7 +405,8 @@ template <int PRODUCT>
 static void go(const MoeParams& p, hipStream_t s) {
   constexpr bool UP = PRODUCT != kMoeDown, GATED = PRODUCT == kMoeGated;
   if (p.rows <= kMoeFewRows) {
-    const int steps = (UP ? p.width : p.ff_max) / 32, units = GATED ? p.ff_max / 16 : (UP ? p.ff_max : p.width) / 32;  // of the largest expert
+    const int steps = (UP ? p.width : p.ff_max) / 32;  // of the largest expert
+    const int units = GATED ? p.ff_max / 16 : (UP ? p.ff_max : p.width) / 32;
     const int smem = (steps < kStreamChunk ? steps : kStreamChunk) * 1024;
     // workgroups with work, were every wave to take whole units
     const int64_t wgs = (int64_t)p.max_tiles * (((GATED ? p.ff_first / 16 : UP ? p.ff_first / 32 : units) + 3) / 4);
